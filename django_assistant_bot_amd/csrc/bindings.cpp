@@ -156,8 +156,100 @@ PYBIND11_MODULE(_native, m) {
                             (const float*)b_next, rows, cols, ST(s)),
           "dyt_residual");
   });
-  m.def("glu_f32", [](u out, u x, long rows, int F, int gelu, u s) {
-    check(dab::glu_f32((float*)out, (const float*)x, rows, F, gelu, ST(s)), "glu_f32");
+  m.def("glu_f32", [](u out, long ldo, u x, long rows, int F, int gelu, u bias, u row_scale, u perm, u s) {
+    check(dab::glu_f32((float*)out, ldo, (const float*)x, rows, F, gelu, (const float*)bias, (const float*)row_scale,
+                       (const int*)perm, ST(s)),
+          "glu_f32");
+  });
+  // chunked / sink attention over the paged cache
+  m.def("flash_attention_chunk",
+        [](u q, long qst, long qsh, u kc, u vc, u bt, int max_blocks, int bs, u out, long ost, long osh, u cu_q, u ctx_k,
+           int batch, int max_sq, int Hq, int Hkv, int D, float scale, int chunk, u sink, float out_scale, u s) {
+          check(dab::flash_attention(CVP(q), qst, qsh, nullptr, nullptr, 0, 0, CVP(kc), CVP(vc), (const int*)bt,
+                                     max_blocks, bs, VP(out), ost, osh, (const int*)cu_q, nullptr, (const int*)ctx_k,
+                                     batch, max_sq, Hq, Hkv, D, 1, 1, scale, ST(s), nullptr, nullptr, 0,
+                                     (const float*)sink, chunk, out_scale),
+                "flash_attention_chunk");
+        });
+  m.def("any_attention", [](u q, u kc, u vc, int f32, u bt, int max_blocks, int bs, u cu, u ctx, int B, int T, int H,
+                            int G, int D, int chunk, float scale, u sink, u out, long o_tok, float out_scale, u s) {
+    check(dab::any_attention(CVP(q), CVP(kc), CVP(vc), f32, (const int*)bt, max_blocks, bs, (const int*)cu,
+                             (const int*)ctx, B, T, H, G, D, chunk, scale, (const float*)sink, VP(out), o_tok, out_scale,
+                             ST(s)),
+          "any_attention");
+  });
+  // a projection is passed as (pointer, fp32, slabs, slab stride, row stride)
+  using P = std::tuple<u, int, int, long, long>;
+  const auto proj = [](const P& t) {
+    return dab::Proj{CVP(std::get<0>(t)), std::get<1>(t), std::get<2>(t), std::get<3>(t), std::get<4>(t)};
+  };
+  m.def("rms_residual", [proj](u x, u h, int act_f32, const P& y, u bias, u pairs, int top, u ids, u table, u gain,
+                               int n_true, float eps, int rows, int cols, int fresh, u s) {
+    check(dab::rms_residual((float*)x, VP(h), act_f32, proj(y), (const float*)bias, CVP(pairs), top, (const int*)ids,
+                            CVP(table), (const float*)gain, n_true, eps, rows, cols, fresh, ST(s)),
+          "rms_residual");
+  });
+  m.def("qk_rope_write", [proj](const P& y, int col0, int H, int G, int D, int dim, int rot, u freq, float eps, int norm,
+                                u positions, u slots, u q, u kc, u vc, int act_f32, int bs, int T, u s) {
+    check(dab::qk_rope_write(proj(y), col0, H, G, D, dim, rot, (const double*)freq, eps, norm, (const int*)positions,
+                             (const int64_t*)slots, VP(q), VP(kc), VP(vc), act_f32, bs, T, ST(s)),
+          "qk_rope_write");
+  });
+  m.def("recurrent_state_width", &dab::recurrent_state_width);
+  m.def("short_conv", [proj](const P& y, int col0, int C, int taps, u w, u bias, u ring, u slot, u pos, u cu, int chunks,
+                             int max_q, u out, int act_f32, u s) {
+    check(dab::short_conv(proj(y), col0, C, taps, (const float*)w, (const float*)bias, VP(ring), (const int*)slot,
+                          (const int*)pos, (const int*)cu, chunks, max_q, VP(out), act_f32, ST(s)),
+          "short_conv");
+  });
+  // shape = (delta, H, G, D, Dp, V, C, q_col, k_col, v_col, a_col, b_col)
+  using R = std::tuple<int, int, int, int, int, int, int, int, int, int, int, int>;
+  const auto shape = [](const R& t) {
+    return dab::RecurrentShape{std::get<0>(t), std::get<1>(t), std::get<2>(t), std::get<3>(t), std::get<4>(t),  std::get<5>(t),
+                               std::get<6>(t), std::get<7>(t), std::get<8>(t), std::get<9>(t), std::get<10>(t), std::get<11>(t)};
+  };
+  m.def("state_scan", [proj, shape](u conv, int act_f32, const R& d, const P& gates, u A, u dt_bias, u skip, u state,
+                                    u slot, u pos, u cu, int chunks, u out, u s) {
+    check(dab::state_scan(CVP(conv), act_f32, shape(d), proj(gates), (const float*)A, (const float*)dt_bias,
+                          (const float*)skip, (float*)state, (const int*)slot, (const int*)pos, (const int*)cu, chunks,
+                          VP(out), ST(s)),
+          "state_scan");
+  });
+  m.def("state_decode", [proj, shape](const P& y, int col0, int taps, u w, u bias, u ring, int act_f32, const R& d,
+                                      const P& gates, u A, u dt_bias, u skip, u state, u slot, u pos, int row0, int B,
+                                      int g_col, u norm, float eps, float out_scale, u out, long ldo, int pad, u s) {
+    check(dab::state_decode(proj(y), col0, taps, (const float*)w, (const float*)bias, VP(ring), act_f32, shape(d),
+                            proj(gates), (const float*)A, (const float*)dt_bias, (const float*)skip, (float*)state,
+                            (const int*)slot, (const int*)pos, row0, B, g_col, (const float*)norm, eps, out_scale,
+                            VP(out), ldo, pad, ST(s)),
+          "state_decode");
+  });
+  m.def("gated_norm", [proj](u y, int act_f32, const P& gate, int g_col, int n, int part, int gate_first, int per_head,
+                             u w, float eps, float scale, u out, long ldo, int pad, int row0, int T, u s) {
+    check(dab::gated_norm(CVP(y), act_f32, proj(gate), g_col, n, part, gate_first, per_head, (const float*)w, eps, scale,
+                          VP(out), ldo, pad, row0, T, ST(s)),
+          "gated_norm");
+  });
+  m.def("moe_route", [proj](const P& z, int col0, int E, int top, float scale, u idx, u wt, int T, u s) {
+    check(dab::moe_route(proj(z), col0, E, top, scale, (int*)idx, (float*)wt, T, ST(s)), "moe_route");
+  });
+  m.def("moe_plan", [](u idx, int pairs, int E, int bm, u perm, u tiles, int max_tiles, u s) {
+    check(dab::moe_plan((const int*)idx, pairs, E, bm, (int*)perm, VP(tiles), max_tiles, ST(s)), "moe_plan");
+  });
+  m.def("shared_glu", [proj](const P& y, int col0, int F, const P& z, int sg_col, u out, long ldo, int act_f32, int T, u s) {
+    check(dab::shared_glu(proj(y), col0, F, proj(z), sg_col, VP(out), ldo, act_f32, T, ST(s)), "shared_glu");
+  });
+  m.def("gemm_grouped", [](u A, long lda, u B, u C, long ldc, int N, int K, u perm, int a_div, int scatter, u tiles,
+                           int n_tiles, int bm, int glu, u row_scale, u s) {
+    check(dab::gemm_grouped(CVP(A), lda, CVP(B), VP(C), ldc, N, K, (const int*)perm, a_div, scatter, CVP(tiles), n_tiles,
+                            bm, glu, (const float*)row_scale, ST(s)),
+          "gemm_grouped");
+  });
+  m.def("gemm_f32_grouped", [](u A, long lda, u B, u C, long ldc, int N, int K, u perm, int a_div, int scatter, u tiles,
+                               int n_tiles, u s) {
+    check(dab::gemm_f32_grouped((const float*)A, lda, (const float*)B, (float*)C, ldc, N, K, (const int*)perm, a_div,
+                                scatter, CVP(tiles), n_tiles, ST(s)),
+          "gemm_f32_grouped");
   });
   m.def("gemm_f32", [](u A, long lda, long sa, u B, long ldb, long sb, u C, long ldc, long sc, int M, int N, int K,
                        int batch, u s) {
@@ -204,17 +296,19 @@ PYBIND11_MODULE(_native, m) {
   m.def("paged_decode_attention", [](u q, u kc, u vc, u bt, int max_blocks, int bs, u ctx, u out, u po, u pm, u pl,
                                      u cnt, int batch, int Hq, int Hkv, int D, int part_size, int max_parts,
                                      float scale, u s, u order, u w0, long w0_bytes, u w1, long w1_bytes,
-                                     int w_blocks) {
+                                     int w_blocks, int chunk, u sink, float out_scale, long o_stride) {
     dab::L3Warm warm{{(const char*)w0, (const char*)w1}, {w0_bytes, w1_bytes}, w_blocks};
     check(dab::paged_decode_attention(CVP(q), CVP(kc), CVP(vc), (const int*)bt, max_blocks, bs, (const int*)ctx, VP(out),
                                       (float*)po, (float*)pm, (float*)pl, (int*)cnt, batch, Hq, Hkv, D, part_size,
-                                      max_parts, scale, ST(s), (const int*)order, &warm),
+                                      max_parts, scale, ST(s), (const int*)order, &warm, chunk, (const float*)sink,
+                                      out_scale, o_stride),
           "paged_decode_attention");
   }, py::arg("q"), py::arg("kc"), py::arg("vc"), py::arg("bt"), py::arg("max_blocks"), py::arg("bs"), py::arg("ctx"),
      py::arg("out"), py::arg("po"), py::arg("pm"), py::arg("pl"), py::arg("cnt"), py::arg("batch"), py::arg("Hq"),
      py::arg("Hkv"), py::arg("D"), py::arg("part_size"), py::arg("max_parts"), py::arg("scale"), py::arg("s"),
      py::arg("order") = 0, py::arg("w0") = 0, py::arg("w0_bytes") = 0, py::arg("w1") = 0, py::arg("w1_bytes") = 0,
-     py::arg("w_blocks") = 0);
+     py::arg("w_blocks") = 0, py::arg("chunk") = 0, py::arg("sink") = 0, py::arg("out_scale") = 1.f,
+     py::arg("o_stride") = 0);
   m.def("gemm_bt", [](u A, long lda, u B, long ldb, u C, long ldc, u bias, u residual, long ldr, int M, int N, int K,
                       int epilogue, int out_f32, u row_group, u q_group, u allow, int allow_words, u s, int b_rows,
                       int b_group) {
@@ -454,7 +548,8 @@ PYBIND11_MODULE(_native, m) {
 
   // ---------------- KV block manager ----------------
   py::class_<dab::KVBlockManager>(m, "KVBlockManager")
-      .def(py::init<int, int, bool>(), py::arg("num_blocks"), py::arg("block_size"), py::arg("prefix_cache") = true)
+      .def(py::init<int, int, bool, int>(), py::arg("num_blocks"), py::arg("block_size"), py::arg("prefix_cache") = true,
+           py::arg("state_slots") = 0)
       .def("add_sequence", &dab::KVBlockManager::add_sequence)
       .def("extend", &dab::KVBlockManager::extend)
       .def("append_tokens", &dab::KVBlockManager::append_tokens)
@@ -468,6 +563,9 @@ PYBIND11_MODULE(_native, m) {
       .def("block_size", &dab::KVBlockManager::block_size)
       .def("prefix_hits", &dab::KVBlockManager::prefix_hits)
       .def("blocks", &dab::KVBlockManager::blocks)
+      .def("num_free_state_slots", &dab::KVBlockManager::num_free_state_slots)
+      .def("state_slots_into", [](const dab::KVBlockManager& k, const std::vector<int64_t>& seqs,
+                                  u out) { k.state_slots(seqs, (int32_t*)out); })
       .def("slot_mapping_into",
            [](const dab::KVBlockManager& k, int64_t seq, int start, int n, u out) {
              k.slot_mapping(seq, start, n, (int64_t*)out);

@@ -66,9 +66,16 @@ struct FlashParams {
   int lpt;
   // flash_fwd WIN only: query i sees keys i - window + 1 .. i (0: all before it); sink[h] joins head h's
   // denominator as one more logit without key or value (null: none)
-  int window;
+  // chunk > 0 instead of a window: query i sees keys i / chunk * chunk .. i.  out_scale multiplies the output
+  int window, chunk;
   const float* sink;
+  float out_scale;
 };
+
+// first key position that the query at position i sees
+__device__ __forceinline__ int first_key(int i, int window, int chunk) {
+  return chunk > 0 ? i / chunk * chunk : window > 0 ? max(0, i - window + 1) : 0;
+}
 
 // One workgroup = 16 QT NW queries (NW waves x QT 16-query sub-tiles) of one (sequence, head);
 // 64-key tiles staged through LDS with register prefetch of the next tile during compute (issue
@@ -155,8 +162,11 @@ __global__ __launch_bounds__(64 * NW, MINW ? MINW : ((QT == 2 && NW == 4) ? 2 : 
     n_keys = min(kv_len, kv_len - seqlen_q + last_q + 1);
   }
   const int n_tiles = div_up(n_keys, KT);
-  const int win = WIN && p.window > 0 ? p.window : kv_len;
-  const int kt0 = WIN ? max(0, kv_len - seqlen_q + q0 - win + 1) / KT : 0;
+  const int kt0 = WIN ? first_key(kv_len - seqlen_q + q0, p.window, p.chunk) / KT : 0;
+  int lo[QT];  // first key this lane's query sees
+#pragma unroll
+  for (int qt = 0; qt < QT; ++qt) lo[qt] = WIN ? first_key(q_pos[qt], p.window, p.chunk) : 0;
+  const int lo_last = WIN ? first_key(kv_len - seqlen_q + min(q0 + QB, seqlen_q) - 1, p.window, p.chunk) : 0;
 
   u32x4 kreg[CH], vreg[CH];
   // Branch-free staging: rows past the end are clamped to the last valid key (finite data, masked
@@ -229,7 +239,7 @@ __global__ __launch_bounds__(64 * NW, MINW ? MINW : ((QT == 2 && NW == 4) ? 2 : 
     }
     // online softmax per query sub-tile; only the tail / diagonal tiles need the mask
     const bool need_mask = (kt + 1) * KT > kv_len || (CAUSAL && (kt + 1) * KT - 1 > kv_len - seqlen_q + q0) ||
-                           (WIN && kt * KT + win <= kv_len - seqlen_q + q0 + QB - 1);
+                           (WIN && kt * KT < lo_last);
     bf16x8 pb[QT][2];
 #pragma unroll
     for (int qt = 0; qt < QT; ++qt) {
@@ -241,7 +251,7 @@ __global__ __launch_bounds__(64 * NW, MINW ? MINW : ((QT == 2 && NW == 4) ? 2 : 
           float v = s[qt][m][r] * p.scale_log2;
           if (need_mask) {
             const int key = kt * KT + 16 * m + 4 * g + r;
-            if (key >= kv_len || (CAUSAL && key > q_pos[qt]) || (WIN && key + win <= q_pos[qt])) v = kNegInf;
+            if (key >= kv_len || (CAUSAL && key > q_pos[qt]) || (WIN && key < lo[qt])) v = kNegInf;
           }
           s[qt][m][r] = v;
           mx = fmaxf(mx, v);
@@ -303,7 +313,7 @@ __global__ __launch_bounds__(64 * NW, MINW ? MINW : ((QT == 2 && NW == 4) ? 2 : 
     l_tot += __shfl_xor(l_tot, 16, 64);
     l_tot += __shfl_xor(l_tot, 32, 64);
     if (!q_valid[qt]) continue;
-    const float inv = l_tot > 0.f ? 1.f / l_tot : 0.f;
+    const float inv = l_tot > 0.f ? (WIN ? p.out_scale : 1.f) / l_tot : 0.f;
     bf16* orow = p.out + (size_t)(q_start + my_q[qt]) * p.o_stride_tok + (size_t)h * p.o_stride_head;
 #pragma unroll
     for (int t = 0; t < NTD; ++t) {
@@ -1525,6 +1535,12 @@ struct DecodeParams {
   const int* order;  // optional [B] sequence visit order (longest first: see paged_decode_attention)
   int Hq, Hkv, part_size, max_parts;
   float scale_log2;
+  // chunk > 0: the new token sees its own chunk's keys only; partitions are counted from the 32-key sub-tile that
+  // holds the chunk's first key.  sink (or null): one more score in head h's denominator
+  int chunk;
+  const float* sink;
+  float out_scale;
+  long o_stride_tok;
   L3Warm warm;  // optional: the next projections' weights, warmed into L3 by appended workgroups
 };
 
@@ -1579,7 +1595,10 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
   // The longest context is a wave max over ctx_lens (B <= a few hundred ints, L2-resident), so the
   // bound holds for any visit order; the longest-first order is only a load-balancing hint.
   int maxc = 0;
-  for (int i = lane; i < BH / p.Hkv; i += 64) maxc = max(maxc, p.ctx_lens[i]);
+  for (int i = lane; i < BH / p.Hkv; i += 64) {
+    const int c = p.ctx_lens[i];
+    maxc = max(maxc, c - (first_key(c - 1, 0, p.chunk) & ~(KT - 1)));
+  }
 #pragma unroll
   for (int off = 32; off; off >>= 1) maxc = max(maxc, __shfl_xor(maxc, off));
   maxc = __builtin_amdgcn_readfirstlane(maxc);
@@ -1589,7 +1608,8 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
     const int bh = item - part * BH;
     const int hk = bh % p.Hkv, b = p.order ? p.order[bh / p.Hkv] : bh / p.Hkv;
     const int ctx = p.ctx_lens[b];
-    const int k_begin = part * p.part_size;
+    const int k_lo = first_key(ctx - 1, 0, p.chunk), k_org = k_lo & ~(KT - 1);
+    const int k_begin = k_org + part * p.part_size;
     if (k_begin >= ctx) continue;
     const int k_end = min(ctx, k_begin + p.part_size);
 
@@ -1659,7 +1679,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
         for (int r = 0; r < 4; ++r) {
           const int key = k0 + 16 * m + 4 * g + r;
           float v = s[m][r] * p.scale_log2;
-          if (key >= k_end) v = kNegInf;
+          if (key >= k_end || key < k_lo) v = kNegInf;
           s[m][r] = v;
           mx = fmaxf(mx, v);
         }
@@ -1785,8 +1805,18 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
       lred[w * 16 + li] = l_run;
     }
     __syncthreads();
-    const int np = min(p.max_parts, div_up(ctx, p.part_size));
+    const int np = min(p.max_parts, div_up(ctx - k_org, p.part_size));
     const bool direct = np == 1;
+    // the finished output of head hq: the sink's term joins the denominator here, once
+    auto finish = [&](int qh, int d, float M, float L, float O) {
+      const int hh = hk * G + qh;
+      if (p.sink) {
+        const float sk = p.sink[hh] * 1.4426950408889634f, M2 = fmaxf(M, sk), f = exp2f(M - M2);
+        L = L * f + exp2f(sk - M2);
+        O *= f;
+      }
+      p.out[(size_t)b * p.o_stride_tok + (size_t)hh * D + d] = f2bf(L > 0.f ? O / L * p.out_scale : 0.f);
+    };
     for (int e = tid; e < G * D; e += 256) {
       const int qh = e / D, d = e % D;
       float M = -1e30f;
@@ -1801,7 +1831,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
       }
       const size_t hq = (size_t)b * p.Hq + hk * G + qh;
       if (direct) {
-        p.out[hq * D + d] = f2bf(L > 0.f ? O / L : 0.f);
+        finish(qh, d, M, L, O);
       } else {
         const size_t pi = hq * p.max_parts + part;
         // write-through (sc1) stores: visible to the combining workgroup on any XCD without a
@@ -1842,7 +1872,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
             L += f * ld(p.part_l + base + i);
             O += f * ld(p.part_o + (base + i) * D + d);
           }
-          p.out[hq * D + d] = f2bf(L > 0.f ? O / L : 0.f);
+          finish(qh, d, M, L, O);
         }
       }
     }
@@ -1857,7 +1887,8 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
                     const int* block_tables, int max_blocks, int block_size, void* out, long o_stride_tok,
                     long o_stride_head, const int* cu_q, const int* cu_k, const int* ctx_k, int batch,
                     int max_seqlen_q, int Hq, int Hkv, int D, int causal, int paged, float scale, hipStream_t s,
-                    const int* rope_pos, const void* rope_cs, int window, const float* sink) {
+                    const int* rope_pos, const void* rope_cs, int window, const float* sink, int chunk,
+                    float out_scale) {
   if (batch <= 0 || max_seqlen_q <= 0) return 0;
   if (Hq % Hkv || (paged && block_size % 64)) return hipErrorInvalidValue;
   FlashParams prm{};
@@ -1885,16 +1916,24 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
   prm.Hkv = Hkv;
   prm.scale_log2 = scale * 1.4426950408889634f;
   prm.pairs_per_wg = 1;
-  if (window > 0 || sink || D == 256) {  // windowed / sink form: packed keys, 16-query sub-tiles
-    if (!causal || paged || rope_cs) return hipErrorInvalidValue;
+  if (window > 0 || chunk > 0 || sink || D == 256 || out_scale != 1.f) {  // windowed / chunked / sink form: 16-query sub-tiles
+    if (!causal || rope_cs || (window > 0 && chunk > 0)) return hipErrorInvalidValue;
     prm.window = window;
+    prm.chunk = chunk;
     prm.sink = sink;
+    prm.out_scale = out_scale;
     const int qw = D >= 128 ? 128 : 64;
     const dim3 gw((max_seqlen_q + qw - 1) / qw, Hq, batch);
-    if (D == 64) hipLaunchKernelGGL((flash_fwd_kernel<64, true, false, 4, 1, 0, true>), gw, dim3(256), 0, s, prm);
-    else if (D == 128) hipLaunchKernelGGL((flash_fwd_kernel<128, true, false, 8, 1, 0, true>), gw, dim3(512), 0, s, prm);
-    else if (D == 256) hipLaunchKernelGGL((flash_fwd_kernel<256, true, false, 8, 1, 0, true>), gw, dim3(512), 0, s, prm);
-    else return hipErrorInvalidValue;
+#define DAB_FLASH_WIN(P)                                                                                                 \
+  do {                                                                                                                   \
+    if (D == 64) hipLaunchKernelGGL((flash_fwd_kernel<64, true, P, 4, 1, 0, true>), gw, dim3(256), 0, s, prm);           \
+    else if (D == 128) hipLaunchKernelGGL((flash_fwd_kernel<128, true, P, 8, 1, 0, true>), gw, dim3(512), 0, s, prm);    \
+    else if (D == 256) hipLaunchKernelGGL((flash_fwd_kernel<256, true, P, 8, 1, 0, true>), gw, dim3(512), 0, s, prm);    \
+    else return hipErrorInvalidValue;                                                                                    \
+  } while (0)
+    if (paged) DAB_FLASH_WIN(true);
+    else DAB_FLASH_WIN(false);
+#undef DAB_FLASH_WIN
     return hipGetLastError();
   }
   // Llama prefill (D = 128 over the paged cache): the 32x32 kernel below
@@ -2028,7 +2067,7 @@ int paged_decode_attention(const void* q, const void* k_cache, const void* v_cac
                            int max_blocks, int block_size, const int* ctx_lens, void* out, float* part_o,
                            float* part_m, float* part_l, int* counters, int batch, int Hq, int Hkv, int D,
                            int part_size, int max_parts, float scale, hipStream_t s, const int* order,
-                           const L3Warm* warm) {
+                           const L3Warm* warm, int chunk, const float* sink, float out_scale, long o_stride_tok) {
   if (batch <= 0) return 0;
   if (Hq % Hkv || Hq / Hkv > 16 || part_size % 128 || max_parts < 1 || block_size % 32) return hipErrorInvalidValue;
   if (max_parts > 1 && !counters) return hipErrorInvalidValue;
@@ -2052,6 +2091,10 @@ int paged_decode_attention(const void* q, const void* k_cache, const void* v_cac
   prm.part_size = part_size;
   prm.max_parts = max_parts;
   prm.scale_log2 = scale * 1.4426950408889634f;
+  prm.chunk = chunk;
+  prm.sink = sink;
+  prm.out_scale = out_scale;
+  prm.o_stride_tok = o_stride_tok ? o_stride_tok : (long)Hq * D;
   prm.warm = warm ? *warm : L3Warm{{nullptr, nullptr}, {0, 0}, 0};
   if (prm.warm.blocks < 0 || prm.warm.blocks > 1024 || ((prm.warm.bytes[0] | prm.warm.bytes[1]) & 15) ||
       (prm.warm.blocks && prm.warm.bytes[0] + prm.warm.bytes[1] <= 0))

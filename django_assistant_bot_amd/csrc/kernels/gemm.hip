@@ -49,11 +49,20 @@ struct GemmParams {
   int cap;
   int rows_b;  // SHUF: rows of the B copy (>= N, multiple of 16)
   int bgrp;    // SHUF: row blocks per group of the copy (shuffle_weights(w, group)), 1 = plain
+  const float* glu_bias;  // GLU over 8-row groups: fp32 [gate N / 2 | up N / 2], or null
+  // GROUP: rows of A and C grouped by expert (gemm_grouped)
+  const int4* tiles;      // {expert, first sorted position, rows, -}
+  const int* perm;        // sorted position -> (token, choice) pair
+  int n_tiles, a_div, scatter;
+  const float* row_scale; // GLU: [pairs] factor of a row
 };
 
 __device__ __forceinline__ int gsw(int r) { return 2 * ((r >> 1) & 3); }
 
-template <int EPI, int BM, int BN, int WGM, int WGN, bool SHUF = false>
+// GROUP (mixture of experts, SHUF): a row tile is a run of rows of one expert; B holds the experts' copies one
+// after the other.  A row: the sorted position itself, or token perm[pos] / a_div; C row: the sorted position, or
+// (scatter) the pair perm[pos].
+template <int EPI, int BM, int BN, int WGM, int WGN, bool SHUF = false, bool GROUP = false>
 __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
   constexpr int BK = 64;
   constexpr int NW = WGM * WGN;            // waves
@@ -62,7 +71,7 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
   constexpr int TILE_A = BM * BK * 2, TILE_B = BN * BK * 2;
   __shared__ __attribute__((aligned(16))) char smem[2 * (TILE_A + TILE_B)];  // [buf][A|B]
 
-  const int tiles_m = (p.M + BM - 1) / BM;
+  const int tiles_m = GROUP ? p.n_tiles : (p.M + BM - 1) / BM;
   const int tiles_n = (p.N + BN - 1) / BN;
   const int nwg = tiles_m * tiles_n;
   // bijective XCD remap: blocks b and b+8 share an XCD; give each XCD a contiguous id range
@@ -70,10 +79,27 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
   const int xcd = bid % 8, q8 = nwg / 8, r8 = nwg % 8;
   const int swz_id = (xcd < r8 ? xcd * (q8 + 1) : r8 * (q8 + 1) + (xcd - r8) * q8) + bid / 8;
   const int tm = swz_id % tiles_m, tn = swz_id / tiles_m;
-  const int m0 = tm * BM, n0 = tn * BN;
+  int m0 = tm * BM;
+  const int n0 = tn * BN;
+  if constexpr (GROUP) {
+    const int4 t = p.tiles[tm];
+    if (t.z <= 0) return;  // whole workgroup
+    m0 = t.y;
+    p.M = t.y + t.z;
+    p.B += (size_t)t.x * p.N * p.K;
+  }
 
   const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, g = lane >> 4, li = lane & 15;
   const int wm = w / WGN, wn = w % WGN;
+  int arow[GROUP ? BM / (8 * NW) : 1];  // GROUP: A rows this lane stages
+  if constexpr (GROUP) {
+#pragma unroll
+    for (int c = 0; c < BM / (8 * NW); ++c) {
+      const int pos = min(m0 + (((c * NW + w) * 64 + lane) >> 3), p.M - 1);
+      arow[c] = p.a_div > 0 ? p.perm[pos] / p.a_div : pos;
+    }
+  }
+  auto c_row = [&](int m) { return GROUP && p.scatter ? p.perm[m] : m; };
 
   // staging: instruction c of wave w writes LDS bytes [(c*NW+w)*1024, +1024) of a tile = rows 8(c*NW+w)..+7
   auto stage = [&](int buf, int k0) {
@@ -83,7 +109,7 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
     for (int c = 0; c < BM / (8 * NW); ++c) {
       const int e = (c * NW + w) * 64 + lane;
       const int r = e >> 3, pos = e & 7;
-      const int ra = min(m0 + r, p.M - 1);
+      const int ra = GROUP ? arow[GROUP ? c : 0] : min(m0 + r, p.M - 1);
       const bf16* ga = p.A + (size_t)ra * p.lda + k0 + (pos ^ gsw(r)) * 8;
       __builtin_amdgcn_global_load_lds((const void*)ga,
                                        (__attribute__((address_space(3))) void*)(As + (c * NW + w) * 1024), 16, 0, 0);
@@ -155,21 +181,27 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
 #pragma unroll
     for (int mi = 0; mi < MI; ++mi) {
       const int m = m0 + wm * TM + 16 * mi + li;
+      const float rs = GROUP && p.row_scale && m < p.M ? p.row_scale[p.perm[m]] : 1.f;
 #pragma unroll
       for (int pi = 0; pi < NI / 2; ++pi) {
+        const int oc = (n0 + wn * TN) / 2 + 16 * pi + 4 * g;
+        f32x4 bg = {0.f, 0.f, 0.f, 0.f}, bu = {0.f, 0.f, 0.f, 0.f};
+        if (p.glu_bias && 2 * oc < p.N) {
+          bg = *reinterpret_cast<const f32x4*>(p.glu_bias + oc);
+          bu = *reinterpret_cast<const f32x4*>(p.glu_bias + p.N / 2 + oc);
+        }
         float o[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const auto sw = __builtin_amdgcn_permlane32_swap(__float_as_uint(acc[2 * pi][mi][r]),
                                                            __float_as_uint(acc[2 * pi + 1][mi][r]), false, false);
-          o[r] = glu_act<EPI == EPI_GEGLU8>(__uint_as_float(sw[0])) * __uint_as_float(sw[1]);
+          o[r] = glu_act<EPI == EPI_GEGLU8>(__uint_as_float(sw[0]) + bg[r]) * (__uint_as_float(sw[1]) + bu[r]) * rs;
         }
-        const int oc = (n0 + wn * TN) / 2 + 16 * pi + 4 * g;
         if (m < p.M && 2 * oc < p.N) {
           u32x2 v;
           v[0] = pack2bf(o[0], o[1]);
           v[1] = pack2bf(o[2], o[3]);
-          *reinterpret_cast<u32x2*>((bf16*)p.C + (size_t)m * p.ldc + oc) = v;
+          *reinterpret_cast<u32x2*>((bf16*)p.C + (size_t)c_row(m) * p.ldc + oc) = v;
         }
       }
     }
@@ -257,7 +289,7 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
         u32x2 v;
         v[0] = pack2bf(o[0], o[1]);
         v[1] = pack2bf(o[2], o[3]);
-        *reinterpret_cast<u32x2*>((bf16*)p.C + (size_t)m * p.ldc + n) = v;
+        *reinterpret_cast<u32x2*>((bf16*)p.C + (size_t)c_row(m) * p.ldc + n) = v;
       }
     }
   }
@@ -287,13 +319,15 @@ int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
   if (K % 64 || N % 4 || lda % 8 || ldb % 8) return hipErrorInvalidValue;
   if (b_group < 1 || (b_group > 1 && (b_rows <= 0 || b_rows % (16 * b_group)))) return hipErrorInvalidValue;
   if (epilogue == EPI_SWIGLU && (N % 32 || out_f32)) return hipErrorInvalidValue;
-  if ((epilogue == EPI_SWIGLU8 || epilogue == EPI_GEGLU8) && (N % 32 || out_f32 || bias || residual)) return hipErrorInvalidValue;
+  if ((epilogue == EPI_SWIGLU8 || epilogue == EPI_GEGLU8) && (N % 32 || out_f32 || residual)) return hipErrorInvalidValue;
   if (b_rows > 0 && (b_rows < N || b_rows % 16 || ldb != K)) return hipErrorInvalidValue;
-  GemmParams p;
+  GemmParams p{};
   p.A = (const bf16*)A;
   p.B = (const bf16*)B;
   p.C = C;
-  p.bias = (const bf16*)bias;
+  const bool glu8 = epilogue == EPI_SWIGLU8 || epilogue == EPI_GEGLU8;  // their bias is fp32 [gate | up]
+  p.bias = glu8 ? nullptr : (const bf16*)bias;
+  p.glu_bias = glu8 ? (const float*)bias : nullptr;
   p.residual = (const bf16*)residual;
   p.row_group = row_group;
   p.q_group = q_group;
@@ -322,6 +356,38 @@ int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
     case EPI_GEGLU8: return launch_gemm<EPI_GEGLU8>(p, big, s, sh);
     default: return hipErrorInvalidValue;
   }
+}
+
+int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int N, int K, const int* perm, int a_div,
+                 int scatter, const void* tiles, int n_tiles, int bm, int glu, const float* row_scale, hipStream_t s) {
+  if (n_tiles <= 0 || N <= 0) return 0;
+  if (K % 64 || N % 32 || lda % 8 || ldc % 4 || !tiles || !perm || (bm != 32 && bm != 128) || (row_scale && !glu))
+    return hipErrorInvalidValue;
+  GemmParams p{};
+  p.A = (const bf16*)A;
+  p.B = (const bf16*)B;
+  p.C = C;
+  p.N = N;
+  p.K = K;
+  p.lda = lda;
+  p.ldc = ldc;
+  p.rows_b = N;
+  p.bgrp = 1;
+  p.tiles = (const int4*)tiles;
+  p.perm = perm;
+  p.n_tiles = n_tiles;
+  p.a_div = a_div;
+  p.scatter = scatter;
+  p.row_scale = row_scale;
+  const dim3 grid((unsigned)n_tiles * ((N + 127) / 128));
+  if (bm == 32) {
+    if (glu) hipLaunchKernelGGL((gemm_bt_kernel<EPI_SWIGLU8, 32, 128, 1, 4, true, true>), grid, dim3(256), 0, s, p);
+    else hipLaunchKernelGGL((gemm_bt_kernel<EPI_NONE, 32, 128, 1, 4, true, true>), grid, dim3(256), 0, s, p);
+  } else {
+    if (glu) hipLaunchKernelGGL((gemm_bt_kernel<EPI_SWIGLU8, 128, 128, 2, 2, true, true>), grid, dim3(256), 0, s, p);
+    else hipLaunchKernelGGL((gemm_bt_kernel<EPI_NONE, 128, 128, 2, 2, true, true>), grid, dim3(256), 0, s, p);
+  }
+  return hipGetLastError();
 }
 
 // b_rows > 0: B is a shuffle_weights copy of b_rows >= N rows (the index's one row layout).

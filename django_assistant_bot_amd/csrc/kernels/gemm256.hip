@@ -561,6 +561,13 @@ __global__ __launch_bounds__(512) void gemm256_kernel(G256 p) {
       if constexpr (BIAS) {
 #pragma unroll
         for (int jh = 0; jh < 2; ++jh) {
+          if constexpr (EPI == G_SWIGLU8 || EPI == G_GEGLU8) {  // fp32 [gate N / 2 | up N / 2]
+            const float* fb = reinterpret_cast<const float*>(p.bias) + (n0 + 128 * jh) / 2 + 16 * e_wc + 4 * e_g;
+            const f32x4 gv = *reinterpret_cast<const f32x4*>(fb), uv = *reinterpret_cast<const f32x4*>(fb + p.N / 2);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) bg[jh][r] = gv[r], bu[jh][r] = uv[r];
+            continue;
+          }
           const bf16* bp = p.bias + n0 + 128 * jh + 32 * e_wc + 4 * e_g;
           const u32x2 gv = *reinterpret_cast<const u32x2*>(bp), uv = *reinterpret_cast<const u32x2*>(bp + 16);
           bg[jh][0] = __uint_as_float(gv[0] << 16), bg[jh][1] = __uint_as_float(gv[0] & 0xffff0000u);
@@ -841,14 +848,13 @@ int gemm256_ok(int M, int N, int K, long lda, long ldb) {
 }
 
 // b_shuf: B is in the shuffle_weights layout (ldb == K).  Epilogues: 0 none, 1 GELU, 2 SwiGLU over
-// 16-row [gate | up] groups, 4 / 6 SwiGLU / tanh-GELU GLU over 8-row groups (no bias); bias / residual optional.
+// 16-row [gate | up] groups, 4 / 6 SwiGLU / tanh-GELU GLU over 8-row groups (bias: fp32 [gate | up]); bias / residual optional.
 int gemm256(const void* A, long lda, const void* B, long ldb, void* C, long ldc, const void* bias,
             const void* residual, long ldr, int M, int N, int K, int epilogue, hipStream_t s, int b_shuf,
             int b_group) {
   if (!gemm256_ok(M, N, K, lda, ldb)) return hipErrorInvalidValue;
   if (b_group != 1 && !(b_group == 8 && b_shuf)) return hipErrorInvalidValue;  // (N % 256: whole groups)
   if ((epilogue == G_SWIGLU || epilogue == G_SWIGLU8 || epilogue == G_GEGLU8) && residual) return hipErrorInvalidValue;
-  if ((epilogue == G_SWIGLU8 || epilogue == G_GEGLU8) && bias) return hipErrorInvalidValue;
   if (b_shuf && ldb != K) return hipErrorInvalidValue;
   G256 p{};
   p.A = (const bf16*)A;
@@ -904,10 +910,12 @@ int gemm256(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
       else G256_LAUNCH(G_SWIGLU, false, false);
       break;
     case G_SWIGLU8:
-      G256_LAUNCH(G_SWIGLU8, false, false);
+      if (hb) G256_LAUNCH(G_SWIGLU8, true, false);
+      else G256_LAUNCH(G_SWIGLU8, false, false);
       break;
     case G_GEGLU8:
-      G256_LAUNCH(G_GEGLU8, false, false);
+      if (hb) G256_LAUNCH(G_GEGLU8, true, false);
+      else G256_LAUNCH(G_GEGLU8, false, false);
       break;
     default: return hipErrorInvalidValue;
   }

@@ -12,8 +12,13 @@ struct GemmF32 {
   float* C;
   long lda, ldb, ldc, sa, sb, sc;
   int M, N, K;
+  // GROUP: as in gemm_bt_kernel
+  const int4* tiles;
+  const int* perm;
+  int a_div, scatter;
 };
 
+template <bool GROUP>
 __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32 p) {
   constexpr int BK = 16, LD = 20;  // LDS row stride in floats (16-B aligned, rows spread over the banks)
   __shared__ __attribute__((aligned(16))) float as[64 * LD];
@@ -21,11 +26,21 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32 p) {
   const float* A = p.A + (size_t)blockIdx.z * p.sa;
   const float* B = p.B + (size_t)blockIdx.z * p.sb;
   float* C = p.C + (size_t)blockIdx.z * p.sc;
-  const int m0 = blockIdx.y * 64, n0 = blockIdx.x * 64;
+  int m0 = blockIdx.y * 64;
+  const int n0 = blockIdx.x * 64;
+  if (GROUP) {
+    const int4 t = p.tiles[blockIdx.y];
+    if (t.z <= 0) return;  // whole workgroup
+    m0 = t.y;
+    p.M = t.y + t.z;
+    B += (size_t)t.x * p.N * p.K;
+  }
   const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, g = lane >> 4, li = lane & 15;
   const int wm = (w >> 1) * 32, wn = (w & 1) * 32;
   const int row = tid >> 2, kq = (tid & 3) * 4;
-  const float* ga = A + (size_t)min(m0 + row, p.M - 1) * p.lda + kq;
+  int ar = min(m0 + row, p.M - 1);
+  if (GROUP && p.a_div > 0) ar = p.perm[ar] / p.a_div;
+  const float* ga = A + (size_t)ar * p.lda + kq;
   const float* gb = B + (size_t)min(n0 + row, p.N - 1) * p.ldb + kq;
   f32x4 acc[2][2];
 #pragma unroll
@@ -61,10 +76,11 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32 p) {
   for (int i = 0; i < 2; ++i) {
     const int m = m0 + wm + 16 * i + li;
     if (m >= p.M) continue;
+    const size_t mc = GROUP && p.scatter ? p.perm[m] : m;
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
       const int n = n0 + wn + 16 * j + 4 * g;
-      if (n < p.N) *reinterpret_cast<f32x4*>(C + (size_t)m * p.ldc + n) = acc[i][j];  // N % 4 == 0
+      if (n < p.N) *reinterpret_cast<f32x4*>(C + mc * p.ldc + n) = acc[i][j];  // N % 4 == 0
     }
   }
 }
@@ -75,8 +91,17 @@ int gemm_f32(const float* A, long lda, long sa, const float* B, long ldb, long s
   if (K <= 0 || K % 16 || N % 4 || lda % 4 || ldb % 4 || ldc % 4 || sa % 4 || sb % 4 || sc % 4 || batch > 65535 ||
       (M + 63) / 64 > 65535)
     return hipErrorInvalidValue;
-  GemmF32 p{A, B, C, lda, ldb, ldc, sa, sb, sc, M, N, K};
-  hipLaunchKernelGGL(gemm_f32_kernel, dim3((N + 63) / 64, (M + 63) / 64, batch), dim3(256), 0, s, p);
+  GemmF32 p{A, B, C, lda, ldb, ldc, sa, sb, sc, M, N, K, nullptr, nullptr, 0, 0};
+  hipLaunchKernelGGL(gemm_f32_kernel<false>, dim3((N + 63) / 64, (M + 63) / 64, batch), dim3(256), 0, s, p);
+  return hipGetLastError();
+}
+
+int gemm_f32_grouped(const float* A, long lda, const float* B, float* C, long ldc, int N, int K, const int* perm, int a_div,
+                     int scatter, const void* tiles, int n_tiles, hipStream_t s) {
+  if (n_tiles <= 0 || N <= 0) return 0;
+  if (K <= 0 || K % 16 || N % 4 || lda % 4 || ldc % 4 || n_tiles > 65535 || !tiles || !perm) return hipErrorInvalidValue;
+  GemmF32 p{A, B, C, lda, K, ldc, 0, 0, 0, 0, N, K, (const int4*)tiles, perm, a_div, scatter};
+  hipLaunchKernelGGL(gemm_f32_kernel<true>, dim3((N + 63) / 64, n_tiles, 1), dim3(256), 0, s, p);
   return hipGetLastError();
 }
 

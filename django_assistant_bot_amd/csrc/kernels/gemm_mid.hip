@@ -43,7 +43,7 @@ struct GMid {
   const bf16* A;
   const bf16* B;  // shuffle_weights layout, [N][K]
   bf16* C;
-  const bf16* residual;
+  const bf16* residual;   // GLU epilogues with RES: fp32 bias [gate N / 2 | up N / 2] instead
   float* slabs;  // [tiles_m][gn][2] partial tiles of 128 x 256 fp32 (in accumulator order)
   int* cnt;      // [tiles_m][gn][2] ready flags of the stored partial tiles, zero at rest
   int M, N, K;
@@ -382,6 +382,17 @@ __global__ __launch_bounds__(512) void gemm_mid_kernel(GMid p) {
       if constexpr (EPI == MID_SWIGLU8 || EPI == MID_GEGLU8) {
         // 8-row [gate | up] groups inside each 16-row block: one permlane32_swap of the (jn, jn + 1)
         // pair gives lanes 0-31 block jn's gate / up rows and lanes 32-63 block jn + 1's
+        f32x4 bg[2], bu[2];
+#pragma unroll
+        for (int pr = 0; pr < 2; ++pr) {
+          bg[pr] = bu[pr] = f32x4{0.f, 0.f, 0.f, 0.f};
+          if constexpr (RES) {
+            const float* fb = reinterpret_cast<const float*>(p.residual) + (n0 + 64 * e_wc + 32 * pr) / 2 + 4 * e_g;
+            bg[pr] = *reinterpret_cast<const f32x4*>(fb);
+            bu[pr] = *reinterpret_cast<const f32x4*>(fb + p.N / 2);
+          }
+        }
+        if constexpr (RES) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int mr = 64 * wr + 16 * i + e_li;
@@ -392,7 +403,7 @@ __global__ __launch_bounds__(512) void gemm_mid_kernel(GMid p) {
             for (int r = 0; r < 4; ++r) {
               const auto s = __builtin_amdgcn_permlane32_swap(__float_as_uint(acc[i][2 * pr][r]),
                                                               __float_as_uint(acc[i][2 * pr + 1][r]), false, false);
-              o[r] = glu_act<EPI == MID_GEGLU8>(__uint_as_float(s[0])) * __uint_as_float(s[1]);
+              o[r] = glu_act<EPI == MID_GEGLU8>(__uint_as_float(s[0]) + bg[pr][r]) * (__uint_as_float(s[1]) + bu[pr][r]);
             }
             u32x2 v;
             v[0] = pack2bf(o[0], o[1]);
@@ -482,7 +493,7 @@ int gemm_mid_counters(int M, int N) {
 }
 
 // epilogue 0: C = A B^T (+ residual, bf16 add after rounding); 4 / 6: SwiGLU / tanh-GELU GLU over
-// 8-row [gate | up] groups (C has N / 2 columns).  slabs: gemm_mid_slab_bytes() bytes; cnt: >= gemm_mid_counters()
+// 8-row [gate | up] groups (C has N / 2 columns; residual: null, or their fp32 bias [gate | up]).  slabs: gemm_mid_slab_bytes() bytes; cnt: >= gemm_mid_counters()
 // ints, zero on first use (the launch leaves them zero).  variant (A/B harness only): 0 default
 // (BK 64), 32 / 64 force the K-step, + 1000 = DIAG 1 (split tiles not combined: timing only).
 // BK 32 (6-stage ring) measured 5-20 % slower than BK 64 on every mid shape, with LDS bank
@@ -493,7 +504,6 @@ int gemm_mid(const void* A, long lda, const void* B, void* C, long ldc, const vo
   if (!gemm_mid_ok(M, N, K, lda)) return hipErrorInvalidValue;
   if (b_group != 1 && b_group != 8) return hipErrorInvalidValue;
   if (epilogue != MID_NONE && epilogue != MID_SWIGLU8 && epilogue != MID_GEGLU8) return hipErrorInvalidValue;
-  if (epilogue != MID_NONE && residual) return hipErrorInvalidValue;
   if (!slabs || !cnt || slab_bytes < gemm_mid_slab_bytes() || n_cnt < gemm_mid_counters(M, N) ||
       slab_bytes >= (1L << 32))
     return hipErrorInvalidValue;
@@ -537,7 +547,9 @@ int gemm_mid(const void* A, long lda, const void* B, void* C, long ldc, const vo
       MID_LAUNCH(E, R, 32, 0);             \
     }                                      \
   } while (0)
-  if (epilogue == MID_SWIGLU8) MID_BK(MID_SWIGLU8, false);
+  if (epilogue == MID_SWIGLU8 && residual) MID_BK(MID_SWIGLU8, true);
+  else if (epilogue == MID_GEGLU8 && residual) MID_BK(MID_GEGLU8, true);
+  else if (epilogue == MID_SWIGLU8) MID_BK(MID_SWIGLU8, false);
   else if (epilogue == MID_GEGLU8) MID_BK(MID_GEGLU8, false);
   else if (residual) MID_BK(MID_NONE, true);
   else MID_BK(MID_NONE, false);

@@ -21,6 +21,15 @@ struct L3Warm {
   int blocks;  // 0: off
 };
 
+// A projection as its consumers see it: rows of ``ld`` columns, finished (S == 1) or as S split-K slabs ``slab``
+// elements apart (proj.h)
+struct Proj {
+  const void* p;
+  int f32;
+  int S;
+  long slab, ld;
+};
+
 // norm.hip
 int rmsnorm(void* out, void* res_out, const void* x, const void* res_in, const void* w, int rows, int cols, float eps,
             hipStream_t s);
@@ -48,12 +57,51 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
                     long o_stride_head, const int* cu_q, const int* cu_k, const int* ctx_k, int batch,
                     int max_seqlen_q, int Hq, int Hkv, int D, int causal, int paged, float scale, hipStream_t s,
                     const int* rope_pos = nullptr, const void* rope_cs = nullptr, int window = 0,
-                    const float* sink = nullptr);
+                    const float* sink = nullptr, int chunk = 0, float out_scale = 1.f);
 int paged_decode_attention(const void* q, const void* k_cache, const void* v_cache, const int* block_tables,
                            int max_blocks, int block_size, const int* ctx_lens, void* out, float* part_o,
                            float* part_m, float* part_l, int* counters, int batch, int Hq, int Hkv, int D,
                            int part_size, int max_parts, float scale, hipStream_t s,
-                           const int* order = nullptr, const L3Warm* warm = nullptr);
+                           const int* order = nullptr, const L3Warm* warm = nullptr, int chunk = 0,
+                           const float* sink = nullptr, float out_scale = 1.f, long o_stride_tok = 0);
+
+// attention_any.hip (any head width, bf16 or fp32, paged)
+int any_attention(const void* q, const void* kc, const void* vc, int f32, const int* bt, int max_blocks, int bs,
+                  const int* cu, const int* ctx, int B, int T, int H, int G, int D, int chunk, float scale,
+                  const float* sink, void* out, long o_tok, float out_scale, hipStream_t s);
+
+// rms_stream.hip (RMS norms around an fp32 residual stream; rotary positions and q / k norm before attention)
+int rms_residual(float* x, void* h, int act_f32, Proj y, const float* bias, const void* pairs, int top, const int* ids,
+                 const void* table, const float* gain, int n_true, float eps, int rows, int cols, int fresh,
+                 hipStream_t s);
+int qk_rope_write(Proj y, int col0, int H, int G, int D, int dim, int rot, const double* freq, float eps, int norm,
+                  const int* positions, const int64_t* slots, void* q, void* kc, void* vc, int act_f32, int bs, int T,
+                  hipStream_t s);
+
+// recurrent.hip (matrix-state recurrences: gated delta rule and state-space duality)
+struct RecurrentShape {
+  int delta;                       // 1: gated delta rule, 0: state-space duality
+  int H, G, D, Dp, V;              // heads, q / k groups, state rows (padded: Dp), value columns
+  int C, q_col, k_col, v_col;      // convolution channels and where q, k, v start among them
+  int a_col, b_col;                // gate columns (decay / step, beta)
+};
+int recurrent_state_width(int D);  // D padded as the state is stored
+int short_conv(Proj y, int col0, int C, int taps, const float* w, const float* bias, void* ring, const int* slot,
+               const int* pos, const int* cu, int chunks, int max_q, void* out, int act_f32, hipStream_t s);
+int state_scan(const void* conv, int act_f32, RecurrentShape d, Proj gates, const float* A, const float* dt_bias,
+               const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, void* out,
+               hipStream_t s);
+int state_decode(Proj y, int col0, int taps, const float* w, const float* bias, void* ring, int act_f32, RecurrentShape d,
+                 Proj gates, const float* A, const float* dt_bias, const float* skip, float* state, const int* slot,
+                 const int* pos, int row0, int B, int g_col, const float* norm, float eps, float out_scale, void* out,
+                 long ldo, int pad, hipStream_t s);
+int gated_norm(const void* y, int act_f32, Proj gate, int g_col, int n, int part, int gate_first, int per_head,
+               const float* w, float eps, float scale, void* out, long ldo, int pad, int row0, int T, hipStream_t s);
+
+// moe.hip
+int moe_route(Proj z, int col0, int E, int top, float scale, int* idx, float* wt, int T, hipStream_t s);
+int moe_plan(const int* idx, int P, int E, int bm, int* perm, void* tiles, int max_tiles, hipStream_t s);
+int shared_glu(Proj y, int col0, int F, Proj z, int sg_col, void* out, long ldo, int act_f32, int T, hipStream_t s);
 
 // dyt.hip (Dynamic Tanh norms around an fp32 residual stream)
 int embed_dyt(float* x, void* h, const int* ids, const void* table, int f32, float scale, float alpha, const float* w,
@@ -61,11 +109,16 @@ int embed_dyt(float* x, void* h, const int* ids, const void* table, int f32, flo
 int dyt_residual(float* x, void* h, int h_f32, const void* y, int y_f32, int S, long slab_stride, float a_post,
                  const float* w_post, const float* b_post, const float* ls, float a_next, const float* w_next,
                  const float* b_next, int rows, int cols, hipStream_t s);
-int glu_f32(float* out, const float* x, long rows, int F, int gelu, hipStream_t s);
+int glu_f32(float* out, long ldo, const float* x, long rows, int F, int gelu, const float* bias, const float* row_scale,
+            const int* perm, hipStream_t s);
 
 // gemm_f32.hip (32-bit mode; batched by strides)
 int gemm_f32(const float* A, long lda, long sa, const float* B, long ldb, long sb, float* C, long ldc, long sc, int M,
              int N, int K, int batch, hipStream_t s);
+// rows of A and C grouped by expert (moe_plan tiles of 64 rows): C[pos] = A[perm[pos] / a_div] . B[expert]^T with
+// a_div > 0, A[pos] otherwise; scatter: C row perm[pos]
+int gemm_f32_grouped(const float* A, long lda, const float* B, float* C, long ldc, int N, int K, const int* perm, int a_div,
+                     int scatter, const void* tiles, int n_tiles, hipStream_t s);
 
 // latent_attention.hip
 int latent_write(const void* y, int y_f32, int S, long slab_stride, long ld, void* q_out, int q_cols, const float* gain,
@@ -89,6 +142,10 @@ int latent_any(void* out, const void* q, const void* cache, int f32, const int* 
 int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc, const void* bias, const void* residual,
             long ldr, int M, int N, int K, int epilogue, int out_f32, const int* row_group, const int* q_group,
             const uint32_t* allow, int allow_words, hipStream_t s, int b_rows = 0, int b_group = 1);
+// experts: like gemm_f32_grouped, bf16, B = per-expert shuffle_weights copies of N rows; glu: SwiGLU over 8-row groups,
+// each row times row_scale[pair].  bm: rows of a tile (32 or 128)
+int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int N, int K, const int* perm, int a_div,
+                 int scatter, const void* tiles, int n_tiles, int bm, int glu, const float* row_scale, hipStream_t s);
 
 // gemm256.hip (large-M prefill / encoder GEMM, 256x256 phased schedule; epilogue 0 none, 1 GELU,
 // 2 SwiGLU on [gate 16 | up 16]-interleaved weight rows; bias / residual optional)

@@ -1,0 +1,97 @@
+// A projection as its consumers see it: T rows of ``ld`` columns, either the finished output (S == 1) or the
+// producing GEMM's split-K slabs (S > 1, ``slab`` elements apart), which the consumer sums in fp32.
+#pragma once
+#include "common.h"
+
+namespace dab {
+
+template <typename T>
+struct ElemIO;
+template <>
+struct ElemIO<bf16> {
+  static __device__ __forceinline__ float load(const bf16* p) { return bf2f(*p); }
+  static __device__ __forceinline__ void store(bf16* p, float v) { *p = f2bf(v); }
+  static __device__ __forceinline__ float round(float v) { return bf2f(f2bf(v)); }
+  static __device__ __forceinline__ float2 load2(const bf16* p) {
+    const uint32_t v = *reinterpret_cast<const uint32_t*>(p);
+    return make_float2(__uint_as_float(v << 16), __uint_as_float(v & 0xffff0000u));
+  }
+  static __device__ __forceinline__ void store2(bf16* p, float a, float b) { *reinterpret_cast<uint32_t*>(p) = pack2bf(a, b); }
+  static __device__ __forceinline__ void load8(const bf16* p, float (&f)[8]) {
+    unpack8(*reinterpret_cast<const u32x4*>(p), f);
+  }
+  static __device__ __forceinline__ void store8(bf16* p, const float (&f)[8]) { *reinterpret_cast<u32x4*>(p) = pack8(f); }
+};
+template <>
+struct ElemIO<float> {
+  static __device__ __forceinline__ float load(const float* p) { return *p; }
+  static __device__ __forceinline__ void store(float* p, float v) { *p = v; }
+  static __device__ __forceinline__ float round(float v) { return v; }
+  static __device__ __forceinline__ float2 load2(const float* p) { return *reinterpret_cast<const float2*>(p); }
+  static __device__ __forceinline__ void store2(float* p, float a, float b) { *reinterpret_cast<float2*>(p) = make_float2(a, b); }
+  static __device__ __forceinline__ void load8(const float* p, float (&f)[8]) {
+    const f32x4 a = *reinterpret_cast<const f32x4*>(p), b = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      f[j] = a[j];
+      f[4 + j] = b[j];
+    }
+  }
+  static __device__ __forceinline__ void store8(float* p, const float (&f)[8]) {
+    *reinterpret_cast<f32x4*>(p) = f32x4{f[0], f[1], f[2], f[3]};
+    *reinterpret_cast<f32x4*>(p + 4) = f32x4{f[4], f[5], f[6], f[7]};
+  }
+};
+
+// element (row, col); rounded to the activation type AT when it was summed from slabs, like a finished output
+template <typename PT, typename AT>
+__device__ __forceinline__ float proj_at(const Proj& p, long row, int col) {
+  const PT* q = (const PT*)p.p + row * p.ld + col;
+  float v = ElemIO<PT>::load(q);
+  for (int s = 1; s < p.S; ++s) v += ElemIO<PT>::load(q + s * p.slab);
+  return ElemIO<AT>::round(v);
+}
+
+// the same without rounding (values that stay in 32 bits)
+template <typename PT>
+__device__ __forceinline__ float proj_f32(const Proj& p, long row, int col) {
+  const PT* q = (const PT*)p.p + row * p.ld + col;
+  float v = ElemIO<PT>::load(q);
+  for (int s = 1; s < p.S; ++s) v += ElemIO<PT>::load(q + s * p.slab);
+  return v;
+}
+
+// 8 consecutive elements (col % 8 == 0, ld % 8 == 0)
+template <typename PT>
+__device__ __forceinline__ void proj8(const Proj& p, long row, int col, float (&f)[8]) {
+  const PT* q = (const PT*)p.p + row * p.ld + col;
+  ElemIO<PT>::load8(q, f);
+  int s = 1;
+  for (; s + 4 <= p.S; s += 4) {
+    SlabVec8<PT> v[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j].load(q + (s + j) * p.slab);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j].add_to(f);
+  }
+  for (; s < p.S; ++s) {
+    SlabVec8<PT> v;
+    v.load(q + s * p.slab);
+    v.add_to(f);
+  }
+}
+
+// Type dispatch of kernels <projection type, activation type>: bf16 rows, fp32 slabs of a bf16 model, fp32 model.
+#define DAB_PROJ_DISPATCH(y, act_f32, CALL)   \
+  do {                                        \
+    if (act_f32) {                            \
+      if (!(y).f32) return hipErrorInvalidValue; \
+      CALL(float, float);                     \
+    } else if ((y).f32) {                     \
+      CALL(float, bf16);                      \
+    } else {                                  \
+      CALL(bf16, bf16);                       \
+    }                                         \
+  } while (0)
+
+}  // namespace dab

@@ -1,0 +1,224 @@
+// RMS norms around an fp32 residual stream, and the step between a layer's input projection and its attention.
+//
+//   embed_rms       x = table[id]; h = x / rms(x) * gain
+//   rms_residual    x += sublayer output (GEMM rows or split-K slabs) + bias + the token's expert rows
+//                   [+ table[id]];  h = x / rms(x) * gain: everything between two layers in one pass
+//   qk_rope_write   [q | k | v] columns of a projection -> interleaved rotary positions on q and k, weightless
+//                   RMS norm per head, q rows out, k / v into the paged cache
+//
+// Gains are fp32 and already hold 1 + w where a model stores them around zero.  The mean is over the true
+// width; padded columns are zeros.
+#include "launchers.h"
+#include "proj.h"
+
+namespace dab {
+
+__device__ __forceinline__ float block_total(float v, float* red) {
+  v = wave_sum(v);
+  const int nw = blockDim.x >> 6;
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float t = 0.f;
+  for (int i = 0; i < nw; ++i) t += red[i];
+  return t;
+}
+
+struct RmsParams {
+  float* x;
+  void* h;
+  Proj y;                // sublayer output (p null: none)
+  const float* bias;     // [cols] or null
+  const void* pairs;     // [rows * top, cols] activation type, or null
+  int top;
+  const int* ids;        // with table: x += table[ids[row]]
+  const void* table;
+  const float* gain;     // null: no h
+  float inv_n, eps;
+  int rows, cols, fresh; // fresh: x starts at zero (embedding)
+};
+
+// one workgroup per row; a thread owns 8 columns at (tid + i blockDim) * 8, i < NV
+template <typename PT, typename AT, int NV>
+__global__ __launch_bounds__(256) void rms_residual_kernel(RmsParams p) {
+  __shared__ float red[4];
+  const int row = blockIdx.x;
+  float x[NV][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + i * blockDim.x) * 8;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[i][j] = 0.f;
+    if (c >= p.cols) continue;
+    float* xr = p.x + (size_t)row * p.cols + c;
+    if (!p.fresh) ElemIO<float>::load8(xr, x[i]);
+    if (p.y.p) {
+      float v[8];
+      proj8<PT>(p.y, row, c, v);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[i][j] += v[j];
+    }
+    if (p.bias) {
+      float v[8];
+      ElemIO<float>::load8(p.bias + c, v);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[i][j] += v[j];
+    }
+    if (p.pairs) {
+      const AT* q = (const AT*)p.pairs + (size_t)row * p.top * p.cols + c;
+      for (int k = 0; k < p.top; ++k) {
+        float v[8];
+        ElemIO<AT>::load8(q + (size_t)k * p.cols, v);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[i][j] += v[j];
+      }
+    }
+    if (p.table) {
+      float v[8];
+      ElemIO<AT>::load8((const AT*)p.table + (size_t)p.ids[row] * p.cols + c, v);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[i][j] += v[j];
+    }
+    ElemIO<float>::store8(xr, x[i]);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ss = fmaf(x[i][j], x[i][j], ss);
+  }
+  if (!p.gain) return;
+  const float r = 1.f / sqrtf(block_total(ss, red) * p.inv_n + p.eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + i * blockDim.x) * 8;
+    if (c >= p.cols) continue;
+    float g[8];
+    ElemIO<float>::load8(p.gain + c, g);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) g[j] *= x[i][j] * r;
+    ElemIO<AT>::store8((AT*)p.h + (size_t)row * p.cols + c, g);
+  }
+}
+
+int rms_residual(float* x, void* h, int act_f32, Proj y, const float* bias, const void* pairs, int top, const int* ids,
+                 const void* table, const float* gain, int n_true, float eps, int rows, int cols, int fresh,
+                 hipStream_t s) {
+  if (rows <= 0) return 0;
+  if (cols <= 0 || cols % 8 || cols > 16384 || !x || (gain && !h) || n_true < 1 || (pairs && top < 1) ||
+      (table && !ids) || (y.p && (y.S < 1 || y.ld % 8)))
+    return hipErrorInvalidValue;
+  const int nv8 = cols / 8;
+  const int bt = nv8 >= 256 ? 256 : (nv8 + 63) / 64 * 64;
+  const int nv = (nv8 + bt - 1) / bt;
+  RmsParams p{x, h, y, bias, pairs, top, ids, table, gain, 1.f / n_true, eps, rows, cols, fresh};
+  if (!y.p) p.y.f32 = act_f32;
+#define RMS_NV(PT, AT)                                                                                                 \
+  do {                                                                                                                 \
+    if (nv <= 1) hipLaunchKernelGGL((rms_residual_kernel<PT, AT, 1>), dim3(rows), dim3(bt), 0, s, p);                  \
+    else if (nv <= 2) hipLaunchKernelGGL((rms_residual_kernel<PT, AT, 2>), dim3(rows), dim3(bt), 0, s, p);             \
+    else if (nv <= 4) hipLaunchKernelGGL((rms_residual_kernel<PT, AT, 4>), dim3(rows), dim3(bt), 0, s, p);             \
+    else hipLaunchKernelGGL((rms_residual_kernel<PT, AT, 8>), dim3(rows), dim3(bt), 0, s, p);                          \
+  } while (0)
+  DAB_PROJ_DISPATCH(p.y, act_f32, RMS_NV);
+#undef RMS_NV
+  return hipGetLastError();
+}
+
+// ----------------------------------------------------------------------------------------------
+
+struct RopeParams {
+  Proj y;
+  int col0;              // q heads, then k heads, then v heads from this column, D columns each
+  int H, G, D;           // D: padded head width
+  int dim;               // true query / key width (RMS statistic)
+  int rot;               // rotated dimensions (even)
+  const double* freq;    // [rot / 2]
+  float inv_dim, eps;
+  int norm;              // 1: q and k over their root mean square
+  const int* positions;
+  const int64_t* slots;
+  void* q;               // [T, H, D]
+  void* kc;              // [blocks, G, bs, D]
+  void* vc;
+  int bs, T;
+};
+
+// one workgroup per token; a wave walks heads, a lane owns the pairs 2 (lane + 64 i), i < NP.  The angle
+// p * f is formed in fp64 and reduced to a half turn before the fp32 sine and cosine, so it is exact to
+// fp32 rounding at any position.
+template <typename PT, typename AT, int NP>
+__global__ __launch_bounds__(256) void qk_rope_kernel(RopeParams p) {
+  const int t = blockIdx.x, w = threadIdx.x >> 6, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+  const int64_t slot = p.slots[t];
+  const double pos = (double)p.positions[t];
+  float cs[NP], sn[NP];
+#pragma unroll
+  for (int i = 0; i < NP; ++i) {
+    const int pr = lane + 64 * i;
+    cs[i] = 1.f;
+    sn[i] = 0.f;
+    if (2 * pr < p.rot) {
+      const double turns = pos * p.freq[pr];
+      const float a = (float)((turns - rint(turns)) * 6.283185307179586476925);
+      sincosf(a, &sn[i], &cs[i]);
+    }
+  }
+  const size_t blk = slot >= 0 ? (size_t)(slot / p.bs) : 0, off = slot >= 0 ? (size_t)(slot % p.bs) : 0;
+  for (int hd = w; hd < p.H + 2 * p.G; hd += nw) {
+    const bool is_v = hd >= p.H + p.G;
+    float u[NP], v[NP], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NP; ++i) {
+      const int d = 2 * (lane + 64 * i);
+      u[i] = v[i] = 0.f;
+      if (d >= p.D) continue;
+      const PT* s = (const PT*)p.y.p + (size_t)t * p.y.ld + p.col0 + (size_t)hd * p.D + d;
+      for (int k = 0; k < p.y.S; ++k, s += p.y.slab) {
+        const float2 e = ElemIO<PT>::load2(s);
+        u[i] += e.x;
+        v[i] += e.y;
+      }
+      u[i] = ElemIO<AT>::round(u[i]);
+      v[i] = ElemIO<AT>::round(v[i]);
+      if (!is_v) {
+        const float a = u[i] * cs[i] - v[i] * sn[i], b = v[i] * cs[i] + u[i] * sn[i];
+        u[i] = a;
+        v[i] = b;
+        ss += a * a + b * b;
+      }
+    }
+    float r = 1.f;
+    if (!is_v && p.norm) r = 1.f / sqrtf(wave_sum(ss) * p.inv_dim + p.eps);
+    AT* dst;
+    if (hd < p.H) dst = (AT*)p.q + ((size_t)t * p.H + hd) * p.D;
+    else if (slot < 0) continue;
+    else {
+      const int gk = is_v ? hd - p.H - p.G : hd - p.H;
+      dst = (AT*)(is_v ? p.vc : p.kc) + ((blk * p.G + gk) * p.bs + off) * p.D;
+    }
+#pragma unroll
+    for (int i = 0; i < NP; ++i) {
+      const int d = 2 * (lane + 64 * i);
+      if (d >= p.D) continue;
+      ElemIO<AT>::store2(dst + d, u[i] * r, v[i] * r);
+    }
+  }
+}
+
+int qk_rope_write(Proj y, int col0, int H, int G, int D, int dim, int rot, const double* freq, float eps, int norm,
+                  const int* positions, const int64_t* slots, void* q, void* kc, void* vc, int act_f32, int bs, int T,
+                  hipStream_t s) {
+  if (T <= 0) return 0;
+  if (H < 1 || G < 1 || D < 2 || D % 2 || D > 1024 || dim < 1 || dim > D || rot % 2 || rot > dim || rot < 0 || bs < 1 ||
+      (rot && !freq) || y.S < 1)
+    return hipErrorInvalidValue;
+  RopeParams p{y, col0, H, G, D, dim, rot, freq, 1.f / dim, eps, norm, positions, slots, q, kc, vc, bs, T};
+#define ROPE_NP(PT, AT)                                                                                      \
+  do {                                                                                                       \
+    if (D <= 128) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 1>), dim3(T), dim3(256), 0, s, p);              \
+    else if (D <= 256) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 2>), dim3(T), dim3(256), 0, s, p);         \
+    else hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 8>), dim3(T), dim3(256), 0, s, p);                       \
+  } while (0)
+  DAB_PROJ_DISPATCH(y, act_f32, ROPE_NP);
+#undef ROPE_NP
+  return hipGetLastError();
+}
+
+}  // namespace dab

@@ -39,7 +39,7 @@ struct StreamParams {
   long ldw;
   void* out;
   long ldo;
-  const bf16* residual;
+  const bf16* residual;   // GLU over 8-row groups: fp32 bias [gate N / 2 | up N / 2] instead, or null
   long ldr;
   int M, N, K, S, kc;
   int epi;       // 0 none, 2 swiglu (16-row gate | up groups), 4 / 6 swiglu / tanh-gelu glu (8-row groups), 8 candidates
@@ -398,7 +398,12 @@ __global__ __launch_bounds__(64 * (NWC + NL), 1) void stream_gemm_kernel(StreamP
       const int m = e / (BN / 8), part = e % (BN / 8);
       if (m >= p.M) continue;
       const int i = part / pp, j0 = (part % pp) * 4;
-      const f32x4 gt = tile4(m, 2 * hg * i + j0), up = tile4(m, 2 * hg * i + hg + j0);
+      f32x4 gt = tile4(m, 2 * hg * i + j0), up = tile4(m, 2 * hg * i + hg + j0);
+      if (p.residual) {
+        const float* fb = reinterpret_cast<const float*>(p.residual) + n0 / 2 + hg * i + j0;
+        gt += *reinterpret_cast<const f32x4*>(fb);
+        up += *reinterpret_cast<const f32x4*>(fb + p.N / 2);
+      }
       float o[4];
 #pragma unroll
       for (int j = 0; j < 4; ++j) o[j] = (p.epi == ST_EPI_GEGLU8 ? gelu_tanh_f(gt[j]) : silu_f(gt[j])) * up[j];
@@ -545,7 +550,7 @@ int stream_gemm(const void* X, long ldx, const void* W, long ldw, void* out, lon
     return hipErrorInvalidValue;
   if (epilogue == ST_EPI_SWIGLU && bn % 32) return hipErrorInvalidValue;  // whole 16 + 16 row pairs per tile
   if (S > 1 && (epilogue != ST_EPI_NONE || residual)) return hipErrorInvalidValue;
-  if (residual && ldr % 8) return hipErrorInvalidValue;
+  if (residual && (ldr % 8 || epilogue == ST_EPI_SWIGLU)) return hipErrorInvalidValue;
   if ((long)bn * ldw * 2 >= (1L << 31)) return hipErrorInvalidValue;  // buffer descriptor range
   if (kStreamCfgs[cfg].shuf && (ldw != K || K % 32)) return hipErrorInvalidValue;
   StreamParams p{};

@@ -7,8 +7,11 @@
 
 namespace dab {
 
-KVBlockManager::KVBlockManager(int num_blocks, int block_size, bool prefix_cache)
-    : num_blocks_(num_blocks), block_size_(block_size), prefix_cache_(prefix_cache) {
+KVBlockManager::KVBlockManager(int num_blocks, int block_size, bool prefix_cache, int state_slots)
+    : num_blocks_(num_blocks), block_size_(block_size), prefix_cache_(prefix_cache), n_slots_(state_slots) {
+  if (state_slots < 0 || (state_slots > 0 && prefix_cache))
+    throw std::invalid_argument("state slots exclude prefix reuse");
+  for (int i = 0; i < state_slots; ++i) free_slots_.push_back(i);
   if (num_blocks <= 0 || block_size <= 0) throw std::invalid_argument("num_blocks and block_size must be > 0");
   free_.reserve(num_blocks);
   for (int b = 0; b < num_blocks; ++b) free_.push_back(b);  // ascending = a valid min-heap
@@ -96,7 +99,13 @@ int KVBlockManager::add_sequence(int64_t seq_id, const std::vector<int32_t>& tok
   for (int32_t b : hit_blocks) reused_from_lru += in_lru_[b] ? 1 : 0;
   const int fresh = need_blocks - (int)hit_blocks.size();
   if (fresh > num_free_blocks() - reused_from_lru) return -1;
+  if (n_slots_ > 0 && free_slots_.empty()) return -1;
   Seq s;
+  if (n_slots_ > 0) {
+    std::pop_heap(free_slots_.begin(), free_slots_.end(), std::greater<int32_t>());
+    s.slot = free_slots_.back();
+    free_slots_.pop_back();
+  }
   for (int32_t b : hit_blocks) {
     if (in_lru_[b]) {
       lru_.erase(lru_pos_[b]);
@@ -157,6 +166,10 @@ void KVBlockManager::free_sequence(int64_t seq_id) {
   auto it = seqs_.find(seq_id);
   if (it == seqs_.end()) return;
   for (int32_t b : it->second.blocks) release_block(b);
+  if (it->second.slot >= 0) {
+    free_slots_.push_back(it->second.slot);
+    std::push_heap(free_slots_.begin(), free_slots_.end(), std::greater<int32_t>());
+  }
   seqs_.erase(it);
 }
 
@@ -174,6 +187,14 @@ const std::vector<int32_t>& KVBlockManager::blocks(int64_t seq_id) const {
   auto it = seqs_.find(seq_id);
   if (it == seqs_.end()) throw std::invalid_argument("unknown sequence");
   return it->second.blocks;
+}
+
+void KVBlockManager::state_slots(const std::vector<int64_t>& seq_ids, int32_t* out) const {
+  for (size_t i = 0; i < seq_ids.size(); ++i) {
+    auto it = seqs_.find(seq_ids[i]);
+    if (it == seqs_.end()) throw std::invalid_argument("unknown sequence");
+    out[i] = it->second.slot;
+  }
 }
 
 void KVBlockManager::slot_mapping(int64_t seq_id, int start, int n, int64_t* out) const {

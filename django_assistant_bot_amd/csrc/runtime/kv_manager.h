@@ -11,6 +11,10 @@
 // out lowest id first (a min-heap), so the live blocks of a batch stay packed at the low end of the
 // pool: decode attention reads every live block each step, and scattered over an engine-sized pool
 // (24k blocks) they streamed ~3 % slower than packed (profiles/decode_round2.md).
+//
+// Models with recurrent layers also need one state slot per live sequence (``state_slots`` > 0): a sequence
+// takes the lowest free slot when it is admitted and gives it back with its blocks.  A slot holds the state
+// of the whole prefix, so block-wise prefix reuse is off for such models.
 #pragma once
 #include <cstdint>
 #include <list>
@@ -21,10 +25,10 @@ namespace dab {
 
 class KVBlockManager {
  public:
-  KVBlockManager(int num_blocks, int block_size, bool prefix_cache);
+  KVBlockManager(int num_blocks, int block_size, bool prefix_cache, int state_slots = 0);
 
   // Admits a sequence: reuses cached prefix blocks, allocates blocks for len(tokens)+reserve.
-  // Returns the number of prompt tokens whose KV is already cached, or -1 if blocks are short
+  // Returns the number of prompt tokens whose KV is already cached, or -1 if blocks (or state slots) are short
   // (nothing is allocated in that case).
   int add_sequence(int64_t seq_id, const std::vector<int32_t>& tokens, int reserve);
   // Makes room for `n` more tokens at the end of the sequence; false if out of blocks.
@@ -43,6 +47,9 @@ class KVBlockManager {
   int block_size() const { return block_size_; }
   int64_t prefix_hits() const { return prefix_hits_; }
   const std::vector<int32_t>& blocks(int64_t seq_id) const;
+  int num_free_state_slots() const { return (int)free_slots_.size(); }
+  // state slot of every sequence (-1: the manager hands out none)
+  void state_slots(const std::vector<int64_t>& seq_ids, int32_t* out) const;
 
   // One decode step for a batch: reserves one slot per sequence (returns the index of the first
   // sequence that cannot get a block, nothing appended then), else appends each sequence's last
@@ -59,10 +66,13 @@ class KVBlockManager {
     std::vector<int32_t> blocks;
     std::vector<int32_t> tokens;
     std::vector<uint64_t> hashes;  // chained hash of each registered full block
+    int32_t slot = -1;             // state slot
   };
   int num_blocks_, block_size_;
   bool prefix_cache_;
+  int n_slots_;
   std::vector<int32_t> free_;  // min-heap (std::greater)
+  std::vector<int32_t> free_slots_;  // min-heap
   int lru_cap_ = 64;
   std::vector<int32_t> ref_;
   std::vector<uint64_t> block_hash_;  // 0 = not registered

@@ -96,6 +96,30 @@ static void test_kv_manager(unsigned seed) {
   CHECK(m.num_free_blocks() == NB, "blocks not returned: %d of %d", m.num_free_blocks(), NB);
 }
 
+static void test_state_slots() {
+  dab::KVBlockManager m(64, 16, false, 3);
+  std::map<int64_t, int32_t> live;
+  std::mt19937 rng(5);
+  for (int64_t id = 0; id < 500; ++id) {
+    if (m.add_sequence(id, std::vector<int32_t>(1 + rng() % 40, 1), 0) < 0) {
+      CHECK(live.size() == 3, "admission refused with %zu live", live.size());
+    } else {
+      int32_t slot = -1;
+      m.state_slots({id}, &slot);
+      CHECK(slot >= 0 && slot < 3, "slot %d", slot);
+      for (auto& kv : live) CHECK(kv.second != slot, "slot %d used twice", slot);
+      live[id] = slot;
+    }
+    if (live.size() == 3 || (rng() & 1)) {
+      auto itr = live.begin();
+      std::advance(itr, rng() % live.size());
+      m.free_sequence(itr->first);
+      live.erase(itr);
+    }
+    CHECK(m.num_free_state_slots() == 3 - (int)live.size(), "slots leaked");
+  }
+}
+
 static void test_tokenizer() {
   dab::TokenizerConfig cfg;
   dab::HashTokenizer tok(cfg);
@@ -179,6 +203,7 @@ static void test_rag() {
 
 int main() {
   for (unsigned seed = 1; seed <= 4; ++seed) test_kv_manager(seed);
+  test_state_slots();
   test_tokenizer();
   test_rag();
   dab::trace::range_push("selftest");  // no-op or real: must not crash either way

@@ -31,7 +31,7 @@ import torch
 
 from .. import ops
 from ..models import AttnMeta, decoder_config, decoder_family
-from ..models.configs import DecoderConfig, VumuvikConfig
+from ..models.configs import DecoderConfig, VugotarConfig, VumuvikConfig
 from ..ops._lib import native
 from ..utils import trace
 from .tokenizer import Tokenizer
@@ -106,7 +106,8 @@ def _bucket_sizes(max_batch):
 
 
 class LLMEngine:
-    def __init__(self, model: str | DecoderConfig | VumuvikConfig = "llama-3-8b", device=None, weights: dict | None = None,
+    def __init__(self, model: str | DecoderConfig | VumuvikConfig | VugotarConfig = "llama-3-8b",
+                 device=None, weights: dict | None = None,
                  checkpoint: str | None = None, seed: int = 0, max_batch: int = 256, block_size: int = 64,
                  max_model_len: int | None = None, kv_cache_gb: float | None = None, num_blocks: int | None = None,
                  max_prefill_tokens: int = 16384, use_graphs: bool = True, prefix_cache: bool = True,
@@ -160,17 +161,22 @@ class LLMEngine:
         self.mixed_prefill_tokens = mixed_prefill_tokens
         self.part_size = part_size
         per_block = self.model.cache_bytes_per_block(block_size)
+        # recurrent layers: a state slot per live sequence and one more for padded decode rows; a slot holds the whole
+        # prefix, so there is no block-wise prefix reuse
+        self.recurrent = self.model.recurrent
+        self.state_slots = max_batch if self.recurrent else 0
+        prefix_cache = prefix_cache and not self.recurrent
         if num_blocks is None:
             if kv_cache_gb:
-                num_blocks = int(kv_cache_gb * (1 << 30) // per_block)
+                num_blocks = int(max(0, kv_cache_gb * (1 << 30) - self.model.state_bytes(self.state_slots + 1)) // per_block)
             elif self.is_gpu:
                 free, _ = torch.cuda.mem_get_info(self.device)
-                num_blocks = int(free * kv_memory_fraction // per_block)
+                num_blocks = int(max(0, free * kv_memory_fraction - self.model.state_bytes(self.state_slots + 1)) // per_block)
             else:
                 num_blocks = 4 * self.max_blocks_per_seq
             num_blocks = max(2, min(num_blocks, max_batch * self.max_blocks_per_seq + 8))
-        self.kv = self.model.make_cache(num_blocks, block_size)
-        self.blocks = native().KVBlockManager(num_blocks, block_size, prefix_cache)
+        self.kv = self.model.make_cache(num_blocks, block_size, self.state_slots + 1)
+        self.blocks = native().KVBlockManager(num_blocks, block_size, prefix_cache, self.state_slots)
         self._prefix_cache = prefix_cache
         self.seed = seed
         self.waiting: deque[_Req] = deque()
@@ -195,6 +201,7 @@ class LLMEngine:
         self._d_cnt = torch.zeros(mb, dtype=torch.int64, device=dev)
         self._d_tokens = torch.zeros(mb, dtype=torch.int32, device=dev)
         self._d_order = torch.arange(mb, dtype=torch.int32, device=dev)  # decode attention dispatch order
+        self._d_state = torch.full((mb,), self.state_slots, dtype=torch.int32, device=dev)  # recurrent state slots
         pin = self.is_gpu
         mk = lambda *a, **k: torch.zeros(*a, **k, pin_memory=pin)  # noqa: E731
         self._h_ids = mk(mb, dtype=torch.int32)
@@ -208,6 +215,7 @@ class LLMEngine:
         self._h_cnt = mk(mb, dtype=torch.int64)
         self._h_tokens = mk(mb, dtype=torch.int32)
         self._h_order = mk(mb, dtype=torch.int32)
+        self._h_state = mk(mb, dtype=torch.int32)
         # pipelined decode (``_step_pipelined``): step t+1 is launched before step t's tokens are read,
         # its input ids copied on the device from step t's sampled tokens, so the host's per-step
         # bookkeeping overlaps the GPU instead of idling it.  Two alternating host buffer sets: the
@@ -215,7 +223,7 @@ class LLMEngine:
         self.pipeline_decode = bool(pipeline_decode) and tp_size == 1
         self._h_alt = {k: mk(*(getattr(self, k).shape,), dtype=getattr(self, k).dtype)
                        for k in ("_h_ids", "_h_pos", "_h_slots", "_h_ctx", "_h_bt", "_h_temp", "_h_topk", "_h_topp",
-                                 "_h_cnt", "_h_tokens", "_h_order")}
+                                 "_h_cnt", "_h_tokens", "_h_order", "_h_state")}
         self._inflight = None  # launched decode step whose tokens are not consumed yet
         self._d_mask = None  # JSON-constrained decoding buffers (allocated on first use)
         self._masked = False
@@ -402,7 +410,7 @@ class LLMEngine:
         self.waiting.clear()
         self.prefilling.clear()
         self.running.clear()
-        self.blocks = native().KVBlockManager(self.blocks.num_blocks(), self.block_size, self._prefix_cache)
+        self.blocks = native().KVBlockManager(self.blocks.num_blocks(), self.block_size, self._prefix_cache, self.state_slots)
         self.timer.collect()
         return ids
 
@@ -455,6 +463,7 @@ class LLMEngine:
                     self._h_ids.data_ptr(), self._h_pos.data_ptr(), self._h_slots.data_ptr(), self._h_ctx.data_ptr(),
                     self._h_bt.data_ptr()) >= 0:
                 raise RuntimeError("cache exhausted")
+            self._fill_state([entries[e][0] for e in rows])
             for e in rows:
                 self._fed[entries[e][0]] += 1
         row0 = {}  # entry -> its first row of the step
@@ -503,7 +512,7 @@ class LLMEngine:
         for d, h in ((self._d_ids, self._h_ids), (self._d_pos, self._h_pos), (self._d_slots, self._h_slots),
                      (self._d_ctx, self._h_ctx), (self._d_temp, self._h_temp), (self._d_topk, self._h_topk),
                      (self._d_topp, self._h_topp), (self._d_cnt, self._h_cnt), (self._d_order, self._h_order),
-                     (self._d_bt, self._h_bt)):
+                     (self._d_bt, self._h_bt), (self._d_state, self._h_state)):
             d[:Bp].copy_(h[:Bp], non_blocking=True)
         key = (Bp, True, False)
         if self.use_graphs and (self._graphs.get(key) or self._capture(Bp)) is not None:
@@ -568,6 +577,19 @@ class LLMEngine:
         self._build_block_tables([c[0] for c in chunks], bt)
         return cu, ctx, bt
 
+    def _fill_state(self, seqs) -> None:
+        """Host: the state slots of the decode rows."""
+        if self.recurrent:
+            self.blocks.state_slots_into(seqs, self._h_state.data_ptr())
+
+    def _chunk_state(self, chunks):
+        """Device tensor of the prefill chunks' state slots (None without recurrent layers)."""
+        if not self.recurrent:
+            return None
+        st = torch.empty(len(chunks), dtype=torch.int32)
+        self.blocks.state_slots_into([c[0] for c in chunks], st.data_ptr())
+        return self._h2d(st)
+
     def _prefill_inputs(self, chunks):
         """Packed prefill step: device ids, host cu_q, batch description."""
         T = sum(c[3] for c in chunks)
@@ -576,7 +598,8 @@ class LLMEngine:
         cu, ctx, bt = self._fill_chunks(chunks, ids, pos, slots)
         to = self._h2d
         meta = AttnMeta(decode=False, positions=to(pos), slots=to(slots), block_tables=to(bt), ctx_lens=to(ctx),
-                        cu_q=to(cu), max_q=max(c[3] for c in chunks), chunk_lens=[(c[3], c[2] + c[3]) for c in chunks])
+                        cu_q=to(cu), max_q=max(c[3] for c in chunks), chunk_lens=[(c[3], c[2] + c[3]) for c in chunks],
+                        state_slots=self._chunk_state(chunks))
         return to(ids), cu, meta
 
     def _run_prefill(self, chunks):
@@ -658,6 +681,7 @@ class LLMEngine:
         to = lambda a: torch.as_tensor(a).to(dev, non_blocking=True)  # noqa: E731
         self._d_ctx[:Bp].copy_(self._h_ctx[:Bp], non_blocking=True)
         self._d_bt[:Bp].copy_(self._h_bt[:Bp], non_blocking=True)
+        self._d_state[:Bp].copy_(self._h_state[:Bp], non_blocking=True)
         order = None
         if self.is_gpu:  # longest first: the decode attention stops at the longest context's partitions
             self._fill_order(Bp)
@@ -667,17 +691,19 @@ class LLMEngine:
                         cu_q=to(cu), max_q=max(c[3] for c in chunks), workspace=self._workspace,
                         part_size=self._decode_part(Bp), n_decode=Bp, dec_block_tables=self._d_bt[:Bp],
                         dec_ctx_lens=self._d_ctx[:Bp], order=order,
-                        chunk_lens=[(c[3], c[2] + c[3]) for c in chunks], max_len=self.max_model_len)
+                        chunk_lens=[(c[3], c[2] + c[3]) for c in chunks], max_len=self.max_model_len,
+                        state_slots=self._chunk_state(chunks), dec_state_slots=self._d_state[:Bp])
         return to(ids), cu, meta
 
     def _pad_decode_rows(self, B: int, Bp: int) -> None:
-        """Host decode rows B..Bp: no cache write, attend to one key of block 0, output ignored."""
+        """Host decode rows B..Bp: no cache write, attend to one key of block 0, the spare state slot, output ignored."""
         if Bp > B:
             self._h_ids[B:Bp] = 0
             self._h_pos[B:Bp] = 0
             self._h_slots[B:Bp] = -1
             self._h_ctx[B:Bp] = 1
             self._h_bt[B:Bp] = 0
+            self._h_state[B:Bp] = self.state_slots
 
     def _run_mixed(self, batch: list, chunks):
         """Prefill chunks + one decode token per running sequence in one forward (see ``step``)."""
@@ -919,6 +945,7 @@ class LLMEngine:
                 self._h_ids.data_ptr(), self._h_pos.data_ptr(), self._h_slots.data_ptr(), self._h_ctx.data_ptr(),
                 self._h_bt.data_ptr())
             if fail < 0:
+                self._fill_state([r.seq for r in nxt])
                 pos = {id(r): i for i, r in enumerate(prev["batch"])}
                 self._launch_decode(nxt, [pos[id(r)] for r in nxt], pending=1)
                 launched = True
@@ -952,7 +979,8 @@ class LLMEngine:
         self._fill_order(Bp)
         pairs = [(self._d_pos, self._h_pos), (self._d_slots, self._h_slots), (self._d_ctx, self._h_ctx),
                  (self._d_temp, self._h_temp), (self._d_topk, self._h_topk), (self._d_topp, self._h_topp),
-                 (self._d_cnt, self._h_cnt), (self._d_bt, self._h_bt), (self._d_order, self._h_order)]
+                 (self._d_cnt, self._h_cnt), (self._d_bt, self._h_bt), (self._d_order, self._h_order),
+                 (self._d_state, self._h_state)]
         if src_rows is None:
             pairs.append((self._d_ids, self._h_ids))
         else:
@@ -1023,6 +1051,7 @@ class LLMEngine:
                 self._h_ids.data_ptr(), self._h_pos.data_ptr(), self._h_slots.data_ptr(), self._h_ctx.data_ptr(),
                 self._h_bt.data_ptr())
             if fail < 0:
+                self._fill_state([r.seq for r in batch])
                 return batch
             if not self._preempt_one(protect=None if B == 1 else batch[fail]):
                 raise RuntimeError("KV cache exhausted")
@@ -1046,7 +1075,8 @@ class LLMEngine:
         self._fill_order(Bp)
         for d, h in ((self._d_ids, self._h_ids), (self._d_pos, self._h_pos), (self._d_slots, self._h_slots),
                      (self._d_ctx, self._h_ctx), (self._d_temp, self._h_temp), (self._d_topk, self._h_topk),
-                     (self._d_topp, self._h_topp), (self._d_cnt, self._h_cnt), (self._d_order, self._h_order)):
+                     (self._d_topp, self._h_topp), (self._d_cnt, self._h_cnt), (self._d_order, self._h_order),
+                     (self._d_state, self._h_state)):
             d[:Bp].copy_(h[:Bp], non_blocking=True)
         self._d_bt[:Bp].copy_(self._h_bt[:Bp], non_blocking=True)
         self._masked = self._fill_masks(batch, Bp)
@@ -1099,7 +1129,7 @@ class LLMEngine:
         meta = AttnMeta(decode=True, positions=self._d_pos[:Bp], slots=self._d_slots[:Bp],
                         block_tables=self._d_bt[:Bp], ctx_lens=self._d_ctx[:Bp], workspace=self._workspace,
                         part_size=self._decode_part(Bp), order=self._d_order[:Bp] if self.is_gpu else None,
-                        max_len=self.max_model_len)
+                        max_len=self.max_model_len, state_slots=self._d_state[:Bp] if self.recurrent else None)
         h = self.model.forward(self._d_ids[:Bp], meta, self.kv)
         logits = self._d_logits = self.model.logits(h)
         if self._masked:
@@ -1124,11 +1154,14 @@ class LLMEngine:
     def _capture(self, Bp: int):
         try:
             s = torch.cuda.Stream(self.device)
+            live = self._d_state[:Bp].clone()
+            self._d_state[:Bp] = self.state_slots  # a recurrence must not advance twice: warm up on the spare slot
             s.wait_stream(torch.cuda.current_stream(self.device))
             with torch.cuda.stream(s):
                 self._decode_body(Bp)  # warm-up (allocator, lazy init) outside the graph
             torch.cuda.current_stream(self.device).wait_stream(s)
             torch.cuda.synchronize(self.device)
+            self._d_state[:Bp].copy_(live)
             self._d_cnt[:Bp].copy_(self._h_cnt[:Bp])  # the warm-up advanced the RNG counters
             g = torch.cuda.CUDAGraph()
             if self._graph_pool is None:

@@ -1,6 +1,7 @@
-"""Model families: BERT-style sentence encoders, Llama-3-style decoders and latent-attention (Vumuvik) decoders."""
+"""Model families: BERT-style sentence encoders, Llama-3-style, latent-attention (Vumuvik) and hybrid (Vugotar)
+decoders."""
 from .bert import BertEncoder, pack_sequences  # noqa: F401
-from .cache import AttnMeta, KVCache, LatentCache  # noqa: F401
+from .cache import AttnMeta, HybridCache, KVCache, LatentCache  # noqa: F401
 from .configs import (  # noqa: F401
     DECODERS,
     ENCODERS,
@@ -8,6 +9,7 @@ from .configs import (  # noqa: F401
     EncoderConfig,
     LatentLayer,
     LatentMixer,
+    VugotarConfig,
     VumuvikConfig,
     decoder_config,
     encoder_config,
@@ -16,13 +18,16 @@ from .configs import (  # noqa: F401
 )
 from .llama import LlamaModel  # noqa: F401
 from .registry import DecoderFamily, decoder_family  # noqa: F401
+from .vugotar import VugotarModel  # noqa: F401
 from .vumuvik import VumuvikModel  # noqa: F401
 from .weights import (  # noqa: F401
     load_decoder_checkpoint,
     load_encoder_checkpoint,
+    load_vugotar_checkpoint,
     load_vumuvik_checkpoint,
     random_decoder_weights,
     random_encoder_weights,
+    random_vugotar_weights,
     random_vumuvik_weights,
     shard_decoder_weights,
 )

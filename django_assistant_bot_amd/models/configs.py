@@ -175,6 +175,187 @@ def vumuvik_uniform(name: str, layers: int, vocab_size: int, hidden: int, ff: in
     return VumuvikConfig(name, vocab_size, hidden, blocks, kw.pop("eps", 1e-6), kw.pop("embed_scale", hidden ** 0.5), **kw)
 
 
+# ------------------------------------------------------------------ hybrid decoders (Vugotar)
+
+
+@dataclass(frozen=True)
+class ChunkedMixer:
+    """Softmax attention inside chunks of positions, with a sink of score 0 in every head's denominator."""
+
+    heads: int
+    kv_heads: int
+    dim: int  # query / key width of a head
+    vdim: int
+    scale: float
+    chunk: int = 0  # positions of a chunk (0: one chunk)
+    rot_dims: int = 0  # rotated dimensions, interleaved pairs
+    rot_base: float = 10000.0
+
+
+@dataclass(frozen=True)
+class DeltaMixer:
+    """Gated delta rule: a dim x vdim state per head, q / k heads shared by groups of value heads."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int  # taps of the short convolution
+
+
+@dataclass(frozen=True)
+class ParallelMixer:
+    """Both mixers read the layer's input; the result is the scaled sum of their outputs."""
+
+    left: ChunkedMixer
+    right: DeltaMixer
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+
+
+@dataclass(frozen=True)
+class Mamba2Mixer:
+    """State-space duality: a state x vdim state per head, B / C shared by groups of heads."""
+
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    conv: int
+    norm_groups: int = 1
+
+
+@dataclass(frozen=True)
+class DenseMlp:
+    """SwiGLU with biases on all three projections."""
+
+    ff: int
+
+
+@dataclass(frozen=True)
+class MoeMlp:
+    """``top`` of ``experts`` SwiGLUs per token plus, with ``shared``, one that every token runs behind a sigmoid gate."""
+
+    experts: int
+    top: int
+    scale: float
+    ff: int
+    shared: int | None = None
+
+
+@dataclass(frozen=True)
+class HybridLayer:
+    """x + mixer(norm(x)) + mlp(norm(x)): one norm, both sublayers read its output."""
+
+    mixer: ParallelMixer | Mamba2Mixer
+    mlp: DenseMlp | MoeMlp | None = None
+
+
+@dataclass(frozen=True)
+class VugotarConfig:
+    """Vugotar decoder: hybrid layers, of which ``loop`` = (start, stop, times) runs a stretch several times with the
+    same weights (every pass with its own cache and state; the embedding is added again before each pass but the
+    first).  The ``padded_*`` sizes are what the kernels see; padding is zeros."""
+
+    name: str
+    vocab_size: int
+    hidden: int
+    blocks: tuple  # of HybridLayer
+    eps: float = 1e-5
+    loop: tuple | None = None
+    max_position: int = 1 << 20  # no positional table: only the cache bounds a sequence
+    default_model_len: int = 8192
+    bos_id: int = 0
+    eos_ids: tuple = ()
+
+    MAX_STATE_ROWS, MAX_TAPS, MAX_HEAD, MAX_EXPERTS, MAX_TOP = 256, 16, 1024, 1024, 64  # of the kernels
+
+    def __post_init__(self):
+        for i, b in enumerate(self.blocks):
+            where = f"{self.name}: layer {i}"
+            m, f = b.mixer, b.mlp
+            if isinstance(m, ParallelMixer):
+                a, d = m.left, m.right
+                if a.heads % a.kv_heads or d.heads % d.kv_heads:
+                    raise ValueError(f"{where}: heads must be whole groups of kv_heads")
+                if a.rot_dims % 2 or a.rot_dims > a.dim or max(a.dim, a.vdim) > self.MAX_HEAD:
+                    raise ValueError(f"{where}: rotated dimensions or head width")
+                rows, taps = d.dim, d.conv
+            else:
+                if m.heads % m.groups or (m.heads * m.vdim) % m.norm_groups:
+                    raise ValueError(f"{where}: heads must be whole groups, channels whole norm groups")
+                rows, taps = m.state, m.conv
+            if not 1 <= rows <= self.MAX_STATE_ROWS or not 1 <= taps <= self.MAX_TAPS:
+                raise ValueError(f"{where}: state rows up to {self.MAX_STATE_ROWS}, taps up to {self.MAX_TAPS}")
+            if isinstance(f, MoeMlp) and not 1 <= f.top <= min(f.experts, self.MAX_TOP) or (
+                    isinstance(f, MoeMlp) and f.experts > self.MAX_EXPERTS):
+                raise ValueError(f"{where}: experts up to {self.MAX_EXPERTS}, of which up to {self.MAX_TOP} per token")
+        if self.loop is not None:
+            a, b, t = self.loop
+            if not 0 <= a <= b <= len(self.blocks) or t < 1:
+                raise ValueError(f"{self.name}: loop {self.loop} outside the layers")
+
+    @property
+    def layers(self) -> int:
+        return len(self.blocks)
+
+    def runs(self) -> list:
+        """(layer, embedding added before it) of every layer run, in order."""
+        a, b, t = self.loop or (0, 0, 1)
+        if a == b:
+            return [(i, False) for i in range(self.layers)]
+        return ([(i, False) for i in range(a)]
+                + [(i, k > 0 and i == a) for k in range(t) for i in range(a, b)]
+                + [(i, False) for i in range(b, self.layers)])
+
+    @property
+    def padded_hidden(self) -> int:
+        return _up(self.hidden, 128)
+
+    @property
+    def padded_vocab(self) -> int:
+        return _up(self.vocab_size, 128)
+
+    @staticmethod
+    def padded_head(m: ChunkedMixer) -> int:
+        """Common padded width of the query / key and value heads."""
+        d = max(m.dim, m.vdim)
+        return next((p for p in (64, 128, 256) if d <= p), _up(d, 64))
+
+    def to_dict(self):
+        return asdict(self)
+
+    def params(self) -> int:
+        W = self.hidden
+        n = 2 * self.vocab_size * W + W
+        for b in self.blocks:
+            m, f = b.mixer, b.mlp
+            n += W
+            if isinstance(m, ParallelMixer):
+                a, d = m.left, m.right
+                n += W * (a.heads * (a.dim + a.vdim) + a.kv_heads * (a.dim + a.vdim))
+                c, v = 2 * d.kv_heads * d.dim + d.heads * d.vdim, d.heads * d.vdim
+                n += W * (c + 2 * v + 2 * d.heads) + c * d.conv + 2 * d.heads + d.vdim
+            else:
+                inner = m.heads * m.vdim
+                c = inner + 2 * m.groups * m.state
+                n += W * (2 * inner + c + m.heads) + c * (m.conv + 1) + 3 * m.heads + inner
+            if isinstance(f, DenseMlp):
+                n += 3 * W * f.ff + 2 * f.ff + W
+            elif f is not None:
+                n += f.experts * (3 * W * f.ff + W) + (3 * W * f.shared + W if f.shared else 0)
+        return n
+
+
+def vugotar_uniform(name: str, layers: int, vocab_size: int, hidden: int, left: ChunkedMixer, right: DeltaMixer,
+                    mamba: Mamba2Mixer, dense: DenseMlp, moe: MoeMlp | None, loop: tuple | None = None, **kw) -> VugotarConfig:
+    """A Vugotar whose layers repeat (mamba2 + dense, parallel + experts, parallel + dense); without ``moe`` every MLP is
+    dense."""
+    par = ParallelMixer(left, right, 0.5, 0.5)
+    cycle = (HybridLayer(mamba, dense), HybridLayer(par, moe or dense), HybridLayer(par, dense))
+    return VugotarConfig(name, vocab_size, hidden, tuple(cycle[i % 3] for i in range(layers)), loop=loop, **kw)
+
+
 ENCODERS = {
     "bge-base-en": EncoderConfig("bge-base-en"),
     "bge-large-en": EncoderConfig("bge-large-en", hidden=1024, layers=24, heads=16, intermediate=4096),
@@ -220,6 +401,25 @@ DECODERS.update({
         LatentLayer(LatentMixer(3, 64, 64, 80, 0.11, 33, kv_from=0), 200),
         LatentLayer(LatentMixer(5, 32, 56, 48, 0.2, 0), None),
         LatentLayer(LatentMixer(2, 40, 24, 48, 0.15, 128, kv_from=2), 256)), 1e-5, 11.0, max_position=2048),
+})
+
+DECODERS.update({
+    # Llama-3-8B's width, MLP, vocabulary and KV heads; 2048-token chunks; a 128 x 128 state per head
+    "vugotar-8b": vugotar_uniform(
+        "vugotar-8b", 24, 128256, 4096, ChunkedMixer(32, 8, 128, 128, 128 ** -0.5, 2048, 64, 500000.0),
+        DeltaMixer(16, 8, 128, 128, 4), Mamba2Mixer(64, 64, 128, 8, 4, 8), DenseMlp(14336), None),
+    # ... and with experts: 64 of 512, 6 per token, at Llama-3.2-1B's width
+    "vugotar-moe": vugotar_uniform(
+        "vugotar-moe", 15, 128256, 2048, ChunkedMixer(16, 4, 128, 128, 128 ** -0.5, 1024, 128, 500000.0),
+        DeltaMixer(16, 8, 128, 128, 4), Mamba2Mixer(64, 64, 128, 8, 4, 8), DenseMlp(8192),
+        MoeMlp(64, 6, 2.0, 1024, 2048)),
+    # test size: every branch at unequal sizes
+    "tiny-vugotar": VugotarConfig("tiny-vugotar", 1000, 200, (
+        HybridLayer(Mamba2Mixer(6, 24, 40, 3, 3, 4), DenseMlp(168)),
+        HybridLayer(ParallelMixer(ChunkedMixer(6, 2, 48, 40, 0.15, 70, 32, 5000.0), DeltaMixer(6, 2, 40, 24, 4), 0.7, 0.4),
+                    MoeMlp(12, 3, 1.7, 40, 72)),
+        HybridLayer(ParallelMixer(ChunkedMixer(3, 3, 64, 64, 0.12, 0, 64), DeltaMixer(2, 2, 64, 64, 2)), None),
+        HybridLayer(Mamba2Mixer(2, 64, 64, 1, 4, 1), MoeMlp(5, 1, 1.0, 24))), 1e-5, loop=(1, 3, 2), max_position=2048),
 })
 
 _ALIASES = {
@@ -338,16 +538,55 @@ def vumuvik_config_from_dir(path: str) -> VumuvikConfig:
                          float(c["embedding"]["scale"]))
 
 
+def vugotar_config_from_dir(path: str) -> VugotarConfig:
+    """config.json of a Vugotar checkpoint: ``architecture``, ``vocab``, ``width``, ``norm.eps``, ``loop`` (or none) and
+    ``layers`` (each ``type``, ``mixer`` sizes and ``mlp`` or null)."""
+    c = _hf(path)
+    blocks = []
+    for i, L in enumerate(c["layers"]):
+        m, f = L["mixer"], L.get("mlp")
+        if L.get("type") == "parallel":
+            a, d = m["left"], m["right"]
+            rot = a.get("rot") or {}
+            mixer = ParallelMixer(
+                ChunkedMixer(int(a["heads"]), int(a["kv_heads"]), int(a["dim"]), int(a["vdim"]), float(a["scale"]),
+                             int((a.get("mask") or {}).get("size") or 0), int(rot.get("dims") or 0),
+                             float(rot.get("base", 10000.0))),
+                DeltaMixer(int(d["heads"]), int(d["kv_heads"]), int(d["dim"]), int(d["vdim"]), int(d["conv"])),
+                float(m["left_scale"]), float(m["right_scale"]))
+        elif L.get("type") == "mamba2":
+            mixer = Mamba2Mixer(int(m["heads"]), int(m["vdim"]), int(m["state"]), int(m["groups"]), int(m["conv"]),
+                                int(m["norm_groups"]))
+        else:
+            raise ValueError(f"{path}: layer {i}: mixer type {L.get('type')!r} is not supported (parallel, mamba2)")
+        if f is None:
+            mlp = None
+        elif f.get("kind") == "dense":
+            mlp = DenseMlp(int(f["ff"]))
+        elif f.get("kind") == "moe":
+            r, sh = f["router"], f.get("shared")
+            mlp = MoeMlp(int(r["experts"]), int(r["top"]), float(r["scale"]), int(f["expert"]["ff"]),
+                         None if sh is None else int(sh["ff"]))
+        else:
+            raise ValueError(f"{path}: layer {i}: mlp kind {f.get('kind')!r} is not supported (dense, moe or null)")
+        blocks.append(HybridLayer(mixer, mlp))
+    lp = c.get("loop")
+    loop = None if lp is None else (int(lp["start"]), int(lp["stop"]), int(lp["times"]))
+    return VugotarConfig(_label(path), int(c["vocab"]), int(c["width"]), tuple(blocks), float(c["norm"]["eps"]), loop)
+
+
+_DIR_CONFIGS = {"vumuvik": vumuvik_config_from_dir, "vugotar": vugotar_config_from_dir}
+
+
 def _dir_architecture(path: str) -> str | None:
     c = _hf(path)
-    if c.get("architecture") == "Vumuvik":
-        return "vumuvik"
-    return c.get("model_type")
+    arch = str(c.get("architecture")).lower()
+    return arch if arch in _DIR_CONFIGS else c.get("model_type")
 
 
-def decoder_config(name: str, **overrides) -> DecoderConfig | VumuvikConfig:
+def decoder_config(name: str, **overrides) -> DecoderConfig | VumuvikConfig | VugotarConfig:
     if checkpoint_dir(name):
-        cfg = vumuvik_config_from_dir(name) if _dir_architecture(name) == "vumuvik" else decoder_config_from_hf(name)
+        cfg = _DIR_CONFIGS.get(_dir_architecture(name), decoder_config_from_hf)(name)
         return replace(cfg, **overrides) if overrides else cfg
     k = _key(name)
     if k not in DECODERS:
@@ -362,4 +601,4 @@ def is_encoder(name: str) -> bool:
 
 def is_decoder(name: str) -> bool:
     d = checkpoint_dir(name)
-    return _dir_architecture(d) in ("llama", "vumuvik") if d else _key(name) in DECODERS
+    return _dir_architecture(d) in ("llama", *_DIR_CONFIGS) if d else _key(name) in DECODERS

@@ -198,7 +198,7 @@ class LlamaModel(FragmentProjections):
         return self.embed.dtype
 
     # ---- what the engine asks of a decoder family
-    def make_cache(self, num_blocks: int, block_size: int) -> KVCache:
+    def make_cache(self, num_blocks: int, block_size: int, slots: int = 0) -> KVCache:
         return KVCache(self.cfg.layers, num_blocks, self.hkv, block_size, self.cfg.head_dim, self.device)
 
     def cache_bytes_per_block(self, block_size: int) -> int:

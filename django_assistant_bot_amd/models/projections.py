@@ -15,6 +15,11 @@ class FragmentProjections:
     frag = False
     tp_size = 1
     interleaved_mlp = True
+    recurrent = False  # the model keeps a state slot per sequence (``models.cache.HybridCache``)
+
+    def state_bytes(self, slots: int) -> int:
+        """Bytes of ``slots`` state slots (none: every layer's memory is paged)."""
+        return 0
 
     # stream_gemm.hip configurations (shuffled weights): BN 128 rows per workgroup at M <= 64 (13)
     # and M <= 128 (10).  Whole-chip tilings at M 65..128: gate_up's 28672 rows / 112 make exactly
@@ -94,13 +99,15 @@ class FragmentProjections:
             return ops.linear(x, w)
         return self._stream_or_tile(x, w, dec, allow_slabs, name, epilogue, self.proj_group.get(name, 1))
 
-    def _stream_or_tile(self, x, w, dec: bool, allow_slabs: bool, name: str, epilogue, grp: int):
+    def _stream_or_tile(self, x, w, dec: bool, allow_slabs: bool, name: str, epilogue, grp: int, out=None, glu_bias=None):
+        """``out`` / ``glu_bias``: of a gated epilogue (a view to write, fp32 [gate | up])."""
         if dec and self.frag:
             cfg, s = self._stream_choice(name, x.shape[0], w.shape[0], w.shape[1])
             if cfg >= 0:
                 if epilogue != ops.EPI_NONE:
-                    return ops.stream_gemm(x, w, epilogue=epilogue, nt=True, cfg=cfg, w_group=grp)
+                    return ops.stream_gemm(x, w, epilogue=epilogue, nt=True, cfg=cfg, w_group=grp, out=out,
+                                           glu_bias=glu_bias)
                 sd = torch.bfloat16 if (self.slab_bf16 and self.tp_size == 1) else torch.float32
                 out = ops.stream_gemm(x, w, splits=s, cfg=cfg, nt=True, slab_dtype=sd, w_group=grp)
                 return ops.slab_reduce(out) if (s > 1 and not allow_slabs) else out
-        return ops.gemm_bt(x, w, epilogue=epilogue, shuffled=self.frag, b_group=grp)
+        return ops.gemm_bt(x, w, epilogue=epilogue, shuffled=self.frag, b_group=grp, out=out, glu_bias=glu_bias)

@@ -6,10 +6,18 @@ from typing import Callable
 
 import torch
 
-from .configs import DecoderConfig, VumuvikConfig
+from .configs import DecoderConfig, VugotarConfig, VumuvikConfig
 from .llama import LlamaModel
+from .vugotar import VugotarModel
 from .vumuvik import VumuvikModel
-from .weights import load_decoder_checkpoint, load_vumuvik_checkpoint, random_decoder_weights, random_vumuvik_weights
+from .weights import (
+    load_decoder_checkpoint,
+    load_vugotar_checkpoint,
+    load_vumuvik_checkpoint,
+    random_decoder_weights,
+    random_vugotar_weights,
+    random_vumuvik_weights,
+)
 
 
 @dataclass(frozen=True)
@@ -36,6 +44,8 @@ def _load_llama(path, cfg, device="cpu", **kw):
 FAMILIES = {
     DecoderConfig: DecoderFamily(LlamaModel, random_decoder_weights, _load_llama),
     VumuvikConfig: DecoderFamily(VumuvikModel, _single(random_vumuvik_weights), _single(load_vumuvik_checkpoint),
+                                 (torch.bfloat16, torch.float32)),
+    VugotarConfig: DecoderFamily(VugotarModel, _single(random_vugotar_weights), _single(load_vugotar_checkpoint),
                                  (torch.bfloat16, torch.float32)),
 }
 

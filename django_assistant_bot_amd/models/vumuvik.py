@@ -143,7 +143,7 @@ class VumuvikModel(FragmentProjections):
     def _widths(self):
         return [L.R for L in self.layers]
 
-    def make_cache(self, num_blocks: int, block_size: int) -> LatentCache:
+    def make_cache(self, num_blocks: int, block_size: int, slots: int = 0) -> LatentCache:
         return LatentCache(self._widths(), self.source, num_blocks, block_size, self.device, self.dtype)
 
     def cache_bytes_per_block(self, block_size: int) -> int:

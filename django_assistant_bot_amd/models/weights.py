@@ -11,10 +11,20 @@ from __future__ import annotations
 import glob
 import os
 import re
+from dataclasses import dataclass
 
 import torch
 
-from .configs import DecoderConfig, EncoderConfig, VumuvikConfig
+from .configs import (
+    DecoderConfig,
+    DenseMlp,
+    EncoderConfig,
+    MoeMlp,
+    ParallelMixer,
+    VugotarConfig,
+    VumuvikConfig,
+    _up,
+)
 
 STD = 0.02
 
@@ -298,8 +308,8 @@ def _vumuvik_layout(cfg: VumuvikConfig, get, device, dtype, interleave_mlp) -> d
     return w
 
 
-def load_vumuvik_checkpoint(path: str, cfg: VumuvikConfig, device="cpu", dtype=torch.bfloat16, interleave_mlp=False,
-                            reader: SafetensorsDir | None = None) -> dict:
+def _checked(path: str, reader: SafetensorsDir | None):
+    """``get(name, shape)`` over a checkpoint directory."""
     st = reader or SafetensorsDir(path)
 
     def get(name, shape):
@@ -308,7 +318,12 @@ def load_vumuvik_checkpoint(path: str, cfg: VumuvikConfig, device="cpu", dtype=t
             raise ValueError(f"{path}: tensor {name} is {tuple(t.shape)}, config.json says {tuple(shape)}")
         return t
 
-    return _vumuvik_layout(cfg, get, torch.device(device), dtype, interleave_mlp)
+    return get
+
+
+def load_vumuvik_checkpoint(path: str, cfg: VumuvikConfig, device="cpu", dtype=torch.bfloat16, interleave_mlp=False,
+                            reader: SafetensorsDir | None = None) -> dict:
+    return _vumuvik_layout(cfg, _checked(path, reader), torch.device(device), dtype, interleave_mlp)
 
 
 def random_vumuvik_tensors(cfg: VumuvikConfig, device="cpu", dtype=torch.bfloat16, seed=0):
@@ -330,3 +345,170 @@ def random_vumuvik_tensors(cfg: VumuvikConfig, device="cpu", dtype=torch.bfloat1
 def random_vumuvik_weights(cfg: VumuvikConfig, device="cpu", dtype=torch.bfloat16, seed=0, interleave_mlp=False) -> dict:
     device = torch.device(device)
     return _vumuvik_layout(cfg, random_vumuvik_tensors(cfg, device, dtype, seed), device, dtype, interleave_mlp)
+
+
+# ------------------------------------------------------------------------------------------------
+# Vugotar
+
+
+class Columns:
+    """Named blocks of output rows of one fused projection, each starting at a multiple of ``align``."""
+
+    def __init__(self, align: int = 16):
+        self.align, self.at, self.width = align, {}, 0
+
+    def add(self, name: str, n: int) -> None:
+        self.at[name] = self.width
+        self.width = _up(self.width + n, self.align)
+
+    def fill(self, parts: dict, cols: int, total: int, like: torch.Tensor) -> torch.Tensor:
+        out = like.new_zeros((total, cols))
+        for name, t in parts.items():
+            out[self.at[name]:self.at[name] + t.shape[0], :t.shape[1]] = t
+        return out
+
+
+@dataclass(frozen=True)
+class HybridLayout:
+    """Where things are in a Vugotar layer's fused tensors."""
+
+    inp: Columns  # input projection: mixer columns, the shared expert's [gate | up]
+    aux: Columns  # fp32 projection: recurrence gates, router, shared gate
+    ff: int  # padded MLP columns at the head of the output projection's input (0: none)
+    mix: int  # its column of the recurrent mixer's output, the last block
+    width: int  # its columns
+    expert_ff: int  # padded expert width
+    conv: int  # convolution channels, a multiple of 8
+
+
+def hybrid_layout(cfg: VugotarConfig, i: int) -> HybridLayout:
+    m, f = cfg.blocks[i].mixer, cfg.blocks[i].mlp
+    inp, aux = Columns(), Columns(1)
+    if isinstance(m, ParallelMixer):
+        a, d = m.left, m.right
+        inp.add("qkv", (a.heads + 2 * a.kv_heads) * cfg.padded_head(a))
+        conv = _up(2 * d.kv_heads * d.dim + d.heads * d.vdim, 8)
+        inp.add("conv", conv)
+        inp.add("gate", d.heads * d.vdim)
+        aux.add("a", d.heads)
+        aux.add("b", d.heads)
+        attn, rec = a.heads * cfg.padded_head(a), d.heads * d.vdim
+    else:
+        rec = m.heads * m.vdim
+        conv = _up(rec + 2 * m.groups * m.state, 8)
+        inp.add("gate", rec)
+        inp.add("conv", conv)
+        aux.add("a", m.heads)
+        attn = 0
+    ff = eff = 0
+    if isinstance(f, DenseMlp):
+        ff = _up(f.ff, 128)
+    elif isinstance(f, MoeMlp):
+        aux.add("router", f.experts)
+        eff = _up(f.ff, 64)
+        if f.shared:
+            ff = _up(f.shared, 128)
+            inp.add("shared", 2 * ff)
+            aux.add("sg", 1)
+    return HybridLayout(inp, aux, ff, ff + attn, _up(ff + attn + rec, 128), eff, conv)
+
+
+def _vugotar_layout(cfg: VugotarConfig, get, device, dtype, interleave_mlp) -> dict:
+    """``get(name, shape)`` -> the engine's tensors.  Both sublayers of a layer read one norm, so a layer has one input
+    projection (``in_w``: attention q | k | v, convolution channels, gates, shared expert), one small fp32 projection
+    (``aux_w``: recurrence gates, router logits) and one output projection over the concatenated activations
+    [MLP | attention | recurrence] (``out_w``); a dense MLP's [gate | up] stays apart for the fused GLU epilogue.
+    Sizes are padded with zeros; gains (1 + w), biases, taps and recurrence constants are fp32."""
+    W, Wp = cfg.hidden, cfg.padded_hidden
+
+    def mat(name, *shape):
+        return get(name, shape).to(device=device, dtype=dtype)
+
+    def vec(name, *shape):
+        return get(name, shape).to(device=device, dtype=torch.float32).contiguous()
+
+    def glu(p, ff, to):
+        return _gate_up(_pad(mat(p + "gate", ff, W), to, Wp), _pad(mat(p + "up", ff, W), to, Wp), interleave_mlp)
+
+    w = {"embed": _pad(mat("embed", cfg.vocab_size, W), cfg.vocab_size, Wp),
+         "lm_head": _pad(mat("head", cfg.vocab_size, W), cfg.padded_vocab, Wp),
+         "final_norm": _pad(1 + vec("final.norm", W), Wp)}
+    for i, blk in enumerate(cfg.blocks):
+        p, m, f, lay = f"l{i}.", blk.mixer, blk.mlp, hybrid_layout(cfg, i)
+        w[p + "norm1"] = _pad(1 + vec(p + "norm1", W), Wp)
+        inp, aux, q = {}, {}, p + "mix."
+        out = w["embed"].new_zeros((Wp, lay.width))
+        if isinstance(m, ParallelMixer):
+            a, d, D = m.left, m.right, cfg.padded_head(m.left)
+            inp["qkv"] = torch.cat([_pad(mat(q + "left." + n, h * c, W).view(h, c, W), h, D, W).reshape(h * D, W)
+                                    for n, h, c in (("q", a.heads, a.dim), ("k", a.kv_heads, a.dim), ("v", a.kv_heads, a.vdim))])
+            out[:W, lay.ff:lay.mix] = _pad(mat(q + "left.o", W, a.heads * a.vdim).view(W, a.heads, a.vdim),
+                                           W, a.heads, D).reshape(W, a.heads * D)
+            q += "right."
+            rows = {"q": d.kv_heads * d.dim, "k": d.kv_heads * d.dim, "v": d.heads * d.vdim}
+            inp["conv"] = torch.cat([mat(q + n, r, W) for n, r in rows.items()])
+            w[p + "conv_w"] = _pad(torch.cat([vec(q + n + ".conv", r, d.conv) for n, r in rows.items()]), lay.conv, d.conv)
+            inp["gate"] = mat(q + "g", d.heads * d.vdim, W)
+            aux["a"], aux["b"] = mat(q + "a", d.heads, W), mat(q + "b", d.heads, W)
+            w[p + "rec_norm"] = vec(q + "norm", d.vdim)
+            heads, rec = d.heads, d.heads * d.vdim
+        else:
+            heads, rec = m.heads, m.heads * m.vdim
+            conv = rec + 2 * m.groups * m.state
+            full = mat(q + "in", rec + conv + heads, W)
+            inp["gate"], inp["conv"], aux["a"] = full[:rec], full[rec:rec + conv], full[rec + conv:]
+            w[p + "conv_w"] = _pad(vec(q + "conv", conv, m.conv), lay.conv, m.conv)
+            w[p + "conv_b"] = _pad(vec(q + "conv.b", conv), lay.conv)
+            w[p + "skip"], w[p + "rec_norm"] = vec(q + "D", heads), vec(q + "norm", rec)
+        out[:W, lay.mix:lay.mix + rec] = mat(q + "o", W, rec)
+        w[p + "A"] = torch.exp(vec(q + "A_log", heads).double()).float()
+        w[p + "dt_bias"] = vec(q + "dt_bias", heads)
+        q = p + "mlp."
+        if isinstance(f, DenseMlp):
+            w[p + "gate_up_w"] = glu(q, f.ff, lay.ff).contiguous()
+            w[p + "gate_up_b"] = torch.cat([_pad(vec(q + n + ".b", f.ff), lay.ff) for n in ("gate", "up")])
+            out[:W, :f.ff] = mat(q + "down", W, f.ff)
+            w[p + "down_b"] = _pad(vec(q + "down.b", W), Wp)
+        elif f is not None:
+            aux["router"] = mat(q + "router", f.experts, W)
+            ex, F = [f"{q}e{e}." for e in range(f.experts)], lay.expert_ff
+            w[p + "expert_gate_up_w"] = torch.cat([glu(e, f.ff, F) for e in ex])
+            w[p + "expert_down_w"] = torch.cat([_pad(mat(e + "down", W, f.ff), Wp, F) for e in ex])
+            if f.shared:
+                inp["shared"] = torch.cat([_pad(mat(q + "shared." + n, f.shared, W), lay.ff, W) for n in ("gate", "up")])
+                aux["sg"] = mat(q + "shared.sg", 1, W)
+                out[:W, :f.shared] = mat(q + "shared.down", W, f.shared)
+        w[p + "in_w"] = lay.inp.fill(inp, Wp, _up(lay.inp.width, 128), out)
+        w[p + "aux_w"] = lay.aux.fill(aux, Wp, _up(lay.aux.width, 128), out)
+        w[p + "out_w"] = out
+    return w
+
+
+def load_vugotar_checkpoint(path: str, cfg: VugotarConfig, device="cpu", dtype=torch.bfloat16, interleave_mlp=False,
+                            reader: SafetensorsDir | None = None) -> dict:
+    return _vugotar_layout(cfg, _checked(path, reader), torch.device(device), dtype, interleave_mlp)
+
+
+def random_vugotar_tensors(cfg: VugotarConfig, device="cpu", dtype=torch.bfloat16, seed=0):
+    """Seeded ``get(name, shape)`` of a random Vugotar: fan-in scaled matrices, small norm weights around zero, plain
+    norms and skips near one, decays between about 0.9 and 0.999 per step."""
+    g = _gen(torch.device(device), seed * 1000003)
+
+    def get(name, shape):
+        if name.endswith(".conv"):
+            return _randn(shape, g, device, torch.float32, std=shape[1] ** -0.5)
+        if len(shape) == 2:
+            return _randn(shape, g, device, dtype, std=STD if name in ("embed", "head") else shape[1] ** -0.5)
+        t = _randn(shape, g, device, torch.float32, std=0.1)
+        if name.endswith(".A_log"):
+            return t
+        if name.endswith(".dt_bias"):
+            return t - 4.0
+        return t + 1.0 if name.endswith((".D", "mix.norm", "right.norm")) else t
+
+    return get
+
+
+def random_vugotar_weights(cfg: VugotarConfig, device="cpu", dtype=torch.bfloat16, seed=0, interleave_mlp=False) -> dict:
+    device = torch.device(device)
+    return _vugotar_layout(cfg, random_vugotar_tensors(cfg, device, dtype, seed), device, dtype, interleave_mlp)

@@ -382,12 +382,13 @@ def use_gemm256(M: int, N: int, K: int, lda: int, ldb: int) -> bool:
 
 
 def gemm_bt(A, B, bias=None, residual=None, epilogue=EPI_NONE, out_f32=False, row_group=None, q_group=None,
-            allow=None, out=None, shuffled=False, n=None, b_group: int = 1):
+            allow=None, out=None, shuffled=False, n=None, b_group: int = 1, glu_bias=None):
     """C = A . B^T (+bias) (+act) (+residual) on MFMA; A [M, K], B [N, K] (K-contiguous rows).
 
     ``shuffled``: B is a ``shuffle_weights`` copy (the layout the decode GEMM streams, so a model
     keeps ONE copy of every projection) of ``B.shape[0]`` rows, of which the first ``n`` (default:
-    all) are the matrix; ``b_group`` 8: a ``shuffle_weights(w, 8)`` copy."""
+    all) are the matrix; ``b_group`` 8: a ``shuffle_weights(w, 8)`` copy.  ``glu_bias`` (GLU8 epilogues):
+    fp32 [N] = [gate | up], added before the gate's activation and the product."""
     expect(b_group == 1 or (shuffled and b_group == 8), "b_group: 1, or 8 with a shuffled copy")
     if shuffled:
         R = B.shape[0]
@@ -396,9 +397,9 @@ def gemm_bt(A, B, bias=None, residual=None, epilogue=EPI_NONE, out_f32=False, ro
                "shuffled B: contiguous [R, K] copy, R % (16 b_group) == 0, K % 32 == 0, R >= n")
         if not A.is_cuda:
             Bu = unshuffle_weights(B, b_group)[:N]
-            return ref.gemm_bt(A, Bu, bias, residual, epilogue, out_f32, row_group, q_group, allow)
+            return ref.gemm_bt(A, Bu, bias, residual, epilogue, out_f32, row_group, q_group, allow, glu_bias)
     if not A.is_cuda:
-        return ref.gemm_bt(A, B, bias, residual, epilogue, out_f32, row_group, q_group, allow)
+        return ref.gemm_bt(A, B, bias, residual, epilogue, out_f32, row_group, q_group, allow, glu_bias)
     expect(A.dtype == torch.bfloat16 and B.dtype == torch.bfloat16, "bf16 operands required")
     expect(A.stride(-1) == 1 and B.stride(-1) == 1, "operands must be K-contiguous")
     M, K = A.shape
@@ -415,6 +416,7 @@ def gemm_bt(A, B, bias=None, residual=None, epilogue=EPI_NONE, out_f32=False, ro
     if epilogue in GLU8:
         expect(N % 32 == 0 and not out_f32 and bias is None and residual is None,
                "swiglu8 epilogue needs N % 32 == 0, bf16 output, no bias / residual")
+    _glu_bias(glu_bias, epilogue, N)
     if residual is not None:
         expect(residual.dtype == torch.bfloat16 and residual.stride(-1) == 1, "residual must be bf16 row-major")
         expect(tuple(residual.shape) == (M, n_out), "residual shape mismatch")
@@ -436,15 +438,22 @@ def gemm_bt(A, B, bias=None, residual=None, epilogue=EPI_NONE, out_f32=False, ro
     plain = not out_f32 and row_group is None and q_group is None and allow is None
     if (plain and shuffled and N == B.shape[0] and bias is None and epilogue in (EPI_NONE, *GLU8)
             and use_gemm_mid(M, N, K, A.stride(0))):
-        return gemm_mid(A, B, residual=residual, epilogue=epilogue, out=out, b_group=b_group)
+        return gemm_mid(A, B, residual=residual, epilogue=epilogue, out=out, b_group=b_group, glu_bias=glu_bias)
     if (epilogue in (EPI_NONE, EPI_GELU, EPI_SWIGLU, *GLU8) and plain and (not shuffled or N == B.shape[0])
             and use_gemm256(M, N, K, A.stride(0), B.stride(0))):
-        return _gemm256_into(A, B, out, bias, residual, epilogue, shuffled, b_group)
-    native().gemm_bt(ptr(A), A.stride(0), ptr(B), B.stride(0), ptr(out), out.stride(0), ptr(bias), ptr(residual),
+        return _gemm256_into(A, B, out, bias if glu_bias is None else glu_bias, residual, epilogue, shuffled, b_group)
+    native().gemm_bt(ptr(A), A.stride(0), ptr(B), B.stride(0), ptr(out), out.stride(0),
+                     ptr(bias if glu_bias is None else glu_bias), ptr(residual),
                      residual.stride(0) if residual is not None else 0, M, N, K, int(epilogue), int(out_f32),
                      ptr(row_group), ptr(q_group), ptr(allow), allow_words, stream(A),
                      B.shape[0] if shuffled else 0, int(b_group))
     return out
+
+
+def _glu_bias(glu_bias, epilogue, N: int) -> None:
+    if glu_bias is not None:
+        expect(epilogue in GLU8 and glu_bias.dtype == torch.float32 and glu_bias.is_contiguous() and glu_bias.numel() == N,
+               "glu_bias: fp32 [gate | up] of a GLU8 epilogue")
 
 
 def _gemm256_into(A, B, out, bias, residual, epilogue, shuffled, b_group=1):
@@ -490,7 +499,7 @@ def gemm_mid_ok(M: int, N: int, K: int, lda: int) -> bool:
     return bool(native().gemm_mid_ok(M, N, K, lda)) and -(-M // 128) * (N // 256) <= (1 << 16)
 
 
-def gemm_mid(A, B, residual=None, epilogue=EPI_NONE, out=None, variant: int = 0, b_group: int = 1):
+def gemm_mid(A, B, residual=None, epilogue=EPI_NONE, out=None, variant: int = 0, b_group: int = 1, glu_bias=None):
     """C = A . B^T (+ residual) or SwiGLU over 8-row [gate | up] groups, B a ``shuffle_weights`` copy:
     the mid-M kernel (``gemm_mid.hip``: grouped stream-K, 128 x 256 tiles, in-launch owner combine) for
     M = 256..4096 (mixed serving steps, single prompts).  Bit-reproducible: the split-K partials are
@@ -507,12 +516,13 @@ def gemm_mid(A, B, residual=None, epilogue=EPI_NONE, out=None, variant: int = 0,
     if residual is not None:
         expect(epilogue == EPI_NONE and residual.dtype == torch.bfloat16 and residual.stride(-1) == 1
                and tuple(residual.shape) == (M, N), "residual must be bf16 [M, N]")
+    _glu_bias(glu_bias, epilogue, N)
     if out is None:
         out = torch.empty((M, n_out), dtype=torch.bfloat16, device=A.device)
     expect(out.dtype == torch.bfloat16 and out.stride(-1) == 1 and tuple(out.shape) == (M, n_out), "bad output")
     s = stream(A)
     slabs, cnt = _mid_workspace(A.device, s)
-    native().gemm_mid(ptr(A), A.stride(0), ptr(B), ptr(out), out.stride(0), ptr(residual),
+    native().gemm_mid(ptr(A), A.stride(0), ptr(B), ptr(out), out.stride(0), ptr(residual if glu_bias is None else glu_bias),
                       residual.stride(0) if residual is not None else 0, M, N, K, int(epilogue), ptr(slabs),
                       slabs.numel() * 4, ptr(cnt), cnt.numel(), s, int(variant), int(b_group))
     return out
@@ -585,7 +595,7 @@ def shuffle_rows_into(dst: torch.Tensor, rows: torch.Tensor, vals: torch.Tensor)
     v5[rows // 16, :, :, rows % 16, :] = vals.to(dst.dtype).reshape(-1, K // 32, 4, 8)
 
 
-def _ref_stream_gemm(x, w, splits=1, epilogue=EPI_NONE, residual=None, norm_eps=0.0):
+def _ref_stream_gemm(x, w, splits=1, epilogue=EPI_NONE, residual=None, norm_eps=0.0, glu_bias=None):
     """CPU semantics of ``stream_gemm`` (row-major ``w``): bf16 [M, N] / SwiGLU / fp32 slabs
     [S, M, N] whose sum is the product (slab 0 holds it, the others are zero).  ``norm_eps`` > 0:
     the product of the RMS-normalised rows of x (gains folded into w) before the epilogue."""
@@ -601,7 +611,7 @@ def _ref_stream_gemm(x, w, splits=1, epilogue=EPI_NONE, residual=None, norm_eps=
         if splits > 1:
             return torch.cat([y[None], torch.zeros((splits - 1,) + tuple(y.shape))], 0)
         return y.to(torch.bfloat16)
-    y = ref.gemm_bt(x, w, None, None, epilogue, out_f32=splits > 1)
+    y = ref.gemm_bt(x, w, None, None, epilogue, out_f32=splits > 1, glu_bias=glu_bias)
     if splits > 1:
         return torch.cat([y[None], torch.zeros((splits - 1,) + tuple(y.shape), dtype=y.dtype)], 0)
     return y if residual is None else (y.float() + residual.float()).to(torch.bfloat16)
@@ -637,7 +647,7 @@ def unshuffle_weights(w: torch.Tensor, group: int = 1) -> torch.Tensor:
 
 
 def stream_gemm(x, w, splits=1, epilogue=EPI_NONE, residual=None, out=None, nt=False, cfg=0, norm_eps: float = 0.0,
-                slab_dtype=torch.float32, w_group: int = 1):
+                slab_dtype=torch.float32, w_group: int = 1, glu_bias=None):
     """Decode GEMM y = x w^T on the warp-specialised streaming kernel (``stream_gemm.hip``): bf16
     [M, N] (optional residual add), SwiGLU [M, N/2] over 16- / 8-row interleaved [gate | up] rows, or
     fp32 K-slice slabs [S, M, N] (their sum is the product; consumers sum them in their prologue or
@@ -649,7 +659,7 @@ def stream_gemm(x, w, splits=1, epilogue=EPI_NONE, residual=None, out=None, nt=F
     partial sums rounded to bf16 (half the bytes for the producer and its consumer; the rounding the TP
     path's all-reduce input has).  On the CPU ``w`` is row-major."""
     if not x.is_cuda:
-        y = _ref_stream_gemm(x, w, splits=splits, epilogue=epilogue, residual=residual, norm_eps=norm_eps)
+        y = _ref_stream_gemm(x, w, splits=splits, epilogue=epilogue, residual=residual, norm_eps=norm_eps, glu_bias=glu_bias)
         return y.to(slab_dtype) if splits > 1 else y
     expect(norm_eps <= 0 or residual is None, "the consumer RMSNorm takes no residual add")
     expect(x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16, "bf16 operands required")
@@ -675,13 +685,15 @@ def stream_gemm(x, w, splits=1, epilogue=EPI_NONE, residual=None, out=None, nt=F
         if residual is not None:
             expect(epilogue == EPI_NONE and residual.dtype == torch.bfloat16 and residual.stride(-1) == 1
                    and tuple(residual.shape) == (M, N), "residual must be bf16 [M, N]")
+        _glu_bias(glu_bias, epilogue, N)
         if epilogue == EPI_SWIGLU:
             expect(bn % 32 == 0, f"stream_gemm cfg {cfg}: EPI_SWIGLU needs 32-row tiles (use EPI_SWIGLU8)")
         if out is None:
             out = torch.empty((M, n_out), dtype=torch.bfloat16, device=x.device)
         expect(out.dtype == torch.bfloat16 and out.stride(-1) == 1 and tuple(out.shape) == (M, n_out), "bad output")
         ldo = out.stride(0)
-    native().stream_gemm(ptr(x), x.stride(0), ptr(w), w.stride(0), ptr(out), ldo, ptr(residual),
+    native().stream_gemm(ptr(x), x.stride(0), ptr(w), w.stride(0), ptr(out), ldo,
+                         ptr(residual if glu_bias is None else glu_bias),
                          residual.stride(0) if residual is not None else 0, M, N, K, splits, int(epilogue), stream(x),
                          int(bool(nt)), int(cfg), float(norm_eps), int(splits > 1 and out.dtype == torch.bfloat16),
                          int(w_group))

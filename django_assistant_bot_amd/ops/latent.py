@@ -74,23 +74,29 @@ def dyt_residual(x, y, post: DytNorm | None, ls, nxt: DytNorm | None, dtype=torc
     return h
 
 
-def glu_f32(x, gelu: bool = True):
-    """fp32 [T, 2F] = [gate | up] -> act(gate) * up [T, F] (tanh-GELU, or SiLU)."""
+def glu_f32(x, gelu: bool = True, bias=None, out=None):
+    """fp32 [T, 2F] = [gate | up] (+ ``bias`` [gate | up]) -> act(gate) * up [T, F] (tanh-GELU, or SiLU)."""
     F2 = x.shape[-1]
     if not x.is_cuda:
+        x = x if bias is None else x + bias
         g, u = x[..., :F2 // 2].float(), x[..., F2 // 2:].float()
         act = torch.nn.functional.gelu(g, approximate="tanh") if gelu else torch.nn.functional.silu(g)
-        return (act * u).to(x.dtype)
+        y = (act * u).to(x.dtype)
+        return y if out is None else out.copy_(y)
     expect(x.dtype == torch.float32 and x.is_contiguous() and F2 % 8 == 0, "contiguous fp32 [T, 2F], F % 4")
-    out = torch.empty((x.shape[0], F2 // 2), dtype=torch.float32, device=x.device)
-    native().glu_f32(ptr(out), ptr(x), x.shape[0], F2 // 2, int(gelu), stream(x))
+    if bias is not None:
+        _f32(F2, bias)
+    out = torch.empty((x.shape[0], F2 // 2), dtype=torch.float32, device=x.device) if out is None else out
+    expect(out.dtype == torch.float32 and tuple(out.shape) == (x.shape[0], F2 // 2) and out.stride(1) == 1
+           and out.stride(0) % 4 == 0, "bad glu output")
+    native().glu_f32(ptr(out), out.stride(0), ptr(x), x.shape[0], F2 // 2, int(gelu), ptr(bias), 0, 0, stream(x))
     return out
 
 
 def gemm_f32(a, b):
     """fp32 a [M, K] . b [N, K]^T."""
     if not a.is_cuda:
-        return ref.gemm_bt(a, b)
+        return ref.gemm_bt(a, b, out_f32=True)
     M, K = a.shape
     N = b.shape[0]
     expect(a.dtype == torch.float32 and b.dtype == torch.float32 and b.is_contiguous() and a.stride(1) == 1, "fp32 rows")

@@ -163,7 +163,7 @@ def paged_decode(q, k_cache, v_cache, block_tables, ctx_lens, scale):
 
 
 def gemm_bt(A, B, bias=None, residual=None, epilogue=EPI_NONE, out_f32=False, row_group=None, q_group=None,
-            allow=None):
+            allow=None, glu_bias=None):
     c = A.float() @ B.float().t()
     if epilogue == EPI_SCORES:
         ok = torch.ones_like(c, dtype=torch.bool)
@@ -187,6 +187,8 @@ def gemm_bt(A, B, bias=None, residual=None, epilogue=EPI_NONE, out_f32=False, ro
     elif epilogue in (EPI_SWIGLU, EPI_SWIGLU8, EPI_GEGLU8):
         N, hg = c.shape[1], 16 if epilogue == EPI_SWIGLU else 8
         c = c.view(c.shape[0], N // (2 * hg), 2, hg)
+        if glu_bias is not None:  # [gate | up]
+            c = c + glu_bias.float().view(2, N // (2 * hg), hg).transpose(0, 1)
         act = F.gelu(c[:, :, 0], approximate="tanh") if epilogue == EPI_GEGLU8 else F.silu(c[:, :, 0])
         c = (act * c[:, :, 1]).reshape(c.shape[0], N // 2)
     if residual is not None:
