@@ -1,0 +1,490 @@
+// Chunked form of the matrix-state recurrences (recurrent.hip) for bf16 prompt portions: 64 tokens at a time on MFMA.
+//
+// Within a chunk let G_i = log-decay summed up to token i (inclusive), S0 the state before it, and k, q the unit
+// vectors.  The recurrence then is (delta; L = strictly lower triangle)
+//     M_ij = beta_i e^(G_i - G_j) k_i.k_j  (j < i)          T = (I + M)^-1
+//     R_i  = beta_i (v_i - e^(G_i) S0^T k_i)                U = T R
+//     o_i  = e^(G_i) S0^T q_i + sum_{j <= i} e^(G_i - G_j) (q_i.k_j) U_j
+//     S    = e^(G_C) S0 + sum_j e^(G_C - G_j) k_j U_j^T
+// and for state-space duality T = I, U = beta v.  T and A_ij = e^(G_i - G_j) q_i.k_j do not depend on the state:
+//   chunk_prepare   every (chunk, head) at once: products of the bf16 inputs, T by forward substitution
+//   chunk_scan      the chunks of a sequence in turn; a wave owns 16 value columns of one head and keeps their state
+//                   in accumulator registers
+//
+// Precision: everything is an fp32 computation.  The convolved q, k are exact bf16 numbers, so their products on the
+// bf16 MFMA are exact fp32 products; unit-norm factors, decays and betas are fp32 row scales applied outside.  An fp32
+// operand X (S, R, U, T) enters as X = hi + mid + lo, three bf16 terms (24 bits): products with a bf16 operand take 3
+// MFMAs, fp32 x fp32 the 6 whose weight exceeds 2^-24.  (A, which only reaches the bf16 output, has two terms.)
+//
+// Operand order: the accumulator layout (lane g = lane / 16 holds rows 4 g + r of a 16-row tile) is fed straight back
+// as a B operand by letting k slot (g, j) of a 32-deep step be row 4 g + j of its first tile for j < 4 and row
+// 4 g + j - 4 of its second tile otherwise; A operands are read in the same order.
+#include "launchers.h"
+#include "proj.h"
+
+namespace dab {
+
+namespace {
+
+constexpr int kC = 64;          // tokens of a chunk
+constexpr int kPairs = 6;       // (16-row tile, 32-deep step) pairs of a lower-triangular 64 x 64 operand
+constexpr int kFrag = 1024;     // bytes of one A fragment
+constexpr int kT = kPairs * 3 * kFrag, kA = kPairs * 2 * kFrag, kScal = 5 * kC * 4;
+constexpr int kWs = kT + kA + kScal;  // workspace of one (chunk, head)
+
+__device__ __forceinline__ int pair_id(int m, int kb) { return m < 2 ? m : 2 + 2 * (m - 2) + kb; }
+
+struct ChunkP {
+  const bf16* conv;
+  int C, q_col, k_col, v_col;
+  int H, G, D, V;
+  Proj gates;
+  int a_col, b_col;
+  const float* A;
+  const float* dt_bias;
+  const float* skip;
+  float* state;
+  const int* slot;
+  const int* pos;
+  const int* cu;
+  bf16* out;
+  char* ws;
+  float qscale;
+};
+
+// x = hi + mid (+ lo), bf16 each
+template <int N>
+__device__ __forceinline__ void split(const float (&x)[8], bf16x8 (&o)[N]) {
+  float r[8];
+#pragma unroll
+  for (int j = 0; j < 8; ++j) r[j] = x[j];
+#pragma unroll
+  for (int n = 0; n < N; ++n) {
+    u32x4 p;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) p[j] = pack2bf(r[2 * j], r[2 * j + 1]);
+    o[n] = __builtin_bit_cast(bf16x8, p);
+    if (n + 1 < N) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        r[2 * j] -= __uint_as_float(p[j] << 16);
+        r[2 * j + 1] -= __uint_as_float(p[j] & 0xffff0000u);
+      }
+    }
+  }
+}
+
+__device__ __forceinline__ bf16x8 cat4(const bf16x4& a, const bf16x4& b) {
+  return bf16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+}
+
+template <int D32, bool DELTA>
+__global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkP p) {
+  constexpr int Dp = 32 * D32, STR = Dp * 2 + 16, LD = 68;
+  constexpr int KQ = 2 * kC * STR, MA = 2 * kC * LD * 4;
+  __shared__ __attribute__((aligned(16))) char smem[KQ > MA ? KQ : MA];
+  __shared__ float gam[kC], be[kC], kk[kC], qq[kC];
+  char* ks = smem;
+  char* qs = smem + kC * STR;
+  float* Mm = reinterpret_cast<float*>(smem);
+  float* Am = Mm + kC * LD;
+  const int c = blockIdx.x, h = blockIdx.y, b = blockIdx.z, hk = h / (p.H / p.G);
+  const int r0 = p.cu[b] + kC * c, n = min(kC, p.cu[b + 1] - r0);
+  if (n <= 0) return;
+  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, g = lane >> 4, li = lane & 15;
+  char* ws = p.ws + ((size_t)(p.cu[b] / kC + b + c) * p.H + h) * kWs;
+  for (int i = tid; i < 2 * kC * (Dp / 8); i += 256) {
+    const int t = i / (Dp / 8) % kC, ch = i % (Dp / 8);
+    const bool q = i >= kC * (Dp / 8);
+    u32x4 v = {0, 0, 0, 0};
+    if (t < n && ch * 8 < p.D)
+      v = *reinterpret_cast<const u32x4*>(p.conv + (size_t)(r0 + t) * p.C + (q ? p.q_col : p.k_col) + hk * p.D + ch * 8);
+    *reinterpret_cast<u32x4*>((q ? qs : ks) + t * STR + ch * 16) = v;
+  }
+  if (w == 0) {
+    float dl = 0.f, beta = 0.f;
+    if (lane < n) {
+      const float z = proj_f32<float>(p.gates, r0 + lane, p.a_col + h) + p.dt_bias[h];
+      const float dt = z > 20.f ? z : log1pf(__expf(z));
+      dl = -p.A[h] * dt;
+      beta = DELTA ? 1.f / (1.f + __expf(-proj_f32<float>(p.gates, r0 + lane, p.b_col + h))) : dt;
+    }
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const float x = __shfl_up(dl, o, 64);
+      if (lane >= o) dl += x;
+    }
+    gam[lane] = dl;
+    be[lane] = beta;
+  }
+  __syncthreads();
+  // rows 16 w .. of K K^T and Q K^T (lower triangle), and the diagonal of Q Q^T
+  f32x4 kkt[4], qkt[4], qqt = {0.f, 0.f, 0.f, 0.f};
+  bf16x8 ka[D32], qa[D32];
+#pragma unroll
+  for (int kb = 0; kb < D32; ++kb) {
+    ka[kb] = *reinterpret_cast<const bf16x8*>(ks + (16 * w + li) * STR + (32 * kb + 8 * g) * 2);
+    qa[kb] = *reinterpret_cast<const bf16x8*>(qs + (16 * w + li) * STR + (32 * kb + 8 * g) * 2);
+    if (DELTA) qqt = mfma16(qa[kb], qa[kb], qqt);
+  }
+#pragma unroll
+  for (int nt = 0; nt < 4; ++nt) {
+    kkt[nt] = qkt[nt] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (nt > w) continue;
+#pragma unroll
+    for (int kb = 0; kb < D32; ++kb) {
+      const bf16x8 kn = *reinterpret_cast<const bf16x8*>(ks + (16 * nt + li) * STR + (32 * kb + 8 * g) * 2);
+      if (DELTA) kkt[nt] = mfma16(ka[kb], kn, kkt[nt]);
+      qkt[nt] = mfma16(qa[kb], kn, qkt[nt]);
+    }
+    if (DELTA && nt == w) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (4 * g + r == li) {
+          kk[16 * w + li] = 1.f / sqrtf(kkt[nt][r] + 1e-6f);
+          qq[16 * w + li] = p.qscale / sqrtf(qqt[r] + 1e-6f);
+        }
+    }
+  }
+  if (!DELTA && tid < kC) kk[tid] = qq[tid] = 1.f;
+  __syncthreads();  // K / Q are done with: M and A take their place
+#pragma unroll
+  for (int nt = 0; nt < 4; ++nt)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = 16 * w + 4 * g + r, j = 16 * nt + li;
+      float m = 0.f, a = 0.f;
+      if (j <= i) {
+        const float e = __expf(gam[i] - gam[j]) * kk[j];
+        a = e * qq[i] * qkt[nt][r];
+        if (DELTA && j < i) m = be[i] * e * kk[i] * kkt[nt][r];
+      }
+      if (DELTA) Mm[i * LD + j] = m;
+      Am[i * LD + j] = a;
+    }
+  __syncthreads();
+  auto frag = [&](const float* src, int m, int kb, float(&x)[8]) {
+    const float* s = src + (16 * m + li) * LD + 32 * kb + 4 * g;
+    const f32x4 lo = *reinterpret_cast<const f32x4*>(s), hi = *reinterpret_cast<const f32x4*>(s + 16);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      x[j] = lo[j];
+      x[4 + j] = hi[j];
+    }
+  };
+  if (w == 0) {
+    float* sc = reinterpret_cast<float*>(ws + kT + kA);
+    const float eg = __expf(gam[lane]);
+    sc[lane] = be[lane];
+    sc[kC + lane] = eg * kk[lane];
+    sc[2 * kC + lane] = eg * qq[lane];
+    sc[3 * kC + lane] = __expf(gam[kC - 1] - gam[lane]) * kk[lane];
+    sc[4 * kC + lane] = eg;
+    if (DELTA) {
+      // column ``lane`` of T: t_i = [i == lane] - sum_{j < i} M_ij t_j
+      float t[kC];
+#pragma unroll
+      for (int i = 0; i < kC; ++i) {
+        float a[4] = {lane == i ? 1.f : 0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int j4 = 0; j4 < (i + 3) / 4; ++j4) {
+          const f32x4 mv = *reinterpret_cast<const f32x4*>(Mm + i * LD + 4 * j4);
+#pragma unroll
+          for (int q = 0; q < 4; ++q)
+            if (4 * j4 + q < i) a[q] = fmaf(-mv[q], t[4 * j4 + q], a[q]);
+        }
+        t[i] = (a[0] + a[1]) + (a[2] + a[3]);
+      }
+#pragma unroll
+      for (int i = 0; i < kC; ++i) Mm[i * LD + lane] = t[i];  // every read of M was this wave's own
+    }
+  }
+  auto put = [&](int pr, auto&& fn) {
+    const int m = pr < 2 ? pr : 2 + (pr - 2) / 2, kb = pr < 2 ? 0 : (pr - 2) % 2;
+    fn(m, kb);
+  };
+  if (w > 0)
+    for (int pr = w - 1; pr < kPairs; pr += 3)
+      put(pr, [&](int m, int kb) {
+        float x[8];
+        bf16x8 o[2];
+        frag(Am, m, kb, x);
+        split(x, o);
+#pragma unroll
+        for (int s = 0; s < 2; ++s) *reinterpret_cast<bf16x8*>(ws + kT + (2 * pr + s) * kFrag + lane * 16) = o[s];
+      });
+  if (!DELTA) return;
+  __syncthreads();
+  for (int pr = w; pr < kPairs; pr += 4)
+    put(pr, [&](int m, int kb) {
+      float x[8];
+      bf16x8 o[3];
+      frag(Mm, m, kb, x);
+      split(x, o);
+#pragma unroll
+      for (int s = 0; s < 3; ++s) *reinterpret_cast<bf16x8*>(ws + (3 * pr + s) * kFrag + lane * 16) = o[s];
+    });
+}
+
+template <int D32, bool DELTA>
+__global__ __launch_bounds__(256) void chunk_scan_kernel(ChunkP p) {
+  constexpr int Dp = 32 * D32, STR = Dp * 2 + 16, MT = 2 * D32;
+  constexpr int CH = 2 * kC * (Dp / 8) / 256;  // 16-B pieces of the K | Q tile per thread
+  static_assert(CH >= 1, "tile too small");
+  __shared__ __attribute__((aligned(16))) char smem[2 * kC * STR];
+  __shared__ __attribute__((aligned(16))) float sc[5][kC];  // beta, e^G k-norm, e^G q-norm, e^(G_C - G) k-norm, e^G
+  const char* ks = smem;
+  const char* qs = smem + kC * STR;
+  const int h = blockIdx.y, b = blockIdx.z, hk = h / (p.H / p.G);
+  const int q0 = p.cu[b], len = p.cu[b + 1] - q0;
+  if (len <= 0) return;
+  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, g = lane >> 4, li = lane & 15;
+  const int col = blockIdx.x * 64 + 16 * w + li;
+  const bool live = blockIdx.x * 64 + 16 * w < p.V, mine = col < p.V;
+  float* sp = p.state + (((size_t)p.slot[b] * p.H + h) * p.V + (mine ? col : 0)) * Dp + 4 * g;
+  const char* ws0 = p.ws + ((size_t)(q0 / kC + b) * p.H + h) * kWs;
+  f32x4 S[MT];
+  const bool fresh = p.pos[q0] == 0;
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+    S[m] = fresh || !mine ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
+  const float skip = !DELTA && p.skip ? p.skip[h] : 0.f;
+  const int nc = (len + kC - 1) / kC;
+  u32x4 pre[CH];
+  auto fetch = [&](int c) {
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+      const int e = tid + 256 * i, t = e / (Dp / 8) % kC, ch = e % (Dp / 8);
+      const bool q = e >= kC * (Dp / 8);
+      pre[i] = u32x4{0, 0, 0, 0};
+      if (kC * c + t < len && ch * 8 < p.D)
+        pre[i] = *reinterpret_cast<const u32x4*>(p.conv + (size_t)(q0 + kC * c + t) * p.C + (q ? p.q_col : p.k_col) +
+                                                 hk * p.D + ch * 8);
+    }
+  };
+  fetch(0);
+  for (int c = 0; c < nc; ++c) {
+    const int n = min(kC, len - kC * c);
+    const char* ws = ws0 + (size_t)c * p.H * kWs;
+    __syncthreads();  // the previous chunk's tile is done with
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+      const int e = tid + 256 * i, t = e / (Dp / 8) % kC, ch = e % (Dp / 8);
+      *reinterpret_cast<u32x4*>(smem + (e >= kC * (Dp / 8) ? kC * STR : 0) + t * STR + ch * 16) = pre[i];
+    }
+    for (int i = tid; i < 5 * kC; i += 256) (&sc[0][0])[i] = reinterpret_cast<const float*>(ws + kT + kA)[i];
+    __syncthreads();
+    if (c + 1 < nc) fetch(c + 1);
+    if (!live) continue;  // (every wave reaches the barriers)
+    // values of this wave's columns in the accumulator layout
+    float R[4][4];
+    const bf16* vp = p.conv + (size_t)(q0 + kC * c) * p.C + p.v_col + h * p.V + (mine ? col : 0);
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = 16 * m + 4 * g + r;
+        R[m][r] = t < n && mine ? bf2f(vp[(size_t)t * p.C]) : 0.f;
+      }
+    bf16x8 ss[D32][3];  // the state as three bf16 terms
+#pragma unroll
+    for (int kb = 0; kb < D32; ++kb) {
+      float x[8];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        x[r] = S[2 * kb][r];
+        x[4 + r] = S[2 * kb + 1][r];
+      }
+      split(x, ss[kb]);
+    }
+    auto rows = [&](const char* src, int m, int kb) {  // A operand: 16 token rows, 32 state rows in slot order
+      const char* s = src + (16 * m + li) * STR + (32 * kb + 4 * g) * 2;
+      return cat4(*reinterpret_cast<const bf16x4*>(s), *reinterpret_cast<const bf16x4*>(s + 32));
+    };
+    auto times_s = [&](const char* src, int m) {
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kb = 0; kb < D32; ++kb) {
+        const bf16x8 a = rows(src, m, kb);
+        acc = mfma16(a, ss[kb][2], acc);
+        acc = mfma16(a, ss[kb][1], acc);
+        acc = mfma16(a, ss[kb][0], acc);
+      }
+      return acc;
+    };
+    f32x4 U[4], O[4];
+    float vskip[4][4];
+    if (!DELTA) {
+#pragma unroll
+      for (int m = 0; m < 4; ++m)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          vskip[m][r] = skip * R[m][r];
+          U[m][r] = sc[0][16 * m + 4 * g + r] * R[m][r];
+        }
+    } else {
+#pragma unroll
+      for (int m = 0; m < 4; ++m) {
+        const f32x4 P = times_s(ks, m);
+        const f32x4 be = *reinterpret_cast<const f32x4*>(&sc[0][16 * m + 4 * g]);
+        const f32x4 ek = *reinterpret_cast<const f32x4*>(&sc[1][16 * m + 4 * g]);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) R[m][r] = be[r] * (R[m][r] - ek[r] * P[r]);
+      }
+      bf16x8 rs[2][3];
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb) {
+        float x[8];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          x[r] = R[2 * kb][r];
+          x[4 + r] = R[2 * kb + 1][r];
+        }
+        split(x, rs[kb]);
+      }
+#pragma unroll
+      for (int m = 0; m < 4; ++m) {
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kb = 0; kb <= m / 2; ++kb) {
+          const char* f = ws + 3 * pair_id(m, kb) * kFrag + lane * 16;
+          const bf16x8 t0 = *reinterpret_cast<const bf16x8*>(f), t1 = *reinterpret_cast<const bf16x8*>(f + kFrag),
+                       t2 = *reinterpret_cast<const bf16x8*>(f + 2 * kFrag);
+          acc = mfma16(t2, rs[kb][0], acc);
+          acc = mfma16(t0, rs[kb][2], acc);
+          acc = mfma16(t1, rs[kb][1], acc);
+          acc = mfma16(t1, rs[kb][0], acc);
+          acc = mfma16(t0, rs[kb][1], acc);
+          acc = mfma16(t0, rs[kb][0], acc);
+        }
+        U[m] = acc;
+      }
+    }
+    // read-out
+    bf16x8 us[2][2];
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb) {
+      float x[8];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        x[r] = U[2 * kb][r];
+        x[4 + r] = U[2 * kb + 1][r];
+      }
+      split(x, us[kb]);
+    }
+#pragma unroll
+    for (int m = 0; m < 4; ++m) {
+      O[m] = times_s(qs, m);
+      O[m] *= *reinterpret_cast<const f32x4*>(&sc[2][16 * m + 4 * g]);
+#pragma unroll
+      for (int kb = 0; kb <= m / 2; ++kb) {
+        const char* f = ws + kT + 2 * pair_id(m, kb) * kFrag + lane * 16;
+        const bf16x8 a0 = *reinterpret_cast<const bf16x8*>(f), a1 = *reinterpret_cast<const bf16x8*>(f + kFrag);
+        O[m] = mfma16(a1, us[kb][0], O[m]);
+        O[m] = mfma16(a0, us[kb][1], O[m]);
+        O[m] = mfma16(a0, us[kb][0], O[m]);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = 16 * m + 4 * g + r;
+        if (t < n && mine)
+          p.out[(size_t)(q0 + kC * c + t) * p.H * p.V + h * p.V + col] = f2bf(DELTA ? O[m][r] : O[m][r] + vskip[m][r]);
+      }
+    }
+    // state: S = e^(G_C) S + K^T (e^(G_C - G) U)
+    bf16x8 wu[2][3];
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb) {
+      float x[8];
+      const f32x4 w0 = *reinterpret_cast<const f32x4*>(&sc[3][32 * kb + 4 * g]);
+      const f32x4 w1 = *reinterpret_cast<const f32x4*>(&sc[3][32 * kb + 16 + 4 * g]);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        x[r] = U[2 * kb][r] * w0[r];
+        x[4 + r] = U[2 * kb + 1][r] * w1[r];
+      }
+      split(x, wu[kb]);
+    }
+    const float ec = sc[4][kC - 1];
+    const int tq = li >> 2, tp = li & 3;
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+      f32x4 acc = S[m] * ec;
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb) {
+        const bf16x4 lo = ds_read_tr16(ks + (32 * kb + 4 * g + tq) * STR + (16 * m + 4 * tp) * 2);
+        const bf16x4 hi = ds_read_tr16(ks + (32 * kb + 16 + 4 * g + tq) * STR + (16 * m + 4 * tp) * 2);
+        const bf16x8 a = cat4(lo, hi);
+        acc = mfma16(a, wu[kb][2], acc);
+        acc = mfma16(a, wu[kb][1], acc);
+        acc = mfma16(a, wu[kb][0], acc);
+      }
+      S[m] = acc;
+    }
+  }
+  if (mine) {
+#pragma unroll
+    for (int m = 0; m < MT; ++m) *reinterpret_cast<f32x4*>(sp + 16 * m) = S[m];
+  }
+}
+
+}  // namespace
+
+long state_chunks_bytes(int T, int chunks, int H) { return (long)(T / kC + chunks) * H * kWs; }
+
+int state_chunks_ok(RecurrentShape d) {
+  return d.D % 8 == 0 && d.Dp <= 128 && d.C % 8 == 0 && d.q_col % 8 == 0 && d.k_col % 8 == 0 && d.H >= 1 && d.G >= 1 &&
+         d.H % d.G == 0 && d.H <= 65535 && d.Dp == recurrent_state_width(d.D);
+}
+
+int state_chunks(const void* conv, RecurrentShape d, Proj gates, const float* A, const float* dt_bias, const float* skip,
+                 float* state, const int* slot, const int* pos, const int* cu, int chunks, int max_q, void* out, void* ws,
+                 hipStream_t s) {
+  if (chunks <= 0 || max_q <= 0) return 0;
+  if (!state_chunks_ok(d) || !gates.f32 || gates.S < 1 || chunks > 65535 || !ws) return hipErrorInvalidValue;
+  ChunkP p{};
+  p.conv = (const bf16*)conv;
+  p.C = d.C;
+  p.q_col = d.q_col;
+  p.k_col = d.k_col;
+  p.v_col = d.v_col;
+  p.H = d.H;
+  p.G = d.G;
+  p.D = d.D;
+  p.V = d.V;
+  p.gates = gates;
+  p.a_col = d.a_col;
+  p.b_col = d.b_col;
+  p.A = A;
+  p.dt_bias = dt_bias;
+  p.skip = skip;
+  p.state = state;
+  p.slot = slot;
+  p.pos = pos;
+  p.cu = cu;
+  p.out = (bf16*)out;
+  p.ws = (char*)ws;
+  p.qscale = 1.f / sqrtf((float)d.D);
+  const dim3 gp((max_q + kC - 1) / kC, d.H, chunks), gs((d.V + 63) / 64, d.H, chunks);
+#define CHUNK_L(D32)                                                                               \
+  do {                                                                                             \
+    if (d.delta) {                                                                                 \
+      hipLaunchKernelGGL((chunk_prepare_kernel<D32, true>), gp, dim3(256), 0, s, p);               \
+      hipLaunchKernelGGL((chunk_scan_kernel<D32, true>), gs, dim3(256), 0, s, p);                  \
+    } else {                                                                                       \
+      hipLaunchKernelGGL((chunk_prepare_kernel<D32, false>), gp, dim3(256), 0, s, p);              \
+      hipLaunchKernelGGL((chunk_scan_kernel<D32, false>), gs, dim3(256), 0, s, p);                 \
+    }                                                                                              \
+  } while (0)
+  switch (d.Dp / 32) {
+    case 1: CHUNK_L(1); break;
+    case 2: CHUNK_L(2); break;
+    case 3: CHUNK_L(3); break;
+    case 4: CHUNK_L(4); break;
+    default: return hipErrorInvalidValue;
+  }
+#undef CHUNK_L
+  return hipGetLastError();
+}
+
+}  // namespace dab

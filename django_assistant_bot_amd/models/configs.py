@@ -406,7 +406,7 @@ DECODERS.update({
 DECODERS.update({
     # Llama-3-8B's width, MLP, vocabulary and KV heads; 2048-token chunks; a 128 x 128 state per head
     "vugotar-8b": vugotar_uniform(
-        "vugotar-8b", 24, 128256, 4096, ChunkedMixer(32, 8, 128, 128, 128 ** -0.5, 2048, 64, 500000.0),
+        "vugotar-8b", 28, 128256, 4096, ChunkedMixer(32, 8, 128, 128, 128 ** -0.5, 2048, 64, 500000.0),
         DeltaMixer(16, 8, 128, 128, 4), Mamba2Mixer(64, 64, 128, 8, 4, 8), DenseMlp(14336), None),
     # ... and with experts: 64 of 512, 6 per token, at Llama-3.2-1B's width
     "vugotar-moe": vugotar_uniform(

@@ -260,7 +260,7 @@ class VugotarModel(FragmentProjections):
         o = None
         if Tp:
             c = ops.short_conv(y, at["conv"], L.conv_w, L.conv_b, ring, meta.state_slots, pos, meta.cu_q, meta.max_q)
-            o = ops.state_scan(c, d, z, L.A, L.dt_bias, L.skip, state, meta.state_slots, pos, meta.cu_q)
+            o = ops.state_scan(c, d, z, L.A, L.dt_bias, L.skip, state, meta.state_slots, pos, meta.cu_q, meta.max_q)
         if Tp < T:
             slot = meta.state_slots if meta.decode else meta.dec_state_slots
             if d.delta:

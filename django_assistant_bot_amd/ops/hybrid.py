@@ -264,9 +264,13 @@ def short_conv(y, col0: int, w, bias, ring, slot, pos, cu, max_q: int):
     return out
 
 
-def state_scan(conv, d: RecurrentShape, z, A, dt_bias, skip, state, slot, pos, cu):
-    """The recurrence over the portions ``cu`` of convolved channels; ``state`` [slots, H, V, Dp] goes on from where the
-    sequence left it (zero at position 0).  -> read-outs [T, H V]."""
+CHUNK_MIN_TOKENS = 24  # portions shorter than this are scanned token by token
+
+
+def state_scan(conv, d: RecurrentShape, z, A, dt_bias, skip, state, slot, pos, cu, max_q: int, chunked: bool | None = None):
+    """The recurrence over the portions ``cu`` (the longest of ``max_q`` tokens) of convolved channels; ``state`` [slots, H,
+    V, Dp] goes on from where the sequence left it (zero at position 0).  -> read-outs [T, H V].  ``chunked``: 64 tokens at a
+    time on MFMA (bf16; default: where the sizes allow and the portions are long enough) or token by token."""
     T = conv.shape[0]
     if not conv.is_cuda:
         return ref.state_scan(conv, d, z, A, dt_bias, skip, state, slot, pos, ref._spans(cu, 0, 0)).to(conv.dtype)
@@ -275,7 +279,18 @@ def state_scan(conv, d: RecurrentShape, z, A, dt_bias, skip, state, slot, pos, c
     expect(conv.is_contiguous() and conv.dtype in _ACT and conv.shape[1] == d.C and pos.numel() >= T, "convolved channels")
     same_device(conv, z, A, dt_bias, skip, state, slot, pos, cu)
     out = torch.empty((T, d.H * d.V), dtype=conv.dtype, device=conv.device)
-    native().state_scan(ptr(conv), int(conv.dtype == torch.float32), d.native(), pz, ptr(A), ptr(dt_bias), ptr(skip),
+    n, nat = cu.numel() - 1, native()
+    expect(slot.numel() >= n, "state slots")
+    fits = conv.dtype == torch.bfloat16 and nat.state_chunks_ok(d.native())
+    if chunked is None:
+        chunked = fits and max_q >= CHUNK_MIN_TOKENS
+    if chunked:
+        expect(fits, "chunked scan: bf16, state rows % 8, at most 128")
+        ws = torch.empty((nat.state_chunks_bytes(T, n, d.H),), dtype=torch.uint8, device=conv.device)
+        nat.state_chunks(ptr(conv), d.native(), pz, ptr(A), ptr(dt_bias), ptr(skip), ptr(state), ptr(slot), ptr(pos), ptr(cu),
+                         n, int(max_q), ptr(out), ptr(ws), stream(conv))
+        return out
+    nat.state_scan(ptr(conv), int(conv.dtype == torch.float32), d.native(), pz, ptr(A), ptr(dt_bias), ptr(skip),
                         ptr(state), ptr(slot), ptr(pos), ptr(cu), cu.numel() - 1, ptr(out), stream(conv))
     return out
 

@@ -1,0 +1,367 @@
+"""RMS-stream, recurrent, chunked-attention and expert kernels against plain formulas in fp64 (tests/vugotar_oracle.py)
+or fp32 (the CPU references, which test_vugotar_model.py holds against the oracle)."""
+import pytest
+import torch
+import vugotar_oracle as oracle
+
+from django_assistant_bot_amd import ops
+from django_assistant_bot_amd.ops import reference as ref
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+BF, F32 = torch.bfloat16, torch.float32
+
+
+def rnd(*shape, seed=0, dtype=BF, scale=1.0):
+    g = torch.Generator().manual_seed(seed + sum(shape))
+    return (torch.randn(shape, generator=g) * scale).to(dtype)
+
+
+def close(got, want, tol):
+    got, want = got.double().cpu(), want.double()
+    assert torch.isfinite(got).all()
+    err = (got - want).abs().max().item() / max(want.abs().max().item(), 1e-6)
+    assert err < tol, err
+
+
+def i32(*v):
+    return torch.tensor(v, dtype=torch.int32)
+
+
+@pytest.mark.parametrize("rows,cols,n", [(1, 128, 100), (7, 4096, 4096), (130, 2048, 2000), (300, 640, 640), (3, 10240, 10000)])
+@pytest.mark.parametrize("yt,dtype", [(BF, BF), (F32, BF), (F32, F32)])
+@pytest.mark.parametrize("form", ["rows", "slabs", "all", "embed"])
+def test_rms_residual(rows, cols, n, yt, dtype, form):
+    x, gain = rnd(rows, cols, dtype=F32), rnd(cols, seed=1, dtype=F32)
+    y = rnd(5, rows, cols, seed=2, dtype=yt) if form in ("slabs", "all") else rnd(rows, cols, seed=2, dtype=yt)
+    bias = pairs = again = None
+    ids, table = torch.randint(0, 9, (rows,), dtype=torch.int32), rnd(9, cols, seed=3, dtype=dtype)
+    for t in (x, gain, table):
+        t[..., n:] = 0
+    y[..., n:] = 0
+    if form == "all":
+        bias, pairs, again = rnd(cols, seed=4, dtype=F32), rnd(rows * 3, cols, seed=5, dtype=dtype), (ids, table)
+        bias[n:], pairs[:, n:] = 0, 0
+    c = lambda t: None if t is None else t.to(DEV)  # noqa: E731
+    if form == "embed":
+        xg, h = ops.rms_embed(ids.to(DEV), table.to(DEV), gain.to(DEV), n, 1e-4)
+        x, hr = ops.rms_embed(ids, table, gain, n, 1e-4)
+    else:
+        xg = x.to(DEV)
+        h = ops.rms_residual(xg, y.to(DEV), gain.to(DEV), n, 1e-4, dtype, c(bias), c(pairs),
+                             None if again is None else (ids.to(DEV), table.to(DEV)))
+        hr = ops.rms_residual(x, y, gain, n, 1e-4, dtype, bias, pairs, again)
+    close(xg, x, 2e-6)
+    close(h, hr, 6e-3 if dtype == BF else 3e-6)
+    assert ops.rms_residual(xg, y.to(DEV), None, n, 1e-4, dtype) is None
+
+
+@pytest.mark.parametrize("H,G,D,dim,rot", [(4, 2, 64, 64, 64), (6, 6, 128, 96, 96), (8, 1, 128, 128, 32), (2, 2, 256, 200, 100),
+                                           (1, 1, 320, 270, 6), (3, 1, 64, 40, 0)])
+@pytest.mark.parametrize("yt,dtype", [(BF, BF), (F32, BF), (F32, F32)])
+def test_qk_rope_write(H, G, D, dim, rot, yt, dtype):
+    T, bs = 9, 16
+    y = rnd(T, 8 + (H + 2 * G) * D + 24, dtype=yt)
+    v = y[:, 8:8 + (H + 2 * G) * D].unflatten(1, (H + 2 * G, D))
+    v[:, :H + G, dim:] = 0
+    pos = i32(0, 1, 2, 63, 64, 1000, 100003, 7, 0)
+    slots = torch.tensor([3, 17, 16, -1, 40, 41, 0, 63, 5])
+    turns = ops.rope_turns(rot, 10000.0, DEV)
+    caches = [torch.zeros(4, G, bs, D, dtype=dtype) for _ in range(2)]
+    dev = [c.to(DEV) for c in caches]
+    q = ops.qk_rope_write(y.to(DEV), 8, H, G, D, dim, rot, turns, 1e-5, True, pos.to(DEV), slots.to(DEV), *dev)
+    qr = ops.qk_rope_write(y, 8, H, G, D, dim, rot, turns.cpu(), 1e-5, True, pos, slots, *caches)
+    tol = 8e-3 if dtype == BF else 3e-6
+    close(q, qr, tol)
+    close(dev[0], caches[0], tol)
+    close(dev[1], caches[1], tol)
+
+
+def paged(n, G, D, bs, dtype, seed):
+    """Random K / V caches with the pages of every sequence shuffled: (k, v, block tables)."""
+    pages = [-(-m // bs) for m in n]
+    total = sum(pages) + 2
+    perm = torch.randperm(total, generator=torch.Generator().manual_seed(seed)).int()
+    bt = torch.zeros(len(n), max(pages) + 1, dtype=torch.int32)
+    at = 0
+    for b, k in enumerate(pages):
+        bt[b, :k] = perm[at:at + k]
+        at += k
+    return rnd(total, G, bs, D, seed=seed, dtype=dtype), rnd(total, G, bs, D, seed=seed + 1, dtype=dtype), bt
+
+
+@pytest.mark.parametrize("H,G,D", [(4, 2, 64), (6, 6, 128), (8, 1, 128), (2, 1, 256), (3, 3, 320), (20, 1, 64)])
+@pytest.mark.parametrize("chunk", [0, 1, 64, 100, 257])
+@pytest.mark.parametrize("dtype", [BF, F32])
+def test_chunk_attention(H, G, D, chunk, dtype):
+    """Prompts, portions and decoded tokens; every query of a chunk's first and last positions is among them."""
+    bs, n = 64, [300, 129, 64, 1, 513]
+    nq = [300, 29, 2, 1, 200]
+    k, v, bt = paged(n, G, D, bs, dtype, 3)
+    k *= 2.0
+    cu, ctx = i32(0, *torch.tensor(nq).cumsum(0).tolist()), i32(*n)
+    T = int(cu[-1])
+    q, sink = rnd(T, H, D, seed=9, dtype=dtype), rnd(H, seed=4, dtype=F32)
+    want, out = torch.zeros(T, H * D + 8, dtype=dtype), torch.zeros(T, H * D + 8, dtype=dtype, device=DEV)
+    scale = 1.5 * D ** -0.5
+    args = (scale, chunk, sink)
+    ops.chunk_prefill(q, k, v, bt, cu, ctx, max(nq), *args, want, 0.6)
+    dev = [t.to(DEV) for t in (q, k, v, bt, cu, ctx, sink)]
+    ops.chunk_prefill(*dev[:6], max(nq), scale, chunk, dev[6], out, 0.6)
+    tol = 1.5e-2 if dtype == BF else 1e-5
+    close(out, want, tol)
+    # decoding at every length around a chunk's edge
+    lens = [1, 2, 63, 64, 65, 99, 100, 101, 200, 201, 256, 257, 258, 400, 513]
+    k, v, bt = paged(lens, G, D, bs, dtype, 5)
+    q = rnd(len(lens), H, D, seed=11, dtype=dtype)
+    want = torch.zeros(len(lens), H * D, dtype=dtype)
+    ops.chunk_decode(q, k, v, bt, i32(*lens), *args, want, 0.6)
+    dev = [t.to(DEV) for t in (q, k, v, bt, i32(*lens))]
+    for part, ws in ((512, None), (128, ops.DecodeWorkspace(len(lens), H, D, 6, DEV))):
+        out = torch.zeros(len(lens), H * D, dtype=dtype, device=DEV)
+        ops.chunk_decode(*dev, scale, chunk, sink.to(DEV), out, 0.6, part, ws)
+        close(out, want, tol)
+
+
+SHAPES = {  # delta, H, G, D, V, taps
+    "delta": (True, 4, 2, 128, 128, 4), "delta_odd": (True, 3, 1, 40, 23, 3), "delta_small": (True, 2, 2, 8, 16, 1),
+    "delta_96": (True, 2, 1, 96, 80, 2), "delta_wide": (True, 2, 2, 200, 72, 4), "delta_tiny": (True, 3, 3, 3, 5, 6),
+    "ssd": (False, 8, 2, 128, 64, 4), "ssd_odd": (False, 6, 3, 24, 40, 5), "ssd_64": (False, 2, 1, 64, 130, 4),
+    "ssd_wide": (False, 2, 1, 256, 33, 9)}
+
+
+def recurrence(name, T, seed=0, decay=-2.0):
+    delta, H, G, D, V, taps = SHAPES[name]
+    n = G * D
+    C = -(-(2 * n + H * V) // 8) * 8
+    cols = (0, n, 2 * n) if delta else (H * V + n, H * V, 0)
+    d = ops.RecurrentShape(delta, H, G, D, V, C, *cols, 1, H + 2)
+    y = rnd(T, 16 + C + H * V, seed=seed)
+    w, bias = rnd(C, taps, seed=seed + 1, dtype=F32, scale=taps ** -0.5), None if delta else rnd(C, seed=seed + 2, dtype=F32, scale=0.2)
+    z = rnd(T, 2 * H + 5, seed=seed + 3, dtype=F32)
+    A, dtb = rnd(H, seed=seed + 4, dtype=F32, scale=0.5).exp(), rnd(H, seed=seed + 5, dtype=F32, scale=0.5) + decay
+    skip = None if delta else rnd(H, seed=seed + 6, dtype=F32)
+    return d, taps, y, w, bias, z, A, dtb, skip
+
+
+def oracle_scan(d, conv, z, A, dtb, skip):
+    """fp64, token by token, from the convolved channels."""
+    c, z, A, dtb = conv.double(), z.double(), A.double(), dtb.double()
+    T, of = c.shape[0], torch.arange(d.H) // (d.H // d.G)
+    q, k = (c[:, s:s + d.G * d.D].view(T, d.G, d.D) for s in (d.q_col, d.k_col))
+    v = c[:, d.v_col:d.v_col + d.H * d.V].view(T, d.H, d.V)
+    dt = oracle.softplus(z[:, d.a_col:d.a_col + d.H] + dtb)
+    if d.delta:
+        o, S = oracle.delta_rule(oracle.unit(q)[:, of] * d.D ** -0.5, oracle.unit(k)[:, of], v, torch.exp(-A * dt),
+                                 torch.sigmoid(z[:, d.b_col:d.b_col + d.H]))
+        return o, S
+    o, S = oracle.ssd_scan(v, k[:, of], q[:, of], dt, A)
+    return o + skip.double()[:, None] * v, S
+
+
+@pytest.mark.parametrize("name", list(SHAPES))
+@pytest.mark.parametrize("dtype", [BF, F32])
+def test_short_conv_and_ring(name, dtype):
+    """Portions of unequal sequences in one launch, down to two tokens, against whole sequences."""
+    n, cuts = [70, 5, 33], [[0, 2, 3, 70], [0, 1, 3, 5], [0, 30, 32, 33]]
+    d, taps, _, w, bias, *_ = recurrence(name, 4)
+    ys = [rnd(m, 16 + d.C + 8, seed=m, dtype=dtype) for m in n]
+    ring = torch.full((5, taps, d.C), 9.0, dtype=dtype, device=DEV)  # what an earlier sequence left
+    slot = i32(3, 0, 4).to(DEV)
+    got = [[], [], []]
+    for step in range(3):
+        part = [ys[b][cuts[b][step]:cuts[b][step + 1]] for b in range(3)]
+        cu = i32(0, *torch.tensor([len(p) for p in part]).cumsum(0).tolist())
+        pos = torch.cat([torch.arange(cuts[b][step], cuts[b][step + 1]) for b in range(3)]).int()
+        out = ops.short_conv(torch.cat(part).to(DEV), 16, w.to(DEV), None if bias is None else bias.to(DEV), ring, slot,
+                             pos.to(DEV), cu.to(DEV), max(len(p) for p in part))
+        for b in range(3):
+            got[b].append(out[cu[b]:cu[b + 1]].cpu())
+    for b in range(3):
+        want = oracle.short_conv(ys[b][:, 16:16 + d.C].double(), w.double(), None if bias is None else bias.double())
+        close(torch.cat(got[b]), want, 6e-3 if dtype == BF else 2e-6)
+
+
+@pytest.mark.parametrize("name", list(SHAPES))
+@pytest.mark.parametrize("form", ["tokens_f32", "tokens_bf16", "chunks"])
+def test_state_scan(name, form):
+    """Two sequences of unequal portions in one launch, going on from their slots; the states come out right too."""
+    d, taps, _, w, bias, _, A, dtb, skip = recurrence(name, 4)
+    dtype = F32 if form == "tokens_f32" else BF
+    if form == "chunks" and not ops.native().state_chunks_ok(d.native()):
+        pytest.skip("sizes that are scanned token by token")
+    n, cuts = [200, 130], [[0, 64, 66, 200], [0, 1, 129, 130]]
+    conv = [rnd(m, d.C, seed=m, dtype=dtype) for m in n]
+    z = [rnd(m, 2 * d.H + 5, seed=m + 1, dtype=F32) for m in n]
+    state = torch.full((4, d.H, d.V, d.Dp), 5.0, device=DEV)
+    slot, c = i32(2, 0).to(DEV), lambda t: None if t is None else t.to(DEV)
+    got = [[], []]
+    for step in range(3):
+        cut = [slice(cuts[b][step], cuts[b][step + 1]) for b in range(2)]
+        m = [s.stop - s.start for s in cut]
+        cu = i32(0, m[0], m[0] + m[1])
+        pos = torch.cat([torch.arange(s.start, s.stop) for s in cut]).int()
+        out = ops.state_scan(torch.cat([conv[b][cut[b]] for b in range(2)]).to(DEV), d, torch.cat([z[b][cut[b]] for b in range(2)]).to(DEV),
+                             c(A), c(dtb), c(skip), state, slot, pos.to(DEV), cu.to(DEV), max(m), chunked=form == "chunks")
+        for b in range(2):
+            got[b].append(out[cu[b]:cu[b + 1]].cpu())
+    for b, s in enumerate((2, 0)):
+        o, S = oracle_scan(d, conv[b], z[b], A, dtb, skip)
+        close(torch.cat(got[b]).view(-1, d.H, d.V), o, 5e-3 if dtype == BF else 5e-6)
+        close(state[s, :, :, :d.D].transpose(1, 2), S, 5e-6)
+        assert float(state[s, :, :, d.D:].abs().sum()) == 0
+    assert bool((state[1] == 5).all()) and bool((state[3] == 5).all())
+
+
+@pytest.mark.parametrize("decay", [-12.0, 3.0])
+@pytest.mark.parametrize("name", ["delta", "ssd"])
+def test_chunked_scan_with_long_and_short_memory(name, decay):
+    """Decays within 1e-5 of one (every write stays) and close to zero (e^(G_i - G_j) underflows inside a chunk)."""
+    d, _, _, _, _, _, A, dtb, skip = recurrence(name, 4, decay=decay)
+    T = 500
+    conv, z = rnd(T, d.C, seed=1), rnd(T, 2 * d.H + 5, seed=2, dtype=F32)
+    state = torch.zeros(1, d.H, d.V, d.Dp, device=DEV)
+    c = lambda t: None if t is None else t.to(DEV)  # noqa: E731
+    out = ops.state_scan(conv.to(DEV), d, z.to(DEV), c(A), c(dtb), c(skip), state, i32(0).to(DEV), torch.arange(T).int().to(DEV),
+                         i32(0, T).to(DEV), T, chunked=True)
+    o, S = oracle_scan(d, conv, z, A, dtb, skip)
+    close(out.view(T, d.H, d.V), o, 5e-3)
+    close(state[0, :, :, :d.D].transpose(1, 2), S, 1e-5)
+
+
+@pytest.mark.parametrize("name", list(SHAPES))
+@pytest.mark.parametrize("yt,dtype", [(BF, BF), (F32, BF), (F32, F32)])
+def test_state_decode(name, yt, dtype):
+    """Token by token through the decode kernel (slots of earlier sequences, padded rows) against whole sequences."""
+    T, B, pad, eps = 12, 3, 5, 1e-3
+    d, taps, _, w, bias, _, A, dtb, skip = recurrence(name, 4)
+    n = d.H * d.V
+    slabs = 4 if (yt, dtype) == (F32, BF) else 1
+    y = rnd(T, B, 16 + d.C + n, seed=1, dtype=dtype)
+    z = rnd(T, B, 2 * d.H + 5, seed=2, dtype=F32)
+    wn = rnd(d.V, seed=8, dtype=F32) + 1
+    ring = torch.full((6, taps, d.C), 4.0, dtype=dtype, device=DEV)
+    state = torch.full((6, d.H, d.V, d.Dp), -3.0, device=DEV)
+    slot = i32(4, 1, 0, 5, 5).to(DEV)  # two padded rows on the spare slot
+    c = lambda t: None if t is None else t.to(DEV)  # noqa: E731
+    got = []
+    for t in range(T):
+        rows = torch.cat([y[t, :1], y[t], y[t, :2]])  # one prompt row ahead (row0 = 1), two padded rows behind
+        yy = rows.to(yt)
+        if slabs > 1:
+            split = rnd(slabs - 1, *rows.shape, seed=t, dtype=F32)
+            yy = torch.cat([split, (rows.float() - split.sum(0))[None]])
+        zz = torch.cat([z[t, :1], z[t], z[t, :2]])
+        out = torch.full((B + 3, n + (pad if d.delta else 0)), 7.0, dtype=dtype, device=DEV)
+        pos = i32(99, t, t, t, 0, 0).to(DEV)
+        ops.state_decode(yy.to(DEV), 16, c(w), c(bias), ring, d, zz.to(DEV), c(A), c(dtb), c(skip), state, slot, pos, 1, out,
+                         16 + d.C, c(wn) if d.delta else None, eps, 0.4 if d.delta else 1.0, pad)
+        assert bool((out[0] == 7).all())
+        if d.delta:
+            assert float(out[1:, n:].abs().sum()) == 0
+        got.append(out[1:1 + B, :n].cpu())
+    got = torch.stack(got)
+    for b in range(B):
+        conv = oracle.short_conv(y[:, b, 16:16 + d.C].double(), w.double(), None if bias is None else bias.double())
+        conv = conv.to(dtype)
+        o, S = oracle_scan(d, conv, z[:, b], A, dtb, skip)
+        if d.delta:
+            o = 0.4 * oracle.rms(o, eps) * wn.double() * oracle.silu(y[:, b, 16 + d.C:].double()).view(T, d.H, d.V)
+        close(got[:, b].view(T, d.H, d.V), o, 2e-2 if dtype == BF else 2e-5)
+        close(state[int(slot[b]), :, :, :d.D].transpose(1, 2), S, 1e-2 if dtype == BF else 1e-5)
+    assert bool((state[2] == -3).all()) and bool((state[3] == -3).all())
+
+
+@pytest.mark.parametrize("n,part", [(512, 128), (96, 32), (60, 15), (2048, 1024), (77, 77), (1200, 600)])
+@pytest.mark.parametrize("first,per_head", [(True, False), (False, True)])
+@pytest.mark.parametrize("yt,dtype", [(BF, BF), (F32, BF), (F32, F32)])
+def test_gated_norm(n, part, first, per_head, yt, dtype):
+    T, row0, pad = 21, 2, 11
+    y, gate, w = rnd(T + row0, n, dtype=dtype), rnd(3, T + row0, n + 8, seed=1, dtype=yt), rnd(part if per_head else n, seed=2, dtype=F32)
+    if yt == BF:
+        gate = gate[0]
+    out = torch.full((T + row0 + 1, n + pad + 2), 3.0, dtype=dtype, device=DEV)
+    ops.gated_norm(y.to(DEV), gate.to(DEV), 8, part, w.to(DEV), 1e-3, out, row0, T, first, per_head, 0.7, pad)
+    g = (gate.double().sum(0) if gate.dim() == 3 else gate.double())[:, 8:]
+    v = y.double()
+    ww = w.double().repeat(n // part) if per_head else w.double()
+    want = oracle.rms((v * oracle.silu(g) if first else v).view(-1, n // part, part), 1e-3).reshape(-1, n) * ww * 0.7
+    want = want if first else want * oracle.silu(g)
+    close(out[row0:row0 + T, :n], want[row0:], 8e-3 if dtype == BF else 3e-6)
+    assert float(out[row0:row0 + T, n:n + pad].abs().sum()) == 0
+    assert bool((out[:row0] == 3).all()) and bool((out[row0 + T:] == 3).all()) and bool((out[:, n + pad:] == 3).all())
+
+
+@pytest.mark.parametrize("T,E,top", [(1, 1, 1), (5, 16, 4), (130, 64, 6), (9, 70, 8), (33, 300, 3), (2, 1000, 64)])
+@pytest.mark.parametrize("S", [1, 4])
+def test_moe_route(T, E, top, S):
+    z = rnd(S, T, E + 7, dtype=F32)
+    z = z[0] if S == 1 else z
+    idx, wt = ops.moe_route(z.to(DEV), 3, E, top, 1.7, T)
+    zz = (z.double() if S == 1 else z.double().sum(0))[:, 3:3 + E]
+    want = oracle.route(zz, top, 1.7)
+    got = torch.zeros(T, E, dtype=torch.float64).scatter(1, idx.cpu().long(), wt.cpu().double())
+    close(got, want, 1e-5)
+    assert all(len(set(r)) == top for r in idx.cpu().tolist())
+
+
+@pytest.mark.parametrize("T,E,top,K,F,W", [(1, 4, 2, 128, 64, 128), (7, 16, 4, 256, 128, 256), (150, 8, 3, 512, 192, 384),
+                                           (600, 5, 2, 256, 64, 256), (40, 70, 5, 128, 64, 128), (1000, 3, 3, 128, 128, 128)])
+@pytest.mark.parametrize("dtype", [BF, F32])
+def test_moe_experts(T, E, top, K, F, W, dtype):
+    """Unequal loads, one expert that nobody chose and one that everybody did."""
+    h = rnd(T, K, dtype=dtype)
+    gate, up, down = (rnd(E, a, b, seed=s, dtype=dtype, scale=b ** -0.5) for a, b, s in ((F, K, 1), (F, K, 2), (W, F, 3)))
+    g = torch.Generator().manual_seed(5)
+    p = torch.rand(T, E, generator=g)
+    p[:, 0] += 2
+    if E > top:
+        p[:, -1] = -1
+    idx = torch.topk(p, top).indices.int()
+    wt = torch.rand(T, top, generator=g)
+    if dtype == BF:
+        gu = torch.cat([ops.shuffle_weights(ops.interleave_gate_up(gate[e], up[e], 8)) for e in range(E)])
+        dn = torch.cat([ops.shuffle_weights(down[e]) for e in range(E)])
+    else:
+        gu, dn = torch.cat([gate, up], 1).reshape(E * 2 * F, K), down.reshape(E * W, F)
+    got = ops.moe_experts(h.to(DEV), idx.to(DEV), wt.to(DEV), gu.to(DEV), dn.to(DEV), E, 8 if dtype == BF else 0)
+    want = torch.zeros(T, top, W, dtype=torch.float64)
+    for e in range(E):
+        t, k = (idx == e).nonzero(as_tuple=True)
+        act = oracle.silu(h[t].double() @ gate[e].double().T) * (h[t].double() @ up[e].double().T) * wt[t, k].double()[:, None]
+        want[t, k] = act.to(dtype).double() @ down[e].double().T
+    close(got, want.view(T * top, W), 1e-2 if dtype == BF else 5e-6)
+
+
+@pytest.mark.parametrize("yt,dtype", [(BF, BF), (F32, BF), (F32, F32)])
+def test_shared_glu(yt, dtype):
+    T, n = 37, 136
+    y, z = rnd(2, T, 16 + 2 * n, dtype=yt), rnd(3, T, 5, dtype=F32)
+    y = y[0] if yt == BF else y
+    out = torch.full((T, n + 24), 2.0, dtype=dtype, device=DEV)
+    ops.shared_glu(y.to(DEV), 16, n, z.to(DEV), 2, out[:, :n])
+    yy = y.double() if y.dim() == 2 else y.double().sum(0)
+    want = oracle.silu(yy[:, 16:16 + n]) * yy[:, 16 + n:] * torch.sigmoid(z.double().sum(0)[:, 2:3])
+    close(out[:, :n], want, 1.5e-2 if dtype == BF else 3e-6)
+    assert bool((out[:, n:] == 2).all())
+
+
+@pytest.mark.parametrize("M,N,K", [(1, 128, 128), (5, 2048, 512), (100, 768, 192), (130, 1024, 256), (300, 512, 512),
+                                   (1100, 1024, 256), (2500, 512, 192)])
+@pytest.mark.parametrize("epi", [ops.EPI_SWIGLU8, ops.EPI_GEGLU8])
+def test_biased_glu_epilogue(M, N, K, epi):
+    """The gated epilogue with a bias in every GEMM kernel a gate|up projection can take, into a strided view."""
+    x, w, b = rnd(M, K), rnd(N, K, seed=2, scale=K ** -0.5), rnd(N, seed=3, dtype=F32)
+    want = ref.gemm_bt(x, w, epilogue=epi, glu_bias=b)
+    wide = torch.full((M, N // 2 + 64), 5.0, dtype=BF, device=DEV)
+    ops.gemm_bt(x.to(DEV), ops.shuffle_weights(w).to(DEV), epilogue=epi, shuffled=True, glu_bias=b.to(DEV), out=wide[:, :N // 2])
+    close(wide[:, :N // 2], want, 1.2e-2)
+    assert bool((wide[:, N // 2:] == 5).all())
+    close(ops.gemm_bt(x.to(DEV), w.to(DEV), epilogue=epi, glu_bias=b.to(DEV)), want, 1.2e-2)
+    if M <= 16 and N % 128 == 0 and K % 128 == 0:
+        got = ops.stream_gemm(x.to(DEV), ops.shuffle_weights(w).to(DEV), epilogue=epi, cfg=30, nt=True, glu_bias=b.to(DEV))
+        close(got, want, 1.2e-2)
+    xf, wf = x.float(), torch.cat([w.view(-1, 2, 8, K)[:, 0].reshape(-1, K), w.view(-1, 2, 8, K)[:, 1].reshape(-1, K)]).float()
+    out = torch.zeros(M, N // 2 + 4, device=DEV)
+    ops.glu_f32(ops.gemm_f32(xf.to(DEV), wf.to(DEV)), epi == ops.EPI_GEGLU8, b.to(DEV), out[:, :N // 2])
+    close(out[:, :N // 2], ref.gemm_bt(x.float(), w.float(), epilogue=epi, glu_bias=b, out_f32=True), 1e-5)

@@ -4,17 +4,27 @@ on the native kernels in 32-bit and bf16."""
 import json
 import os
 import random
-import struct
 
 import numpy as np
 import pytest
 import torch
 import vumuvik_oracle as oracle
+from decoder_helpers import (
+    GREEDY,
+    MODES,
+    TOL,
+    VOCAB,
+    assert_greedy,
+    engine,
+    error,
+    feed_portions,
+    greedy_oracle,
+    prompt,
+    write_checkpoint,
+)
 
 from django_assistant_bot_amd.engine.llm_engine import LLMEngine, SamplingParams
 from django_assistant_bot_amd.models import decoder_config, is_decoder
-
-VOCAB = 211
 
 
 def layer(heads, dim, vdim, rank, window, ff, kv_from=None, scale=None):
@@ -78,19 +88,6 @@ def tensors(cfg, seed=0, share=1.0):
     return {k: v.to(torch.bfloat16) for k, v in w.items()}
 
 
-def write_checkpoint(path, cfg, w):
-    with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(cfg, f)
-    head, blob = {}, b""
-    for k, v in w.items():
-        raw = v.contiguous().view(torch.int16).numpy().tobytes()
-        head[k] = {"dtype": "BF16", "shape": list(v.shape), "data_offsets": [len(blob), len(blob) + len(raw)]}
-        blob += raw
-    h = json.dumps(head).encode()
-    with open(os.path.join(path, "model.safetensors"), "wb") as f:
-        f.write(struct.pack("<Q", len(h)) + h + blob)
-
-
 _DIRS: dict = {}
 
 
@@ -105,43 +102,6 @@ def models(tmp_path_factory):
             _DIRS[name] = (d, cfg, {k: v.double() for k, v in w.items()})
         return _DIRS[name]
     return get
-
-
-MODES = [pytest.param(("cpu", torch.float32), id="cpu-f32"),
-         pytest.param(("cuda", torch.float32), id="gpu-f32", marks=pytest.mark.gpu),
-         pytest.param(("cuda", torch.bfloat16), id="gpu-bf16", marks=pytest.mark.gpu)]
-TOL = {torch.float32: 2e-5, torch.bfloat16: 1.5e-2}
-
-
-def engine(path, mode, tokens=1024, **kw):
-    dev, dtype = mode
-    kw.setdefault("prefix_cache", False)
-    kw.setdefault("max_batch", 4)
-    kw.setdefault("max_model_len", tokens)
-    bs = kw.setdefault("block_size", 64)
-    return LLMEngine(path, dev, dtype=dtype, num_blocks=tokens // bs, **kw)
-
-
-def error(got, want):
-    """rms over the vocabulary of the mean-free difference, per row, over the rms of the wanted logits."""
-    d = got.double() - want
-    d = d - d.mean(-1, keepdim=True)
-    return d.pow(2).mean(-1).sqrt() / want.pow(2).mean().sqrt()
-
-
-def prompt(n, seed=0):
-    r = random.Random(seed)
-    return [r.randrange(VOCAB) for _ in range(n)]
-
-
-def feed_portions(eng, rid, toks, sizes):
-    """Feeds ``toks`` in portions of the given sizes (repeated), every row wanted -> [n, vocab]."""
-    out, at, k = [], 0, 0
-    while at < len(toks):
-        n = min(sizes[k % len(sizes)], len(toks) - at)
-        out.append(eng.feed([(rid, toks[at:at + n], range(n))]))
-        at, k = at + n, k + 1
-    return torch.cat(out)
 
 
 # ------------------------------------------------------------------------------------------------ mechanisms
@@ -349,24 +309,6 @@ def test_small_pages_on_the_cpu(models):
 # ------------------------------------------------------------------------------------------------ generation
 
 
-def greedy_oracle(cfg, w, toks, n):
-    toks = list(toks)
-    for _ in range(n):
-        toks.append(int(oracle.forward(cfg, w, toks)[-1].argmax()))
-    return toks[-n:]
-
-
-def assert_greedy(cfg, w, toks, out, tol):
-    """Every generated token is the oracle's best, up to ``tol`` of the logit spread (rounding ties)."""
-    lg = oracle.forward(cfg, w, list(toks) + list(out))
-    for i, t in enumerate(out):
-        row = lg[len(toks) - 1 + i]
-        assert row.max() - row[t] <= tol * row.std(), (i, float(row.max() - row[t]))
-
-
-GREEDY = dict(do_sample=False, temperature=0.0, ignore_eos=True)
-
-
 @pytest.mark.parametrize("mode", MODES)
 @pytest.mark.parametrize("mixed", [0, 48])
 def test_greedy_generation_through_the_scheduler(models, mode, mixed):
@@ -378,8 +320,8 @@ def test_greedy_generation_through_the_scheduler(models, mode, mixed):
     for p, o, n in zip(prompts, outs, n_new):
         assert len(o.token_ids) == n and o.finish_reason == "length"
         if mode[1] == torch.float32:
-            assert o.token_ids == greedy_oracle(cfg, w, p or [0], n)
-        assert_greedy(cfg, w, p or [0], o.token_ids, 2 * TOL[mode[1]])
+            assert o.token_ids == greedy_oracle(oracle, cfg, w, p or [0], n)
+        assert_greedy(oracle, cfg, w, p or [0], o.token_ids, 2 * TOL[mode[1]])
     assert eng.blocks.num_free_blocks() == eng.blocks.num_blocks()
     if mixed:
         assert eng.stats["mixed_steps"] > 0
@@ -396,10 +338,10 @@ def test_preemption_and_prefix_reuse(models, mode):
     assert eng.blocks.prefix_hits() > 0
     for p, o in zip(prompts + prompts[:1], outs):
         assert len(o.token_ids) == 60
-        assert_greedy(cfg, w, p, o.token_ids, 2 * TOL[mode[1]])
+        assert_greedy(oracle, cfg, w, p, o.token_ids, 2 * TOL[mode[1]])
     tight = engine(path, mode, tokens=9 * 64, max_model_len=256)
     for p, o in zip(prompts, tight.generate(prompts, sp)):
-        assert_greedy(cfg, w, p, o.token_ids, 2 * TOL[mode[1]])
+        assert_greedy(oracle, cfg, w, p, o.token_ids, 2 * TOL[mode[1]])
     assert tight.stats["preemptions"] > 0
 
 
