@@ -83,7 +83,8 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkP p) {
   constexpr int Dp = 32 * D32, STR = Dp * 2 + 16, LD = 68;
   constexpr int KQ = 2 * kC * STR, MA = 2 * kC * LD * 4;
   __shared__ __attribute__((aligned(16))) char smem[KQ > MA ? KQ : MA];
-  __shared__ float gam[kC], be[kC], kk[kC], qq[kC];
+  __shared__ double gam[kC];  // sums in fp64: their small differences are what counts
+  __shared__ float be[kC], kk[kC], qq[kC];
   char* ks = smem;
   char* qs = smem + kC * STR;
   float* Mm = reinterpret_cast<float*>(smem);
@@ -102,7 +103,8 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkP p) {
     *reinterpret_cast<u32x4*>((q ? qs : ks) + t * STR + ch * 16) = v;
   }
   if (w == 0) {
-    float dl = 0.f, beta = 0.f;
+    float beta = 0.f;
+    double dl = 0.;
     if (lane < n) {
       const float z = proj_f32<float>(p.gates, r0 + lane, p.a_col + h) + p.dt_bias[h];
       const float dt = z > 20.f ? z : log1pf(__expf(z));
@@ -111,7 +113,7 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkP p) {
     }
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
-      const float x = __shfl_up(dl, o, 64);
+      const double x = __shfl_up(dl, o, 64);
       if (lane >= o) dl += x;
     }
     gam[lane] = dl;
@@ -155,7 +157,7 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkP p) {
       const int i = 16 * w + 4 * g + r, j = 16 * nt + li;
       float m = 0.f, a = 0.f;
       if (j <= i) {
-        const float e = __expf(gam[i] - gam[j]) * kk[j];
+        const float e = __expf((float)(gam[i] - gam[j])) * kk[j];
         a = e * qq[i] * qkt[nt][r];
         if (DELTA && j < i) m = be[i] * e * kk[i] * kkt[nt][r];
       }
@@ -174,11 +176,11 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkP p) {
   };
   if (w == 0) {
     float* sc = reinterpret_cast<float*>(ws + kT + kA);
-    const float eg = __expf(gam[lane]);
+    const float eg = __expf((float)gam[lane]);
     sc[lane] = be[lane];
     sc[kC + lane] = eg * kk[lane];
     sc[2 * kC + lane] = eg * qq[lane];
-    sc[3 * kC + lane] = __expf(gam[kC - 1] - gam[lane]) * kk[lane];
+    sc[3 * kC + lane] = __expf((float)(gam[kC - 1] - gam[lane])) * kk[lane];
     sc[4 * kC + lane] = eg;
     if (DELTA) {
       // column ``lane`` of T: t_i = [i == lane] - sum_{j < i} M_ij t_j
