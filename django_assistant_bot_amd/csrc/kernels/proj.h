@@ -21,6 +21,17 @@ struct ElemIO<bf16> {
     unpack8(*reinterpret_cast<const u32x4*>(p), f);
   }
   static __device__ __forceinline__ void store8(bf16* p, const float (&f)[8]) { *reinterpret_cast<u32x4*>(p) = pack8(f); }
+  static __device__ __forceinline__ void add4(const bf16* p, float (&f)[4]) {
+    const u32x2 v = *reinterpret_cast<const u32x2*>(p);
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      f[2 * j] += __uint_as_float(v[j] << 16);
+      f[2 * j + 1] += __uint_as_float(v[j] & 0xffff0000u);
+    }
+  }
+  static __device__ __forceinline__ void store4(bf16* p, const float (&f)[4]) {
+    *reinterpret_cast<u32x2*>(p) = u32x2{pack2bf(f[0], f[1]), pack2bf(f[2], f[3])};
+  }
 };
 template <>
 struct ElemIO<float> {
@@ -41,24 +52,37 @@ struct ElemIO<float> {
     *reinterpret_cast<f32x4*>(p) = f32x4{f[0], f[1], f[2], f[3]};
     *reinterpret_cast<f32x4*>(p + 4) = f32x4{f[4], f[5], f[6], f[7]};
   }
+  static __device__ __forceinline__ void add4(const float* p, float (&f)[4]) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) f[j] += v[j];
+  }
+  static __device__ __forceinline__ void store4(float* p, const float (&f)[4]) {
+    *reinterpret_cast<f32x4*>(p) = f32x4{f[0], f[1], f[2], f[3]};
+  }
 };
 
-// element (row, col); rounded to the activation type AT when it was summed from slabs, like a finished output
-template <typename PT, typename AT>
-__device__ __forceinline__ float proj_at(const Proj& p, long row, int col) {
-  const PT* q = (const PT*)p.p + row * p.ld + col;
-  float v = ElemIO<PT>::load(q);
-  for (int s = 1; s < p.S; ++s) v += ElemIO<PT>::load(q + s * p.slab);
-  return ElemIO<AT>::round(v);
-}
-
-// the same without rounding (values that stay in 32 bits)
+// element (row, col) in fp32; the slabs' loads are issued four at a time
 template <typename PT>
 __device__ __forceinline__ float proj_f32(const Proj& p, long row, int col) {
   const PT* q = (const PT*)p.p + row * p.ld + col;
   float v = ElemIO<PT>::load(q);
-  for (int s = 1; s < p.S; ++s) v += ElemIO<PT>::load(q + s * p.slab);
+  int s = 1;
+  for (; s + 4 <= p.S; s += 4) {
+    float x[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) x[j] = ElemIO<PT>::load(q + (s + j) * p.slab);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v += x[j];
+  }
+  for (; s < p.S; ++s) v += ElemIO<PT>::load(q + s * p.slab);
   return v;
+}
+
+// the same rounded to the activation type, like a finished output
+template <typename PT, typename AT>
+__device__ __forceinline__ float proj_at(const Proj& p, long row, int col) {
+  return ElemIO<AT>::round(proj_f32<PT>(p, row, col));
 }
 
 // 8 consecutive elements (col % 8 == 0, ld % 8 == 0)

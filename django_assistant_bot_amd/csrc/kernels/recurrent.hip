@@ -53,49 +53,52 @@ constexpr int kConvTokens = 16;  // tokens a thread walks
 
 template <typename PT, typename AT, int K>
 __global__ __launch_bounds__(256) void short_conv_kernel(ConvParams p) {
-  const int b = blockIdx.z, c = (blockIdx.x * 256 + threadIdx.x) * 2;
+  const int b = blockIdx.z, c = (blockIdx.x * 256 + threadIdx.x) * 8;
   const int r0 = p.cu[b], n = p.cu[b + 1] - r0, t0 = blockIdx.y * kConvTokens;
   if (t0 >= n || c >= p.C) return;
   const int pos0 = p.pos[r0];
   const AT* ring = (const AT*)p.ring + (size_t)p.slot[b] * p.taps * p.C;
-  float w[2][K], win[2][K];  // win[.][K - 1]: the newest input
+  float w[K][8], win[K][8], bias[8];
 #pragma unroll
-  for (int k = 0; k < K; ++k) {
-    const int tap = k - (K - p.taps);
-    w[0][k] = tap >= 0 ? p.w[(size_t)c * p.taps + tap] : 0.f;
-    w[1][k] = tap >= 0 ? p.w[(size_t)(c + 1) * p.taps + tap] : 0.f;
-    win[0][k] = win[1][k] = 0.f;
-  }
-  auto input = [&](int t) {  // input of the chunk's token t, which may lie before the chunk
-    if (t >= 0) return make_float2(proj_at<PT, AT>(p.y, r0 + t, p.col0 + c), proj_at<PT, AT>(p.y, r0 + t, p.col0 + c + 1));
-    const int at = pos0 + t;
-    return at >= 0 ? ElemIO<AT>::load2(ring + (size_t)(at % p.taps) * p.C + c) : make_float2(0.f, 0.f);
-  };
-#pragma unroll
-  for (int k = 1; k < K; ++k) {  // the inputs before t0; win[k] = token t0 - (K - k)
-    if (K - k > p.taps - 1) continue;
-    const float2 v = input(t0 - (K - k));
-    win[0][k] = v.x;
-    win[1][k] = v.y;
-  }
-  const float b0 = p.bias ? p.bias[c] : 0.f, b1 = p.bias ? p.bias[c + 1] : 0.f;
-  const int t1 = min(n, t0 + kConvTokens);
-  for (int t = t0; t < t1; ++t) {
-    const float2 v = input(t);
-#pragma unroll
-    for (int k = 0; k + 1 < K; ++k) {
-      win[0][k] = win[0][k + 1];
-      win[1][k] = win[1][k + 1];
-    }
-    win[0][K - 1] = v.x;
-    win[1][K - 1] = v.y;
-    float s0 = b0, s1 = b1;
+  for (int j = 0; j < 8; ++j) {
+    bias[j] = p.bias ? p.bias[c + j] : 0.f;
 #pragma unroll
     for (int k = 0; k < K; ++k) {
-      s0 = fmaf(w[0][k], win[0][k], s0);
-      s1 = fmaf(w[1][k], win[1][k], s1);
+      const int tap = k - (K - p.taps);
+      w[k][j] = tap >= 0 ? p.w[(size_t)(c + j) * p.taps + tap] : 0.f;
+      win[k][j] = 0.f;
     }
-    ElemIO<AT>::store2((AT*)p.out + (size_t)(r0 + t) * p.C + c, silu_f(s0), silu_f(s1));
+  }
+  auto input = [&](int t, float(&v)[8]) {  // input of the chunk's token t, which may lie before the chunk
+    if (t >= 0) {
+      proj8<PT>(p.y, r0 + t, p.col0 + c, v);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] = ElemIO<AT>::round(v[j]);
+    } else if (pos0 + t >= 0) {
+      ElemIO<AT>::load8(ring + (size_t)((pos0 + t) % p.taps) * p.C + c, v);
+    }
+  };
+#pragma unroll
+  for (int k = 1; k < K; ++k)  // the inputs before t0: win[k] = token t0 - (K - k)
+    if (K - k <= p.taps - 1) input(t0 - (K - k), win[k]);
+  // token t0 + i goes to window entry i % K, so nothing is shifted
+  static_assert(kConvTokens % K == 0, "whole turns of the window");
+  const int t1 = min(n, t0 + kConvTokens);
+  for (int t = t0; t < t1; t += K) {
+#pragma unroll
+    for (int i = 0; i < K; ++i) {
+      if (t + i >= t1) break;  // (uniform in the workgroup)
+      input(t + i, win[i]);
+      float o[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        o[j] = bias[j];
+#pragma unroll
+        for (int k = 0; k < K; ++k) o[j] = fmaf(w[k][j], win[(i + 1 + k) % K][j], o[j]);
+        o[j] = silu_f(o[j]);
+      }
+      ElemIO<AT>::store8((AT*)p.out + (size_t)(r0 + t + i) * p.C + c, o);
+    }
   }
 }
 
@@ -114,11 +117,11 @@ __global__ __launch_bounds__(256) void conv_ring_kernel(ConvParams p) {
 int short_conv(Proj y, int col0, int C, int taps, const float* w, const float* bias, void* ring, const int* slot,
                const int* pos, const int* cu, int chunks, int max_q, void* out, int act_f32, hipStream_t s) {
   if (chunks <= 0 || max_q <= 0) return 0;
-  if (C < 2 || C % 2 || col0 % 2 || y.ld % 2 || taps < 1 || taps > 16 || y.S < 1 || chunks > 65535 ||
+  if (C < 8 || C % 8 || col0 % 8 || y.ld % 8 || taps < 1 || taps > 16 || y.S < 1 || chunks > 65535 ||
       (max_q + kConvTokens - 1) / kConvTokens > 65535)
     return hipErrorInvalidValue;
   ConvParams p{y, col0, C, taps, w, bias, ring, slot, pos, cu, out};
-  const dim3 grid((C / 2 + 255) / 256, (max_q + kConvTokens - 1) / kConvTokens, chunks);
+  const dim3 grid((C / 8 + 255) / 256, (max_q + kConvTokens - 1) / kConvTokens, chunks);
 #define CONV_K(PT, AT)                                                                                        \
   do {                                                                                                        \
     if (taps <= 4) hipLaunchKernelGGL((short_conv_kernel<PT, AT, 4>), grid, dim3(256), 0, s, p);              \
@@ -543,38 +546,63 @@ struct GatedNorm {
   void* out;
   long ldo;
   int pad, row0;      // zero columns after the last channel
+  int lanes;          // VEC, part / 8 a power of two below 64: lanes of a group (0: 64)
 };
 
-// one wave per group; lane owns channel pairs when everything is even, single channels otherwise
-template <typename PT, typename AT>
+// VEC: part, n and every row and column start are multiples of 8.  One wave per group of up to 512 channels (several
+// per workgroup), the whole workgroup on a wider one.
+template <typename PT, typename AT, bool VEC>
 __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNorm p) {
+  constexpr int E = VEC ? 8 : 1;
   __shared__ float red[4];
   const int row = p.row0 + blockIdx.y, lane = threadIdx.x & 63, w = threadIdx.x >> 6;
-  const bool wide = p.part > 512;  // the whole workgroup on one group
-  const int grp = wide ? blockIdx.x : blockIdx.x * 4 + w;
+  // lanes of one group: a whole workgroup, a wave, or (VEC) the part / 8 lanes a narrow group fills
+  const bool wide = p.part > 64 * E;
+  const int gl = wide ? 256 : (VEC && p.lanes) ? p.lanes : 64;
+  const int per = wide ? 1 : 256 / gl;
+  const int grp = blockIdx.x * per + (wide ? 0 : (int)threadIdx.x / gl), i0 = wide ? threadIdx.x : (int)threadIdx.x % gl;
   const int ng = p.n / p.part;
   AT* out = (AT*)p.out + (size_t)row * p.ldo;
   if (blockIdx.x == 0)
     for (int i = threadIdx.x; i < p.pad; i += 256) ElemIO<AT>::store(out + p.n + i, 0.f);
-  if (grp >= ng) return;  // (wide: uniform)
-  const AT* y = (const AT*)p.y + (size_t)row * p.n + (size_t)grp * p.part;
-  const int c0 = grp * p.part, st = wide ? 256 : 64, i0 = wide ? threadIdx.x : lane;
-  float ss = 0.f;
-  for (int i = i0; i < p.part; i += st) {
-    float v = ElemIO<AT>::load(y + i);
-    if (p.gate_first) v *= silu_f(proj_f32<PT>(p.gate, row, p.g_col + c0 + i));
-    ss = fmaf(v, v, ss);
+  const bool on = grp < ng;  // (no early exit: the lanes of a wave reduce together)
+  const AT* y = (const AT*)p.y + (size_t)row * p.n + (size_t)(on ? grp : 0) * p.part;
+  const int c0 = (on ? grp : 0) * p.part;
+  auto value = [&](int i, float(&v)[E], float(&g)[E]) {
+    if constexpr (VEC) {
+      ElemIO<AT>::load8(y + i, v);
+      proj8<PT>(p.gate, row, p.g_col + c0 + i, g);
+    } else {
+      v[0] = ElemIO<AT>::load(y + i);
+      g[0] = proj_f32<PT>(p.gate, row, p.g_col + c0 + i);
+    }
+#pragma unroll
+    for (int j = 0; j < E; ++j) g[j] = silu_f(g[j]);
+  };
+  float ss = 0.f, v[E], g[E];
+  for (int i = i0 * E; i < p.part; i += gl * E) {
+    value(i, v, g);
+#pragma unroll
+    for (int j = 0; j < E; ++j) {
+      const float x = p.gate_first ? v[j] * g[j] : v[j];
+      ss = fmaf(x, x, ss);
+    }
   }
-  ss = wave_sum(ss);
+  for (int o = (wide ? 64 : gl) / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
   if (wide) {
     if (lane == 0) red[w] = ss;
     __syncthreads();
     ss = red[0] + red[1] + red[2] + red[3];
   }
   const float r = p.scale / sqrtf(ss / p.part + p.eps);
-  for (int i = i0; i < p.part; i += st) {
-    const float v = ElemIO<AT>::load(y + i) * silu_f(proj_f32<PT>(p.gate, row, p.g_col + c0 + i));
-    ElemIO<AT>::store(out + c0 + i, v * r * p.w[p.per_head ? i : c0 + i]);
+  if (!on) return;
+  for (int i = i0 * E; i < p.part; i += gl * E) {
+    if (wide || gl * E < p.part) value(i, v, g);  // (one step: still in registers)
+    float o[E];
+#pragma unroll
+    for (int j = 0; j < E; ++j) o[j] = v[j] * g[j] * r * p.w[(p.per_head ? 0 : c0) + i + j];
+    if constexpr (VEC) ElemIO<AT>::store8(out + c0 + i, o);
+    else ElemIO<AT>::store(out + c0 + i, o[0]);
   }
 }
 
@@ -582,14 +610,23 @@ int gated_norm(const void* y, int act_f32, Proj gate, int g_col, int n, int part
                const float* w, float eps, float scale, void* out, long ldo, int pad, int row0, int T, hipStream_t s) {
   if (T <= 0) return 0;
   if (n < 1 || part < 1 || n % part || gate.S < 1 || T > (1 << 20)) return hipErrorInvalidValue;
-  GatedNorm p{y, gate, g_col, n, part, gate_first, per_head, w, eps, scale, out, ldo, pad, row0};
+  GatedNorm p{y, gate, g_col, n, part, gate_first, per_head, w, eps, scale, out, ldo, pad, row0, 0};
   const int ng = n / part;
+  const bool vec = part % 8 == 0 && g_col % 8 == 0 && gate.ld % 8 == 0 && gate.slab % 8 == 0 && ldo % 8 == 0 &&
+                   ((uintptr_t)y | (uintptr_t)out | (uintptr_t)gate.p) % 16 == 0;
+  const int pl = part / 8;
+  if (vec && pl < 64 && (pl & (pl - 1)) == 0) p.lanes = pl;
+  const int e = vec ? 8 : 1, per = part > 64 * e ? 1 : 256 / (p.lanes ? p.lanes : 64);
   // rows in grid.y (65535 limit): walk in slices
   for (int r = 0; r < T; r += 32768) {
     GatedNorm q = p;
     q.row0 = row0 + r;
-    const dim3 grid(part > 512 ? ng : (ng + 3) / 4, T - r < 32768 ? T - r : 32768);
-#define GN_L(PT, AT) hipLaunchKernelGGL((gated_norm_kernel<PT, AT>), grid, dim3(256), 0, s, q)
+    const dim3 grid((ng + per - 1) / per, T - r < 32768 ? T - r : 32768);
+#define GN_L(PT, AT)                                                                                   \
+  do {                                                                                                 \
+    if (vec) hipLaunchKernelGGL((gated_norm_kernel<PT, AT, true>), grid, dim3(256), 0, s, q);          \
+    else hipLaunchKernelGGL((gated_norm_kernel<PT, AT, false>), grid, dim3(256), 0, s, q);             \
+  } while (0)
     DAB_PROJ_DISPATCH(gate, act_f32, GN_L);
 #undef GN_L
   }

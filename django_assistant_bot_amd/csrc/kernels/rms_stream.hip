@@ -140,64 +140,77 @@ struct RopeParams {
   int bs, T;
 };
 
-// one workgroup per token; a wave walks heads, a lane owns the pairs 2 (lane + 64 i), i < NP.  The angle
-// p * f is formed in fp64 and reduced to a half turn before the fp32 sine and cosine, so it is exact to
-// fp32 rounding at any position.
-template <typename PT, typename AT, int NP>
-__global__ __launch_bounds__(256) void qk_rope_kernel(RopeParams p) {
-  const int t = blockIdx.x, w = threadIdx.x >> 6, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+// One workgroup per token.  A group of LPH lanes walks heads, a lane owns the pairs 2 (2 (lane + LPH i) + 0 / 1), i < NP:
+// four consecutive elements.  The angle p * f is formed in fp64 and reduced to a half turn before the fp32 sine and
+// cosine, so it is exact to fp32 rounding at any position; one workgroup forms it once for all heads.
+template <typename PT, typename AT, int LPH, int NP>
+__global__ __launch_bounds__(512) void qk_rope_kernel(RopeParams p) {
+  const int t = blockIdx.x, grp = threadIdx.x / LPH, lane = threadIdx.x % LPH, ng = blockDim.x / LPH;
   const int64_t slot = p.slots[t];
   const double pos = (double)p.positions[t];
-  float cs[NP], sn[NP];
+  float cs[NP][2], sn[NP][2];
 #pragma unroll
-  for (int i = 0; i < NP; ++i) {
-    const int pr = lane + 64 * i;
-    cs[i] = 1.f;
-    sn[i] = 0.f;
-    if (2 * pr < p.rot) {
-      const double turns = pos * p.freq[pr];
-      const float a = (float)((turns - rint(turns)) * 6.283185307179586476925);
-      sincosf(a, &sn[i], &cs[i]);
+  for (int i = 0; i < NP; ++i)
+#pragma unroll
+    for (int e = 0; e < 2; ++e) {
+      const int pr = 2 * (lane + LPH * i) + e;
+      cs[i][e] = 1.f;
+      sn[i][e] = 0.f;
+      if (2 * pr < p.rot) {
+        const double turns = pos * p.freq[pr];
+        sincosf((float)((turns - rint(turns)) * 6.283185307179586476925), &sn[i][e], &cs[i][e]);
+      }
     }
-  }
   const size_t blk = slot >= 0 ? (size_t)(slot / p.bs) : 0, off = slot >= 0 ? (size_t)(slot % p.bs) : 0;
-  for (int hd = w; hd < p.H + 2 * p.G; hd += nw) {
-    const bool is_v = hd >= p.H + p.G;
-    float u[NP], v[NP], ss = 0.f;
+  const int heads = p.H + 2 * p.G;
+  for (int h0 = 0; h0 < heads; h0 += ng) {  // (uniform trip count: the groups of a wave reduce together)
+    const int hd = h0 + grp;
+    const bool on = hd < heads, is_v = hd >= p.H + p.G;
+    float x[NP][4], ss = 0.f;
 #pragma unroll
     for (int i = 0; i < NP; ++i) {
-      const int d = 2 * (lane + 64 * i);
-      u[i] = v[i] = 0.f;
-      if (d >= p.D) continue;
+      const int d = 4 * (lane + LPH * i);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) x[i][e] = 0.f;
+      if (d >= p.D || !on) continue;
       const PT* s = (const PT*)p.y.p + (size_t)t * p.y.ld + p.col0 + (size_t)hd * p.D + d;
-      for (int k = 0; k < p.y.S; ++k, s += p.y.slab) {
-        const float2 e = ElemIO<PT>::load2(s);
-        u[i] += e.x;
-        v[i] += e.y;
+      ElemIO<PT>::add4(s, x[i]);
+      int k = 1;
+      s += p.y.slab;
+      for (; k + 2 <= p.y.S; k += 2, s += 2 * p.y.slab) {
+        float a[4] = {0.f, 0.f, 0.f, 0.f};
+        ElemIO<PT>::add4(s, x[i]);
+        ElemIO<PT>::add4(s + p.y.slab, a);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) x[i][e] += a[e];
       }
-      u[i] = ElemIO<AT>::round(u[i]);
-      v[i] = ElemIO<AT>::round(v[i]);
+      if (k < p.y.S) ElemIO<PT>::add4(s, x[i]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) x[i][e] = ElemIO<AT>::round(x[i][e]);
       if (!is_v) {
-        const float a = u[i] * cs[i] - v[i] * sn[i], b = v[i] * cs[i] + u[i] * sn[i];
-        u[i] = a;
-        v[i] = b;
-        ss += a * a + b * b;
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+          const float u = x[i][2 * e], v = x[i][2 * e + 1];
+          x[i][2 * e] = u * cs[i][e] - v * sn[i][e];
+          x[i][2 * e + 1] = v * cs[i][e] + u * sn[i][e];
+          ss += x[i][2 * e] * x[i][2 * e] + x[i][2 * e + 1] * x[i][2 * e + 1];
+        }
       }
-    }
-    float r = 1.f;
-    if (!is_v && p.norm) r = 1.f / sqrtf(wave_sum(ss) * p.inv_dim + p.eps);
-    AT* dst;
-    if (hd < p.H) dst = (AT*)p.q + ((size_t)t * p.H + hd) * p.D;
-    else if (slot < 0) continue;
-    else {
-      const int gk = is_v ? hd - p.H - p.G : hd - p.H;
-      dst = (AT*)(is_v ? p.vc : p.kc) + ((blk * p.G + gk) * p.bs + off) * p.D;
     }
 #pragma unroll
+    for (int o = LPH / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    const float r = !is_v && p.norm ? 1.f / sqrtf(ss * p.inv_dim + p.eps) : 1.f;
+    if (!on || (hd >= p.H && slot < 0)) continue;
+    const int gk = is_v ? hd - p.H - p.G : hd - p.H;
+    AT* dst = hd < p.H ? (AT*)p.q + ((size_t)t * p.H + hd) * p.D
+                       : (AT*)(is_v ? p.vc : p.kc) + ((blk * p.G + gk) * p.bs + off) * p.D;
+#pragma unroll
     for (int i = 0; i < NP; ++i) {
-      const int d = 2 * (lane + 64 * i);
+      const int d = 4 * (lane + LPH * i);
       if (d >= p.D) continue;
-      ElemIO<AT>::store2(dst + d, u[i] * r, v[i] * r);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) x[i][e] *= r;
+      ElemIO<AT>::store4(dst + d, x[i]);
     }
   }
 }
@@ -206,15 +219,16 @@ int qk_rope_write(Proj y, int col0, int H, int G, int D, int dim, int rot, const
                   const int* positions, const int64_t* slots, void* q, void* kc, void* vc, int act_f32, int bs, int T,
                   hipStream_t s) {
   if (T <= 0) return 0;
-  if (H < 1 || G < 1 || D < 2 || D % 2 || D > 1024 || dim < 1 || dim > D || rot % 2 || rot > dim || rot < 0 || bs < 1 ||
+  if (H < 1 || G < 1 || D < 4 || D % 4 || col0 % 4 || y.ld % 4 || y.slab % 4 || D > 1024 || dim < 1 || dim > D || rot % 2 || rot > dim || rot < 0 || bs < 1 ||
       (rot && !freq) || y.S < 1)
     return hipErrorInvalidValue;
   RopeParams p{y, col0, H, G, D, dim, rot, freq, 1.f / dim, eps, norm, positions, slots, q, kc, vc, bs, T};
 #define ROPE_NP(PT, AT)                                                                                      \
   do {                                                                                                       \
-    if (D <= 128) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 1>), dim3(T), dim3(256), 0, s, p);              \
-    else if (D <= 256) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 2>), dim3(T), dim3(256), 0, s, p);         \
-    else hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 8>), dim3(T), dim3(256), 0, s, p);                       \
+    if (D <= 64) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 16, 1>), dim3(T), dim3(256), 0, s, p);           \
+    else if (D <= 128) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 32, 1>), dim3(T), dim3(512), 0, s, p);     \
+    else if (D <= 256) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 64, 1>), dim3(T), dim3(512), 0, s, p);     \
+    else hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 64, 4>), dim3(T), dim3(512), 0, s, p);                   \
   } while (0)
   DAB_PROJ_DISPATCH(y, act_f32, ROPE_NP);
 #undef ROPE_NP

@@ -105,8 +105,8 @@ def qk_rope_write(y, col0: int, H: int, G: int, D: int, dim: int, rot: int, turn
     expect(dtype in _ACT and kc.is_contiguous() and vc.is_contiguous() and kc.shape == vc.shape and kc.shape[1] == G
            and kc.shape[3] == D and vc.dtype == dtype, "K / V caches [blocks, G, block_size, D]")
     expect(slots.dtype == torch.int64 and slots.is_contiguous() and slots.numel() == T, "slots: int64 [T]")
-    expect(D % 2 == 0 and D <= 1024 and 1 <= dim <= D and rot % 2 == 0 and 0 <= rot <= dim and col0 % 2 == 0
-           and py[4] % 2 == 0, "head sizes")
+    expect(D % 4 == 0 and D <= 1024 and 1 <= dim <= D and rot % 2 == 0 and 0 <= rot <= dim and col0 % 4 == 0
+           and py[4] % 4 == 0, "head sizes")
     expect(rot == 0 or (turns.dtype == torch.float64 and turns.numel() == rot // 2), "turns: fp64 [rot / 2]")
     expect(dtype == torch.bfloat16 or py[1] == 1, "an fp32 cache takes an fp32 projection")
     same_device(y, turns, positions, slots, kc)
@@ -251,8 +251,8 @@ def short_conv(y, col0: int, w, bias, ring, slot, pos, cu, max_q: int):
     py = _proj(y, T, col0 + C)
     _i32(slot), _i32(pos), _i32(cu)
     n = cu.numel() - 1
-    expect(w.dtype == torch.float32 and w.is_contiguous() and taps <= MAX_TAPS and C % 2 == 0 and col0 % 2 == 0
-           and py[4] % 2 == 0, "convolution: fp32 taps, even channels")
+    expect(w.dtype == torch.float32 and w.is_contiguous() and taps <= MAX_TAPS and C % 8 == 0 and col0 % 8 == 0
+           and py[4] % 8 == 0, "convolution: fp32 taps, channels in eights")
     expect(dtype in _ACT and ring.is_contiguous() and tuple(ring.shape[1:]) == (taps, C) and slot.numel() >= n, "ring")
     expect(dtype == torch.bfloat16 or py[1] == 1, "fp32 activations take an fp32 projection")
     if bias is not None:
