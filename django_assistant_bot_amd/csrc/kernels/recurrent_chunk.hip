@@ -29,7 +29,7 @@ namespace {
 constexpr int kC = 64;          // tokens of a chunk
 constexpr int kPairs = 6;       // (16-row tile, 32-deep step) pairs of a lower-triangular 64 x 64 operand
 constexpr int kFrag = 1024;     // bytes of one A fragment
-constexpr int kT = kPairs * 3 * kFrag, kA = kPairs * 2 * kFrag, kScal = 5 * kC * 4;
+constexpr int kT = kPairs * 3 * kFrag, kA = kPairs * 2 * kFrag, kScal = 2048;  // (5 rows of kC floats used)
 constexpr int kWs = kT + kA + kScal;  // workspace of one (chunk, head)
 
 __device__ __forceinline__ int pair_id(int m, int kb) { return m < 2 ? m : 2 + 2 * (m - 2) + kb; }
@@ -78,47 +78,57 @@ __device__ __forceinline__ bf16x8 cat4(const bf16x4& a, const bf16x4& b) {
   return bf16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
 }
 
+// The K | Q tile of a chunk, 16-B pieces e = tid + 256 i.  Loads are unconditional (a load behind a lane mask waits for
+// its data on the spot): rows past the portion repeat its last one, which zero betas and triangles keep out of every
+// result; columns past D become zeros.
+template <int D32>
+constexpr int kPieces = 2 * kC * 4 * D32 / 256;
+
+template <int D32>
+__device__ __forceinline__ void fetch_kq(const ChunkP& p, int row, int n, int hk, int tid, u32x4 (&pre)[kPieces<D32>]) {
+  constexpr int PR = 4 * D32;
+#pragma unroll
+  for (int i = 0; i < kPieces<D32>; ++i) {
+    const int e = tid + 256 * i, t = min(e / PR % kC, n - 1), ch = e % PR;
+    const int c = min(ch * 8, p.D - 8) + (e >= kC * PR ? p.q_col : p.k_col) + hk * p.D;
+    pre[i] = *reinterpret_cast<const u32x4*>(p.conv + (size_t)(row + t) * p.C + c);
+    if (ch * 8 >= p.D) pre[i] = u32x4{0, 0, 0, 0};
+  }
+}
+
+template <int D32>
+__device__ __forceinline__ void store_kq(char* lds, int tid, const u32x4 (&pre)[kPieces<D32>]) {
+  constexpr int PR = 4 * D32, STR = 64 * D32 + 16;
+#pragma unroll
+  for (int i = 0; i < kPieces<D32>; ++i) {
+    const int e = tid + 256 * i;
+    *reinterpret_cast<u32x4*>(lds + (e >= kC * PR ? kC * STR : 0) + e / PR % kC * STR + e % PR * 16) = pre[i];
+  }
+}
+
+// ssd: one workgroup per (chunk, q / k group), its products once, then decays and output head by head; delta: one
+// workgroup per (chunk, head), whose triangular solve is the longer part.
 template <int D32, bool DELTA>
 __global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkP p) {
   constexpr int Dp = 32 * D32, STR = Dp * 2 + 16, LD = 68;
-  constexpr int KQ = 2 * kC * STR, MA = 2 * kC * LD * 4;
+  constexpr int KQ = 2 * kC * STR, MA = (DELTA ? 2 : 1) * kC * LD * 4;
   __shared__ __attribute__((aligned(16))) char smem[KQ > MA ? KQ : MA];
   __shared__ double gam[kC];  // sums in fp64: their small differences are what counts
   __shared__ float be[kC], kk[kC], qq[kC];
   char* ks = smem;
   char* qs = smem + kC * STR;
-  float* Mm = reinterpret_cast<float*>(smem);
-  float* Am = Mm + kC * LD;
-  const int c = blockIdx.x, h = blockIdx.y, b = blockIdx.z, hk = h / (p.H / p.G);
+  float* Am = reinterpret_cast<float*>(smem);
+  float* Mm = Am + kC * LD;
+  const int rep = p.H / p.G;
+  const int c = blockIdx.x, hk = DELTA ? blockIdx.y / rep : blockIdx.y, b = blockIdx.z;
+  const int h_first = DELTA ? blockIdx.y : hk * rep, h_last = DELTA ? h_first : h_first + rep - 1;
   const int r0 = p.cu[b] + kC * c, n = min(kC, p.cu[b + 1] - r0);
   if (n <= 0) return;
   const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, g = lane >> 4, li = lane & 15;
-  char* ws = p.ws + ((size_t)(p.cu[b] / kC + b + c) * p.H + h) * kWs;
-  for (int i = tid; i < 2 * kC * (Dp / 8); i += 256) {
-    const int t = i / (Dp / 8) % kC, ch = i % (Dp / 8);
-    const bool q = i >= kC * (Dp / 8);
-    u32x4 v = {0, 0, 0, 0};
-    if (t < n && ch * 8 < p.D)
-      v = *reinterpret_cast<const u32x4*>(p.conv + (size_t)(r0 + t) * p.C + (q ? p.q_col : p.k_col) + hk * p.D + ch * 8);
-    *reinterpret_cast<u32x4*>((q ? qs : ks) + t * STR + ch * 16) = v;
-  }
-  if (w == 0) {
-    float beta = 0.f;
-    double dl = 0.;
-    if (lane < n) {
-      const float z = proj_f32<float>(p.gates, r0 + lane, p.a_col + h) + p.dt_bias[h];
-      const float dt = z > 20.f ? z : log1pf(__expf(z));
-      dl = -p.A[h] * dt;
-      beta = DELTA ? 1.f / (1.f + __expf(-proj_f32<float>(p.gates, r0 + lane, p.b_col + h))) : dt;
-    }
-#pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-      const double x = __shfl_up(dl, o, 64);
-      if (lane >= o) dl += x;
-    }
-    gam[lane] = dl;
-    be[lane] = beta;
-  }
+  u32x4 pre[kPieces<D32>];
+  fetch_kq<D32>(p, r0, n, hk, tid, pre);
+  store_kq<D32>(smem, tid, pre);
+  if (!DELTA && tid < kC) kk[tid] = qq[tid] = 1.f;
   __syncthreads();
   // rows 16 w .. of K K^T and Q K^T (lower triangle), and the diagonal of Q Q^T
   f32x4 kkt[4], qkt[4], qqt = {0.f, 0.f, 0.f, 0.f};
@@ -148,23 +158,6 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkP p) {
         }
     }
   }
-  if (!DELTA && tid < kC) kk[tid] = qq[tid] = 1.f;
-  __syncthreads();  // K / Q are done with: M and A take their place
-#pragma unroll
-  for (int nt = 0; nt < 4; ++nt)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int i = 16 * w + 4 * g + r, j = 16 * nt + li;
-      float m = 0.f, a = 0.f;
-      if (j <= i) {
-        const float e = __expf((float)(gam[i] - gam[j])) * kk[j];
-        a = e * qq[i] * qkt[nt][r];
-        if (DELTA && j < i) m = be[i] * e * kk[i] * kkt[nt][r];
-      }
-      if (DELTA) Mm[i * LD + j] = m;
-      Am[i * LD + j] = a;
-    }
-  __syncthreads();
   auto frag = [&](const float* src, int m, int kb, float(&x)[8]) {
     const float* s = src + (16 * m + li) * LD + 32 * kb + 4 * g;
     const f32x4 lo = *reinterpret_cast<const f32x4*>(s), hi = *reinterpret_cast<const f32x4*>(s + 16);
@@ -174,73 +167,109 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkP p) {
       x[4 + j] = hi[j];
     }
   };
-  if (w == 0) {
-    float* sc = reinterpret_cast<float*>(ws + kT + kA);
-    const float eg = __expf((float)gam[lane]);
-    sc[lane] = be[lane];
-    sc[kC + lane] = eg * kk[lane];
-    sc[2 * kC + lane] = eg * qq[lane];
-    sc[3 * kC + lane] = __expf((float)(gam[kC - 1] - gam[lane])) * kk[lane];
-    sc[4 * kC + lane] = eg;
-    if (DELTA) {
-      // column ``lane`` of T: t_i = [i == lane] - sum_{j < i} M_ij t_j
-      float t[kC];
-#pragma unroll
-      for (int i = 0; i < kC; ++i) {
-        float a[4] = {lane == i ? 1.f : 0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int j4 = 0; j4 < (i + 3) / 4; ++j4) {
-          const f32x4 mv = *reinterpret_cast<const f32x4*>(Mm + i * LD + 4 * j4);
-#pragma unroll
-          for (int q = 0; q < 4; ++q)
-            if (4 * j4 + q < i) a[q] = fmaf(-mv[q], t[4 * j4 + q], a[q]);
-        }
-        t[i] = (a[0] + a[1]) + (a[2] + a[3]);
+  auto row_of = [](int pr) { return pr < 2 ? pr : 2 + (pr - 2) / 2; };
+  auto step_of = [](int pr) { return pr < 2 ? 0 : (pr - 2) % 2; };
+  for (int h = h_first; h <= h_last; ++h) {
+    char* ws = p.ws + ((size_t)(p.cu[b] / kC + b + c) * p.H + h) * kWs;
+    __syncthreads();  // K / Q, or the previous head's matrices, are done with
+    if (w == 0) {
+      float beta = 0.f;
+      double dl = 0.;
+      if (lane < n) {
+        const float z = proj_f32<float>(p.gates, r0 + lane, p.a_col + h) + p.dt_bias[h];
+        const float dt = z > 20.f ? z : log1pf(__expf(z));
+        dl = -p.A[h] * dt;
+        beta = DELTA ? 1.f / (1.f + __expf(-proj_f32<float>(p.gates, r0 + lane, p.b_col + h))) : dt;
       }
 #pragma unroll
-      for (int i = 0; i < kC; ++i) Mm[i * LD + lane] = t[i];  // every read of M was this wave's own
+      for (int o = 1; o < 64; o <<= 1) {
+        const double x = __shfl_up(dl, o, 64);
+        if (lane >= o) dl += x;
+      }
+      gam[lane] = dl;
+      be[lane] = beta;
     }
-  }
-  auto put = [&](int pr, auto&& fn) {
-    const int m = pr < 2 ? pr : 2 + (pr - 2) / 2, kb = pr < 2 ? 0 : (pr - 2) % 2;
-    fn(m, kb);
-  };
-  if (w > 0)
-    for (int pr = w - 1; pr < kPairs; pr += 3)
-      put(pr, [&](int m, int kb) {
+    __syncthreads();
+#pragma unroll
+    for (int nt = 0; nt < 4; ++nt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = 16 * w + 4 * g + r, j = 16 * nt + li;
+        float m = 0.f, a = 0.f;
+        if (j <= i) {
+          const float e = __expf((float)(gam[i] - gam[j])) * kk[j];
+          a = e * qq[i] * qkt[nt][r];
+          if (DELTA && j < i) m = be[i] * e * kk[i] * kkt[nt][r];
+        }
+        if (DELTA) Mm[i * LD + j] = m;
+        Am[i * LD + j] = a;
+      }
+    __syncthreads();
+    if (w == 0) {
+      float* sc = reinterpret_cast<float*>(ws + kT + kA);
+      const float eg = __expf((float)gam[lane]);
+      sc[lane] = be[lane];
+      sc[kC + lane] = eg * kk[lane];
+      sc[2 * kC + lane] = eg * qq[lane];
+      sc[3 * kC + lane] = __expf((float)(gam[kC - 1] - gam[lane])) * kk[lane];
+      sc[4 * kC + lane] = eg;
+      if (DELTA) {
+        // column ``lane`` of T: t_i = [i == lane] - sum_{j < i} M_ij t_j
+        float t[kC];
+#pragma unroll
+        for (int i = 0; i < kC; ++i) {
+          float a[4] = {lane == i ? 1.f : 0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int j4 = 0; j4 < (i + 3) / 4; ++j4) {
+            const f32x4 mv = *reinterpret_cast<const f32x4*>(Mm + i * LD + 4 * j4);
+#pragma unroll
+            for (int q = 0; q < 4; ++q)
+              if (4 * j4 + q < i) a[q] = fmaf(-mv[q], t[4 * j4 + q], a[q]);
+          }
+          t[i] = (a[0] + a[1]) + (a[2] + a[3]);
+        }
+#pragma unroll
+        for (int i = 0; i < kC; ++i) Mm[i * LD + lane] = t[i];  // every read of M was this wave's own
+      }
+    }
+    if (w > 0 || !DELTA)
+      for (int pr = DELTA ? w - 1 : w; pr < kPairs; pr += DELTA ? 3 : 4) {
         float x[8];
         bf16x8 o[2];
-        frag(Am, m, kb, x);
+        frag(Am, row_of(pr), step_of(pr), x);
         split(x, o);
 #pragma unroll
         for (int s = 0; s < 2; ++s) *reinterpret_cast<bf16x8*>(ws + kT + (2 * pr + s) * kFrag + lane * 16) = o[s];
-      });
-  if (!DELTA) return;
-  __syncthreads();
-  for (int pr = w; pr < kPairs; pr += 4)
-    put(pr, [&](int m, int kb) {
+      }
+    if constexpr (!DELTA) continue;
+    __syncthreads();
+    for (int pr = w; pr < kPairs; pr += 4) {
       float x[8];
       bf16x8 o[3];
-      frag(Mm, m, kb, x);
+      frag(Mm, row_of(pr), step_of(pr), x);
       split(x, o);
 #pragma unroll
       for (int s = 0; s < 3; ++s) *reinterpret_cast<bf16x8*>(ws + (3 * pr + s) * kFrag + lane * 16) = o[s];
-    });
+    }
+  }
 }
 
+// LDS: the chunk's K | Q tile (rows prefetched into registers a chunk ahead) and its workspace block (T and A fragments,
+// row scales), copied by LDS-DMA as soon as every wave is done with the previous one.
 template <int D32, bool DELTA>
-__global__ __launch_bounds__(256) void chunk_scan_kernel(ChunkP p) {
+__global__ __launch_bounds__(256, 2) void chunk_scan_kernel(ChunkP p) {
   constexpr int Dp = 32 * D32, STR = Dp * 2 + 16, MT = 2 * D32;
-  constexpr int CH = 2 * kC * (Dp / 8) / 256;  // 16-B pieces of the K | Q tile per thread
-  static_assert(CH >= 1, "tile too small");
-  __shared__ __attribute__((aligned(16))) char smem[2 * kC * STR];
-  __shared__ __attribute__((aligned(16))) float sc[5][kC];  // beta, e^G k-norm, e^G q-norm, e^(G_C - G) k-norm, e^G
-  const char* ks = smem;
-  const char* qs = smem + kC * STR;
+  constexpr int P0 = DELTA ? 0 : kT / 1024, P1 = kWs / 1024;  // 1-KB pieces of the workspace block that are needed
+  __shared__ __attribute__((aligned(16))) char smem[2 * kC * STR + kWs];
+  char* const ks = smem;
+  char* const qs = smem + kC * STR;
+  char* const wl = smem + 2 * kC * STR;
+  const float* const sc = reinterpret_cast<const float*>(wl + kT + kA);  // beta, e^G k-norm, e^G q-norm, e^(G_C - G) k-norm, e^G
   const int h = blockIdx.y, b = blockIdx.z, hk = h / (p.H / p.G);
   const int q0 = p.cu[b], len = p.cu[b + 1] - q0;
   if (len <= 0) return;
-  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, g = lane >> 4, li = lane & 15;
+  const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, li = lane & 15;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int col = blockIdx.x * 64 + 16 * w + li;
   const bool live = blockIdx.x * 64 + 16 * w < p.V, mine = col < p.V;
   float* sp = p.state + (((size_t)p.slot[b] * p.H + h) * p.V + (mine ? col : 0)) * Dp + 4 * g;
@@ -252,176 +281,161 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(ChunkP p) {
     S[m] = fresh || !mine ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
   const float skip = !DELTA && p.skip ? p.skip[h] : 0.f;
   const int nc = (len + kC - 1) / kC;
-  u32x4 pre[CH];
-  auto fetch = [&](int c) {
+  u32x4 pre[kPieces<D32>];
+  auto fetch = [&](int c) { fetch_kq<D32>(p, q0 + kC * c, min(kC, len - kC * c), hk, tid, pre); };
+  auto copy_ws = [&](int c) {
+    const char* src = ws0 + (size_t)c * p.H * kWs + lane * 16;
+    for (int i = P0 + w; i < P1; i += 4)
+      __builtin_amdgcn_global_load_lds((const void*)(src + i * 1024),
+                                       (__attribute__((address_space(3))) void*)(wl + i * 1024), 16, 0, 0);
+  };
+  auto gather8 = [](const f32x4& a, const f32x4& c, float(&x)[8]) {
 #pragma unroll
-    for (int i = 0; i < CH; ++i) {
-      const int e = tid + 256 * i, t = e / (Dp / 8) % kC, ch = e % (Dp / 8);
-      const bool q = e >= kC * (Dp / 8);
-      pre[i] = u32x4{0, 0, 0, 0};
-      if (kC * c + t < len && ch * 8 < p.D)
-        pre[i] = *reinterpret_cast<const u32x4*>(p.conv + (size_t)(q0 + kC * c + t) * p.C + (q ? p.q_col : p.k_col) +
-                                                 hk * p.D + ch * 8);
+    for (int r = 0; r < 4; ++r) {
+      x[r] = a[r];
+      x[4 + r] = c[r];
     }
   };
+  auto scale4 = [&](int row, int m) { return *reinterpret_cast<const f32x4*>(sc + row * kC + 16 * m + 4 * g); };
   fetch(0);
+  copy_ws(0);
   for (int c = 0; c < nc; ++c) {
     const int n = min(kC, len - kC * c);
-    const char* ws = ws0 + (size_t)c * p.H * kWs;
     __syncthreads();  // the previous chunk's tile is done with
-#pragma unroll
-    for (int i = 0; i < CH; ++i) {
-      const int e = tid + 256 * i, t = e / (Dp / 8) % kC, ch = e % (Dp / 8);
-      *reinterpret_cast<u32x4*>(smem + (e >= kC * (Dp / 8) ? kC * STR : 0) + t * STR + ch * 16) = pre[i];
-    }
-    for (int i = tid; i < 5 * kC; i += 256) (&sc[0][0])[i] = reinterpret_cast<const float*>(ws + kT + kA)[i];
+    store_kq<D32>(smem, tid, pre);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's workspace pieces landed
     __syncthreads();
-    if (c + 1 < nc) fetch(c + 1);
-    if (!live) continue;  // (every wave reaches the barriers)
-    // values of this wave's columns in the accumulator layout
-    float R[4][4];
+    f32x4 R[4];  // values of this wave's columns in the accumulator layout
     const bf16* vp = p.conv + (size_t)(q0 + kC * c) * p.C + p.v_col + h * p.V + (mine ? col : 0);
 #pragma unroll
     for (int m = 0; m < 4; ++m)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = 16 * m + 4 * g + r;
-        R[m][r] = t < n && mine ? bf2f(vp[(size_t)t * p.C]) : 0.f;
-      }
-    bf16x8 ss[D32][3];  // the state as three bf16 terms
-#pragma unroll
-    for (int kb = 0; kb < D32; ++kb) {
-      float x[8];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        x[r] = S[2 * kb][r];
-        x[4 + r] = S[2 * kb + 1][r];
-      }
-      split(x, ss[kb]);
-    }
-    auto rows = [&](const char* src, int m, int kb) {  // A operand: 16 token rows, 32 state rows in slot order
-      const char* s = src + (16 * m + li) * STR + (32 * kb + 4 * g) * 2;
-      return cat4(*reinterpret_cast<const bf16x4*>(s), *reinterpret_cast<const bf16x4*>(s + 32));
-    };
-    auto times_s = [&](const char* src, int m) {
-      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+      for (int r = 0; r < 4; ++r) R[m][r] = bf2f(vp[(size_t)min(16 * m + 4 * g + r, n - 1) * p.C]);
+    if (c + 1 < nc) fetch(c + 1);
+    bf16x8 wu[2][3];
+    float ec = 0.f;
+    if (live) {
+      bf16x8 ss[D32][3];  // the state as three bf16 terms
 #pragma unroll
       for (int kb = 0; kb < D32; ++kb) {
-        const bf16x8 a = rows(src, m, kb);
-        acc = mfma16(a, ss[kb][2], acc);
-        acc = mfma16(a, ss[kb][1], acc);
-        acc = mfma16(a, ss[kb][0], acc);
+        float x[8];
+        gather8(S[2 * kb], S[2 * kb + 1], x);
+        split(x, ss[kb]);
       }
-      return acc;
-    };
-    f32x4 U[4], O[4];
-    float vskip[4][4];
-    if (!DELTA) {
+      auto times_s = [&](const char* src, int m) {  // A operand: 16 token rows, 32 state rows in slot order
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int m = 0; m < 4; ++m)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          vskip[m][r] = skip * R[m][r];
-          U[m][r] = sc[0][16 * m + 4 * g + r] * R[m][r];
+        for (int kb = 0; kb < D32; ++kb) {
+          const char* s = src + (16 * m + li) * STR + (32 * kb + 4 * g) * 2;
+          const bf16x8 a = cat4(*reinterpret_cast<const bf16x4*>(s), *reinterpret_cast<const bf16x4*>(s + 32));
+          acc = mfma16(a, ss[kb][2], acc);
+          acc = mfma16(a, ss[kb][1], acc);
+          acc = mfma16(a, ss[kb][0], acc);
         }
-    } else {
+        return acc;
+      };
+      f32x4 U[4], O[4];
+      if (DELTA) {
+        f32x4 P[4];
 #pragma unroll
-      for (int m = 0; m < 4; ++m) {
-        const f32x4 P = times_s(ks, m);
-        const f32x4 be = *reinterpret_cast<const f32x4*>(&sc[0][16 * m + 4 * g]);
-        const f32x4 ek = *reinterpret_cast<const f32x4*>(&sc[1][16 * m + 4 * g]);
+        for (int m = 0; m < 4; ++m) P[m] = times_s(ks, m);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) R[m][r] = be[r] * (R[m][r] - ek[r] * P[r]);
+        for (int m = 0; m < 4; ++m) O[m] = times_s(qs, m) * scale4(2, m);
+#pragma unroll
+        for (int m = 0; m < 4; ++m) R[m] = scale4(0, m) * (R[m] - scale4(1, m) * P[m]);
+        bf16x8 rs[2][3];
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb) {
+          float x[8];
+          gather8(R[2 * kb], R[2 * kb + 1], x);
+          split(x, rs[kb]);
+        }
+#pragma unroll
+        for (int m = 0; m < 4; ++m) {
+          f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int kb = 0; kb <= m / 2; ++kb) {
+            const char* f = wl + 3 * pair_id(m, kb) * kFrag + lane * 16;
+            const bf16x8 t0 = *reinterpret_cast<const bf16x8*>(f), t1 = *reinterpret_cast<const bf16x8*>(f + kFrag),
+                         t2 = *reinterpret_cast<const bf16x8*>(f + 2 * kFrag);
+            acc = mfma16(t2, rs[kb][0], acc);
+            acc = mfma16(t0, rs[kb][2], acc);
+            acc = mfma16(t1, rs[kb][1], acc);
+            acc = mfma16(t1, rs[kb][0], acc);
+            acc = mfma16(t0, rs[kb][1], acc);
+            acc = mfma16(t0, rs[kb][0], acc);
+          }
+          U[m] = acc;
+        }
+      } else {
+#pragma unroll
+        for (int m = 0; m < 4; ++m) {
+          O[m] = times_s(qs, m) * scale4(2, m) + skip * R[m];
+          U[m] = scale4(0, m) * R[m];
+        }
       }
-      bf16x8 rs[2][3];
+      // read-out
+      bf16x8 us[2][2];
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb) {
         float x[8];
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          x[r] = R[2 * kb][r];
-          x[4 + r] = R[2 * kb + 1][r];
-        }
-        split(x, rs[kb]);
+        gather8(U[2 * kb], U[2 * kb + 1], x);
+        split(x, us[kb]);
       }
 #pragma unroll
       for (int m = 0; m < 4; ++m) {
-        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int kb = 0; kb <= m / 2; ++kb) {
-          const char* f = ws + 3 * pair_id(m, kb) * kFrag + lane * 16;
-          const bf16x8 t0 = *reinterpret_cast<const bf16x8*>(f), t1 = *reinterpret_cast<const bf16x8*>(f + kFrag),
-                       t2 = *reinterpret_cast<const bf16x8*>(f + 2 * kFrag);
-          acc = mfma16(t2, rs[kb][0], acc);
-          acc = mfma16(t0, rs[kb][2], acc);
-          acc = mfma16(t1, rs[kb][1], acc);
-          acc = mfma16(t1, rs[kb][0], acc);
-          acc = mfma16(t0, rs[kb][1], acc);
-          acc = mfma16(t0, rs[kb][0], acc);
+          const char* f = wl + kT + 2 * pair_id(m, kb) * kFrag + lane * 16;
+          const bf16x8 a0 = *reinterpret_cast<const bf16x8*>(f), a1 = *reinterpret_cast<const bf16x8*>(f + kFrag);
+          O[m] = mfma16(a1, us[kb][0], O[m]);
+          O[m] = mfma16(a0, us[kb][1], O[m]);
+          O[m] = mfma16(a0, us[kb][0], O[m]);
         }
-        U[m] = acc;
       }
-    }
-    // read-out
-    bf16x8 us[2][2];
+      if (mine) {
+        bf16* op = p.out + (size_t)(q0 + kC * c) * p.H * p.V + h * p.V + col;
+        const size_t ld = (size_t)p.H * p.V;
+        if (n == kC) {
 #pragma unroll
-    for (int kb = 0; kb < 2; ++kb) {
-      float x[8];
+          for (int m = 0; m < 4; ++m)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        x[r] = U[2 * kb][r];
-        x[4 + r] = U[2 * kb + 1][r];
+            for (int r = 0; r < 4; ++r) op[(16 * m + 4 * g + r) * ld] = f2bf(O[m][r]);
+        } else {
+#pragma unroll
+          for (int m = 0; m < 4; ++m)
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+              if (16 * m + 4 * g + r < n) op[(16 * m + 4 * g + r) * ld] = f2bf(O[m][r]);
+        }
       }
-      split(x, us[kb]);
-    }
-#pragma unroll
-    for (int m = 0; m < 4; ++m) {
-      O[m] = times_s(qs, m);
-      O[m] *= *reinterpret_cast<const f32x4*>(&sc[2][16 * m + 4 * g]);
-#pragma unroll
-      for (int kb = 0; kb <= m / 2; ++kb) {
-        const char* f = ws + kT + 2 * pair_id(m, kb) * kFrag + lane * 16;
-        const bf16x8 a0 = *reinterpret_cast<const bf16x8*>(f), a1 = *reinterpret_cast<const bf16x8*>(f + kFrag);
-        O[m] = mfma16(a1, us[kb][0], O[m]);
-        O[m] = mfma16(a0, us[kb][1], O[m]);
-        O[m] = mfma16(a0, us[kb][0], O[m]);
-      }
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = 16 * m + 4 * g + r;
-        if (t < n && mine)
-          p.out[(size_t)(q0 + kC * c + t) * p.H * p.V + h * p.V + col] = f2bf(DELTA ? O[m][r] : O[m][r] + vskip[m][r]);
-      }
-    }
-    // state: S = e^(G_C) S + K^T (e^(G_C - G) U)
-    bf16x8 wu[2][3];
-#pragma unroll
-    for (int kb = 0; kb < 2; ++kb) {
-      float x[8];
-      const f32x4 w0 = *reinterpret_cast<const f32x4*>(&sc[3][32 * kb + 4 * g]);
-      const f32x4 w1 = *reinterpret_cast<const f32x4*>(&sc[3][32 * kb + 16 + 4 * g]);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        x[r] = U[2 * kb][r] * w0[r];
-        x[4 + r] = U[2 * kb + 1][r] * w1[r];
-      }
-      split(x, wu[kb]);
-    }
-    const float ec = sc[4][kC - 1];
-    const int tq = li >> 2, tp = li & 3;
-#pragma unroll
-    for (int m = 0; m < MT; ++m) {
-      f32x4 acc = S[m] * ec;
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb) {
-        const bf16x4 lo = ds_read_tr16(ks + (32 * kb + 4 * g + tq) * STR + (16 * m + 4 * tp) * 2);
-        const bf16x4 hi = ds_read_tr16(ks + (32 * kb + 16 + 4 * g + tq) * STR + (16 * m + 4 * tp) * 2);
-        const bf16x8 a = cat4(lo, hi);
-        acc = mfma16(a, wu[kb][2], acc);
-        acc = mfma16(a, wu[kb][1], acc);
-        acc = mfma16(a, wu[kb][0], acc);
+        float x[8];
+        gather8(U[2 * kb] * scale4(3, 2 * kb), U[2 * kb + 1] * scale4(3, 2 * kb + 1), x);
+        split(x, wu[kb]);
       }
-      S[m] = acc;
+      ec = sc[4 * kC + kC - 1];
+    }
+    __syncthreads();  // every wave is done with the workspace block
+    if (c + 1 < nc) copy_ws(c + 1);
+    if (live) {
+      // state: S = e^(G_C) S + K^T (e^(G_C - G) U)
+      const int tq = li >> 2, tp = li & 3;
+#pragma unroll
+      for (int m = 0; m < MT; ++m) {
+        f32x4 acc = S[m] * ec;
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb) {
+          const bf16x4 lo = ds_read_tr16(ks + (32 * kb + 4 * g + tq) * STR + (16 * m + 4 * tp) * 2);
+          const bf16x4 hi = ds_read_tr16(ks + (32 * kb + 16 + 4 * g + tq) * STR + (16 * m + 4 * tp) * 2);
+          const bf16x8 a = cat4(lo, hi);
+          acc = mfma16(a, wu[kb][2], acc);
+          acc = mfma16(a, wu[kb][1], acc);
+          acc = mfma16(a, wu[kb][0], acc);
+        }
+        S[m] = acc;
+      }
     }
   }
   if (mine) {
@@ -467,7 +481,7 @@ int state_chunks(const void* conv, RecurrentShape d, Proj gates, const float* A,
   p.out = (bf16*)out;
   p.ws = (char*)ws;
   p.qscale = 1.f / sqrtf((float)d.D);
-  const dim3 gp((max_q + kC - 1) / kC, d.H, chunks), gs((d.V + 63) / 64, d.H, chunks);
+  const dim3 gp((max_q + kC - 1) / kC, d.delta ? d.H : d.G, chunks), gs((d.V + 63) / 64, d.H, chunks);
 #define CHUNK_L(D32)                                                                               \
   do {                                                                                             \
     if (d.delta) {                                                                                 \
