@@ -297,6 +297,13 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
 
 template <int EPI, bool SHUF>
 static int launch_gemm(const GemmParams& p, bool big, hipStream_t s) {
+  if constexpr (EPI == EPI_NONE && SHUF) {
+    // a narrow product (router logits, recurrence gates): 32-row tiles, or its few workgroups leave most CUs idle
+    if (p.N <= 128 && p.M > 128) {
+      hipLaunchKernelGGL((gemm_bt_kernel<EPI, 32, 128, 1, 4, SHUF>), dim3((p.M + 31) / 32), dim3(256), 0, s, p);
+      return hipGetLastError();
+    }
+  }
   if (big) {
     const int nwg = ((p.M + 255) / 256) * ((p.N + 255) / 256);
     hipLaunchKernelGGL((gemm_bt_kernel<EPI, 256, 256, 2, 4, SHUF>), dim3(nwg), dim3(512), 0, s, p);
@@ -361,7 +368,7 @@ int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
 int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int N, int K, const int* perm, int a_div,
                  int scatter, const void* tiles, int n_tiles, int bm, int glu, const float* row_scale, hipStream_t s) {
   if (n_tiles <= 0 || N <= 0) return 0;
-  if (K % 64 || N % 32 || lda % 8 || ldc % 4 || !tiles || !perm || (bm != 32 && bm != 128) || (row_scale && !glu))
+  if (K % 64 || N % 32 || lda % 8 || ldc % 4 || !tiles || !perm || (bm != 32 && bm != 128 && bm != 256) || (row_scale && !glu))
     return hipErrorInvalidValue;
   GemmParams p{};
   p.A = (const bf16*)A;
@@ -379,10 +386,14 @@ int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int 
   p.a_div = a_div;
   p.scatter = scatter;
   p.row_scale = row_scale;
-  const dim3 grid((unsigned)n_tiles * ((N + 127) / 128));
+  const int bn = bm == 256 ? 256 : 128;
+  const dim3 grid((unsigned)n_tiles * ((N + bn - 1) / bn));
   if (bm == 32) {
     if (glu) hipLaunchKernelGGL((gemm_bt_kernel<EPI_SWIGLU8, 32, 128, 1, 4, true, true>), grid, dim3(256), 0, s, p);
     else hipLaunchKernelGGL((gemm_bt_kernel<EPI_NONE, 32, 128, 1, 4, true, true>), grid, dim3(256), 0, s, p);
+  } else if (bm == 256) {
+    if (glu) hipLaunchKernelGGL((gemm_bt_kernel<EPI_SWIGLU8, 256, 256, 2, 4, true, true>), grid, dim3(512), 0, s, p);
+    else hipLaunchKernelGGL((gemm_bt_kernel<EPI_NONE, 256, 256, 2, 4, true, true>), grid, dim3(512), 0, s, p);
   } else {
     if (glu) hipLaunchKernelGGL((gemm_bt_kernel<EPI_SWIGLU8, 128, 128, 2, 2, true, true>), grid, dim3(256), 0, s, p);
     else hipLaunchKernelGGL((gemm_bt_kernel<EPI_NONE, 128, 128, 2, 2, true, true>), grid, dim3(256), 0, s, p);

@@ -149,7 +149,7 @@ int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
             long ldr, int M, int N, int K, int epilogue, int out_f32, const int* row_group, const int* q_group,
             const uint32_t* allow, int allow_words, hipStream_t s, int b_rows = 0, int b_group = 1);
 // experts: like gemm_f32_grouped, bf16, B = per-expert shuffle_weights copies of N rows; glu: SwiGLU over 8-row groups,
-// each row times row_scale[pair].  bm: rows of a tile (32 or 128)
+// each row times row_scale[pair].  bm: rows of a tile (32, 128 or 256)
 int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int N, int K, const int* perm, int a_div,
                  int scatter, const void* tiles, int n_tiles, int bm, int glu, const float* row_scale, hipStream_t s);
 

@@ -40,7 +40,7 @@ __device__ __forceinline__ float sum8(float v) {
 struct ConvParams {
   Proj y;
   int col0, C, taps;
-  const float* w;     // [C, taps]
+  const float* w;     // [taps, C]
   const float* bias;  // [C] or null
   void* ring;         // [slots, taps, C]
   const int* slot;    // [chunks]
@@ -49,7 +49,7 @@ struct ConvParams {
   void* out;          // [T, C]
 };
 
-constexpr int kConvTokens = 16;  // tokens a thread walks
+constexpr int kConvTokens = 32;  // tokens a thread walks
 
 template <typename PT, typename AT, int K>
 __global__ __launch_bounds__(256) void short_conv_kernel(ConvParams p) {
@@ -60,44 +60,65 @@ __global__ __launch_bounds__(256) void short_conv_kernel(ConvParams p) {
   const AT* ring = (const AT*)p.ring + (size_t)p.slot[b] * p.taps * p.C;
   float w[K][8], win[K][8], bias[8];
 #pragma unroll
-  for (int j = 0; j < 8; ++j) {
-    bias[j] = p.bias ? p.bias[c + j] : 0.f;
+  for (int j = 0; j < 8; ++j) bias[j] = 0.f;
+  if (p.bias) ElemIO<float>::load8(p.bias + c, bias);
 #pragma unroll
-    for (int k = 0; k < K; ++k) {
-      const int tap = k - (K - p.taps);
-      w[k][j] = tap >= 0 ? p.w[(size_t)(c + j) * p.taps + tap] : 0.f;
+  for (int k = 0; k < K; ++k) {
+    const int tap = k - (K - p.taps);
+    ElemIO<float>::load8(p.w + (size_t)max(tap, 0) * p.C + c, w[k]);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      if (tap < 0) w[k][j] = 0.f;
       win[k][j] = 0.f;
     }
   }
-  auto input = [&](int t, float(&v)[8]) {  // input of the chunk's token t, which may lie before the chunk
-    if (t >= 0) {
-      proj8<PT>(p.y, r0 + t, p.col0 + c, v);
+  auto token = [&](int t, float(&v)[8]) {  // input of the chunk's token t
+    proj8<PT>(p.y, r0 + t, p.col0 + c, v);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) v[j] = ElemIO<AT>::round(v[j]);
-    } else if (pos0 + t >= 0) {
-      ElemIO<AT>::load8(ring + (size_t)((pos0 + t) % p.taps) * p.C + c, v);
-    }
+    for (int j = 0; j < 8; ++j) v[j] = ElemIO<AT>::round(v[j]);
   };
 #pragma unroll
-  for (int k = 1; k < K; ++k)  // the inputs before t0: win[k] = token t0 - (K - k)
-    if (K - k <= p.taps - 1) input(t0 - (K - k), win[k]);
-  // token t0 + i goes to window entry i % K, so nothing is shifted
-  static_assert(kConvTokens % K == 0, "whole turns of the window");
+  for (int k = 1; k < K; ++k) {  // the inputs before t0: win[k] = token t0 - (K - k), which may lie before the chunk
+    const int t = t0 - (K - k);
+    if (K - k > p.taps - 1) continue;
+    if (t >= 0) token(t, win[k]);
+    else if (pos0 + t >= 0) ElemIO<AT>::load8(ring + (size_t)((pos0 + t) % p.taps) * p.C + c, win[k]);
+  }
+  // token t0 + i goes to window entry i % K, so nothing is shifted; inputs are requested PF tokens ahead
+  constexpr int PF = K < 4 || K > 8 ? 2 : 4;
+  static_assert(kConvTokens % K == 0 && K % PF == 0, "whole turns of the window");
   const int t1 = min(n, t0 + kConvTokens);
+  float nx[PF][8];
+#pragma unroll
+  for (int i = 0; i < PF; ++i) token(min(t0 + i, t1 - 1), nx[i]);
   for (int t = t0; t < t1; t += K) {
 #pragma unroll
-    for (int i = 0; i < K; ++i) {
-      if (t + i >= t1) break;  // (uniform in the workgroup)
-      input(t + i, win[i]);
-      float o[8];
+    for (int i0 = 0; i0 < K; i0 += PF) {
+      if (t + i0 >= t1) break;  // (uniform in the workgroup)
+      float in[PF][8];
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        o[j] = bias[j];
+      for (int i = 0; i < PF; ++i)
 #pragma unroll
-        for (int k = 0; k < K; ++k) o[j] = fmaf(w[k][j], win[(i + 1 + k) % K][j], o[j]);
-        o[j] = silu_f(o[j]);
+        for (int j = 0; j < 8; ++j) in[i][j] = nx[i][j];
+#pragma unroll
+      for (int i = 0; i < PF; ++i) token(min(t + i0 + PF + i, t1 - 1), nx[i]);
+#pragma unroll
+      for (int i = 0; i < PF; ++i) {
+        if (t + i0 + i >= t1) break;
+        float o[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          win[i0 + i][j] = in[i][j];
+          o[j] = bias[j];
+        }
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+#pragma unroll
+          for (int k = 0; k < K; ++k) o[j] = fmaf(w[k][j], win[(i0 + i + 1 + k) % K][j], o[j]);
+          o[j] = silu_f(o[j]);
+        }
+        ElemIO<AT>::store8((AT*)p.out + (size_t)(r0 + t + i0 + i) * p.C + c, o);
       }
-      ElemIO<AT>::store8((AT*)p.out + (size_t)(r0 + t + i) * p.C + c, o);
     }
   }
 }
@@ -124,7 +145,8 @@ int short_conv(Proj y, int col0, int C, int taps, const float* w, const float* b
   const dim3 grid((C / 8 + 255) / 256, (max_q + kConvTokens - 1) / kConvTokens, chunks);
 #define CONV_K(PT, AT)                                                                                        \
   do {                                                                                                        \
-    if (taps <= 4) hipLaunchKernelGGL((short_conv_kernel<PT, AT, 4>), grid, dim3(256), 0, s, p);              \
+    if (taps <= 2) hipLaunchKernelGGL((short_conv_kernel<PT, AT, 2>), grid, dim3(256), 0, s, p);              \
+    else if (taps <= 4) hipLaunchKernelGGL((short_conv_kernel<PT, AT, 4>), grid, dim3(256), 0, s, p);              \
     else if (taps <= 8) hipLaunchKernelGGL((short_conv_kernel<PT, AT, 8>), grid, dim3(256), 0, s, p);         \
     else hipLaunchKernelGGL((short_conv_kernel<PT, AT, 16>), grid, dim3(256), 0, s, p);                       \
     hipLaunchKernelGGL((conv_ring_kernel<PT, AT>), dim3((C + 255) / 256, taps, chunks), dim3(256), 0, s, p);  \
@@ -399,10 +421,10 @@ __global__ __launch_bounds__(256) void state_decode_kernel(DecodeStep a) {
     float v = 0.f;
     if (ch >= 0) {
       const float cur = proj_at<PT, AT>(a.y, row, a.col0 + ch);
-      const float* cw = a.w + (size_t)ch * a.taps;
-      float acc = fmaf(cw[a.taps - 1], cur, a.bias ? a.bias[ch] : 0.f);
+      const float* cw = a.w + ch;
+      float acc = fmaf(cw[(size_t)(a.taps - 1) * p.C], cur, a.bias ? a.bias[ch] : 0.f);
       for (int j = 1; j < a.taps && j <= pos; ++j)
-        acc = fmaf(cw[a.taps - 1 - j], ElemIO<AT>::load(ring + (size_t)((pos - j) % a.taps) * p.C + ch), acc);
+        acc = fmaf(cw[(size_t)(a.taps - 1 - j) * p.C], ElemIO<AT>::load(ring + (size_t)((pos - j) % a.taps) * p.C + ch), acc);
       ElemIO<AT>::store(ring + (size_t)(pos % a.taps) * p.C + ch, cur);
       v = ElemIO<AT>::round(silu_f(acc));
     }

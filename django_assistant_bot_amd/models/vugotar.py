@@ -103,7 +103,7 @@ class VugotarModel(FragmentProjections):
             return ops.shuffle_weights(t, g)
 
         def vec(key):
-            return take(key).to(self.device) if key in weights else None
+            return take(key).to(self.device).contiguous() if key in weights else None
 
         self.embed = take("embed").to(self.device)
         self.lm_head = mat("lm_head")
@@ -140,7 +140,7 @@ class VugotarModel(FragmentProjections):
     # ------------------------------------------------------------------ what the engine asks of a family
     def _specs(self):
         L = [self.layers[li] for li, _ in self.runs]
-        return [((x.attn.kv_heads, x.D) if x.attn else None, (x.conv_w.shape[1], x.rec)) for x in L]
+        return [((x.attn.kv_heads, x.D) if x.attn else None, (x.conv_w.shape[0], x.rec)) for x in L]
 
     def make_cache(self, num_blocks: int, block_size: int, slots: int = 1) -> HybridCache:
         return HybridCache(self._specs(), num_blocks, block_size, slots, self.device, self.dtype)

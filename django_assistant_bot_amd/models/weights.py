@@ -447,7 +447,7 @@ def _vugotar_layout(cfg: VugotarConfig, get, device, dtype, interleave_mlp) -> d
             q += "right."
             rows = {"q": d.kv_heads * d.dim, "k": d.kv_heads * d.dim, "v": d.heads * d.vdim}
             inp["conv"] = torch.cat([mat(q + n, r, W) for n, r in rows.items()])
-            w[p + "conv_w"] = _pad(torch.cat([vec(q + n + ".conv", r, d.conv) for n, r in rows.items()]), lay.conv, d.conv)
+            w[p + "conv_w"] = _pad(torch.cat([vec(q + n + ".conv", r, d.conv) for n, r in rows.items()]).t(), d.conv, lay.conv)
             inp["gate"] = mat(q + "g", d.heads * d.vdim, W)
             aux["a"], aux["b"] = mat(q + "a", d.heads, W), mat(q + "b", d.heads, W)
             w[p + "rec_norm"] = vec(q + "norm", d.vdim)
@@ -457,7 +457,7 @@ def _vugotar_layout(cfg: VugotarConfig, get, device, dtype, interleave_mlp) -> d
             conv = rec + 2 * m.groups * m.state
             full = mat(q + "in", rec + conv + heads, W)
             inp["gate"], inp["conv"], aux["a"] = full[:rec], full[rec:rec + conv], full[rec + conv:]
-            w[p + "conv_w"] = _pad(vec(q + "conv", conv, m.conv), lay.conv, m.conv)
+            w[p + "conv_w"] = _pad(vec(q + "conv", conv, m.conv).t(), m.conv, lay.conv)
             w[p + "conv_b"] = _pad(vec(q + "conv.b", conv), lay.conv)
             w[p + "skip"], w[p + "rec_norm"] = vec(q + "D", heads), vec(q + "norm", rec)
         out[:W, lay.mix:lay.mix + rec] = mat(q + "o", W, rec)

@@ -241,10 +241,10 @@ def _check_state(d: RecurrentShape, z, T, A, dt_bias, skip, state, slot, ring=No
 
 
 def short_conv(y, col0: int, w, bias, ring, slot, pos, cu, max_q: int):
-    """Causal convolution (``w`` fp32 [C, taps], last tap = the token) and silu of the portions ``cu`` of columns
+    """Causal convolution (``w`` fp32 [taps, C], last tap = the token) and silu of the portions ``cu`` of columns
     col0.. of a projection; inputs before a portion come from ``ring`` [slots, taps, C], which is brought up to
     date.  -> [T, C]."""
-    C, taps = w.shape
+    taps, C = w.shape
     T, dtype = pos.numel(), ring.dtype
     if not y.is_cuda:
         return ref.short_conv(y, col0, C, w, bias, ring, slot, pos, ref._spans(cu, 0, 0), dtype)
@@ -300,7 +300,7 @@ def state_decode(y, col0: int, w, bias, ring, d: RecurrentShape, z, A, dt_bias, 
     """One decoded token per sequence, rows row0.. of the projections: convolution, ring, gates, state update and
     read-out.  delta: also the per-head norm (``norm`` [V]) and the silu gate (columns g_col..), out_scale * result into
     ``out`` [T, >= H V + pad] (``pad`` zero columns behind it); ssd: the read-out into ``out`` [T, H V]."""
-    B, taps, dtype = slot.numel(), w.shape[1], ring.dtype
+    B, taps, dtype = slot.numel(), w.shape[0], ring.dtype
     n = d.H * d.V
     if not y.is_cuda:
         spans = ref._spans(None, B, row0)
@@ -315,7 +315,7 @@ def state_decode(y, col0: int, w, bias, ring, d: RecurrentShape, z, A, dt_bias, 
     py = _proj(y, T, max(col0 + d.C, g_col + n if d.delta else 0))
     pz = _check_state(d, z, T, A, dt_bias, skip, state, slot, ring, taps)
     _i32(pos)
-    expect(w.dtype == torch.float32 and w.is_contiguous() and tuple(w.shape) == (d.C, taps) and taps <= MAX_TAPS, "taps")
+    expect(w.dtype == torch.float32 and w.is_contiguous() and tuple(w.shape) == (taps, d.C) and taps <= MAX_TAPS, "taps")
     expect(dtype == torch.bfloat16 or py[1] == 1, "fp32 activations take an fp32 projection")
     expect(pos.numel() >= T, "positions")
     if bias is not None:
@@ -388,7 +388,7 @@ def moe_experts(h, idx, wt, gate_up, down, E: int, group: int):
     expect(wt.dtype == torch.float32 and wt.is_contiguous() and tuple(wt.shape) == (T, top), "expert weights per token")
     same_device(h, idx, wt, gate_up, down)
     f32 = h.dtype == torch.float32
-    bm = 64 if f32 else 32 if P <= 48 * E else 128
+    bm = 64 if f32 else 32 if P <= 48 * E else 128 if P <= 400 * E else 256  # rows of a tile, by the mean load
     n_tiles = min(P, E) + P // bm
     dev, s, nat = h.device, stream(h), native()
     perm = torch.empty((P,), dtype=torch.int32, device=dev)

@@ -77,13 +77,13 @@ def _spans(cu, T, row0):
 def short_conv(y, col0, C, w, bias, ring, slot, pos, cu, dtype):
     """Convolves every portion (``cu``) or one token per sequence and updates the rings; -> [T, C]."""
     x = total(y)[:, col0:col0 + C].to(dtype)
-    taps = w.shape[1]
+    taps = w.shape[0]
     out = torch.zeros(x.shape[0], C)
     for b, (a, e) in enumerate(cu):
         p0, s = int(pos[a]), int(slot[b])
         past = [ring[s, p % taps].float() if p >= 0 else torch.zeros(C) for p in range(p0 - taps + 1, p0)]
         xs = torch.cat([torch.stack(past) if past else torch.zeros(0, C), x[a:e].float()])
-        o = sum(xs[k:k + e - a] * w[:, k] for k in range(taps))
+        o = sum(xs[k:k + e - a] * w[k] for k in range(taps))
         out[a:e] = F.silu(o if bias is None else o + bias)
         for t in range(max(0, e - a - taps), e - a):
             ring[s, (p0 + t) % taps] = x[a + t]

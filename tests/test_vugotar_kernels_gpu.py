@@ -137,7 +137,7 @@ def recurrence(name, T, seed=0, decay=-2.0):
     cols = (0, n, 2 * n) if delta else (H * V + n, H * V, 0)
     d = ops.RecurrentShape(delta, H, G, D, V, C, *cols, 1, H + 2)
     y = rnd(T, 16 + C + H * V, seed=seed)
-    w, bias = rnd(C, taps, seed=seed + 1, dtype=F32, scale=taps ** -0.5), None if delta else rnd(C, seed=seed + 2, dtype=F32, scale=0.2)
+    w, bias = rnd(taps, C, seed=seed + 1, dtype=F32, scale=taps ** -0.5), None if delta else rnd(C, seed=seed + 2, dtype=F32, scale=0.2)
     z = rnd(T, 2 * H + 5, seed=seed + 3, dtype=F32)
     A, dtb = rnd(H, seed=seed + 4, dtype=F32, scale=0.5).exp(), rnd(H, seed=seed + 5, dtype=F32, scale=0.5) + decay
     skip = None if delta else rnd(H, seed=seed + 6, dtype=F32)
@@ -178,7 +178,7 @@ def test_short_conv_and_ring(name, dtype):
         for b in range(3):
             got[b].append(out[cu[b]:cu[b + 1]].cpu())
     for b in range(3):
-        want = oracle.short_conv(ys[b][:, 16:16 + d.C].double(), w.double(), None if bias is None else bias.double())
+        want = oracle.short_conv(ys[b][:, 16:16 + d.C].double(), w.double().T, None if bias is None else bias.double())
         close(torch.cat(got[b]), want, 6e-3 if dtype == BF else 2e-6)
 
 
@@ -262,7 +262,7 @@ def test_state_decode(name, yt, dtype):
         got.append(out[1:1 + B, :n].cpu())
     got = torch.stack(got)
     for b in range(B):
-        conv = oracle.short_conv(y[:, b, 16:16 + d.C].double(), w.double(), None if bias is None else bias.double())
+        conv = oracle.short_conv(y[:, b, 16:16 + d.C].double(), w.double().T, None if bias is None else bias.double())
         conv = conv.to(dtype)
         o, S = oracle_scan(d, conv, z[:, b], A, dtb, skip)
         if d.delta:
@@ -306,7 +306,8 @@ def test_moe_route(T, E, top, S):
 
 
 @pytest.mark.parametrize("T,E,top,K,F,W", [(1, 4, 2, 128, 64, 128), (7, 16, 4, 256, 128, 256), (150, 8, 3, 512, 192, 384),
-                                           (600, 5, 2, 256, 64, 256), (40, 70, 5, 128, 64, 128), (1000, 3, 3, 128, 128, 128)])
+                                           (600, 5, 2, 256, 64, 256), (40, 70, 5, 128, 64, 128), (1000, 3, 3, 128, 128, 128),
+                                           (900, 3, 2, 192, 192, 320)])
 @pytest.mark.parametrize("dtype", [BF, F32])
 def test_moe_experts(T, E, top, K, F, W, dtype):
     """Unequal loads, one expert that nobody chose and one that everybody did."""

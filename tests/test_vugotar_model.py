@@ -229,7 +229,7 @@ def test_mechanisms_against_the_oracle():
     xin, taps_w, b = R(9, C), R(C, taps), R(C)
     ring, out = torch.zeros(2, taps, C), []
     for a, e in ((0, 2), (2, 3), (3, 9)):
-        out.append(ops.short_conv(xin[a:e].float(), 0, taps_w.float(), b.float(), ring, torch.tensor([1]),
+        out.append(ops.short_conv(xin[a:e].float(), 0, taps_w.t().float(), b.float(), ring, torch.tensor([1]),
                                   torch.arange(a, e, dtype=torch.int32), torch.tensor([0, e - a]), e - a))
     near(torch.cat(out), oracle.short_conv(xin, taps_w, b))
     # both recurrences, a portion and then decoded tokens
