@@ -65,7 +65,9 @@ def decode_step(eng, batch, ctx):
     for i in range(batch):
         assert eng.blocks.add_sequence(i, [rng.randrange(eng.cfg.vocab_size) for _ in range(ctx - 1)], 0) == 0
     h = (eng._h_ids, eng._h_pos, eng._h_slots, eng._h_ctx, eng._h_bt)
-    assert eng.blocks.prepare_decode_into(list(range(batch)), [1] * batch, eng.max_blocks_per_seq,
+    # tokens of their own, so that experts are loaded as unequal requests load them
+    assert eng.blocks.prepare_decode_into(list(range(batch)), [rng.randrange(eng.cfg.vocab_size) for _ in range(batch)],
+                                          eng.max_blocks_per_seq,
                                           *(t.data_ptr() for t in h)) < 0
     eng._decode_logits(batch)
     key = (next(b for b in eng._buckets if b >= batch), True, False)

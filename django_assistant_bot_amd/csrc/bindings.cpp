@@ -248,6 +248,9 @@ PYBIND11_MODULE(_native, m) {
   m.def("shared_glu", [proj](const P& y, int col0, int F, const P& z, int sg_col, u out, long ldo, int act_f32, int T, u s) {
     check(dab::shared_glu(proj(y), col0, F, proj(z), sg_col, VP(out), ldo, act_f32, T, ST(s)), "shared_glu");
   });
+  m.def("gemm_narrow", [](u A, long lda, u B, u C, int M, int N, int K, int S, u s) {
+    check(dab::gemm_narrow(CVP(A), lda, CVP(B), (float*)C, M, N, K, S, ST(s)), "gemm_narrow");
+  });
   m.def("gemm_grouped", [](u A, long lda, u B, u C, long ldc, int N, int K, u perm, int a_div, int scatter, u tiles,
                            int n_tiles, int bm, int glu, u row_scale, u s) {
     check(dab::gemm_grouped(CVP(A), lda, CVP(B), VP(C), ldc, N, K, (const int*)perm, a_div, scatter, CVP(tiles), n_tiles,

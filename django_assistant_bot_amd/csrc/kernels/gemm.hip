@@ -139,12 +139,14 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
 #pragma unroll
     for (int j = 0; j < MI; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
 
-  const int nk = p.K / BK;
-  stage(0, 0);
+  // gridDim.y > 1 (gemm_narrow): slab blockIdx.y of the K range, into C [slabs][M][ldc]
+  const int nk = p.K / BK / gridDim.y, kb = blockIdx.y * nk * BK;
+  if (blockIdx.y) p.C = (float*)p.C + (size_t)blockIdx.y * p.M * p.ldc;
+  stage(0, kb);
   for (int kt = 0; kt < nk; ++kt) {
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
-    if (kt + 1 < nk) stage((kt + 1) & 1, (kt + 1) * BK);
+    if (kt + 1 < nk) stage((kt + 1) & 1, kb + (kt + 1) * BK);
     const char* As = smem + (kt & 1) * (TILE_A + TILE_B);
     const char* Bs = As + TILE_A;
 #pragma unroll
@@ -297,13 +299,6 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
 
 template <int EPI, bool SHUF>
 static int launch_gemm(const GemmParams& p, bool big, hipStream_t s) {
-  if constexpr (EPI == EPI_NONE && SHUF) {
-    // a narrow product (router logits, recurrence gates): 32-row tiles, or its few workgroups leave most CUs idle
-    if (p.N <= 128 && p.M > 128) {
-      hipLaunchKernelGGL((gemm_bt_kernel<EPI, 32, 128, 1, 4, SHUF>), dim3((p.M + 31) / 32), dim3(256), 0, s, p);
-      return hipGetLastError();
-    }
-  }
   if (big) {
     const int nwg = ((p.M + 255) / 256) * ((p.N + 255) / 256);
     hipLaunchKernelGGL((gemm_bt_kernel<EPI, 256, 256, 2, 4, SHUF>), dim3(nwg), dim3(512), 0, s, p);
@@ -363,6 +358,27 @@ int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
     case EPI_GEGLU8: return launch_gemm<EPI_GEGLU8>(p, big, s, sh);
     default: return hipErrorInvalidValue;
   }
+}
+
+int gemm_narrow(const void* A, long lda, const void* B, float* C, int M, int N, int K, int S, hipStream_t s) {
+  if (M <= 0 || N <= 0) return 0;
+  if (S < 1 || S > 64 || K % (64 * S) || N % 16 || lda % 8) return hipErrorInvalidValue;
+  GemmParams p{};
+  p.A = (const bf16*)A;
+  p.B = (const bf16*)B;
+  p.C = C;
+  p.M = M;
+  p.N = N;
+  p.K = K;
+  p.lda = lda;
+  p.ldb = K;
+  p.ldc = N;
+  p.out_f32 = 1;
+  p.rows_b = N;
+  p.bgrp = 1;
+  hipLaunchKernelGGL((gemm_bt_kernel<EPI_NONE, 32, 128, 1, 4, true>), dim3(((M + 31) / 32) * ((N + 127) / 128), S), dim3(256), 0,
+                     s, p);
+  return hipGetLastError();
 }
 
 int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int N, int K, const int* perm, int a_div,

@@ -148,6 +148,8 @@ int latent_any(void* out, const void* q, const void* cache, int f32, const int* 
 int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc, const void* bias, const void* residual,
             long ldr, int M, int N, int K, int epilogue, int out_f32, const int* row_group, const int* q_group,
             const uint32_t* allow, int allow_words, hipStream_t s, int b_rows = 0, int b_group = 1);
+// a narrow fp32 product (router logits, recurrence gates) as S split-K slabs [S][M][N]: 32-row tiles, B a shuffle_weights copy
+int gemm_narrow(const void* A, long lda, const void* B, float* C, int M, int N, int K, int S, hipStream_t s);
 // experts: like gemm_f32_grouped, bf16, B = per-expert shuffle_weights copies of N rows; glu: SwiGLU over 8-row groups,
 // each row times row_scale[pair].  bm: rows of a tile (32, 128 or 256)
 int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int N, int K, const int* perm, int a_div,

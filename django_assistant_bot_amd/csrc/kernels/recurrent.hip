@@ -47,14 +47,13 @@ struct ConvParams {
   const int* pos;     // [T]
   const int* cu;      // [chunks + 1]
   void* out;          // [T, C]
+  int span;           // tokens a thread walks, whole turns of the window
 };
-
-constexpr int kConvTokens = 32;  // tokens a thread walks
 
 template <typename PT, typename AT, int K>
 __global__ __launch_bounds__(256) void short_conv_kernel(ConvParams p) {
   const int b = blockIdx.z, c = (blockIdx.x * 256 + threadIdx.x) * 8;
-  const int r0 = p.cu[b], n = p.cu[b + 1] - r0, t0 = blockIdx.y * kConvTokens;
+  const int r0 = p.cu[b], n = p.cu[b + 1] - r0, t0 = blockIdx.y * p.span;
   if (t0 >= n || c >= p.C) return;
   const int pos0 = p.pos[r0];
   const AT* ring = (const AT*)p.ring + (size_t)p.slot[b] * p.taps * p.C;
@@ -86,8 +85,8 @@ __global__ __launch_bounds__(256) void short_conv_kernel(ConvParams p) {
   }
   // token t0 + i goes to window entry i % K, so nothing is shifted; inputs are requested PF tokens ahead
   constexpr int PF = K < 4 || K > 8 ? 2 : 4;
-  static_assert(kConvTokens % K == 0 && K % PF == 0, "whole turns of the window");
-  const int t1 = min(n, t0 + kConvTokens);
+  static_assert(K % PF == 0, "whole turns of the window");
+  const int t1 = min(n, t0 + p.span);
   float nx[PF][8];
 #pragma unroll
   for (int i = 0; i < PF; ++i) token(min(t0 + i, t1 - 1), nx[i]);
@@ -138,11 +137,12 @@ __global__ __launch_bounds__(256) void conv_ring_kernel(ConvParams p) {
 int short_conv(Proj y, int col0, int C, int taps, const float* w, const float* bias, void* ring, const int* slot,
                const int* pos, const int* cu, int chunks, int max_q, void* out, int act_f32, hipStream_t s) {
   if (chunks <= 0 || max_q <= 0) return 0;
-  if (C < 8 || C % 8 || col0 % 8 || y.ld % 8 || taps < 1 || taps > 16 || y.S < 1 || chunks > 65535 ||
-      (max_q + kConvTokens - 1) / kConvTokens > 65535)
+  if (C < 8 || C % 8 || col0 % 8 || y.ld % 8 || taps < 1 || taps > 16 || y.S < 1 || y.slab % 8 || chunks > 65535 || max_q > (1 << 19))
     return hipErrorInvalidValue;
-  ConvParams p{y, col0, C, taps, w, bias, ring, slot, pos, cu, out};
-  const dim3 grid((C / 8 + 255) / 256, (max_q + kConvTokens - 1) / kConvTokens, chunks);
+  // long walks amortise the taps and the inputs before them; short ones keep a single prompt's latency down
+  const int wide = (C / 8 + 255) / 256, span = (long)wide * ((max_q + 31) / 32) * chunks >= 1024 ? 32 : taps <= 8 ? 8 : 16;
+  ConvParams p{y, col0, C, taps, w, bias, ring, slot, pos, cu, out, span};
+  const dim3 grid(wide, (max_q + span - 1) / span, chunks);
 #define CONV_K(PT, AT)                                                                                        \
   do {                                                                                                        \
     if (taps <= 2) hipLaunchKernelGGL((short_conv_kernel<PT, AT, 2>), grid, dim3(256), 0, s, p);              \

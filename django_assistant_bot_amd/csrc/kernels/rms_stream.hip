@@ -140,40 +140,45 @@ struct RopeParams {
   int bs, T;
 };
 
-// One workgroup per token.  A group of LPH lanes walks heads, a lane owns the pairs 2 (2 (lane + LPH i) + 0 / 1), i < NP:
-// four consecutive elements.  The angle p * f is formed in fp64 and reduced to a half turn before the fp32 sine and
-// cosine, so it is exact to fp32 rounding at any position; one workgroup forms it once for all heads.
+// cosine and sine of a whole number of turns' fraction r in [-1/2, 1/2]: the nearest quarter turn is taken off, then the
+// Taylor series on [-pi/4, pi/4] to fp32 rounding
+__device__ __forceinline__ void sincos_turn(double r, float& sn, float& cs) {
+  const double q = rint(4. * r);
+  const float a = (float)((r - 0.25 * q) * 6.283185307179586476925), z = a * a;
+  float s = fmaf(z, -2.5052108e-8f, 2.7557319e-6f);
+  s = fmaf(z, s, -1.9841270e-4f);
+  s = fmaf(z, s, 8.3333333e-3f);
+  s = fmaf(z, s, -1.6666667e-1f);
+  s = fmaf(a * z, s, a);
+  float c = fmaf(z, 2.0876757e-9f, -2.7557319e-7f);
+  c = fmaf(z, c, 2.4801587e-5f);
+  c = fmaf(z, c, -1.3888889e-3f);
+  c = fmaf(z, c, 4.1666667e-2f);
+  c = fmaf(z, c, -0.5f);
+  c = fmaf(z, c, 1.f);
+  const int k = (int)q & 3;
+  const float s1 = k & 1 ? c : s, c1 = k & 1 ? s : c;
+  sn = k & 2 ? -s1 : s1;
+  cs = (k == 1 || k == 2) ? -c1 : c1;
+}
+
+// One workgroup per token: the angles once (p * f formed in fp64, so they are exact to fp32 rounding at any position), then
+// groups of LPH lanes walk heads, the next head's elements requested under the current one.  A lane owns the elements
+// 4 (lane + LPH i) .. + 3, i < NP.
 template <typename PT, typename AT, int LPH, int NP>
-__global__ __launch_bounds__(512) void qk_rope_kernel(RopeParams p) {
-  const int t = blockIdx.x, grp = threadIdx.x / LPH, lane = threadIdx.x % LPH, ng = blockDim.x / LPH;
-  const int64_t slot = p.slots[t];
-  const double pos = (double)p.positions[t];
-  float cs[NP][2], sn[NP][2];
-#pragma unroll
-  for (int i = 0; i < NP; ++i)
-#pragma unroll
-    for (int e = 0; e < 2; ++e) {
-      const int pr = 2 * (lane + LPH * i) + e;
-      cs[i][e] = 1.f;
-      sn[i][e] = 0.f;
-      if (2 * pr < p.rot) {
-        const double turns = pos * p.freq[pr];
-        sincosf((float)((turns - rint(turns)) * 6.283185307179586476925), &sn[i][e], &cs[i][e]);
-      }
-    }
-  const size_t blk = slot >= 0 ? (size_t)(slot / p.bs) : 0, off = slot >= 0 ? (size_t)(slot % p.bs) : 0;
+__global__ __launch_bounds__(256) void qk_rope_kernel(RopeParams p) {
+  __shared__ __attribute__((aligned(16))) float2 cs[2 * LPH * NP];
+  const int t = blockIdx.x, grp = threadIdx.x / LPH, lane = threadIdx.x % LPH;
+  constexpr int ng = 256 / LPH;
   const int heads = p.H + 2 * p.G;
-  for (int h0 = 0; h0 < heads; h0 += ng) {  // (uniform trip count: the groups of a wave reduce together)
-    const int hd = h0 + grp;
-    const bool on = hd < heads, is_v = hd >= p.H + p.G;
-    float x[NP][4], ss = 0.f;
+  auto load = [&](int hd, float(&x)[NP][4]) {
+    hd = min(hd, heads - 1);
 #pragma unroll
     for (int i = 0; i < NP; ++i) {
-      const int d = 4 * (lane + LPH * i);
+      const int d = min(4 * (lane + LPH * i), p.D - 4);
+      const PT* s = (const PT*)p.y.p + (size_t)t * p.y.ld + p.col0 + (size_t)hd * p.D + d;
 #pragma unroll
       for (int e = 0; e < 4; ++e) x[i][e] = 0.f;
-      if (d >= p.D || !on) continue;
-      const PT* s = (const PT*)p.y.p + (size_t)t * p.y.ld + p.col0 + (size_t)hd * p.D + d;
       ElemIO<PT>::add4(s, x[i]);
       int k = 1;
       s += p.y.slab;
@@ -185,15 +190,42 @@ __global__ __launch_bounds__(512) void qk_rope_kernel(RopeParams p) {
         for (int e = 0; e < 4; ++e) x[i][e] += a[e];
       }
       if (k < p.y.S) ElemIO<PT>::add4(s, x[i]);
+    }
+  };
+  float nx[NP][4];
+  load(grp, nx);
+  const int64_t slot = p.slots[t];
+  const double pos = (double)p.positions[t];
+  for (int pr = threadIdx.x; pr < 2 * LPH * NP; pr += 256) {
+    float c = 1.f, s = 0.f;
+    if (2 * pr < p.rot) {
+      const double turns = pos * p.freq[pr];
+      sincos_turn(turns - rint(turns), s, c);
+    }
+    cs[pr] = make_float2(c, s);
+  }
+  const size_t blk = slot >= 0 ? (size_t)(slot / p.bs) : 0, off = slot >= 0 ? (size_t)(slot % p.bs) : 0;
+  __syncthreads();
+  for (int h0 = 0; h0 < heads; h0 += ng) {  // (uniform trip count: the groups of a wave reduce together)
+    const int hd = h0 + grp;
+    const bool on = hd < heads, is_v = hd >= p.H + p.G;
+    float x[NP][4], ss = 0.f;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) x[i][e] = ElemIO<AT>::round(x[i][e]);
-      if (!is_v) {
+    for (int i = 0; i < NP; ++i)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) x[i][e] = ElemIO<AT>::round(nx[i][e]);
+    if (h0 + ng < heads) load(hd + ng, nx);
+    if (!is_v) {
+#pragma unroll
+      for (int i = 0; i < NP; ++i) {
+        const f32x4 w = *reinterpret_cast<const f32x4*>(&cs[2 * (lane + LPH * i)]);
+        const bool in = 4 * (lane + LPH * i) < p.D;
 #pragma unroll
         for (int e = 0; e < 2; ++e) {
           const float u = x[i][2 * e], v = x[i][2 * e + 1];
-          x[i][2 * e] = u * cs[i][e] - v * sn[i][e];
-          x[i][2 * e + 1] = v * cs[i][e] + u * sn[i][e];
-          ss += x[i][2 * e] * x[i][2 * e] + x[i][2 * e + 1] * x[i][2 * e + 1];
+          x[i][2 * e] = u * w[2 * e] - v * w[2 * e + 1];
+          x[i][2 * e + 1] = v * w[2 * e] + u * w[2 * e + 1];
+          if (in) ss += x[i][2 * e] * x[i][2 * e] + x[i][2 * e + 1] * x[i][2 * e + 1];
         }
       }
     }
@@ -226,9 +258,9 @@ int qk_rope_write(Proj y, int col0, int H, int G, int D, int dim, int rot, const
 #define ROPE_NP(PT, AT)                                                                                      \
   do {                                                                                                       \
     if (D <= 64) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 16, 1>), dim3(T), dim3(256), 0, s, p);           \
-    else if (D <= 128) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 32, 1>), dim3(T), dim3(512), 0, s, p);     \
-    else if (D <= 256) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 64, 1>), dim3(T), dim3(512), 0, s, p);     \
-    else hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 64, 4>), dim3(T), dim3(512), 0, s, p);                   \
+    else if (D <= 128) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 32, 1>), dim3(T), dim3(256), 0, s, p);     \
+    else if (D <= 256) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 64, 1>), dim3(T), dim3(256), 0, s, p);     \
+    else hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 64, 4>), dim3(T), dim3(256), 0, s, p);                   \
   } while (0)
   DAB_PROJ_DISPATCH(y, act_f32, ROPE_NP);
 #undef ROPE_NP

@@ -180,7 +180,7 @@ class VugotarModel(FragmentProjections):
             s = next((s for s in (16, 8, 4, 2) if w.shape[1] % (128 * s) == 0), 1)
             if cfg >= 0 and s > 1:
                 return ops.stream_gemm(h, w, splits=s, cfg=cfg, nt=True)
-        return ops.gemm_bt(h, w, out_f32=True, shuffled=True)
+        return ops.gemm_narrow(h, w)
 
     def _glu(self, h, L: HybridDecoderLayer, dec: bool, out) -> None:
         w, b = L.gate_up_w, L.gate_up_b

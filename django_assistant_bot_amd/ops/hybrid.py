@@ -195,6 +195,27 @@ def chunk_decode(q, kc, vc, bt, ctx, scale: float, chunk: int, sink, out, out_sc
 
 
 # ----------------------------------------------------------------------------------------------
+# narrow fp32 projection
+
+
+def gemm_narrow(x, w):
+    """x [M, K] . w [N, K]^T for a few columns that stay in fp32 (router logits, recurrence gates): fp32 [M, N], or split-K
+    slabs [S, M, N] where the row tiles alone would leave CUs idle.  bf16 on the GPU (``w`` a ``shuffle_weights`` copy)."""
+    if not x.is_cuda:
+        return x.float() @ w.float().t()
+    M, K = x.shape
+    N = w.shape[0]
+    expect(x.dtype == w.dtype == torch.bfloat16 and x.stride(1) == 1 and w.is_contiguous() and w.shape[1] == K, "bf16 operands")
+    expect(K % 64 == 0 and N % 16 == 0 and x.stride(0) % 8 == 0, "gemm_narrow: K % 64, N % 16")
+    tiles, S = -(-M // 32) * -(-N // 128), 1
+    while S < 16 and tiles * S < 1024 and K % (128 * S) == 0 and K // (2 * S) >= 256:
+        S *= 2
+    out = torch.empty((S, M, N) if S > 1 else (M, N), dtype=torch.float32, device=x.device)
+    native().gemm_narrow(ptr(x), x.stride(0), ptr(w), ptr(out), M, N, K, S, stream(x))
+    return out
+
+
+# ----------------------------------------------------------------------------------------------
 # recurrent mixers
 
 

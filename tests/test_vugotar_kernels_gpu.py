@@ -366,3 +366,25 @@ def test_biased_glu_epilogue(M, N, K, epi):
     out = torch.zeros(M, N // 2 + 4, device=DEV)
     ops.glu_f32(ops.gemm_f32(xf.to(DEV), wf.to(DEV)), epi == ops.EPI_GEGLU8, b.to(DEV), out[:, :N // 2])
     close(out[:, :N // 2], ref.gemm_bt(x.float(), w.float(), epilogue=epi, glu_bias=b, out_f32=True), 1e-5)
+
+
+@pytest.mark.parametrize("M,N,K", [(1, 128, 128), (130, 128, 256), (1000, 128, 4096), (33, 144, 192), (3000, 16, 1024), (70, 256, 2048)])
+def test_gemm_narrow(M, N, K):
+    x, w = rnd(M, K), rnd(N, K, seed=2, scale=K ** -0.5)
+    got = ops.gemm_narrow(x.to(DEV), ops.shuffle_weights(w).to(DEV))
+    got = got.sum(0) if got.dim() == 3 else got
+    close(got, x.double() @ w.double().T, 3e-6)
+
+
+def test_rotations_are_exact_to_fp32():
+    """cos and sin of every quadrant, of angles near the axes and of positions past 2^20."""
+    D, T = 128, 600
+    pos = torch.cat([torch.arange(300), torch.randint(1 << 20, 1 << 24, (300,), generator=torch.Generator().manual_seed(1))]).int()
+    y = torch.zeros(T, 3 * D, dtype=F32)
+    y[:, 0:D:2] = 1.0  # unit pairs: the rotated pair is (cos, sin)
+    kc = torch.zeros(1, 1, 16, D, device=DEV)
+    turns = ops.rope_turns(D, 10000.0, DEV)
+    q = ops.qk_rope_write(y.to(DEV), 0, 1, 1, D, D, D, turns, 0.0, False, pos.to(DEV), torch.full((T,), -1).to(DEV), kc, kc.clone())
+    a = pos.double()[:, None] * turns.cpu() * 2 * torch.pi
+    got = q[:, 0].double().cpu()
+    assert float((got[:, 0::2] - a.cos()).abs().max()) < 2e-7 and float((got[:, 1::2] - a.sin()).abs().max()) < 2e-7
