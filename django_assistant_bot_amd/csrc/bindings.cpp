@@ -216,12 +216,13 @@ PYBIND11_MODULE(_native, m) {
           "state_scan");
   });
   m.def("state_chunks_ok", [shape](const R& d) { return dab::state_chunks_ok(shape(d)) != 0; });
-  m.def("state_chunks_bytes", &dab::state_chunks_bytes);
+  m.def("state_chunks_segments", [shape](const R& d, int chunks, int max_q) { return dab::state_chunks_segments(shape(d), chunks, max_q); });
+  m.def("state_chunks_bytes", [shape](const R& d, int T, int chunks, int segs) { return dab::state_chunks_bytes(shape(d), T, chunks, segs); });
   m.def("state_chunks", [proj, shape](u conv, const R& d, const P& gates, u A, u dt_bias, u skip, u state, u slot, u pos,
-                                      u cu, int chunks, int max_q, u out, u ws, u s) {
+                                      u cu, int chunks, int max_q, int T, int segs, u out, u ws, u s) {
     check(dab::state_chunks(CVP(conv), shape(d), proj(gates), (const float*)A, (const float*)dt_bias, (const float*)skip,
-                            (float*)state, (const int*)slot, (const int*)pos, (const int*)cu, chunks, max_q, VP(out),
-                            VP(ws), ST(s)),
+                            (float*)state, (const int*)slot, (const int*)pos, (const int*)cu, chunks, max_q, T, segs,
+                            VP(out), VP(ws), ST(s)),
           "state_chunks");
   });
   m.def("state_decode", [proj, shape](const P& y, int col0, int taps, u w, u bias, u ring, int act_f32, const R& d,

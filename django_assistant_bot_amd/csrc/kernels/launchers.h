@@ -93,10 +93,11 @@ int state_scan(const void* conv, int act_f32, RecurrentShape d, Proj gates, cons
                hipStream_t s);
 // recurrent_chunk.hip: the scan of bf16 portions 64 tokens at a time (prepare + scan); ws: state_chunks_bytes
 int state_chunks_ok(RecurrentShape d);
-long state_chunks_bytes(int T, int chunks, int H);
+int state_chunks_segments(RecurrentShape d, int chunks, int max_q);
+long state_chunks_bytes(RecurrentShape d, int T, int chunks, int segs);
 int state_chunks(const void* conv, RecurrentShape d, Proj gates, const float* A, const float* dt_bias, const float* skip,
-                 float* state, const int* slot, const int* pos, const int* cu, int chunks, int max_q, void* out, void* ws,
-                 hipStream_t s);
+                 float* state, const int* slot, const int* pos, const int* cu, int chunks, int max_q, int T, int segs, void* out,
+                 void* ws, hipStream_t s);
 int state_decode(Proj y, int col0, int taps, const float* w, const float* bias, void* ring, int act_f32, RecurrentShape d,
                  Proj gates, const float* A, const float* dt_bias, const float* skip, float* state, const int* slot,
                  const int* pos, int row0, int B, int g_col, const float* norm, float eps, float out_scale, void* out,

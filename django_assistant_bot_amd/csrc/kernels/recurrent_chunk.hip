@@ -11,6 +11,12 @@
 //   chunk_scan      the chunks of a sequence in turn; a wave owns 16 value columns of one head and keeps their state
 //                   in accumulator registers
 //
+// Few sequences leave the chip idle while their chunks wait for each other, so long portions are cut into segments of
+// kSeg chunks that run side by side: chunk_scan in its SUMMARY form first computes what a segment does to any state,
+// S_end = P S_start + S_loc (delta: P by scanning the columns of the identity without values; ssd: P is the scalar
+// e^(G of the segment)), chunk_combine walks the segments with it, and the segments are then scanned from their own
+// start states.
+//
 // Precision: everything is an fp32 computation.  The convolved q, k are exact bf16 numbers, so their products on the
 // bf16 MFMA are exact fp32 products; unit-norm factors, decays and betas are fp32 row scales applied outside.  An fp32
 // operand X (S, R, U, T) enters as X = hi + mid + lo, three bf16 terms (24 bits): products with a bf16 operand take 3
@@ -50,7 +56,12 @@ struct ChunkP {
   bf16* out;
   char* ws;
   float qscale;
+  int segs;          // segments per sequence (1: whole sequences)
+  float* seg_start;  // [chunks, segs, H, V, Dp] state before each segment but a sequence's first
+  float* seg_loc;    // [chunks, segs, H, V (+ Dp), Dp] summaries
 };
+
+constexpr int kSeg = 16;  // chunks of a segment
 
 // x = hi + mid (+ lo), bf16 each
 template <int N>
@@ -256,7 +267,7 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkP p) {
 
 // LDS: the chunk's K | Q tile (rows prefetched into registers a chunk ahead) and its workspace block (T and A fragments,
 // row scales), copied by LDS-DMA as soon as every wave is done with the previous one.
-template <int D32, bool DELTA>
+template <int D32, bool DELTA, bool SUMMARY>
 __global__ __launch_bounds__(256, 2) void chunk_scan_kernel(ChunkP p) {
   constexpr int Dp = 32 * D32, STR = Dp * 2 + 16, MT = 2 * D32;
   constexpr int P0 = DELTA ? 0 : kT / 1024, P1 = kWs / 1024;  // 1-KB pieces of the workspace block that are needed
@@ -265,22 +276,33 @@ __global__ __launch_bounds__(256, 2) void chunk_scan_kernel(ChunkP p) {
   char* const qs = smem + kC * STR;
   char* const wl = smem + 2 * kC * STR;
   const float* const sc = reinterpret_cast<const float*>(wl + kT + kA);  // beta, e^G k-norm, e^G q-norm, e^(G_C - G) k-norm, e^G
-  const int h = blockIdx.y, b = blockIdx.z, hk = h / (p.H / p.G);
+  const int h = blockIdx.y, b = blockIdx.z / p.segs, seg = blockIdx.z % p.segs, hk = h / (p.H / p.G);
   const int q0 = p.cu[b], len = p.cu[b + 1] - q0;
-  if (len <= 0) return;
+  const int nca = (len + kC - 1) / kC;  // chunks of the portion; this workgroup's are c0 .. nc - 1
+  const int c0 = p.segs > 1 ? seg * kSeg : 0, nc = p.segs > 1 ? min(nca, c0 + kSeg) : nca;
+  if (c0 >= nca || (SUMMARY && nc == nca)) return;  // (nothing needs the last segment's summary)
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, li = lane & 15;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int col = blockIdx.x * 64 + 16 * w + li;
-  const bool live = blockIdx.x * 64 + 16 * w < p.V, mine = col < p.V;
-  float* sp = p.state + (((size_t)p.slot[b] * p.H + h) * p.V + (mine ? col : 0)) * Dp + 4 * g;
+  const int vb = (p.V + 63) / 64;
+  const bool ident = SUMMARY && (int)blockIdx.x >= vb;  // columns of the identity
+  const int ncol = ident ? Dp : p.V, bx = ident ? blockIdx.x - vb : blockIdx.x;
+  const int col = bx * 64 + 16 * w + li;
+  const bool live = bx * 64 + 16 * w < ncol, mine = col < ncol;
+  const size_t bs = (size_t)(b * p.segs + seg) * p.H + h;
+  float* const slot_state = p.state + (((size_t)p.slot[b] * p.H + h) * p.V + (mine ? col : 0)) * Dp + 4 * g;
+  const float* sp = seg > 0 ? p.seg_start + (bs * p.V + (mine ? col : 0)) * Dp + 4 * g : slot_state;
   const char* ws0 = p.ws + ((size_t)(q0 / kC + b) * p.H + h) * kWs;
   f32x4 S[MT];
-  const bool fresh = p.pos[q0] == 0;
+  const bool fresh = SUMMARY || !mine || (seg == 0 && p.pos[q0] == 0);
 #pragma unroll
-  for (int m = 0; m < MT; ++m)
-    S[m] = fresh || !mine ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
+  for (int m = 0; m < MT; ++m) {
+    S[m] = fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
+    if (SUMMARY && ident) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[m][r] = 16 * m + 4 * g + r == col ? 1.f : 0.f;
+    }
+  }
   const float skip = !DELTA && p.skip ? p.skip[h] : 0.f;
-  const int nc = (len + kC - 1) / kC;
   u32x4 pre[kPieces<D32>];
   auto fetch = [&](int c) { fetch_kq<D32>(p, q0 + kC * c, min(kC, len - kC * c), hk, tid, pre); };
   auto copy_ws = [&](int c) {
@@ -297,20 +319,21 @@ __global__ __launch_bounds__(256, 2) void chunk_scan_kernel(ChunkP p) {
     }
   };
   auto scale4 = [&](int row, int m) { return *reinterpret_cast<const f32x4*>(sc + row * kC + 16 * m + 4 * g); };
-  fetch(0);
-  copy_ws(0);
-  for (int c = 0; c < nc; ++c) {
+  fetch(c0);
+  copy_ws(c0);
+  for (int c = c0; c < nc; ++c) {
     const int n = min(kC, len - kC * c);
     __syncthreads();  // the previous chunk's tile is done with
     store_kq<D32>(smem, tid, pre);
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's workspace pieces landed
     __syncthreads();
     f32x4 R[4];  // values of this wave's columns in the accumulator layout
-    const bf16* vp = p.conv + (size_t)(q0 + kC * c) * p.C + p.v_col + h * p.V + (mine ? col : 0);
+    const bf16* vp = p.conv + (size_t)(q0 + kC * c) * p.C + p.v_col + h * p.V + (mine && !ident ? col : 0);
+    const float von = ident ? 0.f : 1.f;
 #pragma unroll
     for (int m = 0; m < 4; ++m)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) R[m][r] = bf2f(vp[(size_t)min(16 * m + 4 * g + r, n - 1) * p.C]);
+      for (int r = 0; r < 4; ++r) R[m][r] = von * bf2f(vp[(size_t)min(16 * m + 4 * g + r, n - 1) * p.C]);
     if (c + 1 < nc) fetch(c + 1);
     bf16x8 wu[2][3];
     float ec = 0.f;
@@ -339,8 +362,10 @@ __global__ __launch_bounds__(256, 2) void chunk_scan_kernel(ChunkP p) {
         f32x4 P[4];
 #pragma unroll
         for (int m = 0; m < 4; ++m) P[m] = times_s(ks, m);
+        if (!SUMMARY) {
 #pragma unroll
-        for (int m = 0; m < 4; ++m) O[m] = times_s(qs, m) * scale4(2, m);
+          for (int m = 0; m < 4; ++m) O[m] = times_s(qs, m) * scale4(2, m);
+        }
 #pragma unroll
         for (int m = 0; m < 4; ++m) R[m] = scale4(0, m) * (R[m] - scale4(1, m) * P[m]);
         bf16x8 rs[2][3];
@@ -370,11 +395,11 @@ __global__ __launch_bounds__(256, 2) void chunk_scan_kernel(ChunkP p) {
       } else {
 #pragma unroll
         for (int m = 0; m < 4; ++m) {
-          O[m] = times_s(qs, m) * scale4(2, m) + skip * R[m];
+          if (!SUMMARY) O[m] = times_s(qs, m) * scale4(2, m) + skip * R[m];
           U[m] = scale4(0, m) * R[m];
         }
       }
-      // read-out
+      if constexpr (!SUMMARY) {  // read-out
       bf16x8 us[2][2];
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb) {
@@ -409,6 +434,7 @@ __global__ __launch_bounds__(256, 2) void chunk_scan_kernel(ChunkP p) {
               if (16 * m + 4 * g + r < n) op[(16 * m + 4 * g + r) * ld] = f2bf(O[m][r]);
         }
       }
+      }
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb) {
         float x[8];
@@ -438,15 +464,88 @@ __global__ __launch_bounds__(256, 2) void chunk_scan_kernel(ChunkP p) {
       }
     }
   }
-  if (mine) {
+  if (mine && (SUMMARY || nc == nca)) {
+    float* dst = SUMMARY ? p.seg_loc + (bs * (DELTA ? p.V + Dp : p.V) + (ident ? p.V : 0) + col) * Dp + 4 * g : slot_state;
 #pragma unroll
-    for (int m = 0; m < MT; ++m) *reinterpret_cast<f32x4*>(sp + 16 * m) = S[m];
+    for (int m = 0; m < MT; ++m) *reinterpret_cast<f32x4*>(dst + 16 * m) = S[m];
+  }
+}
+
+// Start states of a sequence's segments, one after the other; a workgroup owns 16 value columns of one head.
+template <int D32, bool DELTA>
+__global__ __launch_bounds__(256) void chunk_combine_kernel(ChunkP p) {
+  constexpr int Dp = 32 * D32;
+  __shared__ __attribute__((aligned(16))) float st[16][Dp];
+  const int h = blockIdx.y, b = blockIdx.z, col0 = blockIdx.x * 16;
+  const int q0 = p.cu[b], len = p.cu[b + 1] - q0, nca = (len + kC - 1) / kC, ns = (nca + kSeg - 1) / kSeg;
+  if (ns < 2) return;
+  const int d = threadIdx.x % 128, half = threadIdx.x / 128;  // this thread's state row, and columns 8 half .. + 7
+  const bool fresh = p.pos[q0] == 0, on = d < Dp;
+  const float* s0 = p.state + ((size_t)p.slot[b] * p.H + h) * p.V * Dp;
+  float x[8];
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int c = min(col0 + 8 * half + i, p.V - 1);
+    x[i] = fresh || !on ? 0.f : s0[(size_t)c * Dp + d];
+  }
+  for (int s = 0; s + 1 < ns; ++s) {
+    const size_t bs = (size_t)(b * p.segs + s) * p.H + h;
+    const float* loc = p.seg_loc + bs * (DELTA ? p.V + Dp : p.V) * Dp;
+    float y[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) y[i] = on ? loc[(size_t)min(col0 + 8 * half + i, p.V - 1) * Dp + d] : 0.f;
+    if (DELTA) {
+      __syncthreads();
+      if (on)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) st[8 * half + i][d] = x[i];
+      __syncthreads();
+      const float* P = loc + (size_t)p.V * Dp + (on ? d : 0);
+#pragma unroll 2
+      for (int j = 0; j < Dp; j += 4) {
+        float pc[4];
+#pragma unroll
+        for (int q = 0; q < 4; ++q) pc[q] = P[(size_t)(j + q) * Dp];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          const f32x4 v = *reinterpret_cast<const f32x4*>(&st[8 * half + i][j]);
+#pragma unroll
+          for (int q = 0; q < 4; ++q) y[i] = fmaf(pc[q], v[q], y[i]);
+        }
+      }
+    } else {
+      float gseg = 1.f;
+      const char* ws = p.ws + ((size_t)(q0 / kC + b + s * kSeg) * p.H + h) * kWs + kT + kA;
+#pragma unroll
+      for (int c = 0; c < kSeg; ++c) gseg *= reinterpret_cast<const float*>(ws + (size_t)c * p.H * kWs)[4 * kC + kC - 1];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) y[i] = fmaf(gseg, x[i], y[i]);
+    }
+    float* nx = p.seg_start + (bs + p.H) * p.V * Dp;  // (segment s + 1)
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      x[i] = y[i];
+      if (on && col0 + 8 * half + i < p.V) nx[(size_t)(col0 + 8 * half + i) * Dp + d] = y[i];
+    }
   }
 }
 
 }  // namespace
 
-long state_chunks_bytes(int T, int chunks, int H) { return (long)(T / kC + chunks) * H * kWs; }
+// Segments per sequence of a launch: 1, unless whole sequences would leave most CUs idle
+int state_chunks_segments(RecurrentShape d, int chunks, int max_q) {
+  const int nca = (max_q + kC - 1) / kC;
+  const long wgs = (long)((d.V + 63) / 64) * d.H * chunks;
+  return wgs <= 128 && nca >= 2 * kSeg ? (nca + kSeg - 1) / kSeg : 1;
+}
+
+static long seg_floats(RecurrentShape d, int chunks, int segs, bool loc) {
+  return segs < 2 ? 0 : (long)chunks * segs * d.H * (d.V + (loc && d.delta ? d.Dp : 0)) * d.Dp;
+}
+
+long state_chunks_bytes(RecurrentShape d, int T, int chunks, int segs) {
+  return (long)(T / kC + chunks) * d.H * kWs + 4 * (seg_floats(d, chunks, segs, false) + seg_floats(d, chunks, segs, true));
+}
 
 int state_chunks_ok(RecurrentShape d) {
   return d.D % 8 == 0 && d.Dp <= 128 && d.C % 8 == 0 && d.q_col % 8 == 0 && d.k_col % 8 == 0 && d.H >= 1 && d.G >= 1 &&
@@ -454,10 +553,12 @@ int state_chunks_ok(RecurrentShape d) {
 }
 
 int state_chunks(const void* conv, RecurrentShape d, Proj gates, const float* A, const float* dt_bias, const float* skip,
-                 float* state, const int* slot, const int* pos, const int* cu, int chunks, int max_q, void* out, void* ws,
-                 hipStream_t s) {
+                 float* state, const int* slot, const int* pos, const int* cu, int chunks, int max_q, int T, int segs, void* out,
+                 void* ws, hipStream_t s) {
   if (chunks <= 0 || max_q <= 0) return 0;
-  if (!state_chunks_ok(d) || !gates.f32 || gates.S < 1 || chunks > 65535 || !ws) return hipErrorInvalidValue;
+  if (!state_chunks_ok(d) || !gates.f32 || gates.S < 1 || segs < 1 || (long)chunks * segs > 65535 || !ws ||
+      (segs > 1 && segs < (max_q + kC * kSeg - 1) / (kC * kSeg)))
+    return hipErrorInvalidValue;
   ChunkP p{};
   p.conv = (const bf16*)conv;
   p.C = d.C;
@@ -480,17 +581,26 @@ int state_chunks(const void* conv, RecurrentShape d, Proj gates, const float* A,
   p.cu = cu;
   p.out = (bf16*)out;
   p.ws = (char*)ws;
+  p.segs = segs;
+  p.seg_start = (float*)((char*)ws + (long)(T / kC + chunks) * d.H * kWs);
+  p.seg_loc = p.seg_start + seg_floats(d, chunks, segs, false);
   p.qscale = 1.f / sqrtf((float)d.D);
-  const dim3 gp((max_q + kC - 1) / kC, d.delta ? d.H : d.G, chunks), gs((d.V + 63) / 64, d.H, chunks);
-#define CHUNK_L(D32)                                                                               \
+  const int vb = (d.V + 63) / 64;
+  const dim3 gp((max_q + kC - 1) / kC, d.delta ? d.H : d.G, chunks), gs(vb, d.H, chunks * segs);
+  const dim3 gm(vb + (d.delta ? (d.Dp + 63) / 64 : 0), d.H, chunks * segs), gc((d.V + 15) / 16, d.H, chunks);
+#define CHUNK_D(D32, DELTA)                                                                        \
   do {                                                                                             \
-    if (d.delta) {                                                                                 \
-      hipLaunchKernelGGL((chunk_prepare_kernel<D32, true>), gp, dim3(256), 0, s, p);               \
-      hipLaunchKernelGGL((chunk_scan_kernel<D32, true>), gs, dim3(256), 0, s, p);                  \
-    } else {                                                                                       \
-      hipLaunchKernelGGL((chunk_prepare_kernel<D32, false>), gp, dim3(256), 0, s, p);              \
-      hipLaunchKernelGGL((chunk_scan_kernel<D32, false>), gs, dim3(256), 0, s, p);                 \
+    hipLaunchKernelGGL((chunk_prepare_kernel<D32, DELTA>), gp, dim3(256), 0, s, p);                \
+    if (segs > 1) {                                                                                \
+      hipLaunchKernelGGL((chunk_scan_kernel<D32, DELTA, true>), gm, dim3(256), 0, s, p);           \
+      hipLaunchKernelGGL((chunk_combine_kernel<D32, DELTA>), gc, dim3(256), 0, s, p);              \
     }                                                                                              \
+    hipLaunchKernelGGL((chunk_scan_kernel<D32, DELTA, false>), gs, dim3(256), 0, s, p);            \
+  } while (0)
+#define CHUNK_L(D32)                 \
+  do {                               \
+    if (d.delta) CHUNK_D(D32, true); \
+    else CHUNK_D(D32, false);        \
   } while (0)
   switch (d.Dp / 32) {
     case 1: CHUNK_L(1); break;
@@ -500,6 +610,7 @@ int state_chunks(const void* conv, RecurrentShape d, Proj gates, const float* A,
     default: return hipErrorInvalidValue;
   }
 #undef CHUNK_L
+#undef CHUNK_D
   return hipGetLastError();
 }
 

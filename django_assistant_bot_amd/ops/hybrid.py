@@ -288,10 +288,12 @@ def short_conv(y, col0: int, w, bias, ring, slot, pos, cu, max_q: int):
 CHUNK_MIN_TOKENS = 24  # portions shorter than this are scanned token by token
 
 
-def state_scan(conv, d: RecurrentShape, z, A, dt_bias, skip, state, slot, pos, cu, max_q: int, chunked: bool | None = None):
+def state_scan(conv, d: RecurrentShape, z, A, dt_bias, skip, state, slot, pos, cu, max_q: int, chunked: bool | None = None,
+               segments: int | None = None):
     """The recurrence over the portions ``cu`` (the longest of ``max_q`` tokens) of convolved channels; ``state`` [slots, H,
     V, Dp] goes on from where the sequence left it (zero at position 0).  -> read-outs [T, H V].  ``chunked``: 64 tokens at a
-    time on MFMA (bf16; default: where the sizes allow and the portions are long enough) or token by token."""
+    time on MFMA (bf16; default: where the sizes allow and the portions are long enough) or token by token.  ``segments``: of
+    1024 tokens that a long portion is cut into so that they run side by side (default: when the launch would be small)."""
     T = conv.shape[0]
     if not conv.is_cuda:
         return ref.state_scan(conv, d, z, A, dt_bias, skip, state, slot, pos, ref._spans(cu, 0, 0)).to(conv.dtype)
@@ -307,9 +309,10 @@ def state_scan(conv, d: RecurrentShape, z, A, dt_bias, skip, state, slot, pos, c
         chunked = fits and max_q >= CHUNK_MIN_TOKENS
     if chunked:
         expect(fits, "chunked scan: bf16, state rows % 8, at most 128")
-        ws = torch.empty((nat.state_chunks_bytes(T, n, d.H),), dtype=torch.uint8, device=conv.device)
+        segs = nat.state_chunks_segments(d.native(), n, int(max_q)) if segments is None else segments
+        ws = torch.empty((nat.state_chunks_bytes(d.native(), T, n, segs),), dtype=torch.uint8, device=conv.device)
         nat.state_chunks(ptr(conv), d.native(), pz, ptr(A), ptr(dt_bias), ptr(skip), ptr(state), ptr(slot), ptr(pos), ptr(cu),
-                         n, int(max_q), ptr(out), ptr(ws), stream(conv))
+                         n, int(max_q), T, segs, ptr(out), ptr(ws), stream(conv))
         return out
     nat.state_scan(ptr(conv), int(conv.dtype == torch.float32), d.native(), pz, ptr(A), ptr(dt_bias), ptr(skip),
                         ptr(state), ptr(slot), ptr(pos), ptr(cu), cu.numel() - 1, ptr(out), stream(conv))

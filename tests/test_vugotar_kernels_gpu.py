@@ -126,7 +126,7 @@ def test_chunk_attention(H, G, D, chunk, dtype):
 SHAPES = {  # delta, H, G, D, V, taps
     "delta": (True, 4, 2, 128, 128, 4), "delta_odd": (True, 3, 1, 40, 23, 3), "delta_small": (True, 2, 2, 8, 16, 1),
     "delta_96": (True, 2, 1, 96, 80, 2), "delta_wide": (True, 2, 2, 200, 72, 4), "delta_tiny": (True, 3, 3, 3, 5, 6),
-    "ssd": (False, 8, 2, 128, 64, 4), "ssd_odd": (False, 6, 3, 24, 40, 5), "ssd_64": (False, 2, 1, 64, 130, 4),
+    "ssd": (False, 8, 2, 128, 64, 4), "ssd_odd": (False, 6, 3, 24, 40, 5), "ssd_64": (False, 2, 1, 64, 132, 4),
     "ssd_wide": (False, 2, 1, 256, 33, 9)}
 
 
@@ -225,6 +225,36 @@ def test_chunked_scan_with_long_and_short_memory(name, decay):
     out = ops.state_scan(conv.to(DEV), d, z.to(DEV), c(A), c(dtb), c(skip), state, i32(0).to(DEV), torch.arange(T).int().to(DEV),
                          i32(0, T).to(DEV), T, chunked=True)
     o, S = oracle_scan(d, conv, z, A, dtb, skip)
+    close(out.view(T, d.H, d.V), o, 5e-3)
+    close(state[0, :, :, :d.D].transpose(1, 2), S, 1e-5)
+
+
+@pytest.mark.parametrize("name", ["delta", "delta_odd", "delta_96", "ssd", "ssd_odd", "ssd_64"])
+def test_state_scan_in_segments(name):
+    """A long portion cut into segments that run side by side, beside a short one, both going on from a state: the whole
+    scan's results, and those of one pass over the sequence."""
+    d, _, _, _, _, _, A, dtb, skip = recurrence(name, 4, decay=-5.0)
+    n = [2500, 700]
+    c = lambda t: None if t is None else t.to(DEV)  # noqa: E731
+    conv = rnd(sum(n), d.C, seed=1)
+    z = rnd(sum(n), 2 * d.H + 5, seed=2, dtype=F32)
+    pos = torch.cat([torch.arange(3, 3 + m) for m in n]).int().to(DEV)
+    got = []
+    for segs in (1, 3):
+        state = rnd(2, d.H, d.V, d.Dp, seed=3, dtype=F32)
+        state[..., d.D:] = 0
+        state = state.to(DEV)
+        out = ops.state_scan(conv.to(DEV), d, z.to(DEV), c(A), c(dtb), c(skip), state, i32(1, 0).to(DEV), pos,
+                             i32(0, n[0], sum(n)).to(DEV), max(n), chunked=True, segments=segs)
+        got.append((out, state))
+    close(got[1][0], got[0][0].cpu(), 5e-3)
+    close(got[1][1], got[0][1].cpu(), 1e-5)
+    # from position 0, against the oracle
+    T = 2100
+    state = torch.full((1, d.H, d.V, d.Dp), 9.0, device=DEV)
+    out = ops.state_scan(conv[:T].to(DEV), d, z[:T].to(DEV), c(A), c(dtb), c(skip), state, i32(0).to(DEV), torch.arange(T).int().to(DEV),
+                         i32(0, T).to(DEV), T, chunked=True, segments=3)
+    o, S = oracle_scan(d, conv[:T], z[:T], A, dtb, skip)
     close(out.view(T, d.H, d.V), o, 5e-3)
     close(state[0, :, :, :d.D].transpose(1, 2), S, 1e-5)
 
