@@ -409,10 +409,8 @@ __global__ __launch_bounds__(256) void state_decode_kernel(DecodeStep a) {
   const int h = blockIdx.x, b = blockIdx.y, hk = h / (p.H / p.G), row = a.row0 + b;
   const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, part = lane & 7;
   const int slot = p.slot[b], pos = p.pos[row];
-  float dl, beta;
-  step_gates<float, DELTA>(p, row, h, dl, beta);
-  const float g = __expf(dl);
   AT* ring = (AT*)a.ring + (size_t)slot * a.taps * p.C;
+  const int now = pos % a.taps;  // ring entry of this token
   for (int i = tid; i < 2 * Dp + p.V; i += 256) {
     int ch = -1;
     if (i < Dp) ch = i < p.D ? p.k_col + hk * p.D + i : -1;
@@ -423,13 +421,28 @@ __global__ __launch_bounds__(256) void state_decode_kernel(DecodeStep a) {
       const float cur = proj_at<PT, AT>(a.y, row, a.col0 + ch);
       const float* cw = a.w + ch;
       float acc = fmaf(cw[(size_t)(a.taps - 1) * p.C], cur, a.bias ? a.bias[ch] : 0.f);
-      for (int j = 1; j < a.taps && j <= pos; ++j)
-        acc = fmaf(cw[(size_t)(a.taps - 1 - j) * p.C], ElemIO<AT>::load(ring + (size_t)((pos - j) % a.taps) * p.C + ch), acc);
-      ElemIO<AT>::store(ring + (size_t)(pos % a.taps) * p.C + ch, cur);
+      for (int j0 = 1; j0 < a.taps; j0 += 4) {  // four past inputs requested at a time
+        float past[4], tap[4];
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          const int j = j0 + q;
+          const bool ok = j < a.taps && j <= pos;
+          const int e = ok ? (now >= j ? now - j : now - j + a.taps) : now;
+          past[q] = ElemIO<AT>::load(ring + (size_t)e * p.C + ch);
+          tap[q] = cw[(size_t)(ok ? a.taps - 1 - j : 0) * p.C];
+          if (!ok) past[q] = tap[q] = 0.f;
+        }
+#pragma unroll
+        for (int q = 0; q < 4; ++q) acc = fmaf(tap[q], past[q], acc);
+      }
+      ElemIO<AT>::store(ring + (size_t)now * p.C + ch, cur);
       v = ElemIO<AT>::round(silu_f(acc));
     }
     sm[i] = v;
   }
+  float dl, beta;
+  step_gates<float, DELTA>(p, row, h, dl, beta);
+  const float g = __expf(dl);
   __syncthreads();
   float nk = 1.f, nq = 1.f;
   if (DELTA) {

@@ -166,10 +166,10 @@ __device__ __forceinline__ void sincos_turn(double r, float& sn, float& cs) {
 // groups of LPH lanes walk heads, the next head's elements requested under the current one.  A lane owns the elements
 // 4 (lane + LPH i) .. + 3, i < NP.
 template <typename PT, typename AT, int LPH, int NP>
-__global__ __launch_bounds__(256) void qk_rope_kernel(RopeParams p) {
+__global__ __launch_bounds__(512) void qk_rope_kernel(RopeParams p) {
   __shared__ __attribute__((aligned(16))) float2 cs[2 * LPH * NP];
   const int t = blockIdx.x, grp = threadIdx.x / LPH, lane = threadIdx.x % LPH;
-  constexpr int ng = 256 / LPH;
+  const int ng = blockDim.x / LPH;
   const int heads = p.H + 2 * p.G;
   auto load = [&](int hd, float(&x)[NP][4]) {
     hd = min(hd, heads - 1);
@@ -196,7 +196,7 @@ __global__ __launch_bounds__(256) void qk_rope_kernel(RopeParams p) {
   load(grp, nx);
   const int64_t slot = p.slots[t];
   const double pos = (double)p.positions[t];
-  for (int pr = threadIdx.x; pr < 2 * LPH * NP; pr += 256) {
+  for (int pr = threadIdx.x; pr < 2 * LPH * NP; pr += blockDim.x) {
     float c = 1.f, s = 0.f;
     if (2 * pr < p.rot) {
       const double turns = pos * p.freq[pr];
@@ -255,12 +255,13 @@ int qk_rope_write(Proj y, int col0, int H, int G, int D, int dim, int rot, const
       (rot && !freq) || y.S < 1)
     return hipErrorInvalidValue;
   RopeParams p{y, col0, H, G, D, dim, rot, freq, 1.f / dim, eps, norm, positions, slots, q, kc, vc, bs, T};
+  const int bt = T <= 2048 ? 512 : 256;  // decoded tokens: fewer turns of the head loop; prompts: more workgroups a CU
 #define ROPE_NP(PT, AT)                                                                                      \
   do {                                                                                                       \
-    if (D <= 64) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 16, 1>), dim3(T), dim3(256), 0, s, p);           \
-    else if (D <= 128) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 32, 1>), dim3(T), dim3(256), 0, s, p);     \
-    else if (D <= 256) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 64, 1>), dim3(T), dim3(256), 0, s, p);     \
-    else hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 64, 4>), dim3(T), dim3(256), 0, s, p);                   \
+    if (D <= 64) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 16, 1>), dim3(T), dim3(bt), 0, s, p);            \
+    else if (D <= 128) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 32, 1>), dim3(T), dim3(bt), 0, s, p);      \
+    else if (D <= 256) hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 64, 1>), dim3(T), dim3(bt), 0, s, p);      \
+    else hipLaunchKernelGGL((qk_rope_kernel<PT, AT, 64, 4>), dim3(T), dim3(bt), 0, s, p);                    \
   } while (0)
   DAB_PROJ_DISPATCH(y, act_f32, ROPE_NP);
 #undef ROPE_NP
