@@ -209,6 +209,29 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
     }
     return;
   }
+  if constexpr (GROUP) {
+    // v_permlane16_swap of blocks (2 pi, 2 pi + 1): a lane then holds 8 consecutive columns, one 16-B store
+    const int cq = 16 * (g & 1) + 8 * (g >> 1);
+#pragma unroll
+    for (int mi = 0; mi < MI; ++mi) {
+      const int m = m0 + wm * TM + 16 * mi + li;
+      bf16* row = (bf16*)p.C + (size_t)c_row(min(m, p.M - 1)) * p.ldc;
+#pragma unroll
+      for (int pi = 0; pi < NI / 2; ++pi) {
+        float o[8];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const auto sw = __builtin_amdgcn_permlane16_swap(__float_as_uint(acc[2 * pi][mi][r]),
+                                                           __float_as_uint(acc[2 * pi + 1][mi][r]), false, false);
+          o[r] = __uint_as_float(sw[0]);
+          o[4 + r] = __uint_as_float(sw[1]);
+        }
+        const int n = n0 + wn * TN + 32 * pi + cq;
+        if (m < p.M && n < p.N) *reinterpret_cast<u32x4*>(row + n) = pack8(o);
+      }
+    }
+    return;
+  }
 #pragma unroll
   for (int mi = 0; mi < MI; ++mi) {
     const int m = m0 + wm * TM + 16 * mi + li;
@@ -384,7 +407,7 @@ int gemm_narrow(const void* A, long lda, const void* B, float* C, int M, int N, 
 int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int N, int K, const int* perm, int a_div,
                  int scatter, const void* tiles, int n_tiles, int bm, int glu, const float* row_scale, hipStream_t s) {
   if (n_tiles <= 0 || N <= 0) return 0;
-  if (K % 64 || N % 32 || lda % 8 || ldc % 4 || !tiles || !perm || (bm != 32 && bm != 128 && bm != 256) || (row_scale && !glu))
+  if (K % 64 || N % 32 || lda % 8 || ldc % 8 || !tiles || !perm || (bm != 32 && bm != 128 && bm != 256) || (row_scale && !glu))
     return hipErrorInvalidValue;
   GemmParams p{};
   p.A = (const bf16*)A;
