@@ -1,6 +1,6 @@
 """Prefill and decode throughput of decoder presets at the engine's own step functions (random weights).
 
-    python bench.py --decoder-bench vumuvik-8b,llama-3-8b [--decoder-shapes ...]
+    python bench.py --decoder-bench vugotar-8b,llama-3-8b [--decoder-shapes ...]
 
 Per model: prefill steps of packed prompts (model forward + last-token logits, as ``LLMEngine._run_prefill``
 enqueues them) and decode steps replayed from the engine's HIP graphs (forward + LM head + sampling) at a

@@ -83,7 +83,7 @@ CONFIGS = {
     # projection sizes that take the streaming decode GEMM (K % 128) and a split-K of several slabs
     "stream": config(512, [
         mamba(8, 64, 128, 2, 4, 1, dense(1024)),
-        parallel((8, 2, 64, 64, 0.3, 96, 64), (4, 2, 128, 128, 4), moe(16, 4, 1.5, 256, 512)),
+        parallel((8, 2, 64, 64, 0.3, 96, 64), (4, 2, 128, 128, 4), moe(14, 5, 1.3, 256, 512)),
         parallel((8, 8, 64, 64, 0.3, 200, 32), (8, 4, 64, 64, 4), dense(1024))], loop=(1, 2, 2)),
 }
 
