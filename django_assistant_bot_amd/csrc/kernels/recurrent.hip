@@ -174,7 +174,6 @@ struct ScanParams {
   const int* cu;
   void* out;          // [T, H * V]
   float qscale;
-  int nc;             // column groups per wave step (decode)
 };
 
 template <typename GT, bool DELTA>

@@ -65,6 +65,25 @@ def test_kv_manager_alloc_extend_free(n):
     assert m.num_free_blocks() == 8
 
 
+def test_kv_manager_state_slots(n):
+    m = n.KVBlockManager(16, 4, False, 2)
+    out = np.zeros(2, dtype=np.int32)
+    assert m.add_sequence(7, [1, 2], 0) == 0 and m.add_sequence(8, [3], 0) == 0
+    m.state_slots_into([8, 7], out.ctypes.data)
+    assert list(out) == [1, 0] and m.num_free_state_slots() == 0
+    assert m.add_sequence(9, [4], 0) == -1 and m.num_free_blocks() == 14  # no slot: nothing allocated
+    m.free_sequence(7)
+    assert m.add_sequence(9, [4], 0) == 0
+    m.state_slots_into([9, 8], out.ctypes.data)
+    assert list(out) == [0, 1]
+    with pytest.raises(ValueError, match="prefix"):
+        n.KVBlockManager(16, 4, True, 2)
+    plain = n.KVBlockManager(16, 4, False)
+    plain.add_sequence(1, [1], 0)
+    plain.state_slots_into([1], out.ctypes.data)
+    assert out[0] == -1
+
+
 def test_kv_manager_prefix_cache(n):
     m = n.KVBlockManager(16, 4, True)
     prompt = list(range(100, 111))  # 11 tokens -> 2 full blocks registrable

@@ -80,6 +80,8 @@ CONFIGS = {
         parallel((20, 1, 16, 16, 0.7, 90, 16), (4, 4, 96, 40, 9), None),
         mamba(2, 70, 136, 1, 4, 2, moe(70, 5, 1.5, 16, 24)),
         parallel((2, 2, 160, 136, 0.2, 70, 160), (1, 1, 200, 33, 4), dense(72))]),
+    # no attention anywhere: nothing is paged
+    "recurrent": config(96, [mamba(4, 16, 24, 2, 4, 4, dense(64)), mamba(2, 48, 8, 1, 2, 1, moe(6, 2, 1.1, 24))], loop=(0, 2, 1)),
     # projection sizes that take the streaming decode GEMM (K % 128) and a split-K of several slabs
     "stream": config(512, [
         mamba(8, 64, 128, 2, 4, 1, dense(1024)),
