@@ -183,6 +183,7 @@ class LLMEngine:
         self.prefilling: list[_Req] = []
         self.running: list[_Req] = []
         self.finished: dict[int, _Req] = {}
+        self._newly_finished: list[int] = []  # ids the next step() return reports (abort finishes some too)
         self._ids = itertools.count()
         self.stats = {"prefill_tokens": 0, "decode_tokens": 0, "decode_steps": 0, "prefill_steps": 0,
                       "preemptions": 0, "graph_replays": 0, "mixed_steps": 0}
@@ -306,7 +307,7 @@ class LLMEngine:
                                          "prefill_s": 0.0})
 
     def has_unfinished(self) -> bool:
-        return bool(self.waiting or self.prefilling or self.running)
+        return bool(self.waiting or self.prefilling or self.running or self._newly_finished)
 
     def generate(self, prompts: list, params: SamplingParams | list | None = None) -> list[GenerationOutput]:
         """Batch generate: token-id lists or strings -> outputs in input order."""
@@ -332,7 +333,8 @@ class LLMEngine:
         )
 
     def step(self) -> list[int]:
-        """One scheduler iteration. Returns the ids finished by it.
+        """One scheduler iteration. Returns the ids finished since the previous one (by this step, or
+        by an ``abort`` before it, which reads the tokens in flight), unless popped already.
 
         * nothing running: a prefill step (chunks of up to ``max_prefill_tokens``);
         * running sequences and pending prompts with ``mixed_prefill_tokens`` > 0: ONE mixed forward
@@ -342,7 +344,12 @@ class LLMEngine:
           stalling all decodes for a whole prefill step;
         * otherwise a decode step (HIP-graph replay).
         """
-        done_before = set(self.finished)
+        self._step()
+        done = [rid for rid in dict.fromkeys(self._newly_finished) if rid in self.finished]
+        self._newly_finished.clear()
+        return done
+
+    def _step(self) -> None:
         if self.fault_hook is not None:
             self.fault_hook(self)
         if self.auto_expire:
@@ -354,7 +361,7 @@ class LLMEngine:
                 prev, self._pending_prefill = self._pending_prefill, None
                 self._run_prefill(chunks)
                 self._finish_prefill(prev)
-                return [k for k in self.finished if k not in done_before]
+                return
             self._finish_prefill(self._pending_prefill)
             self._pending_prefill = None
         if self._inflight is not None and not self._can_pipeline():
@@ -378,7 +385,6 @@ class LLMEngine:
                 batch = self._reserve_decode()
                 if batch:
                     self._run_decode(batch)
-        return [k for k in self.finished if k not in done_before]
 
     def abort(self, rid: int, reason: str = "abort") -> bool:
         """Stops a request wherever it is (queued, prefilling or decoding) and frees its KV blocks;
@@ -397,6 +403,7 @@ class LLMEngine:
                     r.finish_reason = reason
                     r.finish_t = time.perf_counter()
                     self.finished[rid] = r
+                    self._newly_finished.append(rid)
                     self.stats["aborted"] = self.stats.get("aborted", 0) + 1
                     return True
         return False
@@ -410,8 +417,9 @@ class LLMEngine:
         self.waiting.clear()
         self.prefilling.clear()
         self.running.clear()
+        self._newly_finished.clear()
         self.blocks = native().KVBlockManager(self.blocks.num_blocks(), self.block_size, self._prefix_cache, self.state_slots)
-        self.timer.collect()
+        self.timer.discard()  # the fault may have left events that cannot be read
         return ids
 
     def expired(self) -> list[int]:
@@ -892,6 +900,7 @@ class LLMEngine:
             self.running.remove(r)
             self.blocks.free_sequence(r.seq)
             self.finished[r.rid] = r
+            self._newly_finished.append(r.rid)
 
     def _preempt_one(self, protect: _Req | None) -> bool:
         for victim in reversed(self.running):
@@ -1152,21 +1161,25 @@ class LLMEngine:
             self._h_tokens[:Bp] = self._d_tokens[:Bp]
 
     def _capture(self, Bp: int):
+        """Records a decode step of Bp rows.  Other threads (an embedding worker) use the GPU
+        meanwhile: the capture is thread-local, so that their allocations and synchronisations
+        neither fail nor invalidate it."""
+        current = torch.cuda.current_stream(self.device)
+        live = self._d_state[:Bp].clone()
         try:
             s = torch.cuda.Stream(self.device)
-            live = self._d_state[:Bp].clone()
             self._d_state[:Bp] = self.state_slots  # a recurrence must not advance twice: warm up on the spare slot
-            s.wait_stream(torch.cuda.current_stream(self.device))
+            s.wait_stream(current)
             with torch.cuda.stream(s):
                 self._decode_body(Bp)  # warm-up (allocator, lazy init) outside the graph
-            torch.cuda.current_stream(self.device).wait_stream(s)
+            current.wait_stream(s)
             torch.cuda.synchronize(self.device)
             self._d_state[:Bp].copy_(live)
             self._d_cnt[:Bp].copy_(self._h_cnt[:Bp])  # the warm-up advanced the RNG counters
             g = torch.cuda.CUDAGraph()
             if self._graph_pool is None:
                 self._graph_pool = torch.cuda.graph_pool_handle()
-            with torch.cuda.graph(g, pool=self._graph_pool, stream=s):
+            with torch.cuda.graph(g, pool=self._graph_pool, stream=s, capture_error_mode="thread_local"):
                 self._decode_body(Bp)
             torch.cuda.synchronize(self.device)
             self._graphs[(Bp, self._fast, self._masked)] = g
@@ -1177,6 +1190,10 @@ class LLMEngine:
 
             logging.getLogger(__name__).warning("HIP graph capture failed (%s); decode runs eagerly", exc)
             self.use_graphs = False
+            # a capture that fails at its end leaves its side stream current
+            torch.cuda.set_stream(current)
+            self._d_state[:Bp].copy_(live)
+            self._d_cnt[:Bp].copy_(self._h_cnt[:Bp])
             return None
 
     def capture_all(self, sizes=None):

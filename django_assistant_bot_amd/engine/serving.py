@@ -19,9 +19,20 @@ import logging
 import queue
 import threading
 import time
-from concurrent.futures import Future
+from concurrent.futures import Future, InvalidStateError
 
 logger = logging.getLogger(__name__)
+
+
+def _answer(fut: Future, result=None, error: BaseException | None = None) -> None:
+    """Resolves a caller's future; a caller that is gone (a cancelled future) is skipped."""
+    try:
+        if error is not None:
+            fut.set_exception(error)
+        else:
+            fut.set_result(result)
+    except InvalidStateError:
+        pass
 
 
 class LLMWorker:
@@ -34,6 +45,7 @@ class LLMWorker:
         self._lock = threading.Lock()
         self.requests = 0
         self.faults = 0
+        self._down = False  # the reset after a fault failed: requests are refused
         self.healthy = True  # False after a sticky device error: /health reports 503 for a restart
         self.last_error = ""
         self._thread = threading.Thread(target=self._run, name="dab-llm-worker", daemon=True)
@@ -64,6 +76,8 @@ class LLMWorker:
             except queue.Empty:
                 return
             if ids == "__cancel__":
+                if self._down:
+                    continue
                 for rid, f in list(self._futures.items()):
                     if f is fut:
                         self.engine.abort(rid, "cancelled")
@@ -71,43 +85,58 @@ class LLMWorker:
                         del self._futures[rid]
                 continue
             try:
+                if self._down:
+                    raise RuntimeError(f"the engine is down ({self.last_error})")
                 rid = self.engine.add_request(ids, params)
                 self._futures[rid] = fut
                 self.requests += 1
             except Exception as exc:  # invalid request: fail only this caller
-                fut.set_exception(exc)
+                _answer(fut, error=exc)
 
     def _run(self):
         while not self._stop:
-            self._drain()
-            if not self.engine.has_unfinished():
+            try:
+                self._drain()
+            except Exception as exc:  # an abort reads the tokens in flight: a step's failure
+                self._fault(exc)
+            if self._down or not self.engine.has_unfinished():
                 self._wake.wait(0.05)
                 self._wake.clear()
                 continue
             try:
                 finished = self.engine.step()
-            except Exception as exc:  # engine fault: fail every in-flight request, keep serving
-                logger.exception("engine step failed")
-                self.faults += 1
-                self.last_error = f"{type(exc).__name__}: {exc}"
-                if _sticky_device_error(exc):
-                    # a HIP fault poisons the context: stop taking work, let the supervisor restart
-                    self.healthy = False
-                for fut in self._futures.values():
-                    if not fut.done():
-                        fut.set_exception(exc)
-                self._futures.clear()
-                self.engine.fail_all()
+            except Exception as exc:
+                self._fault(exc)
                 continue
             for rid in finished:
                 fut = self._futures.pop(rid, None)
                 out = self.engine.pop_output(rid)
-                if fut is None or fut.done():
+                if fut is None:
                     continue
                 if out is not None and out.finish_reason.startswith("error:"):  # refused by a replica
-                    fut.set_exception(RuntimeError(f"request refused by the engine ({out.finish_reason})"))
+                    _answer(fut, error=RuntimeError(f"request refused by the engine ({out.finish_reason})"))
                 else:
-                    fut.set_result(out)
+                    _answer(fut, out)
+
+    def _fault(self, exc: Exception) -> None:
+        """Engine fault: fails every in-flight request and resets the engine; the worker goes on
+        serving, or refuses requests if the reset failed.  It never raises: without its thread every later caller would wait for ever."""
+        logger.error("engine step failed", exc_info=exc)
+        self.faults += 1
+        self.last_error = f"{type(exc).__name__}: {exc}"
+        if _sticky_device_error(exc):
+            # a HIP fault poisons the context: stop taking work, let the supervisor restart
+            self.healthy = False
+        try:
+            self.engine.fail_all()
+        except Exception as reset:
+            logger.error("engine reset failed", exc_info=reset)
+            self.healthy = False
+            self._down = True
+            self.last_error += f"; reset failed: {type(reset).__name__}: {reset}"
+        for fut in self._futures.values():
+            _answer(fut, error=exc)
+        self._futures.clear()
 
     def stop(self):
         self._stop = True
@@ -177,11 +206,11 @@ class EmbedWorker:
                     vecs = self.engine.embed(flat, normalize=norm).float().cpu().tolist() if flat else []
                 except Exception as exc:
                     for _, fut in items:
-                        fut.set_exception(exc)
+                        _answer(fut, error=exc)
                     continue
                 o = 0
                 for texts, fut in items:
-                    fut.set_result(vecs[o:o + len(texts)])
+                    _answer(fut, vecs[o:o + len(texts)])
                     o += len(texts)
                 self.requests += len(items)
 

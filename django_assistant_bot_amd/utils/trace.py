@@ -102,6 +102,10 @@ class GpuTimer:
         self._pending = keep
         return out
 
+    def discard(self) -> None:
+        """Forgets the recorded spans without reading them."""
+        self._pending = []
+
     def reset(self) -> None:
         self.collect()
         self.totals.clear()

@@ -151,6 +151,86 @@ def test_worker_marks_a_broken_tp_group_unhealthy():
         worker.stop()
 
 
+def test_worker_answers_later_callers_when_the_reset_after_a_fault_fails():
+    """A step fails and so does the engine reset: the worker's thread lives on and refuses requests,
+    instead of ending silently with every later caller waiting for ever."""
+    from django_assistant_bot_amd.engine import serving
+
+    eng = _engine(0, _weights())
+    worker = serving.LLMWorker(eng)
+
+    def fail(*_):
+        raise RuntimeError("injected failure")
+    try:
+        sp = SamplingParams(max_new_tokens=5, do_sample=False, temperature=0.0, ignore_eos=True)
+        eng.fault_hook, eng.fail_all = fail, fail
+        with pytest.raises(RuntimeError, match="injected"):
+            worker.submit(list(range(5, 25)), sp).result(timeout=60)
+        with pytest.raises(RuntimeError, match="engine is down"):
+            worker.submit(list(range(5, 25)), sp).result(timeout=60)
+        assert not worker.healthy and "reset failed" in worker.last_error and worker._thread.is_alive()
+    finally:
+        worker.stop()
+
+
+def test_workers_outlive_callers_that_are_gone():
+    """A future cancelled before its answer (a client that disconnected) is skipped by both workers."""
+    import threading
+
+    from django_assistant_bot_amd.engine import serving
+
+    gate = threading.Event()
+
+    class Encoder:
+        def embed(self, texts, normalize=None):
+            gate.wait(60)
+            return torch.ones(len(texts), 2)
+
+    emb = serving.EmbedWorker(Encoder())
+    gone = emb.submit(["a"])
+    assert gone.cancel()
+    gate.set()
+    assert emb.submit(["b"]).result(timeout=60) == [[1.0, 1.0]]
+
+    eng = _engine(0, _weights())
+    llm = serving.LLMWorker(eng)
+    try:
+        sp = SamplingParams(max_new_tokens=5, do_sample=False, temperature=0.0, ignore_eos=True)
+        eng.fault_hook = lambda e: gate.wait(60)
+        gate.clear()
+        gone = llm.submit(list(range(5, 25)), sp)
+        assert gone.cancel()  # its request runs to the end unread
+        gate.set()
+        assert len(llm.submit(list(range(5, 25)), sp).result(timeout=60).token_ids) == 5
+    finally:
+        llm.stop()
+
+
+@pytest.mark.parametrize("pipeline", [True, False])
+def test_requests_finished_by_an_abort_are_still_reported(pipeline):
+    """abort() reads the tokens in flight, which can finish other requests: the next step reports them."""
+    eng = _pipe_engine(pipeline, _weights())
+    sp = SamplingParams(max_new_tokens=6, do_sample=False, temperature=0.0, ignore_eos=True)
+    keep = [eng.add_request(list(range(5, 25 + i)), sp) for i in range(2)]
+    drop = eng.add_request(list(range(40, 60)), SamplingParams(max_new_tokens=60, do_sample=False, temperature=0.0,
+                                                               ignore_eos=True))
+    reported = []
+    for _ in range(20):
+        if all(len(r.out) == 5 for r in eng.running if r.rid in keep) and len(eng.running) == 3:
+            break
+        reported += eng.step()
+    assert not reported
+    assert eng.abort(drop)
+    eng.pop_output(drop)
+    if pipeline:
+        assert not eng.running  # the token in flight was the last of both
+    while eng.has_unfinished():
+        reported += eng.step()
+    assert sorted(reported) == keep
+    assert all(len(eng.pop_output(r).token_ids) == 6 for r in keep)
+    assert eng.step() == [] and not eng.has_unfinished()
+
+
 def _pipe_engine(pipeline: bool, weights):
     return LLMEngine(decoder_config("tiny-llama"), device="cpu", weights=dict(weights), max_batch=8, block_size=16,
                      num_blocks=64, max_prefill_tokens=256, use_graphs=False, pipeline_decode=pipeline)
