@@ -156,9 +156,10 @@ PYBIND11_MODULE(_native, m) {
                             (const float*)b_next, rows, cols, ST(s)),
           "dyt_residual");
   });
-  m.def("glu_f32", [](u out, long ldo, u x, long rows, int F, int gelu, u bias, u row_scale, u perm, u s) {
-    check(dab::glu_f32((float*)out, ldo, (const float*)x, rows, F, gelu, (const float*)bias, (const float*)row_scale,
-                       (const int*)perm, ST(s)),
+  m.def("glu_f32", [](u out, long ldo, u x, long rows, int F, int act, u bias, u row_scale, u perm, int scale_in,
+                      u s) {
+    check(dab::glu_f32((float*)out, ldo, (const float*)x, rows, F, act, (const float*)bias, (const float*)row_scale,
+                       (const int*)perm, scale_in, ST(s)),
           "glu_f32");
   });
   // chunked / sink attention over the paged cache
@@ -183,11 +184,18 @@ PYBIND11_MODULE(_native, m) {
   const auto proj = [](const P& t) {
     return dab::Proj{CVP(std::get<0>(t)), std::get<1>(t), std::get<2>(t), std::get<3>(t), std::get<4>(t)};
   };
-  m.def("rms_residual", [proj](u x, u h, int act_f32, const P& y, u bias, u pairs, int top, u ids, u table, u gain,
-                               int n_true, float eps, int rows, int cols, int fresh, u s) {
+  m.def("rms_residual", [proj](u x, u h, int act_f32, const P& y, u bias, u pairs, int top, u ids, u table,
+                               int table_f32, u post, u gain, int n_true, float eps, int rows, int cols, int fresh, u s) {
     check(dab::rms_residual((float*)x, VP(h), act_f32, proj(y), (const float*)bias, CVP(pairs), top, (const int*)ids,
-                            CVP(table), (const float*)gain, n_true, eps, rows, cols, fresh, ST(s)),
+                            CVP(table), table_f32, (const float*)post, (const float*)gain, n_true, eps, rows, cols, fresh,
+                            ST(s)),
           "rms_residual");
+  });
+  m.def("sigmoid_gate", [proj](const P& y, int col0, u x, long ldx, int act_f32, int n, int T, u s) {
+    check(dab::sigmoid_gate(proj(y), col0, VP(x), ldx, act_f32, n, T, ST(s)), "sigmoid_gate");
+  });
+  m.def("softcap", [proj](const P& y, float cap, u out, int n, int T, u s) {
+    check(dab::softcap(proj(y), cap, (float*)out, n, T, ST(s)), "softcap");
   });
   m.def("qk_rope_write", [proj](const P& y, int col0, int H, int G, int D, int dim, int rot, u freq, float eps, int norm,
                                 u positions, u slots, u q, u kc, u vc, int act_f32, int bs, int T, u s) {
@@ -201,6 +209,34 @@ PYBIND11_MODULE(_native, m) {
     check(dab::short_conv(proj(y), col0, C, taps, (const float*)w, (const float*)bias, VP(ring), (const int*)slot,
                           (const int*)pos, (const int*)cu, chunks, max_q, VP(out), act_f32, ST(s)),
           "short_conv");
+  });
+  m.def("short_conv_step", [proj](const P& y, int col0, int C, int taps, u w, u bias, u ring, u slot, u pos, int row0, int B,
+                                  u out, int act_f32, u s) {
+    check(dab::short_conv_step(proj(y), col0, C, taps, (const float*)w, (const float*)bias, VP(ring), (const int*)slot,
+                               (const int*)pos, row0, B, VP(out), act_f32, ST(s)),
+          "short_conv_step");
+  });
+  m.def("selective_state_width", &dab::selective_state_width);
+  m.def("narrow_rows", [proj](const P& z, u out, u low, int N, int R, int T, u s) {
+    check(dab::narrow_rows(proj(z), (float*)out, VP(low), N, R, T, ST(s)), "narrow_rows");
+  });
+  // shape = (C, Np, rank, b_col, c_col, z_col)
+  using SS = std::tuple<int, int, int, int, int, int>;
+  const auto sel = [](const SS& t) {
+    return dab::SelectiveShape{std::get<0>(t), std::get<1>(t), std::get<2>(t), std::get<3>(t), std::get<4>(t), std::get<5>(t)};
+  };
+  m.def("selective_scan", [proj, sel](u x, int act_f32, const SS& d, const P& dt, const P& bc, const P& y, u A, u dt_bias,
+                                      u skip, u state, u slot, u pos, u cu, int chunks, u out, u s) {
+    check(dab::selective_scan(CVP(x), act_f32, sel(d), proj(dt), proj(bc), proj(y), (const float*)A, (const float*)dt_bias,
+                              (const float*)skip, (float*)state, (const int*)slot, (const int*)pos, (const int*)cu, chunks,
+                              VP(out), ST(s)),
+          "selective_scan");
+  });
+  m.def("selective_step", [proj, sel](u x, int act_f32, const SS& d, u dt_w, const P& low, const P& y, u A, u dt_bias, u skip,
+                                      u state, u slot, u pos, int row0, int B, u out, u s) {
+    check(dab::selective_step(CVP(x), act_f32, sel(d), CVP(dt_w), proj(low), proj(y), (const float*)A, (const float*)dt_bias,
+                              (const float*)skip, (float*)state, (const int*)slot, (const int*)pos, row0, B, VP(out), ST(s)),
+          "selective_step");
   });
   // shape = (delta, H, G, D, Dp, V, C, q_col, k_col, v_col, a_col, b_col)
   using R = std::tuple<int, int, int, int, int, int, int, int, int, int, int, int>;
@@ -240,8 +276,8 @@ PYBIND11_MODULE(_native, m) {
                           VP(out), ldo, pad, row0, T, ST(s)),
           "gated_norm");
   });
-  m.def("moe_route", [proj](const P& z, int col0, int E, int top, float scale, u idx, u wt, int T, u s) {
-    check(dab::moe_route(proj(z), col0, E, top, scale, (int*)idx, (float*)wt, T, ST(s)), "moe_route");
+  m.def("moe_route", [proj](const P& z, int col0, int E, int top, float scale, int sigmoid, u idx, u wt, int T, u s) {
+    check(dab::moe_route(proj(z), col0, E, top, scale, sigmoid, (int*)idx, (float*)wt, T, ST(s)), "moe_route");
   });
   m.def("moe_plan", [](u idx, int pairs, int E, int bm, u perm, u tiles, int max_tiles, u s) {
     check(dab::moe_plan((const int*)idx, pairs, E, bm, (int*)perm, VP(tiles), max_tiles, ST(s)), "moe_plan");
@@ -253,9 +289,9 @@ PYBIND11_MODULE(_native, m) {
     check(dab::gemm_narrow(CVP(A), lda, CVP(B), (float*)C, M, N, K, S, ST(s)), "gemm_narrow");
   });
   m.def("gemm_grouped", [](u A, long lda, u B, u C, long ldc, int N, int K, u perm, int a_div, int scatter, u tiles,
-                           int n_tiles, int bm, int glu, u row_scale, u s) {
+                           int n_tiles, int bm, int glu, u row_scale, int scale_in, u s) {
     check(dab::gemm_grouped(CVP(A), lda, CVP(B), VP(C), ldc, N, K, (const int*)perm, a_div, scatter, CVP(tiles), n_tiles,
-                            bm, glu, (const float*)row_scale, ST(s)),
+                            bm, glu, (const float*)row_scale, scale_in, ST(s)),
           "gemm_grouped");
   });
   m.def("gemm_f32_grouped", [](u A, long lda, u B, u C, long ldc, int N, int K, u perm, int a_div, int scatter, u tiles,
@@ -270,9 +306,12 @@ PYBIND11_MODULE(_native, m) {
           "gemm_f32");
   });
   m.def("latent_write", [](u y, int y_f32, int S, long slab_stride, long ld, u q_out, int q_cols, u gain, u cache,
-                           int cache_f32, u slots, int T, int R, int rank, float eps, u s) {
+                           int cache_f32, u slots, int T, int R, int rank, float eps,
+                           const std::tuple<u, u, int, int, int, int, float>& rope, u s) {
+    const auto& [freq, positions, rot, D, q_at, c_at, mul] = rope;
     check(dab::latent_write(CVP(y), y_f32, S, slab_stride, ld, VP(q_out), q_cols, (const float*)gain, VP(cache),
-                            cache_f32, (const int64_t*)slots, T, R, rank, eps, ST(s)),
+                            cache_f32, (const int64_t*)slots, T, R, rank, eps,
+                            dab::LatentRope{(const double*)freq, (const int*)positions, rot, D, q_at, c_at, mul}, ST(s)),
           "latent_write");
   });
   m.def("latent_gather", [](u out, u cache, u bt, int max_blocks, int bs, u cu_k, u ctx, int B, int total,

@@ -86,11 +86,15 @@ __device__ __forceinline__ float gelu_tanh_f(float x) {
   return x * __builtin_amdgcn_rcpf(1.f + __expf(-u2));
 }
 
-// gate activation of the fused GLU epilogues
-template <bool GELU>
+// gate activation of the gated epilogues
+enum GluAct { GLU_SILU = 0, GLU_GELU = 1, GLU_RELU = 2 };
+template <int ACT>
 __device__ __forceinline__ float glu_act(float x) {
-  return GELU ? gelu_tanh_f(x) : silu_f(x);
+  return ACT == GLU_RELU ? fmaxf(x, 0.f) : ACT == GLU_GELU ? gelu_tanh_f(x) : silu_f(x);
 }
+// ... of the 8-row-group epilogues 4 (SiLU), 6 (tanh-GELU) and 7 (ReLU), the same numbers in every GEMM
+constexpr bool glu8_epilogue(int epi) { return epi == 4 || epi == 6 || epi == 7; }
+constexpr int glu8_act(int epi) { return epi == 7 ? GLU_RELU : epi == 6 ? GLU_GELU : GLU_SILU; }
 
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

@@ -186,11 +186,12 @@ int dyt_residual(float* x, void* h, int h_f32, const void* y, int y_f32, int S, 
   return hipGetLastError();
 }
 
-// 32-bit path of the gated MLP: x [rows, 2F] = [gate | up] (+ bias [gate | up]) -> gelu_tanh(gate) up (silu with
-// gelu == 0), times row_scale[perm[row]]
+// 32-bit path of the gated MLP: x [rows, 2F] = [gate | up] (+ bias [gate | up]) -> act(gate) up (``act``: GluAct),
+// times row_scale[perm[row]] (scale_in: the factor multiplies gate and up instead, before the bias)
 __global__ __launch_bounds__(256) void glu_f32_kernel(float* __restrict__ out, long ldo, const float* __restrict__ x,
-                                                      long rows, int F, int gelu, const float* __restrict__ bias,
-                                                      const float* __restrict__ row_scale, const int* __restrict__ perm) {
+                                                      long rows, int F, int act, const float* __restrict__ bias,
+                                                      const float* __restrict__ row_scale, const int* __restrict__ perm,
+                                                      int scale_in) {
   const int fv = F >> 2;
   const long n = rows * fv;
   for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n; i += (long)gridDim.x * 256) {
@@ -198,25 +199,30 @@ __global__ __launch_bounds__(256) void glu_f32_kernel(float* __restrict__ out, l
     const int c = (int)(i - r * fv) * 4;
     f32x4 g = *reinterpret_cast<const f32x4*>(x + r * 2 * F + c);
     f32x4 u = *reinterpret_cast<const f32x4*>(x + r * 2 * F + F + c);
+    const float rf = row_scale ? row_scale[perm[r]] : 1.f, rs = scale_in ? 1.f : rf;
+    if (scale_in) {
+      g *= rf;
+      u *= rf;
+    }
     if (bias) {
       g += *reinterpret_cast<const f32x4*>(bias + c);
       u += *reinterpret_cast<const f32x4*>(bias + F + c);
     }
-    const float rs = row_scale ? row_scale[perm[r]] : 1.f;
     f32x4 o;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) o[j] = (gelu ? gelu_tanh_f(g[j]) : silu_f(g[j])) * u[j] * rs;
+    for (int j = 0; j < 4; ++j) o[j] = (act == GLU_RELU ? fmaxf(g[j], 0.f) : act == GLU_GELU ? gelu_tanh_f(g[j]) : silu_f(g[j])) * u[j] * rs;
     *reinterpret_cast<f32x4*>(out + r * ldo + c) = o;
   }
 }
 
-int glu_f32(float* out, long ldo, const float* x, long rows, int F, int gelu, const float* bias, const float* row_scale,
-            const int* perm, hipStream_t s) {
+int glu_f32(float* out, long ldo, const float* x, long rows, int F, int act, const float* bias, const float* row_scale,
+            const int* perm, int scale_in, hipStream_t s) {
   if (rows <= 0) return 0;
   if (F <= 0 || F % 4 || ldo % 4 || (row_scale && !perm)) return hipErrorInvalidValue;
   const long n = rows * (F / 4);
   const unsigned grid = (unsigned)((n + 255) / 256 < 4096 ? (n + 255) / 256 : 4096);
-  hipLaunchKernelGGL(glu_f32_kernel, dim3(grid), dim3(256), 0, s, out, ldo, x, rows, F, gelu, bias, row_scale, perm);
+  hipLaunchKernelGGL(glu_f32_kernel, dim3(grid), dim3(256), 0, s, out, ldo, x, rows, F, act, bias, row_scale, perm,
+                     scale_in);
   return hipGetLastError();
 }
 

@@ -24,8 +24,11 @@
 
 namespace dab {
 
-// EPI_SWIGLU8 / EPI_GEGLU8: SiLU / tanh-GELU gate over 8-row [gate | up] groups; EPI_CANDIDATES is internal (gemm_score_candidates)
-enum EpiMode { EPI_NONE = 0, EPI_GELU = 1, EPI_SWIGLU = 2, EPI_SCORES = 3, EPI_SWIGLU8 = 4, EPI_CANDIDATES = 5, EPI_GEGLU8 = 6 };
+// EPI_SWIGLU8 / EPI_GEGLU8 / EPI_REGLU8: SiLU / tanh-GELU / ReLU gate over 8-row [gate | up] groups; EPI_CANDIDATES is
+// internal (gemm_score_candidates)
+enum EpiMode {
+  EPI_NONE = 0, EPI_GELU = 1, EPI_SWIGLU = 2, EPI_SCORES = 3, EPI_SWIGLU8 = 4, EPI_CANDIDATES = 5, EPI_GEGLU8 = 6, EPI_REGLU8 = 7
+};
 
 struct GemmParams {
   const bf16* A;
@@ -54,7 +57,8 @@ struct GemmParams {
   const int4* tiles;      // {expert, first sorted position, rows, -}
   const int* perm;        // sorted position -> (token, choice) pair
   int n_tiles, a_div, scatter;
-  const float* row_scale; // GLU: [pairs] factor of a row
+  const float* row_scale; // GLU: [pairs] factor of a row, of the result or (scale_in) of gate and up before the activation
+  int scale_in;
 };
 
 __device__ __forceinline__ int gsw(int r) { return 2 * ((r >> 1) & 3); }
@@ -176,14 +180,15 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
   }
 
   // epilogue: acc[ni][mi][r] = C[m = m0 + wm*TM + 16 mi + li][n = n0 + wn*TN + 16 ni + 4 g + r]
-  if constexpr (EPI == EPI_SWIGLU8 || EPI == EPI_GEGLU8) {
+  if constexpr (glu8_epilogue(EPI)) {
     // 8-row [gate | up] groups inside each 16-row block: v_permlane32_swap of blocks (2 pi, 2 pi + 1)
     // hands lanes 0-31 block 2 pi's gate / up rows and lanes 32-63 block 2 pi + 1's (gemm256.hip);
     // the swap runs with every lane active, the row / column bounds only guard the stores
 #pragma unroll
     for (int mi = 0; mi < MI; ++mi) {
       const int m = m0 + wm * TM + 16 * mi + li;
-      const float rs = GROUP && p.row_scale && m < p.M ? p.row_scale[p.perm[m]] : 1.f;
+      const float rf = GROUP && p.row_scale && m < p.M ? p.row_scale[p.perm[m]] : 1.f;
+      const float ri = GROUP && p.scale_in ? rf : 1.f, rs = GROUP && p.scale_in ? 1.f : rf;
 #pragma unroll
       for (int pi = 0; pi < NI / 2; ++pi) {
         const int oc = (n0 + wn * TN) / 2 + 16 * pi + 4 * g;
@@ -197,7 +202,8 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bt_kernel(GemmParams p) {
         for (int r = 0; r < 4; ++r) {
           const auto sw = __builtin_amdgcn_permlane32_swap(__float_as_uint(acc[2 * pi][mi][r]),
                                                            __float_as_uint(acc[2 * pi + 1][mi][r]), false, false);
-          o[r] = glu_act<EPI == EPI_GEGLU8>(__uint_as_float(sw[0]) + bg[r]) * (__uint_as_float(sw[1]) + bu[r]) * rs;
+          const float gt = __uint_as_float(sw[0]) * ri + bg[r], up = __uint_as_float(sw[1]) * ri + bu[r];
+          o[r] = glu_act<glu8_act(EPI)>(gt) * up * rs;
         }
         if (m < p.M && 2 * oc < p.N) {
           u32x2 v;
@@ -344,13 +350,13 @@ int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
   if (K % 64 || N % 4 || lda % 8 || ldb % 8) return hipErrorInvalidValue;
   if (b_group < 1 || (b_group > 1 && (b_rows <= 0 || b_rows % (16 * b_group)))) return hipErrorInvalidValue;
   if (epilogue == EPI_SWIGLU && (N % 32 || out_f32)) return hipErrorInvalidValue;
-  if ((epilogue == EPI_SWIGLU8 || epilogue == EPI_GEGLU8) && (N % 32 || out_f32 || residual)) return hipErrorInvalidValue;
+  if (glu8_epilogue(epilogue) && (N % 32 || out_f32 || residual)) return hipErrorInvalidValue;
   if (b_rows > 0 && (b_rows < N || b_rows % 16 || ldb != K)) return hipErrorInvalidValue;
   GemmParams p{};
   p.A = (const bf16*)A;
   p.B = (const bf16*)B;
   p.C = C;
-  const bool glu8 = epilogue == EPI_SWIGLU8 || epilogue == EPI_GEGLU8;  // their bias is fp32 [gate | up]
+  const bool glu8 = glu8_epilogue(epilogue);  // their bias is fp32 [gate | up]
   p.bias = glu8 ? nullptr : (const bf16*)bias;
   p.glu_bias = glu8 ? (const float*)bias : nullptr;
   p.residual = (const bf16*)residual;
@@ -379,6 +385,7 @@ int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
     case EPI_SCORES: return launch_gemm<EPI_SCORES>(p, big, s, sh);
     case EPI_SWIGLU8: return launch_gemm<EPI_SWIGLU8>(p, big, s, sh);
     case EPI_GEGLU8: return launch_gemm<EPI_GEGLU8>(p, big, s, sh);
+    case EPI_REGLU8: return launch_gemm<EPI_REGLU8>(p, big, s, sh);
     default: return hipErrorInvalidValue;
   }
 }
@@ -405,7 +412,8 @@ int gemm_narrow(const void* A, long lda, const void* B, float* C, int M, int N, 
 }
 
 int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int N, int K, const int* perm, int a_div,
-                 int scatter, const void* tiles, int n_tiles, int bm, int glu, const float* row_scale, hipStream_t s) {
+                 int scatter, const void* tiles, int n_tiles, int bm, int glu, const float* row_scale, int scale_in,
+                 hipStream_t s) {
   if (n_tiles <= 0 || N <= 0) return 0;
   if (K % 64 || N % 32 || lda % 8 || ldc % 8 || !tiles || !perm || (bm != 32 && bm != 128 && bm != 256) || (row_scale && !glu))
     return hipErrorInvalidValue;
@@ -425,6 +433,7 @@ int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int 
   p.a_div = a_div;
   p.scatter = scatter;
   p.row_scale = row_scale;
+  p.scale_in = scale_in;
   const int bn = bm == 256 ? 256 : 128;
   const dim3 grid((unsigned)n_tiles * ((N + bn - 1) / bn));
   if (bm == 32) {

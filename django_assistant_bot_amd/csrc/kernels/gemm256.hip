@@ -45,7 +45,7 @@ namespace dab {
 
 namespace {
 
-enum { G_NONE = 0, G_GELU = 1, G_SWIGLU = 2, G_CAND = 3, G_SWIGLU8 = 4, G_GEGLU8 = 6 };
+enum { G_NONE = 0, G_GELU = 1, G_SWIGLU = 2, G_CAND = 3, G_SWIGLU8 = 4, G_GEGLU8 = 6, G_REGLU8 = 7 };
 
 struct G256 {
   const bf16* A;
@@ -551,9 +551,9 @@ __global__ __launch_bounds__(512) void gemm256_kernel(G256 p) {
             }
           }
       }
-    } else if constexpr (EPI == G_SWIGLU || EPI == G_SWIGLU8 || EPI == G_GEGLU8) {
+    } else if constexpr (EPI == G_SWIGLU || glu8_epilogue(EPI)) {
       // G_SWIGLU: weight rows interleaved in 16-row groups [gate 16 | up 16]: jn = 0 gate, jn = 1 up.
-      // G_SWIGLU8 (G_GEGLU8: tanh-GELU gate): 8-row groups [gate 8 | up 8] inside every 16-row MFMA block (the decode layout:
+      // G_SWIGLU8 (G_GEGLU8 / G_REGLU8: tanh-GELU / ReLU gate): 8-row groups [gate 8 | up 8] inside every 16-row MFMA block (the decode layout:
       // any 16-row multiple tiles it): lane g holds rows 4g..4g+3 of both blocks, so one
       // v_permlane32_swap of the (jn 0, jn 1) pair gives lanes 0-31 block 0's gate / up rows and
       // lanes 32-63 block 1's -- the same output column 16 wc + 4 g as the 16-row form.
@@ -561,7 +561,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(G256 p) {
       if constexpr (BIAS) {
 #pragma unroll
         for (int jh = 0; jh < 2; ++jh) {
-          if constexpr (EPI == G_SWIGLU8 || EPI == G_GEGLU8) {  // fp32 [gate N / 2 | up N / 2]
+          if constexpr (glu8_epilogue(EPI)) {  // fp32 [gate N / 2 | up N / 2]
             const float* fb = reinterpret_cast<const float*>(p.bias) + (n0 + 128 * jh) / 2 + 16 * e_wc + 4 * e_g;
             const f32x4 gv = *reinterpret_cast<const f32x4*>(fb), uv = *reinterpret_cast<const f32x4*>(fb + p.N / 2);
 #pragma unroll
@@ -588,7 +588,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(G256 p) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               float gt = acc[ih][jh][i][0][r], up = acc[ih][jh][i][1][r];
-              if constexpr (EPI == G_SWIGLU8 || EPI == G_GEGLU8) {
+              if constexpr (glu8_epilogue(EPI)) {
                 const auto sw = __builtin_amdgcn_permlane32_swap(__float_as_uint(gt), __float_as_uint(up), false, false);
                 gt = __uint_as_float(sw[0]);
                 up = __uint_as_float(sw[1]);
@@ -597,7 +597,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(G256 p) {
                 gt += bg[jh][r];
                 up += bu[jh][r];
               }
-              o[r] = glu_act<EPI == G_GEGLU8>(gt) * up;
+              o[r] = glu_act<glu8_act(EPI)>(gt) * up;
             }
             u32x2 v;
             v[0] = pack2bf(o[0], o[1]);
@@ -854,7 +854,7 @@ int gemm256(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
             int b_group) {
   if (!gemm256_ok(M, N, K, lda, ldb)) return hipErrorInvalidValue;
   if (b_group != 1 && !(b_group == 8 && b_shuf)) return hipErrorInvalidValue;  // (N % 256: whole groups)
-  if ((epilogue == G_SWIGLU || epilogue == G_SWIGLU8 || epilogue == G_GEGLU8) && residual) return hipErrorInvalidValue;
+  if ((epilogue == G_SWIGLU || glu8_epilogue(epilogue)) && residual) return hipErrorInvalidValue;
   if (b_shuf && ldb != K) return hipErrorInvalidValue;
   G256 p{};
   p.A = (const bf16*)A;
@@ -916,6 +916,10 @@ int gemm256(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
     case G_GEGLU8:
       if (hb) G256_LAUNCH(G_GEGLU8, true, false);
       else G256_LAUNCH(G_GEGLU8, false, false);
+      break;
+    case G_REGLU8:
+      if (hb) G256_LAUNCH(G_REGLU8, true, false);
+      else G256_LAUNCH(G_REGLU8, false, false);
       break;
     default: return hipErrorInvalidValue;
   }

@@ -37,7 +37,7 @@ namespace dab {
 
 namespace {
 
-enum { MID_NONE = 0, MID_SWIGLU8 = 4, MID_GEGLU8 = 6 };
+enum { MID_NONE = 0, MID_SWIGLU8 = 4, MID_GEGLU8 = 6, MID_REGLU8 = 7 };
 
 struct GMid {
   const bf16* A;
@@ -379,7 +379,7 @@ __global__ __launch_bounds__(512) void gemm_mid_kernel(GMid p) {
       asm volatile("" : "+v"(e_li), "+v"(e_g), "+v"(e_wc));
       const long c_rows = min(128, p.M - m0);
       const __amdgpu_buffer_rsrc_t rC = mk_rsrc(p.C + (size_t)m0 * p.ldc, (unsigned)(c_rows * p.ldc * 2));
-      if constexpr (EPI == MID_SWIGLU8 || EPI == MID_GEGLU8) {
+      if constexpr (glu8_epilogue(EPI)) {
         // 8-row [gate | up] groups inside each 16-row block: one permlane32_swap of the (jn, jn + 1)
         // pair gives lanes 0-31 block jn's gate / up rows and lanes 32-63 block jn + 1's
         f32x4 bg[2], bu[2];
@@ -403,7 +403,7 @@ __global__ __launch_bounds__(512) void gemm_mid_kernel(GMid p) {
             for (int r = 0; r < 4; ++r) {
               const auto s = __builtin_amdgcn_permlane32_swap(__float_as_uint(acc[i][2 * pr][r]),
                                                               __float_as_uint(acc[i][2 * pr + 1][r]), false, false);
-              o[r] = glu_act<EPI == MID_GEGLU8>(__uint_as_float(s[0]) + bg[pr][r]) * (__uint_as_float(s[1]) + bu[pr][r]);
+              o[r] = glu_act<glu8_act(EPI)>(__uint_as_float(s[0]) + bg[pr][r]) * (__uint_as_float(s[1]) + bu[pr][r]);
             }
             u32x2 v;
             v[0] = pack2bf(o[0], o[1]);
@@ -503,7 +503,7 @@ int gemm_mid(const void* A, long lda, const void* B, void* C, long ldc, const vo
              int b_group) {
   if (!gemm_mid_ok(M, N, K, lda)) return hipErrorInvalidValue;
   if (b_group != 1 && b_group != 8) return hipErrorInvalidValue;
-  if (epilogue != MID_NONE && epilogue != MID_SWIGLU8 && epilogue != MID_GEGLU8) return hipErrorInvalidValue;
+  if (epilogue != MID_NONE && !glu8_epilogue(epilogue)) return hipErrorInvalidValue;
   if (!slabs || !cnt || slab_bytes < gemm_mid_slab_bytes() || n_cnt < gemm_mid_counters(M, N) ||
       slab_bytes >= (1L << 32))
     return hipErrorInvalidValue;
@@ -551,6 +551,8 @@ int gemm_mid(const void* A, long lda, const void* B, void* C, long ldc, const vo
   else if (epilogue == MID_GEGLU8 && residual) MID_BK(MID_GEGLU8, true);
   else if (epilogue == MID_SWIGLU8) MID_BK(MID_SWIGLU8, false);
   else if (epilogue == MID_GEGLU8) MID_BK(MID_GEGLU8, false);
+  else if (epilogue == MID_REGLU8 && residual) MID_BK(MID_REGLU8, true);
+  else if (epilogue == MID_REGLU8) MID_BK(MID_REGLU8, false);
   else if (residual) MID_BK(MID_NONE, true);
   else MID_BK(MID_NONE, false);
 #undef MID_BK

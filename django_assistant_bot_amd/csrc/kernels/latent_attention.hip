@@ -10,7 +10,11 @@
 // Masks: a sliding window of `window` keys (self included; 0 = unlimited).  Softmax sink: one extra
 // logit per head that joins the denominator and has neither key nor value.
 //
-//   latent_write   : split-K slabs of the [q | latent] projection -> q rows, RMS norm, cache write
+// Rotary positions (optional): a rotated part of every query head and one rotated key part shared by the heads.  The
+// cached row then is [c | rotated key] and the expansions carry an identity block for the rotated columns, so both forms
+// stay what they are.
+//
+//   latent_write   : split-K slabs of the [q | latent] projection -> q rows, RMS norm, rotation, cache write
 //   latent_gather  : packed copy of the cached latents a prefill chunk sees (K / V expansion input)
 //   head_gemm      : Y[t, h, :] = W[h] X[t, h, :], weights in the ops.shuffle_weights layout
 //   latent_decode  : MFMA decode over key partitions, and the combine of the partitions
@@ -18,6 +22,7 @@
 //                    and shapes outside the MFMA kernels' tiles
 #include "common.h"
 #include "launchers.h"
+#include "proj.h"
 
 namespace dab {
 
@@ -25,13 +30,40 @@ namespace dab {
 
 // One workgroup per token.  Wave 0: latent columns [q_cols, q_cols + R) summed over the slabs, RMS over
 // the first `rank` of them, gain, cache row (slot < 0: no write).  Waves 1-3: the q columns (q_out set).
-template <typename YT, typename CT>
+// ROPE: latent columns c_at .. c_at + rot and the columns q_at .. q_at + rot of every D-wide head are rotated, neighbours
+// (2i, 2i + 1) being a pair; they take no part in the norm.  Heads and rotated parts start at multiples of 8.
+template <typename YT, typename CT, bool ROPE>
 __global__ __launch_bounds__(256) void latent_write_kernel(const YT* __restrict__ y, int S, long slab_stride, long ld,
                                                            CT* __restrict__ q_out, int q_cols,
                                                            const float* __restrict__ gain, CT* __restrict__ cache,
                                                            const int64_t* __restrict__ slots, int R, int rank,
-                                                           float eps) {
+                                                           float eps, LatentRope rope) {
+  extern __shared__ __attribute__((aligned(16))) float2 turn[];  // (cosine, sine) of every pair, 1 / 0 past the last
   const int t = blockIdx.x, tid = threadIdx.x;
+  const int rot8 = (rope.rot + 7) & ~7;
+  if constexpr (ROPE) {
+    const double pos = (double)rope.positions[t];
+    for (int i = tid; i < rot8 / 2; i += 256) {
+      float s = 0.f, c = 1.f;
+      if (2 * i < rope.rot) {
+        const double turns = pos * rope.freq[i];
+        sincos_turn(turns - rint(turns), s, c);
+        s *= rope.mul;
+        c *= rope.mul;
+      }
+      turn[i] = make_float2(c, s);
+    }
+    __syncthreads();
+  }
+  auto rotate = [&](int d, float(&v)[8]) {  // columns d .. d + 7 of a rotated part
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const float2 w = turn[d / 2 + j];
+      const float a = v[2 * j], b = v[2 * j + 1];
+      v[2 * j] = a * w.x - b * w.y;
+      v[2 * j + 1] = b * w.x + a * w.y;
+    }
+  };
   const YT* row = y + (size_t)t * ld;
   auto sum8 = [&](int c, float(&v)[8]) {
 #pragma unroll
@@ -65,6 +97,7 @@ __global__ __launch_bounds__(256) void latent_write_kernel(const YT* __restrict_
     float ss = 0.f;
     for (int c = tid * 8; c < R; c += 512) {  // columns past `rank` are exact zeros
       float v[8];
+      if (ROPE && c >= rope.c_at) break;
       sum8(q_cols + c, v);
 #pragma unroll
       for (int j = 0; j < 8; ++j) ss = fmaf(v[j], v[j], ss);
@@ -74,32 +107,51 @@ __global__ __launch_bounds__(256) void latent_write_kernel(const YT* __restrict_
     for (int c = tid * 8; c < R; c += 512) {
       float v[8];
       sum8(q_cols + c, v);
+      if (ROPE && c >= rope.c_at) {
+        if (c < rope.c_at + rot8) rotate(c - rope.c_at, v);
+      } else {
 #pragma unroll
-      for (int j = 0; j < 8; ++j) v[j] *= inv * gain[c + j];
+        for (int j = 0; j < 8; ++j) v[j] *= inv * gain[c + j];
+      }
       put8(out + c, v);
     }
   } else if (q_out) {
     for (int c = (tid - 64) * 8; c < q_cols; c += 192 * 8) {
       float v[8];
       sum8(c, v);
+      if constexpr (ROPE) {
+        const int d = c % rope.D - rope.q_at;
+        if (d >= 0 && d < rot8) rotate(d, v);
+      }
       put8(q_out + (size_t)t * q_cols + c, v);
     }
   }
 }
 
 int latent_write(const void* y, int y_f32, int S, long slab_stride, long ld, void* q_out, int q_cols, const float* gain,
-                 void* cache, int cache_f32, const int64_t* slots, int T, int R, int rank, float eps, hipStream_t s) {
+                 void* cache, int cache_f32, const int64_t* slots, int T, int R, int rank, float eps, LatentRope rope,
+                 hipStream_t s) {
   if (T <= 0) return 0;
+  if (rope.rot && (!q_out || !cache || !rope.freq || !rope.positions || rope.rot < 0 || rope.rot % 2 || rope.D < 8 || rope.D % 8 ||
+                   rope.q_at % 8 || rope.c_at % 8 || rope.q_at + rope.rot > rope.D || rope.c_at < rank || q_cols % rope.D ||
+                   rope.c_at + rope.rot > R || rope.rot > 4096))
+    return hipErrorInvalidValue;
   if (S < 1 || ld % 8 || q_cols % 8 || (cache && (R % 8 || rank < 1 || rank > R || !gain || !slots)) || !slots)
     return hipErrorInvalidValue;
   if (cache_f32 && !y_f32) return hipErrorInvalidValue;
-#define DAB_LW(YT, CT)                                                                                             \
-  hipLaunchKernelGGL((latent_write_kernel<YT, CT>), dim3(T), dim3(256), 0, s, (const YT*)y, S, slab_stride, ld,    \
-                     (CT*)q_out, q_cols, gain, (CT*)cache, slots, R, rank, eps)
+#define DAB_LW1(YT, CT, RO)                                                                                        \
+  hipLaunchKernelGGL((latent_write_kernel<YT, CT, RO>), dim3(T), dim3(256), RO ? (rope.rot + 7) / 8 * 32 : 0, s,   \
+                     (const YT*)y, S, slab_stride, ld, (CT*)q_out, q_cols, gain, (CT*)cache, slots, R, rank, eps, rope)
+#define DAB_LW(YT, CT)                    \
+  do {                                    \
+    if (rope.rot) DAB_LW1(YT, CT, true);  \
+    else DAB_LW1(YT, CT, false);          \
+  } while (0)
   if (y_f32 && cache_f32) DAB_LW(float, float);
   else if (y_f32) DAB_LW(float, bf16);
   else DAB_LW(bf16, bf16);
 #undef DAB_LW
+#undef DAB_LW1
   return hipGetLastError();
 }
 

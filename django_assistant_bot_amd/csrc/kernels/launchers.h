@@ -72,8 +72,10 @@ int any_attention(const void* q, const void* kc, const void* vc, int f32, const 
 
 // rms_stream.hip (RMS norms around an fp32 residual stream; rotary positions and q / k norm before attention)
 int rms_residual(float* x, void* h, int act_f32, Proj y, const float* bias, const void* pairs, int top, const int* ids,
-                 const void* table, const float* gain, int n_true, float eps, int rows, int cols, int fresh,
-                 hipStream_t s);
+                 const void* table, int table_f32, const float* post, const float* gain, int n_true, float eps, int rows,
+                 int cols, int fresh, hipStream_t s);
+int sigmoid_gate(Proj y, int col0, void* x, long ldx, int act_f32, int n, int T, hipStream_t s);
+int softcap(Proj y, float cap, float* out, int n, int T, hipStream_t s);
 int qk_rope_write(Proj y, int col0, int H, int G, int D, int dim, int rot, const double* freq, float eps, int norm,
                   const int* positions, const int64_t* slots, void* q, void* kc, void* vc, int act_f32, int bs, int T,
                   hipStream_t s);
@@ -88,6 +90,9 @@ struct RecurrentShape {
 int recurrent_state_width(int D);  // D padded as the state is stored
 int short_conv(Proj y, int col0, int C, int taps, const float* w, const float* bias, void* ring, const int* slot,
                const int* pos, const int* cu, int chunks, int max_q, void* out, int act_f32, hipStream_t s);
+// one decoded token per sequence, rows row0..
+int short_conv_step(Proj y, int col0, int C, int taps, const float* w, const float* bias, void* ring, const int* slot,
+                    const int* pos, int row0, int B, void* out, int act_f32, hipStream_t s);
 int state_scan(const void* conv, int act_f32, RecurrentShape d, Proj gates, const float* A, const float* dt_bias,
                const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, void* out,
                hipStream_t s);
@@ -105,8 +110,24 @@ int state_decode(Proj y, int col0, int taps, const float* w, const float* bias, 
 int gated_norm(const void* y, int act_f32, Proj gate, int g_col, int n, int part, int gate_first, int per_head,
                const float* w, float eps, float scale, void* out, long ldo, int pad, int row0, int T, hipStream_t s);
 
+// selective_scan.hip (diagonal state-space recurrence with a step size, input and read-out of every token)
+struct SelectiveShape {
+  int C, Np;                 // channels, stored states of a channel (selective_state_width)
+  int rank, b_col, c_col;    // columns of the low-rank projection: step [0, rank), input, read-out
+  int z_col;                 // gate columns of the input projection
+};
+int selective_state_width(int N);  // N padded as the state is stored (0: too many)
+int narrow_rows(Proj z, float* out, void* low, int N, int R, int T, hipStream_t s);
+int selective_scan(const void* u, int act_f32, SelectiveShape d, Proj dt, Proj bc, Proj y, const float* A, const float* dt_bias,
+                   const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, void* out,
+                   hipStream_t s);
+int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, Proj low, Proj y, const float* A,
+                   const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos, int row0, int B,
+                   void* out, hipStream_t s);
+
 // moe.hip
-int moe_route(Proj z, int col0, int E, int top, float scale, int* idx, float* wt, int T, hipStream_t s);
+// sigmoid 0: softmax scores, weights over their sum; 1: sigmoid scores as they are
+int moe_route(Proj z, int col0, int E, int top, float scale, int sigmoid, int* idx, float* wt, int T, hipStream_t s);
 int moe_plan(const int* idx, int P, int E, int bm, int* perm, void* tiles, int max_tiles, hipStream_t s);
 int shared_glu(Proj y, int col0, int F, Proj z, int sg_col, void* out, long ldo, int act_f32, int T, hipStream_t s);
 
@@ -116,8 +137,8 @@ int embed_dyt(float* x, void* h, const int* ids, const void* table, int f32, flo
 int dyt_residual(float* x, void* h, int h_f32, const void* y, int y_f32, int S, long slab_stride, float a_post,
                  const float* w_post, const float* b_post, const float* ls, float a_next, const float* w_next,
                  const float* b_next, int rows, int cols, hipStream_t s);
-int glu_f32(float* out, long ldo, const float* x, long rows, int F, int gelu, const float* bias, const float* row_scale,
-            const int* perm, hipStream_t s);
+int glu_f32(float* out, long ldo, const float* x, long rows, int F, int act, const float* bias, const float* row_scale,
+            const int* perm, int scale_in, hipStream_t s);
 
 // gemm_f32.hip (32-bit mode; batched by strides)
 int gemm_f32(const float* A, long lda, long sa, const float* B, long ldb, long sb, float* C, long ldc, long sc, int M,
@@ -128,8 +149,17 @@ int gemm_f32_grouped(const float* A, long lda, const float* B, float* C, long ld
                      int scatter, const void* tiles, int n_tiles, hipStream_t s);
 
 // latent_attention.hip
+// rotary positions of latent_write: turns per position of the rot / 2 pairs, factor on cosine and sine, head width of the q
+// columns and where its rotated part starts in a head and in the latent row
+struct LatentRope {
+  const double* freq;
+  const int* positions;
+  int rot, D, q_at, c_at;
+  float mul;
+};
 int latent_write(const void* y, int y_f32, int S, long slab_stride, long ld, void* q_out, int q_cols, const float* gain,
-                 void* cache, int cache_f32, const int64_t* slots, int T, int R, int rank, float eps, hipStream_t s);
+                 void* cache, int cache_f32, const int64_t* slots, int T, int R, int rank, float eps, LatentRope rope,
+                 hipStream_t s);
 int latent_gather(void* out, const void* cache, const int* block_tables, int max_blocks, int block_size,
                   const int* cu_k, const int* ctx, int B, int total, int row_bytes, hipStream_t s);
 int head_gemm(void* y, long y_tok, long y_head, const void* x, long x_tok, long x_head, const void* w, int row0, int T,
@@ -144,17 +174,18 @@ int latent_any(void* out, const void* q, const void* cache, int f32, const int* 
                int window, float scale, hipStream_t s);
 
 // gemm.hip
-// b_rows > 0: B is an ops.shuffle_weights copy of b_rows (>= N) rows; epilogue 4 = SwiGLU over 8-row
-// [gate | up] groups
+// b_rows > 0: B is an ops.shuffle_weights copy of b_rows (>= N) rows; epilogue 4 / 6 / 7 = SiLU /
+// tanh-GELU / ReLU gate over 8-row [gate | up] groups
 int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc, const void* bias, const void* residual,
             long ldr, int M, int N, int K, int epilogue, int out_f32, const int* row_group, const int* q_group,
             const uint32_t* allow, int allow_words, hipStream_t s, int b_rows = 0, int b_group = 1);
 // a narrow fp32 product (router logits, recurrence gates) as S split-K slabs [S][M][N]: 32-row tiles, B a shuffle_weights copy
 int gemm_narrow(const void* A, long lda, const void* B, float* C, int M, int N, int K, int S, hipStream_t s);
 // experts: like gemm_f32_grouped, bf16, B = per-expert shuffle_weights copies of N rows; glu: SwiGLU over 8-row groups,
-// each row times row_scale[pair].  bm: rows of a tile (32, 128 or 256)
+// each row times row_scale[pair] (scale_in: gate and up times it, before the activation).  bm: rows of a tile (32, 128 or 256)
 int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int N, int K, const int* perm, int a_div,
-                 int scatter, const void* tiles, int n_tiles, int bm, int glu, const float* row_scale, hipStream_t s);
+                 int scatter, const void* tiles, int n_tiles, int bm, int glu, const float* row_scale, int scale_in,
+                 hipStream_t s);
 
 // gemm256.hip (large-M prefill / encoder GEMM, 256x256 phased schedule; epilogue 0 none, 1 GELU,
 // 2 SwiGLU on [gate 16 | up 16]-interleaved weight rows; bias / residual optional)

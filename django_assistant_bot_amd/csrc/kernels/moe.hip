@@ -1,7 +1,8 @@
 // Mixture of experts: routing, the row plan of the grouped GEMMs, and the shared expert's gated activation.
 //
 //   route        fp32 logits -> softmax over all experts -> the ``top`` largest, weights over their sum (+ 1e-20)
-//                times ``scale``; one wave per token
+//                times ``scale``; or (sigmoid) the scores' sigmoids, their ``top`` largest as they are times ``scale``;
+//                one wave per token
 //   plan         (token, expert) pairs grouped by expert: perm[sorted position] = pair, and the row tiles of
 //                the grouped GEMM, each {expert, first sorted position, rows}; one workgroup
 //   shared_glu   silu(gate) up sigmoid(w_sg h) of the expert that every token runs
@@ -14,8 +15,8 @@
 namespace dab {
 
 template <typename GT, int EI>
-__global__ __launch_bounds__(256) void moe_route_kernel(Proj z, int col0, int E, int top, float scale, int* idx, float* wt,
-                                                        int T) {
+__global__ __launch_bounds__(256) void moe_route_kernel(Proj z, int col0, int E, int top, float scale, int sigmoid, int* idx,
+                                                        float* wt, int T) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= T) return;
   float s[EI];
@@ -30,12 +31,12 @@ __global__ __launch_bounds__(256) void moe_route_kernel(Proj z, int col0, int E,
   float sum = 0.f;
 #pragma unroll
   for (int i = 0; i < EI; ++i) {
-    s[i] = __expf(s[i] - mx);
+    s[i] = sigmoid ? 1.f / (1.f + __expf(-s[i])) : __expf(s[i] - mx);
     sum += s[i];
   }
   sum = wave_sum(sum);
 #pragma unroll
-  for (int i = 0; i < EI; ++i) s[i] = lane + 64 * i < E ? s[i] / sum : -1.f;
+  for (int i = 0; i < EI; ++i) s[i] = lane + 64 * i < E ? (sigmoid ? s[i] : s[i] / sum) : -1.f;
   float total = 0.f, mine = 0.f;  // lane k keeps the k-th choice
   int mine_e = 0;
   for (int k = 0; k < top; ++k) {
@@ -67,17 +68,20 @@ __global__ __launch_bounds__(256) void moe_route_kernel(Proj z, int col0, int E,
   }
   if (lane < top) {
     idx[(size_t)t * top + lane] = mine_e;
-    wt[(size_t)t * top + lane] = mine / (total + 1e-20f) * scale;
+    wt[(size_t)t * top + lane] = (sigmoid ? mine : mine / (total + 1e-20f)) * scale;
   }
 }
 
-int moe_route(Proj z, int col0, int E, int top, float scale, int* idx, float* wt, int T, hipStream_t s) {
+int moe_route(Proj z, int col0, int E, int top, float scale, int sigmoid, int* idx, float* wt, int T, hipStream_t s) {
   if (T <= 0) return 0;
   if (E < 1 || E > 1024 || top < 1 || top > 64 || top > E || !z.f32 || z.S < 1) return hipErrorInvalidValue;
   const dim3 grid((T + 3) / 4);
-  if (E <= 64) hipLaunchKernelGGL((moe_route_kernel<float, 1>), grid, dim3(256), 0, s, z, col0, E, top, scale, idx, wt, T);
-  else if (E <= 256) hipLaunchKernelGGL((moe_route_kernel<float, 4>), grid, dim3(256), 0, s, z, col0, E, top, scale, idx, wt, T);
-  else hipLaunchKernelGGL((moe_route_kernel<float, 16>), grid, dim3(256), 0, s, z, col0, E, top, scale, idx, wt, T);
+  if (E <= 64) hipLaunchKernelGGL((moe_route_kernel<float, 1>), grid, dim3(256), 0, s, z, col0, E, top, scale, sigmoid, idx, wt,
+                                  T);
+  else if (E <= 256) hipLaunchKernelGGL((moe_route_kernel<float, 4>), grid, dim3(256), 0, s, z, col0, E, top, scale, sigmoid, idx, wt,
+                                  T);
+  else hipLaunchKernelGGL((moe_route_kernel<float, 16>), grid, dim3(256), 0, s, z, col0, E, top, scale, sigmoid, idx, wt,
+                                  T);
   return hipGetLastError();
 }
 

@@ -105,6 +105,30 @@ __device__ __forceinline__ void proj8(const Proj& p, long row, int col, float (&
   }
 }
 
+// cosine and sine of a whole number of turns' fraction r in [-1/2, 1/2]: the nearest quarter turn is taken off, then the
+// Taylor series on [-pi/4, pi/4] to fp32 rounding
+__device__ __forceinline__ void sincos_turn(double r, float& sn, float& cs) {
+  const double q = rint(4. * r);
+  const float a = (float)((r - 0.25 * q) * 6.283185307179586476925), z = a * a;
+  float s = fmaf(z, -2.5052108e-8f, 2.7557319e-6f);
+  s = fmaf(z, s, -1.9841270e-4f);
+  s = fmaf(z, s, 8.3333333e-3f);
+  s = fmaf(z, s, -1.6666667e-1f);
+  s = fmaf(a * z, s, a);
+  float c = fmaf(z, 2.0876757e-9f, -2.7557319e-7f);
+  c = fmaf(z, c, 2.4801587e-5f);
+  c = fmaf(z, c, -1.3888889e-3f);
+  c = fmaf(z, c, 4.1666667e-2f);
+  c = fmaf(z, c, -0.5f);
+  c = fmaf(z, c, 1.f);
+  const int k = (int)q & 3;
+  const float s1 = k & 1 ? c : s, c1 = k & 1 ? s : c;
+  sn = k & 2 ? -s1 : s1;
+  cs = (k == 1 || k == 2) ? -c1 : c1;
+}
+
+__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(__expf(z)); }
+
 // Type dispatch of kernels <projection type, activation type>: bf16 rows, fp32 slabs of a bf16 model, fp32 model.
 #define DAB_PROJ_DISPATCH(y, act_f32, CALL)   \
   do {                                        \

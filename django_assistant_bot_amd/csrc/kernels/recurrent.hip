@@ -23,7 +23,6 @@
 
 namespace dab {
 
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(__expf(z)); }
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + __expf(-z)); }
 
 // sum over the 8 lanes that share a column
@@ -153,6 +152,57 @@ int short_conv(Proj y, int col0, int C, int taps, const float* w, const float* b
   } while (0)
   DAB_PROJ_DISPATCH(y, act_f32, CONV_K);
 #undef CONV_K
+  return hipGetLastError();
+}
+
+// one decoded token per sequence: 8 channels a thread
+template <typename PT, typename AT>
+__global__ __launch_bounds__(64) void conv_step_kernel(ConvParams p, int row0) {
+  const int b = blockIdx.y, c = (blockIdx.x * 64 + threadIdx.x) * 8, row = row0 + b;
+  if (c >= p.C) return;
+  const int pos = p.pos[row], now = pos % p.taps;
+  AT* ring = (AT*)p.ring + (size_t)p.slot[b] * p.taps * p.C + c;
+  float cur[8], o[8], w[8];
+  proj8<PT>(p.y, row, p.col0 + c, cur);
+  ElemIO<float>::load8(p.w + (size_t)(p.taps - 1) * p.C + c, w);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) o[j] = 0.f;
+  if (p.bias) ElemIO<float>::load8(p.bias + c, o);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    cur[j] = ElemIO<AT>::round(cur[j]);
+    o[j] = fmaf(w[j], cur[j], o[j]);
+  }
+  for (int k0 = 1; k0 < p.taps; k0 += 4) {  // four past inputs requested at a time
+    float past[4][8], tap[4][8];
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int k = k0 + q, e = k < p.taps ? (now >= k ? now - k : now - k + p.taps) : now;
+      ElemIO<AT>::load8(ring + (size_t)e * p.C, past[q]);
+      ElemIO<float>::load8(p.w + (size_t)(k < p.taps ? p.taps - 1 - k : 0) * p.C + c, tap[q]);
+    }
+#pragma unroll
+    for (int q = 0; q < 4; ++q)
+      if (k0 + q < p.taps && k0 + q <= pos) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) o[j] = fmaf(tap[q][j], past[q][j], o[j]);
+      }
+  }
+  ElemIO<AT>::store8(ring + (size_t)now * p.C, cur);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) o[j] = silu_f(o[j]);
+  ElemIO<AT>::store8((AT*)p.out + (size_t)row * p.C + c, o);
+}
+
+int short_conv_step(Proj y, int col0, int C, int taps, const float* w, const float* bias, void* ring, const int* slot,
+                    const int* pos, int row0, int B, void* out, int act_f32, hipStream_t s) {
+  if (B <= 0) return 0;
+  if (C < 8 || C % 8 || col0 % 8 || y.ld % 8 || taps < 1 || taps > 16 || y.S < 1 || y.slab % 8 || B > 65535) return hipErrorInvalidValue;
+  ConvParams p{y, col0, C, taps, w, bias, ring, slot, pos, nullptr, out, 0};
+  const dim3 grid((C / 8 + 63) / 64, B);
+#define CSTEP_L(PT, AT) hipLaunchKernelGGL((conv_step_kernel<PT, AT>), grid, dim3(64), 0, s, p, row0)
+  DAB_PROJ_DISPATCH(y, act_f32, CSTEP_L);
+#undef CSTEP_L
   return hipGetLastError();
 }
 

@@ -2,7 +2,11 @@
 //
 //   embed_rms       x = table[id]; h = x / rms(x) * gain
 //   rms_residual    x += sublayer output (GEMM rows or split-K slabs) + bias + the token's expert rows
-//                   [+ table[id]];  h = x / rms(x) * gain: everything between two layers in one pass
+//                   [+ table[id]];  h = x / rms(x) * gain: everything between two layers in one pass.  With ``post``,
+//                   output + bias + expert rows pass an RMS norm of their own before they are added; without ``gain``
+//                   h is x as it is
+//   sigmoid_gate    x *= sigmoid(columns of a projection)
+//   softcap         cap tanh(y / cap) of the logits
 //   qk_rope_write   [q | k | v] columns of a projection -> interleaved rotary positions on q and k, weightless
 //                   RMS norm per head, q rows out, k / v into the paged cache
 //
@@ -31,27 +35,28 @@ struct RmsParams {
   const void* pairs;     // [rows * top, cols] activation type, or null
   int top;
   const int* ids;        // with table: x += table[ids[row]]
-  const void* table;
-  const float* gain;     // null: no h
+  const void* table;     // activation type, or fp32 (table_f32)
+  int table_f32;
+  const float* post;     // [cols] gain of the norm of what is added, or null
+  const float* gain;     // null: h = x
   float inv_n, eps;
   int rows, cols, fresh; // fresh: x starts at zero (embedding)
 };
 
 // one workgroup per row; a thread owns 8 columns at (tid + i blockDim) * 8, i < NV
-template <typename PT, typename AT, int NV>
+template <typename PT, typename AT, int NV, bool POST>
 __global__ __launch_bounds__(256) void rms_residual_kernel(RmsParams p) {
-  __shared__ float red[4];
+  __shared__ float red[4], red_post[4];
   const int row = blockIdx.x;
   float x[NV][8];
-  float ss = 0.f;
+  float ss = 0.f, sp = 0.f;
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
     const int c = (threadIdx.x + i * blockDim.x) * 8;
 #pragma unroll
     for (int j = 0; j < 8; ++j) x[i][j] = 0.f;
     if (c >= p.cols) continue;
-    float* xr = p.x + (size_t)row * p.cols + c;
-    if (!p.fresh) ElemIO<float>::load8(xr, x[i]);
+    if (!POST && !p.fresh) ElemIO<float>::load8(p.x + (size_t)row * p.cols + c, x[i]);
     if (p.y.p) {
       float v[8];
       proj8<PT>(p.y, row, c, v);
@@ -73,13 +78,36 @@ __global__ __launch_bounds__(256) void rms_residual_kernel(RmsParams p) {
         for (int j = 0; j < 8; ++j) x[i][j] += v[j];
       }
     }
+    if (POST) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) sp = fmaf(x[i][j], x[i][j], sp);
+    }
+  }
+  const float rp = POST ? 1.f / sqrtf(block_total(sp, red_post) * p.inv_n + p.eps) : 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + i * blockDim.x) * 8;
+    if (c >= p.cols) continue;
+    float* xr = p.x + (size_t)row * p.cols + c;
+    if (POST) {
+      float v[8], g[8];
+      ElemIO<float>::load8(xr, v);
+      ElemIO<float>::load8(p.post + c, g);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[i][j] = (p.fresh ? 0.f : v[j]) + x[i][j] * rp * g[j];
+    }
     if (p.table) {
       float v[8];
-      ElemIO<AT>::load8((const AT*)p.table + (size_t)p.ids[row] * p.cols + c, v);
+      if (p.table_f32) ElemIO<float>::load8((const float*)p.table + (size_t)p.ids[row] * p.cols + c, v);
+      else ElemIO<AT>::load8((const AT*)p.table + (size_t)p.ids[row] * p.cols + c, v);
 #pragma unroll
       for (int j = 0; j < 8; ++j) x[i][j] += v[j];
     }
     ElemIO<float>::store8(xr, x[i]);
+    if (!p.gain) {
+      if (p.h) ElemIO<AT>::store8((AT*)p.h + (size_t)row * p.cols + c, x[i]);
+      continue;
+    }
 #pragma unroll
     for (int j = 0; j < 8; ++j) ss = fmaf(x[i][j], x[i][j], ss);
   }
@@ -98,26 +126,95 @@ __global__ __launch_bounds__(256) void rms_residual_kernel(RmsParams p) {
 }
 
 int rms_residual(float* x, void* h, int act_f32, Proj y, const float* bias, const void* pairs, int top, const int* ids,
-                 const void* table, const float* gain, int n_true, float eps, int rows, int cols, int fresh,
-                 hipStream_t s) {
+                 const void* table, int table_f32, const float* post, const float* gain, int n_true, float eps, int rows,
+                 int cols, int fresh, hipStream_t s) {
   if (rows <= 0) return 0;
   if (cols <= 0 || cols % 8 || cols > 16384 || !x || (gain && !h) || n_true < 1 || (pairs && top < 1) ||
-      (table && !ids) || (y.p && (y.S < 1 || y.ld % 8)))
+      (table && !ids) || (post && !y.p && !pairs) || (y.p && (y.S < 1 || y.ld % 8)))
     return hipErrorInvalidValue;
   const int nv8 = cols / 8;
   const int bt = nv8 >= 256 ? 256 : (nv8 + 63) / 64 * 64;
   const int nv = (nv8 + bt - 1) / bt;
-  RmsParams p{x, h, y, bias, pairs, top, ids, table, gain, 1.f / n_true, eps, rows, cols, fresh};
+  RmsParams p{x, h, y, bias, pairs, top, ids, table, table_f32, post, gain, 1.f / n_true, eps, rows, cols, fresh};
   if (!y.p) p.y.f32 = act_f32;
-#define RMS_NV(PT, AT)                                                                                                 \
-  do {                                                                                                                 \
-    if (nv <= 1) hipLaunchKernelGGL((rms_residual_kernel<PT, AT, 1>), dim3(rows), dim3(bt), 0, s, p);                  \
-    else if (nv <= 2) hipLaunchKernelGGL((rms_residual_kernel<PT, AT, 2>), dim3(rows), dim3(bt), 0, s, p);             \
-    else if (nv <= 4) hipLaunchKernelGGL((rms_residual_kernel<PT, AT, 4>), dim3(rows), dim3(bt), 0, s, p);             \
-    else hipLaunchKernelGGL((rms_residual_kernel<PT, AT, 8>), dim3(rows), dim3(bt), 0, s, p);                          \
+#define RMS_L(PT, AT, NV)                                                                                      \
+  do {                                                                                                         \
+    if (post) hipLaunchKernelGGL((rms_residual_kernel<PT, AT, NV, true>), dim3(rows), dim3(bt), 0, s, p);      \
+    else hipLaunchKernelGGL((rms_residual_kernel<PT, AT, NV, false>), dim3(rows), dim3(bt), 0, s, p);          \
+  } while (0)
+#define RMS_NV(PT, AT)                  \
+  do {                                  \
+    if (nv <= 1) RMS_L(PT, AT, 1);      \
+    else if (nv <= 2) RMS_L(PT, AT, 2); \
+    else if (nv <= 4) RMS_L(PT, AT, 4); \
+    else RMS_L(PT, AT, 8);              \
   } while (0)
   DAB_PROJ_DISPATCH(p.y, act_f32, RMS_NV);
 #undef RMS_NV
+#undef RMS_L
+  return hipGetLastError();
+}
+
+// ----------------------------------------------------------------------------------------------
+
+template <typename PT, typename AT>
+__global__ __launch_bounds__(256) void sigmoid_gate_kernel(Proj y, int col0, AT* x, long ldx, int n) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 8, t = blockIdx.y;
+  if (c >= n) return;
+  float g[8], v[8];
+  proj8<PT>(y, t, col0 + c, g);
+  ElemIO<AT>::load8(x + (size_t)t * ldx + c, v);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] /= 1.f + __expf(-g[j]);
+  ElemIO<AT>::store8(x + (size_t)t * ldx + c, v);
+}
+
+int sigmoid_gate(Proj y, int col0, void* x, long ldx, int act_f32, int n, int T, hipStream_t s) {
+  if (T <= 0) return 0;
+  if (n < 8 || n % 8 || col0 % 8 || y.ld % 8 || y.slab % 8 || ldx % 8 || y.S < 1 || T > (1 << 20)) return hipErrorInvalidValue;
+  for (int r = 0; r < T; r += 32768) {
+    Proj yr = y;
+    yr.p = (const char*)y.p + (size_t)r * y.ld * (y.f32 ? 4 : 2);
+    const dim3 grid((n / 8 + 255) / 256, T - r < 32768 ? T - r : 32768);
+#define SGATE_L(PT, AT) \
+  hipLaunchKernelGGL((sigmoid_gate_kernel<PT, AT>), grid, dim3(256), 0, s, yr, col0, (AT*)x + (size_t)r * ldx, ldx, n)
+    DAB_PROJ_DISPATCH(y, act_f32, SGATE_L);
+#undef SGATE_L
+  }
+  return hipGetLastError();
+}
+
+// tanh to fp32 rounding: odd Taylor polynomial near zero, the exp form (no cancellation there) elsewhere
+__device__ __forceinline__ float tanh_exact(float x) {
+  const float a = fabsf(x), z = x * x;
+  if (a < 0.25f) {
+    float s = fmaf(z, 8.8632355e-3f, -2.1869489e-2f);
+    s = fmaf(z, s, 5.3968254e-2f);
+    s = fmaf(z, s, -1.3333333e-1f);
+    s = fmaf(z, s, 3.3333333e-1f);
+    return x - x * z * s;
+  }
+  const float t = 1.f - 2.f / (1.f + __expf(2.f * a));
+  return x < 0.f ? -t : t;
+}
+
+template <typename PT>
+__global__ __launch_bounds__(256) void softcap_kernel(Proj y, float cap, float inv, float* __restrict__ out, int n) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 8, t = blockIdx.y;
+  if (c >= n) return;
+  float v[8];
+  proj8<PT>(y, t, c, v);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] = cap * tanh_exact(v[j] * inv);
+  ElemIO<float>::store8(out + (size_t)t * n + c, v);
+}
+
+int softcap(Proj y, float cap, float* out, int n, int T, hipStream_t s) {
+  if (T <= 0) return 0;
+  if (n < 8 || n % 8 || y.ld % 8 || y.slab % 8 || y.S < 1 || T > 65535 || !(cap > 0.f)) return hipErrorInvalidValue;
+  const dim3 grid((n / 8 + 255) / 256, T);
+  if (y.f32) hipLaunchKernelGGL(softcap_kernel<float>, grid, dim3(256), 0, s, y, cap, 1.f / cap, out, n);
+  else hipLaunchKernelGGL(softcap_kernel<bf16>, grid, dim3(256), 0, s, y, cap, 1.f / cap, out, n);
   return hipGetLastError();
 }
 
@@ -139,28 +236,6 @@ struct RopeParams {
   void* vc;
   int bs, T;
 };
-
-// cosine and sine of a whole number of turns' fraction r in [-1/2, 1/2]: the nearest quarter turn is taken off, then the
-// Taylor series on [-pi/4, pi/4] to fp32 rounding
-__device__ __forceinline__ void sincos_turn(double r, float& sn, float& cs) {
-  const double q = rint(4. * r);
-  const float a = (float)((r - 0.25 * q) * 6.283185307179586476925), z = a * a;
-  float s = fmaf(z, -2.5052108e-8f, 2.7557319e-6f);
-  s = fmaf(z, s, -1.9841270e-4f);
-  s = fmaf(z, s, 8.3333333e-3f);
-  s = fmaf(z, s, -1.6666667e-1f);
-  s = fmaf(a * z, s, a);
-  float c = fmaf(z, 2.0876757e-9f, -2.7557319e-7f);
-  c = fmaf(z, c, 2.4801587e-5f);
-  c = fmaf(z, c, -1.3888889e-3f);
-  c = fmaf(z, c, 4.1666667e-2f);
-  c = fmaf(z, c, -0.5f);
-  c = fmaf(z, c, 1.f);
-  const int k = (int)q & 3;
-  const float s1 = k & 1 ? c : s, c1 = k & 1 ? s : c;
-  sn = k & 2 ? -s1 : s1;
-  cs = (k == 1 || k == 2) ? -c1 : c1;
-}
 
 // One workgroup per token: the angles once (p * f formed in fp64, so they are exact to fp32 rounding at any position), then
 // groups of LPH lanes walk heads, the next head's elements requested under the current one.  A lane owns the elements

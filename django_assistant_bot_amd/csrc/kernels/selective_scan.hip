@@ -1,0 +1,374 @@
+// Selective scan (Mamba): a diagonal state of N entries per channel, carried in fp32 from step to step in per-sequence
+// slots.  Per channel c and entry n, with step dt_c > 0, input B_n and read-out C_n of the token:
+//   S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c u_c B_n;   y_c = (sum_n S[c, n] C_n + D_c u_c) silu(z_c)
+// u is the convolved input, dt = softplus(W_dt low + bias), and low | B | C come from one narrow projection of u.
+//
+//   narrow_rows     slabs of that projection -> fp32 rows, and its first columns in bf16 (operand of W_dt)
+//   selective_scan  prompt portions: a workgroup walks one sequence for a block of channels, a tile of tokens at a time
+//   selective_step  one decoded token per sequence; W_dt low is formed in the kernel, its weights read once for SB sequences
+//
+// A channel is shared by L neighbouring lanes, NS entries each, so a step's read-out is a sum over L lanes; four tokens'
+// sums are transposed across a quad, so each lane finishes one of them.  The state is stored [slot][channel][Np], Np = L NS
+// (zeros past N); A holds -exp(A_log) log2(e), so a decay is one v_exp.  Everything but u, z and the output is fp32.
+#include "launchers.h"
+#include "proj.h"
+
+namespace dab {
+
+// values of the lane whose quad index is ^1 / ^2, and of the lane 4 / 8 further in its row of 16
+template <int CTRL>
+__device__ __forceinline__ float dpp(float v) {
+  return __uint_as_float((unsigned)__builtin_amdgcn_update_dpp(0, (int)__float_as_uint(v), CTRL, 0xf, 0xf, true));
+}
+__device__ __forceinline__ float quad_xor1(float v) { return dpp<0xB1>(v); }
+__device__ __forceinline__ float quad_xor2(float v) { return dpp<0x4E>(v); }
+
+// sum over the quads of a group of L lanes (each lane's quad index kept)
+template <int L>
+__device__ __forceinline__ float across_quads(float v) {
+  if (L == 8) v += __shfl_xor(v, 4, 64);
+  if (L == 16) {
+    v += dpp<0x124>(v);  // row_ror:4
+    v += dpp<0x128>(v);  // row_ror:8
+  }
+  return v;
+}
+
+int selective_state_width(int N) {
+  if (N < 1 || N > 256) return 0;
+  return N <= 64 ? (N + 15) / 16 * 16 : N <= 128 ? 128 : 256;
+}
+
+// ----------------------------------------------------------------------------------------------
+
+template <bool LOW>
+__global__ __launch_bounds__(256) void narrow_rows_kernel(Proj z, float* __restrict__ out, bf16* __restrict__ low, int N, int R,
+                                                          long total) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= total) return;
+  const int w = N / 8;
+  const long t = i / w;
+  const int c = (int)(i - t * w) * 8;
+  float v[8];
+  proj8<float>(z, t, c, v);
+  ElemIO<float>::store8(out + t * N + c, v);
+  if (LOW && c < R) ElemIO<bf16>::store8(low + t * R + c, v);
+}
+
+int narrow_rows(Proj z, float* out, void* low, int N, int R, int T, hipStream_t s) {
+  if (T <= 0) return 0;
+  if (!z.f32 || z.S < 1 || N < 8 || N % 8 || R % 8 || R > N || z.ld % 4 || z.slab % 4) return hipErrorInvalidValue;
+  const long total = (long)T * (N / 8);
+  if (total > (1l << 38)) return hipErrorInvalidValue;
+  const dim3 grid((unsigned)((total + 255) / 256));
+  if (low) hipLaunchKernelGGL(narrow_rows_kernel<true>, grid, dim3(256), 0, s, z, out, (bf16*)low, N, R, total);
+  else hipLaunchKernelGGL(narrow_rows_kernel<false>, grid, dim3(256), 0, s, z, out, (bf16*)low, N, R, total);
+  return hipGetLastError();
+}
+
+// ----------------------------------------------------------------------------------------------
+// prompt portions
+
+struct SelScan {
+  const void* u;        // [T, C] convolved input
+  SelectiveShape d;
+  Proj dt;              // fp32 [T, C]: W_dt low
+  Proj bc;              // fp32 rows of the narrow projection (one slab)
+  Proj y;               // input projection, gate columns from z_col
+  const float* A;       // [C, Np]
+  const float* bias;    // [C]
+  const float* skip;    // [C]
+  float* state;
+  const int* slot;
+  const int* pos;
+  const int* cu;
+  void* out;            // [T, C]
+};
+
+template <typename PT, typename AT, int L, int NS, int TB>
+__global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
+  constexpr int CH = 256 / L, Np = L * NS, ITEMS = TB * CH / 8, BCV = TB * 2 * Np / 1024;
+  static_assert(ITEMS <= 256 && BCV * 1024 == TB * 2 * Np && TB % 4 == 0, "tile");
+  __shared__ __attribute__((aligned(16))) float2 dtx[TB][CH];    // (dt, dt u); then (y, -)
+  __shared__ __attribute__((aligned(16))) float bc[TB][2 * Np];  // B | C
+  const int tid = threadIdx.x, ch = tid / L, part = tid % L, c0 = blockIdx.x * CH, b = blockIdx.y;
+  const int r0 = p.cu[b], n = p.cu[b + 1] - r0;
+  if (n <= 0) return;
+  const int C = p.d.C, c = min(c0 + ch, C - 1);
+  float S[NS], A[NS];
+  float* sp = p.state + ((size_t)p.slot[b] * C + c) * Np + part * NS;
+  const float* ap = p.A + (size_t)c * Np + part * NS;
+  const bool fresh = p.pos[r0] == 0;
+#pragma unroll
+  for (int j = 0; j < NS; ++j) {
+    const float v = sp[j];
+    S[j] = fresh ? 0.f : v;
+    A[j] = ap[j];
+  }
+  // this thread's 8 channels of one token of a tile (CH and C are multiples of 8)
+  const int it = tid / (CH / 8), ic = (tid % (CH / 8)) * 8, cc = c0 + ic;
+  const bool item = tid < ITEMS && cc < C;
+  const int ccl = min(cc, C - 8);
+  float nu[8], nd[8], nz[8], bias[8], skip[8];
+  f32x4 nb[BCV];
+  ElemIO<float>::load8(p.bias + ccl, bias);
+  ElemIO<float>::load8(p.skip + ccl, skip);
+  auto fetch = [&](int t0) {  // rows past the portion are clamped, and nulled when they are used
+    const long row = r0 + min(t0 + min(it, TB - 1), n - 1);
+    ElemIO<AT>::load8((const AT*)p.u + row * C + ccl, nu);
+    proj8<float>(p.dt, row, ccl, nd);
+    proj8<PT>(p.y, row, p.d.z_col + ccl, nz);
+#pragma unroll
+    for (int k = 0; k < BCV; ++k) {
+      const int e = (k * 256 + tid) * 4, t = e / (2 * Np), j = e % (2 * Np);
+      const int col = j < Np ? p.d.b_col + j : p.d.c_col + j - Np;
+      nb[k] = *reinterpret_cast<const f32x4*>((const float*)p.bc.p + (long)(r0 + min(t0 + t, n - 1)) * p.bc.ld + col);
+    }
+  };
+  fetch(0);
+  for (int t0 = 0; t0 < n; t0 += TB) {
+    float u[8], z[8];
+    const bool live = item && t0 + it < n;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      u[j] = nu[j];
+      z[j] = nz[j];
+    }
+    if (item) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const float dt = live ? softplus_f(nd[j] + bias[j]) : 0.f;
+        dtx[it][ic + j] = make_float2(dt, dt * u[j]);
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < BCV; ++k) *reinterpret_cast<f32x4*>(&bc[0][0] + (k * 256 + tid) * 4) = nb[k];
+    __syncthreads();
+    if (t0 + TB < n) fetch(t0 + TB);
+#pragma unroll 1
+    for (int t = 0; t < TB; t += 4) {
+      float y[4];
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const float2 v = dtx[t + q][ch];
+        const float* br = &bc[t + q][part * NS];
+        const float* cr = &bc[t + q][Np + part * NS];
+        y[q] = 0.f;
+#pragma unroll
+        for (int j = 0; j < NS; ++j) {
+          S[j] = fmaf(__builtin_amdgcn_exp2f(v.x * A[j]), S[j], v.y * br[j]);
+          y[q] = fmaf(S[j], cr[j], y[q]);
+        }
+      }
+      const bool b0 = part & 1, b1 = part & 2;
+      const float v0 = (b0 ? y[1] : y[0]) + quad_xor1(b0 ? y[0] : y[1]);
+      const float v1 = (b0 ? y[3] : y[2]) + quad_xor1(b0 ? y[2] : y[3]);
+      const float r = across_quads<L>((b1 ? v1 : v0) + quad_xor2(b1 ? v0 : v1));
+      if (part < 4) dtx[t + part][ch].x = r;
+    }
+    __syncthreads();
+    if (live) {
+      float o[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) o[j] = fmaf(skip[j], u[j], dtx[it][ic + j].x) * silu_f(z[j]);
+      ElemIO<AT>::store8((AT*)p.out + (size_t)(r0 + t0 + it) * C + cc, o);
+    }
+  }
+  if (c0 + ch < C) {
+#pragma unroll
+    for (int j = 0; j < NS; ++j) sp[j] = S[j];
+  }
+}
+
+static bool bad_shape(const SelectiveShape& d, const Proj& y) {
+  return d.C < 8 || d.C % 8 || d.Np != selective_state_width(d.Np) || d.rank < 0 || d.b_col % 4 || d.c_col % 4 || d.z_col % 8 ||
+         y.S < 1 || y.ld % 8 || y.slab % 8;
+}
+
+int selective_scan(const void* u, int act_f32, SelectiveShape d, Proj dt, Proj bc, Proj y, const float* A, const float* dt_bias,
+                   const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, void* out,
+                   hipStream_t s) {
+  if (chunks <= 0) return 0;
+  if (bad_shape(d, y) || !dt.f32 || dt.S != 1 || dt.ld % 4 || !bc.f32 || bc.S != 1 || bc.ld % 4 || chunks > 65535)
+    return hipErrorInvalidValue;
+  SelScan p{u, d, dt, bc, y, A, dt_bias, skip, state, slot, pos, cu, out};
+  // lanes per channel: more of them when the channels alone leave SIMDs without a wave
+  const long waves = (long)chunks * d.C / 16;
+#define SEL_L(PT, AT, L, NS, TB)                                                                                   \
+  hipLaunchKernelGGL((selective_scan_kernel<PT, AT, L, NS, TB>), dim3((d.C + 256 / L - 1) / (256 / L), chunks),    \
+                     dim3(256), 0, s, p)
+#define SEL_N(PT, AT)                                     \
+  do {                                                    \
+    switch (d.Np) {                                       \
+      case 16:                                            \
+        if (waves >= 1024) SEL_L(PT, AT, 4, 4, 32);       \
+        else if (waves >= 256) SEL_L(PT, AT, 8, 2, 64);   \
+        else SEL_L(PT, AT, 16, 1, 64);                    \
+        break;                                            \
+      case 32:                                            \
+        if (waves >= 1024) SEL_L(PT, AT, 4, 8, 32);       \
+        else SEL_L(PT, AT, 16, 2, 64);                    \
+        break;                                            \
+      case 48: SEL_L(PT, AT, 4, 12, 32); break;           \
+      case 64: SEL_L(PT, AT, 8, 8, 32); break;            \
+      case 128: SEL_L(PT, AT, 16, 8, 32); break;          \
+      case 256: SEL_L(PT, AT, 16, 16, 16); break;         \
+      default: return hipErrorInvalidValue;               \
+    }                                                     \
+  } while (0)
+  DAB_PROJ_DISPATCH(y, act_f32, SEL_N);
+#undef SEL_N
+#undef SEL_L
+  return hipGetLastError();
+}
+
+// ----------------------------------------------------------------------------------------------
+// one decoded token per sequence
+
+struct SelStep {
+  const void* u;        // [*, C]
+  SelectiveShape d;
+  const void* dt_w;     // [C, rank padded]: bf16 fragments (ops.shuffle_weights) or fp32 rows
+  Proj low;             // fp32 rows of the narrow projection: low | B | C
+  Proj y;
+  const float* A;
+  const float* bias;
+  const float* skip;
+  float* state;
+  const int* slot;
+  const int* pos;
+  int row0, B;
+  void* out;
+};
+
+constexpr int kMaxRank = 2048;
+
+// 64 channels (4 lanes each, NS state entries a lane) of SB sequences
+template <typename PT, typename AT, int NS, int SB>
+__global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
+  constexpr int Np = 4 * NS;
+  extern __shared__ __attribute__((aligned(16))) float sm[];  // low [SB][rank] | B, C [SB][2 Np] | dt [SB][64]
+  const int tid = threadIdx.x, ch = tid >> 2, part = tid & 3, c0 = blockIdx.x * 64, b0 = blockIdx.y * SB;
+  const int C = p.d.C, R = p.d.rank, c = min(c0 + ch, C - 1);
+  float* low = sm;
+  float* bc = sm + SB * R;
+  float* dts = bc + SB * 2 * Np;
+  float S[SB][NS], uv[SB], zv[SB];
+  float* sp[SB];
+  bool fresh[SB];
+#pragma unroll
+  for (int s = 0; s < SB; ++s) {
+    const int b = min(b0 + s, p.B - 1), row = p.row0 + b;
+    sp[s] = p.state + ((size_t)p.slot[b] * C + c) * Np + part * NS;
+    fresh[s] = p.pos[row] == 0;
+#pragma unroll
+    for (int j = 0; j < NS; j += 4) {
+      const f32x4 v = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(sp[s] + j));
+#pragma unroll
+      for (int e = 0; e < 4; ++e) S[s][j + e] = v[e];
+    }
+    uv[s] = ElemIO<AT>::load((const AT*)p.u + (size_t)row * C + c);
+    zv[s] = proj_f32<PT>(p.y, row, p.d.z_col + c);
+  }
+  for (int s = 0; s < SB; ++s) {
+    const float* src = (const float*)p.low.p + (long)(p.row0 + min(b0 + s, p.B - 1)) * p.low.ld;
+    for (int i = tid * 4; i < R; i += 1024)
+      *reinterpret_cast<f32x4*>(low + s * R + i) = *reinterpret_cast<const f32x4*>(src + i);
+    for (int i = tid * 4; i < 2 * Np; i += 1024)
+      *reinterpret_cast<f32x4*>(bc + s * 2 * Np + i) =
+          *reinterpret_cast<const f32x4*>(src + (i < Np ? p.d.b_col + i : p.d.c_col + i - Np));
+  }
+  __syncthreads();
+  // W_dt low: a lane holds 8 of every 32 columns of channel li; the four lane groups are summed
+  const int w = tid >> 6, lane = tid & 63, g = lane >> 4, li = lane & 15, cw = c0 + 16 * w;
+  if (cw < C) {  // (C is a multiple of 16 here: whole blocks)
+    float acc[SB];
+#pragma unroll
+    for (int s = 0; s < SB; ++s) acc[s] = 0.f;
+#pragma unroll 4
+    for (int k = 0; k < R / 32; ++k) {
+      float wv[8];
+      if constexpr (sizeof(AT) == 2) ElemIO<bf16>::load8((const bf16*)p.dt_w + ((size_t)(cw / 16) * (R / 32) + k) * 512 + lane * 8, wv);
+      else ElemIO<float>::load8((const float*)p.dt_w + (size_t)(cw + li) * R + 32 * k + 8 * g, wv);
+#pragma unroll
+      for (int s = 0; s < SB; ++s) {
+        float lv[8];
+        ElemIO<float>::load8(low + s * R + 32 * k + 8 * g, lv);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) acc[s] = fmaf(wv[j], lv[j], acc[s]);
+      }
+    }
+#pragma unroll
+    for (int s = 0; s < SB; ++s) {
+      acc[s] += __shfl_xor(acc[s], 16, 64);
+      acc[s] += __shfl_xor(acc[s], 32, 64);
+      if (g == 0) dts[s * 64 + 16 * w + li] = acc[s];
+    }
+  }
+  __syncthreads();
+  if (c0 + ch >= C) return;
+  const float bias = p.bias[c], skip = p.skip[c];
+  float A[NS];
+#pragma unroll
+  for (int j = 0; j < NS; ++j) A[j] = p.A[(size_t)c * Np + part * NS + j];
+#pragma unroll
+  for (int s = 0; s < SB; ++s) {
+    if (b0 + s >= p.B) break;
+    const float dt = softplus_f(dts[s * 64 + ch] + bias), x = dt * uv[s];
+    const float* br = bc + s * 2 * Np + part * NS;
+    float y = 0.f;
+#pragma unroll
+    for (int j = 0; j < NS; ++j) {
+      const float prev = fresh[s] ? 0.f : S[s][j];
+      S[s][j] = fmaf(__builtin_amdgcn_exp2f(dt * A[j]), prev, x * br[j]);
+      y = fmaf(S[s][j], br[Np + j], y);
+    }
+#pragma unroll
+    for (int j = 0; j < NS; j += 4)
+      __builtin_nontemporal_store(f32x4{S[s][j], S[s][j + 1], S[s][j + 2], S[s][j + 3]}, reinterpret_cast<f32x4*>(sp[s] + j));
+    y += quad_xor1(y);
+    y += quad_xor2(y);
+    if (part == 0)
+      ElemIO<AT>::store((AT*)p.out + (size_t)(p.row0 + b0 + s) * C + c, fmaf(skip, uv[s], y) * silu_f(zv[s]));
+  }
+}
+
+int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, Proj low, Proj y, const float* A,
+                   const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos, int row0, int B,
+                   void* out, hipStream_t s) {
+  if (B <= 0) return 0;
+  if (bad_shape(d, y) || d.C % 16 || d.rank < 32 || d.rank % 32 || d.rank > kMaxRank || !low.f32 || low.S != 1 || low.ld % 4 ||
+      B > 65535)
+    return hipErrorInvalidValue;
+  SelStep p{u, d, dt_w, low, y, A, dt_bias, skip, state, slot, pos, row0, B, out};
+  const int cb = (d.C + 63) / 64;
+  // several sequences a workgroup (one pass over W_dt) once there are workgroups enough
+  const int sb = d.Np <= 32 && d.rank <= 1024 && (long)cb * B >= 4096 ? 4 : 1;
+  const dim3 grid(cb, (B + sb - 1) / sb);
+  const size_t lds = (size_t)sb * (d.rank + 2 * d.Np + 64) * sizeof(float);
+#define STEP_L(PT, AT, NS, SB) hipLaunchKernelGGL((selective_step_kernel<PT, AT, NS, SB>), grid, dim3(256), lds, s, p)
+#define STEP_N(PT, AT)                          \
+  do {                                          \
+    switch (d.Np) {                             \
+      case 16:                                  \
+        if (sb == 4) STEP_L(PT, AT, 4, 4);      \
+        else STEP_L(PT, AT, 4, 1);              \
+        break;                                  \
+      case 32:                                  \
+        if (sb == 4) STEP_L(PT, AT, 8, 4);      \
+        else STEP_L(PT, AT, 8, 1);              \
+        break;                                  \
+      case 48: STEP_L(PT, AT, 12, 1); break;    \
+      case 64: STEP_L(PT, AT, 16, 1); break;    \
+      case 128: STEP_L(PT, AT, 32, 1); break;   \
+      case 256: STEP_L(PT, AT, 64, 1); break;   \
+      default: return hipErrorInvalidValue;     \
+    }                                           \
+  } while (0)
+  DAB_PROJ_DISPATCH(y, act_f32, STEP_N);
+#undef STEP_N
+#undef STEP_L
+  return hipGetLastError();
+}
+
+}  // namespace dab

@@ -64,7 +64,7 @@ struct StreamParams {
   int cap;
 };
 
-constexpr int ST_EPI_NONE = 0, ST_EPI_SWIGLU = 2, ST_EPI_SWIGLU8 = 4, ST_EPI_GEGLU8 = 6, ST_EPI_CAND = 8;
+constexpr int ST_EPI_NONE = 0, ST_EPI_SWIGLU = 2, ST_EPI_SWIGLU8 = 4, ST_EPI_GEGLU8 = 6, ST_EPI_REGLU8 = 7, ST_EPI_CAND = 8;
 
 constexpr int cgcd(int a, int b) { return b == 0 ? a : cgcd(b, a % b); }
 constexpr int clcm(int a, int b) { return a / cgcd(a, b) * b; }
@@ -390,7 +390,7 @@ __global__ __launch_bounds__(64 * (NWC + NL), 1) void stream_gemm_kernel(StreamP
     return;
   }
   bf16* out = (bf16*)p.out;
-  if (p.epi == ST_EPI_SWIGLU || p.epi == ST_EPI_SWIGLU8 || p.epi == ST_EPI_GEGLU8) {
+  if (p.epi == ST_EPI_SWIGLU || glu8_epilogue(p.epi)) {
     // hg-row groups: rows [2 hg i, 2 hg i + hg) gate, [2 hg i + hg, 2 hg (i + 1)) up -> output
     // columns n0/2 + hg i + j; each thread makes 4 outputs
     const int hg = p.epi == ST_EPI_SWIGLU ? 16 : 8, pp = hg / 4;
@@ -406,7 +406,7 @@ __global__ __launch_bounds__(64 * (NWC + NL), 1) void stream_gemm_kernel(StreamP
       }
       float o[4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[j] = (p.epi == ST_EPI_GEGLU8 ? gelu_tanh_f(gt[j]) : silu_f(gt[j])) * up[j];
+      for (int j = 0; j < 4; ++j) o[j] = (p.epi == ST_EPI_REGLU8 ? fmaxf(gt[j], 0.f) : p.epi == ST_EPI_GEGLU8 ? gelu_tanh_f(gt[j]) : silu_f(gt[j])) * up[j];
       u32x2 v;
       v[0] = pack2bf(o[0], o[1]);
       v[1] = pack2bf(o[2], o[3]);
@@ -546,7 +546,7 @@ int stream_gemm(const void* X, long ldx, const void* W, long ldw, void* out, lon
   const int bn = stream_gemm_bn(cfg);
   if (!bn || M > stream_gemm_max_m(cfg)) return hipErrorInvalidValue;
   if (N % bn || S < 1 || K % (S * KS) || ldx % 8 || ldw % 8 || ldo % 8) return hipErrorInvalidValue;
-  if (epilogue != ST_EPI_NONE && epilogue != ST_EPI_SWIGLU && epilogue != ST_EPI_SWIGLU8 && epilogue != ST_EPI_GEGLU8)
+  if (epilogue != ST_EPI_NONE && epilogue != ST_EPI_SWIGLU && !glu8_epilogue(epilogue))
     return hipErrorInvalidValue;
   if (epilogue == ST_EPI_SWIGLU && bn % 32) return hipErrorInvalidValue;  // whole 16 + 16 row pairs per tile
   if (S > 1 && (epilogue != ST_EPI_NONE || residual)) return hipErrorInvalidValue;

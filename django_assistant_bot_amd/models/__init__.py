@@ -1,5 +1,5 @@
-"""Model families: BERT-style sentence encoders, Llama-3-style, latent-attention (Vumuvik) and hybrid (Vugotar)
-decoders."""
+"""Model families: BERT-style sentence encoders, Llama-3-style, latent-attention (Vumuvik) and hybrid
+(Vugotar, Vunelix) decoders."""
 from .bert import BertEncoder, pack_sequences  # noqa: F401
 from .cache import AttnMeta, HybridCache, KVCache, LatentCache  # noqa: F401
 from .configs import (  # noqa: F401
@@ -11,6 +11,7 @@ from .configs import (  # noqa: F401
     LatentMixer,
     VugotarConfig,
     VumuvikConfig,
+    VunelixConfig,
     decoder_config,
     encoder_config,
     is_decoder,
@@ -20,14 +21,17 @@ from .llama import LlamaModel  # noqa: F401
 from .registry import DecoderFamily, decoder_family  # noqa: F401
 from .vugotar import VugotarModel  # noqa: F401
 from .vumuvik import VumuvikModel  # noqa: F401
+from .vunelix import VunelixModel  # noqa: F401
 from .weights import (  # noqa: F401
     load_decoder_checkpoint,
     load_encoder_checkpoint,
     load_vugotar_checkpoint,
     load_vumuvik_checkpoint,
+    load_vunelix_checkpoint,
     random_decoder_weights,
     random_encoder_weights,
     random_vugotar_weights,
     random_vumuvik_weights,
+    random_vunelix_weights,
     shard_decoder_weights,
 )

@@ -7,7 +7,9 @@ layers carry: a state slot per sequence, handed out by the same manager.
 """
 from __future__ import annotations
 
+import math
 from dataclasses import dataclass
+from typing import NamedTuple
 
 import torch
 
@@ -74,27 +76,41 @@ class LatentCache:
         return own * block_size * torch.finfo(dtype).bits // 8
 
 
+class RunMemory(NamedTuple):
+    """What one layer run keeps (None: nothing of the kind)."""
+
+    kv: tuple | None = None  # per-head keys and values: (kv_heads, D)
+    latent: int | None = None  # latent row: its padded width
+    ring: tuple | None = None  # convolution inputs per slot: (taps, channels)
+    state: tuple | None = None  # fp32 state per slot: its shape
+
+
 class HybridCache:
     """Memory of a decoder whose layers mix attention and recurrence, one entry per layer RUN (a looped layer has
-    its own in every pass).  Attention: paged K and V [num_blocks, kv_heads, block_size, D].  Recurrence: per slot
-    the ring of the last ``taps`` convolution inputs [slots, taps, channels] and the fp32 state [slots, heads, V,
-    Dp].  The last slot takes the writes of padded decode rows.  ``specs``: per run (attention (kv_heads, D) or None,
-    (taps, ``ops.RecurrentShape``))."""
+    its own in every pass).  Attention: paged K and V [num_blocks, kv_heads, block_size, D], or paged latent rows ``c``
+    [num_blocks, block_size, width].  Recurrence: per slot the ring of the last ``taps`` convolution inputs [slots, taps,
+    channels] and the fp32 state [slots, *shape].  The last slot takes the writes of padded decode rows."""
 
-    def __init__(self, specs, num_blocks, block_size, slots, device, dtype=torch.bfloat16):
+    def __init__(self, runs: list, num_blocks, block_size, slots, device, dtype=torch.bfloat16):
         self.num_blocks, self.block_size, self.slots = num_blocks, block_size, slots
-        z = lambda *shape, dt=dtype: torch.zeros(shape, device=device, dtype=dt)  # noqa: E731
-        self.k, self.v, self.ring, self.state = [], [], [], []
-        for attn, (taps, d) in specs:
+
+        def z(on, *shape, dt=dtype):
+            return None if on is None else torch.zeros(shape, device=device, dtype=dt)
+
+        self.k, self.v, self.c, self.ring, self.state = [], [], [], [], []
+        for m in runs:
             for c in (self.k, self.v):
-                c.append(None if attn is None else z(num_blocks, attn[0], block_size, attn[1]))
-            self.ring.append(z(slots, taps, d.C))
-            self.state.append(z(slots, d.H, d.V, d.Dp, dt=torch.float32))
+                c.append(m.kv and z(m.kv, num_blocks, m.kv[0], block_size, m.kv[1]))
+            self.c.append(z(m.latent, num_blocks, block_size, m.latent))
+            self.ring.append(z(m.ring, slots, *(m.ring or ())))
+            self.state.append(z(m.state, slots, *(m.state or ()), dt=torch.float32))
 
     @staticmethod
-    def bytes_per_block(specs, block_size, dtype=torch.bfloat16):
-        return sum(2 * a[0] * a[1] * block_size * torch.finfo(dtype).bits // 8 for a, _ in specs if a is not None)
+    def bytes_per_block(runs, block_size, dtype=torch.bfloat16):
+        cells = sum(2 * m.kv[0] * m.kv[1] for m in runs if m.kv) + sum(m.latent for m in runs if m.latent)
+        return cells * block_size * torch.finfo(dtype).bits // 8
 
     @staticmethod
-    def bytes_per_slot(specs, dtype=torch.bfloat16):
-        return sum(t * d.C * torch.finfo(dtype).bits // 8 + 4 * d.H * d.V * d.Dp for _, (t, d) in specs)
+    def bytes_per_slot(runs, dtype=torch.bfloat16):
+        ring = sum(math.prod(m.ring) for m in runs if m.ring) * torch.finfo(dtype).bits // 8
+        return ring + 4 * sum(math.prod(m.state) for m in runs if m.state)

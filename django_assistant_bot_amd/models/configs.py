@@ -8,6 +8,7 @@ directory is given.
 from __future__ import annotations
 
 import json
+import math
 import os
 from dataclasses import asdict, dataclass, field, replace
 
@@ -69,10 +70,44 @@ class DecoderConfig:
 
 # ------------------------------------------------------------------ latent-attention decoders (Vumuvik)
 
+# cached row widths of the MFMA decode kernel, and rows of (width, latent part) whose rest is a rotated key
+LATENT_TILES = (64, 128, 192, 256, 384, 512)
+ROTARY_TILES = ((320, 256), (576, 512))
+
+
+def _up(n: int, m: int) -> int:
+    return -(-n // m) * m
+
+
+@dataclass(frozen=True)
+class Yarn:
+    """YaRN scaling of rotary frequencies: divided by ``factor`` where a pair turns fewer than ``slow`` times in ``original``
+    positions, as they are where it turns more than ``fast`` times, a ramp over the pairs between."""
+
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
+class Rotary:
+    """Rotary positions on ``dims`` dimensions, neighbours (2i, 2i + 1) being a pair."""
+
+    dims: int
+    base: float = 10000.0
+    scaling: Yarn | None = None
+
+    @property
+    def gain(self) -> float:
+        """Factor on cosine and sine."""
+        return 1.0 if self.scaling is None else 0.1 * math.log(self.scaling.factor) + 1.0
+
 
 @dataclass(frozen=True)
 class LatentMixer:
-    """One latent-attention mixer: every head's keys and values are images of one ``rank``-wide latent."""
+    """One latent-attention mixer: every head's keys and values are images of one ``rank``-wide latent.  With ``rot`` a
+    head also has ``rot.dims`` rotated query dimensions, which meet one rotated key part that all heads share."""
 
     heads: int
     dim: int  # query / key width of a head
@@ -81,16 +116,41 @@ class LatentMixer:
     scale: float
     window: int = 0  # keys a query sees, itself included (0: all before it)
     kv_from: int | None = None  # layer whose cached latent this mixer reads (None: its own)
+    rot: Rotary | None = None
+    gate: bool = False  # the heads' output is multiplied with the sigmoid of a projection of the layer's input
+
+    # where the rotated parts start in a head and in a cached row (multiples of 8), and the widths up to their ends
+    @property
+    def q_at(self) -> int:
+        return _up(self.dim, 8)
+
+    @property
+    def c_at(self) -> int:
+        return _up(self.rank, 8)
+
+    @property
+    def head_width(self) -> int:
+        return max(self.q_at + self.rot.dims if self.rot else self.dim, self.vdim)
+
+    @property
+    def row_width(self) -> int:
+        return self.c_at + self.rot.dims if self.rot else self.rank
+
+    def padded_head(self) -> int:
+        """Common padded width of the query / key and value heads."""
+        return next((p for p in (64, 128, 256) if self.head_width <= p), _up(self.head_width, 64))
+
+    def padded_row(self) -> int:
+        """Padded width of a cached row: a tile of the MFMA decode kernel where one fits."""
+        tiles = LATENT_TILES if self.rot is None else sorted(LATENT_TILES + tuple(r for r, _ in ROTARY_TILES))
+        values = dict(ROTARY_TILES)
+        return next((p for p in tiles if self.row_width <= p and self.rank <= values.get(p, p)), _up(self.row_width, 64))
 
 
 @dataclass(frozen=True)
 class LatentLayer:
     mixer: LatentMixer
     ff: int | None  # hidden width of the gated MLP (None: the layer has no feed-forward)
-
-
-def _up(n: int, m: int) -> int:
-    return -(-n // m) * m
 
 
 @dataclass(frozen=True)
@@ -109,8 +169,6 @@ class VumuvikConfig:
     default_model_len: int = 8192  # engine default when max_model_len is not given
     bos_id: int = 0
     eos_ids: tuple = ()
-
-    RANK_TILES = (64, 128, 192, 256, 384, 512)  # latent widths of the MFMA decode kernel
 
     def __post_init__(self):
         for i, b in enumerate(self.blocks):
@@ -142,14 +200,10 @@ class VumuvikConfig:
         return _up(self.vocab_size, 128)
 
     def padded_head(self, i: int) -> int:
-        """Common padded width of the query / key and value heads of layer ``i``."""
-        m = self.blocks[i].mixer
-        d = max(m.dim, m.vdim)
-        return next((p for p in (64, 128, 256) if d <= p), _up(d, 64))
+        return self.blocks[i].mixer.padded_head()
 
     def padded_rank(self, i: int) -> int:
-        r = self.blocks[i].mixer.rank
-        return next((p for p in self.RANK_TILES if r <= p), _up(r, 64))
+        return self.blocks[i].mixer.padded_row()
 
     def padded_ff(self, i: int) -> int:
         return _up(self.blocks[i].ff, 64)
@@ -226,28 +280,62 @@ class Mamba2Mixer:
 
 
 @dataclass(frozen=True)
+class SelectiveMixer:
+    """Mamba's selective scan: a diagonal state of ``state`` entries per channel; step, input and read-out are projections
+    of the convolved channels, the step through ``dt_rank`` dimensions."""
+
+    inner: int
+    state: int
+    dt_rank: int
+    conv: int  # taps of the short convolution
+
+
+@dataclass(frozen=True)
 class DenseMlp:
-    """SwiGLU with biases on all three projections."""
+    """Gated MLP (in a Vugotar with biases on all three projections)."""
 
     ff: int
+    act: str = "silu"
 
 
 @dataclass(frozen=True)
 class MoeMlp:
-    """``top`` of ``experts`` SwiGLUs per token plus, with ``shared``, one that every token runs behind a sigmoid gate."""
+    """``top`` of ``experts`` SwiGLUs per token plus, with ``shared``, one that every token runs (in a Vugotar behind a
+    sigmoid gate).  ``scores``: of the router, "softmax" (weights over their sum) or "sigmoid" (weights as they are);
+    ``weigh``: what the weight multiplies, the expert's "output" or its "input"."""
 
     experts: int
     top: int
     scale: float
     ff: int
     shared: int | None = None
+    scores: str = "softmax"
+    weigh: str = "output"
+
+
+def loop_runs(layers: int, loop: tuple | None) -> list:
+    """(layer, pass that starts right before it or None) of every layer run, in order; ``loop`` = (start, stop, times)."""
+    a, b, t = loop or (0, 0, 1)
+    if a == b:
+        return [(i, None) for i in range(layers)]
+    return ([(i, None) for i in range(a)]
+            + [(i, k if i == a else None) for k in range(t) for i in range(a, b)]
+            + [(i, None) for i in range(b, layers)])
+
+
+def _check_loop(name: str, layers: int, loop: tuple | None) -> None:
+    if loop is not None:
+        a, b, t = loop
+        if not 0 <= a <= b <= layers or t < 1:
+            raise ValueError(f"{name}: loop {loop} outside the layers")
 
 
 @dataclass(frozen=True)
 class HybridLayer:
-    """x + mixer(norm(x)) + mlp(norm(x)): one norm, both sublayers read its output."""
+    """A mixer and a feed-forward.  Vugotar: x + mixer(norm(x)) + mlp(norm(x)), one norm that both read.  Vunelix: a norm
+    before and after each of the two."""
 
-    mixer: ParallelMixer | Mamba2Mixer
+    mixer: ParallelMixer | Mamba2Mixer | SelectiveMixer | LatentMixer
     mlp: DenseMlp | MoeMlp | None = None
 
 
@@ -290,10 +378,7 @@ class VugotarConfig:
             if isinstance(f, MoeMlp) and not 1 <= f.top <= min(f.experts, self.MAX_TOP) or (
                     isinstance(f, MoeMlp) and f.experts > self.MAX_EXPERTS):
                 raise ValueError(f"{where}: experts up to {self.MAX_EXPERTS}, of which up to {self.MAX_TOP} per token")
-        if self.loop is not None:
-            a, b, t = self.loop
-            if not 0 <= a <= b <= len(self.blocks) or t < 1:
-                raise ValueError(f"{self.name}: loop {self.loop} outside the layers")
+        _check_loop(self.name, len(self.blocks), self.loop)
 
     @property
     def layers(self) -> int:
@@ -301,12 +386,7 @@ class VugotarConfig:
 
     def runs(self) -> list:
         """(layer, embedding added before it) of every layer run, in order."""
-        a, b, t = self.loop or (0, 0, 1)
-        if a == b:
-            return [(i, False) for i in range(self.layers)]
-        return ([(i, False) for i in range(a)]
-                + [(i, k > 0 and i == a) for k in range(t) for i in range(a, b)]
-                + [(i, False) for i in range(b, self.layers)])
+        return [(i, bool(k)) for i, k in loop_runs(self.layers, self.loop)]
 
     @property
     def padded_hidden(self) -> int:
@@ -354,6 +434,100 @@ def vugotar_uniform(name: str, layers: int, vocab_size: int, hidden: int, left: 
     par = ParallelMixer(left, right, 0.5, 0.5)
     cycle = (HybridLayer(mamba, dense), HybridLayer(par, moe or dense), HybridLayer(par, dense))
     return VugotarConfig(name, vocab_size, hidden, tuple(cycle[i % 3] for i in range(layers)), loop=loop, **kw)
+
+
+# ------------------------------------------------------------------ recurrent / latent decoders (Vunelix)
+
+
+@dataclass(frozen=True)
+class VunelixConfig:
+    """Vunelix decoder: selective scans and rotary latent attention, dense ReLU-gated MLPs and sigmoid-routed experts, an RMS
+    norm before and after each.  ``loop`` = (start, stop, times) runs a stretch of layers several times with the same
+    weights (every pass with its own cache and state); before each pass the stream is mixed with the embedding by a
+    projection and a vector of the pass is added.  Logits: the tied embedding, softly capped."""
+
+    name: str
+    vocab_size: int
+    hidden: int
+    blocks: tuple  # of HybridLayer
+    eps: float = 1e-5
+    loop: tuple | None = None
+    softcap: float | None = None
+    max_position: int = 1 << 20  # no positional table: only the cache bounds a sequence
+    default_model_len: int = 8192
+    bos_id: int = 0
+    eos_ids: tuple = ()
+
+    MAX_STATE, MAX_STEP_RANK, MAX_TAPS, MAX_ROW, MAX_EXPERTS, MAX_TOP = 256, 2048, 16, 2048, 1024, 64  # of the kernels
+
+    def __post_init__(self):
+        for i, b in enumerate(self.blocks):
+            where, m, f = f"{self.name}: layer {i}", b.mixer, b.mlp
+            if isinstance(m, SelectiveMixer):
+                if not (1 <= m.state <= self.MAX_STATE and 1 <= m.dt_rank <= self.MAX_STEP_RANK and 1 <= m.conv <= self.MAX_TAPS):
+                    raise ValueError(f"{where}: state up to {self.MAX_STATE}, step rank up to {self.MAX_STEP_RANK}, taps up "
+                                     f"to {self.MAX_TAPS}")
+            else:
+                if m.rot is not None and (m.rot.dims % 2 or m.rot.dims < 2):
+                    raise ValueError(f"{where}: rotated dimensions come in pairs")
+                if m.padded_row() > self.MAX_ROW:
+                    raise ValueError(f"{where}: latent and rotated key up to {self.MAX_ROW} wide")
+            if isinstance(f, MoeMlp) and not 1 <= f.top <= min(f.experts, self.MAX_TOP) or (
+                    isinstance(f, MoeMlp) and f.experts > self.MAX_EXPERTS):
+                raise ValueError(f"{where}: experts up to {self.MAX_EXPERTS}, of which up to {self.MAX_TOP} per token")
+        _check_loop(self.name, len(self.blocks), self.loop)
+
+    @property
+    def layers(self) -> int:
+        return len(self.blocks)
+
+    def runs(self) -> list:
+        """(layer, pass that starts right before it or None) of every layer run, in order."""
+        return loop_runs(self.layers, self.loop)
+
+    @property
+    def passes(self) -> int:
+        """Passes of the loop (0: there is nothing to loop)."""
+        return sum(k is not None for _, k in self.runs())
+
+    @property
+    def padded_hidden(self) -> int:
+        return _up(self.hidden, 128)
+
+    @property
+    def padded_vocab(self) -> int:
+        return _up(self.vocab_size, 128)
+
+    def to_dict(self):
+        return asdict(self)
+
+    def params(self) -> int:
+        W = self.hidden
+        n = self.vocab_size * W + W + (2 * W * W + self.loop[2] * W if self.loop else 0)
+        for b in self.blocks:
+            m, f = b.mixer, b.mlp
+            n += 2 * W
+            if isinstance(m, SelectiveMixer):
+                n += m.inner * (3 * W + m.conv + 1 + 2 * m.dt_rank + 3 * m.state + 2)
+            else:
+                P = m.rot.dims if m.rot else 0
+                n += W * (m.heads * (m.dim + P + (2 if m.gate else 1) * m.vdim) + m.rank + P) + m.rank * (1 + m.heads * (m.dim + m.vdim))
+            if f is not None:
+                n += 2 * W
+            if isinstance(f, DenseMlp):
+                n += 3 * W * f.ff
+            elif f is not None:
+                n += f.experts * (3 * W * f.ff + W) + (3 * W * f.shared if f.shared else 0)
+        return n
+
+
+def vunelix_uniform(name: str, layers: int, vocab_size: int, hidden: int, mamba: SelectiveMixer, latent: LatentMixer,
+                    dense: DenseMlp, moe: MoeMlp | None, loop: tuple | None = None, **kw) -> VunelixConfig:
+    """A Vunelix whose layers repeat (scan + dense, latent attention + experts, latent attention + experts); without ``moe``
+    every MLP is dense."""
+    cycle = (HybridLayer(mamba, dense), HybridLayer(latent, moe or dense), HybridLayer(latent, moe or dense))
+    return VunelixConfig(name, vocab_size, hidden, tuple(cycle[i % 3] for i in range(layers)), loop=loop,
+                         softcap=kw.pop("softcap", 30.0), **kw)
 
 
 ENCODERS = {
@@ -420,6 +594,27 @@ DECODERS.update({
                     MoeMlp(12, 3, 1.7, 40, 72)),
         HybridLayer(ParallelMixer(ChunkedMixer(3, 3, 64, 64, 0.12, 0, 64), DeltaMixer(2, 2, 64, 64, 2)), None),
         HybridLayer(Mamba2Mixer(2, 64, 64, 1, 4, 1), MoeMlp(5, 1, 1.0, 24))), 1e-5, loop=(1, 3, 2), max_position=2048),
+})
+
+_YARN = Yarn(4.0, 4096, 32.0, 1.0)
+
+DECODERS.update({
+    # Llama-3-8B's width, MLP, vocabulary and head count; a 512-wide latent, 96 + 32 dimensions a head, 16-entry states
+    "vunelix-8b": vunelix_uniform(
+        "vunelix-8b", 28, 128256, 4096, SelectiveMixer(8192, 16, 256, 4),
+        LatentMixer(32, 96, 128, 512, 128 ** -0.5, rot=Rotary(32, 500000.0, _YARN), gate=True), DenseMlp(14336, "relu"), None),
+    # ... and with experts: 64 of 1024, 6 per token beside a shared one, at Llama-3.2-1B's width
+    "vunelix-moe": vunelix_uniform(
+        "vunelix-moe", 15, 128256, 2048, SelectiveMixer(4096, 16, 128, 4),
+        LatentMixer(16, 96, 128, 256, 128 ** -0.5, rot=Rotary(32, 500000.0, _YARN), gate=True), DenseMlp(8192, "relu"),
+        MoeMlp(64, 6, 1.0, 1024, 2048, "sigmoid", "input")),
+    # test size: every branch at unequal sizes
+    "tiny-vunelix": VunelixConfig("tiny-vunelix", 1000, 200, (
+        HybridLayer(SelectiveMixer(152, 20, 9, 3), MoeMlp(12, 3, 1.0, 40, 72, "sigmoid", "input")),
+        HybridLayer(LatentMixer(3, 40, 24, 80, 0.15, rot=Rotary(12, 5000.0, Yarn(3.0, 100, 16.0, 2.0)), gate=True), DenseMlp(168, "relu")),
+        HybridLayer(SelectiveMixer(96, 8, 4, 4), None),
+        HybridLayer(LatentMixer(5, 16, 56, 48, 0.2, rot=Rotary(32), gate=True), MoeMlp(5, 1, 1.0, 24, None, "sigmoid", "input"))),
+        1e-5, loop=(1, 3, 2), softcap=20.0, max_position=2048),
 })
 
 _ALIASES = {
@@ -575,7 +770,45 @@ def vugotar_config_from_dir(path: str) -> VugotarConfig:
     return VugotarConfig(_label(path), int(c["vocab"]), int(c["width"]), tuple(blocks), float(c["norm"]["eps"]), loop)
 
 
-_DIR_CONFIGS = {"vumuvik": vumuvik_config_from_dir, "vugotar": vugotar_config_from_dir}
+def vunelix_config_from_dir(path: str) -> VunelixConfig:
+    """config.json of a Vunelix checkpoint: ``architecture``, ``vocab``, ``width``, ``norm.eps``, ``loop`` and
+    ``logit_softcap`` (or none) and ``layers`` (each ``type``, ``mixer`` sizes and ``mlp`` or null)."""
+    c = _hf(path)
+    blocks = []
+    for i, L in enumerate(c["layers"]):
+        m, f = L["mixer"], L.get("mlp")
+        if L.get("type") == "mamba1":
+            mixer = SelectiveMixer(int(m["inner"]), int(m["state"]), int(m["dt_rank"]), int(m["conv"]))
+        elif L.get("type") == "latent_attention":
+            rot, P = m.get("rot"), int(m.get("rot_dim") or 0)
+            if P and (rot is None or int(rot["dims"]) != P):
+                raise ValueError(f"{path}: layer {i}: rot.dims must be rot_dim")
+            if P:
+                sc = rot.get("scaling")
+                rot = Rotary(P, float(rot["base"]), None if sc is None else Yarn(
+                    float(sc["factor"]), float(sc["original"]), float(sc["fast"]), float(sc["slow"])))
+            mixer = LatentMixer(int(m["heads"]), int(m["dim"]), int(m["vdim"]), int(m["kv_rank"]), float(m["scale"]),
+                                rot=rot if P else None, gate=True)
+        else:
+            raise ValueError(f"{path}: layer {i}: mixer type {L.get('type')!r} is not supported (mamba1, latent_attention)")
+        if f is None:
+            mlp = None
+        elif f.get("kind") == "dense":
+            mlp = DenseMlp(int(f["ff"]), "relu")
+        elif f.get("kind") == "moe":
+            r, sh = f["router"], f.get("shared")
+            mlp = MoeMlp(int(r["experts"]), int(r["top"]), 1.0, int(f["expert"]["ff"]), None if sh is None else int(sh["ff"]),
+                         "sigmoid", "input")
+        else:
+            raise ValueError(f"{path}: layer {i}: mlp kind {f.get('kind')!r} is not supported (dense, moe or null)")
+        blocks.append(HybridLayer(mixer, mlp))
+    lp, cap = c.get("loop"), c.get("logit_softcap")
+    loop = None if lp is None else (int(lp["start"]), int(lp["stop"]), int(lp["times"]))
+    return VunelixConfig(_label(path), int(c["vocab"]), int(c["width"]), tuple(blocks), float(c["norm"]["eps"]), loop,
+                         None if not cap else float(cap))
+
+
+_DIR_CONFIGS = {"vumuvik": vumuvik_config_from_dir, "vugotar": vugotar_config_from_dir, "vunelix": vunelix_config_from_dir}
 
 
 def _dir_architecture(path: str) -> str | None:
@@ -584,7 +817,7 @@ def _dir_architecture(path: str) -> str | None:
     return arch if arch in _DIR_CONFIGS else c.get("model_type")
 
 
-def decoder_config(name: str, **overrides) -> DecoderConfig | VumuvikConfig | VugotarConfig:
+def decoder_config(name: str, **overrides) -> DecoderConfig | VumuvikConfig | VugotarConfig | VunelixConfig:
     if checkpoint_dir(name):
         cfg = _DIR_CONFIGS.get(_dir_architecture(name), decoder_config_from_hf)(name)
         return replace(cfg, **overrides) if overrides else cfg

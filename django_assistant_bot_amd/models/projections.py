@@ -111,3 +111,47 @@ class FragmentProjections:
                 out = ops.stream_gemm(x, w, splits=s, cfg=cfg, nt=True, slab_dtype=sd, w_group=grp)
                 return ops.slab_reduce(out) if (s > 1 and not allow_slabs) else out
         return ops.gemm_bt(x, w, epilogue=epilogue, shuffled=self.frag, b_group=grp, out=out, glu_bias=glu_bias)
+
+
+class HybridProjections(FragmentProjections):
+    """The projections of a decoder that runs in bf16 (fragment layout on the GPU) or, with ``f32``, in 32-bit."""
+
+    f32 = False
+    GLU8 = {"silu": ops.EPI_SWIGLU8, "gelu": ops.EPI_GEGLU8, "relu": ops.EPI_REGLU8}
+
+    def _place(self, t, name: str = ""):
+        """A projection's weights as its GEMMs read them."""
+        if not self.frag:
+            return t
+        g = self.PROJ_GROUPS.get(name, 1)
+        g = g if t.shape[0] % (16 * g) == 0 and t.numel() * 2 < (1 << 31) else 1
+        if self.proj_group.setdefault((name, *t.shape), g) != g:
+            raise AssertionError("one grouping per projection shape")
+        return ops.shuffle_weights(t, g)
+
+    def _proj(self, x, w, dec: bool, allow_slabs: bool = True, name: str = ""):
+        if x.is_cuda and not self.f32:
+            return self._stream_or_tile(x, w, dec, allow_slabs, name, ops.EPI_NONE, self.proj_group.get((name, *w.shape), 1))
+        return ops.gemm_f32(x, w) if self.f32 else ops.gemm_bt(x, w)
+
+    def _aux(self, h, w, dec: bool, wide: bool = False):
+        """A projection whose result stays in 32 bits: decode-sized steps as split-K slabs; ``wide``: as many columns as
+        the large ones."""
+        if not (h.is_cuda and not self.f32):
+            return ops.gemm_f32(h, w)
+        if dec:
+            cfg, _ = self._stream_choice("aux", h.shape[0], w.shape[0], w.shape[1])
+            s = next((s for s in (16, 8, 4, 2) if w.shape[1] % (128 * s) == 0), 1)
+            if cfg >= 0 and s > 1:
+                return ops.stream_gemm(h, w, splits=s, cfg=cfg, nt=True)
+        return ops.gemm_bt(h, w, out_f32=True, shuffled=True) if wide else ops.gemm_narrow(h, w)
+
+    def _glu(self, h, w, act: str, dec: bool, out=None, bias=None):
+        """act(gate) * up of a [gate | up] projection (``bias`` fp32 [gate | up])."""
+        if h.is_cuda and not self.f32:
+            return self._stream_or_tile(h, w, dec, False, "gate_up", self.GLU8[act],
+                                        self.proj_group.get(("gate_up", *w.shape), 1), out=out, glu_bias=bias)
+        if self.interleaved_mlp:
+            y = ops.gemm_bt(h, w, epilogue=self.GLU8[act], glu_bias=bias)
+            return y if out is None else out.copy_(y)
+        return ops.glu_f32(ops.gemm_f32(h, w), act, bias=bias, out=out)

@@ -6,17 +6,20 @@ from typing import Callable
 
 import torch
 
-from .configs import DecoderConfig, VugotarConfig, VumuvikConfig
+from .configs import DecoderConfig, VugotarConfig, VumuvikConfig, VunelixConfig
 from .llama import LlamaModel
 from .vugotar import VugotarModel
 from .vumuvik import VumuvikModel
+from .vunelix import VunelixModel
 from .weights import (
     load_decoder_checkpoint,
     load_vugotar_checkpoint,
     load_vumuvik_checkpoint,
+    load_vunelix_checkpoint,
     random_decoder_weights,
     random_vugotar_weights,
     random_vumuvik_weights,
+    random_vunelix_weights,
 )
 
 
@@ -46,6 +49,8 @@ FAMILIES = {
     VumuvikConfig: DecoderFamily(VumuvikModel, _single(random_vumuvik_weights), _single(load_vumuvik_checkpoint),
                                  (torch.bfloat16, torch.float32)),
     VugotarConfig: DecoderFamily(VugotarModel, _single(random_vugotar_weights), _single(load_vugotar_checkpoint),
+                                 (torch.bfloat16, torch.float32)),
+    VunelixConfig: DecoderFamily(VunelixModel, _single(random_vunelix_weights), _single(load_vunelix_checkpoint),
                                  (torch.bfloat16, torch.float32)),
 }
 

@@ -23,9 +23,9 @@ from dataclasses import dataclass
 import torch
 
 from .. import ops
-from .cache import AttnMeta, HybridCache
+from .cache import AttnMeta, HybridCache, RunMemory
 from .configs import ChunkedMixer, DenseMlp, MoeMlp, ParallelMixer, VugotarConfig
-from .projections import FragmentProjections
+from .projections import HybridProjections
 from .weights import HybridLayout, hybrid_layout
 
 
@@ -70,7 +70,7 @@ def _recurrent_shape(mixer, lay: HybridLayout) -> ops.RecurrentShape:
                               a["a"], 0)
 
 
-class VugotarModel(FragmentProjections):
+class VugotarModel(HybridProjections):
     vocab_parallel = False
     custom_ar = None
     recurrent = True
@@ -93,14 +93,7 @@ class VugotarModel(FragmentProjections):
         self.proj_group = {}
 
         def mat(key, name=""):
-            t = take(key).to(self.device)
-            if not self.frag:
-                return t
-            g = self.PROJ_GROUPS.get(name, 1)
-            g = g if t.shape[0] % (16 * g) == 0 and t.numel() * 2 < (1 << 31) else 1
-            if self.proj_group.setdefault((name, *t.shape), g) != g:
-                raise AssertionError("one grouping per projection shape")
-            return ops.shuffle_weights(t, g)
+            return self._place(take(key).to(self.device), name)
 
         def vec(key):
             return take(key).to(self.device).contiguous() if key in weights else None
@@ -140,7 +133,8 @@ class VugotarModel(FragmentProjections):
     # ------------------------------------------------------------------ what the engine asks of a family
     def _specs(self):
         L = [self.layers[li] for li, _ in self.runs]
-        return [((x.attn.kv_heads, x.D) if x.attn else None, (x.conv_w.shape[0], x.rec)) for x in L]
+        return [RunMemory(kv=(x.attn.kv_heads, x.D) if x.attn else None, ring=(x.conv_w.shape[0], x.rec.C),
+                          state=(x.rec.H, x.rec.V, x.rec.Dp)) for x in L]
 
     def make_cache(self, num_blocks: int, block_size: int, slots: int = 1) -> HybridCache:
         return HybridCache(self._specs(), num_blocks, block_size, slots, self.device, self.dtype)
@@ -166,32 +160,6 @@ class VugotarModel(FragmentProjections):
                                    self.device)
 
     # ------------------------------------------------------------------ forward
-    def _proj(self, x, w, dec: bool, allow_slabs: bool = True, name: str = ""):
-        if x.is_cuda and not self.f32:
-            return self._stream_or_tile(x, w, dec, allow_slabs, name, ops.EPI_NONE, self.proj_group.get((name, *w.shape), 1))
-        return ops.gemm_f32(x, w) if self.f32 else ops.gemm_bt(x, w)
-
-    def _aux(self, h, w, dec: bool):
-        """The small fp32 projection: decode-sized steps as fp32 split-K slabs."""
-        if not (h.is_cuda and not self.f32):
-            return ops.gemm_f32(h, w)
-        if dec:
-            cfg, _ = self._stream_choice("aux", h.shape[0], w.shape[0], w.shape[1])
-            s = next((s for s in (16, 8, 4, 2) if w.shape[1] % (128 * s) == 0), 1)
-            if cfg >= 0 and s > 1:
-                return ops.stream_gemm(h, w, splits=s, cfg=cfg, nt=True)
-        return ops.gemm_narrow(h, w)
-
-    def _glu(self, h, L: HybridDecoderLayer, dec: bool, out) -> None:
-        w, b = L.gate_up_w, L.gate_up_b
-        if h.is_cuda and not self.f32:
-            self._stream_or_tile(h, w, dec, False, "gate_up", ops.EPI_SWIGLU8, self.proj_group.get(("gate_up", *w.shape), 1),
-                                 out=out, glu_bias=b)
-        elif self.interleaved_mlp:
-            out.copy_(ops.gemm_bt(h, w, epilogue=ops.EPI_SWIGLU8, glu_bias=b))
-        else:
-            ops.glu_f32(ops.gemm_f32(h, w), gelu=False, bias=b, out=out)
-
     def forward(self, ids: torch.Tensor, meta: AttnMeta, kv: HybridCache) -> torch.Tensor:
         """ids int32 [T] -> final hidden states [T, padded width] (after the last norm)."""
         T, cfg, n = ids.numel(), self.cfg, len(self.runs)
@@ -225,7 +193,7 @@ class VugotarModel(FragmentProjections):
         cat = torch.empty((T, lay.width), dtype=self.dtype, device=h.device)
         pairs = None
         if L.gate_up_w is not None:
-            self._glu(h, L, sk, cat[:, :lay.ff])
+            self._glu(h, L.gate_up_w, "silu", sk, cat[:, :lay.ff], L.gate_up_b)
         elif L.moe is not None:
             m = L.moe
             idx, wt = ops.moe_route(z, lay.aux.at["router"], m.experts, m.top, m.scale, T)

@@ -9,10 +9,8 @@ Per layer:  [q | latent] GEMM -> latent write (slab sum, RMS norm, cache) -> att
 norm1b, ls1, residual, norm2 (one launch) -> gate|up GEMM (+ tanh-GELU GLU) -> down GEMM -> norm2b, ls2,
 residual, next norm1 (one launch).
 
-Attention takes the cheaper exact form of the same scores: prefill expands K and V of the visible context
-from the cached latents and runs the windowed flash kernel; decode folds W_uk into the query and W_uv
-behind the softmax, so each cached latent is read once for all heads.  Layers that share a latent
-(``kv_from``) read the owner's cache with their own expansion, window and sink.
+Attention is ``latent_attn.LatentAttention``.  Layers that share a latent (``kv_from``) read the owner's cache with
+their own expansion, window and sink.
 
 The 32-bit mode (``dtype=torch.float32``) runs the same steps with fp32 weights, activations and cache on
 the fp32 MFMA GEMM and the absorbed attention kernel.
@@ -21,13 +19,13 @@ from __future__ import annotations
 
 from dataclasses import dataclass
 
-import numpy as np
 import torch
 
 from .. import ops
-from ..ops.latent import FLASH_WINDOW_DIMS, DytNorm, decode_split
+from ..ops.latent import DytNorm
 from .cache import AttnMeta, LatentCache
 from .configs import LatentMixer, VumuvikConfig
+from .latent_attn import LatentAttention, PrefillPlan
 from .projections import FragmentProjections
 
 
@@ -52,34 +50,7 @@ class LatentDecoderLayer:
     down_w: torch.Tensor | None = None
 
 
-class _PrefillPlan:
-    """What the chunks of one forward see: per window, the packed context rows (cu_k), and the latents
-    gathered for them (shared by the layers that read one cache)."""
-
-    def __init__(self, meta: AttnMeta, device):
-        self.meta, self.device = meta, device
-        self._cu: dict = {}
-        self._c: dict = {}
-
-    def context(self, window: int):
-        if window not in self._cu:
-            n = [min(ctx, q + window - 1) if window else ctx for q, ctx in self.meta.chunk_lens]
-            cu = torch.from_numpy(np.concatenate([[0], np.cumsum(n)]).astype(np.int32))
-            if self.device.type == "cuda":
-                cu = cu.pin_memory().to(self.device, non_blocking=True)
-            self._cu[window] = (cu, int(sum(n)))
-        return self._cu[window]
-
-    def latents(self, src: int, window: int, cache: LatentCache):
-        if (src, window) not in self._c:
-            cu, total = self.context(window)
-            # one source's rows stay live at a time: the layers that share them are neighbours
-            self._c = {k: v for k, v in self._c.items() if k[0] == src}
-            self._c[src, window] = ops.latent_gather(cache.c[src], self.meta.block_tables, cu, self.meta.ctx_lens, total)
-        return self._c[src, window]
-
-
-class VumuvikModel(FragmentProjections):
+class VumuvikModel(LatentAttention, FragmentProjections):
     vocab_parallel = False
     custom_ar = None
 
@@ -152,13 +123,8 @@ class VumuvikModel(FragmentProjections):
     def decode_part(self, batch: int, part_size: int) -> int:
         return part_size  # (the latent decode splits by partition count, ``_split``)
 
-    def _split(self, L: LatentDecoderLayer, batch: int, max_len: int) -> tuple[int, int]:
-        return decode_split(batch, L.mixer.heads, L.R, L.mixer.window, max_len) if self.frag else (1, 128)
-
     def make_workspace(self, max_batch: int, max_len: int, part_size: int):
-        rows = [(b * L.mixer.heads * self._split(L, b, max_len)[0], L.R) for L in self.layers
-                for b in range(1, max_batch + 1)]
-        return ops.LatentWorkspace(max(r for r, _ in rows), max(r * R for r, R in rows), self.device)
+        return self._latent_workspace(self.layers, max_batch, max_len)
 
     # ------------------------------------------------------------------ forward
     def _proj(self, x, w, dec: bool, allow_slabs: bool = True, name: str = "", epilogue=ops.EPI_NONE):
@@ -179,7 +145,7 @@ class VumuvikModel(FragmentProjections):
         # element-wise pass sums; short prefill steps do the same
         small_pf = not meta.decode and not meta.n_decode and T <= self.PREFILL_STREAM_MAX_M
         sk = self.frag and (meta.decode and T <= self.STREAM_MAX_M or small_pf)
-        plan = None if meta.decode else _PrefillPlan(meta, self.device)
+        plan = None if meta.decode else PrefillPlan(meta, self.device)
         x, h = ops.embed_dyt(ids, self.embed, self.cfg.embed_scale, self.layers[0].norm1)
         for li, L in enumerate(self.layers):
             nxt = self.layers[li + 1].norm1 if li + 1 < nl else self.final_norm
@@ -200,35 +166,7 @@ class VumuvikModel(FragmentProjections):
         qd = self._proj(h, L.qd_w, sk, name="qd")
         q = ops.latent_write(qd, HD, L.latent_norm, kv.c[li] if own else None, meta.slots, m.rank, self.cfg.eps)
         q = q.unflatten(1, (m.heads, L.D))
-        Tp = 0 if meta.decode else T - meta.n_decode
-        if Tp == T:
-            return self._prefill(L, q, src, meta, kv, plan)
-        if meta.decode:
-            return self._decode(L, q, kv.c[src], meta.block_tables, meta.ctx_lens, meta)
-        out = torch.empty((T, m.heads, L.D), dtype=self.dtype, device=q.device)
-        if Tp:
-            self._prefill(L, q[:Tp], src, meta, kv, plan, out[:Tp])
-        self._decode(L, q[Tp:], kv.c[src], meta.dec_block_tables, meta.dec_ctx_lens, meta, out[Tp:])
-        return out
-
-    def _decode(self, L: LatentDecoderLayer, q, cache, block_tables, ctx_lens, meta: AttnMeta, out=None):
-        m = L.mixer
-        qa = ops.head_gemm(q, L.absorb_w, L.R)
-        parts, min_part = self._split(L, q.shape[0], meta.max_len) if meta.workspace is not None else (1, 128)
-        oa = ops.latent_decode(qa, cache, block_tables, ctx_lens, m.scale, m.window, L.sink, parts, meta.workspace,
-                               meta.order, min_part)
-        return ops.head_gemm(oa, L.kv_w, L.D, row0=m.heads * L.D, out=out)
-
-    def _prefill(self, L: LatentDecoderLayer, q, src: int, meta: AttnMeta, kv: LatentCache, plan, out=None):
-        m, HD = L.mixer, L.mixer.heads * L.D
-        if self.f32 or L.D not in FLASH_WINDOW_DIMS:
-            oa = ops.latent_attention(ops.head_gemm(q, L.absorb_w, L.R), kv.c[src], meta.block_tables, meta.cu_q,
-                                      meta.ctx_lens, m.scale, m.window, L.sink)
-            return ops.head_gemm(oa, L.kv_w, L.D, row0=HD, out=out)
-        cu_k, total = plan.context(m.window)
-        kvx = self._proj(plan.latents(src, m.window, kv), L.kv_w, False, name="kv").view(total, 2, m.heads, L.D)
-        return ops.flash_attention_window(q, kvx[:, 0], kvx[:, 1], meta.cu_q, cu_k, meta.max_q, m.scale, m.window,
-                                          L.sink, out=out)
+        return self._latent_attend(L, q, src, meta, kv, plan)
 
     def logits(self, h: torch.Tensor) -> torch.Tensor:
         """[n, padded width] -> [n, vocab]."""

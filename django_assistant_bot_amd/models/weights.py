@@ -9,11 +9,14 @@ and slices the tensor-parallel shard of each projection (Megatron column / row s
 from __future__ import annotations
 
 import glob
+import math
 import os
 import re
 from dataclasses import dataclass
 
 import torch
+
+from ..ops.selective import state_width
 
 from .configs import (
     DecoderConfig,
@@ -21,8 +24,10 @@ from .configs import (
     EncoderConfig,
     MoeMlp,
     ParallelMixer,
+    SelectiveMixer,
     VugotarConfig,
     VumuvikConfig,
+    VunelixConfig,
     _up,
 )
 
@@ -512,3 +517,142 @@ def random_vugotar_tensors(cfg: VugotarConfig, device="cpu", dtype=torch.bfloat1
 def random_vugotar_weights(cfg: VugotarConfig, device="cpu", dtype=torch.bfloat16, seed=0, interleave_mlp=False) -> dict:
     device = torch.device(device)
     return _vugotar_layout(cfg, random_vugotar_tensors(cfg, device, dtype, seed), device, dtype, interleave_mlp)
+
+
+# ------------------------------------------------------------------------------------------------
+# Vunelix
+
+
+@dataclass(frozen=True)
+class SelectiveLayout:
+    """Padded sizes of a selective-scan layer: channels, state entries, step dimensions; columns of the narrow projection."""
+
+    inner: int
+    state: int
+    rank: int
+    b_col: int
+    c_col: int
+    narrow: int
+
+
+def selective_layout(m: SelectiveMixer) -> SelectiveLayout:
+    Np, R = state_width(m.state), _up(m.dt_rank, 64)
+    return SelectiveLayout(_up(m.inner, 128), Np, R, R, R + Np, R + 2 * Np)
+
+
+def _vunelix_layout(cfg: VunelixConfig, get, device, dtype, interleave_mlp) -> dict:
+    """``get(name, shape)`` -> the engine's tensors.  Scan layers: ``in_w`` [x; z], ``x_w`` (step | input | read-out, the fp32
+    projection), ``dt_w``, ``o_w``; attention layers: ``in_w`` [q; latent | rotated key; output gate], ``kv_w`` (K rows with an
+    identity block for the rotated key, then V rows), ``absorb_w`` (the K rows of every head transposed), ``o_w``.  Sizes
+    are padded with zeros; gains, biases, taps and recurrence constants are fp32, decays as -exp(A_log) log2(e)."""
+    W, Wp = cfg.hidden, cfg.padded_hidden
+
+    def mat(name, *shape):
+        return get(name, shape).to(device=device, dtype=dtype)
+
+    def vec(name, *shape):
+        return get(name, shape).to(device=device, dtype=torch.float32).contiguous()
+
+    def glu(p, ff, to):
+        return _gate_up(_pad(mat(p + "gate", ff, W), to, Wp), _pad(mat(p + "up", ff, W), to, Wp), interleave_mlp).contiguous()
+
+    def heads(t, H, n, at, D, cols):
+        """Rows of H heads of n -> H heads of D, from row ``at`` of each; columns padded to ``cols``."""
+        out = t.new_zeros((H, D, cols))
+        out[:, at:at + n, :t.shape[1]] = t.view(H, n, t.shape[1])
+        return out
+
+    embed = _pad(mat("embed", cfg.vocab_size, W), cfg.vocab_size, Wp)
+    w = {"embed": embed, "lm_head": _pad(embed, cfg.padded_vocab, Wp), "final_norm": _pad(vec("final.norm", W), Wp)}
+    if cfg.passes:
+        mix = mat("loop.in", W, 2 * W)
+        w["loop_w"] = torch.stack([_pad(mix[:, :W], Wp, Wp), _pad(mix[:, W:], Wp, Wp)])
+        w["loop_step"] = _pad(vec("loop.step", cfg.loop[2], W), cfg.loop[2], Wp)
+    for i, blk in enumerate(cfg.blocks):
+        p, m, f = f"l{i}.", blk.mixer, blk.mlp
+        q = p + "mix."
+        for n in ("norm1", "norm1b") + (("norm2", "norm2b") if f is not None else ()):
+            w[p + n] = _pad(vec(p + n, W), Wp)
+        if isinstance(m, SelectiveMixer):
+            lay, N, R = selective_layout(m), m.state, m.dt_rank
+            I = lay.inner
+            w[p + "in_w"] = _pad(mat(q + "in", 2 * m.inner, W).view(2, m.inner, W), 2, I, Wp).reshape(2 * I, Wp)
+            w[p + "conv_w"] = _pad(vec(q + "conv", m.inner, m.conv).t(), m.conv, I).contiguous()
+            w[p + "conv_b"] = _pad(vec(q + "conv.b", m.inner), I)
+            x, xw = mat(q + "x", R + 2 * N, m.inner), embed.new_zeros((_up(lay.narrow, 128), I))
+            for at, a, b in ((0, 0, R), (lay.b_col, R, R + N), (lay.c_col, R + N, R + 2 * N)):
+                xw[at:at + b - a, :m.inner] = x[a:b]
+            w[p + "x_w"] = xw
+            w[p + "dt_w"] = _pad(mat(q + "dt", m.inner, R), I, lay.rank)
+            w[p + "dt_bias"] = _pad(vec(q + "dt.b", m.inner), I)
+            decay = -torch.exp(vec(q + "A_log", m.inner, N).double()) * math.log2(math.e)
+            w[p + "A"] = _pad(decay.float(), I, lay.state).contiguous()
+            w[p + "skip"] = _pad(vec(q + "D", m.inner), I)
+            w[p + "o_w"] = _pad(mat(q + "o", W, m.inner), Wp, I)
+        else:
+            H, D, R, P = m.heads, m.padded_head(), m.padded_row(), m.rot.dims if m.rot else 0
+            full = mat(q + "q", H * (m.dim + P), W).view(H, m.dim + P, W)
+            qw = embed.new_zeros((H, D, Wp))
+            qw[:, :m.dim, :W] = full[:, :m.dim]
+            qw[:, m.q_at:m.q_at + P, :W] = full[:, m.dim:]
+            dkv = mat(q + "dkv", m.rank + P, W)
+            row = embed.new_zeros((R, Wp))
+            row[:m.rank, :W] = dkv[:m.rank]
+            row[m.c_at:m.c_at + P, :W] = dkv[m.rank:]
+            parts = [qw.reshape(H * D, Wp), row]
+            if m.gate:
+                parts.append(heads(mat(q + "g", H * m.vdim, W), H, m.vdim, 0, D, Wp).reshape(H * D, Wp))
+            fused = torch.cat(parts)
+            w[p + "in_w"] = _pad(fused, _up(fused.shape[0], 128), Wp)
+            w[p + "latent_norm"] = _pad(vec(q + "dkv.norm", m.rank), R)
+            uk = heads(mat(q + "uk", H * m.dim, m.rank), H, m.dim, 0, D, R)
+            for k in range(P):  # the rotated key part passes through
+                uk[:, m.q_at + k, m.c_at + k] = 1.0
+            uv = heads(mat(q + "uv", H * m.vdim, m.rank), H, m.vdim, 0, D, R)
+            w[p + "kv_w"] = torch.cat([uk.reshape(H * D, R), uv.reshape(H * D, R)])
+            w[p + "absorb_w"] = uk.transpose(1, 2).reshape(H * R, D).contiguous()
+            w[p + "o_w"] = _pad(mat(q + "o", W, H * m.vdim).view(W, H, m.vdim), Wp, H, D).reshape(Wp, H * D)
+        q = p + "mlp."
+        if isinstance(f, DenseMlp):
+            F = _up(f.ff, 128)
+            w[p + "gate_up_w"], w[p + "down_w"] = glu(q, f.ff, F), _pad(mat(q + "down", W, f.ff), Wp, F)
+        elif f is not None:
+            w[p + "router_w"] = _pad(mat(q + "router", f.experts, W), _up(f.experts, 128), Wp)
+            ex, F = [f"{q}e{e}." for e in range(f.experts)], _up(f.ff, 64)
+            w[p + "expert_gate_up_w"] = torch.cat([glu(e, f.ff, F) for e in ex])
+            w[p + "expert_down_w"] = torch.cat([_pad(mat(e + "down", W, f.ff), Wp, F) for e in ex])
+            if f.shared:
+                F = _up(f.shared, 128)
+                w[p + "gate_up_w"] = glu(q + "shared.", f.shared, F)
+                w[p + "down_w"] = _pad(mat(q + "shared.down", W, f.shared), Wp, F)
+    return w
+
+
+def load_vunelix_checkpoint(path: str, cfg: VunelixConfig, device="cpu", dtype=torch.bfloat16, interleave_mlp=False,
+                            reader: SafetensorsDir | None = None) -> dict:
+    return _vunelix_layout(cfg, _checked(path, reader), torch.device(device), dtype, interleave_mlp)
+
+
+def random_vunelix_tensors(cfg: VunelixConfig, device="cpu", dtype=torch.bfloat16, seed=0):
+    """Seeded ``get(name, shape)`` of a random Vunelix: fan-in scaled matrices, norms and skips near one, small biases, decays
+    between about 0.9 and 0.999 per step."""
+    g = _gen(torch.device(device), seed * 1000003)
+
+    def get(name, shape):
+        if name.endswith(".conv"):
+            return _randn(shape, g, device, torch.float32, std=shape[1] ** -0.5)
+        if name.endswith(".A_log"):
+            return _randn(shape, g, device, torch.float32, std=0.1)
+        if len(shape) == 2 and name != "loop.step":
+            return _randn(shape, g, device, dtype, std=STD if name == "embed" else shape[1] ** -0.5)
+        t = _randn(shape, g, device, torch.float32, std=0.1)
+        if name.endswith(".dt.b"):
+            return t - 4.0
+        return t if name == "loop.step" or name.endswith(".conv.b") else t + 1.0
+
+    return get
+
+
+def random_vunelix_weights(cfg: VunelixConfig, device="cpu", dtype=torch.bfloat16, seed=0, interleave_mlp=False) -> dict:
+    device = torch.device(device)
+    return _vunelix_layout(cfg, random_vunelix_tensors(cfg, device, dtype, seed), device, dtype, interleave_mlp)

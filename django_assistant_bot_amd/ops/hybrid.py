@@ -8,6 +8,7 @@ finished output [T, N] or its split-K slabs [S, T, N].
 """
 from __future__ import annotations
 
+import math
 from typing import NamedTuple
 
 import torch
@@ -51,13 +52,17 @@ def rms_embed(ids, table, gain, n: int, eps: float):
     return x, rms_residual(x, None, gain, n, eps, table.dtype, again=(ids, table), fresh=True)
 
 
-def rms_residual(x, y, gain, n: int, eps: float, dtype=torch.bfloat16, bias=None, pairs=None, again=None, fresh=False):
+def rms_residual(x, y, gain, n: int, eps: float, dtype=torch.bfloat16, bias=None, pairs=None, again=None, fresh=False,
+                 post=None, raw=False):
     """x += y (rows or slabs) + bias + the token's expert rows (``pairs`` [T * top, C]) + table[ids] (``again`` = (ids,
     table)), in place (fp32 [T, C]; ``fresh``: x starts at zero); returns x / rms(x) * gain as ``dtype`` (None without
-    ``gain``).  The mean square is over the first ``n`` columns; the padded ones are zero."""
+    ``gain``; ``raw``: x itself).  ``post``: y + bias + expert rows are divided by their root mean square and multiplied with
+    it before they are added.  The mean squares are over the first ``n`` columns; the padded ones are zero.  The table may
+    be fp32."""
     ids, table = again if again is not None else (None, None)
+    expect(not (raw and gain is not None), "raw: without a gain")
     if not x.is_cuda:
-        return ref.rms_residual(x, y, gain, n, eps, dtype, bias, pairs, ids, table)
+        return ref.rms_residual(x, y, gain, n, eps, dtype, bias, pairs, ids, table, post, raw, fresh)
     rows, cols = x.shape
     expect(x.dtype == torch.float32 and x.is_contiguous() and cols % 8 == 0 and 1 <= n <= cols and cols <= 16384,
            "the residual stream is contiguous fp32, width % 8")
@@ -66,7 +71,8 @@ def rms_residual(x, y, gain, n: int, eps: float, dtype=torch.bfloat16, bias=None
     if y is not None:
         py = _proj(y, rows, cols, "sublayer output")
         expect(py[4] % 8 == 0 and (dtype == torch.bfloat16 or py[1] == 1), "sublayer output rows")
-    _f32v(cols, gain, bias)
+    _f32v(cols, gain, bias, post)
+    expect(post is None or y is not None or pairs is not None, "post: of a sublayer's output")
     top = 0
     if pairs is not None:
         expect(pairs.dtype == dtype and pairs.is_contiguous() and pairs.shape[1] == cols and pairs.shape[0] % rows == 0,
@@ -74,11 +80,11 @@ def rms_residual(x, y, gain, n: int, eps: float, dtype=torch.bfloat16, bias=None
         top = pairs.shape[0] // rows
     if ids is not None:
         _i32(ids)
-        expect(ids.numel() == rows and table.dtype == dtype and table.is_contiguous() and table.shape[1] == cols, "embedding")
-    same_device(x, y, gain, bias, pairs, ids, table)
-    h = torch.empty((rows, cols), dtype=dtype, device=x.device) if gain is not None else None
+        expect(ids.numel() == rows and table.dtype in (dtype, torch.float32) and table.is_contiguous() and table.shape[1] == cols, "embedding")
+    same_device(x, y, gain, bias, pairs, ids, table, post)
+    h = torch.empty((rows, cols), dtype=dtype, device=x.device) if gain is not None or raw else None
     native().rms_residual(ptr(x), ptr(h), int(dtype == torch.float32), py, ptr(bias), ptr(pairs), top, ptr(ids),
-                          ptr(table), ptr(gain), int(n), float(eps), rows, cols, int(fresh), stream(x))
+                          ptr(table), int(table is not None and table.dtype == torch.float32), ptr(post), ptr(gain), int(n), float(eps), rows, cols, int(fresh), stream(x))
     return h
 
 
@@ -86,10 +92,21 @@ def rms_residual(x, y, gain, n: int, eps: float, dtype=torch.bfloat16, bias=None
 # attention in chunks, interleaved rotary positions
 
 
-def rope_turns(dims: int, base: float, device) -> torch.Tensor:
-    """fp64 turns per position of the ``dims / 2`` rotated pairs: base^(-2i / dims) / 2 pi."""
+def rope_turns(dims: int, base: float, device, scaling=None) -> torch.Tensor:
+    """fp64 turns per position of the ``dims / 2`` rotated pairs: base^(-2i / dims) / 2 pi.  ``scaling`` (``configs.Yarn``):
+    pairs that turn less than ``slow`` times in ``original`` positions are slowed down by ``factor``, those that turn more
+    than ``fast`` times are not, with a ramp over the pairs between."""
     i = torch.arange(dims // 2, dtype=torch.float64)
-    return (torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / max(dims, 1)) / (2 * torch.pi)).to(device)
+    turns = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / max(dims, 1)) / (2 * torch.pi)
+    if scaling is not None:
+        def pair(times):  # the (fractional) pair that turns so often
+            return dims * math.log(scaling.original / (2 * math.pi * times)) / (2 * math.log(base))
+
+        lo = max(math.floor(pair(scaling.fast)), 0)
+        hi = min(math.ceil(pair(scaling.slow)), dims - 1)
+        ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+        turns = turns / scaling.factor * ramp + turns * (1.0 - ramp)
+    return turns.to(device)
 
 
 def qk_rope_write(y, col0: int, H: int, G: int, D: int, dim: int, rot: int, turns, eps: float, norm: bool, positions,
@@ -261,6 +278,36 @@ def _check_state(d: RecurrentShape, z, T, A, dt_bias, skip, state, slot, ring=No
     return pz
 
 
+def _conv_args(y, col0: int, w, bias, ring, rows: int):
+    taps, C = w.shape
+    py = _proj(y, rows, col0 + C)
+    expect(w.dtype == torch.float32 and w.is_contiguous() and taps <= MAX_TAPS and C % 8 == 0 and col0 % 8 == 0
+           and py[4] % 8 == 0, "convolution: fp32 taps, channels in eights")
+    expect(ring.dtype in _ACT and ring.is_contiguous() and tuple(ring.shape[1:]) == (taps, C), "ring")
+    expect(ring.dtype == torch.bfloat16 or py[1] == 1, "fp32 activations take an fp32 projection")
+    if bias is not None:
+        _f32v(C, bias)
+    return py
+
+
+def short_conv_step(y, col0: int, w, bias, ring, slot, pos, row0: int, out):
+    """``short_conv`` of one decoded token per sequence: rows row0.. of the projection, into the same rows of ``out``."""
+    taps, C = w.shape
+    B, dtype = slot.numel(), ring.dtype
+    if not y.is_cuda:
+        c = ref.short_conv(y, col0, C, w, bias, ring, slot, pos, ref._spans(None, B, row0), dtype)
+        out[row0:row0 + B] = c[row0:row0 + B]
+        return out
+    py = _conv_args(y, col0, w, bias, ring, row0 + B)
+    _i32(slot), _i32(pos)
+    expect(pos.numel() >= row0 + B and out.is_contiguous() and out.shape[1] == C, "positions / output rows")
+    _rows(out, row0 + B, C, dtype)
+    same_device(y, w, bias, ring, slot, pos, out)
+    native().short_conv_step(py, int(col0), C, taps, ptr(w), ptr(bias), ptr(ring), ptr(slot), ptr(pos), int(row0), B, ptr(out),
+                             int(dtype == torch.float32), stream(y))
+    return out
+
+
 def short_conv(y, col0: int, w, bias, ring, slot, pos, cu, max_q: int):
     """Causal convolution (``w`` fp32 [taps, C], last tap = the token) and silu of the portions ``cu`` of columns
     col0.. of a projection; inputs before a portion come from ``ring`` [slots, taps, C], which is brought up to
@@ -269,15 +316,10 @@ def short_conv(y, col0: int, w, bias, ring, slot, pos, cu, max_q: int):
     T, dtype = pos.numel(), ring.dtype
     if not y.is_cuda:
         return ref.short_conv(y, col0, C, w, bias, ring, slot, pos, ref._spans(cu, 0, 0), dtype)
-    py = _proj(y, T, col0 + C)
+    py = _conv_args(y, col0, w, bias, ring, T)
     _i32(slot), _i32(pos), _i32(cu)
     n = cu.numel() - 1
-    expect(w.dtype == torch.float32 and w.is_contiguous() and taps <= MAX_TAPS and C % 8 == 0 and col0 % 8 == 0
-           and py[4] % 8 == 0, "convolution: fp32 taps, channels in eights")
-    expect(dtype in _ACT and ring.is_contiguous() and tuple(ring.shape[1:]) == (taps, C) and slot.numel() >= n, "ring")
-    expect(dtype == torch.bfloat16 or py[1] == 1, "fp32 activations take an fp32 projection")
-    if bias is not None:
-        _f32v(C, bias)
+    expect(slot.numel() >= n, "state slots")
     same_device(y, w, bias, ring, slot, pos, cu)
     out = torch.empty((T, C), dtype=dtype, device=y.device)
     native().short_conv(py, int(col0), C, taps, ptr(w), ptr(bias), ptr(ring), ptr(slot), ptr(pos), ptr(cu), n, int(max_q),
@@ -382,27 +424,31 @@ def gated_norm(y, gate, g_col: int, part: int, w, eps: float, out, row0: int, T:
 MAX_EXPERTS, MAX_TOP = 1024, 64
 
 
-def moe_route(z, col0: int, E: int, top: int, scale: float, T: int):
+def moe_route(z, col0: int, E: int, top: int, scale: float, T: int, scores: str = "softmax"):
     """fp32 router logits (columns col0..) -> (experts int32 [T, top], weights fp32 [T, top]): softmax over all experts,
-    the ``top`` largest, over their sum, times ``scale``."""
+    the ``top`` largest, over their sum, times ``scale``; ``scores`` "sigmoid": the ``top`` largest sigmoids as they are,
+    times ``scale``."""
+    expect(scores in ("softmax", "sigmoid"), "scores: softmax or sigmoid")
     if not z.is_cuda:
-        idx, wt = ref.moe_route(z, col0, E, top, scale)
+        idx, wt = ref.moe_route(z, col0, E, top, scale, scores)
         return idx[:T].int(), wt[:T]
     pz = _proj(z, T, col0 + E, "router logits")
     expect(pz[1] == 1 and 1 <= top <= min(E, MAX_TOP) and E <= MAX_EXPERTS, "router: fp32 logits, top <= experts")
     idx = torch.empty((T, top), dtype=torch.int32, device=z.device)
     wt = torch.empty((T, top), dtype=torch.float32, device=z.device)
-    native().moe_route(pz, int(col0), E, top, float(scale), ptr(idx), ptr(wt), T, stream(z))
+    native().moe_route(pz, int(col0), E, top, float(scale), int(scores == "sigmoid"), ptr(idx), ptr(wt), T, stream(z))
     return idx, wt
 
 
-def moe_experts(h, idx, wt, gate_up, down, E: int, group: int):
+def moe_experts(h, idx, wt, gate_up, down, E: int, group: int, weigh: str = "output"):
     """Each token's chosen experts: ``gate_up`` [E * 2F, K] and ``down`` [E * W, F] hold the experts one after the other
     (bf16 on the GPU: ``shuffle_weights`` copies with gate / up in 8-row groups; fp32: row-major, stacked).  -> [T * top,
-    W], row t * top + k = weight * expert output."""
+    W], row t * top + k = weight * expert output (``weigh`` "input": the expert of weight * h)."""
     T, top = idx.shape
+    expect(weigh in ("output", "input"), "weigh: output or input")
     if not h.is_cuda:
-        return ref.moe_experts(h, idx, wt, gate_up, down, E, group)
+        return ref.moe_experts(h, idx, wt, gate_up, down, E, group, weigh)
+    win = int(weigh == "input")
     K, F2, W = h.shape[1], gate_up.shape[0] // E, down.shape[0] // E
     P = T * top
     expect(h.stride(1) == 1 and h.dtype in _ACT and gate_up.dtype == h.dtype == down.dtype, "one type")
@@ -424,13 +470,13 @@ def moe_experts(h, idx, wt, gate_up, down, E: int, group: int):
         expect(K % 16 == 0 and (F2 // 2) % 16 == 0 and W % 4 == 0 and h.stride(0) % 4 == 0, "fp32 experts: K % 16, F % 16")
         gu = torch.empty((P, F2), dtype=h.dtype, device=dev)
         nat.gemm_f32_grouped(ptr(h), h.stride(0), ptr(gate_up), ptr(gu), F2, F2, K, ptr(perm), top, 0, ptr(tiles), n_tiles, s)
-        nat.glu_f32(ptr(act), F2 // 2, ptr(gu), P, F2 // 2, 0, 0, ptr(wt), ptr(perm), s)
+        nat.glu_f32(ptr(act), F2 // 2, ptr(gu), P, F2 // 2, 0, 0, ptr(wt), ptr(perm), win, s)
         nat.gemm_f32_grouped(ptr(act), F2 // 2, ptr(down), ptr(out), W, W, F2 // 2, ptr(perm), 0, 1, ptr(tiles), n_tiles, s)
         return out
     expect(group == 8 and K % 64 == 0 and F2 % 128 == 0 and W % 32 == 0 and h.stride(0) % 8 == 0, "experts: K % 64, F % 64, W % 32")
     nat.gemm_grouped(ptr(h), h.stride(0), ptr(gate_up), ptr(act), F2 // 2, F2, K, ptr(perm), top, 0, ptr(tiles), n_tiles, bm,
-                     1, ptr(wt), s)
-    nat.gemm_grouped(ptr(act), F2 // 2, ptr(down), ptr(out), W, W, F2 // 2, ptr(perm), 0, 1, ptr(tiles), n_tiles, bm, 0, 0, s)
+                     1, ptr(wt), win, s)
+    nat.gemm_grouped(ptr(act), F2 // 2, ptr(down), ptr(out), W, W, F2 // 2, ptr(perm), 0, 1, ptr(tiles), n_tiles, bm, 0, 0, 0, s)
     return out
 
 
@@ -447,4 +493,34 @@ def shared_glu(y, col0: int, n: int, z, sg_col: int, out):
     same_device(y, z, out)
     native().shared_glu(py, int(col0), int(n), pz, int(sg_col), ptr(out), out.stride(0), int(out.dtype == torch.float32), T,
                         stream(y))
+    return out
+
+
+# ----------------------------------------------------------------------------------------------
+# gates and caps
+
+
+def sigmoid_gate(y, col0: int, x):
+    """x [T, n] *= sigmoid(columns col0 .. col0 + n of a projection), in place."""
+    T, n = x.shape
+    if not x.is_cuda:
+        return x.copy_((x.float() * torch.sigmoid(ref.total(y)[:T, col0:col0 + n])).to(x.dtype))
+    py = _proj(y, T, col0 + n, "gate")
+    expect(x.dtype in _ACT and x.stride(1) == 1 and x.stride(0) % 8 == 0 and n % 8 == 0 and col0 % 8 == 0 and py[4] % 8 == 0,
+           "rows and columns in eights")
+    expect(x.dtype == torch.bfloat16 or py[1] == 1, "fp32 activations take an fp32 projection")
+    same_device(y, x)
+    native().sigmoid_gate(py, int(col0), ptr(x), x.stride(0), int(x.dtype == torch.float32), n, T, stream(x))
+    return x
+
+
+def softcap(y, cap: float):
+    """cap * tanh(y / cap), fp32, of logits [T, n] or their slabs."""
+    T, n = y.shape[-2:]
+    if not y.is_cuda:
+        return cap * torch.tanh(ref.total(y) / cap)
+    py = _proj(y, T, n, "logits")
+    expect(n % 8 == 0 and py[4] % 8 == 0 and cap > 0, "columns in eights, a positive cap")
+    out = torch.empty((T, n), dtype=torch.float32, device=y.device)
+    native().softcap(py, float(cap), ptr(out), n, T, stream(y))
     return out

@@ -15,8 +15,8 @@ from . import reference as ref
 from ._lib import expect, expect_bf16_contig, native, ptr, same_device, stream
 
 EPI_NONE, EPI_GELU, EPI_SWIGLU, EPI_SCORES = ref.EPI_NONE, ref.EPI_GELU, ref.EPI_SWIGLU, ref.EPI_SCORES
-EPI_SWIGLU8, EPI_GEGLU8 = ref.EPI_SWIGLU8, ref.EPI_GEGLU8
-GLU8 = (EPI_SWIGLU8, EPI_GEGLU8)  # gated epilogues over 8-row [gate | up] groups
+EPI_SWIGLU8, EPI_GEGLU8, EPI_REGLU8 = ref.EPI_SWIGLU8, ref.EPI_GEGLU8, ref.EPI_REGLU8
+GLU8 = (EPI_SWIGLU8, EPI_GEGLU8, EPI_REGLU8)  # gated epilogues over 8-row [gate | up] groups
 
 
 def _i32(t: torch.Tensor) -> None:
@@ -606,7 +606,7 @@ def _ref_stream_gemm(x, w, splits=1, epilogue=EPI_NONE, residual=None, norm_eps=
         if epilogue in (EPI_SWIGLU, *GLU8):
             grp = 16 if epilogue == EPI_SWIGLU else 8
             v = y.view(y.shape[0], -1, 2, grp)
-            act = F.gelu(v[:, :, 0], approximate="tanh") if epilogue == EPI_GEGLU8 else F.silu(v[:, :, 0])
+            act = ref.glu_act(v[:, :, 0], ref.epilogue_act(epilogue))
             y = (act * v[:, :, 1]).reshape(y.shape[0], -1)
         if splits > 1:
             return torch.cat([y[None], torch.zeros((splits - 1,) + tuple(y.shape))], 0)

@@ -74,14 +74,13 @@ def dyt_residual(x, y, post: DytNorm | None, ls, nxt: DytNorm | None, dtype=torc
     return h
 
 
-def glu_f32(x, gelu: bool = True, bias=None, out=None):
-    """fp32 [T, 2F] = [gate | up] (+ ``bias`` [gate | up]) -> act(gate) * up [T, F] (tanh-GELU, or SiLU)."""
+def glu_f32(x, act: str = "gelu", bias=None, out=None):
+    """fp32 [T, 2F] = [gate | up] (+ ``bias`` [gate | up]) -> act(gate) * up [T, F] (``act``: gelu (tanh), silu, relu)."""
     F2 = x.shape[-1]
     if not x.is_cuda:
         x = x if bias is None else x + bias
         g, u = x[..., :F2 // 2].float(), x[..., F2 // 2:].float()
-        act = torch.nn.functional.gelu(g, approximate="tanh") if gelu else torch.nn.functional.silu(g)
-        y = (act * u).to(x.dtype)
+        y = (ref.glu_act(g, act) * u).to(x.dtype)
         return y if out is None else out.copy_(y)
     expect(x.dtype == torch.float32 and x.is_contiguous() and F2 % 8 == 0, "contiguous fp32 [T, 2F], F % 4")
     if bias is not None:
@@ -89,7 +88,8 @@ def glu_f32(x, gelu: bool = True, bias=None, out=None):
     out = torch.empty((x.shape[0], F2 // 2), dtype=torch.float32, device=x.device) if out is None else out
     expect(out.dtype == torch.float32 and tuple(out.shape) == (x.shape[0], F2 // 2) and out.stride(1) == 1
            and out.stride(0) % 4 == 0, "bad glu output")
-    native().glu_f32(ptr(out), out.stride(0), ptr(x), x.shape[0], F2 // 2, int(gelu), ptr(bias), 0, 0, stream(x))
+    native().glu_f32(ptr(out), out.stride(0), ptr(x), x.shape[0], F2 // 2, ref.GLU_ACTS.index(act), ptr(bias), 0, 0, 0,
+                     stream(x))
     return out
 
 
@@ -111,13 +111,28 @@ def gemm_f32(a, b):
 # latent attention
 
 
-def latent_write(y, q_cols: int, gain, cache, slots, rank: int, eps: float):
-    """``y``: the [q | latent] projection, [T, q_cols (+ R)] or its split-K slabs [S, T, ...].  Writes the
+class LatentRope(NamedTuple):
+    """Rotary positions of ``latent_write``: the neighbours (2i, 2i + 1) of columns q_at .. q_at + dims of every D-wide query
+    head and of columns c_at .. c_at + dims of the latent row are a pair; ``turns`` fp64 [dims / 2] per position, ``gain`` on
+    cosine and sine."""
+
+    turns: torch.Tensor
+    gain: float
+    dims: int
+    D: int
+    q_at: int
+    c_at: int
+    positions: torch.Tensor  # int32 [T]
+
+
+def latent_write(y, q_cols: int, gain, cache, slots, rank: int, eps: float, rope: LatentRope | None = None):
+    """``y``: the [q | latent] projection, [T, q_cols (+ R ..)] or its split-K slabs [S, T, ...].  Writes the
     RMS-normed latents (statistic over ``rank`` <= R columns) into ``cache`` [blocks, block_size, R] at
     ``slots`` (int64, < 0 skipped) unless ``cache`` is None, and returns the q rows [T, q_cols] (a view of
-    ``y`` when there is nothing to sum)."""
+    ``y`` when there is nothing to sum or rotate).  ``rope``: rotates a part of every head and of the row, which then is
+    [latent | rotated key]."""
     if not y.is_cuda:
-        return ref.latent_write(y, q_cols, gain, cache, slots, rank, eps)
+        return ref.latent_write(y, q_cols, gain, cache, slots, rank, eps, rope)
     T, N = y.shape[-2:]
     slabs = y.dim() == 3
     expect(y.dtype in _ACT and y.is_contiguous() and N % 8 == 0 and q_cols % 8 == 0, "bad projection")
@@ -127,19 +142,29 @@ def latent_write(y, q_cols: int, gain, cache, slots, rank: int, eps: float):
     R = 0
     if cache is not None:
         R = cache.shape[-1]
-        expect(cache.is_contiguous() and cache.dtype in _ACT and N == q_cols + R and 1 <= rank <= R and R % 8 == 0,
+        expect(cache.is_contiguous() and cache.dtype in _ACT and N >= q_cols + R and 1 <= rank <= R and R % 8 == 0,
                "latent cache does not fit the projection")
         expect(cache.dtype == torch.bfloat16 or y.dtype == torch.float32, "an fp32 cache takes an fp32 projection")
         _f32(R, gain)
     else:
         expect(N == q_cols, "a projection without latents is q only")
+    ro = (0, 0, 0, 8, 0, 0, 1.0)
+    if rope is not None:
+        expect(cache is not None and rope.dims % 2 == 0 and rope.dims >= 2 and rope.D % 8 == rope.q_at % 8 == rope.c_at % 8 == 0
+               and rope.q_at + rope.dims <= rope.D and rank <= rope.c_at and rope.c_at + rope.dims <= R and q_cols % rope.D == 0,
+               "rotated columns")
+        expect(rope.turns.dtype == torch.float64 and rope.turns.numel() == rope.dims // 2, "turns: fp64 [dims / 2]")
+        _i32(rope.positions)
+        expect(rope.positions.numel() == T, "positions")
+        same_device(y, rope.turns, rope.positions)
+        ro = (ptr(rope.turns), ptr(rope.positions), rope.dims, rope.D, rope.q_at, rope.c_at, float(rope.gain))
     q = None
-    if slabs:
+    if slabs or rope is not None:
         dt = torch.bfloat16 if cache is None else cache.dtype
         q = torch.empty((T, q_cols), dtype=dt, device=y.device)
     native().latent_write(ptr(y), int(y.dtype == torch.float32), y.shape[0] if slabs else 1, T * N, N, ptr(q), q_cols,
                           ptr(gain), ptr(cache), int(cache is not None and cache.dtype == torch.float32), ptr(slots), T,
-                          R, int(rank), float(eps), stream(y))
+                          R, int(rank), float(eps), ro, stream(y))
     return y[:, :q_cols] if q is None else q
 
 

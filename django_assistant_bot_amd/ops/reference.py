@@ -14,6 +14,17 @@ import torch.nn.functional as F
 EPI_NONE, EPI_GELU, EPI_SWIGLU, EPI_SCORES = 0, 1, 2, 3
 EPI_SWIGLU8 = 4  # SwiGLU over 8-row [gate | up] groups (decode copies of whole-chip stream_gemm tilings)
 EPI_GEGLU8 = 6  # the same groups with a tanh-GELU gate
+EPI_REGLU8 = 7  # ... with a ReLU gate
+GLU_ACTS = ("silu", "gelu", "relu")  # gate activations, in the kernels' order
+
+
+def glu_act(x, act: str):
+    return F.gelu(x, approximate="tanh") if act == "gelu" else F.relu(x) if act == "relu" else F.silu(x)
+
+
+def epilogue_act(epilogue: int) -> str:
+    return {EPI_GEGLU8: "gelu", EPI_REGLU8: "relu"}.get(epilogue, "silu")
+
 
 
 def rmsnorm(x, w, eps, residual=None):
@@ -184,12 +195,12 @@ def gemm_bt(A, B, bias=None, residual=None, epilogue=EPI_NONE, out_f32=False, ro
         c = c + bias.float()
     if epilogue == EPI_GELU:
         c = F.gelu(c)
-    elif epilogue in (EPI_SWIGLU, EPI_SWIGLU8, EPI_GEGLU8):
+    elif epilogue in (EPI_SWIGLU, EPI_SWIGLU8, EPI_GEGLU8, EPI_REGLU8):
         N, hg = c.shape[1], 16 if epilogue == EPI_SWIGLU else 8
         c = c.view(c.shape[0], N // (2 * hg), 2, hg)
         if glu_bias is not None:  # [gate | up]
             c = c + glu_bias.float().view(2, N // (2 * hg), hg).transpose(0, 1)
-        act = F.gelu(c[:, :, 0], approximate="tanh") if epilogue == EPI_GEGLU8 else F.silu(c[:, :, 0])
+        act = glu_act(c[:, :, 0], epilogue_act(epilogue))
         c = (act * c[:, :, 1]).reshape(c.shape[0], N // 2)
     if residual is not None:
         # a bf16 output is the rounded projection plus the residual, rounded again (HF's
@@ -273,14 +284,28 @@ def dyt_residual(x, y, post, ls, nxt, dtype):
     return None if nxt is None else dyt(x, nxt).to(dtype)
 
 
-def latent_write(y, q_cols, gain, cache, slots, rank, eps):
+def latent_write(y, q_cols, gain, cache, slots, rank, eps, rope=None):
     y = y.float().sum(0).to(y.dtype) if y.dim() == 3 else y
+    q = y[:, :q_cols]
     if cache is not None:
-        c = y[:, q_cols:].float()
-        c = c * torch.rsqrt(c.pow(2).sum(-1, keepdim=True) / rank + eps) * gain
+        raw = y[:, q_cols:q_cols + cache.shape[-1]].float()
+        c = raw * torch.rsqrt(raw[:, :rank].pow(2).sum(-1, keepdim=True) / rank + eps) * gain
+        if rope is not None:
+            a = (rope.positions.double()[:, None] * rope.turns) * (2 * torch.pi)
+            cs, sn = a.cos().float() * rope.gain, a.sin().float() * rope.gain
+
+            def turn(x, at):  # columns at .. at + dims of the last dimension
+                u, v = x[..., at:at + rope.dims:2], x[..., at + 1:at + rope.dims:2]
+                c2, s2 = (t.view(t.shape[0], *(1,) * (x.dim() - 2), -1) for t in (cs, sn))
+                out = x.float().clone()
+                out[..., at:at + rope.dims:2], out[..., at + 1:at + rope.dims:2] = u * c2 - v * s2, v * c2 + u * s2
+                return out
+
+            c[:, rope.c_at:] = turn(raw, rope.c_at)[:, rope.c_at:]
+            q = turn(q.unflatten(1, (-1, rope.D)), rope.q_at).flatten(1).to(y.dtype)
         live = slots >= 0
         cache.view(-1, cache.shape[-1])[slots[live]] = c[live].to(cache.dtype)
-    return y[:, :q_cols]
+    return q
 
 
 def gather_latent(cache, block_table, start, end):

@@ -13,17 +13,23 @@ def total(y):
     return y.float().sum(0) if y.dim() == 3 else y.float()
 
 
-def rms_residual(x, y, gain, n, eps, dtype, bias, pairs, ids, table):
+def rms_residual(x, y, gain, n, eps, dtype, bias, pairs, ids, table, post=None, raw=False, fresh=False):
+    add = torch.zeros_like(x)
     if y is not None:
-        x += total(y)
+        add += total(y)
     if bias is not None:
-        x += bias
+        add += bias
     if pairs is not None:
-        x += pairs.float().view(x.shape[0], -1, x.shape[1]).sum(1)
+        add += pairs.float().view(x.shape[0], -1, x.shape[1]).sum(1)
+    if post is not None:
+        add = add * torch.rsqrt(add.pow(2).sum(-1, keepdim=True) / n + eps) * post
+    if fresh:
+        x.zero_()
+    x += add
     if ids is not None:
         x += table[ids.long()].float()
     if gain is None:
-        return None
+        return x.to(dtype, copy=True) if raw else None
     r = torch.rsqrt(x.pow(2).sum(-1, keepdim=True) / n + eps)
     return (x * r * gain).to(dtype)
 
@@ -133,13 +139,15 @@ def gated_norm(y, gate, g_col, part, gate_first, per_head, w, eps, scale):
     return v if gate_first else v * g
 
 
-def moe_route(z, col0, E, top, scale):
-    s = torch.softmax(total(z)[:, col0:col0 + E], -1)
-    v, idx = torch.topk(s, top, -1)
+def moe_route(z, col0, E, top, scale, scores="softmax"):
+    z = total(z)[:, col0:col0 + E]
+    v, idx = torch.topk(torch.sigmoid(z) if scores == "sigmoid" else torch.softmax(z, -1), top, -1)
+    if scores == "sigmoid":
+        return idx, v * scale
     return idx, v / (v.sum(-1, keepdim=True) + 1e-20) * scale
 
 
-def moe_experts(h, idx, wt, gate_up, down, E, group):
+def moe_experts(h, idx, wt, gate_up, down, E, group, weigh="output"):
     """-> [T * top, W]: each choice's weighted expert output."""
     T, top = idx.shape
     F2, W = gate_up.shape[0] // E, down.shape[0] // E
@@ -148,16 +156,34 @@ def moe_experts(h, idx, wt, gate_up, down, E, group):
         t, k = (idx == e).nonzero(as_tuple=True)
         if not t.numel():
             continue
+        f = wt[t, k][:, None]
         y = h[t].float() @ gate_up[e * F2:(e + 1) * F2].float().T
+        y, f = (y * f, 1.0) if weigh == "input" else (y, f)
         if group:
             y = y.view(-1, F2 // (2 * group), 2, group)
             act = (F.silu(y[:, :, 0]) * y[:, :, 1]).reshape(-1, F2 // 2)
         else:
             act = F.silu(y[:, :F2 // 2]) * y[:, F2 // 2:]
-        out[t, k] = (act * wt[t, k][:, None]).to(h.dtype).float() @ down[e * W:(e + 1) * W].float().T
+        out[t, k] = (act * f).to(h.dtype).float() @ down[e * W:(e + 1) * W].float().T
     return out.view(T * top, W).to(h.dtype)
 
 
 def shared_glu(y, col0, n, z, sg_col):
     y, z = total(y), total(z)
     return F.silu(y[:, col0:col0 + n]) * y[:, col0 + n:col0 + 2 * n] * torch.sigmoid(z[:, sg_col:sg_col + 1])
+
+
+def selective_scan(u, d, dt, low, y, A, dt_bias, skip, state, slot, pos, spans, dtype):
+    """-> [T, C] (rows outside ``spans`` are zero); ``dt`` [T, C]: the step's projection."""
+    dt = F.softplus(total(dt) + dt_bias)
+    low, z, x = total(low), total(y)[:, d.z_col:d.z_col + d.C], u.float()
+    B, Cn = low[:, d.b_col:d.b_col + d.Np], low[:, d.c_col:d.c_col + d.Np]
+    out = torch.zeros(x.shape[0], d.C)
+    for b, (a, e) in enumerate(spans):
+        s = int(slot[b])
+        S = state[s].clone() if int(pos[a]) else torch.zeros(d.C, d.Np)
+        for t in range(a, e):
+            S = torch.exp2(dt[t][:, None] * A) * S + (dt[t] * x[t])[:, None] * B[t]
+            out[t] = ((S @ Cn[t]) + skip * x[t]) * F.silu(z[t])
+        state[s] = S
+    return out.to(dtype)

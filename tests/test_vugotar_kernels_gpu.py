@@ -394,7 +394,7 @@ def test_biased_glu_epilogue(M, N, K, epi):
         close(got, want, 1.2e-2)
     xf, wf = x.float(), torch.cat([w.view(-1, 2, 8, K)[:, 0].reshape(-1, K), w.view(-1, 2, 8, K)[:, 1].reshape(-1, K)]).float()
     out = torch.zeros(M, N // 2 + 4, device=DEV)
-    ops.glu_f32(ops.gemm_f32(xf.to(DEV), wf.to(DEV)), epi == ops.EPI_GEGLU8, b.to(DEV), out[:, :N // 2])
+    ops.glu_f32(ops.gemm_f32(xf.to(DEV), wf.to(DEV)), "gelu" if epi == ops.EPI_GEGLU8 else "silu", b.to(DEV), out[:, :N // 2])
     close(out[:, :N // 2], ref.gemm_bt(x.float(), w.float(), epilogue=epi, glu_bias=b, out_f32=True), 1e-5)
 
 

@@ -78,8 +78,8 @@ def test_gemm_f32(M, N, K):
 
 def test_glu_f32():
     x = rnd(37, 2 * 200, dtype=torch.float32, scale=3)
-    for gelu in (True, False):
-        close(ops.glu_f32(x.to(DEV), gelu), ops.glu_f32(x, gelu), 2e-6)
+    for act in ("gelu", "silu", "relu"):
+        close(ops.glu_f32(x.to(DEV), act), ops.glu_f32(x, act), 2e-6)
 
 
 @pytest.mark.parametrize("M,N,K", [(1, 128, 128), (5, 2048, 512), (100, 768, 192), (130, 1024, 256), (300, 512, 512),
