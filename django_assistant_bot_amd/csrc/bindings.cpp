@@ -232,9 +232,9 @@ PYBIND11_MODULE(_native, m) {
                               VP(out), ST(s)),
           "selective_scan");
   });
-  m.def("selective_step", [proj, sel](u x, int act_f32, const SS& d, u dt_w, const P& low, const P& y, u A, u dt_bias, u skip,
-                                      u state, u slot, u pos, int row0, int B, u out, u s) {
-    check(dab::selective_step(CVP(x), act_f32, sel(d), CVP(dt_w), proj(low), proj(y), (const float*)A, (const float*)dt_bias,
+  m.def("selective_step", [proj, sel](u x, int act_f32, const SS& d, u dt_w, u low, const P& bc, const P& y, u A, u dt_bias,
+                                      u skip, u state, u slot, u pos, int row0, int B, u out, u s) {
+    check(dab::selective_step(CVP(x), act_f32, sel(d), CVP(dt_w), CVP(low), proj(bc), proj(y), (const float*)A, (const float*)dt_bias,
                               (const float*)skip, (float*)state, (const int*)slot, (const int*)pos, row0, B, VP(out), ST(s)),
           "selective_step");
   });
@@ -285,8 +285,8 @@ PYBIND11_MODULE(_native, m) {
   m.def("shared_glu", [proj](const P& y, int col0, int F, const P& z, int sg_col, u out, long ldo, int act_f32, int T, u s) {
     check(dab::shared_glu(proj(y), col0, F, proj(z), sg_col, VP(out), ldo, act_f32, T, ST(s)), "shared_glu");
   });
-  m.def("gemm_narrow", [](u A, long lda, u B, u C, int M, int N, int K, int S, u s) {
-    check(dab::gemm_narrow(CVP(A), lda, CVP(B), (float*)C, M, N, K, S, ST(s)), "gemm_narrow");
+  m.def("gemm_narrow", [](u A, long lda, u B, u C, int M, int N, int K, int S, int tall, u s) {
+    check(dab::gemm_narrow(CVP(A), lda, CVP(B), (float*)C, M, N, K, S, tall, ST(s)), "gemm_narrow");
   });
   m.def("gemm_grouped", [](u A, long lda, u B, u C, long ldc, int N, int K, u perm, int a_div, int scatter, u tiles,
                            int n_tiles, int bm, int glu, u row_scale, int scale_in, u s) {
@@ -324,7 +324,11 @@ PYBIND11_MODULE(_native, m) {
                         int K, u s) {
     check(dab::head_gemm(VP(y), y_tok, y_head, CVP(x), x_tok, x_head, CVP(w), row0, T, H, N, K, ST(s)), "head_gemm");
   });
+  m.def("latent_key_fill", [](u k, long k_tok, int D, u rows, int R, int q_at, int c_at, int rot, int H, int T, u s) {
+    check(dab::latent_key_fill(VP(k), k_tok, D, CVP(rows), R, q_at, c_at, rot, H, T, ST(s)), "latent_key_fill");
+  });
   m.def("latent_decode_ok", &dab::latent_decode_ok);
+  m.def("latent_decode_values", &dab::latent_decode_values);
   m.def("latent_decode_groups", &dab::latent_decode_groups);
   m.def("latent_decode", [](u q, u cache, u bt, int max_blocks, int bs, u ctx, u sink, u out, u po, u pml, int B,
                             int H, int R, int window, int parts, int min_part, float scale, u order, u s) {

@@ -390,7 +390,7 @@ int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc,
   }
 }
 
-int gemm_narrow(const void* A, long lda, const void* B, float* C, int M, int N, int K, int S, hipStream_t s) {
+int gemm_narrow(const void* A, long lda, const void* B, float* C, int M, int N, int K, int S, int tall, hipStream_t s) {
   if (M <= 0 || N <= 0) return 0;
   if (S < 1 || S > 64 || K % (64 * S) || N % 16 || lda % 8) return hipErrorInvalidValue;
   GemmParams p{};
@@ -406,8 +406,12 @@ int gemm_narrow(const void* A, long lda, const void* B, float* C, int M, int N, 
   p.out_f32 = 1;
   p.rows_b = N;
   p.bgrp = 1;
-  hipLaunchKernelGGL((gemm_bt_kernel<EPI_NONE, 32, 128, 1, 4, true>), dim3(((M + 31) / 32) * ((N + 127) / 128), S), dim3(256), 0,
-                     s, p);
+  if (tall)
+    hipLaunchKernelGGL((gemm_bt_kernel<EPI_NONE, 128, 128, 2, 2, true>), dim3(((M + 127) / 128) * ((N + 127) / 128), S), dim3(256),
+                       0, s, p);
+  else
+    hipLaunchKernelGGL((gemm_bt_kernel<EPI_NONE, 32, 128, 1, 4, true>), dim3(((M + 31) / 32) * ((N + 127) / 128), S), dim3(256), 0,
+                       s, p);
   return hipGetLastError();
 }
 

@@ -11,11 +11,12 @@
 // logit per head that joins the denominator and has neither key nor value.
 //
 // Rotary positions (optional): a rotated part of every query head and one rotated key part shared by the heads.  The
-// cached row then is [c | rotated key] and the expansions carry an identity block for the rotated columns, so both forms
-// stay what they are.
+// cached row then is [c | rotated key].  The absorbed query carries its rotated part along (an identity block in its
+// weights); the expanded keys do the same, or latent_key_fill copies the part to every head.
 //
 //   latent_write   : split-K slabs of the [q | latent] projection -> q rows, RMS norm, rotation, cache write
 //   latent_gather  : packed copy of the cached latents a prefill chunk sees (K / V expansion input)
+//   latent_key_fill: the gathered rotated key part into every expanded key head
 //   head_gemm      : Y[t, h, :] = W[h] X[t, h, :], weights in the ops.shuffle_weights layout
 //   latent_decode  : MFMA decode over key partitions, and the combine of the partitions
 //   latent_any     : one (token, head) per workgroup, any rank <= 2048, bf16 or fp32: the 32-bit mode
@@ -186,6 +187,31 @@ int latent_gather(void* out, const void* cache, const int* block_tables, int max
   return hipGetLastError();
 }
 
+// ------------------------------------------------------------------------------- latent_key_fill
+
+// K[i, h, q_at + j] = rows[i, c_at + j] for j < 8 units; one 16-B chunk a thread
+__global__ __launch_bounds__(256) void latent_key_fill_kernel(bf16* __restrict__ k, long k_tok, int D, const bf16* __restrict__ rows,
+                                                              int R, int q_at, int c_at, int units, int H, long total) {
+  const long e = (long)blockIdx.x * 256 + threadIdx.x;
+  if (e >= total) return;
+  const long i = e / (H * units);
+  const int r = (int)(e - i * H * units), h = r / units, u = r % units;
+  *reinterpret_cast<u32x4*>(k + i * k_tok + (long)h * D + q_at + 8 * u) =
+      *reinterpret_cast<const u32x4*>(rows + i * R + c_at + 8 * u);
+}
+
+int latent_key_fill(void* k, long k_tok, int D, const void* rows, int R, int q_at, int c_at, int rot, int H, int T, hipStream_t s) {
+  if (T <= 0) return 0;
+  const int units = (rot + 7) / 8;
+  if (rot < 1 || H < 1 || q_at % 8 || c_at % 8 || D % 8 || R % 8 || k_tok % 8 || q_at + 8 * units > D || c_at + 8 * units > R)
+    return hipErrorInvalidValue;
+  const long total = (long)T * H * units;
+  if (total > (1l << 38)) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(latent_key_fill_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, s, (bf16*)k, k_tok, D,
+                     (const bf16*)rows, R, q_at, c_at, units, H, total);
+  return hipGetLastError();
+}
+
 // -------------------------------------------------------------------------------------- head_gemm
 
 // Y[t, h, n] = sum_k X[t, h, k] W[row0 + h N + n, k]; W in the fragment layout [rows/16][K/32][64 lanes][8],
@@ -284,7 +310,8 @@ int head_gemm(void* y, long y_tok, long y_head, const void* x, long x_tok, long 
 //                   the fp32 scores go to LDS;
 //   softmax       : every wave redoes the (cheap) softmax of all HT head tiles from those scores, so its
 //                   probabilities are born in the B-operand layout and no maximum is exchanged;
-//   O^T += C^T P^T: wave w owns latent columns [w R/4, (w+1) R/4) of every head tile; C^T fragments by
+//   O^T += C^T P^T: wave w owns columns [w VR/4, (w+1) VR/4) of the latent part (the row without a rotated key, which has
+//                   no value) of every head tile; C^T fragments by
 //                   ds_read_b64_tr_b16 from the same tile.
 // One tile buffer per workgroup and two workgroups per CU: one streams while the other computes (a second
 // buffer per workgroup was no faster: a tile's math, not its copy, is the chain).  The
@@ -300,8 +327,8 @@ struct LatentDecodeParams {
   int max_blocks, block_size;
   const int* ctx_lens;
   const float* sink;  // [H], or null
-  bf16* out;          // [B, H, R]
-  float* part_o;      // [B, H, parts, R] un-normalised
+  bf16* out;          // [B, H, VR]
+  float* part_o;      // [B, H, parts, VR] un-normalised
   float* part_ml;     // [B, H, parts, 2] maximum (log2 domain), denominator
   const int* order;
   int H, groups, window, parts, min_part;
@@ -332,11 +359,11 @@ __device__ __forceinline__ int lat_off(int r, int c) {  // byte offset of 16-B c
   return r * R * 2 + 16 * (c ^ lat_swz<R>(r));
 }
 
-template <int R, int HT>
+template <int R, int VR, int HT>
 __global__ __launch_bounds__(256, 2) void latent_decode_kernel(LatentDecodeParams p) {
-  constexpr int KT = kLatTile, NKK = R / 32, NT = R / 64, CPR = R / 8;
+  constexpr int KT = kLatTile, NKK = R / 32, NT = VR / 64, CPR = R / 8;
   constexpr int NKG = 4 / HT, NS = 4 / NKG;        // waves per head tile, 16-key sub-tiles a wave scores
-  constexpr int SROW = KT + 4;                     // floats per head row of the score buffer
+  constexpr int SROW = KT;                         // floats per head row of the score buffer; 16-B chunk c of row r is at c ^ r % 16
   constexpr int TILE = KT * R * 2, PIECES = TILE / 4096;  // 1-KB DMA pieces per wave and tile
   __shared__ __attribute__((aligned(16))) char smem[TILE + 16 * HT * SROW * 4];
   float* sbuf = reinterpret_cast<float*>(smem + TILE);
@@ -434,18 +461,18 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(LatentDecodeParam
         const int key = k0 + 16 * sub + 4 * g + r;
         s0[r] = key >= sp.lo && key < k_end ? (s0[r] + s1[r]) * p.scale_log2 : -__builtin_huge_valf();
       }
-      *reinterpret_cast<f32x4*>(sbuf + (16 * ht + li) * SROW + 16 * sub + 4 * g) = s0;
+      *reinterpret_cast<f32x4*>(sbuf + (16 * ht + li) * SROW + 4 * ((4 * sub + g) ^ li)) = s0;
     }
     __syncthreads();
     bf16x8 pf[HT][2];
 #pragma unroll
     for (int i = 0; i < HT; ++i) {
-      const float* srow = sbuf + (16 * i + li) * SROW + 8 * g;
+      const float* srow = sbuf + (16 * i + li) * SROW;
       float e[16];
       float mx = -__builtin_huge_valf();
 #pragma unroll
       for (int j = 0; j < 4; ++j) {  // keys 32 (j / 2) + 8 g + 4 (j % 2) .. + 4
-        const f32x4 v = *reinterpret_cast<const f32x4*>(srow + 32 * (j >> 1) + 4 * (j & 1));
+        const f32x4 v = *reinterpret_cast<const f32x4*>(srow + 4 * ((8 * (j >> 1) + 2 * g + (j & 1)) ^ li));
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           e[4 * j + r] = v[r];
@@ -481,11 +508,11 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(LatentDecodeParam
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
         const char *pl, *ph;
-        if constexpr (R % 256 == 0) {  // (rows + 4 flip bit 3 of the chunk: the neighbouring 8-chunk group)
+        if constexpr (R % 256 == 0 && VR == R) {  // (rows + 4 flip bit 3 of the chunk: the neighbouring 8-chunk group)
           pl = smem + va[t & 3] + 32 * ks * R * 2 + 128 * (t >> 2);
           ph = smem + vb[t & 3] + 32 * ks * R * 2 + (R == 256 ? 0 : 128 * ((t >> 2) ^ 1));
         } else {
-          const int ch = w * (CPR / 4) + 2 * t + (pp >> 1), row = 32 * ks + 8 * g + qq;
+          const int ch = w * (VR / 32) + 2 * t + (pp >> 1), row = 32 * ks + 8 * g + qq;
           pl = smem + lat_off<R>(row, ch) + 8 * (pp & 1);
           ph = smem + lat_off<R>(row + 4, ch) + 8 * (pp & 1);
         }
@@ -506,10 +533,10 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(LatentDecodeParam
     L += __shfl_xor(L, 16, 64);
     L += __shfl_xor(L, 32, 64);
     if (h >= p.H) continue;
-    const int col = w * (R / 4) + 4 * g;
+    const int col = w * (VR / 4) + 4 * g;
     if (sp.np == 1) {
       const float inv = L > 0.f ? 1.f / L : 0.f;
-      bf16* orow = p.out + (hrow + h) * R + col;
+      bf16* orow = p.out + (hrow + h) * VR + col;
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
         u32x2 v;
@@ -520,7 +547,7 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(LatentDecodeParam
     } else {
       const size_t pi = (hrow + h) * p.parts + part;
 #pragma unroll
-      for (int t = 0; t < NT; ++t) *reinterpret_cast<f32x4*>(p.part_o + pi * R + col + 16 * t) = o[i][t];
+      for (int t = 0; t < NT; ++t) *reinterpret_cast<f32x4*>(p.part_o + pi * VR + col + 16 * t) = o[i][t];
       if (w == 0 && g == 0) {
         p.part_ml[2 * pi] = m_run[i];
         p.part_ml[2 * pi + 1] = L;
@@ -559,8 +586,11 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(LatentDecodeParams 
   *reinterpret_cast<u32x2*>(p.out + hrow * R + c) = v;
 }
 
-// Ranks (padded) the MFMA decode tiles.
-int latent_decode_ok(int R) { return R == 64 || R == 128 || R == 192 || R == 256 || R == 384 || R == 512; }
+// Rows (padded) the MFMA decode tiles, and the width of a row's latent part: 320 and 576 end with a rotated key.
+int latent_decode_ok(int R) {
+  return R == 64 || R == 128 || R == 192 || R == 256 || R == 320 || R == 384 || R == 512 || R == 576;
+}
+int latent_decode_values(int R) { return R == 320 ? 256 : R == 576 ? 512 : R; }
 
 // 16-head tiles of a workgroup: up to 64 heads share one staged latent tile (32 above R = 192: registers)
 static int decode_head_tiles(int H, int R) { return H <= 16 ? 1 : (H <= 32 || R > 192 ? 2 : 4); }
@@ -582,13 +612,14 @@ int latent_decode(const void* q, const void* cache, const int* block_tables, int
                        scale * 1.4426950408889634f};
   const int ht = decode_head_tiles(H, R);
   const dim3 grid(B * p.groups, parts);
-#define DAB_LD1(RR, HH) hipLaunchKernelGGL((latent_decode_kernel<RR, HH>), grid, dim3(256), 0, s, p)
-#define DAB_LD(RR)                                 \
-  case RR:                                         \
-    if (ht == 1) DAB_LD1(RR, 1);                   \
-    else if (ht == 2) DAB_LD1(RR, 2);              \
-    else if constexpr (RR <= 192) DAB_LD1(RR, 4);  \
+#define DAB_LD1(RR, VV, HH) hipLaunchKernelGGL((latent_decode_kernel<RR, VV, HH>), grid, dim3(256), 0, s, p)
+#define DAB_LDV(RR, VV)                                \
+  case RR:                                             \
+    if (ht == 1) DAB_LD1(RR, VV, 1);                   \
+    else if (ht == 2) DAB_LD1(RR, VV, 2);              \
+    else if constexpr (RR <= 192) DAB_LD1(RR, VV, 4);  \
     break;
+#define DAB_LD(RR) DAB_LDV(RR, RR)
   switch (R) {
     DAB_LD(64)
     DAB_LD(128)
@@ -596,12 +627,16 @@ int latent_decode(const void* q, const void* cache, const int* block_tables, int
     DAB_LD(256)
     DAB_LD(384)
     DAB_LD(512)
+    DAB_LDV(320, 256)
+    DAB_LDV(576, 512)
   }
 #undef DAB_LD
+#undef DAB_LDV
 #undef DAB_LD1
   const int err = hipGetLastError();
   if (err || parts == 1) return err;
-  hipLaunchKernelGGL(latent_combine_kernel, dim3(H, B), dim3(R <= 256 ? 64 : 128), 0, s, p, R);
+  const int VR = latent_decode_values(R);
+  hipLaunchKernelGGL(latent_combine_kernel, dim3(H, B), dim3(VR <= 256 ? 64 : 128), 0, s, p, VR);
   return hipGetLastError();
 }
 

@@ -121,8 +121,8 @@ int narrow_rows(Proj z, float* out, void* low, int N, int R, int T, hipStream_t 
 int selective_scan(const void* u, int act_f32, SelectiveShape d, Proj dt, Proj bc, Proj y, const float* A, const float* dt_bias,
                    const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, void* out,
                    hipStream_t s);
-int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, Proj low, Proj y, const float* A,
-                   const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos, int row0, int B,
+int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, const void* low, Proj bc, Proj y,
+                   const float* A, const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos, int row0, int B,
                    void* out, hipStream_t s);
 
 // moe.hip
@@ -164,7 +164,9 @@ int latent_gather(void* out, const void* cache, const int* block_tables, int max
                   const int* cu_k, const int* ctx, int B, int total, int row_bytes, hipStream_t s);
 int head_gemm(void* y, long y_tok, long y_head, const void* x, long x_tok, long x_head, const void* w, int row0, int T,
               int H, int N, int K, hipStream_t s);
+int latent_key_fill(void* k, long k_tok, int D, const void* rows, int R, int q_at, int c_at, int rot, int H, int T, hipStream_t s);
 int latent_decode_ok(int R);
+int latent_decode_values(int R);
 int latent_decode_groups(int H, int R);
 int latent_decode(const void* q, const void* cache, const int* block_tables, int max_blocks, int block_size,
                   const int* ctx_lens, const float* sink, void* out, float* part_o, float* part_ml, int B, int H, int R,
@@ -179,8 +181,9 @@ int latent_any(void* out, const void* q, const void* cache, int f32, const int* 
 int gemm_bt(const void* A, long lda, const void* B, long ldb, void* C, long ldc, const void* bias, const void* residual,
             long ldr, int M, int N, int K, int epilogue, int out_f32, const int* row_group, const int* q_group,
             const uint32_t* allow, int allow_words, hipStream_t s, int b_rows = 0, int b_group = 1);
-// a narrow fp32 product (router logits, recurrence gates) as S split-K slabs [S][M][N]: 32-row tiles, B a shuffle_weights copy
-int gemm_narrow(const void* A, long lda, const void* B, float* C, int M, int N, int K, int S, hipStream_t s);
+// a narrow fp32 product (router logits, recurrence gates) as S split-K slabs [S][M][N]: tiles of 32 or (tall) 128
+// rows, B a shuffle_weights copy
+int gemm_narrow(const void* A, long lda, const void* B, float* C, int M, int N, int K, int S, int tall, hipStream_t s);
 // experts: like gemm_f32_grouped, bf16, B = per-expert shuffle_weights copies of N rows; glu: SwiGLU over 8-row groups,
 // each row times row_scale[pair] (scale_in: gate and up times it, before the activation).  bm: rows of a tile (32, 128 or 256)
 int gemm_grouped(const void* A, long lda, const void* B, void* C, long ldc, int N, int K, const int* perm, int a_div,

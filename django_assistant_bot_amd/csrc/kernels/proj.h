@@ -127,7 +127,17 @@ __device__ __forceinline__ void sincos_turn(double r, float& sn, float& cs) {
   cs = (k == 1 || k == 2) ? -c1 : c1;
 }
 
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(__expf(z)); }
+// log(1 + e^z) = max(z, 0) + log1p(e), e = e^-|z|, with log1p(e) = 2 atanh(s), s = e / (2 + e) <= 1/3, by its power series:
+// fp32 rounding for any z, no branch
+__device__ __forceinline__ float softplus_f(float z) {
+  const float e = __expf(-fabsf(z)), s = e * __builtin_amdgcn_rcpf(2.f + e), q = s * s;
+  float p = fmaf(q, 1.f / 13.f, 1.f / 11.f);
+  p = fmaf(q, p, 1.f / 9.f);
+  p = fmaf(q, p, 1.f / 7.f);
+  p = fmaf(q, p, 1.f / 5.f);
+  p = fmaf(q, p, 1.f / 3.f);
+  return fmaxf(z, 0.f) + 2.f * fmaf(s * q, p, s);
+}
 
 // Type dispatch of kernels <projection type, activation type>: bf16 rows, fp32 slabs of a bf16 model, fp32 model.
 #define DAB_PROJ_DISPATCH(y, act_f32, CALL)   \

@@ -5,7 +5,7 @@
 //
 //   narrow_rows     slabs of that projection -> fp32 rows, and its first columns in bf16 (operand of W_dt)
 //   selective_scan  prompt portions: a workgroup walks one sequence for a block of channels, a tile of tokens at a time
-//   selective_step  one decoded token per sequence; W_dt low is formed in the kernel, its weights read once for SB sequences
+//   selective_step  one decoded token per sequence; W_dt low is formed in the kernel on MFMA, for up to 16 sequences at once
 //
 // A channel is shared by L neighbouring lanes, NS entries each, so a step's read-out is a sum over L lanes; four tokens'
 // sums are transposed across a quad, so each lane finishes one of them.  The state is stored [slot][channel][Np], Np = L NS
@@ -88,6 +88,7 @@ struct SelScan {
 template <typename PT, typename AT, int L, int NS, int TB>
 __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
   constexpr int CH = 256 / L, Np = L * NS, ITEMS = TB * CH / 8, BCV = TB * 2 * Np / 1024;
+  constexpr bool AHEAD = NS <= 4;  // (registers)
   static_assert(ITEMS <= 256 && BCV * 1024 == TB * 2 * Np && TB % 4 == 0, "tile");
   __shared__ __attribute__((aligned(16))) float2 dtx[TB][CH];    // (dt, dt u); then (y, -)
   __shared__ __attribute__((aligned(16))) float bc[TB][2 * Np];  // B | C
@@ -145,19 +146,43 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
     for (int k = 0; k < BCV; ++k) *reinterpret_cast<f32x4*>(&bc[0][0] + (k * 256 + tid) * 4) = nb[k];
     __syncthreads();
     if (t0 + TB < n) fetch(t0 + TB);
-#pragma unroll 1
-    for (int t = 0; t < TB; t += 4) {
-      float y[4];
+    // the values of the next four tokens are read under the current ones
+    float2 vn[4];
+    float bn[4][NS], cn[4][NS];
+    auto read4 = [&](int t) {
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
-        const float2 v = dtx[t + q][ch];
-        const float* br = &bc[t + q][part * NS];
-        const float* cr = &bc[t + q][Np + part * NS];
+        vn[q] = dtx[t + q][ch];
+#pragma unroll
+        for (int j = 0; j < NS; ++j) {
+          bn[q][j] = bc[t + q][part * NS + j];
+          cn[q][j] = bc[t + q][Np + part * NS + j];
+        }
+      }
+    };
+    if (AHEAD) read4(0);
+#pragma unroll 1
+    for (int t = 0; t < TB; t += 4) {
+      if (!AHEAD) read4(t);
+      float2 v[4];
+      float br[4][NS], cr[4][NS], y[4];
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        v[q] = vn[q];
+#pragma unroll
+        for (int j = 0; j < NS; ++j) {
+          br[q][j] = bn[q][j];
+          cr[q][j] = cn[q][j];
+        }
+      }
+      if (AHEAD) read4(min(t + 4, TB - 4));
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
         y[q] = 0.f;
 #pragma unroll
         for (int j = 0; j < NS; ++j) {
-          S[j] = fmaf(__builtin_amdgcn_exp2f(v.x * A[j]), S[j], v.y * br[j]);
-          y[q] = fmaf(S[j], cr[j], y[q]);
+          S[j] = fmaf(__builtin_amdgcn_exp2f(v[q].x * A[j]), S[j], v[q].y * br[q][j]);
+          y[q] = fmaf(S[j], cr[q][j], y[q]);
         }
       }
       const bool b0 = part & 1, b1 = part & 2;
@@ -229,7 +254,8 @@ struct SelStep {
   const void* u;        // [*, C]
   SelectiveShape d;
   const void* dt_w;     // [C, rank padded]: bf16 fragments (ops.shuffle_weights) or fp32 rows
-  Proj low;             // fp32 rows of the narrow projection: low | B | C
+  const void* low;      // [*, rank padded] low-rank steps: bf16, or fp32 with bc's row stride
+  Proj bc;              // fp32 rows of the narrow projection
   Proj y;
   const float* A;
   const float* bias;
@@ -241,121 +267,113 @@ struct SelStep {
   void* out;
 };
 
-constexpr int kMaxRank = 2048;
-
-// 64 channels (4 lanes each, NS state entries a lane) of SB sequences
-template <typename PT, typename AT, int NS, int SB>
+// 16 channels (4 lanes each, NS state entries a lane) of 4 SW sequences, SW a wave.  bf16: W_dt low of the 16 channels and
+// all the sequences is one MFMA tile (every wave forms it, no exchange but through its own LDS rows).
+template <typename PT, typename AT, int NS, int SW>
 __global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
   constexpr int Np = 4 * NS;
-  extern __shared__ __attribute__((aligned(16))) float sm[];  // low [SB][rank] | B, C [SB][2 Np] | dt [SB][64]
-  const int tid = threadIdx.x, ch = tid >> 2, part = tid & 3, c0 = blockIdx.x * 64, b0 = blockIdx.y * SB;
-  const int C = p.d.C, R = p.d.rank, c = min(c0 + ch, C - 1);
-  float* low = sm;
-  float* bc = sm + SB * R;
-  float* dts = bc + SB * 2 * Np;
-  float S[SB][NS], uv[SB], zv[SB];
-  float* sp[SB];
-  bool fresh[SB];
+  __shared__ float dts[4][SW][16];
+  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, g = lane >> 4, li = lane & 15;
+  const int c0 = blockIdx.x * 16, c = c0 + (lane >> 2), part = lane & 3;
+  const int C = p.d.C, R = p.d.rank, s0 = (blockIdx.y * 4 + w) * SW, sw0 = blockIdx.y * 4 * SW;
+  if (s0 >= p.B) return;  // the whole wave (no barrier follows)
+  float S[SW][NS], uv[SW], zv[SW], A[NS];
+  float* sp[SW];
+  bool fresh[SW];
+  int row[SW];
 #pragma unroll
-  for (int s = 0; s < SB; ++s) {
-    const int b = min(b0 + s, p.B - 1), row = p.row0 + b;
+  for (int s = 0; s < SW; ++s) {
+    const int b = min(s0 + s, p.B - 1);
+    row[s] = p.row0 + b;
     sp[s] = p.state + ((size_t)p.slot[b] * C + c) * Np + part * NS;
-    fresh[s] = p.pos[row] == 0;
+    fresh[s] = p.pos[row[s]] == 0;
 #pragma unroll
     for (int j = 0; j < NS; j += 4) {
       const f32x4 v = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(sp[s] + j));
 #pragma unroll
       for (int e = 0; e < 4; ++e) S[s][j + e] = v[e];
     }
-    uv[s] = ElemIO<AT>::load((const AT*)p.u + (size_t)row * C + c);
-    zv[s] = proj_f32<PT>(p.y, row, p.d.z_col + c);
+    uv[s] = ElemIO<AT>::load((const AT*)p.u + (size_t)row[s] * C + c);
+    zv[s] = proj_f32<PT>(p.y, row[s], p.d.z_col + c);
   }
-  for (int s = 0; s < SB; ++s) {
-    const float* src = (const float*)p.low.p + (long)(p.row0 + min(b0 + s, p.B - 1)) * p.low.ld;
-    for (int i = tid * 4; i < R; i += 1024)
-      *reinterpret_cast<f32x4*>(low + s * R + i) = *reinterpret_cast<const f32x4*>(src + i);
-    for (int i = tid * 4; i < 2 * Np; i += 1024)
-      *reinterpret_cast<f32x4*>(bc + s * 2 * Np + i) =
-          *reinterpret_cast<const f32x4*>(src + (i < Np ? p.d.b_col + i : p.d.c_col + i - Np));
+#pragma unroll
+  for (int j = 0; j < NS; j += 4) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(p.A + (size_t)c * Np + part * NS + j);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) A[j + e] = v[e];
   }
-  __syncthreads();
-  // W_dt low: a lane holds 8 of every 32 columns of channel li; the four lane groups are summed
-  const int w = tid >> 6, lane = tid & 63, g = lane >> 4, li = lane & 15, cw = c0 + 16 * w;
-  if (cw < C) {  // (C is a multiple of 16 here: whole blocks)
-    float acc[SB];
-#pragma unroll
-    for (int s = 0; s < SB; ++s) acc[s] = 0.f;
-#pragma unroll 4
-    for (int k = 0; k < R / 32; ++k) {
-      float wv[8];
-      if constexpr (sizeof(AT) == 2) ElemIO<bf16>::load8((const bf16*)p.dt_w + ((size_t)(cw / 16) * (R / 32) + k) * 512 + lane * 8, wv);
-      else ElemIO<float>::load8((const float*)p.dt_w + (size_t)(cw + li) * R + 32 * k + 8 * g, wv);
-#pragma unroll
-      for (int s = 0; s < SB; ++s) {
-        float lv[8];
-        ElemIO<float>::load8(low + s * R + 32 * k + 8 * g, lv);
-#pragma unroll
-        for (int j = 0; j < 8; ++j) acc[s] = fmaf(wv[j], lv[j], acc[s]);
-      }
-    }
-#pragma unroll
-    for (int s = 0; s < SB; ++s) {
-      acc[s] += __shfl_xor(acc[s], 16, 64);
-      acc[s] += __shfl_xor(acc[s], 32, 64);
-      if (g == 0) dts[s * 64 + 16 * w + li] = acc[s];
-    }
-  }
-  __syncthreads();
-  if (c0 + ch >= C) return;
   const float bias = p.bias[c], skip = p.skip[c];
-  float A[NS];
+  if constexpr (sizeof(AT) == 2) {
+    const bf16* wp = (const bf16*)p.dt_w + (size_t)blockIdx.x * (R / 32) * 512 + lane * 8;
+    const bf16* lp = (const bf16*)p.low + (size_t)(p.row0 + min(sw0 + li, p.B - 1)) * R + 8 * g;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k = 0; k < R / 32; ++k)
+      acc = mfma16(*reinterpret_cast<const bf16x8*>(wp + (size_t)k * 512), *reinterpret_cast<const bf16x8*>(lp + 32 * k), acc);
+    if (li / SW == w) {  // channel c0 + 4 g + r of sequence sw0 + li
 #pragma unroll
-  for (int j = 0; j < NS; ++j) A[j] = p.A[(size_t)c * Np + part * NS + j];
+      for (int r = 0; r < 4; ++r) dts[w][li % SW][4 * g + r] = acc[r];
+    }
+  } else {
+#pragma unroll 1
+    for (int s = 0; s < SW; ++s) {
+      const float* wp = (const float*)p.dt_w + (size_t)c * R;
+      const float* lp = (const float*)p.low + (size_t)(p.row0 + min(s0 + s, p.B - 1)) * p.bc.ld;
+      float a = 0.f;
+      for (int k = part * 4; k < R; k += 16)
 #pragma unroll
-  for (int s = 0; s < SB; ++s) {
-    if (b0 + s >= p.B) break;
-    const float dt = softplus_f(dts[s * 64 + ch] + bias), x = dt * uv[s];
-    const float* br = bc + s * 2 * Np + part * NS;
+        for (int e = 0; e < 4; ++e) a = fmaf(wp[k + e], lp[k + e], a);
+      a += quad_xor1(a);
+      a += quad_xor2(a);
+      if (part == 0) dts[w][s][lane >> 2] = a;
+    }
+  }
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+#pragma unroll
+  for (int s = 0; s < SW; ++s) {
+    if (s0 + s >= p.B) break;
+    const float dt = softplus_f(dts[w][s][lane >> 2] + bias), x = dt * uv[s];
+    const float* br = (const float*)p.bc.p + (size_t)row[s] * p.bc.ld + part * NS;
     float y = 0.f;
 #pragma unroll
-    for (int j = 0; j < NS; ++j) {
-      const float prev = fresh[s] ? 0.f : S[s][j];
-      S[s][j] = fmaf(__builtin_amdgcn_exp2f(dt * A[j]), prev, x * br[j]);
-      y = fmaf(S[s][j], br[Np + j], y);
-    }
+    for (int j = 0; j < NS; j += 4) {
+      const f32x4 bv = *reinterpret_cast<const f32x4*>(br + p.d.b_col + j);
+      const f32x4 cv = *reinterpret_cast<const f32x4*>(br + p.d.c_col + j);
+      f32x4 nv;
 #pragma unroll
-    for (int j = 0; j < NS; j += 4)
-      __builtin_nontemporal_store(f32x4{S[s][j], S[s][j + 1], S[s][j + 2], S[s][j + 3]}, reinterpret_cast<f32x4*>(sp[s] + j));
+      for (int e = 0; e < 4; ++e) {
+        const float prev = fresh[s] ? 0.f : S[s][j + e];
+        nv[e] = fmaf(__builtin_amdgcn_exp2f(dt * A[j + e]), prev, x * bv[e]);
+        y = fmaf(nv[e], cv[e], y);
+      }
+      __builtin_nontemporal_store(nv, reinterpret_cast<f32x4*>(sp[s] + j));
+    }
     y += quad_xor1(y);
     y += quad_xor2(y);
-    if (part == 0)
-      ElemIO<AT>::store((AT*)p.out + (size_t)(p.row0 + b0 + s) * C + c, fmaf(skip, uv[s], y) * silu_f(zv[s]));
+    if (part == 0) ElemIO<AT>::store((AT*)p.out + (size_t)row[s] * C + c, fmaf(skip, uv[s], y) * silu_f(zv[s]));
   }
 }
 
-int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, Proj low, Proj y, const float* A,
-                   const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos, int row0, int B,
-                   void* out, hipStream_t s) {
+int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, const void* low, Proj bc, Proj y,
+                   const float* A, const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos,
+                   int row0, int B, void* out, hipStream_t s) {
   if (B <= 0) return 0;
-  if (bad_shape(d, y) || d.C % 16 || d.rank < 32 || d.rank % 32 || d.rank > kMaxRank || !low.f32 || low.S != 1 || low.ld % 4 ||
-      B > 65535)
+  if (bad_shape(d, y) || d.C % 16 || d.rank < 32 || d.rank % 32 || !bc.f32 || bc.S != 1 || bc.ld % 4 || B > 65535)
     return hipErrorInvalidValue;
-  SelStep p{u, d, dt_w, low, y, A, dt_bias, skip, state, slot, pos, row0, B, out};
-  const int cb = (d.C + 63) / 64;
-  // several sequences a workgroup (one pass over W_dt) once there are workgroups enough
-  const int sb = d.Np <= 32 && d.rank <= 1024 && (long)cb * B >= 4096 ? 4 : 1;
-  const dim3 grid(cb, (B + sb - 1) / sb);
-  const size_t lds = (size_t)sb * (d.rank + 2 * d.Np + 64) * sizeof(float);
-#define STEP_L(PT, AT, NS, SB) hipLaunchKernelGGL((selective_step_kernel<PT, AT, NS, SB>), grid, dim3(256), lds, s, p)
+  SelStep p{u, d, dt_w, low, bc, y, A, dt_bias, skip, state, slot, pos, row0, B, out};
+#define STEP_L(PT, AT, NS, SW) \
+  hipLaunchKernelGGL((selective_step_kernel<PT, AT, NS, SW>), dim3(d.C / 16, (B + 4 * SW - 1) / (4 * SW)), dim3(256), 0, s, p)
 #define STEP_N(PT, AT)                          \
   do {                                          \
     switch (d.Np) {                             \
       case 16:                                  \
-        if (sb == 4) STEP_L(PT, AT, 4, 4);      \
+        if (B > 16) STEP_L(PT, AT, 4, 4);       \
         else STEP_L(PT, AT, 4, 1);              \
         break;                                  \
       case 32:                                  \
-        if (sb == 4) STEP_L(PT, AT, 8, 4);      \
+        if (B > 16) STEP_L(PT, AT, 8, 4);       \
         else STEP_L(PT, AT, 8, 1);              \
         break;                                  \
       case 48: STEP_L(PT, AT, 12, 1); break;    \

@@ -146,6 +146,10 @@ class LatentMixer:
         values = dict(ROTARY_TILES)
         return next((p for p in tiles if self.row_width <= p and self.rank <= values.get(p, p)), _up(self.row_width, 64))
 
+    def padded_latent(self) -> int:
+        """Columns of a cached row that values come from (all of them where latent and rotated key share a tile)."""
+        return dict(ROTARY_TILES).get(self.padded_row(), self.padded_row()) if self.rot else self.padded_row()
+
 
 @dataclass(frozen=True)
 class LatentLayer:

@@ -2,10 +2,11 @@
 
 Two exact forms of the same scores: prefill expands K and V of the visible context from the cached rows and runs the
 windowed flash kernel; decode folds W_uk into the query and W_uv behind the softmax, so each cached row is read once for
-all heads.  A rotated key part that the heads share is a part of the cached row; the expansions carry an identity block
-for it, so neither form knows of it.
+all heads.  A rotated key part that the heads share is a part of the cached row.  ``absorb_w`` carries an identity block
+for it; ``kv_w`` does too where it spans whole rows, and where it spans their latent part only the rotated part is copied
+to the expanded keys.
 
-A layer provides ``mixer`` (heads, scale, window), ``D`` (padded head width), ``R`` (padded row width), ``kv_w`` [K rows; V
+A layer provides ``mixer`` (``configs.LatentMixer``), ``D`` (padded head width), ``R`` (padded row width), ``kv_w`` [K rows; V
 rows], ``absorb_w`` (the K rows of every head transposed) and ``sink`` (or None).
 """
 from __future__ import annotations
@@ -74,16 +75,19 @@ class LatentAttention:
         qa = ops.head_gemm(q, L.absorb_w, L.R)
         parts, min_part = self._split(L, q.shape[0], meta.max_len) if meta.workspace is not None else (1, 128)
         oa = ops.latent_decode(qa, cache, block_tables, ctx_lens, m.scale, m.window, L.sink, parts, meta.workspace,
-                               meta.order, min_part)
-        return ops.head_gemm(oa, L.kv_w, L.D, row0=m.heads * L.D, out=out)
+                               meta.order, min_part, values=L.kv_w.shape[1])
+        return ops.head_gemm(oa[..., :L.kv_w.shape[1]], L.kv_w, L.D, row0=m.heads * L.D, out=out)
 
     def _latent_prefill(self, L, q, src: int, meta: AttnMeta, kv, plan, out=None):
         m, HD = L.mixer, L.mixer.heads * L.D
         if self.f32 or L.D not in FLASH_WINDOW_DIMS:
             oa = ops.latent_attention(ops.head_gemm(q, L.absorb_w, L.R), kv.c[src], meta.block_tables, meta.cu_q,
                                       meta.ctx_lens, m.scale, m.window, L.sink)
-            return ops.head_gemm(oa, L.kv_w, L.D, row0=HD, out=out)
+            return ops.head_gemm(oa[..., :L.kv_w.shape[1]], L.kv_w, L.D, row0=HD, out=out)
         cu_k, total = plan.context(m.window)
-        kvx = self._proj(plan.latents(src, m.window, kv), L.kv_w, False, name="kv").view(total, 2, m.heads, L.D)
+        rows, n = plan.latents(src, m.window, kv), L.kv_w.shape[1]
+        kvx = self._proj(rows[:, :n], L.kv_w, False, name="kv").view(total, 2, m.heads, L.D)
+        if n < L.R:
+            ops.latent_key_fill(kvx[:, 0], rows, m.q_at, m.c_at, m.rot.dims)
         return ops.flash_attention_window(q, kvx[:, 0], kvx[:, 1], meta.cu_q, cu_k, meta.max_q, m.scale, m.window,
                                           L.sink, out=out)

@@ -212,7 +212,7 @@ class VunelixModel(LatentAttention, HybridProjections):
             dt = self._aux(step[:Tp], L.dt_w, False, wide=True)
             ops.selective_scan(u, d, dt, low, y, L.A, L.dt_bias, L.skip, state, meta.state_slots, pos, meta.cu_q, out)
         if Tp < T:
-            ops.selective_step(u, d, L.dt_w, low, y, L.A, L.dt_bias, L.skip, state, slot, pos, Tp, out)
+            ops.selective_step(u, d, L.dt_w, step, low, y, L.A, L.dt_bias, L.skip, state, slot, pos, Tp, out)
         return self._proj(out, L.o_w, sk, name="o")
 
     def _attention(self, r: int, L: VunelixLayer, h, meta: AttnMeta, kv: HybridCache, plan, sk: bool):

@@ -542,8 +542,8 @@ def selective_layout(m: SelectiveMixer) -> SelectiveLayout:
 
 def _vunelix_layout(cfg: VunelixConfig, get, device, dtype, interleave_mlp) -> dict:
     """``get(name, shape)`` -> the engine's tensors.  Scan layers: ``in_w`` [x; z], ``x_w`` (step | input | read-out, the fp32
-    projection), ``dt_w``, ``o_w``; attention layers: ``in_w`` [q; latent | rotated key; output gate], ``kv_w`` (K rows with an
-    identity block for the rotated key, then V rows), ``absorb_w`` (the K rows of every head transposed), ``o_w``.  Sizes
+    projection), ``dt_w``, ``o_w``; attention layers: ``in_w`` [q; latent | rotated key; output gate], ``kv_w`` (K rows, with an
+    identity block for a rotated key among their columns, then V rows), ``absorb_w`` (the K rows of every head transposed), ``o_w``.  Sizes
     are padded with zeros; gains, biases, taps and recurrence constants are fp32, decays as -exp(A_log) log2(e)."""
     W, Wp = cfg.hidden, cfg.padded_hidden
 
@@ -591,6 +591,7 @@ def _vunelix_layout(cfg: VunelixConfig, get, device, dtype, interleave_mlp) -> d
             w[p + "o_w"] = _pad(mat(q + "o", W, m.inner), Wp, I)
         else:
             H, D, R, P = m.heads, m.padded_head(), m.padded_row(), m.rot.dims if m.rot else 0
+            V = m.padded_latent()
             full = mat(q + "q", H * (m.dim + P), W).view(H, m.dim + P, W)
             qw = embed.new_zeros((H, D, Wp))
             qw[:, :m.dim, :W] = full[:, :m.dim]
@@ -603,13 +604,13 @@ def _vunelix_layout(cfg: VunelixConfig, get, device, dtype, interleave_mlp) -> d
             if m.gate:
                 parts.append(heads(mat(q + "g", H * m.vdim, W), H, m.vdim, 0, D, Wp).reshape(H * D, Wp))
             fused = torch.cat(parts)
-            w[p + "in_w"] = _pad(fused, _up(fused.shape[0], 128), Wp)
+            w[p + "in_w"] = _pad(fused, _up(fused.shape[0], 256 if fused.shape[0] > 2048 else 128), Wp)
             w[p + "latent_norm"] = _pad(vec(q + "dkv.norm", m.rank), R)
             uk = heads(mat(q + "uk", H * m.dim, m.rank), H, m.dim, 0, D, R)
             for k in range(P):  # the rotated key part passes through
                 uk[:, m.q_at + k, m.c_at + k] = 1.0
-            uv = heads(mat(q + "uv", H * m.vdim, m.rank), H, m.vdim, 0, D, R)
-            w[p + "kv_w"] = torch.cat([uk.reshape(H * D, R), uv.reshape(H * D, R)])
+            uv = heads(mat(q + "uv", H * m.vdim, m.rank), H, m.vdim, 0, D, V)
+            w[p + "kv_w"] = torch.cat([uk[:, :, :V].reshape(H * D, V), uv.reshape(H * D, V)])
             w[p + "absorb_w"] = uk.transpose(1, 2).reshape(H * R, D).contiguous()
             w[p + "o_w"] = _pad(mat(q + "o", W, H * m.vdim).view(W, H, m.vdim), Wp, H, D).reshape(Wp, H * D)
         q = p + "mlp."

@@ -210,6 +210,23 @@ def head_gemm(x, w, n: int, row0: int = 0, out=None):
     return out
 
 
+def latent_key_fill(k, rows, q_at: int, c_at: int, dims: int):
+    """Copies the rotated key part, columns c_at .. c_at + dims of the gathered ``rows`` [T, R], to columns q_at.. of every
+    head of ``k`` [T, H, D] (heads adjacent), in place.  Columns up to the next multiple of 8 are copied along."""
+    T, H, D = k.shape
+    if not k.is_cuda:
+        k[:, :, q_at:q_at + dims] = rows[:, None, c_at:c_at + dims]
+        return k
+    R = rows.shape[1]
+    expect(k.dtype == rows.dtype == torch.bfloat16 and rows.is_contiguous() and rows.shape[0] == T and k.stride(2) == 1
+           and k.stride(1) == D and k.stride(0) % 8 == 0, "bf16 rows, adjacent heads")
+    expect(all(v % 8 == 0 for v in (D, R, q_at, c_at)) and dims >= 1 and q_at + -(-dims // 8) * 8 <= D
+           and c_at + -(-dims // 8) * 8 <= R, "rotated columns")
+    same_device(k, rows)
+    native().latent_key_fill(ptr(k), k.stride(0), D, ptr(rows), R, int(q_at), int(c_at), int(dims), H, T, stream(k))
+    return k
+
+
 FLASH_WINDOW_DIMS = (64, 128, 256)
 
 
@@ -259,14 +276,14 @@ class LatentWorkspace:
 
 
 def latent_decode(q, cache, block_tables, ctx_lens, scale: float, window: int = 0, sink=None, parts: int = 1,
-                  workspace: LatentWorkspace | None = None, order=None, min_part: int = 128):
-    """q [B, H, R] absorbed queries (one new token per sequence) over the paged latents -> [B, H, R].  Each
-    sequence's visible keys are split into up to ``parts`` partitions of >= ``min_part`` keys (``decode_split``)."""
+                  workspace: LatentWorkspace | None = None, order=None, min_part: int = 128, values: int | None = None):
+    """q [B, H, R] absorbed queries (one new token per sequence) over the paged latents -> [B, H, R], or
+    at least the first ``values`` columns of it (rows that end with a rotated key).  Each sequence's visible keys are split into up to ``parts`` partitions of >= ``min_part`` keys (``decode_split``)."""
     if not q.is_cuda:
         return ref.latent_attention(q, cache, block_tables, None, ctx_lens, scale, window, sink)
     B, H, R = q.shape
     bs = cache.shape[1]
-    if q.dtype == torch.float32 or not native().latent_decode_ok(R) or bs % 64:
+    if q.dtype == torch.float32 or not native().latent_decode_ok(R) or native().latent_decode_values(R) < (values or R) or bs % 64:
         return latent_attention(q, cache, block_tables, None, ctx_lens, scale, window, sink)
     _i32(block_tables)
     _i32(ctx_lens)
@@ -280,7 +297,7 @@ def latent_decode(q, cache, block_tables, ctx_lens, scale: float, window: int = 
         expect(order.numel() >= B, "decode order must hold the batch")
     expect(parts == 1 or (workspace is not None and workspace.o.numel() >= B * H * parts * R
                           and workspace.ml.numel() >= 2 * B * H * parts), "latent decode workspace too small")
-    out = torch.empty_like(q)
+    out = torch.empty((B, H, native().latent_decode_values(R)), dtype=q.dtype, device=q.device)
     ws = (ptr(workspace.o), ptr(workspace.ml)) if parts > 1 else (0, 0)
     native().latent_decode(ptr(q), ptr(cache), ptr(block_tables), block_tables.shape[1], bs, ptr(ctx_lens), ptr(sink),
                            ptr(out), *ws, B, H, R, int(window), int(parts), int(min_part), float(scale), ptr(order),

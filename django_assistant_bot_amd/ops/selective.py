@@ -86,18 +86,20 @@ def selective_scan(u, d: SelectiveShape, dt, low, y, A, dt_bias, skip, state, sl
     return out
 
 
-def selective_step(u, d: SelectiveShape, dt_w, low, y, A, dt_bias, skip, state, slot, pos, row0: int, out):
+def selective_step(u, d: SelectiveShape, dt_w, step, low, y, A, dt_bias, skip, state, slot, pos, row0: int, out):
     """The same for one decoded token per sequence, rows row0..; ``dt_w`` [C, rank] (bf16 on the GPU: a ``shuffle_weights``
-    copy) is applied to the first columns of ``low`` here."""
+    copy) is applied to ``step`` [*, rank] (``narrow_rows``) here."""
     B = slot.numel()
     if not u.is_cuda:
-        dt = low[:, :d.rank].float() @ dt_w.float().t()
+        dt = step.float() @ dt_w.float().t()
         c = ref.selective_scan(u, d, dt, low, y, A, dt_bias, skip, state, slot, pos, ref._spans(None, B, row0), out.dtype)
         out[row0:row0 + B] = c[row0:row0 + B]
         return out
     pl, py = _check(u, d, low, y, A, dt_bias, skip, state, slot, pos, out, row0 + B)
     expect(d.C % 16 == 0 and d.rank % 32 == 0 and d.rank <= MAX_STEP_RANK and dt_w.dtype == u.dtype and dt_w.is_contiguous()
            and tuple(dt_w.shape) == (d.C, d.rank), "step weights [C, rank]")
-    native().selective_step(ptr(u), int(u.dtype == torch.float32), tuple(d), ptr(dt_w), pl, py, ptr(A), ptr(dt_bias), ptr(skip),
+    expect(step.dtype == u.dtype and step.shape[0] >= row0 + B and step.shape[1] == d.rank and step.stride(1) == 1
+           and step.stride(0) == (d.rank if step.dtype == torch.bfloat16 else pl[4]), "low-rank steps")
+    native().selective_step(ptr(u), int(u.dtype == torch.float32), tuple(d), ptr(dt_w), ptr(step), pl, py, ptr(A), ptr(dt_bias), ptr(skip),
                             ptr(state), ptr(slot), ptr(pos), int(row0), B, ptr(out), stream(u))
     return out
