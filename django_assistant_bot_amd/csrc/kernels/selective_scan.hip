@@ -85,26 +85,32 @@ struct SelScan {
   void* out;            // [T, C]
 };
 
-template <typename PT, typename AT, int L, int NS, int TB>
+// A lane holds its NS entries of CPT channels, 256 / L apart, so that a token's B and C are read once for all of them.
+template <typename PT, typename AT, int L, int NS, int CPT, int TB>
 __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
-  constexpr int CH = 256 / L, Np = L * NS, ITEMS = TB * CH / 8, BCV = TB * 2 * Np / 1024;
-  constexpr bool AHEAD = NS <= 4;  // (registers)
-  static_assert(ITEMS <= 256 && BCV * 1024 == TB * 2 * Np && TB % 4 == 0, "tile");
-  __shared__ __attribute__((aligned(16))) float2 dtx[TB][CH];    // (dt, dt u); then (y, -)
+  constexpr int CG = 256 / L, CH = CG * CPT, Np = L * NS, ITEMS = TB * CH / 8, BCN = TB * 2 * Np / 4, BCV = (BCN + 255) / 256;
+  constexpr bool AHEAD = NS * CPT <= 4;  // (registers)
+  static_assert(ITEMS <= 256 && TB % 4 == 0, "tile");
+  __shared__ __attribute__((aligned(16))) float ds[TB][CH];      // dt; then y
+  __shared__ __attribute__((aligned(16))) float xs[TB][CH];      // dt u
   __shared__ __attribute__((aligned(16))) float bc[TB][2 * Np];  // B | C
   const int tid = threadIdx.x, ch = tid / L, part = tid % L, c0 = blockIdx.x * CH, b = blockIdx.y;
   const int r0 = p.cu[b], n = p.cu[b + 1] - r0;
   if (n <= 0) return;
-  const int C = p.d.C, c = min(c0 + ch, C - 1);
-  float S[NS], A[NS];
-  float* sp = p.state + ((size_t)p.slot[b] * C + c) * Np + part * NS;
-  const float* ap = p.A + (size_t)c * Np + part * NS;
+  const int C = p.d.C;
+  float S[CPT][NS], A[CPT][NS];
+  float* sp[CPT];
   const bool fresh = p.pos[r0] == 0;
 #pragma unroll
-  for (int j = 0; j < NS; ++j) {
-    const float v = sp[j];
-    S[j] = fresh ? 0.f : v;
-    A[j] = ap[j];
+  for (int i = 0; i < CPT; ++i) {
+    const size_t c = min(c0 + ch + i * CG, C - 1);
+    sp[i] = p.state + ((size_t)p.slot[b] * C + c) * Np + part * NS;
+#pragma unroll
+    for (int j = 0; j < NS; ++j) {
+      const float v = sp[i][j];
+      S[i][j] = fresh ? 0.f : v;
+      A[i][j] = p.A[c * Np + part * NS + j];
+    }
   }
   // this thread's 8 channels of one token of a tile (CH and C are multiples of 8)
   const int it = tid / (CH / 8), ic = (tid % (CH / 8)) * 8, cc = c0 + ic;
@@ -121,7 +127,7 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
     proj8<PT>(p.y, row, p.d.z_col + ccl, nz);
 #pragma unroll
     for (int k = 0; k < BCV; ++k) {
-      const int e = (k * 256 + tid) * 4, t = e / (2 * Np), j = e % (2 * Np);
+      const int e = min(k * 256 + tid, BCN - 1) * 4, t = e / (2 * Np), j = e % (2 * Np);
       const int col = j < Np ? p.d.b_col + j : p.d.c_col + j - Np;
       nb[k] = *reinterpret_cast<const f32x4*>((const float*)p.bc.p + (long)(r0 + min(t0 + t, n - 1)) * p.bc.ld + col);
     }
@@ -138,21 +144,27 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
     if (item) {
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
-        const float dt = live ? softplus_f(nd[j] + bias[j]) : 0.f;
-        dtx[it][ic + j] = make_float2(dt, dt * u[j]);
+        nd[j] = live ? softplus_f(nd[j] + bias[j]) : 0.f;
+        nu[j] = nd[j] * u[j];
       }
+      ElemIO<float>::store8(&ds[it][ic], nd);
+      ElemIO<float>::store8(&xs[it][ic], nu);
     }
 #pragma unroll
-    for (int k = 0; k < BCV; ++k) *reinterpret_cast<f32x4*>(&bc[0][0] + (k * 256 + tid) * 4) = nb[k];
+    for (int k = 0; k < BCV; ++k)
+      if (BCN % 256 == 0 || k * 256 + tid < BCN) *reinterpret_cast<f32x4*>(&bc[0][0] + (k * 256 + tid) * 4) = nb[k];
     __syncthreads();
     if (t0 + TB < n) fetch(t0 + TB);
     // the values of the next four tokens are read under the current ones
-    float2 vn[4];
-    float bn[4][NS], cn[4][NS];
+    float dn[4][CPT], xn[4][CPT], bn[4][NS], cn[4][NS];
     auto read4 = [&](int t) {
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
-        vn[q] = dtx[t + q][ch];
+#pragma unroll
+        for (int i = 0; i < CPT; ++i) {
+          dn[q][i] = ds[t + q][ch + i * CG];
+          xn[q][i] = xs[t + q][ch + i * CG];
+        }
 #pragma unroll
         for (int j = 0; j < NS; ++j) {
           bn[q][j] = bc[t + q][part * NS + j];
@@ -164,11 +176,14 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
 #pragma unroll 1
     for (int t = 0; t < TB; t += 4) {
       if (!AHEAD) read4(t);
-      float2 v[4];
-      float br[4][NS], cr[4][NS], y[4];
+      float dv[4][CPT], xv[4][CPT], br[4][NS], cr[4][NS], y[CPT][4];
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
-        v[q] = vn[q];
+#pragma unroll
+        for (int i = 0; i < CPT; ++i) {
+          dv[q][i] = dn[q][i];
+          xv[q][i] = xn[q][i];
+        }
 #pragma unroll
         for (int j = 0; j < NS; ++j) {
           br[q][j] = bn[q][j];
@@ -177,32 +192,40 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
       }
       if (AHEAD) read4(min(t + 4, TB - 4));
 #pragma unroll
-      for (int q = 0; q < 4; ++q) {
-        y[q] = 0.f;
+      for (int q = 0; q < 4; ++q)
 #pragma unroll
-        for (int j = 0; j < NS; ++j) {
-          S[j] = fmaf(__builtin_amdgcn_exp2f(v[q].x * A[j]), S[j], v[q].y * br[q][j]);
-          y[q] = fmaf(S[j], cr[q][j], y[q]);
+        for (int i = 0; i < CPT; ++i) {
+          y[i][q] = 0.f;
+#pragma unroll
+          for (int j = 0; j < NS; ++j) {
+            S[i][j] = fmaf(__builtin_amdgcn_exp2f(dv[q][i] * A[i][j]), S[i][j], xv[q][i] * br[q][j]);
+            y[i][q] = fmaf(S[i][j], cr[q][j], y[i][q]);
+          }
         }
-      }
       const bool b0 = part & 1, b1 = part & 2;
-      const float v0 = (b0 ? y[1] : y[0]) + quad_xor1(b0 ? y[0] : y[1]);
-      const float v1 = (b0 ? y[3] : y[2]) + quad_xor1(b0 ? y[2] : y[3]);
-      const float r = across_quads<L>((b1 ? v1 : v0) + quad_xor2(b1 ? v0 : v1));
-      if (part < 4) dtx[t + part][ch].x = r;
+#pragma unroll
+      for (int i = 0; i < CPT; ++i) {
+        const float v0 = (b0 ? y[i][1] : y[i][0]) + quad_xor1(b0 ? y[i][0] : y[i][1]);
+        const float v1 = (b0 ? y[i][3] : y[i][2]) + quad_xor1(b0 ? y[i][2] : y[i][3]);
+        const float r = across_quads<L>((b1 ? v1 : v0) + quad_xor2(b1 ? v0 : v1));
+        if (part < 4) ds[t + part][ch + i * CG] = r;
+      }
     }
     __syncthreads();
     if (live) {
       float o[8];
+      ElemIO<float>::load8(&ds[it][ic], o);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) o[j] = fmaf(skip[j], u[j], dtx[it][ic + j].x) * silu_f(z[j]);
+      for (int j = 0; j < 8; ++j) o[j] = fmaf(skip[j], u[j], o[j]) * silu_f(z[j]);
       ElemIO<AT>::store8((AT*)p.out + (size_t)(r0 + t0 + it) * C + cc, o);
     }
   }
-  if (c0 + ch < C) {
 #pragma unroll
-    for (int j = 0; j < NS; ++j) sp[j] = S[j];
-  }
+  for (int i = 0; i < CPT; ++i)
+    if (c0 + ch + i * CG < C) {
+#pragma unroll
+      for (int j = 0; j < NS; ++j) sp[i][j] = S[i][j];
+    }
 }
 
 static bool bad_shape(const SelectiveShape& d, const Proj& y) {
@@ -219,27 +242,28 @@ int selective_scan(const void* u, int act_f32, SelectiveShape d, Proj dt, Proj b
   SelScan p{u, d, dt, bc, y, A, dt_bias, skip, state, slot, pos, cu, out};
   // lanes per channel: more of them when the channels alone leave SIMDs without a wave
   const long waves = (long)chunks * d.C / 16;
-#define SEL_L(PT, AT, L, NS, TB)                                                                                   \
-  hipLaunchKernelGGL((selective_scan_kernel<PT, AT, L, NS, TB>), dim3((d.C + 256 / L - 1) / (256 / L), chunks),    \
-                     dim3(256), 0, s, p)
-#define SEL_N(PT, AT)                                     \
-  do {                                                    \
-    switch (d.Np) {                                       \
-      case 16:                                            \
-        if (waves >= 1024) SEL_L(PT, AT, 4, 4, 32);       \
-        else if (waves >= 256) SEL_L(PT, AT, 8, 2, 64);   \
-        else SEL_L(PT, AT, 16, 1, 64);                    \
-        break;                                            \
-      case 32:                                            \
-        if (waves >= 1024) SEL_L(PT, AT, 4, 8, 32);       \
-        else SEL_L(PT, AT, 16, 2, 64);                    \
-        break;                                            \
-      case 48: SEL_L(PT, AT, 4, 12, 32); break;           \
-      case 64: SEL_L(PT, AT, 8, 8, 32); break;            \
-      case 128: SEL_L(PT, AT, 16, 8, 32); break;          \
-      case 256: SEL_L(PT, AT, 16, 16, 16); break;         \
-      default: return hipErrorInvalidValue;               \
-    }                                                     \
+#define SEL_L(PT, AT, L, NS, CPT, TB)                                                                              \
+  hipLaunchKernelGGL((selective_scan_kernel<PT, AT, L, NS, CPT, TB>),                                              \
+                     dim3((d.C + 256 / L * CPT - 1) / (256 / L * CPT), chunks), dim3(256), 0, s, p)
+#define SEL_N(PT, AT)                                      \
+  do {                                                     \
+    switch (d.Np) {                                        \
+      case 16:                                             \
+        if (waves >= 4096) SEL_L(PT, AT, 4, 4, 2, 16);     \
+        else if (waves >= 1024) SEL_L(PT, AT, 4, 4, 1, 32); \
+        else if (waves >= 256) SEL_L(PT, AT, 8, 2, 1, 64); \
+        else SEL_L(PT, AT, 16, 1, 1, 64);                  \
+        break;                                             \
+      case 32:                                             \
+        if (waves >= 1024) SEL_L(PT, AT, 4, 8, 1, 32);     \
+        else SEL_L(PT, AT, 16, 2, 1, 64);                  \
+        break;                                             \
+      case 48: SEL_L(PT, AT, 4, 12, 1, 32); break;         \
+      case 64: SEL_L(PT, AT, 8, 8, 1, 32); break;          \
+      case 128: SEL_L(PT, AT, 16, 8, 1, 32); break;        \
+      case 256: SEL_L(PT, AT, 16, 16, 1, 16); break;       \
+      default: return hipErrorInvalidValue;                \
+    }                                                      \
   } while (0)
   DAB_PROJ_DISPATCH(y, act_f32, SEL_N);
 #undef SEL_N
@@ -278,6 +302,7 @@ __global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
   const int C = p.d.C, R = p.d.rank, s0 = (blockIdx.y * 4 + w) * SW, sw0 = blockIdx.y * 4 * SW;
   if (s0 >= p.B) return;  // the whole wave (no barrier follows)
   float S[SW][NS], uv[SW], zv[SW], A[NS];
+  f32x4 bv[SW][NS / 4], cv[SW][NS / 4];
   float* sp[SW];
   bool fresh[SW];
   int row[SW];
@@ -292,6 +317,12 @@ __global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
       const f32x4 v = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(sp[s] + j));
 #pragma unroll
       for (int e = 0; e < 4; ++e) S[s][j + e] = v[e];
+    }
+    const float* br = (const float*)p.bc.p + (size_t)row[s] * p.bc.ld + part * NS;
+#pragma unroll
+    for (int j = 0; j < NS / 4; ++j) {
+      bv[s][j] = *reinterpret_cast<const f32x4*>(br + p.d.b_col + 4 * j);
+      cv[s][j] = *reinterpret_cast<const f32x4*>(br + p.d.c_col + 4 * j);
     }
     uv[s] = ElemIO<AT>::load((const AT*)p.u + (size_t)row[s] * C + c);
     zv[s] = proj_f32<PT>(p.y, row[s], p.d.z_col + c);
@@ -335,18 +366,15 @@ __global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
   for (int s = 0; s < SW; ++s) {
     if (s0 + s >= p.B) break;
     const float dt = softplus_f(dts[w][s][lane >> 2] + bias), x = dt * uv[s];
-    const float* br = (const float*)p.bc.p + (size_t)row[s] * p.bc.ld + part * NS;
     float y = 0.f;
 #pragma unroll
     for (int j = 0; j < NS; j += 4) {
-      const f32x4 bv = *reinterpret_cast<const f32x4*>(br + p.d.b_col + j);
-      const f32x4 cv = *reinterpret_cast<const f32x4*>(br + p.d.c_col + j);
       f32x4 nv;
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const float prev = fresh[s] ? 0.f : S[s][j + e];
-        nv[e] = fmaf(__builtin_amdgcn_exp2f(dt * A[j + e]), prev, x * bv[e]);
-        y = fmaf(nv[e], cv[e], y);
+        nv[e] = fmaf(__builtin_amdgcn_exp2f(dt * A[j + e]), prev, x * bv[s][j / 4][e]);
+        y = fmaf(nv[e], cv[s][j / 4][e], y);
       }
       __builtin_nontemporal_store(nv, reinterpret_cast<f32x4*>(sp[s] + j));
     }
