@@ -291,65 +291,66 @@ struct SelStep {
   void* out;
 };
 
-// 16 channels (4 lanes each, NS state entries a lane) of 4 SW sequences, SW a wave.  bf16: W_dt low of the 16 channels and
-// all the sequences is one MFMA tile (every wave forms it, no exchange but through its own LDS rows).
-template <typename PT, typename AT, int NS, int SW>
+// What a wave needs of SW sequences for its 16 channels, requested at once
+template <int NS, int SW>
+struct StepRegs {
+  f32x4 S[SW][NS / 4];
+  float u[SW], z[SW];
+};
+
+// A wave: 16 channels (4 lanes each, NS state entries a lane).  WIDE: the four waves hold neighbouring channels and walk 16
+// sequences, SW at a time, the next ones requested under the current; else they hold the same channels, SW sequences each.
+// bf16: W_dt low of a wave's channels and up to 16 sequences is one MFMA tile.
+template <typename PT, typename AT, int NS, int SW, bool WIDE>
 __global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
-  constexpr int Np = 4 * NS;
-  __shared__ float dts[4][SW][16];
-  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, g = lane >> 4, li = lane & 15;
-  const int c0 = blockIdx.x * 16, c = c0 + (lane >> 2), part = lane & 3;
-  const int C = p.d.C, R = p.d.rank, s0 = (blockIdx.y * 4 + w) * SW, sw0 = blockIdx.y * 4 * SW;
-  if (s0 >= p.B) return;  // the whole wave (no barrier follows)
-  float S[SW][NS], uv[SW], zv[SW], A[NS];
-  f32x4 bv[SW][NS / 4], cv[SW][NS / 4];
-  float* sp[SW];
-  bool fresh[SW];
-  int row[SW];
+  constexpr int Np = 4 * NS, SEQS = WIDE ? 16 : SW;  // sequences of a wave
+  __shared__ float dts[4][SEQS][16];
+  __shared__ __attribute__((aligned(16))) float bcs[4][SEQS][2 * Np];  // B | C
+  const int tid = threadIdx.x, w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int lane = tid & 63, g = lane >> 4, li = lane & 15, part = lane & 3;
+  const int blk = WIDE ? blockIdx.x * 4 + w : blockIdx.x, c = blk * 16 + (lane >> 2);
+  const int C = p.d.C, R = p.d.rank, sw0 = blockIdx.y * (WIDE ? 16 : 4 * SW), s0 = WIDE ? sw0 : sw0 + w * SW;
+  if (s0 >= p.B || blk * 16 >= C) return;  // the whole wave (no barrier follows)
+  const int cell = c * Np + part * NS;  // of a slot's state
+  auto state = [&](int seq) { return p.state + (size_t)p.slot[seq] * C * Np + cell; };
+  auto request = [&](int at, StepRegs<NS, SW>& q) {
 #pragma unroll
-  for (int s = 0; s < SW; ++s) {
-    const int b = min(s0 + s, p.B - 1);
-    row[s] = p.row0 + b;
-    sp[s] = p.state + ((size_t)p.slot[b] * C + c) * Np + part * NS;
-    fresh[s] = p.pos[row[s]] == 0;
+    for (int s = 0; s < SW; ++s) {
+      const int b = min(at + s, p.B - 1);
+      const float* sp = state(b);
 #pragma unroll
-    for (int j = 0; j < NS; j += 4) {
-      const f32x4 v = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(sp[s] + j));
-#pragma unroll
-      for (int e = 0; e < 4; ++e) S[s][j + e] = v[e];
+      for (int j = 0; j < NS / 4; ++j) q.S[s][j] = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(sp + 4 * j));
+      q.u[s] = ElemIO<AT>::load((const AT*)p.u + (size_t)(p.row0 + b) * C + c);
+      q.z[s] = proj_f32<PT>(p.y, p.row0 + b, p.d.z_col + c);
     }
-    const float* br = (const float*)p.bc.p + (size_t)row[s] * p.bc.ld + part * NS;
-#pragma unroll
-    for (int j = 0; j < NS / 4; ++j) {
-      bv[s][j] = *reinterpret_cast<const f32x4*>(br + p.d.b_col + 4 * j);
-      cv[s][j] = *reinterpret_cast<const f32x4*>(br + p.d.c_col + 4 * j);
-    }
-    uv[s] = ElemIO<AT>::load((const AT*)p.u + (size_t)row[s] * C + c);
-    zv[s] = proj_f32<PT>(p.y, row[s], p.d.z_col + c);
+  };
+  StepRegs<NS, SW> q;
+  request(s0, q);
+  for (int i = lane * 4; i < SEQS * 2 * Np; i += 256) {
+    const int s = i / (2 * Np), j = i % (2 * Np);
+    const float* br = (const float*)p.bc.p + (size_t)(p.row0 + min(s0 + s, p.B - 1)) * p.bc.ld;
+    *reinterpret_cast<f32x4*>(&bcs[w][0][0] + i) = *reinterpret_cast<const f32x4*>(br + (j < Np ? p.d.b_col + j : p.d.c_col + j - Np));
   }
+  f32x4 A[NS / 4];
 #pragma unroll
-  for (int j = 0; j < NS; j += 4) {
-    const f32x4 v = *reinterpret_cast<const f32x4*>(p.A + (size_t)c * Np + part * NS + j);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) A[j + e] = v[e];
-  }
+  for (int j = 0; j < NS / 4; ++j) A[j] = *reinterpret_cast<const f32x4*>(p.A + (size_t)c * Np + part * NS + 4 * j);
   const float bias = p.bias[c], skip = p.skip[c];
   if constexpr (sizeof(AT) == 2) {
-    const bf16* wp = (const bf16*)p.dt_w + (size_t)blockIdx.x * (R / 32) * 512 + lane * 8;
+    const bf16* wp = (const bf16*)p.dt_w + (size_t)blk * (R / 32) * 512 + lane * 8;
     const bf16* lp = (const bf16*)p.low + (size_t)(p.row0 + min(sw0 + li, p.B - 1)) * R + 8 * g;
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
     for (int k = 0; k < R / 32; ++k)
       acc = mfma16(*reinterpret_cast<const bf16x8*>(wp + (size_t)k * 512), *reinterpret_cast<const bf16x8*>(lp + 32 * k), acc);
-    if (li / SW == w) {  // channel c0 + 4 g + r of sequence sw0 + li
+    if (WIDE || li / SW == w) {  // channel 4 g + r of sequence sw0 + li
 #pragma unroll
-      for (int r = 0; r < 4; ++r) dts[w][li % SW][4 * g + r] = acc[r];
+      for (int r = 0; r < 4; ++r) dts[w][li % SEQS][4 * g + r] = acc[r];
     }
   } else {
 #pragma unroll 1
-    for (int s = 0; s < SW; ++s) {
+    for (int s = 0; s < SEQS && s0 + s < p.B; ++s) {
       const float* wp = (const float*)p.dt_w + (size_t)c * R;
-      const float* lp = (const float*)p.low + (size_t)(p.row0 + min(s0 + s, p.B - 1)) * p.bc.ld;
+      const float* lp = (const float*)p.low + (size_t)(p.row0 + s0 + s) * p.bc.ld;
       float a = 0.f;
       for (int k = part * 4; k < R; k += 16)
 #pragma unroll
@@ -359,28 +360,40 @@ __global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
       if (part == 0) dts[w][s][lane >> 2] = a;
     }
   }
-  __builtin_amdgcn_wave_barrier();
+  // (a wave reads what it wrote itself)
   __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+#pragma unroll 1
+  for (int at = 0; at < SEQS; at += SW) {
+    if (s0 + at >= p.B) break;
+    StepRegs<NS, SW> cur = q;
+    if (WIDE && at + SW < SEQS && s0 + at + SW < p.B) request(s0 + at + SW, q);
 #pragma unroll
-  for (int s = 0; s < SW; ++s) {
-    if (s0 + s >= p.B) break;
-    const float dt = softplus_f(dts[w][s][lane >> 2] + bias), x = dt * uv[s];
-    float y = 0.f;
+    for (int s = 0; s < SW; ++s) {
+      const int b = s0 + at + s;
+      if (b >= p.B) break;
+      const float dt = softplus_f(dts[w][at + s][lane >> 2] + bias), x = dt * cur.u[s];
+      const float* bc = &bcs[w][at + s][part * NS];
+      const bool fresh = p.pos[p.row0 + b] == 0;
+      float* sp = state(b);
+      float y = 0.f;
 #pragma unroll
-    for (int j = 0; j < NS; j += 4) {
-      f32x4 nv;
+      for (int j = 0; j < NS / 4; ++j) {
+        const f32x4 bv = *reinterpret_cast<const f32x4*>(bc + 4 * j), cv = *reinterpret_cast<const f32x4*>(bc + Np + 4 * j);
+        f32x4 nv;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const float prev = fresh[s] ? 0.f : S[s][j + e];
-        nv[e] = fmaf(__builtin_amdgcn_exp2f(dt * A[j + e]), prev, x * bv[s][j / 4][e]);
-        y = fmaf(nv[e], cv[s][j / 4][e], y);
+        for (int e = 0; e < 4; ++e) {
+          const float prev = fresh ? 0.f : cur.S[s][j][e];
+          nv[e] = fmaf(__builtin_amdgcn_exp2f(dt * A[j][e]), prev, x * bv[e]);
+          y = fmaf(nv[e], cv[e], y);
+        }
+        __builtin_nontemporal_store(nv, reinterpret_cast<f32x4*>(sp + 4 * j));
       }
-      __builtin_nontemporal_store(nv, reinterpret_cast<f32x4*>(sp[s] + j));
+      y += quad_xor1(y);
+      y += quad_xor2(y);
+      if (part == 0) ElemIO<AT>::store((AT*)p.out + (size_t)(p.row0 + b) * C + c, fmaf(skip, cur.u[s], y) * silu_f(cur.z[s]));
     }
-    y += quad_xor1(y);
-    y += quad_xor2(y);
-    if (part == 0) ElemIO<AT>::store((AT*)p.out + (size_t)row[s] * C + c, fmaf(skip, uv[s], y) * silu_f(zv[s]));
   }
 }
 
@@ -391,25 +404,27 @@ int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_
   if (bad_shape(d, y) || d.C % 16 || d.rank < 32 || d.rank % 32 || !bc.f32 || bc.S != 1 || bc.ld % 4 || B > 65535)
     return hipErrorInvalidValue;
   SelStep p{u, d, dt_w, low, bc, y, A, dt_bias, skip, state, slot, pos, row0, B, out};
-#define STEP_L(PT, AT, NS, SW) \
-  hipLaunchKernelGGL((selective_step_kernel<PT, AT, NS, SW>), dim3(d.C / 16, (B + 4 * SW - 1) / (4 * SW)), dim3(256), 0, s, p)
-#define STEP_N(PT, AT)                          \
-  do {                                          \
-    switch (d.Np) {                             \
-      case 16:                                  \
-        if (B > 16) STEP_L(PT, AT, 4, 4);       \
-        else STEP_L(PT, AT, 4, 1);              \
-        break;                                  \
-      case 32:                                  \
-        if (B > 16) STEP_L(PT, AT, 8, 4);       \
-        else STEP_L(PT, AT, 8, 1);              \
-        break;                                  \
-      case 48: STEP_L(PT, AT, 12, 1); break;    \
-      case 64: STEP_L(PT, AT, 16, 1); break;    \
-      case 128: STEP_L(PT, AT, 32, 1); break;   \
-      case 256: STEP_L(PT, AT, 64, 1); break;   \
-      default: return hipErrorInvalidValue;     \
-    }                                           \
+  const bool wide = B > 16 && d.C % 64 == 0;
+#define STEP_L(PT, AT, NS, SW, WIDE)                                                                                   \
+  hipLaunchKernelGGL((selective_step_kernel<PT, AT, NS, SW, WIDE>),                                                    \
+                     WIDE ? dim3((d.C + 63) / 64, (B + 15) / 16) : dim3(d.C / 16, (B + 4 * SW - 1) / (4 * SW)), dim3(256), 0, s, p)
+#define STEP_N(PT, AT)                              \
+  do {                                              \
+    switch (d.Np) {                                 \
+      case 16:                                      \
+        if (wide) STEP_L(PT, AT, 4, 4, true);       \
+        else STEP_L(PT, AT, 4, 1, false);           \
+        break;                                      \
+      case 32:                                      \
+        if (wide) STEP_L(PT, AT, 8, 2, true);       \
+        else STEP_L(PT, AT, 8, 1, false);           \
+        break;                                      \
+      case 48: STEP_L(PT, AT, 12, 1, false); break; \
+      case 64: STEP_L(PT, AT, 16, 1, false); break; \
+      case 128: STEP_L(PT, AT, 32, 1, false); break; \
+      case 256: STEP_L(PT, AT, 64, 1, false); break; \
+      default: return hipErrorInvalidValue;         \
+    }                                               \
   } while (0)
   DAB_PROJ_DISPATCH(y, act_f32, STEP_N);
 #undef STEP_N
