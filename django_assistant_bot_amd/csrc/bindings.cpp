@@ -211,9 +211,9 @@ PYBIND11_MODULE(_native, m) {
           "short_conv");
   });
   m.def("short_conv_step", [proj](const P& y, int col0, int C, int taps, u w, u bias, u ring, u slot, u pos, int row0, int B,
-                                  u out, int act_f32, u s) {
+                                  u out, int z_col, u z_out, int act_f32, u s) {
     check(dab::short_conv_step(proj(y), col0, C, taps, (const float*)w, (const float*)bias, VP(ring), (const int*)slot,
-                               (const int*)pos, row0, B, VP(out), act_f32, ST(s)),
+                               (const int*)pos, row0, B, VP(out), z_col, VP(z_out), act_f32, ST(s)),
           "short_conv_step");
   });
   m.def("selective_state_width", &dab::selective_state_width);
@@ -232,9 +232,9 @@ PYBIND11_MODULE(_native, m) {
                               VP(out), ST(s)),
           "selective_scan");
   });
-  m.def("selective_step", [proj, sel](u x, int act_f32, const SS& d, u dt_w, u low, const P& bc, const P& y, u A, u dt_bias,
+  m.def("selective_step", [proj, sel](u x, int act_f32, const SS& d, u dt_w, u low, const P& bc, u A, u dt_bias,
                                       u skip, u state, u slot, u pos, int row0, int B, u out, u s) {
-    check(dab::selective_step(CVP(x), act_f32, sel(d), CVP(dt_w), CVP(low), proj(bc), proj(y), (const float*)A, (const float*)dt_bias,
+    check(dab::selective_step(CVP(x), act_f32, sel(d), CVP(dt_w), CVP(low), proj(bc), (const float*)A, (const float*)dt_bias,
                               (const float*)skip, (float*)state, (const int*)slot, (const int*)pos, row0, B, VP(out), ST(s)),
           "selective_step");
   });

@@ -90,9 +90,9 @@ struct RecurrentShape {
 int recurrent_state_width(int D);  // D padded as the state is stored
 int short_conv(Proj y, int col0, int C, int taps, const float* w, const float* bias, void* ring, const int* slot,
                const int* pos, const int* cu, int chunks, int max_q, void* out, int act_f32, hipStream_t s);
-// one decoded token per sequence, rows row0..
+// one decoded token per sequence, rows row0..; with z_out also the C columns z_col.. of the projection as finished rows
 int short_conv_step(Proj y, int col0, int C, int taps, const float* w, const float* bias, void* ring, const int* slot,
-                    const int* pos, int row0, int B, void* out, int act_f32, hipStream_t s);
+                    const int* pos, int row0, int B, void* out, int z_col, void* z_out, int act_f32, hipStream_t s);
 int state_scan(const void* conv, int act_f32, RecurrentShape d, Proj gates, const float* A, const float* dt_bias,
                const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, void* out,
                hipStream_t s);
@@ -121,8 +121,8 @@ int narrow_rows(Proj z, float* out, void* low, int N, int R, int T, hipStream_t 
 int selective_scan(const void* u, int act_f32, SelectiveShape d, Proj dt, Proj bc, Proj y, const float* A, const float* dt_bias,
                    const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, void* out,
                    hipStream_t s);
-int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, const void* low, Proj bc, Proj y,
-                   const float* A, const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos, int row0, int B,
+int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, const void* low, Proj bc, const float* A,
+                   const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos, int row0, int B,
                    void* out, hipStream_t s);
 
 // moe.hip

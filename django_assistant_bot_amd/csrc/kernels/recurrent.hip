@@ -157,7 +157,7 @@ int short_conv(Proj y, int col0, int C, int taps, const float* w, const float* b
 
 // one decoded token per sequence: 8 channels a thread
 template <typename PT, typename AT>
-__global__ __launch_bounds__(64) void conv_step_kernel(ConvParams p, int row0) {
+__global__ __launch_bounds__(64) void conv_step_kernel(ConvParams p, int row0, int z_col, AT* z_out) {
   const int b = blockIdx.y, c = (blockIdx.x * 64 + threadIdx.x) * 8, row = row0 + b;
   if (c >= p.C) return;
   const int pos = p.pos[row], now = pos % p.taps;
@@ -192,15 +192,19 @@ __global__ __launch_bounds__(64) void conv_step_kernel(ConvParams p, int row0) {
 #pragma unroll
   for (int j = 0; j < 8; ++j) o[j] = silu_f(o[j]);
   ElemIO<AT>::store8((AT*)p.out + (size_t)row * p.C + c, o);
+  if (z_out) {
+    proj8<PT>(p.y, row, z_col + c, o);
+    ElemIO<AT>::store8(z_out + (size_t)row * p.C + c, o);
+  }
 }
 
 int short_conv_step(Proj y, int col0, int C, int taps, const float* w, const float* bias, void* ring, const int* slot,
-                    const int* pos, int row0, int B, void* out, int act_f32, hipStream_t s) {
+                    const int* pos, int row0, int B, void* out, int z_col, void* z_out, int act_f32, hipStream_t s) {
   if (B <= 0) return 0;
-  if (C < 8 || C % 8 || col0 % 8 || y.ld % 8 || taps < 1 || taps > 16 || y.S < 1 || y.slab % 8 || B > 65535) return hipErrorInvalidValue;
+  if (C < 8 || C % 8 || col0 % 8 || z_col % 8 || y.ld % 8 || taps < 1 || taps > 16 || y.S < 1 || y.slab % 8 || B > 65535) return hipErrorInvalidValue;
   ConvParams p{y, col0, C, taps, w, bias, ring, slot, pos, nullptr, out, 0};
   const dim3 grid((C / 8 + 63) / 64, B);
-#define CSTEP_L(PT, AT) hipLaunchKernelGGL((conv_step_kernel<PT, AT>), grid, dim3(64), 0, s, p, row0)
+#define CSTEP_L(PT, AT) hipLaunchKernelGGL((conv_step_kernel<PT, AT>), grid, dim3(64), 0, s, p, row0, z_col, (AT*)z_out)
   DAB_PROJ_DISPATCH(y, act_f32, CSTEP_L);
 #undef CSTEP_L
   return hipGetLastError();

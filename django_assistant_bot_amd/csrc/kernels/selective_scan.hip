@@ -5,7 +5,7 @@
 //
 //   narrow_rows     slabs of that projection -> fp32 rows, and its first columns in bf16 (operand of W_dt)
 //   selective_scan  prompt portions: a workgroup walks one sequence for a block of channels, a tile of tokens at a time
-//   selective_step  one decoded token per sequence; W_dt low is formed in the kernel on MFMA, for up to 16 sequences at once
+//   selective_step  one decoded token per sequence, the gate's rows being replaced by the result; W_dt low is formed in the kernel on MFMA, for up to 16 sequences at once
 //
 // A channel is shared by L neighbouring lanes, NS entries each, so a step's read-out is a sum over L lanes; four tokens'
 // sums are transposed across a quad, so each lane finishes one of them.  The state is stored [slot][channel][Np], Np = L NS
@@ -228,16 +228,15 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
     }
 }
 
-static bool bad_shape(const SelectiveShape& d, const Proj& y) {
-  return d.C < 8 || d.C % 8 || d.Np != selective_state_width(d.Np) || d.rank < 0 || d.b_col % 4 || d.c_col % 4 || d.z_col % 8 ||
-         y.S < 1 || y.ld % 8 || y.slab % 8;
+static bool bad_shape(const SelectiveShape& d) {
+  return d.C < 8 || d.C % 8 || d.Np != selective_state_width(d.Np) || d.rank < 0 || d.b_col % 4 || d.c_col % 4 || d.z_col % 8;
 }
 
 int selective_scan(const void* u, int act_f32, SelectiveShape d, Proj dt, Proj bc, Proj y, const float* A, const float* dt_bias,
                    const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, void* out,
                    hipStream_t s) {
   if (chunks <= 0) return 0;
-  if (bad_shape(d, y) || !dt.f32 || dt.S != 1 || dt.ld % 4 || !bc.f32 || bc.S != 1 || bc.ld % 4 || chunks > 65535)
+  if (bad_shape(d) || y.S < 1 || y.ld % 8 || y.slab % 8 || !dt.f32 || dt.S != 1 || dt.ld % 4 || !bc.f32 || bc.S != 1 || bc.ld % 4 || chunks > 65535)
     return hipErrorInvalidValue;
   SelScan p{u, d, dt, bc, y, A, dt_bias, skip, state, slot, pos, cu, out};
   // lanes per channel: more of them when the channels alone leave SIMDs without a wave
@@ -280,7 +279,6 @@ struct SelStep {
   const void* dt_w;     // [C, rank padded]: bf16 fragments (ops.shuffle_weights) or fp32 rows
   const void* low;      // [*, rank padded] low-rank steps: bf16, or fp32 with bc's row stride
   Proj bc;              // fp32 rows of the narrow projection
-  Proj y;
   const float* A;
   const float* bias;
   const float* skip;
@@ -288,7 +286,7 @@ struct SelStep {
   const int* slot;
   const int* pos;
   int row0, B;
-  void* out;
+  void* out;            // [*, C]: the gate on entry
 };
 
 // What a wave needs of SW sequences for its 16 channels, requested at once
@@ -301,7 +299,7 @@ struct StepRegs {
 // A wave: 16 channels (4 lanes each, NS state entries a lane).  WIDE: the four waves hold neighbouring channels and walk 16
 // sequences, SW at a time, the next ones requested under the current; else they hold the same channels, SW sequences each.
 // bf16: W_dt low of a wave's channels and up to 16 sequences is one MFMA tile.
-template <typename PT, typename AT, int NS, int SW, bool WIDE>
+template <typename AT, int NS, int SW, bool WIDE>
 __global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
   constexpr int Np = 4 * NS, SEQS = WIDE ? 16 : SW;  // sequences of a wave
   __shared__ float dts[4][SEQS][16];
@@ -311,21 +309,23 @@ __global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
   const int blk = WIDE ? blockIdx.x * 4 + w : blockIdx.x, c = blk * 16 + (lane >> 2);
   const int C = p.d.C, R = p.d.rank, sw0 = blockIdx.y * (WIDE ? 16 : 4 * SW), s0 = WIDE ? sw0 : sw0 + w * SW;
   if (s0 >= p.B || blk * 16 >= C) return;  // the whole wave (no barrier follows)
+  // slots and positions of the wave's sequences, a lane each (read back as scalars); sequences past the last are the last
+  const int mine = min(s0 + min(li, SEQS - 1), p.B - 1), slots = p.slot[mine], places = p.pos[p.row0 + mine];
   const int cell = c * Np + part * NS;  // of a slot's state
-  auto state = [&](int seq) { return p.state + (size_t)p.slot[seq] * C * Np + cell; };
+  auto state = [&](int s) { return p.state + (size_t)__builtin_amdgcn_readlane(slots, s) * C * Np + cell; };
   auto request = [&](int at, StepRegs<NS, SW>& q) {
 #pragma unroll
     for (int s = 0; s < SW; ++s) {
-      const int b = min(at + s, p.B - 1);
-      const float* sp = state(b);
+      const float* sp = state(at + s);
+      const size_t cell = (size_t)(p.row0 + min(s0 + at + s, p.B - 1)) * C + c;
 #pragma unroll
       for (int j = 0; j < NS / 4; ++j) q.S[s][j] = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(sp + 4 * j));
-      q.u[s] = ElemIO<AT>::load((const AT*)p.u + (size_t)(p.row0 + b) * C + c);
-      q.z[s] = proj_f32<PT>(p.y, p.row0 + b, p.d.z_col + c);
+      q.u[s] = ElemIO<AT>::load((const AT*)p.u + cell);
+      q.z[s] = ElemIO<AT>::load((const AT*)p.out + cell);
     }
   };
   StepRegs<NS, SW> q;
-  request(s0, q);
+  request(0, q);
   for (int i = lane * 4; i < SEQS * 2 * Np; i += 256) {
     const int s = i / (2 * Np), j = i % (2 * Np);
     const float* br = (const float*)p.bc.p + (size_t)(p.row0 + min(s0 + s, p.B - 1)) * p.bc.ld;
@@ -368,15 +368,13 @@ __global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
   for (int at = 0; at < SEQS; at += SW) {
     if (s0 + at >= p.B) break;
     StepRegs<NS, SW> cur = q;
-    if (WIDE && at + SW < SEQS && s0 + at + SW < p.B) request(s0 + at + SW, q);
+    if (at + SW < SEQS) request(at + SW, q);
 #pragma unroll
     for (int s = 0; s < SW; ++s) {
-      const int b = s0 + at + s;
-      if (b >= p.B) break;
       const float dt = softplus_f(dts[w][at + s][lane >> 2] + bias), x = dt * cur.u[s];
       const float* bc = &bcs[w][at + s][part * NS];
-      const bool fresh = p.pos[p.row0 + b] == 0;
-      float* sp = state(b);
+      const bool fresh = __builtin_amdgcn_readlane(places, at + s) == 0, live = s0 + at + s < p.B;
+      float* sp = state(at + s);
       float y = 0.f;
 #pragma unroll
       for (int j = 0; j < NS / 4; ++j) {
@@ -388,45 +386,47 @@ __global__ __launch_bounds__(256) void selective_step_kernel(SelStep p) {
           nv[e] = fmaf(__builtin_amdgcn_exp2f(dt * A[j][e]), prev, x * bv[e]);
           y = fmaf(nv[e], cv[e], y);
         }
-        __builtin_nontemporal_store(nv, reinterpret_cast<f32x4*>(sp + 4 * j));
+        if (live) __builtin_nontemporal_store(nv, reinterpret_cast<f32x4*>(sp + 4 * j));
       }
       y += quad_xor1(y);
       y += quad_xor2(y);
-      if (part == 0) ElemIO<AT>::store((AT*)p.out + (size_t)(p.row0 + b) * C + c, fmaf(skip, cur.u[s], y) * silu_f(cur.z[s]));
+      if (live && part == 0)
+        ElemIO<AT>::store((AT*)p.out + (size_t)(p.row0 + s0 + at + s) * C + c, fmaf(skip, cur.u[s], y) * silu_f(cur.z[s]));
     }
   }
 }
 
-int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, const void* low, Proj bc, Proj y,
-                   const float* A, const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos,
+int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, const void* low, Proj bc, const float* A,
+                   const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos,
                    int row0, int B, void* out, hipStream_t s) {
   if (B <= 0) return 0;
-  if (bad_shape(d, y) || d.C % 16 || d.rank < 32 || d.rank % 32 || !bc.f32 || bc.S != 1 || bc.ld % 4 || B > 65535)
+  if (bad_shape(d) || d.C % 16 || d.rank < 32 || d.rank % 32 || !bc.f32 || bc.S != 1 || bc.ld % 4 || B > 65535)
     return hipErrorInvalidValue;
-  SelStep p{u, d, dt_w, low, bc, y, A, dt_bias, skip, state, slot, pos, row0, B, out};
+  SelStep p{u, d, dt_w, low, bc, A, dt_bias, skip, state, slot, pos, row0, B, out};
   const bool wide = B > 16 && d.C % 64 == 0;
-#define STEP_L(PT, AT, NS, SW, WIDE)                                                                                   \
-  hipLaunchKernelGGL((selective_step_kernel<PT, AT, NS, SW, WIDE>),                                                    \
+#define STEP_L(AT, NS, SW, WIDE)                                                                                   \
+  hipLaunchKernelGGL((selective_step_kernel<AT, NS, SW, WIDE>),                                                    \
                      WIDE ? dim3((d.C + 63) / 64, (B + 15) / 16) : dim3(d.C / 16, (B + 4 * SW - 1) / (4 * SW)), dim3(256), 0, s, p)
-#define STEP_N(PT, AT)                              \
+#define STEP_N(AT)                              \
   do {                                              \
     switch (d.Np) {                                 \
       case 16:                                      \
-        if (wide) STEP_L(PT, AT, 4, 4, true);       \
-        else STEP_L(PT, AT, 4, 1, false);           \
+        if (wide) STEP_L(AT, 4, 4, true);       \
+        else STEP_L(AT, 4, 1, false);           \
         break;                                      \
       case 32:                                      \
-        if (wide) STEP_L(PT, AT, 8, 2, true);       \
-        else STEP_L(PT, AT, 8, 1, false);           \
+        if (wide) STEP_L(AT, 8, 2, true);       \
+        else STEP_L(AT, 8, 1, false);           \
         break;                                      \
-      case 48: STEP_L(PT, AT, 12, 1, false); break; \
-      case 64: STEP_L(PT, AT, 16, 1, false); break; \
-      case 128: STEP_L(PT, AT, 32, 1, false); break; \
-      case 256: STEP_L(PT, AT, 64, 1, false); break; \
+      case 48: STEP_L(AT, 12, 1, false); break; \
+      case 64: STEP_L(AT, 16, 1, false); break; \
+      case 128: STEP_L(AT, 32, 1, false); break; \
+      case 256: STEP_L(AT, 64, 1, false); break; \
       default: return hipErrorInvalidValue;         \
     }                                               \
   } while (0)
-  DAB_PROJ_DISPATCH(y, act_f32, STEP_N);
+  if (act_f32) STEP_N(float);
+  else STEP_N(bf16);
 #undef STEP_N
 #undef STEP_L
   return hipGetLastError();

@@ -204,15 +204,15 @@ class VunelixModel(LatentAttention, HybridProjections):
             u = ops.short_conv(y, 0, L.conv_w, L.conv_b, ring, meta.state_slots, pos, meta.cu_q, meta.max_q)
         else:
             u = torch.empty((T, d.C), dtype=self.dtype, device=h.device)
-        if Tp < T:
-            ops.short_conv_step(y, 0, L.conv_w, L.conv_b, ring, slot, pos, Tp, u)
-        low, step = ops.narrow_rows(self._aux(u, L.x_w, sk), L.narrow, d.rank, T, self.dtype)
         out = torch.empty_like(u)
+        if Tp < T:  # the gate's rows wait in ``out``
+            ops.short_conv_step(y, 0, L.conv_w, L.conv_b, ring, slot, pos, Tp, u, d.z_col, out)
+        low, step = ops.narrow_rows(self._aux(u, L.x_w, sk), L.narrow, d.rank, T, self.dtype)
         if Tp:
             dt = self._aux(step[:Tp], L.dt_w, False, wide=True)
             ops.selective_scan(u, d, dt, low, y, L.A, L.dt_bias, L.skip, state, meta.state_slots, pos, meta.cu_q, out)
         if Tp < T:
-            ops.selective_step(u, d, L.dt_w, step, low, y, L.A, L.dt_bias, L.skip, state, slot, pos, Tp, out)
+            ops.selective_step(u, d, L.dt_w, step, low, L.A, L.dt_bias, L.skip, state, slot, pos, Tp, out)
         return self._proj(out, L.o_w, sk, name="o")
 
     def _attention(self, r: int, L: VunelixLayer, h, meta: AttnMeta, kv: HybridCache, plan, sk: bool):

@@ -291,21 +291,28 @@ def _conv_args(y, col0: int, w, bias, ring, rows: int):
     return py
 
 
-def short_conv_step(y, col0: int, w, bias, ring, slot, pos, row0: int, out):
-    """``short_conv`` of one decoded token per sequence: rows row0.. of the projection, into the same rows of ``out``."""
+def short_conv_step(y, col0: int, w, bias, ring, slot, pos, row0: int, out, z_col: int = 0, z_out=None):
+    """``short_conv`` of one decoded token per sequence: rows row0.. of the projection, into the same rows of ``out``.  With
+    ``z_out`` also the columns z_col .. z_col + C (a gate) as finished rows."""
     taps, C = w.shape
     B, dtype = slot.numel(), ring.dtype
     if not y.is_cuda:
         c = ref.short_conv(y, col0, C, w, bias, ring, slot, pos, ref._spans(None, B, row0), dtype)
         out[row0:row0 + B] = c[row0:row0 + B]
+        if z_out is not None:
+            z_out[row0:row0 + B] = ref.total(y)[row0:row0 + B, z_col:z_col + C].to(dtype)
         return out
     py = _conv_args(y, col0, w, bias, ring, row0 + B)
+    if z_out is not None:
+        _proj(y, row0 + B, z_col + C, "gate")
+        expect(z_col % 8 == 0 and z_out.is_contiguous() and z_out.shape[1] == C, "gate columns / rows")
+        _rows(z_out, row0 + B, C, dtype)
     _i32(slot), _i32(pos)
     expect(pos.numel() >= row0 + B and out.is_contiguous() and out.shape[1] == C, "positions / output rows")
     _rows(out, row0 + B, C, dtype)
     same_device(y, w, bias, ring, slot, pos, out)
     native().short_conv_step(py, int(col0), C, taps, ptr(w), ptr(bias), ptr(ring), ptr(slot), ptr(pos), int(row0), B, ptr(out),
-                             int(dtype == torch.float32), stream(y))
+                             int(z_col), ptr(z_out), int(dtype == torch.float32), stream(y))
     return out
 
 

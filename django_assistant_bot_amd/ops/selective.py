@@ -49,7 +49,7 @@ def narrow_rows(z, n: int, low: int, T: int, dtype=torch.bfloat16):
     return out, lo
 
 
-def _check(u, d: SelectiveShape, low, y, A, dt_bias, skip, state, slot, pos, out, rows: int):
+def _check(u, d: SelectiveShape, low, A, dt_bias, skip, state, slot, pos, out, rows: int):
     expect(u.dtype in _ACT and u.is_contiguous() and u.shape[0] >= rows and u.shape[1] == d.C and d.C % 8 == 0, "channels")
     expect(d.Np == state_width(d.Np) and d.Np <= MAX_STATE and d.b_col % 4 == d.c_col % 4 == d.z_col % 8 == 0, "selective sizes")
     expect(state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (d.C, d.Np), "state slots")
@@ -58,12 +58,10 @@ def _check(u, d: SelectiveShape, low, y, A, dt_bias, skip, state, slot, pos, out
     _i32(slot), _i32(pos)
     pl = _proj(low, rows, max(d.rank, d.b_col + d.Np, d.c_col + d.Np), "narrow projection")
     expect(pl[1] == 1 and pl[2] == 1 and pl[4] % 4 == 0, "finished fp32 rows")
-    py = _proj(y, rows, d.z_col + d.C, "gate")
-    expect(py[4] % 8 == 0 and (u.dtype == torch.bfloat16 or py[1] == 1), "gate rows")
     expect(pos.numel() >= rows and out.is_contiguous() and out.shape[1] == d.C, "positions / output rows")
     _rows(out, rows, d.C, u.dtype)
-    same_device(u, low, y, A, dt_bias, skip, state, slot, pos, out)
-    return pl, py
+    same_device(u, low, A, dt_bias, skip, state, slot, pos, out)
+    return pl
 
 
 def selective_scan(u, d: SelectiveShape, dt, low, y, A, dt_bias, skip, state, slot, pos, cu, out):
@@ -77,7 +75,10 @@ def selective_scan(u, d: SelectiveShape, dt, low, y, A, dt_bias, skip, state, sl
         return out
     _i32(cu)
     n = cu.numel() - 1
-    pl, py = _check(u, d, low, y, A, dt_bias, skip, state, slot, pos, out, dt.shape[0])
+    pl = _check(u, d, low, A, dt_bias, skip, state, slot, pos, out, dt.shape[0])
+    py = _proj(y, dt.shape[0], d.z_col + d.C, "gate")
+    expect(py[4] % 8 == 0 and (u.dtype == torch.bfloat16 or py[1] == 1), "gate rows")
+    same_device(u, y, dt, cu)
     expect(dt.dtype == torch.float32 and dt.dim() == 2 and dt.shape[1] == d.C and dt.stride(1) == 1 and dt.stride(0) % 4 == 0,
            "steps: fp32 [T, C]")
     expect(slot.numel() >= n, "state slots")
@@ -86,20 +87,20 @@ def selective_scan(u, d: SelectiveShape, dt, low, y, A, dt_bias, skip, state, sl
     return out
 
 
-def selective_step(u, d: SelectiveShape, dt_w, step, low, y, A, dt_bias, skip, state, slot, pos, row0: int, out):
+def selective_step(u, d: SelectiveShape, dt_w, step, low, A, dt_bias, skip, state, slot, pos, row0: int, out):
     """The same for one decoded token per sequence, rows row0..; ``dt_w`` [C, rank] (bf16 on the GPU: a ``shuffle_weights``
-    copy) is applied to ``step`` [*, rank] (``narrow_rows``) here."""
+    copy) is applied to ``step`` [*, rank] (``narrow_rows``) here.  The rows of ``out`` hold the gate on entry."""
     B = slot.numel()
     if not u.is_cuda:
         dt = step.float() @ dt_w.float().t()
-        c = ref.selective_scan(u, d, dt, low, y, A, dt_bias, skip, state, slot, pos, ref._spans(None, B, row0), out.dtype)
+        c = ref.selective_scan(u, d._replace(z_col=0), dt, low, out.float(), A, dt_bias, skip, state, slot, pos, ref._spans(None, B, row0), out.dtype)
         out[row0:row0 + B] = c[row0:row0 + B]
         return out
-    pl, py = _check(u, d, low, y, A, dt_bias, skip, state, slot, pos, out, row0 + B)
+    pl = _check(u, d, low, A, dt_bias, skip, state, slot, pos, out, row0 + B)
     expect(d.C % 16 == 0 and d.rank % 32 == 0 and d.rank <= MAX_STEP_RANK and dt_w.dtype == u.dtype and dt_w.is_contiguous()
            and tuple(dt_w.shape) == (d.C, d.rank), "step weights [C, rank]")
     expect(step.dtype == u.dtype and step.shape[0] >= row0 + B and step.shape[1] == d.rank and step.stride(1) == 1
            and step.stride(0) == (d.rank if step.dtype == torch.bfloat16 else pl[4]), "low-rank steps")
-    native().selective_step(ptr(u), int(u.dtype == torch.float32), tuple(d), ptr(dt_w), ptr(step), pl, py, ptr(A), ptr(dt_bias), ptr(skip),
+    native().selective_step(ptr(u), int(u.dtype == torch.float32), tuple(d), ptr(dt_w), ptr(step), pl, ptr(A), ptr(dt_bias), ptr(skip),
                             ptr(state), ptr(slot), ptr(pos), int(row0), B, ptr(out), stream(u))
     return out

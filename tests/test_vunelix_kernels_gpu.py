@@ -95,15 +95,17 @@ def test_selective_step(C, N, K, B, dtype, slabs):
     R = c["d"].rank
     w = rnd(C, R, seed=11, dtype=dtype, scale=R ** -0.5)
     slot = c["slot"][row0:].contiguous()
-    out, want = torch.zeros(row0 + B, C, dtype=dtype, device=DEV), torch.zeros(row0 + B, C, dtype=dtype)
+    want = c["y"][..., C:].float().sum(0).to(dtype) if slabs > 1 else c["y"][:, C:].contiguous()
+    want[:row0] = 0
+    out = want.to(DEV)
     step = c["low"][:, :R].to(dtype)
     step = step.contiguous() if dtype == BF else c["low"][:, :R]
     g = to(c)
     gstep = step.to(DEV) if dtype == BF else g["low"][:, :R]
     gw = ops.shuffle_weights(w.to(DEV)) if dtype == BF else w.to(DEV)
-    ops.selective_step(g["u"], g["d"], gw, gstep, g["low"], g["y"], g["A"], g["dt_bias"], g["skip"], g["state"], slot.to(DEV),
+    ops.selective_step(g["u"], g["d"], gw, gstep, g["low"], g["A"], g["dt_bias"], g["skip"], g["state"], slot.to(DEV),
                        g["pos"], row0, out)
-    ops.selective_step(c["u"], c["d"], w, step, c["low"], c["y"], c["A"], c["dt_bias"], c["skip"], c["state"], slot, c["pos"],
+    ops.selective_step(c["u"], c["d"], w, step, c["low"], c["A"], c["dt_bias"], c["skip"], c["state"], slot, c["pos"],
                        row0, want)
     close(out, want, 8e-3 if dtype == BF else 3e-5)
     close(g["state"], c["state"], 2e-5)
@@ -126,8 +128,9 @@ def test_scan_continued_by_steps_matches_one_scan():
             ops.selective_scan(g["u"][s], g["d"], dt.to(DEV)[s], g["low"][s], g["y"][s], g["A"], g["dt_bias"], g["skip"], g["state"],
                                g["slot"], g["pos"][s].contiguous(), i32(0, m).to(DEV), o)
             out[s], at = o, at + m
+        out[at:] = g["y"][at:, C:]
         for t in range(at, n):
-            ops.selective_step(g["u"], g["d"], w.to(DEV), g["low"][:, :64], g["low"], g["y"], g["A"], g["dt_bias"], g["skip"],
+            ops.selective_step(g["u"], g["d"], w.to(DEV), g["low"][:, :64], g["low"], g["A"], g["dt_bias"], g["skip"],
                                g["state"], g["slot"], g["pos"], t, out)
         outs.append((out.cpu(), g["state"].cpu()))
     close(outs[1][0], outs[0][0], 1e-5)
@@ -172,8 +175,10 @@ def test_short_conv_step(C, taps, B, dtype, yt, slabs):
     slot = torch.randperm(B + 1, generator=torch.Generator().manual_seed(1))[:B].int()
     pos = torch.cat([torch.zeros(row0), torch.arange(B) * 3 % 23]).int()
     gr, out, want = ring.to(DEV), torch.zeros(row0 + B, C, dtype=dtype, device=DEV), torch.zeros(row0 + B, C, dtype=dtype)
-    ops.short_conv_step(y.to(DEV), col0, w.to(DEV), b.to(DEV), gr, slot.to(DEV), pos.to(DEV), row0, out)
-    ops.short_conv_step(y, col0, w, b, ring, slot, pos, row0, want)
+    z, zw = torch.zeros_like(out), torch.zeros_like(want)
+    ops.short_conv_step(y.to(DEV), col0, w.to(DEV), b.to(DEV), gr, slot.to(DEV), pos.to(DEV), row0, out, 8, z)
+    ops.short_conv_step(y, col0, w, b, ring, slot, pos, row0, want, 8, zw)
+    close(z, zw, 4e-3 if dtype == BF else 1e-6)
     close(out, want, 8e-3 if dtype == BF else 3e-6)
     close(gr, ring, 4e-3 if dtype == BF else 1e-6)
 

@@ -216,7 +216,11 @@ def test_selective_scan_mechanisms():
     u[:4] = ops.short_conv(x[:4].float(), 0, cw.t().contiguous().float(), cb.float(), ring, torch.tensor([1]), pos[:4],
                            torch.tensor([0, 4]), 4)
     for t in range(4, T):
-        ops.short_conv_step(x.float(), 0, cw.t().contiguous().float(), cb.float(), ring, torch.tensor([1]), pos, t, u)
+        z = torch.zeros(T, C)
+        both = torch.cat([x, 2 * x], 1).float()
+        ops.short_conv_step(both, 0, cw.t().contiguous().float(), cb.float(), ring, torch.tensor([1]), pos, t, u, C, z)
+        near(z[t], 2 * x[t])
+        assert float(z.abs().sum(1).gt(0).sum()) == 1
     near(u, oracle.short_conv(x, cw, cb))
     Np = 16
     d = ops.SelectiveShape(C, Np, K, K, K + Np, C)
@@ -236,8 +240,9 @@ def test_selective_scan_mechanisms():
                            torch.tensor([0, hi - lo]), o)
         out[lo:hi] = o
     step = low[:, :K].float()
+    out[5:] = y[5:, C:].float()
     for t in range(5, T):
-        ops.selective_step(ux.float(), d, dtw.float(), step, low.float(), y.float(), *a, t, out)
+        ops.selective_step(ux.float(), d, dtw.float(), step, low.float(), *a, t, out)
     S, want = oracle.selective_scan(ux, oracle.softplus(dt + dtb), A, low[:, K:K + N], low[:, K + Np:K + Np + N])[::-1]
     near(out, (want + skip * ux) * oracle.silu(y[:, C:]))
     near(st[2, :, :N], S)
