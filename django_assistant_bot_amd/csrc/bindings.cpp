@@ -226,12 +226,13 @@ PYBIND11_MODULE(_native, m) {
     return dab::SelectiveShape{std::get<0>(t), std::get<1>(t), std::get<2>(t), std::get<3>(t), std::get<4>(t), std::get<5>(t)};
   };
   m.def("selective_scan", [proj, sel](u x, int act_f32, const SS& d, const P& dt, const P& bc, const P& y, u A, u dt_bias,
-                                      u skip, u state, u slot, u pos, u cu, int chunks, u out, u s) {
+                                      u skip, u state, u slot, u pos, u cu, int chunks, int max_q, int segs, u ws, u out, u s) {
     check(dab::selective_scan(CVP(x), act_f32, sel(d), proj(dt), proj(bc), proj(y), (const float*)A, (const float*)dt_bias,
                               (const float*)skip, (float*)state, (const int*)slot, (const int*)pos, (const int*)cu, chunks,
-                              VP(out), ST(s)),
+                              max_q, segs, (float*)ws, VP(out), ST(s)),
           "selective_scan");
   });
+  m.def("selective_segments", [sel](const SS& d, int chunks, int max_q) { return dab::selective_segments(sel(d), chunks, max_q); });
   m.def("selective_step", [proj, sel](u x, int act_f32, const SS& d, u dt_w, u low, const P& bc, u A, u dt_bias,
                                       u skip, u state, u slot, u pos, int row0, int B, u out, u s) {
     check(dab::selective_step(CVP(x), act_f32, sel(d), CVP(dt_w), CVP(low), proj(bc), (const float*)A, (const float*)dt_bias,

@@ -119,8 +119,9 @@ struct SelectiveShape {
 int selective_state_width(int N);  // N padded as the state is stored (0: too many)
 int narrow_rows(Proj z, float* out, void* low, int N, int R, int T, hipStream_t s);
 int selective_scan(const void* u, int act_f32, SelectiveShape d, Proj dt, Proj bc, Proj y, const float* A, const float* dt_bias,
-                   const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, void* out,
-                   hipStream_t s);
+                   const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, int max_q,
+                   int segs, float* ws, void* out, hipStream_t s);  // ws (segs > 1): chunks * segs * C * (Np + 1) floats
+int selective_segments(SelectiveShape d, int chunks, int max_q);
 int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_w, const void* low, Proj bc, const float* A,
                    const float* dt_bias, const float* skip, float* state, const int* slot, const int* pos, int row0, int B,
                    void* out, hipStream_t s);

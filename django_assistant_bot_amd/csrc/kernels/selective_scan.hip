@@ -5,6 +5,9 @@
 //
 //   narrow_rows     slabs of that projection -> fp32 rows, and its first columns in bf16 (operand of W_dt)
 //   selective_scan  prompt portions: a workgroup walks one sequence for a block of channels, a tile of tokens at a time
+//                   (few long portions are cut into segments that run side by side: each is summed up from a zero state,
+//                   selective_combine walks the summaries -- a segment takes S to exp(A sum dt) S + S_loc --, and then
+//                   all are scanned from their own start states)
 //   selective_step  one decoded token per sequence, the gate's rows being replaced by the result; W_dt low is formed in the kernel on MFMA, for up to 16 sequences at once
 //
 // A channel is shared by L neighbouring lanes, NS entries each, so a step's read-out is a sum over L lanes; four tokens'
@@ -83,10 +86,17 @@ struct SelScan {
   const int* pos;
   const int* cu;
   void* out;            // [T, C]
+  // segments: tokens of one, their number, start states (and before: summaries) [chunks, segs, C, Np], step sums
+  // [chunks, segs, C]
+  int seg_len, segs;
+  float* starts;
+  float* sums;
 };
 
+enum ScanMode { SCAN_WHOLE, SCAN_SUMMARY, SCAN_SEGMENT };
+
 // A lane holds its NS entries of CPT channels, 256 / L apart, so that a token's B and C are read once for all of them.
-template <typename PT, typename AT, int L, int NS, int CPT, int TB>
+template <typename PT, typename AT, int L, int NS, int CPT, int TB, int MODE>
 __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
   constexpr int CG = 256 / L, CH = CG * CPT, Np = L * NS, ITEMS = TB * CH / 8, BCN = TB * 2 * Np / 4, BCV = (BCN + 255) / 256;
   constexpr bool AHEAD = NS * CPT <= 4;  // (registers)
@@ -95,20 +105,26 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
   __shared__ __attribute__((aligned(16))) float xs[TB][CH];      // dt u
   __shared__ __attribute__((aligned(16))) float bc[TB][2 * Np];  // B | C
   const int tid = threadIdx.x, ch = tid / L, part = tid % L, c0 = blockIdx.x * CH, b = blockIdx.y;
-  const int r0 = p.cu[b], n = p.cu[b + 1] - r0;
-  if (n <= 0) return;
+  const int seg = MODE == SCAN_WHOLE ? 0 : blockIdx.z, t_seg = seg * p.seg_len;
+  const int r0 = p.cu[b] + t_seg, left = p.cu[b + 1] - r0;
+  const bool last = MODE == SCAN_WHOLE || left <= p.seg_len;
+  if (left <= 0 || (MODE == SCAN_SUMMARY && last)) return;
+  const int n = last ? left : p.seg_len;
   const int C = p.d.C;
-  float S[CPT][NS], A[CPT][NS];
+  float S[CPT][NS], A[CPT][NS], total[CPT];
   float* sp[CPT];
-  const bool fresh = p.pos[r0] == 0;
+  const bool fresh = MODE == SCAN_SUMMARY || (MODE == SCAN_WHOLE && p.pos[r0] == 0);
 #pragma unroll
   for (int i = 0; i < CPT; ++i) {
     const size_t c = min(c0 + ch + i * CG, C - 1);
     sp[i] = p.state + ((size_t)p.slot[b] * C + c) * Np + part * NS;
+    float* at = MODE == SCAN_WHOLE ? sp[i] : p.starts + (((size_t)b * p.segs + seg) * C + c) * Np + part * NS;
+    if (MODE == SCAN_SUMMARY) sp[i] = at;
+    total[i] = 0.f;
 #pragma unroll
     for (int j = 0; j < NS; ++j) {
-      const float v = sp[i][j];
-      S[i][j] = fresh ? 0.f : v;
+      const float v = fresh ? 0.f : at[j];
+      S[i][j] = v;
       A[i][j] = p.A[c * Np + part * NS + j];
     }
   }
@@ -196,12 +212,14 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
 #pragma unroll
         for (int i = 0; i < CPT; ++i) {
           y[i][q] = 0.f;
+          if (MODE == SCAN_SUMMARY) total[i] += dv[q][i];
 #pragma unroll
           for (int j = 0; j < NS; ++j) {
             S[i][j] = fmaf(__builtin_amdgcn_exp2f(dv[q][i] * A[i][j]), S[i][j], xv[q][i] * br[q][j]);
-            y[i][q] = fmaf(S[i][j], cr[q][j], y[i][q]);
+            if (MODE != SCAN_SUMMARY) y[i][q] = fmaf(S[i][j], cr[q][j], y[i][q]);
           }
         }
+      if (MODE == SCAN_SUMMARY) continue;
       const bool b0 = part & 1, b1 = part & 2;
 #pragma unroll
       for (int i = 0; i < CPT; ++i) {
@@ -212,7 +230,7 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
       }
     }
     __syncthreads();
-    if (live) {
+    if (MODE != SCAN_SUMMARY && live) {
       float o[8];
       ElemIO<float>::load8(&ds[it][ic], o);
 #pragma unroll
@@ -222,10 +240,38 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelScan p) {
   }
 #pragma unroll
   for (int i = 0; i < CPT; ++i)
-    if (c0 + ch + i * CG < C) {
+    if (c0 + ch + i * CG < C && (last || MODE == SCAN_SUMMARY)) {
 #pragma unroll
       for (int j = 0; j < NS; ++j) sp[i][j] = S[i][j];
+      if (MODE == SCAN_SUMMARY && part == 0) p.sums[((size_t)b * p.segs + seg) * C + c0 + ch + i * CG] = total[i];
     }
+}
+
+// the segments' summaries -> their start states; four state entries a thread
+__global__ __launch_bounds__(256) void selective_combine_kernel(SelScan p) {
+  const int Np = p.d.Np, C = p.d.C, b = blockIdx.y, e = (blockIdx.x * 256 + threadIdx.x) * 4;
+  const int r0 = p.cu[b], n = p.cu[b + 1] - r0;
+  if (n <= 0 || e >= C * Np) return;
+  f32x4 S = {0.f, 0.f, 0.f, 0.f};
+  if (p.pos[r0] != 0) S = *reinterpret_cast<const f32x4*>(p.state + (size_t)p.slot[b] * C * Np + e);
+  const f32x4 A = *reinterpret_cast<const f32x4*>(p.A + e);
+  for (int g = 0; g * p.seg_len < n; ++g) {
+    float* at = p.starts + ((size_t)b * p.segs + g) * C * Np + e;
+    const bool more = (g + 1) * p.seg_len < n;
+    const f32x4 loc = more ? *reinterpret_cast<const f32x4*>(at) : S;
+    const float sum = more ? p.sums[((size_t)b * p.segs + g) * C + e / Np] : 0.f;
+    *reinterpret_cast<f32x4*>(at) = S;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) S[j] = fmaf(__builtin_amdgcn_exp2f(sum * A[j]), S[j], loc[j]);
+  }
+}
+
+// Segments of the longest portion: enough that every SIMD has several waves, none shorter than 256 tokens.  1: not cut.
+int selective_segments(SelectiveShape d, int chunks, int max_q) {
+  const long waves = (long)chunks * d.C / 16;  // four lanes a channel
+  if (waves < 1 || waves >= 2048 || max_q < 512) return 1;
+  const long want = (4096 + waves - 1) / waves, most = max_q / 256;
+  return (int)(want < most ? want : most);
 }
 
 static bool bad_shape(const SelectiveShape& d) {
@@ -233,17 +279,33 @@ static bool bad_shape(const SelectiveShape& d) {
 }
 
 int selective_scan(const void* u, int act_f32, SelectiveShape d, Proj dt, Proj bc, Proj y, const float* A, const float* dt_bias,
-                   const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, void* out,
-                   hipStream_t s) {
-  if (chunks <= 0) return 0;
+                   const float* skip, float* state, const int* slot, const int* pos, const int* cu, int chunks, int max_q,
+                   int segs, float* ws, void* out, hipStream_t s) {
+  if (chunks <= 0 || max_q <= 0) return 0;
+  if (segs < 1 || segs > 65535 || (segs > 1 && !ws)) return hipErrorInvalidValue;
   if (bad_shape(d) || y.S < 1 || y.ld % 8 || y.slab % 8 || !dt.f32 || dt.S != 1 || dt.ld % 4 || !bc.f32 || bc.S != 1 || bc.ld % 4 || chunks > 65535)
     return hipErrorInvalidValue;
-  SelScan p{u, d, dt, bc, y, A, dt_bias, skip, state, slot, pos, cu, out};
+  SelScan p{u, d, dt, bc, y, A, dt_bias, skip, state, slot, pos, cu, out, 0, segs, nullptr, nullptr};
+  p.seg_len = segs > 1 ? ((max_q + segs - 1) / segs + 63) / 64 * 64 : max_q;
+  if (segs > 1) {
+    p.starts = ws;
+    p.sums = ws + (size_t)chunks * segs * d.C * d.Np;
+  }
   // lanes per channel: more of them when the channels alone leave SIMDs without a wave
-  const long waves = (long)chunks * d.C / 16;
-#define SEL_L(PT, AT, L, NS, CPT, TB)                                                                              \
-  hipLaunchKernelGGL((selective_scan_kernel<PT, AT, L, NS, CPT, TB>),                                              \
-                     dim3((d.C + 256 / L * CPT - 1) / (256 / L * CPT), chunks), dim3(256), 0, s, p)
+  const long waves = (long)chunks * d.C / 16 * segs;
+#define SEL_M(PT, AT, L, NS, CPT, TB, MODE)                                                                          \
+  hipLaunchKernelGGL((selective_scan_kernel<PT, AT, L, NS, CPT, TB, MODE>),                                          \
+                     dim3((d.C + 256 / L * CPT - 1) / (256 / L * CPT), chunks, segs), dim3(256), 0, s, p)
+#define SEL_L(PT, AT, L, NS, CPT, TB)                                                                                \
+  do {                                                                                                               \
+    if (segs == 1) {                                                                                                 \
+      SEL_M(PT, AT, L, NS, CPT, TB, SCAN_WHOLE);                                                                     \
+    } else {                                                                                                         \
+      SEL_M(PT, AT, L, NS, CPT, TB, SCAN_SUMMARY);                                                                   \
+      hipLaunchKernelGGL(selective_combine_kernel, dim3((d.C * d.Np / 4 + 255) / 256, chunks), dim3(256), 0, s, p);  \
+      SEL_M(PT, AT, L, NS, CPT, TB, SCAN_SEGMENT);                                                                   \
+    }                                                                                                                \
+  } while (0)
 #define SEL_N(PT, AT)                                      \
   do {                                                     \
     switch (d.Np) {                                        \
@@ -267,6 +329,7 @@ int selective_scan(const void* u, int act_f32, SelectiveShape d, Proj dt, Proj b
   DAB_PROJ_DISPATCH(y, act_f32, SEL_N);
 #undef SEL_N
 #undef SEL_L
+#undef SEL_M
   return hipGetLastError();
 }
 

@@ -210,7 +210,7 @@ class VunelixModel(LatentAttention, HybridProjections):
         low, step = ops.narrow_rows(self._aux(u, L.x_w, sk), L.narrow, d.rank, T, self.dtype)
         if Tp:
             dt = self._aux(step[:Tp], L.dt_w, False, wide=True)
-            ops.selective_scan(u, d, dt, low, y, L.A, L.dt_bias, L.skip, state, meta.state_slots, pos, meta.cu_q, out)
+            ops.selective_scan(u, d, dt, low, y, L.A, L.dt_bias, L.skip, state, meta.state_slots, pos, meta.cu_q, meta.max_q, out)
         if Tp < T:
             ops.selective_step(u, d, L.dt_w, step, low, L.A, L.dt_bias, L.skip, state, slot, pos, Tp, out)
         return self._proj(out, L.o_w, sk, name="o")

@@ -64,10 +64,11 @@ def _check(u, d: SelectiveShape, low, A, dt_bias, skip, state, slot, pos, out, r
     return pl
 
 
-def selective_scan(u, d: SelectiveShape, dt, low, y, A, dt_bias, skip, state, slot, pos, cu, out):
+def selective_scan(u, d: SelectiveShape, dt, low, y, A, dt_bias, skip, state, slot, pos, cu, max_q: int, out, segments: int | None = None):
     """The recurrence over the portions ``cu`` of the convolved channels ``u``, read-out, skip and silu gate, into the same
     rows of ``out`` [T, C]; ``state`` [slots, C, Np] goes on from where the sequence left it (zero at position 0).  ``dt``
-    fp32 [T, C]: the step before bias and softplus; ``A``: -exp(A_log) log2(e)."""
+    fp32 [T, C]: the step before bias and softplus; ``A``: -exp(A_log) log2(e).  ``max_q``: the longest portion;
+    ``segments`` it is cut into, which run side by side (default: when the launch would be small)."""
     if not u.is_cuda:
         spans = ref._spans(cu, 0, 0)
         n = spans[-1][1]
@@ -82,8 +83,11 @@ def selective_scan(u, d: SelectiveShape, dt, low, y, A, dt_bias, skip, state, sl
     expect(dt.dtype == torch.float32 and dt.dim() == 2 and dt.shape[1] == d.C and dt.stride(1) == 1 and dt.stride(0) % 4 == 0,
            "steps: fp32 [T, C]")
     expect(slot.numel() >= n, "state slots")
+    segs = native().selective_segments(tuple(d), n, int(max_q)) if segments is None else int(segments)
+    ws = torch.empty((n * segs * d.C * (d.Np + 1),), dtype=torch.float32, device=u.device) if segs > 1 else None
     native().selective_scan(ptr(u), int(u.dtype == torch.float32), tuple(d), _proj(dt, dt.shape[0], d.C), pl, py, ptr(A),
-                            ptr(dt_bias), ptr(skip), ptr(state), ptr(slot), ptr(pos), ptr(cu), n, ptr(out), stream(u))
+                            ptr(dt_bias), ptr(skip), ptr(state), ptr(slot), ptr(pos), ptr(cu), n, int(max_q), segs,
+                            ptr(ws), ptr(out), stream(u))
     return out
 
 

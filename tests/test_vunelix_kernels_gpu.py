@@ -77,8 +77,9 @@ def test_selective_scan(C, N, lens, dtype):
     dt = rnd(sum(lens), C, seed=9, dtype=F32)
     g, out, want = to(c), torch.zeros(sum(lens), C, dtype=dtype, device=DEV), torch.zeros(sum(lens), C, dtype=dtype)
     before = c["state"].clone()
-    ops.selective_scan(g["u"], g["d"], dt.to(DEV), *(g[k] for k in ("low", "y", "A", "dt_bias", "skip", "state", "slot", "pos", "cu")), out)
-    ops.selective_scan(c["u"], c["d"], dt, *(c[k] for k in ("low", "y", "A", "dt_bias", "skip", "state", "slot", "pos", "cu")), want)
+    names = ("low", "y", "A", "dt_bias", "skip", "state", "slot", "pos", "cu")
+    ops.selective_scan(g["u"], g["d"], dt.to(DEV), *(g[k] for k in names), max(lens), out)
+    ops.selective_scan(c["u"], c["d"], dt, *(c[k] for k in names), max(lens), want)
     close(out, want, 6e-3 if dtype == BF else 3e-5)
     close(g["state"], c["state"], 3e-5)
     idle = [s for s in range(len(before)) if s not in c["slot"].tolist()]
@@ -112,6 +113,29 @@ def test_selective_step(C, N, K, B, dtype, slabs):
     assert float(out[:row0].abs().sum()) == 0
 
 
+@pytest.mark.parametrize("C,N", [(128, 16), (512, 24), (128, 64), (128, 200)])
+@pytest.mark.parametrize("segs", [2, 3, 5])
+@pytest.mark.parametrize("dtype", [BF, F32])
+def test_segmented_scan(C, N, segs, dtype):
+    """Portions of unequal lengths cut into segments: some fill all of them, some end inside one or at an edge."""
+    lens = [64 * segs + 7, 1, 64, 65, 130, 64 * segs]
+    c = scan_case(C, N, 20, lens, dtype, 1, starts=[0, 5, 0, 9, 300, 2])
+    c["A"] *= 0.05  # slow decays: what a segment hands on counts to the end
+    dt = rnd(sum(lens), C, seed=9, dtype=F32) - 2
+    g, out, want = to(c), torch.zeros(sum(lens), C, dtype=dtype, device=DEV), torch.zeros(sum(lens), C, dtype=dtype)
+    names = ("low", "y", "A", "dt_bias", "skip", "state", "slot", "pos", "cu")
+    ops.selective_scan(g["u"], g["d"], dt.to(DEV), *(g[k] for k in names), max(lens), out, segments=segs)
+    ops.selective_scan(c["u"], c["d"], dt, *(c[k] for k in names), max(lens), want)
+    close(out, want, 6e-3 if dtype == BF else 3e-5)
+    close(g["state"], c["state"], 3e-5)
+
+
+def test_segment_choice():
+    seg = lambda C, n, q: ops.native().selective_segments((C, 16, 64, 64, 80, C), n, q)  # noqa: E731
+    assert seg(8192, 16, 1024) == seg(8192, 4, 4096) == seg(128, 1, 511) == 1
+    assert seg(8192, 1, 8192) == 8 and seg(4096, 1, 8192) == 16 and seg(128, 1, 1024) == 4
+
+
 def test_scan_continued_by_steps_matches_one_scan():
     C, N, K, n = 256, 16, 64, 70
     c = scan_case(C, N, K, [n], F32, 1)
@@ -126,7 +150,7 @@ def test_scan_continued_by_steps_matches_one_scan():
             o = torch.zeros(m, C, device=DEV)
             s = slice(at, at + m)
             ops.selective_scan(g["u"][s], g["d"], dt.to(DEV)[s], g["low"][s], g["y"][s], g["A"], g["dt_bias"], g["skip"], g["state"],
-                               g["slot"], g["pos"][s].contiguous(), i32(0, m).to(DEV), o)
+                               g["slot"], g["pos"][s].contiguous(), i32(0, m).to(DEV), m, o)
             out[s], at = o, at + m
         out[at:] = g["y"][at:, C:]
         for t in range(at, n):
@@ -147,7 +171,7 @@ def test_scan_against_the_oracle_at_extreme_steps():
     c["A"][:, :N] = a / math.log(2)
     c["dt_bias"].zero_()
     g, out = to(c), torch.zeros(T, C, device=DEV)
-    ops.selective_scan(g["u"], g["d"], dt.to(DEV), *(g[k] for k in ("low", "y", "A", "dt_bias", "skip", "state", "slot", "pos", "cu")), out)
+    ops.selective_scan(g["u"], g["d"], dt.to(DEV), *(g[k] for k in ("low", "y", "A", "dt_bias", "skip", "state", "slot", "pos", "cu")), T, out)
     D = lambda t: t.double()  # noqa: E731
     y, S = oracle.selective_scan(D(c["u"]), oracle.softplus(D(dt)), D(a), D(c["low"][:, 64:64 + N]), D(c["low"][:, 80:80 + N]))
     want = (y + D(c["skip"]) * D(c["u"])) * oracle.silu(D(c["y"][:, C:]))
@@ -159,7 +183,7 @@ def test_scan_against_the_oracle_at_extreme_steps():
     for t in range(0, T, 7):
         o = torch.zeros(1, C, device=DEV)
         ops.selective_scan(g["u"][t:t + 1], g["d"], dt[t:t + 1].to(DEV), g["low"][t:t + 1], g["y"][t:t + 1], g["A"], g["dt_bias"],
-                           g["skip"], g["state"], g["slot"], i32(0).to(DEV), i32(0, 1).to(DEV), o)
+                           g["skip"], g["state"], g["slot"], i32(0).to(DEV), i32(0, 1).to(DEV), 1, o)
         w = oracle.softplus(D(dt[t])) * D(c["u"][t]) * (D(c["low"][t, 64:64 + N]) * D(c["low"][t, 80:80 + N])).sum() * oracle.silu(D(c["y"][t, C:]))
         rel = ((o.cpu()[0].double() - w) / w).abs()[small[t]]
         assert rel.numel() == 0 or rel.max() < 2e-5
@@ -371,9 +395,9 @@ def test_shapes_are_refused_on_the_host():
         a = list(args)
         a[i] = bad
         with pytest.raises((ValueError, TypeError)):
-            ops.selective_scan(c["u"], c["d"], dt, *a, out)
+            ops.selective_scan(c["u"], c["d"], dt, *a, 4, out)
     with pytest.raises(ValueError):
-        ops.selective_scan(c["u"], c["d"], dt.to(BF), *args, out)
+        ops.selective_scan(c["u"], c["d"], dt.to(BF), *args, 4, out)
     with pytest.raises(ValueError):
         ops.softcap(torch.zeros(2, 12, device=DEV), 1.0)
     with pytest.raises(ValueError):

@@ -237,7 +237,7 @@ def test_selective_scan_mechanisms():
     for lo, hi in ((0, 3), (3, 5)):
         o = torch.zeros(hi - lo, C)
         ops.selective_scan(ux[lo:hi].float(), d, dt[lo:hi].float(), low[lo:hi].float(), y[lo:hi].float(), *a[:5], pos[lo:hi],
-                           torch.tensor([0, hi - lo]), o)
+                           torch.tensor([0, hi - lo]), hi - lo, o)
         out[lo:hi] = o
     step = low[:, :K].float()
     out[5:] = y[5:, C:].float()
