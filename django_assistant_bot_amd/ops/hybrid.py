@@ -226,7 +226,8 @@ def gemm_narrow(x, w):
     expect(K % 64 == 0 and N % 16 == 0 and x.stride(0) % 8 == 0, "gemm_narrow: K % 64, N % 16")
     tall = M >= 2048 and N > 128  # several column tiles read the same rows
     tiles, S = -(-M // (128 if tall else 32)) * -(-N // 128), 1
-    while S < 16 and tiles * S < 1024 and K % (128 * S) == 0 and K // (2 * S) >= 256:
+    want = 512 if tall else 1024  # (a slab of tall tiles is as many bytes as the rows it saves waiting for)
+    while S < 16 and tiles * S < want and K % (128 * S) == 0 and K // (2 * S) >= 256:
         S *= 2
     out = torch.empty((S, M, N) if S > 1 else (M, N), dtype=torch.float32, device=x.device)
     native().gemm_narrow(ptr(x), x.stride(0), ptr(w), ptr(out), M, N, K, S, int(tall), stream(x))
