@@ -226,7 +226,7 @@ def gemm_narrow(x, w):
     expect(K % 64 == 0 and N % 16 == 0 and x.stride(0) % 8 == 0, "gemm_narrow: K % 64, N % 16")
     tall = M >= 2048 and N > 128  # several column tiles read the same rows
     tiles, S = -(-M // (128 if tall else 32)) * -(-N // 128), 1
-    want = 512 if tall else 1024  # (a slab of tall tiles is as many bytes as the rows it saves waiting for)
+    want = 384 if tall else 1024  # (a tall launch fills the chip sooner, and its slabs are many bytes)
     while S < 16 and tiles * S < want and K % (128 * S) == 0 and K // (2 * S) >= 256:
         S *= 2
     out = torch.empty((S, M, N) if S > 1 else (M, N), dtype=torch.float32, device=x.device)
