@@ -68,6 +68,8 @@ def _body(rank, world, layout, port, out_path):
                         max_batch=8, block_size=64, num_blocks=96, max_prefill_tokens=256, tp_group=group,
                         tp_size=world, tp_rank=tp_rank)
         assert eng.model.custom_ar is not None and eng.model.frag
+        # ranks that share one card also share its time and the host's CPUs: a peer may arrive seconds late
+        eng.model.custom_ar.spin_limit = 1 << 26
         # vocab-parallel LM head: this rank's V / tp rows (+ zero pad rows)
         assert eng.vp and eng.model.vocab_local == cfg.vocab_size // world
         assert eng.model.lm_head.shape[0] == -(-cfg.vocab_size // world // 384) * 384
