@@ -165,17 +165,18 @@ PYBIND11_MODULE(_native, m) {
   // chunked / sink attention over the paged cache
   m.def("flash_attention_chunk",
         [](u q, long qst, long qsh, u kc, u vc, u bt, int max_blocks, int bs, u out, long ost, long osh, u cu_q, u ctx_k,
-           int batch, int max_sq, int Hq, int Hkv, int D, float scale, int chunk, u sink, float out_scale, u s) {
+           int batch, int max_sq, int Hq, int Hkv, int D, float scale, int chunk, u sink, u slopes, float out_scale, u s) {
           check(dab::flash_attention(CVP(q), qst, qsh, nullptr, nullptr, 0, 0, CVP(kc), CVP(vc), (const int*)bt,
                                      max_blocks, bs, VP(out), ost, osh, (const int*)cu_q, nullptr, (const int*)ctx_k,
                                      batch, max_sq, Hq, Hkv, D, 1, 1, scale, ST(s), nullptr, nullptr, 0,
-                                     (const float*)sink, chunk, out_scale),
+                                     (const float*)sink, chunk, out_scale, (const float*)slopes),
                 "flash_attention_chunk");
         });
   m.def("any_attention", [](u q, u kc, u vc, int f32, u bt, int max_blocks, int bs, u cu, u ctx, int B, int T, int H,
-                            int G, int D, int chunk, float scale, u sink, u out, long o_tok, float out_scale, u s) {
+                            int G, int D, int chunk, float scale, u sink, u slopes, u out, long o_tok, float out_scale,
+                            u s) {
     check(dab::any_attention(CVP(q), CVP(kc), CVP(vc), f32, (const int*)bt, max_blocks, bs, (const int*)cu,
-                             (const int*)ctx, B, T, H, G, D, chunk, scale, (const float*)sink, VP(out), o_tok, out_scale,
+                             (const int*)ctx, B, T, H, G, D, chunk, scale, (const float*)sink, (const float*)slopes, VP(out), o_tok, out_scale,
                              ST(s)),
           "any_attention");
   });
@@ -191,8 +192,8 @@ PYBIND11_MODULE(_native, m) {
                             ST(s)),
           "rms_residual");
   });
-  m.def("sigmoid_gate", [proj](const P& y, int col0, u x, long ldx, int act_f32, int n, int T, u s) {
-    check(dab::sigmoid_gate(proj(y), col0, VP(x), ldx, act_f32, n, T, ST(s)), "sigmoid_gate");
+  m.def("sigmoid_gate", [proj](const P& y, int col0, int per, u x, long ldx, int act_f32, int n, int T, u s) {
+    check(dab::sigmoid_gate(proj(y), col0, per, VP(x), ldx, act_f32, n, T, ST(s)), "sigmoid_gate");
   });
   m.def("softcap", [proj](const P& y, float cap, u out, int n, int T, u s) {
     check(dab::softcap(proj(y), cap, (float*)out, n, T, ST(s)), "softcap");
@@ -202,6 +203,46 @@ PYBIND11_MODULE(_native, m) {
     check(dab::qk_rope_write(proj(y), col0, H, G, D, dim, rot, (const double*)freq, eps, norm, (const int*)positions,
                              (const int64_t*)slots, VP(q), VP(kc), VP(vc), act_f32, bs, T, ST(s)),
           "qk_rope_write");
+  });
+  // routed = (expert rows, indices, weights, choices per token, experts); gate = (projection, column, bias);
+  // depth = (results, weights, stride, n, keep)
+  m.def("gated_residual", [proj](u src, u x, u h, int act_f32, const P& y, u ids, const std::tuple<u, u, u, int, int>& routed,
+                                 const P& g, int g_col, u g_bias, u post, const std::tuple<u, u, long, int, int>& depth, u gain,
+                                 int n_true, float eps, int rows, int cols, u s) {
+    dab::GatedResidual p{};
+    p.src = (const float*)src, p.x = (float*)x, p.h = VP(h), p.y = proj(y), p.ids = (const int*)ids;
+    p.pairs = CVP(std::get<0>(routed)), p.idx = (const int*)std::get<1>(routed), p.wt = (const float*)std::get<2>(routed);
+    p.top = std::get<3>(routed), p.experts = std::get<4>(routed);
+    p.g = proj(g), p.g_col = g_col, p.g_bias = (const float*)g_bias, p.post = (const float*)post;
+    p.depth = (float*)std::get<0>(depth), p.weights = (const float*)std::get<1>(depth), p.depth_stride = std::get<2>(depth);
+    p.n = std::get<3>(depth), p.keep = std::get<4>(depth);
+    p.gain = (const float*)gain, p.inv_n = 1.f / n_true, p.eps = eps, p.cols = cols;
+    check(dab::gated_residual(p, act_f32, rows, ST(s)), "gated_residual");
+  });
+  m.def("poly_norm", [proj](const P& y, int n, int cols, float a, float b, float c, float e, float eps, u out, int act_f32, int T,
+                            u s) {
+    check(dab::poly_norm(proj(y), n, cols, a, b, c, e, eps, VP(out), act_f32, T, ST(s)), "poly_norm");
+  });
+  // heads = (H, G, D, dim, whole); conv = (taps, weights, ring, slots); rot = (dims, turns, factor); temp = (coef, every);
+  // cache = (k, v, block size); mix = (first values, their width, mode, weight)
+  m.def("attn_inputs", [proj](const P& y, int col0, const std::tuple<int, int, int, int, int>& heads, float eps, u gain, u bias,
+                              const std::tuple<int, u, u, u>& conv, const std::tuple<int, u, float>& rot,
+                              const std::tuple<float, int>& temp, u positions, u slots, u q, const std::tuple<u, u, int>& cache,
+                              const std::tuple<u, int, int, float>& mix, u cu, int row0, int rows, int max_q, int act_f32, u s) {
+    dab::AttnInputs p{};
+    const int dim = std::get<3>(heads);
+    p.y = proj(y), p.col0 = col0, p.H = std::get<0>(heads), p.G = std::get<1>(heads), p.D = std::get<2>(heads);
+    p.whole = std::get<4>(heads), p.eps = eps, p.gain = (const float*)gain, p.bias = (const float*)bias;
+    p.inv_q = 1.f / (p.whole ? p.H * dim : dim), p.inv_k = 1.f / (p.whole ? p.G * dim : dim);
+    p.taps = std::get<0>(conv), p.conv = (const float*)std::get<1>(conv), p.ring = VP(std::get<2>(conv));
+    p.slot = (const int*)std::get<3>(conv);
+    p.rot = std::get<0>(rot), p.turns = (const double*)std::get<1>(rot), p.rot_mul = std::get<2>(rot);
+    p.t_coef = std::get<0>(temp), p.t_every = std::get<1>(temp);
+    p.positions = (const int*)positions, p.slots = (const int64_t*)slots, p.q = VP(q);
+    p.kc = VP(std::get<0>(cache)), p.vc = VP(std::get<1>(cache)), p.bs = std::get<2>(cache);
+    p.first = VP(std::get<0>(mix)), p.first_w = std::get<1>(mix), p.mix = std::get<2>(mix), p.lam = std::get<3>(mix);
+    p.cu = (const int*)cu, p.row0 = row0;
+    check(dab::attn_inputs(p, act_f32, rows, max_q, ST(s)), "attn_inputs");
   });
   m.def("recurrent_state_width", &dab::recurrent_state_width);
   m.def("short_conv", [proj](const P& y, int col0, int C, int taps, u w, u bias, u ring, u slot, u pos, u cu, int chunks,
@@ -277,8 +318,9 @@ PYBIND11_MODULE(_native, m) {
                           VP(out), ldo, pad, row0, T, ST(s)),
           "gated_norm");
   });
-  m.def("moe_route", [proj](const P& z, int col0, int E, int top, float scale, int sigmoid, u idx, u wt, int T, u s) {
-    check(dab::moe_route(proj(z), col0, E, top, scale, sigmoid, (int*)idx, (float*)wt, T, ST(s)), "moe_route");
+  m.def("moe_route", [proj](const P& z, int col0, int E, int top, float scale, int scores, u correction, u idx, u wt, int T,
+                            u s) {
+    check(dab::moe_route(proj(z), col0, E, top, scale, scores, (const float*)correction, (int*)idx, (float*)wt, T, ST(s)), "moe_route");
   });
   m.def("moe_plan", [](u idx, int pairs, int E, int bm, u perm, u tiles, int max_tiles, u s) {
     check(dab::moe_plan((const int*)idx, pairs, E, bm, (int*)perm, VP(tiles), max_tiles, ST(s)), "moe_plan");
@@ -353,19 +395,19 @@ PYBIND11_MODULE(_native, m) {
   m.def("paged_decode_attention", [](u q, u kc, u vc, u bt, int max_blocks, int bs, u ctx, u out, u po, u pm, u pl,
                                      u cnt, int batch, int Hq, int Hkv, int D, int part_size, int max_parts,
                                      float scale, u s, u order, u w0, long w0_bytes, u w1, long w1_bytes,
-                                     int w_blocks, int chunk, u sink, float out_scale, long o_stride) {
+                                     int w_blocks, int chunk, u sink, float out_scale, long o_stride, u slopes) {
     dab::L3Warm warm{{(const char*)w0, (const char*)w1}, {w0_bytes, w1_bytes}, w_blocks};
     check(dab::paged_decode_attention(CVP(q), CVP(kc), CVP(vc), (const int*)bt, max_blocks, bs, (const int*)ctx, VP(out),
                                       (float*)po, (float*)pm, (float*)pl, (int*)cnt, batch, Hq, Hkv, D, part_size,
                                       max_parts, scale, ST(s), (const int*)order, &warm, chunk, (const float*)sink,
-                                      out_scale, o_stride),
+                                      out_scale, o_stride, (const float*)slopes),
           "paged_decode_attention");
   }, py::arg("q"), py::arg("kc"), py::arg("vc"), py::arg("bt"), py::arg("max_blocks"), py::arg("bs"), py::arg("ctx"),
      py::arg("out"), py::arg("po"), py::arg("pm"), py::arg("pl"), py::arg("cnt"), py::arg("batch"), py::arg("Hq"),
      py::arg("Hkv"), py::arg("D"), py::arg("part_size"), py::arg("max_parts"), py::arg("scale"), py::arg("s"),
      py::arg("order") = 0, py::arg("w0") = 0, py::arg("w0_bytes") = 0, py::arg("w1") = 0, py::arg("w1_bytes") = 0,
      py::arg("w_blocks") = 0, py::arg("chunk") = 0, py::arg("sink") = 0, py::arg("out_scale") = 1.f,
-     py::arg("o_stride") = 0);
+     py::arg("o_stride") = 0, py::arg("slopes") = 0);
   m.def("gemm_bt", [](u A, long lda, u B, long ldb, u C, long ldc, u bias, u residual, long ldr, int M, int N, int K,
                       int epilogue, int out_f32, u row_group, u q_group, u allow, int allow_words, u s, int b_rows,
                       int b_group) {

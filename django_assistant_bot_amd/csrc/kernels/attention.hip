@@ -70,6 +70,7 @@ struct FlashParams {
   int window, chunk;
   const float* sink;
   float out_scale;
+  const float* slopes;  // slopes[h] times the distance i - j is taken off the score of key j (null: none)
 };
 
 // first key position that the query at position i sees
@@ -97,7 +98,8 @@ constexpr float kDeferLog2 = 8.f;
 // SIMD, no spills) instead of 112 (4).
 // WIN (causal): sliding window and softmax sink (FlashParams).  Key tiles before the block's first visible
 // key are skipped; the running maximum starts at the sink, whose own term is then 1.
-template <int D, bool CAUSAL, bool PAGED, int NW, int QT, int MINW = 0, bool WIN = false>
+// SLOPE: scores fall with distance (FlashParams).
+template <int D, bool CAUSAL, bool PAGED, int NW, int QT, int MINW = 0, bool WIN = false, bool SLOPE = false>
 __global__ __launch_bounds__(64 * NW, MINW ? MINW : ((QT == 2 && NW == 4) ? 2 : 1)) void flash_fwd_kernel(FlashParams p) {
   constexpr int KT = 64;
   constexpr int NT = 64 * NW;
@@ -217,6 +219,7 @@ __global__ __launch_bounds__(64 * NW, MINW ? MINW : ((QT == 2 && NW == 4) ? 2 : 
     }
   }
 
+  const float slope = SLOPE ? p.slopes[h] * 1.4426950408889634f : 0.f;
   if (n_tiles > kt0) {
     load_tile(kt0);
     store_tile();
@@ -249,6 +252,7 @@ __global__ __launch_bounds__(64 * NW, MINW ? MINW : ((QT == 2 && NW == 4) ? 2 : 
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           float v = s[qt][m][r] * p.scale_log2;
+          if (SLOPE) v = fmaf(slope, (float)(kt * KT + 4 * g - q_pos[qt]) + (float)(16 * m + r), v);
           if (need_mask) {
             const int key = kt * KT + 16 * m + 4 * g + r;
             if (key >= kv_len || (CAUSAL && key > q_pos[qt]) || (WIN && key < lo[qt])) v = kNegInf;
@@ -1539,6 +1543,7 @@ struct DecodeParams {
   // holds the chunk's first key.  sink (or null): one more score in head h's denominator
   int chunk;
   const float* sink;
+  const float* slopes;  // SLOPE: slopes[h] times the distance is taken off a key's score
   float out_scale;
   long o_stride_tok;
   L3Warm warm;  // optional: the next projections' weights, warmed into L3 by appended workgroups
@@ -1555,7 +1560,7 @@ struct DecodeParams {
 // the first copy.  At batch 1 - 8 a workgroup's waves walk their sub-tiles back to back with the
 // whole GPU otherwise idle: one copy round trip per sub-tile was the critical path.  128 KB of LDS:
 // one workgroup per CU, which small batches never fill anyway.
-template <int D, bool KV_NT, bool DMA = false, int NSLOT = 1>
+template <int D, bool KV_NT, bool DMA = false, int NSLOT = 1, bool SLOPE = false>
 __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(DecodeParams p, int total_items) {
   static_assert(NSLOT == 1 || (NSLOT == 2 && DMA), "two slots: DMA staging only");
   // appended workgroups (small batches leave most CUs idle during this latency-bound launch): warm
@@ -1658,6 +1663,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
 #pragma unroll
     for (int t = 0; t < NTD; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m_run = -1e30f, l_run = 0.f;
+    const float slope = SLOPE ? p.slopes[hk * G + min(li, G - 1)] * 1.4426950408889634f : 0.f;
 
     auto compute = [&](const int k0) {
       __builtin_amdgcn_s_waitcnt(0xc07f);  // lgkmcnt(0): this wave's LDS writes landed
@@ -1679,6 +1685,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
         for (int r = 0; r < 4; ++r) {
           const int key = k0 + 16 * m + 4 * g + r;
           float v = s[m][r] * p.scale_log2;
+          if (SLOPE) v = fmaf(slope, (float)(key - (ctx - 1)), v);
           if (key >= k_end || key < k_lo) v = kNegInf;
           s[m][r] = v;
           mx = fmaxf(mx, v);
@@ -1888,7 +1895,7 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
                     long o_stride_head, const int* cu_q, const int* cu_k, const int* ctx_k, int batch,
                     int max_seqlen_q, int Hq, int Hkv, int D, int causal, int paged, float scale, hipStream_t s,
                     const int* rope_pos, const void* rope_cs, int window, const float* sink, int chunk,
-                    float out_scale) {
+                    float out_scale, const float* slopes) {
   if (batch <= 0 || max_seqlen_q <= 0) return 0;
   if (Hq % Hkv || (paged && block_size % 64)) return hipErrorInvalidValue;
   FlashParams prm{};
@@ -1916,8 +1923,9 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
   prm.Hkv = Hkv;
   prm.scale_log2 = scale * 1.4426950408889634f;
   prm.pairs_per_wg = 1;
-  if (window > 0 || chunk > 0 || sink || D == 256 || out_scale != 1.f) {  // windowed / chunked / sink form: 16-query sub-tiles
-    if (!causal || rope_cs || (window > 0 && chunk > 0)) return hipErrorInvalidValue;
+  if (window > 0 || chunk > 0 || sink || slopes || D == 256 || out_scale != 1.f) {  // windowed / chunked / sink form: 16-query sub-tiles
+    if (!causal || rope_cs || (window > 0 && chunk > 0) || (slopes && !paged)) return hipErrorInvalidValue;
+    prm.slopes = slopes;
     prm.window = window;
     prm.chunk = chunk;
     prm.sink = sink;
@@ -1931,7 +1939,12 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
     else if (D == 256) hipLaunchKernelGGL((flash_fwd_kernel<256, true, P, 8, 1, 0, true>), gw, dim3(512), 0, s, prm);    \
     else return hipErrorInvalidValue;                                                                                    \
   } while (0)
-    if (paged) DAB_FLASH_WIN(true);
+    if (slopes) {
+      if (D == 64) hipLaunchKernelGGL((flash_fwd_kernel<64, true, true, 4, 1, 0, true, true>), gw, dim3(256), 0, s, prm);
+      else if (D == 128) hipLaunchKernelGGL((flash_fwd_kernel<128, true, true, 8, 1, 0, true, true>), gw, dim3(512), 0, s, prm);
+      else if (D == 256) hipLaunchKernelGGL((flash_fwd_kernel<256, true, true, 8, 1, 0, true, true>), gw, dim3(512), 0, s, prm);
+      else return hipErrorInvalidValue;
+    } else if (paged) DAB_FLASH_WIN(true);
     else DAB_FLASH_WIN(false);
 #undef DAB_FLASH_WIN
     return hipGetLastError();
@@ -2067,7 +2080,8 @@ int paged_decode_attention(const void* q, const void* k_cache, const void* v_cac
                            int max_blocks, int block_size, const int* ctx_lens, void* out, float* part_o,
                            float* part_m, float* part_l, int* counters, int batch, int Hq, int Hkv, int D,
                            int part_size, int max_parts, float scale, hipStream_t s, const int* order,
-                           const L3Warm* warm, int chunk, const float* sink, float out_scale, long o_stride_tok) {
+                           const L3Warm* warm, int chunk, const float* sink, float out_scale, long o_stride_tok,
+                           const float* slopes) {
   if (batch <= 0) return 0;
   if (Hq % Hkv || Hq / Hkv > 16 || part_size % 128 || max_parts < 1 || block_size % 32) return hipErrorInvalidValue;
   if (max_parts > 1 && !counters) return hipErrorInvalidValue;
@@ -2093,6 +2107,7 @@ int paged_decode_attention(const void* q, const void* k_cache, const void* v_cac
   prm.scale_log2 = scale * 1.4426950408889634f;
   prm.chunk = chunk;
   prm.sink = sink;
+  prm.slopes = slopes;
   prm.out_scale = out_scale;
   prm.o_stride_tok = o_stride_tok ? o_stride_tok : (long)Hq * D;
   prm.warm = warm ? *warm : L3Warm{{nullptr, nullptr}, {0, 0}, 0};
@@ -2108,11 +2123,17 @@ int paged_decode_attention(const void* q, const void* k_cache, const void* v_cac
   if (D == 128) {
     // small batches: two LDS slots per wave (at batch 128 the one-slot kernel's two workgroups per CU
     // are 2.8 % faster per step: 7.44 vs 7.65 ms, profiles/low_load_latency.md)
-    if (batch * Hkv <= 64 && part_size <= 64 * 4 * 32)
-      hipLaunchKernelGGL((paged_decode_kernel<128, true, true, 2>), grid, dim3(256), 0, s, prm, total_items);
+    const bool two = batch * Hkv <= 64 && part_size <= 64 * 4 * 32;
+    if (two && slopes)
+      hipLaunchKernelGGL((paged_decode_kernel<128, true, true, 2, true>), grid, dim3(256), 0, s, prm, total_items);
+    else if (two) hipLaunchKernelGGL((paged_decode_kernel<128, true, true, 2>), grid, dim3(256), 0, s, prm, total_items);
+    else if (slopes)
+      hipLaunchKernelGGL((paged_decode_kernel<128, true, true, 1, true>), grid, dim3(256), 0, s, prm, total_items);
     else hipLaunchKernelGGL((paged_decode_kernel<128, true, true>), grid, dim3(256), 0, s, prm, total_items);
   } else if (D == 64) {
-    hipLaunchKernelGGL((paged_decode_kernel<64, true>), grid, dim3(256), 0, s, prm, total_items);
+    if (slopes)
+      hipLaunchKernelGGL((paged_decode_kernel<64, true, false, 1, true>), grid, dim3(256), 0, s, prm, total_items);
+    else hipLaunchKernelGGL((paged_decode_kernel<64, true>), grid, dim3(256), 0, s, prm, total_items);
   } else {
     return hipErrorInvalidValue;
   }

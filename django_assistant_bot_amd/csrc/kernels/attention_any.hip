@@ -2,7 +2,8 @@
 // 32-bit mode and of sizes that the MFMA kernels do not tile.  One wave per (token, query head), 64 keys a
 // step with a lane per key for the scores and a lane per value column for the sum; online softmax in fp32.
 // ``chunk`` > 0: query i sees keys of its own chunk only, floor(i / chunk) chunk .. i.  ``sink`` (or null)
-// joins head h's denominator as one more score.
+// joins head h's denominator as one more score.  ``slopes`` (or null): slopes[h] times the distance i - j is taken off the
+// score of key j.
 #include "launchers.h"
 #include "proj.h"
 
@@ -19,6 +20,7 @@ struct AnyAttn {
   int B, H, G, D, chunk;
   float scale, out_scale;
   const float* sink;
+  const float* slopes;
   void* out;
   long o_tok;
 };
@@ -52,6 +54,7 @@ __global__ __launch_bounds__(64) void any_attention_kernel(AnyAttn p) {
     m = p.sink[h];
     l = 1.f;
   }
+  const float slope = p.slopes ? p.slopes[h] : 0.f;
   const int first = p.chunk > 0 ? pos / p.chunk * p.chunk : 0;
   for (int k0 = first; k0 <= pos; k0 += 64) {
     const int key = k0 + lane, n = min(64, pos - k0 + 1);
@@ -66,6 +69,7 @@ __global__ __launch_bounds__(64) void any_attention_kernel(AnyAttn p) {
       s = fmaf(qs[d], e.x, s);
       s = fmaf(qs[d + 1], e.y, s);
     }
+    s -= slope * (float)(pos - key);
     if (key > pos) s = -__builtin_huge_valf();
     const float mn = fmaxf(m, wave_max(s));
     const float a = __expf(m - mn), w = __expf(s - mn);
@@ -91,10 +95,10 @@ __global__ __launch_bounds__(64) void any_attention_kernel(AnyAttn p) {
 
 int any_attention(const void* q, const void* kc, const void* vc, int f32, const int* bt, int max_blocks, int bs,
                   const int* cu, const int* ctx, int B, int T, int H, int G, int D, int chunk, float scale,
-                  const float* sink, void* out, long o_tok, float out_scale, hipStream_t s) {
+                  const float* sink, const float* slopes, void* out, long o_tok, float out_scale, hipStream_t s) {
   if (T <= 0) return 0;
   if (B < 1 || H < 1 || G < 1 || H % G || D < 2 || D % 2 || D > 1024 || H > 65535 || chunk < 0 || bs < 1) return hipErrorInvalidValue;
-  AnyAttn p{q, kc, vc, bt, max_blocks, bs, cu, ctx, B, H, G, D, chunk, scale, out_scale, sink, out, o_tok};
+  AnyAttn p{q, kc, vc, bt, max_blocks, bs, cu, ctx, B, H, G, D, chunk, scale, out_scale, sink, slopes, out, o_tok};
   const dim3 grid(T, H);
   const size_t lds = (D + 128) * sizeof(float);
 #define ANY_NV(AT)                                                                                     \

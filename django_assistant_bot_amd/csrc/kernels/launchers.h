@@ -57,28 +57,84 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
                     long o_stride_head, const int* cu_q, const int* cu_k, const int* ctx_k, int batch,
                     int max_seqlen_q, int Hq, int Hkv, int D, int causal, int paged, float scale, hipStream_t s,
                     const int* rope_pos = nullptr, const void* rope_cs = nullptr, int window = 0,
-                    const float* sink = nullptr, int chunk = 0, float out_scale = 1.f);
+                    const float* sink = nullptr, int chunk = 0, float out_scale = 1.f, const float* slopes = nullptr);
 int paged_decode_attention(const void* q, const void* k_cache, const void* v_cache, const int* block_tables,
                            int max_blocks, int block_size, const int* ctx_lens, void* out, float* part_o,
                            float* part_m, float* part_l, int* counters, int batch, int Hq, int Hkv, int D,
                            int part_size, int max_parts, float scale, hipStream_t s,
                            const int* order = nullptr, const L3Warm* warm = nullptr, int chunk = 0,
-                           const float* sink = nullptr, float out_scale = 1.f, long o_stride_tok = 0);
+                           const float* sink = nullptr, float out_scale = 1.f, long o_stride_tok = 0,
+                           const float* slopes = nullptr);
 
 // attention_any.hip (any head width, bf16 or fp32, paged)
 int any_attention(const void* q, const void* kc, const void* vc, int f32, const int* bt, int max_blocks, int bs,
                   const int* cu, const int* ctx, int B, int T, int H, int G, int D, int chunk, float scale,
-                  const float* sink, void* out, long o_tok, float out_scale, hipStream_t s);
+                  const float* sink, const float* slopes, void* out, long o_tok, float out_scale, hipStream_t s);
 
 // rms_stream.hip (RMS norms around an fp32 residual stream; rotary positions and q / k norm before attention)
 int rms_residual(float* x, void* h, int act_f32, Proj y, const float* bias, const void* pairs, int top, const int* ids,
                  const void* table, int table_f32, const float* post, const float* gain, int n_true, float eps, int rows,
                  int cols, int fresh, hipStream_t s);
-int sigmoid_gate(Proj y, int col0, void* x, long ldx, int act_f32, int n, int T, hipStream_t s);
+int sigmoid_gate(Proj y, int col0, int per, void* x, long ldx, int act_f32, int n, int T, hipStream_t s);
 int softcap(Proj y, float cap, float* out, int n, int T, hipStream_t s);
 int qk_rope_write(Proj y, int col0, int H, int G, int D, int dim, int rot, const double* freq, float eps, int norm,
                   const int* positions, const int64_t* slots, void* q, void* kc, void* vc, int act_f32, int bs, int T,
                   hipStream_t s);
+
+// gated_stream.hip (sublayers whose result passes a gate and a norm, sums over depth, PolyNorm)
+struct GatedResidual {
+  const float* src;          // the stream before (null: zeros)
+  float* x;                  // the stream after
+  void* h;                   // x, or with ``gain`` its norm, in the activation type
+  Proj y;                    // sublayer output (p null: none); row ids[row] with ``ids``
+  const int* ids;
+  const void* pairs;         // [rows * top, cols] expert rows or null; index >= experts: weight * src instead
+  const int* idx;
+  const float* wt;
+  int top, experts;
+  Proj g;                    // gate columns g_col.. (p null: none), their bias
+  int g_col;
+  const float* g_bias;
+  const float* post;         // gain of the norm of what is added
+  float* depth;              // n > 0: results 0 .. n - 1, depth_stride apart; keep: x becomes result n
+  const float* weights;      // [n + 1]
+  long depth_stride;
+  int n, keep;
+  const float* gain;         // or null
+  float inv_n, eps;
+  int cols;
+};
+int gated_residual(GatedResidual p, int act_f32, int rows, hipStream_t s);
+int poly_norm(Proj y, int n, int cols, float a, float b, float c, float e, float eps, void* out, int act_f32, int T, hipStream_t s);
+
+// attn_inputs.hip (input projection -> bias, convolution, norm, rotation, temperature, value mix -> q rows and paged cache)
+struct AttnInputs {
+  Proj y;
+  int col0, H, G, D;         // q, k, v heads of D columns from col0
+  float inv_q, inv_k, eps;   // 1 / elements of a norm's mean
+  int whole;                 // 1: one norm over all q heads and one over all k heads
+  const float* gain;         // [(H + G) D]
+  const float* bias;         // [(H + 2 G) D] or null
+  const float* conv;         // [taps, (H + 2 G) D] or null
+  int taps;
+  const double* turns;       // turns per position of the rot / 2 pairs
+  int rot;
+  float rot_mul;             // factor on cosine and sine
+  float t_coef;              // query temperature 1 + t_coef ln(floor((p + 1) / t_every) + 1)
+  int t_every;
+  const int* positions;
+  const int64_t* slots;
+  void *q, *kc, *vc;         // [T, H, D], caches [blocks, G, bs, D]
+  int bs;
+  void* ring;                // [slots, taps, (H + 2 G) D]
+  const int* slot;           // state slot of every portion / decoded token
+  const int* cu;             // portions, or null: decoded tokens from row0
+  int row0;
+  void* first;               // [T, G, first_w]: mix 1: the values are written here; 2: v += lam (first - v)
+  int first_w, mix;
+  float lam;
+};
+int attn_inputs(AttnInputs p, int act_f32, int rows, int max_q, hipStream_t s);
 
 // recurrent.hip (matrix-state recurrences: gated delta rule and state-space duality)
 struct RecurrentShape {
@@ -127,8 +183,11 @@ int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_
                    void* out, hipStream_t s);
 
 // moe.hip
-// sigmoid 0: softmax scores, weights over their sum; 1: sigmoid scores as they are
-int moe_route(Proj z, int col0, int E, int top, float scale, int sigmoid, int* idx, float* wt, int T, hipStream_t s);
+// scores 0: softmax, weights over their sum; 1: sigmoid scores as they are;
+// 2: softmax scores as they are; correction [E] (or null) joins a score where the experts are chosen, not in its weight
+int moe_route(Proj z, int col0, int E, int top, float scale, int scores, const float* correction, int* idx, float* wt, int T,
+              hipStream_t s);
+// pairs whose index is E or more (identity experts) come last in perm and are in no tile
 int moe_plan(const int* idx, int P, int E, int bm, int* perm, void* tiles, int max_tiles, hipStream_t s);
 int shared_glu(Proj y, int col0, int F, Proj z, int sg_col, void* out, long ldo, int act_f32, int T, hipStream_t s);
 

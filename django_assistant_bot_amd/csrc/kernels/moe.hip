@@ -1,10 +1,11 @@
 // Mixture of experts: routing, the row plan of the grouped GEMMs, and the shared expert's gated activation.
 //
 //   route        fp32 logits -> softmax over all experts -> the ``top`` largest, weights over their sum (+ 1e-20)
-//                times ``scale``; or (sigmoid) the scores' sigmoids, their ``top`` largest as they are times ``scale``;
-//                one wave per token
+//                times ``scale``; or (sigmoid, raw softmax) the ``top`` largest as they are times ``scale``.  A correction
+//                per expert joins the score where the experts are chosen, not in the weight; one wave per token
 //   plan         (token, expert) pairs grouped by expert: perm[sorted position] = pair, and the row tiles of
-//                the grouped GEMM, each {expert, first sorted position, rows}; one workgroup
+//                the grouped GEMM, each {expert, first sorted position, rows}; one workgroup.  Pairs of identity experts
+//                (index >= E) come last and are in no tile
 //   shared_glu   silu(gate) up sigmoid(w_sg h) of the expert that every token runs
 //
 // Which rows an expert gets does not change a row's result, so the order within an expert is left to the
@@ -15,11 +16,12 @@
 namespace dab {
 
 template <typename GT, int EI>
-__global__ __launch_bounds__(256) void moe_route_kernel(Proj z, int col0, int E, int top, float scale, int sigmoid, int* idx,
-                                                        float* wt, int T) {
+__global__ __launch_bounds__(256) void moe_route_kernel(Proj z, int col0, int E, int top, float scale, int scores,
+                                                        const float* correction, int* idx, float* wt, int T) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= T) return;
-  float s[EI];
+  const bool sigmoid = scores == 1;
+  float s[EI], w[EI];  // scores as experts are chosen by them, as weights
   float mx = -__builtin_huge_valf();
 #pragma unroll
   for (int i = 0; i < EI; ++i) {
@@ -36,63 +38,71 @@ __global__ __launch_bounds__(256) void moe_route_kernel(Proj z, int col0, int E,
   }
   sum = wave_sum(sum);
 #pragma unroll
-  for (int i = 0; i < EI; ++i) s[i] = lane + 64 * i < E ? (sigmoid ? s[i] : s[i] / sum) : -1.f;
+  for (int i = 0; i < EI; ++i) {
+    const int e = lane + 64 * i;
+    w[i] = sigmoid ? s[i] : s[i] / sum;
+    s[i] = e < E ? w[i] + (correction ? correction[e] : 0.f) : -__builtin_huge_valf();
+  }
   float total = 0.f, mine = 0.f;  // lane k keeps the k-th choice
   int mine_e = 0;
   for (int k = 0; k < top; ++k) {
-    float best = -2.f;
-    int be = 0;
+    float best = -__builtin_huge_valf(), bw = 0.f;
+    int be = E;  // (behind every expert: a lane without one left)
 #pragma unroll
     for (int i = 0; i < EI; ++i)
       if (s[i] > best) {
         best = s[i];
+        bw = w[i];
         be = lane + 64 * i;
       }
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) {
       const float ob = __shfl_xor(best, o, 64);
       const int oe = __shfl_xor(be, o, 64);
+      const float ow = __shfl_xor(bw, o, 64);
       if (ob > best || (ob == best && oe < be)) {
         best = ob;
         be = oe;
+        bw = ow;
       }
     }
-    total += best;
+    total += bw;
     if (lane == k) {
-      mine = best;
+      mine = bw;
       mine_e = be;
     }
 #pragma unroll
     for (int i = 0; i < EI; ++i)
-      if (be == lane + 64 * i) s[i] = -1.f;
+      if (be == lane + 64 * i) s[i] = -__builtin_huge_valf();
   }
   if (lane < top) {
     idx[(size_t)t * top + lane] = mine_e;
-    wt[(size_t)t * top + lane] = (sigmoid ? mine : mine / (total + 1e-20f)) * scale;
+    wt[(size_t)t * top + lane] = (scores ? mine : mine / (total + 1e-20f)) * scale;
   }
 }
 
-int moe_route(Proj z, int col0, int E, int top, float scale, int sigmoid, int* idx, float* wt, int T, hipStream_t s) {
+int moe_route(Proj z, int col0, int E, int top, float scale, int scores, const float* correction, int* idx, float* wt, int T,
+              hipStream_t s) {
   if (T <= 0) return 0;
-  if (E < 1 || E > 1024 || top < 1 || top > 64 || top > E || !z.f32 || z.S < 1) return hipErrorInvalidValue;
+  if (E < 1 || E > 1024 || top < 1 || top > 64 || top > E || !z.f32 || z.S < 1 || scores < 0 || scores > 2) return hipErrorInvalidValue;
   const dim3 grid((T + 3) / 4);
-  if (E <= 64) hipLaunchKernelGGL((moe_route_kernel<float, 1>), grid, dim3(256), 0, s, z, col0, E, top, scale, sigmoid, idx, wt,
-                                  T);
-  else if (E <= 256) hipLaunchKernelGGL((moe_route_kernel<float, 4>), grid, dim3(256), 0, s, z, col0, E, top, scale, sigmoid, idx, wt,
-                                  T);
-  else hipLaunchKernelGGL((moe_route_kernel<float, 16>), grid, dim3(256), 0, s, z, col0, E, top, scale, sigmoid, idx, wt,
-                                  T);
+  if (E <= 64) hipLaunchKernelGGL((moe_route_kernel<float, 1>), grid, dim3(256), 0, s, z, col0, E, top, scale, scores,
+                                  correction, idx, wt, T);
+  else if (E <= 256) hipLaunchKernelGGL((moe_route_kernel<float, 4>), grid, dim3(256), 0, s, z, col0, E, top, scale, scores,
+                                  correction, idx, wt, T);
+  else hipLaunchKernelGGL((moe_route_kernel<float, 16>), grid, dim3(256), 0, s, z, col0, E, top, scale, scores,
+                                  correction, idx, wt, T);
   return hipGetLastError();
 }
 
 // tiles[i] = {expert, first sorted position, rows, 0}; rows 0 past the last tile
 __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ idx, int P, int E, int bm, int* perm,
                                                         int4* tiles, int max_tiles) {
-  __shared__ int cnt[1024], off[1025], tof[1025];
+  __shared__ int cnt[1025], off[1025], tof[1025];  // entry E: identity experts
   const int tid = threadIdx.x;
-  for (int e = tid; e < E; e += 1024) cnt[e] = 0;
+  for (int e = tid; e <= E; e += 1024) cnt[e] = 0;
   __syncthreads();
-  for (int i = tid; i < P; i += 1024) atomicAdd(&cnt[idx[i]], 1);
+  for (int i = tid; i < P; i += 1024) atomicAdd(&cnt[min(idx[i], E)], 1);
   __syncthreads();
   if (tid < 64) {  // prefix sums of rows and tiles, 64 experts a step
     int base = 0, tbase = 0;
@@ -115,7 +125,10 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
       base += __shfl(a, 63, 64);
       tbase += __shfl(b, 63, 64);
     }
-    if (tid == 0) tof[E] = tbase;
+    if (tid == 0) {
+      off[E] = base;
+      tof[E] = tbase;
+    }
   }
   __syncthreads();
   for (int e = tid; e < E; e += 1024) {
@@ -125,7 +138,7 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
   }
   for (int t = tof[E] + tid; t < max_tiles; t += 1024) tiles[t] = make_int4(0, 0, 0, 0);
   __syncthreads();
-  for (int i = tid; i < P; i += 1024) perm[atomicAdd(&off[idx[i]], 1)] = i;
+  for (int i = tid; i < P; i += 1024) perm[atomicAdd(&off[min(idx[i], E)], 1)] = i;
 }
 
 int moe_plan(const int* idx, int P, int E, int bm, int* perm, void* tiles, int max_tiles, hipStream_t s) {

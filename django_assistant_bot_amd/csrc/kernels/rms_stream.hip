@@ -5,7 +5,7 @@
 //                   [+ table[id]];  h = x / rms(x) * gain: everything between two layers in one pass.  With ``post``,
 //                   output + bias + expert rows pass an RMS norm of their own before they are added; without ``gain``
 //                   h is x as it is
-//   sigmoid_gate    x *= sigmoid(columns of a projection)
+//   sigmoid_gate    x *= sigmoid(columns of a projection), a column for every one or (per > 1) for ``per`` of x
 //   softcap         cap tanh(y / cap) of the logits
 //   qk_rope_write   [q | k | v] columns of a projection -> interleaved rotary positions on q and k, weightless
 //                   RMS norm per head, q rows out, k / v into the paged cache
@@ -158,26 +158,32 @@ int rms_residual(float* x, void* h, int act_f32, Proj y, const float* bias, cons
 // ----------------------------------------------------------------------------------------------
 
 template <typename PT, typename AT>
-__global__ __launch_bounds__(256) void sigmoid_gate_kernel(Proj y, int col0, AT* x, long ldx, int n) {
+__global__ __launch_bounds__(256) void sigmoid_gate_kernel(Proj y, int col0, int per, AT* x, long ldx, int n) {
   const int c = (blockIdx.x * 256 + threadIdx.x) * 8, t = blockIdx.y;
   if (c >= n) return;
   float g[8], v[8];
-  proj8<PT>(y, t, col0 + c, g);
+  if (per > 1) {
+    g[0] = proj_f32<PT>(y, t, col0 + c / per);
+#pragma unroll
+    for (int j = 1; j < 8; ++j) g[j] = g[0];
+  } else {
+    proj8<PT>(y, t, col0 + c, g);
+  }
   ElemIO<AT>::load8(x + (size_t)t * ldx + c, v);
 #pragma unroll
   for (int j = 0; j < 8; ++j) v[j] /= 1.f + __expf(-g[j]);
   ElemIO<AT>::store8(x + (size_t)t * ldx + c, v);
 }
 
-int sigmoid_gate(Proj y, int col0, void* x, long ldx, int act_f32, int n, int T, hipStream_t s) {
+int sigmoid_gate(Proj y, int col0, int per, void* x, long ldx, int act_f32, int n, int T, hipStream_t s) {
   if (T <= 0) return 0;
-  if (n < 8 || n % 8 || col0 % 8 || y.ld % 8 || y.slab % 8 || ldx % 8 || y.S < 1 || T > (1 << 20)) return hipErrorInvalidValue;
+  if (n < 8 || n % 8 || (per > 1 ? per % 8 : per != 1 || col0 % 8) || y.ld % 8 || y.slab % 8 || ldx % 8 || y.S < 1 || T > (1 << 20)) return hipErrorInvalidValue;
   for (int r = 0; r < T; r += 32768) {
     Proj yr = y;
     yr.p = (const char*)y.p + (size_t)r * y.ld * (y.f32 ? 4 : 2);
     const dim3 grid((n / 8 + 255) / 256, T - r < 32768 ? T - r : 32768);
 #define SGATE_L(PT, AT) \
-  hipLaunchKernelGGL((sigmoid_gate_kernel<PT, AT>), grid, dim3(256), 0, s, yr, col0, (AT*)x + (size_t)r * ldx, ldx, n)
+  hipLaunchKernelGGL((sigmoid_gate_kernel<PT, AT>), grid, dim3(256), 0, s, yr, col0, per, (AT*)x + (size_t)r * ldx, ldx, n)
     DAB_PROJ_DISPATCH(y, act_f32, SGATE_L);
 #undef SGATE_L
   }

@@ -31,7 +31,7 @@ import torch
 
 from .. import ops
 from ..models import AttnMeta, decoder_config, decoder_family
-from ..models.configs import DecoderConfig, VugotarConfig, VumuvikConfig, VunelixConfig
+from ..models.configs import BizetarConfig, DecoderConfig, VugotarConfig, VumuvikConfig, VunelixConfig
 from ..ops._lib import native
 from ..utils import trace
 from .tokenizer import Tokenizer
@@ -106,7 +106,7 @@ def _bucket_sizes(max_batch):
 
 
 class LLMEngine:
-    def __init__(self, model: str | DecoderConfig | VumuvikConfig | VugotarConfig | VunelixConfig = "llama-3-8b",
+    def __init__(self, model: str | DecoderConfig | VumuvikConfig | VugotarConfig | VunelixConfig | BizetarConfig = "llama-3-8b",
                  device=None, weights: dict | None = None,
                  checkpoint: str | None = None, seed: int = 0, max_batch: int = 256, block_size: int = 64,
                  max_model_len: int | None = None, kv_cache_gb: float | None = None, num_blocks: int | None = None,
@@ -171,6 +171,7 @@ class LLMEngine:
                 num_blocks = int(max(0, kv_cache_gb * (1 << 30) - self.model.state_bytes(self.state_slots + 1)) // per_block)
             elif self.is_gpu:
                 free, _ = torch.cuda.mem_get_info(self.device)
+                free -= self.model.step_bytes(max_prefill_tokens)
                 num_blocks = int(max(0, free * kv_memory_fraction - self.model.state_bytes(self.state_slots + 1)) // per_block)
             else:
                 num_blocks = 4 * self.max_blocks_per_seq

@@ -295,6 +295,47 @@ class SelectiveMixer:
 
 
 @dataclass(frozen=True)
+class QueryTemp:
+    """Queries at position p are multiplied by 1 + coef ln(floor((p + 1) / every) + 1)."""
+
+    coef: float
+    every: int
+
+
+@dataclass(frozen=True)
+class SinkMixer:
+    """Softmax attention over per-head keys and values, with a learned sink per head in the denominator and a sigmoid gate on
+    the output.  What positions do is said by ``rot`` (rotation), ``temp`` (query temperature) and ``slopes`` (every head
+    takes slope * distance off its scores)."""
+
+    heads: int
+    kv_heads: int
+    dim: int  # query / key width of a head
+    vdim: int
+    scale: float
+    norm: str = "head"  # RMS norm of q and k, with weights: "head" (each head, shared weights) or "whole" (all rows at once)
+    gate: str = "element"  # output gate: a number per "element" or per "head"
+    bias: bool = False  # q, k and v have biases
+    conv: int = 0  # taps of the short causal convolution on q, k and v (0: none)
+    rot: Rotary | None = None
+    temp: QueryTemp | None = None
+    slopes: bool = False
+    v_mix: bool = False  # values are mixed with those of the first layer that says so
+
+    def padded_head(self) -> int:
+        """Common padded width of the query / key and value heads."""
+        d = max(self.dim, self.vdim)
+        return next((p for p in (64, 128, 256) if d <= p), _up(d, 64))
+
+
+@dataclass(frozen=True)
+class PolyMlp:
+    """Ungated MLP with PolyNorm: a combination of the normalised first three powers of the hidden values."""
+
+    ff: int
+
+
+@dataclass(frozen=True)
 class DenseMlp:
     """Gated MLP (in a Vugotar with biases on all three projections)."""
 
@@ -305,8 +346,10 @@ class DenseMlp:
 @dataclass(frozen=True)
 class MoeMlp:
     """``top`` of ``experts`` SwiGLUs per token plus, with ``shared``, one that every token runs (in a Vugotar behind a
-    sigmoid gate).  ``scores``: of the router, "softmax" (weights over their sum) or "sigmoid" (weights as they are);
-    ``weigh``: what the weight multiplies, the expert's "output" or its "input"."""
+    sigmoid gate).  ``scores``: of the router, "softmax" (weights over their sum), "softmax_raw" or "sigmoid" (weights as they
+    are); ``weigh``: what the weight multiplies, the expert's "output" or its "input".  ``correction``: a number per expert
+    joins its score where the experts are chosen, not in the weight.  ``identity``: further router outputs whose expert is the
+    layer's input itself."""
 
     experts: int
     top: int
@@ -315,6 +358,18 @@ class MoeMlp:
     shared: int | None = None
     scores: str = "softmax"
     weigh: str = "output"
+    correction: bool = False
+    identity: int = 0
+
+    @property
+    def outputs(self) -> int:
+        """Router outputs."""
+        return self.experts + self.identity
+
+
+def _check_moe(where: str, f, max_experts: int = 1024, max_top: int = 64) -> None:
+    if isinstance(f, MoeMlp) and (not 1 <= f.top <= min(f.outputs, max_top) or f.outputs > max_experts):
+        raise ValueError(f"{where}: experts up to {max_experts}, of which up to {max_top} per token")
 
 
 def loop_runs(layers: int, loop: tuple | None) -> list:
@@ -337,10 +392,10 @@ def _check_loop(name: str, layers: int, loop: tuple | None) -> None:
 @dataclass(frozen=True)
 class HybridLayer:
     """A mixer and a feed-forward.  Vugotar: x + mixer(norm(x)) + mlp(norm(x)), one norm that both read.  Vunelix: a norm
-    before and after each of the two."""
+    before and after each of the two.  Bizetar: a gate and a norm after each."""
 
-    mixer: ParallelMixer | Mamba2Mixer | SelectiveMixer | LatentMixer
-    mlp: DenseMlp | MoeMlp | None = None
+    mixer: ParallelMixer | Mamba2Mixer | SelectiveMixer | LatentMixer | SinkMixer
+    mlp: DenseMlp | MoeMlp | PolyMlp | None = None
 
 
 @dataclass(frozen=True)
@@ -379,9 +434,7 @@ class VugotarConfig:
                 rows, taps = m.state, m.conv
             if not 1 <= rows <= self.MAX_STATE_ROWS or not 1 <= taps <= self.MAX_TAPS:
                 raise ValueError(f"{where}: state rows up to {self.MAX_STATE_ROWS}, taps up to {self.MAX_TAPS}")
-            if isinstance(f, MoeMlp) and not 1 <= f.top <= min(f.experts, self.MAX_TOP) or (
-                    isinstance(f, MoeMlp) and f.experts > self.MAX_EXPERTS):
-                raise ValueError(f"{where}: experts up to {self.MAX_EXPERTS}, of which up to {self.MAX_TOP} per token")
+            _check_moe(where, f, self.MAX_EXPERTS, self.MAX_TOP)
         _check_loop(self.name, len(self.blocks), self.loop)
 
     @property
@@ -476,9 +529,7 @@ class VunelixConfig:
                     raise ValueError(f"{where}: rotated dimensions come in pairs")
                 if m.padded_row() > self.MAX_ROW:
                     raise ValueError(f"{where}: latent and rotated key up to {self.MAX_ROW} wide")
-            if isinstance(f, MoeMlp) and not 1 <= f.top <= min(f.experts, self.MAX_TOP) or (
-                    isinstance(f, MoeMlp) and f.experts > self.MAX_EXPERTS):
-                raise ValueError(f"{where}: experts up to {self.MAX_EXPERTS}, of which up to {self.MAX_TOP} per token")
+            _check_moe(where, f, self.MAX_EXPERTS, self.MAX_TOP)
         _check_loop(self.name, len(self.blocks), self.loop)
 
     @property
@@ -532,6 +583,92 @@ def vunelix_uniform(name: str, layers: int, vocab_size: int, hidden: int, mamba:
     cycle = (HybridLayer(mamba, dense), HybridLayer(latent, moe or dense), HybridLayer(latent, moe or dense))
     return VunelixConfig(name, vocab_size, hidden, tuple(cycle[i % 3] for i in range(layers)), loop=loop,
                          softcap=kw.pop("softcap", 30.0), **kw)
+
+
+# ------------------------------------------------------------------ depth-averaged decoders (Bizetar)
+
+
+@dataclass(frozen=True)
+class BizetarConfig:
+    """Bizetar decoder: softmax attention with sinks (distance slopes and query temperature, or short convolutions and rotary
+    positions), PolyNorm MLPs and experts with identity experts.  A sublayer reads the stream itself; its result passes a
+    sigmoid gate of the same input and a norm before it is added.  After every layer the stream becomes a weighted sum of the
+    embedding and all layers' results; from the first such layer on, values are mixed with that layer's."""
+
+    name: str
+    vocab_size: int
+    hidden: int
+    blocks: tuple  # of HybridLayer
+    eps: float = 1e-5
+    max_position: int = 1 << 20  # no positional table: only the cache bounds a sequence
+    default_model_len: int = 8192
+    bos_id: int = 0
+    eos_ids: tuple = ()
+
+    MAX_TAPS, MAX_HEAD, MAX_WIDTH, MAX_FF = 16, 1024, 16384, 65536  # of the kernels
+
+    def __post_init__(self):
+        if self.hidden > self.MAX_WIDTH:
+            raise ValueError(f"{self.name}: width up to {self.MAX_WIDTH}")
+        for i, b in enumerate(self.blocks):
+            where, m, f = f"{self.name}: layer {i}", b.mixer, b.mlp
+            if m.heads % m.kv_heads or max(m.dim, m.vdim) > self.MAX_HEAD or not 0 <= m.conv <= self.MAX_TAPS:
+                raise ValueError(f"{where}: whole groups of kv_heads, heads up to {self.MAX_HEAD} wide, taps up to {self.MAX_TAPS}")
+            if m.rot is not None and (m.rot.dims % 2 or m.rot.dims > m.dim):
+                raise ValueError(f"{where}: rotated dimensions come in pairs, at most {m.dim}")
+            if m.temp is not None and m.temp.every < 1:
+                raise ValueError(f"{where}: the query temperature's period is a positive number")
+            if isinstance(f, PolyMlp) and f.ff > self.MAX_FF:
+                raise ValueError(f"{where}: MLP up to {self.MAX_FF} wide")
+            _check_moe(where, f)
+        mixed = [b.mixer for b in self.blocks if b.mixer.v_mix]
+        if len({(m.kv_heads, m.vdim) for m in mixed}) > 1:
+            raise ValueError(f"{self.name}: layers that mix values have equal value heads")
+
+    @property
+    def layers(self) -> int:
+        return len(self.blocks)
+
+    @property
+    def first_mix(self) -> int | None:
+        """The layer whose values later layers mix in."""
+        return next((i for i, b in enumerate(self.blocks) if b.mixer.v_mix), None)
+
+    @property
+    def padded_hidden(self) -> int:
+        return _up(self.hidden, 128)
+
+    @property
+    def padded_vocab(self) -> int:
+        return _up(self.vocab_size, 128)
+
+    def to_dict(self):
+        return asdict(self)
+
+    def params(self) -> int:
+        W = self.hidden
+        n = 2 * self.vocab_size * W + 2 * W
+        for i, b in enumerate(self.blocks):
+            m, f = b.mixer, b.mlp
+            qkv = (m.heads + m.kv_heads) * m.dim + m.kv_heads * m.vdim
+            whole = m.norm == "whole"
+            n += W * (qkv + 2 * m.heads * m.vdim if m.gate == "element" else qkv + m.heads * (m.vdim + 1)) + m.heads
+            n += ((m.heads + m.kv_heads) * m.dim if whole else 2 * m.dim) + qkv * (m.conv + m.bias) + m.v_mix
+            n += W * W + 2 * W + i + 2
+            if f is not None:
+                n += W * W + 2 * W
+            if isinstance(f, PolyMlp):
+                n += 2 * W * f.ff + 4
+            elif f is not None:
+                n += f.experts * 3 * W * f.ff + f.outputs * (W + 1)
+        return n
+
+
+def bizetar_uniform(name: str, layers: int, vocab_size: int, hidden: int, first: SinkMixer, second: SinkMixer, dense: PolyMlp,
+                    moe: MoeMlp | None, **kw) -> BizetarConfig:
+    """A Bizetar whose mixers alternate; with ``moe`` the feed-forwards do too (dense, experts)."""
+    blocks = tuple(HybridLayer((first, second)[i % 2], dense if moe is None or i % 2 == 0 else moe) for i in range(layers))
+    return BizetarConfig(name, vocab_size, hidden, blocks, **kw)
 
 
 ENCODERS = {
@@ -619,6 +756,29 @@ DECODERS.update({
         HybridLayer(SelectiveMixer(96, 8, 4, 4), None),
         HybridLayer(LatentMixer(5, 16, 56, 48, 0.2, rot=Rotary(32), gate=True), MoeMlp(5, 1, 1.0, 24, None, "sigmoid", "input"))),
         1e-5, loop=(1, 3, 2), softcap=20.0, max_position=2048),
+})
+
+DECODERS.update({
+    # Llama-3-8B's width, vocabulary and heads; distance slopes and convolved rotary attention in turn
+    "bizetar-8b": bizetar_uniform(
+        "bizetar-8b", 32, 128256, 4096,
+        SinkMixer(32, 8, 128, 128, 128 ** -0.5, "head", "element", True, 4, Rotary(128, 500000.0, _YARN), v_mix=True),
+        SinkMixer(32, 8, 128, 128, 128 ** -0.5, "whole", "head", temp=QueryTemp(0.1, 8192), slopes=True, v_mix=True),
+        PolyMlp(14336), None),
+    # ... and with experts: 64 of 1024 beside 8 identity experts, 8 per token, at Llama-3.2-1B's width
+    "bizetar-moe": bizetar_uniform(
+        "bizetar-moe", 16, 128256, 2048,
+        SinkMixer(16, 4, 128, 128, 128 ** -0.5, "head", "element", True, 4, Rotary(128, 500000.0, _YARN), v_mix=True),
+        SinkMixer(16, 4, 128, 128, 128 ** -0.5, "whole", "head", temp=QueryTemp(0.1, 8192), slopes=True, v_mix=True),
+        PolyMlp(8192), MoeMlp(64, 8, 1.0, 1024, scores="softmax_raw", correction=True, identity=8)),
+    # test size: every branch at unequal sizes
+    "tiny-bizetar": BizetarConfig("tiny-bizetar", 1000, 200, (
+        HybridLayer(SinkMixer(6, 2, 40, 24, 0.2, "whole", "head", temp=QueryTemp(0.3, 50), slopes=True, v_mix=True),
+                    MoeMlp(7, 3, 1.0, 40, scores="softmax_raw", correction=True, identity=3)),
+        HybridLayer(SinkMixer(4, 2, 48, 24, 0.15, "head", "element", True, 3, Rotary(32, 5000.0, Yarn(3.0, 100, 16.0, 2.0)),
+                              v_mix=True), PolyMlp(168)),
+        HybridLayer(SinkMixer(3, 1, 64, 72, 0.12, "head", "element", True, 4, Rotary(64, 1000.0)), None)),
+        1e-5, max_position=2048),
 })
 
 _ALIASES = {
@@ -812,7 +972,44 @@ def vunelix_config_from_dir(path: str) -> VunelixConfig:
                          None if not cap else float(cap))
 
 
-_DIR_CONFIGS = {"vumuvik": vumuvik_config_from_dir, "vugotar": vugotar_config_from_dir, "vunelix": vunelix_config_from_dir}
+def bizetar_config_from_dir(path: str) -> BizetarConfig:
+    """config.json of a Bizetar checkpoint: ``architecture``, ``vocab``, ``width``, ``norm.eps`` and ``layers`` (each ``type``,
+    ``mixer`` sizes and ``mlp`` or null)."""
+    c = _hf(path)
+    blocks = []
+    for i, L in enumerate(c["layers"]):
+        m, f = L["mixer"], L.get("mlp")
+        kw = dict(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                  scale=float(m["scale"]), v_mix=bool(m.get("v_mix")))
+        if L.get("type") == "attention":
+            t = m.get("q_temp")
+            mixer = SinkMixer(norm="whole", gate="head", slopes=True,
+                              temp=None if t is None else QueryTemp(float(t["coef"]), int(t["every"])), **kw)
+        elif L.get("type") == "attention_2":
+            rot = m.get("rot")
+            if rot is not None:
+                sc = rot.get("scaling")
+                rot = Rotary(int(rot["dims"]), float(rot["base"]), None if sc is None else Yarn(
+                    float(sc["factor"]), float(sc["original"]), float(sc["fast"]), float(sc["slow"])))
+            mixer = SinkMixer(norm="head", gate="element", bias=True, conv=int(m.get("conv") or 0), rot=rot, **kw)
+        else:
+            raise ValueError(f"{path}: layer {i}: mixer type {L.get('type')!r} is not supported (attention, attention_2)")
+        if f is None:
+            mlp = None
+        elif f.get("kind") == "dense":
+            mlp = PolyMlp(int(f["ff"]))
+        elif f.get("kind") == "moe":
+            r = f["router"]
+            mlp = MoeMlp(int(r["experts"]), int(r["top"]), 1.0, int(f["expert"]["ff"]), scores="softmax_raw", correction=True,
+                         identity=int(r.get("identity") or 0))
+        else:
+            raise ValueError(f"{path}: layer {i}: mlp kind {f.get('kind')!r} is not supported (dense, moe or null)")
+        blocks.append(HybridLayer(mixer, mlp))
+    return BizetarConfig(_label(path), int(c["vocab"]), int(c["width"]), tuple(blocks), float(c["norm"]["eps"]))
+
+
+_DIR_CONFIGS = {"vumuvik": vumuvik_config_from_dir, "vugotar": vugotar_config_from_dir, "vunelix": vunelix_config_from_dir,
+                "bizetar": bizetar_config_from_dir}
 
 
 def _dir_architecture(path: str) -> str | None:
@@ -821,7 +1018,7 @@ def _dir_architecture(path: str) -> str | None:
     return arch if arch in _DIR_CONFIGS else c.get("model_type")
 
 
-def decoder_config(name: str, **overrides) -> DecoderConfig | VumuvikConfig | VugotarConfig | VunelixConfig:
+def decoder_config(name: str, **overrides) -> DecoderConfig | VumuvikConfig | VugotarConfig | VunelixConfig | BizetarConfig:
     if checkpoint_dir(name):
         cfg = _DIR_CONFIGS.get(_dir_architecture(name), decoder_config_from_hf)(name)
         return replace(cfg, **overrides) if overrides else cfg

@@ -21,6 +21,10 @@ class FragmentProjections:
         """Bytes of ``slots`` state slots (none: every layer's memory is paged)."""
         return 0
 
+    def step_bytes(self, tokens: int) -> int:
+        """Bytes that a step over ``tokens`` tokens keeps from its first layer to its last (nothing worth planning for)."""
+        return 0
+
     # stream_gemm.hip configurations (shuffled weights): BN 128 rows per workgroup at M <= 64 (13)
     # and M <= 128 (10).  Whole-chip tilings at M 65..128: gate_up's 28672 rows / 112 make exactly
     # 256 workgroups where BN 128 left 32 of the 256 CUs idle (cfg 20: 54.9 -> 51.5 us cold); the LM

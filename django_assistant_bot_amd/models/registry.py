@@ -6,16 +6,19 @@ from typing import Callable
 
 import torch
 
-from .configs import DecoderConfig, VugotarConfig, VumuvikConfig, VunelixConfig
+from .bizetar import BizetarModel
+from .configs import BizetarConfig, DecoderConfig, VugotarConfig, VumuvikConfig, VunelixConfig
 from .llama import LlamaModel
 from .vugotar import VugotarModel
 from .vumuvik import VumuvikModel
 from .vunelix import VunelixModel
 from .weights import (
+    load_bizetar_checkpoint,
     load_decoder_checkpoint,
     load_vugotar_checkpoint,
     load_vumuvik_checkpoint,
     load_vunelix_checkpoint,
+    random_bizetar_weights,
     random_decoder_weights,
     random_vugotar_weights,
     random_vumuvik_weights,
@@ -51,6 +54,8 @@ FAMILIES = {
     VugotarConfig: DecoderFamily(VugotarModel, _single(random_vugotar_weights), _single(load_vugotar_checkpoint),
                                  (torch.bfloat16, torch.float32)),
     VunelixConfig: DecoderFamily(VunelixModel, _single(random_vunelix_weights), _single(load_vunelix_checkpoint),
+                                 (torch.bfloat16, torch.float32)),
+    BizetarConfig: DecoderFamily(BizetarModel, _single(random_bizetar_weights), _single(load_bizetar_checkpoint),
                                  (torch.bfloat16, torch.float32)),
 }
 

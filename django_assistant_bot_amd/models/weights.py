@@ -19,11 +19,13 @@ import torch
 from ..ops.selective import state_width
 
 from .configs import (
+    BizetarConfig,
     DecoderConfig,
     DenseMlp,
     EncoderConfig,
     MoeMlp,
     ParallelMixer,
+    PolyMlp,
     SelectiveMixer,
     VugotarConfig,
     VumuvikConfig,
@@ -657,3 +659,123 @@ def random_vunelix_tensors(cfg: VunelixConfig, device="cpu", dtype=torch.bfloat1
 def random_vunelix_weights(cfg: VunelixConfig, device="cpu", dtype=torch.bfloat16, seed=0, interleave_mlp=False) -> dict:
     device = torch.device(device)
     return _vunelix_layout(cfg, random_vunelix_tensors(cfg, device, dtype, seed), device, dtype, interleave_mlp)
+
+
+# ------------------------------------------------------------------------------------------------
+# Bizetar
+
+
+def bizetar_columns(cfg: BizetarConfig, i: int) -> Columns:
+    """Output rows of a layer's input projection: queries, keys and values, output gate, gate of the mixer's result."""
+    m, inp = cfg.blocks[i].mixer, Columns()
+    inp.add("qkv", (m.heads + 2 * m.kv_heads) * m.padded_head())
+    inp.add("g", m.heads * (m.padded_head() if m.gate == "element" else 1))
+    inp.add("rg", cfg.padded_hidden)
+    return inp
+
+
+def _bizetar_layout(cfg: BizetarConfig, get, device, dtype, interleave_mlp) -> dict:
+    """``get(name, shape)`` -> the engine's tensors.  Everything that reads a sublayer's input is one projection: ``in_w``
+    (``bizetar_columns``) for the mixer, ``up_w`` [up; gate of the result] or, with experts, ``rg_w`` (the gate alone) beside
+    the fp32 ``router_w``.  Sizes are padded with zeros; gains (``qk_norm``: of every query and key head), biases, taps,
+    sinks and the weights over depth are fp32; single numbers are floats."""
+    W, Wp = cfg.hidden, cfg.padded_hidden
+
+    def mat(name, *shape):
+        return get(name, shape).to(device=device, dtype=dtype)
+
+    def vec(name, *shape):
+        return get(name, shape).to(device=device, dtype=torch.float32).contiguous()
+
+    def glu(p, ff, to):
+        return _gate_up(_pad(mat(p + "gate", ff, W), to, Wp), _pad(mat(p + "up", ff, W), to, Wp), interleave_mlp).contiguous()
+
+    embed = _pad(mat("embed", cfg.vocab_size, W), cfg.vocab_size, Wp)
+    w = {"embed": embed, "embed_norm": _pad(vec("embed.norm", W), Wp),
+         "lm_head": _pad(mat("head", cfg.vocab_size, W), cfg.padded_vocab, Wp), "final_norm": _pad(vec("final.norm", W), Wp)}
+    for i, blk in enumerate(cfg.blocks):
+        p, m, f = f"l{i}.", blk.mixer, blk.mlp
+        q, H, G, D = p + "mix.", m.heads, m.kv_heads, m.padded_head()
+        parts = (("q", H, m.dim), ("k", G, m.dim), ("v", G, m.vdim))
+
+        def heads(of, cols):  # rows of every q, k and v head, each padded to D
+            return torch.cat([_pad(of(n, h * d).view(h, d, cols), h, D, cols).reshape(h * D, cols) for n, h, d in parts])
+
+        inp = bizetar_columns(cfg, i)
+        rows = {"qkv": heads(lambda n, r: mat(q + n, r, W), W), "rg": mat(p + "rg1", W, W)}
+        if m.gate == "element":
+            rows["g"] = _pad(mat(q + "g", H * m.vdim, W).view(H, m.vdim, W), H, D, W).reshape(H * D, W)
+        else:
+            rows["g"] = mat(q + "g", H, W)
+        w[p + "in_w"] = inp.fill(rows, Wp, _up(inp.width, 256 if inp.width > 2048 else 128), embed)
+        if m.bias:
+            w[p + "qkv_b"] = heads(lambda n, r: vec(q + n + ".b", r), 1).view(-1).contiguous()
+        if m.conv:
+            w[p + "conv_w"] = heads(lambda n, r: vec(q + n + ".conv", r, m.conv), m.conv).t().contiguous()
+        if m.norm == "whole":
+            gains = [_pad(vec(q + n + ".norm", h * m.dim).view(h, m.dim), h, D) for n, h in (("q", H), ("k", G))]
+        else:
+            gains = [_pad(vec(q + n + ".norm", m.dim), D).expand(h, D) for n, h in (("q", H), ("k", G))]
+        w[p + "qk_norm"] = torch.cat(gains).reshape(-1).contiguous()
+        w[p + "sink"] = vec(q + "sink", H)
+        if m.slopes:
+            w[p + "slopes"] = torch.tensor([2.0 ** (-8.0 * (h + 1) / H) for h in range(H)], dtype=torch.float32, device=device)
+        if m.v_mix:
+            w[p + "vmix"] = float(get(q + "vmix", ()))
+        w[p + "o_w"] = _pad(mat(q + "o", W, H * m.vdim).view(W, H, m.vdim), Wp, H, D).reshape(Wp, H * D)
+        w[p + "norm1"], w[p + "rg1_b"] = _pad(vec(p + "norm1", W), Wp), _pad(vec(p + "rg1.b", W), Wp)
+        w[p + "depth"] = vec(p + "dwa", i + 2)
+        if f is None:
+            continue
+        w[p + "norm2"], w[p + "rg2_b"] = _pad(vec(p + "norm2", W), Wp), _pad(vec(p + "rg2.b", W), Wp)
+        gate = _pad(mat(p + "rg2", W, W), Wp, Wp)
+        q = p + "mlp."
+        if isinstance(f, PolyMlp):
+            F = _up(f.ff, 128)
+            w[p + "up_w"] = torch.cat([_pad(mat(q + "up", f.ff, W), F, Wp), gate])
+            w[p + "down_w"] = _pad(mat(q + "down", W, f.ff), Wp, F)
+            w[p + "act"] = tuple(float(x) for x in get(q + "act", (4,)))
+        else:
+            w[p + "rg_w"] = gate
+            w[p + "router_w"] = _pad(mat(q + "router", f.outputs, W), _up(f.outputs, 128), Wp)
+            w[p + "correction"] = vec(q + "correction", f.outputs)
+            ex, F = [f"{q}e{e}." for e in range(f.experts)], _up(f.ff, 64)
+            w[p + "expert_gate_up_w"] = torch.cat([glu(e, f.ff, F) for e in ex])
+            w[p + "expert_down_w"] = torch.cat([_pad(mat(e + "down", W, f.ff), Wp, F) for e in ex])
+    return w
+
+
+def load_bizetar_checkpoint(path: str, cfg: BizetarConfig, device="cpu", dtype=torch.bfloat16, interleave_mlp=False,
+                            reader: SafetensorsDir | None = None) -> dict:
+    return _bizetar_layout(cfg, _checked(path, reader), torch.device(device), dtype, interleave_mlp)
+
+
+def random_bizetar_tensors(cfg: BizetarConfig, device="cpu", dtype=torch.bfloat16, seed=0):
+    """Seeded ``get(name, shape)`` of a random Bizetar: fan-in scaled matrices, norms near one, small biases and sinks, weights
+    over depth that keep most of the newest result."""
+    g = _gen(torch.device(device), seed * 1000003)
+
+    def get(name, shape):
+        if name.endswith(".vmix"):
+            return torch.tensor(0.3)
+        if name.endswith(".act"):
+            return torch.tensor([0.8, 0.4, 0.3, 0.1])
+        if name.endswith(".dwa"):
+            t = _randn(shape, g, device, torch.float32, std=0.2 / shape[0])
+            t[-1] += 0.9
+            return t
+        if name.endswith(".conv"):
+            return _randn(shape, g, device, torch.float32, std=shape[1] ** -0.5)
+        if len(shape) == 2:
+            return _randn(shape, g, device, dtype, std=STD if name in ("embed", "head") else shape[1] ** -0.5)
+        t = _randn(shape, g, device, torch.float32, std=0.1)
+        if name.endswith(".correction"):
+            return t / shape[0]
+        return t if name.endswith((".b", ".sink")) else t + 1.0
+
+    return get
+
+
+def random_bizetar_weights(cfg: BizetarConfig, device="cpu", dtype=torch.bfloat16, seed=0, interleave_mlp=False) -> dict:
+    device = torch.device(device)
+    return _bizetar_layout(cfg, random_bizetar_tensors(cfg, device, dtype, seed), device, dtype, interleave_mlp)

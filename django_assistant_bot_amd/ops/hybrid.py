@@ -136,61 +136,63 @@ def qk_rope_write(y, col0: int, H: int, G: int, D: int, dim: int, rot: int, turn
 CHUNK_FLASH_DIMS = (64, 128, 256)
 
 
-def _any(q, kc, vc, bt, cu, ctx, B, scale, chunk, sink, out, out_scale):
+def _any(q, kc, vc, bt, cu, ctx, B, scale, chunk, sink, out, out_scale, slopes):
     T, H, D = q.shape
     expect(D % 2 == 0 and D <= 1024, "head width")
     native().any_attention(ptr(q), ptr(kc), ptr(vc), int(q.dtype == torch.float32), ptr(bt), bt.shape[1], kc.shape[2],
-                           ptr(cu), ptr(ctx), B, T, H, kc.shape[1], D, int(chunk), float(scale), ptr(sink), ptr(out),
+                           ptr(cu), ptr(ctx), B, T, H, kc.shape[1], D, int(chunk), float(scale), ptr(sink), ptr(slopes), ptr(out),
                            out.stride(0), float(out_scale), stream(q))
     return out
 
 
-def _check_attn(q, kc, vc, bt, ctx, B, sink, out):
+def _check_attn(q, kc, vc, bt, ctx, B, sink, out, slopes=None):
     T, H, D = q.shape
     _i32(bt)
     _i32(ctx)
     expect(q.is_contiguous() and kc.is_contiguous() and vc.is_contiguous() and q.dtype == kc.dtype == vc.dtype
            and q.dtype in _ACT and kc.shape == vc.shape and kc.shape[3] == D and H % kc.shape[1] == 0, "q / cache shapes")
     expect(bt.shape[0] >= B and ctx.numel() >= B, "block table / ctx_lens rows < batch")
-    if sink is not None:
-        _f32v(H, sink)
+    _f32v(H, sink, slopes)
     expect(out.shape[0] >= T and out.stride(-1) == 1 and out.shape[1] >= H * D and out.dtype == q.dtype
            and out.stride(0) % 8 == 0, "output rows")
-    same_device(q, kc, bt, ctx, sink, out)
+    same_device(q, kc, bt, ctx, sink, slopes, out)
 
 
-def chunk_prefill(q, kc, vc, bt, cu, ctx, max_q: int, scale: float, chunk: int, sink, out, out_scale: float = 1.0):
+def chunk_prefill(q, kc, vc, bt, cu, ctx, max_q: int, scale: float, chunk: int, sink, out, out_scale: float = 1.0,
+                  slopes=None):
     """Causal attention of prompt portions over the paged cache in which query i sees the keys of its own chunk,
-    i // chunk * chunk .. i (0: all before it).  ``sink`` fp32 [H]: one more score in the denominator.  Writes
-    out_scale * result to ``out``, rows [T, >= H D]."""
+    i // chunk * chunk .. i (0: all before it).  ``sink`` fp32 [H]: one more score in the denominator.  ``slopes`` fp32
+    [H]: slope * (i - j) is taken off the score of key j.  Writes out_scale * result to ``out``, rows [T, >= H D]."""
     if not q.is_cuda:
         T = q.shape[0]
-        out[:T, :q.shape[1] * q.shape[2]] = ref.chunk_attention(q, kc, vc, bt, cu, ctx, scale, chunk, sink, out_scale).view(T, -1).to(out.dtype)
+        out[:T, :q.shape[1] * q.shape[2]] = ref.chunk_attention(
+            q, kc, vc, bt, cu, ctx, scale, chunk, sink, out_scale, slopes).view(T, -1).to(out.dtype)
         return out
     T, H, D = q.shape
     _i32(cu)
     B = cu.numel() - 1
-    _check_attn(q, kc, vc, bt, ctx, B, sink, out)
+    _check_attn(q, kc, vc, bt, ctx, B, sink, out, slopes)
     if q.dtype == torch.float32 or D not in CHUNK_FLASH_DIMS or kc.shape[2] % 64:
-        return _any(q, kc, vc, bt, cu, ctx, B, scale, chunk, sink, out, out_scale)
+        return _any(q, kc, vc, bt, cu, ctx, B, scale, chunk, sink, out, out_scale, slopes)
     qst, qsh = _head_strides(q)
     native().flash_attention_chunk(ptr(q), qst, qsh, ptr(kc), ptr(vc), ptr(bt), bt.shape[1], kc.shape[2], ptr(out),
                                    out.stride(0), D, ptr(cu), ptr(ctx), B, int(max_q), H, kc.shape[1], D, float(scale),
-                                   int(chunk), ptr(sink), float(out_scale), stream(q))
+                                   int(chunk), ptr(sink), ptr(slopes), float(out_scale), stream(q))
     return out
 
 
 def chunk_decode(q, kc, vc, bt, ctx, scale: float, chunk: int, sink, out, out_scale: float = 1.0, part_size: int = 512,
-                 workspace=None, order=None):
+                 workspace=None, order=None, slopes=None):
     """The same for one new token per sequence (split over key partitions counted from the chunk's start)."""
     B, H, D = q.shape
     if not q.is_cuda:
-        out[:B, :H * D] = ref.chunk_attention(q, kc, vc, bt, None, ctx, scale, chunk, sink, out_scale).view(B, -1).to(out.dtype)
+        out[:B, :H * D] = ref.chunk_attention(
+            q, kc, vc, bt, None, ctx, scale, chunk, sink, out_scale, slopes).view(B, -1).to(out.dtype)
         return out
-    _check_attn(q, kc, vc, bt, ctx, B, sink, out)
+    _check_attn(q, kc, vc, bt, ctx, B, sink, out, slopes)
     G, bs = kc.shape[1], kc.shape[2]
     if q.dtype == torch.float32 or D not in (64, 128) or H // G > 16 or bs % 32:
-        return _any(q, kc, vc, bt, None, ctx, B, scale, chunk, sink, out, out_scale)
+        return _any(q, kc, vc, bt, None, ctx, B, scale, chunk, sink, out, out_scale, slopes)
     expect(part_size % 128 == 0, "part_size must be a multiple of 128")
     parts = workspace.max_parts if workspace is not None else 1
     if workspace is None:
@@ -207,7 +209,7 @@ def chunk_decode(q, kc, vc, bt, ctx, scale: float, chunk: int, sink, out, out_sc
         expect(order.numel() >= B, "decode order must hold the batch")
     native().paged_decode_attention(ptr(q), ptr(kc), ptr(vc), ptr(bt), bt.shape[1], bs, ptr(ctx), ptr(out), *ws, B, H, G,
                                     D, int(part_size), int(parts), float(scale), stream(q), ptr(order), chunk=int(chunk),
-                                    sink=ptr(sink), out_scale=float(out_scale), o_stride=out.stride(0))
+                                    sink=ptr(sink), out_scale=float(out_scale), o_stride=out.stride(0), slopes=ptr(slopes))
     return out
 
 
@@ -433,26 +435,32 @@ def gated_norm(y, gate, g_col: int, part: int, w, eps: float, out, row0: int, T:
 MAX_EXPERTS, MAX_TOP = 1024, 64
 
 
-def moe_route(z, col0: int, E: int, top: int, scale: float, T: int, scores: str = "softmax"):
+MOE_SCORES = ("softmax", "sigmoid", "softmax_raw")
+
+
+def moe_route(z, col0: int, E: int, top: int, scale: float, T: int, scores: str = "softmax", correction=None):
     """fp32 router logits (columns col0..) -> (experts int32 [T, top], weights fp32 [T, top]): softmax over all experts,
-    the ``top`` largest, over their sum, times ``scale``; ``scores`` "sigmoid": the ``top`` largest sigmoids as they are,
-    times ``scale``."""
-    expect(scores in ("softmax", "sigmoid"), "scores: softmax or sigmoid")
+    the ``top`` largest, over their sum, times ``scale``; ``scores`` "sigmoid", "softmax_raw": the ``top`` largest sigmoids /
+    softmax scores as they are, times ``scale``.  ``correction`` fp32 [E] joins the scores where the experts are chosen, not
+    in the weights."""
+    expect(scores in MOE_SCORES, f"scores: one of {MOE_SCORES}")
+    _f32v(E, correction)
     if not z.is_cuda:
-        idx, wt = ref.moe_route(z, col0, E, top, scale, scores)
+        idx, wt = ref.moe_route(z, col0, E, top, scale, scores, correction)
         return idx[:T].int(), wt[:T]
     pz = _proj(z, T, col0 + E, "router logits")
     expect(pz[1] == 1 and 1 <= top <= min(E, MAX_TOP) and E <= MAX_EXPERTS, "router: fp32 logits, top <= experts")
     idx = torch.empty((T, top), dtype=torch.int32, device=z.device)
     wt = torch.empty((T, top), dtype=torch.float32, device=z.device)
-    native().moe_route(pz, int(col0), E, top, float(scale), int(scores == "sigmoid"), ptr(idx), ptr(wt), T, stream(z))
+    native().moe_route(pz, int(col0), E, top, float(scale), MOE_SCORES.index(scores), ptr(correction), ptr(idx), ptr(wt), T, stream(z))
     return idx, wt
 
 
 def moe_experts(h, idx, wt, gate_up, down, E: int, group: int, weigh: str = "output"):
     """Each token's chosen experts: ``gate_up`` [E * 2F, K] and ``down`` [E * W, F] hold the experts one after the other
     (bf16 on the GPU: ``shuffle_weights`` copies with gate / up in 8-row groups; fp32: row-major, stacked).  -> [T * top,
-    W], row t * top + k = weight * expert output (``weigh`` "input": the expert of weight * h)."""
+    W], row t * top + k = weight * expert output (``weigh`` "input": the expert of weight * h).  A choice of ``E`` or more is an
+    identity expert: its row is not written."""
     T, top = idx.shape
     expect(weigh in ("output", "input"), "weigh: output or input")
     if not h.is_cuda:
@@ -509,17 +517,18 @@ def shared_glu(y, col0: int, n: int, z, sg_col: int, out):
 # gates and caps
 
 
-def sigmoid_gate(y, col0: int, x):
-    """x [T, n] *= sigmoid(columns col0 .. col0 + n of a projection), in place."""
+def sigmoid_gate(y, col0: int, x, per: int = 1):
+    """x [T, n] *= sigmoid(columns col0 .. of a projection), in place; a column gates ``per`` neighbours of x."""
     T, n = x.shape
+    expect(n % per == 0, "whole groups of columns")
     if not x.is_cuda:
-        return x.copy_((x.float() * torch.sigmoid(ref.total(y)[:T, col0:col0 + n])).to(x.dtype))
-    py = _proj(y, T, col0 + n, "gate")
-    expect(x.dtype in _ACT and x.stride(1) == 1 and x.stride(0) % 8 == 0 and n % 8 == 0 and col0 % 8 == 0 and py[4] % 8 == 0,
-           "rows and columns in eights")
+        return x.copy_((x.float() * torch.sigmoid(ref.total(y)[:T, col0:col0 + n // per]).repeat_interleave(per, 1)).to(x.dtype))
+    py = _proj(y, T, col0 + n // per, "gate")
+    expect(x.dtype in _ACT and x.stride(1) == 1 and x.stride(0) % 8 == 0 and n % 8 == 0 and py[4] % 8 == 0
+           and (per % 8 == 0 or per == 1 and col0 % 8 == 0), "rows and columns in eights")
     expect(x.dtype == torch.bfloat16 or py[1] == 1, "fp32 activations take an fp32 projection")
     same_device(y, x)
-    native().sigmoid_gate(py, int(col0), ptr(x), x.stride(0), int(x.dtype == torch.float32), n, T, stream(x))
+    native().sigmoid_gate(py, int(col0), int(per), ptr(x), x.stride(0), int(x.dtype == torch.float32), n, T, stream(x))
     return x
 
 

@@ -54,7 +54,7 @@ def qk_rope_write(y, col0, H, G, D, dim, rot, freq, eps, norm, positions, slots,
     return qk[:, :H].to(dtype).contiguous()
 
 
-def chunk_attention(q, kc, vc, bt, cu, ctx, scale, chunk, sink, out_scale):
+def chunk_attention(q, kc, vc, bt, cu, ctx, scale, chunk, sink, out_scale, slopes=None):
     T, H, D = q.shape
     G, bs = kc.shape[1], kc.shape[2]
     out = torch.empty(T, H, D)
@@ -66,6 +66,8 @@ def chunk_attention(q, kc, vc, bt, cu, ctx, scale, chunk, sink, out_scale):
         k, v = (c[blk, :, pos % bs].float().repeat_interleave(H // G, 1) for c in (kc, vc))
         s = torch.einsum("qhd,khd->hqk", q[rows[b]:rows[b + 1]].float(), k) * scale
         i = torch.arange(m - n, m)[:, None]
+        if slopes is not None:
+            s = s - slopes.float().view(-1, 1, 1) * (i - pos[None])
         bad = pos[None] > i
         if chunk:
             bad = bad | (pos[None] // chunk != i // chunk)
@@ -139,10 +141,12 @@ def gated_norm(y, gate, g_col, part, gate_first, per_head, w, eps, scale):
     return v if gate_first else v * g
 
 
-def moe_route(z, col0, E, top, scale, scores="softmax"):
+def moe_route(z, col0, E, top, scale, scores="softmax", correction=None):
     z = total(z)[:, col0:col0 + E]
-    v, idx = torch.topk(torch.sigmoid(z) if scores == "sigmoid" else torch.softmax(z, -1), top, -1)
-    if scores == "sigmoid":
+    s = torch.sigmoid(z) if scores == "sigmoid" else torch.softmax(z, -1)
+    idx = torch.topk(s if correction is None else s + correction, top, -1).indices
+    v = s.gather(-1, idx)
+    if scores != "softmax":
         return idx, v * scale
     return idx, v / (v.sum(-1, keepdim=True) + 1e-20) * scale
 
