@@ -169,7 +169,7 @@ __global__ __launch_bounds__(1024) void poly_norm_kernel(Proj y, int n, int cols
     proj8<PT>(y, row, c, z[i]);
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      z[i][j] = ElemIO<AT>::round(z[i][j]);
+      z[i][j] = c + j < n ? ElemIO<AT>::round(z[i][j]) : 0.f;
       const float q = z[i][j] * z[i][j], q2 = q * q;
       m2 += q;
       m4 += q2;

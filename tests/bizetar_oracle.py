@@ -100,7 +100,8 @@ def attention(h, kind, m, w, p, eps, first, planted=()):
         if "head_norm" in planted:
             q = norm(q.view(n, H, D), w[p + "q.norm"].view(H, D), eps)
             k = norm(k.view(n, G, D), w[p + "k.norm"].view(G, D), eps)
-        q, k = norm(q, w[p + "q.norm"], eps).view(n, H, D), norm(k, w[p + "k.norm"], eps).view(n, G, D)
+        else:
+            q, k = norm(q, w[p + "q.norm"], eps).view(n, H, D), norm(k, w[p + "k.norm"], eps).view(n, G, D)
         if "q_temp" not in planted:
             q = q * temperature(n, m["q_temp"])[:, None, None]
     else:
