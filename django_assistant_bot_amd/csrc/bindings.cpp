@@ -205,9 +205,9 @@ PYBIND11_MODULE(_native, m) {
           "qk_rope_write");
   });
   // routed = (expert rows, indices, weights, choices per token, experts); gate = (projection, column, bias);
-  // depth = (results, weights, stride, n, keep)
+  // depth = (results, weights, stride, n, keep, sum ahead, results in it)
   m.def("gated_residual", [proj](u src, u x, u h, int act_f32, const P& y, u ids, const std::tuple<u, u, u, int, int>& routed,
-                                 const P& g, int g_col, u g_bias, u post, const std::tuple<u, u, long, int, int>& depth, u gain,
+                                 const P& g, int g_col, u g_bias, u post, const std::tuple<u, u, long, int, int, u, int>& depth, u gain,
                                  int n_true, float eps, int rows, int cols, u s) {
     dab::GatedResidual p{};
     p.src = (const float*)src, p.x = (float*)x, p.h = VP(h), p.y = proj(y), p.ids = (const int*)ids;
@@ -215,9 +215,12 @@ PYBIND11_MODULE(_native, m) {
     p.top = std::get<3>(routed), p.experts = std::get<4>(routed);
     p.g = proj(g), p.g_col = g_col, p.g_bias = (const float*)g_bias, p.post = (const float*)post;
     p.depth = (float*)std::get<0>(depth), p.weights = (const float*)std::get<1>(depth), p.depth_stride = std::get<2>(depth);
-    p.n = std::get<3>(depth), p.keep = std::get<4>(depth);
+    p.n = std::get<3>(depth), p.keep = std::get<4>(depth), p.ahead = (const float*)std::get<5>(depth), p.from = std::get<6>(depth);
     p.gain = (const float*)gain, p.inv_n = 1.f / n_true, p.eps = eps, p.cols = cols;
     check(dab::gated_residual(p, act_f32, rows, ST(s)), "gated_residual");
+  });
+  m.def("depth_ahead", [](u over, long stride, u w, int n, int m, u out, u s) {
+    check(dab::depth_ahead((const float*)over, stride, (const float*)w, n, m, (float*)out, ST(s)), "depth_ahead");
   });
   m.def("poly_norm", [proj](const P& y, int n, int cols, float a, float b, float c, float e, float eps, u out, int act_f32, int T,
                             u s) {
@@ -395,19 +398,24 @@ PYBIND11_MODULE(_native, m) {
   m.def("paged_decode_attention", [](u q, u kc, u vc, u bt, int max_blocks, int bs, u ctx, u out, u po, u pm, u pl,
                                      u cnt, int batch, int Hq, int Hkv, int D, int part_size, int max_parts,
                                      float scale, u s, u order, u w0, long w0_bytes, u w1, long w1_bytes,
-                                     int w_blocks, int chunk, u sink, float out_scale, long o_stride, u slopes) {
+                                     int w_blocks, int chunk, u sink, float out_scale, long o_stride, u slopes,
+                                     const std::tuple<u, int, int, long, long, int, int>& gate) {
     dab::L3Warm warm{{(const char*)w0, (const char*)w1}, {w0_bytes, w1_bytes}, w_blocks};
+    // gate = (projection, column, columns of the output it covers each)
+    const dab::OutputGate og{{CVP(std::get<0>(gate)), std::get<1>(gate), std::get<2>(gate), std::get<3>(gate), std::get<4>(gate)},
+                             std::get<5>(gate), std::get<6>(gate)};
     check(dab::paged_decode_attention(CVP(q), CVP(kc), CVP(vc), (const int*)bt, max_blocks, bs, (const int*)ctx, VP(out),
                                       (float*)po, (float*)pm, (float*)pl, (int*)cnt, batch, Hq, Hkv, D, part_size,
                                       max_parts, scale, ST(s), (const int*)order, &warm, chunk, (const float*)sink,
-                                      out_scale, o_stride, (const float*)slopes),
+                                      out_scale, o_stride, (const float*)slopes, &og),
           "paged_decode_attention");
   }, py::arg("q"), py::arg("kc"), py::arg("vc"), py::arg("bt"), py::arg("max_blocks"), py::arg("bs"), py::arg("ctx"),
      py::arg("out"), py::arg("po"), py::arg("pm"), py::arg("pl"), py::arg("cnt"), py::arg("batch"), py::arg("Hq"),
      py::arg("Hkv"), py::arg("D"), py::arg("part_size"), py::arg("max_parts"), py::arg("scale"), py::arg("s"),
      py::arg("order") = 0, py::arg("w0") = 0, py::arg("w0_bytes") = 0, py::arg("w1") = 0, py::arg("w1_bytes") = 0,
      py::arg("w_blocks") = 0, py::arg("chunk") = 0, py::arg("sink") = 0, py::arg("out_scale") = 1.f,
-     py::arg("o_stride") = 0, py::arg("slopes") = 0);
+     py::arg("o_stride") = 0, py::arg("slopes") = 0,
+     py::arg("gate") = std::make_tuple((u)0, 0, 1, 0L, 0L, 0, 1));
   m.def("gemm_bt", [](u A, long lda, u B, long ldb, u C, long ldc, u bias, u residual, long ldr, int M, int N, int K,
                       int epilogue, int out_f32, u row_group, u q_group, u allow, int allow_words, u s, int b_rows,
                       int b_group) {

@@ -20,6 +20,7 @@
 
 #include "common.h"
 #include "launchers.h"
+#include "proj.h"
 
 #include <type_traits>
 
@@ -447,12 +448,16 @@ __device__ __forceinline__ unsigned lds_addr(const char* p) {
 // SGB (A/B): the S^T phase's 16 K-fragment LDS reads and 16 MFMAs interleaved by
 // sched_group_barrier (4 reads ahead, then one MFMA per read) instead of hipcc's own order; same
 // instructions and accumulation order (bit-identical).
+//
+// BIAS: softmax sink and slopes (FlashParams, either may be null; no window).  The accumulators of S^T start at the key's
+// distance term, the running maximum at the sink, whose own term is then 1.
 template <bool CAUSAL, bool VPIPE = false, int NW = 4, bool STAG = false, bool PAIR = false, bool ONEBAR = false,
-          bool SMS = false, bool SGB = false>
+          bool SMS = false, bool SGB = false, bool BIAS = false>
 __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void flash_d128_kernel(FlashParams p) {
   static_assert(NW == 4 || NW == 8, "4 or 8 waves");
   static_assert(!STAG || NW == 8, "staggered groups: 8 waves");
   static_assert(!PAIR || (NW == 4 && CAUSAL), "paired blocks: 4 waves, causal");
+  static_assert(!BIAS || (CAUSAL && !STAG), "sink and slopes: causal, no staggered groups");
   constexpr int D = 128, KT = 64, QB = 32 * NW;
   constexpr int TILE = KT * D * 2;  // 16 KB
   constexpr int BUF = 2 * TILE;     // K | V
@@ -614,8 +619,11 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void flash_d128_kernel(Fl
   for (int db = 0; db < 4; ++db)
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[db][r] = 0.f;
-  float m_run = -1e30f, l_run = 0.f;  // running max in log2 units (scores x scale_log2)
   const float sc = p.scale_log2;
+  const float m_start = BIAS && p.sink ? p.sink[h] * 1.4426950408889634f : -1e30f;
+  const float l_start = BIAS && p.sink && hi == 0 ? 1.f : 0.f;
+  const float slope = BIAS && p.slopes ? p.slopes[h] * 1.4426950408889634f / sc : 0.f;  // (of the unscaled score)
+  float m_run = m_start, l_run = l_start;  // running max in log2 units (scores x scale_log2)
 
   // Loop-invariant LDS addresses (the tile buffer and the key block go in the instruction offset).
   // K reads of k-step st: row lq (and 32 + lq: +8 KB), logical chunk 2 st + hi at (2 st + hi) ^ f(lq).
@@ -651,6 +659,14 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void flash_d128_kernel(Fl
     f32x16 s0, s1;
 #pragma unroll
     for (int r = 0; r < 16; ++r) s0[r] = s1[r] = 0.f;
+    if constexpr (BIAS) {
+      const float base = slope * (float)(k0 + 4 * hi - q_pos);
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        s0[r] = fmaf(slope, (float)((r & 3) + 8 * (r >> 2)), base);
+        s1[r] = fmaf(slope, (float)((r & 3) + 8 * (r >> 2) + 32), base);
+      }
+    }
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
       bf16x8 ka[4], kb2[4];
@@ -996,8 +1012,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void flash_d128_kernel(Fl
       for (int db = 0; db < 4; ++db)
 #pragma unroll
         for (int r = 0; r < 16; ++r) o[db][r] = 0.f;
-      m_run = -1e30f;
-      l_run = 0.f;
+      m_run = m_start;
+      l_run = l_start;
 #pragma unroll
       for (int st = 0; st < 8; ++st) qf[st] = qfB[st];
       rope_q = p.rope_cs && q_valid;
@@ -1546,6 +1562,7 @@ struct DecodeParams {
   const float* slopes;  // SLOPE: slopes[h] times the distance is taken off a key's score
   float out_scale;
   long o_stride_tok;
+  OutputGate gate;  // optional (gate.y.p): the finished output times its sigmoid
   L3Warm warm;  // optional: the next projections' weights, warmed into L3 by appended workgroups
 };
 
@@ -1822,6 +1839,10 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
         L = L * f + exp2f(sk - M2);
         O *= f;
       }
+      if (p.gate.y.p) {
+        const int c = p.gate.col + (hh * D + d) / p.gate.per;
+        O /= 1.f + __expf(-(p.gate.y.f32 ? proj_f32<float>(p.gate.y, b, c) : proj_f32<bf16>(p.gate.y, b, c)));
+      }
       p.out[(size_t)b * p.o_stride_tok + (size_t)hh * D + d] = f2bf(L > 0.f ? O / L * p.out_scale : 0.f);
     };
     for (int e = tid; e < G * D; e += 256) {
@@ -1923,6 +1944,24 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
   prm.Hkv = Hkv;
   prm.scale_log2 = scale * 1.4426950408889634f;
   prm.pairs_per_wg = 1;
+  if (D == 128 && paged && causal && !rope_cs && (sink || slopes) && window == 0 && chunk == 0 && out_scale == 1.f && scale > 0.f) {
+    prm.sink = sink;
+    prm.slopes = slopes;
+    // query blocks in pairs and walked heaviest-first as below, unless that leaves CUs idle
+    const int npairs = ((max_seqlen_q + 127) / 128 + 1) / 2;
+    const long wgs = (long)npairs * Hq * batch;
+    if (wgs >= 256) {
+      const int G = wgs >= 2048 && npairs > 1 ? 2 : 1;
+      prm.pairs_per_wg = G;
+      prm.lpt = ((long)Hq * batch) % 8 == 0;
+      hipLaunchKernelGGL((flash_d128_kernel<true, true, 4, false, true, false, false, false, true>),
+                         dim3((npairs + G - 1) / G, Hq, batch), dim3(256), 0, s, prm);
+    } else {
+      hipLaunchKernelGGL((flash_d128_kernel<true, true, 4, false, false, false, false, false, true>),
+                         dim3((max_seqlen_q + 127) / 128, Hq, batch), dim3(256), 0, s, prm);
+    }
+    return hipGetLastError();
+  }
   if (window > 0 || chunk > 0 || sink || slopes || D == 256 || out_scale != 1.f) {  // windowed / chunked / sink form: 16-query sub-tiles
     if (!causal || rope_cs || (window > 0 && chunk > 0) || (slopes && !paged)) return hipErrorInvalidValue;
     prm.slopes = slopes;
@@ -2081,7 +2120,7 @@ int paged_decode_attention(const void* q, const void* k_cache, const void* v_cac
                            float* part_m, float* part_l, int* counters, int batch, int Hq, int Hkv, int D,
                            int part_size, int max_parts, float scale, hipStream_t s, const int* order,
                            const L3Warm* warm, int chunk, const float* sink, float out_scale, long o_stride_tok,
-                           const float* slopes) {
+                           const float* slopes, const OutputGate* gate) {
   if (batch <= 0) return 0;
   if (Hq % Hkv || Hq / Hkv > 16 || part_size % 128 || max_parts < 1 || block_size % 32) return hipErrorInvalidValue;
   if (max_parts > 1 && !counters) return hipErrorInvalidValue;
@@ -2108,6 +2147,8 @@ int paged_decode_attention(const void* q, const void* k_cache, const void* v_cac
   prm.chunk = chunk;
   prm.sink = sink;
   prm.slopes = slopes;
+  prm.gate = gate ? *gate : OutputGate{};
+  if (prm.gate.y.p && (prm.gate.per < 1 || prm.gate.y.S < 1)) return hipErrorInvalidValue;
   prm.out_scale = out_scale;
   prm.o_stride_tok = o_stride_tok ? o_stride_tok : (long)Hq * D;
   prm.warm = warm ? *warm : L3Warm{{nullptr, nullptr}, {0, 0}, 0};

@@ -3,8 +3,10 @@
 //   gated_residual  f = sublayer output (GEMM rows or split-K slabs), or the token's expert rows, of which identity experts
 //                   (index >= experts) are weight * stream;  f *= sigmoid(gate columns of a projection + bias);
 //                   x = stream + f / rms(f) * post.  At a layer's end also: x is kept as result ``n`` of the depth buffer and
-//                   becomes sum_j w[j] * result j (j <= n).  h = x, or x / rms(x) * gain.  Everything between a sublayer's
+//                   becomes sum_j w[j] * result j (j <= n), of which a part may be there already (``ahead``).  h = x, or x / rms(x) * gain.  Everything between a sublayer's
 //                   last projection and the next one's first in one pass
+//   depth_ahead     for several layers at once, their sums over the results there are so far: a block of layers reads the
+//                   results before it once instead of each layer all of them
 //   norm_embed      the same over rows of the embedding table: x = norm(table[id])
 //   poly_norm       a N(z) + b N(z^2) + c N(z^3) + e over the first n columns of a projection, N(v) = v / rms(v)
 //
@@ -65,7 +67,8 @@ __global__ __launch_bounds__(1024) void gated_residual_kernel(GatedResidual p) {
     }
     if (DEPTH) {
       const float* q = p.depth + at;
-      int k = 0;
+      int k = p.from;
+      if (p.ahead) ElemIO<float>::load8(p.ahead + at, d[i]);
       for (; k + 4 <= p.n; k += 4) {
         float v[4][8];
 #pragma unroll
@@ -128,7 +131,7 @@ int gated_residual(GatedResidual p, int act_f32, int rows, hipStream_t s) {
   if (p.cols <= 0 || p.cols % 8 || p.cols > 16384 || !p.x || !p.h || !p.post || (!p.y.p && !p.pairs) ||
       (p.pairs && (p.top < 1 || !p.idx || !p.wt || !p.src)) || (p.g.p && (!p.g_bias || p.g_col % 8 || p.g.ld % 8 || p.g.S < 1)) ||
       (p.y.p && (p.y.S < 1 || p.y.ld % 8)) || (p.y.p && p.g.p && p.y.f32 != p.g.f32) || p.n < 0 ||
-      (p.n && (!p.depth || !p.weights || p.depth_stride % 8)))
+      (p.n && (!p.depth || !p.weights || p.depth_stride % 8 || p.from < 0 || p.from > p.n)))
     return hipErrorInvalidValue;
   const Proj& like = p.y.p ? p.y : p.g;
   if (!like.p) return hipErrorInvalidValue;
@@ -149,6 +152,59 @@ int gated_residual(GatedResidual p, int act_f32, int rows, hipStream_t s) {
   DAB_PROJ_DISPATCH(like, act_f32, GR_NV);
 #undef GR_NV
 #undef GR_L
+  return hipGetLastError();
+}
+
+template <int M>
+__global__ __launch_bounds__(256) void depth_ahead_kernel(const float* __restrict__ over, long stride, const float* __restrict__ w,
+                                                          int n, float* __restrict__ out, long vecs) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= vecs) return;
+  f32x4 acc[M];
+#pragma unroll
+  for (int m = 0; m < M; ++m) acc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const float* q = over + i * 4;
+  int k = 0;
+  for (; k + 4 <= n; k += 4) {
+    f32x4 v[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) v[u] = *reinterpret_cast<const f32x4*>(q + (k + u) * stride);
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+#pragma unroll
+      for (int m = 0; m < M; ++m)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[m][j] = fmaf(w[m * n + k + u], v[u][j], acc[m][j]);
+  }
+  for (; k < n; ++k) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(q + k * stride);
+#pragma unroll
+    for (int m = 0; m < M; ++m)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[m][j] = fmaf(w[m * n + k], v[j], acc[m][j]);
+  }
+#pragma unroll
+  for (int m = 0; m < M; ++m) *reinterpret_cast<f32x4*>(out + m * stride + i * 4) = acc[m];
+}
+
+int depth_ahead(const float* over, long stride, const float* w, int n, int m, float* out, hipStream_t s) {
+  if (stride <= 0) return 0;
+  if (stride % 4 || n < 1 || m < 1 || m > 8 || (stride / 4 + 255) / 256 > (1u << 31) - 1) return hipErrorInvalidValue;
+  const long vecs = stride / 4;
+  const dim3 grid((unsigned)((vecs + 255) / 256));
+#define DA_L(M) \
+  case M: hipLaunchKernelGGL(depth_ahead_kernel<M>, grid, dim3(256), 0, s, over, stride, w, n, out, vecs); break
+  switch (m) {
+    DA_L(1);
+    DA_L(2);
+    DA_L(3);
+    DA_L(4);
+    DA_L(5);
+    DA_L(6);
+    DA_L(7);
+    DA_L(8);
+  }
+#undef DA_L
   return hipGetLastError();
 }
 

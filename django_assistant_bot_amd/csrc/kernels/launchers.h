@@ -30,6 +30,12 @@ struct Proj {
   long slab, ld;
 };
 
+// A sigmoid gate of an attention's output: columns ``col`` .. of a projection, one for ``per`` neighbours of the output
+struct OutputGate {
+  Proj y;
+  int col, per;
+};
+
 // norm.hip
 int rmsnorm(void* out, void* res_out, const void* x, const void* res_in, const void* w, int rows, int cols, float eps,
             hipStream_t s);
@@ -64,7 +70,7 @@ int paged_decode_attention(const void* q, const void* k_cache, const void* v_cac
                            int part_size, int max_parts, float scale, hipStream_t s,
                            const int* order = nullptr, const L3Warm* warm = nullptr, int chunk = 0,
                            const float* sink = nullptr, float out_scale = 1.f, long o_stride_tok = 0,
-                           const float* slopes = nullptr);
+                           const float* slopes = nullptr, const OutputGate* gate = nullptr);
 
 // attention_any.hip (any head width, bf16 or fp32, paged)
 int any_attention(const void* q, const void* kc, const void* vc, int f32, const int* bt, int max_blocks, int bs,
@@ -100,11 +106,15 @@ struct GatedResidual {
   const float* weights;      // [n + 1]
   long depth_stride;
   int n, keep;
+  const float* ahead;        // the sum over results 0 .. from - 1 (null: none, from is 0)
+  int from;
   const float* gain;         // or null
   float inv_n, eps;
   int cols;
 };
 int gated_residual(GatedResidual p, int act_f32, int rows, hipStream_t s);
+// out[m] = sum over j < n of w[m][j] result j, for up to 8 rows of w; ``stride`` elements a result
+int depth_ahead(const float* over, long stride, const float* w, int n, int m, float* out, hipStream_t s);
 int poly_norm(Proj y, int n, int cols, float a, float b, float c, float e, float eps, void* out, int act_f32, int T, hipStream_t s);
 
 // attn_inputs.hip (input projection -> bias, convolution, norm, rotation, temperature, value mix -> q rows and paged cache)

@@ -12,7 +12,9 @@ and sublayers read it as it is, so everything that reads a sublayer's input is o
 
 What follows a sublayer's last projection is one pass (``ops.gated_residual``): slab or expert-row sum, identity experts,
 gate, norm, residual and, at a layer's end, the sum over the results of all earlier layers.  Those results are kept for the
-step in fp32 (``depth``); only the convolution's past inputs outlive a step, in state slots.
+step in fp32 (``depth``); every few layers the sums of the next ones over all results so far are formed at once
+(``ops.depth_ahead``), so a layer reads the newest results only.  What outlives a step beside the pages is the convolution's
+past inputs, in state slots.
 
 The 32-bit mode (``dtype=torch.float32``) runs the same steps with fp32 weights, activations and cache.
 """
@@ -106,6 +108,9 @@ class BizetarModel(HybridProjections):
             self.layers.append(L)
         if gpu and consume:
             torch.cuda.empty_cache()
+        # the weights of a block of layers over the results before it: [layers, results]
+        self.ahead = {b: torch.stack([L.depth[:b + 1] for L in self.layers[b:b + ops.MAX_AHEAD]]).contiguous()
+                      for b in range(ops.MAX_AHEAD, len(self.layers), ops.MAX_AHEAD)}
         self.recurrent = any(L.inputs.conv is not None for L in self.layers)
         self.layer_tap = None  # called as tap(layer, residual stream) after every layer (numerics tests)
 
@@ -127,7 +132,7 @@ class BizetarModel(HybridProjections):
         return slots * HybridCache.bytes_per_slot(self._specs(), self.dtype)
 
     def step_bytes(self, tokens: int) -> int:
-        return 4 * tokens * len(self.layers) * self.embed.shape[1]  # (``depth``)
+        return 4 * tokens * (len(self.layers) + (ops.MAX_AHEAD if self.ahead else 0)) * self.embed.shape[1]  # (``depth``)
 
     long_part = 2048
 
@@ -147,10 +152,15 @@ class BizetarModel(HybridProjections):
         small_pf = not meta.decode and not meta.n_decode and T <= self.PREFILL_STREAM_MAX_M
         sk = self.frag and (meta.decode and T <= self.STREAM_MAX_M or small_pf)
         depth = torch.empty((n, T, self.embed.shape[1]), dtype=torch.float32, device=ids.device)
+        sums = torch.empty((ops.MAX_AHEAD, *depth.shape[1:]), dtype=torch.float32, device=ids.device) if self.ahead else None
         h = ops.norm_embed(ids, self.embed, self.embed_norm, W, eps, depth[0])
         x, src, first = torch.empty_like(depth[0]), depth[0], None
         for i, L in enumerate(self.layers):
-            close = dict(depth=(depth, L.depth, i + 1), gain=self.final_norm if i + 1 == n else None)
+            b = i - i % ops.MAX_AHEAD  # the first layer of the block
+            if i in self.ahead:
+                ops.depth_ahead(depth, self.ahead[i], sums)
+            ahead = (sums[i - b], b + 1) if b else (None, 0)
+            close = dict(depth=(depth, L.depth, i + 1, *ahead), gain=self.final_norm if i + 1 == n else None)
             y, z, first = self._attention(i, L, h, meta, kv, sk, first)
             h = ops.gated_residual(src, x, z, (y, L.cols.at["rg"], L.rg1_b), L.norm1, W, eps, self.dtype,
                                    **(close if L.norm2 is None else {}))
@@ -177,15 +187,16 @@ class BizetarModel(HybridProjections):
         Tp = 0 if meta.decode else T - meta.n_decode
         q = ops.attn_inputs(y, at["qkv"], a, meta.positions, meta.slots, kc, vc, kv.ring[i], meta.cu_q if Tp else None, meta.max_q,
                             meta.state_slots if Tp else None, meta.state_slots if meta.decode else meta.dec_state_slots, Tp, mix)
+        per = a.D if L.mixer.gate == "head" else 1
         o = torch.empty((T, a.H * a.D), dtype=self.dtype, device=h.device)
         if Tp:
             ops.chunk_prefill(q[:Tp], kc, vc, meta.block_tables, meta.cu_q, meta.ctx_lens, meta.max_q, L.mixer.scale, 0, L.sink,
                               o[:Tp], slopes=L.slopes)
-        if Tp < T:
+            ops.sigmoid_gate(y, at["g"], o[:Tp], per)
+        if Tp < T:  # (mixed steps have finished projections)
             bt, ctx = (meta.block_tables, meta.ctx_lens) if meta.decode else (meta.dec_block_tables, meta.dec_ctx_lens)
             ops.chunk_decode(q[Tp:], kc, vc, bt, ctx, L.mixer.scale, 0, L.sink, o[Tp:], 1.0, meta.part_size, meta.workspace,
-                             meta.order, L.slopes)
-        ops.sigmoid_gate(y, at["g"], o, a.D if L.mixer.gate == "head" else 1)
+                             meta.order, L.slopes, (y[Tp:] if Tp else y, at["g"], per))
         return y, self._proj(o, L.o_w, sk, name="o"), first
 
     def _mlp(self, L: BizetarLayer, h, sk: bool):

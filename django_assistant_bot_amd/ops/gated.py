@@ -42,7 +42,7 @@ def norm_embed(ids, table, gain, n: int, eps: float, x):
     h = torch.empty((T, cols), dtype=table.dtype, device=x.device)
     f32 = int(table.dtype == torch.float32)
     native().gated_residual(0, ptr(x), ptr(h), f32, (ptr(table), f32, 1, 0, cols), ptr(ids), (0, 0, 0, 0, 0), _NONE, 0, 0, ptr(gain),
-                            (0, 0, 0, 0, 0), 0, int(n), float(eps), T, cols, stream(x))
+                            (0, 0, 0, 0, 0, 0, 0), 0, int(n), float(eps), T, cols, stream(x))
     return h
 
 
@@ -50,8 +50,9 @@ def gated_residual(src, x, y, gate, post, n: int, eps: float, dtype=torch.bfloat
                    gain=None):
     """x = src + f' / rms(f') * post with f' = f * sigmoid(columns col.. of a projection + bias), ``gate`` = (projection, col,
     bias), and f = the sublayer output ``y`` (rows or slabs) or the token's expert rows (``own``), in which identity experts
-    give weight * src.  ``depth`` = (results fp32 [N, T, C], weights [k + 1], k): x becomes result k (kept if k < N) and then
-    sum over j <= k of weights[j] * result j.  fp32 [T, C]; ``x`` may be ``src``.  -> x, or with ``gain`` x / rms(x) * gain, as
+    give weight * src.  ``depth`` = (results fp32 [N, T, C], weights [k + 1], k, ahead, n): x becomes result k (kept if k < N)
+    and then the sum over j <= k of weights[j] * result j, the first ``n`` of which are in ``ahead`` [T, C] (``depth_ahead``;
+    None: none, n = 0).  fp32 [T, C]; ``x`` may be ``src``.  -> x, or with ``gain`` x / rms(x) * gain, as
     ``dtype``.  Mean squares are over the first ``n`` columns; the padded ones are zero."""
     expect((y is None) != (own is None), "a sublayer output or expert rows")
     if not x.is_cuda:
@@ -75,18 +76,38 @@ def gated_residual(src, x, y, gate, post, n: int, eps: float, dtype=torch.bfloat
                and tuple(own.idx.shape) == tuple(own.wt.shape) == (T, top) and own.wt.dtype == torch.float32
                and own.wt.is_contiguous(), "expert rows")
         routed = (ptr(own.rows), ptr(own.idx), ptr(own.wt), top, int(own.experts))
-    over, w, k = depth if depth is not None else (None, None, 0)
+    over, w, k, ahead, n_ahead = depth if depth is not None else (None, None, 0, None, 0)
     if depth is not None:
         expect(over.dtype == torch.float32 and over.is_contiguous() and over.dim() == 3 and tuple(over.shape[1:]) == (T, cols)
                and 1 <= k <= over.shape[0], "results over depth")
         _f32v(k + 1, w)
+        _f32v(T * cols, ahead)
+        expect(0 <= n_ahead <= k and (ahead is not None or n_ahead == 0), "results ahead")
         expect(x.data_ptr() != over.data_ptr(), "the stream is not a result")
     same_device(x, src, y, g, bias, post, over, w, gain)
     h = torch.empty((T, cols), dtype=dtype, device=x.device)
     native().gated_residual(ptr(src), ptr(x), ptr(h), int(dtype == torch.float32), py, 0, routed, pg, int(col), ptr(bias), ptr(post),
-                            (ptr(over), ptr(w), T * cols, k, int(depth is not None and k < over.shape[0])), ptr(gain), int(n),
+                            (ptr(over), ptr(w), T * cols, k, int(depth is not None and k < over.shape[0]), ptr(ahead), n_ahead), ptr(gain), int(n),
                             float(eps), T, cols, stream(x))
     return h
+
+
+MAX_AHEAD = 8  # layers whose sums are formed at once
+
+
+def depth_ahead(over, w, out):
+    """out[m] = sum over j of w[m][j] * over[j]: results fp32 [n, T, C], weights fp32 [m, n], out fp32 [>= m, T, C]."""
+    m, n = w.shape
+    if not over.is_cuda:
+        out[:m] = torch.einsum("mn,ntc->mtc", w, over[:n])
+        return out
+    expect(over.dtype == out.dtype == torch.float32 and over.is_contiguous() and out.is_contiguous() and over.shape[0] >= n
+           and out.shape[0] >= m and over.shape[1:] == out.shape[1:] and over.shape[2] % 8 == 0 and 1 <= m <= MAX_AHEAD and n >= 1,
+           "results and sums")
+    _f32v(m * n, w)
+    same_device(over, w, out)
+    native().depth_ahead(ptr(over), over.shape[1] * over.shape[2], ptr(w), n, m, ptr(out), stream(over))
+    return out
 
 
 def poly_norm(y, T: int, n: int, cols: int, act, eps: float, dtype):

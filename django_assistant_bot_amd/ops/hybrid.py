@@ -182,17 +182,23 @@ def chunk_prefill(q, kc, vc, bt, cu, ctx, max_q: int, scale: float, chunk: int, 
 
 
 def chunk_decode(q, kc, vc, bt, ctx, scale: float, chunk: int, sink, out, out_scale: float = 1.0, part_size: int = 512,
-                 workspace=None, order=None, slopes=None):
-    """The same for one new token per sequence (split over key partitions counted from the chunk's start)."""
+                 workspace=None, order=None, slopes=None, gate=None):
+    """The same for one new token per sequence (split over key partitions counted from the chunk's start).  ``gate`` =
+    (projection, column, per): the output times the sigmoid of its columns, as ``sigmoid_gate``."""
     B, H, D = q.shape
     if not q.is_cuda:
         out[:B, :H * D] = ref.chunk_attention(
             q, kc, vc, bt, None, ctx, scale, chunk, sink, out_scale, slopes).view(B, -1).to(out.dtype)
+        if gate is not None:
+            sigmoid_gate(gate[0], gate[1], out[:B, :H * D], gate[2])
         return out
     _check_attn(q, kc, vc, bt, ctx, B, sink, out, slopes)
     G, bs = kc.shape[1], kc.shape[2]
     if q.dtype == torch.float32 or D not in (64, 128) or H // G > 16 or bs % 32:
-        return _any(q, kc, vc, bt, None, ctx, B, scale, chunk, sink, out, out_scale, slopes)
+        _any(q, kc, vc, bt, None, ctx, B, scale, chunk, sink, out, out_scale, slopes)
+        if gate is not None:
+            sigmoid_gate(gate[0], gate[1], out[:B, :H * D], gate[2])
+        return out
     expect(part_size % 128 == 0, "part_size must be a multiple of 128")
     parts = workspace.max_parts if workspace is not None else 1
     if workspace is None:
@@ -207,9 +213,16 @@ def chunk_decode(q, kc, vc, bt, ctx, scale: float, chunk: int, sink, out, out_sc
     if order is not None:
         _i32(order)
         expect(order.numel() >= B, "decode order must hold the batch")
+    og = (0, 0, 1, 0, 0, 0, 1)
+    if gate is not None:
+        y, col, per = gate
+        expect(per >= 1 and H * D % per == 0, "whole groups of gated columns")
+        og = (*_proj(y, B, col + H * D // per, "gate"), int(col), int(per))
+        same_device(q, y)
     native().paged_decode_attention(ptr(q), ptr(kc), ptr(vc), ptr(bt), bt.shape[1], bs, ptr(ctx), ptr(out), *ws, B, H, G,
                                     D, int(part_size), int(parts), float(scale), stream(q), ptr(order), chunk=int(chunk),
-                                    sink=ptr(sink), out_scale=float(out_scale), o_stride=out.stride(0), slopes=ptr(slopes))
+                                    sink=ptr(sink), out_scale=float(out_scale), o_stride=out.stride(0), slopes=ptr(slopes),
+                                    gate=og)
     return out
 
 

@@ -28,10 +28,12 @@ def gated_residual(src, x, y, gate, post, n, eps, dtype, own, depth, gain):
     f = f * torch.sigmoid(total(g)[:T, col:col + C] + bias)
     out = src + _unit(f, n, eps) * post
     if depth is not None:
-        over, w, k = depth
+        over, w, k, ahead, n0 = depth
         if k < over.shape[0]:
             over[k] = out
-        out = w[k] * out + (w[:k, None, None] * over[:k]).sum(0)
+        out = w[k] * out + (w[n0:k, None, None] * over[n0:k]).sum(0)
+        if ahead is not None:
+            out = out + ahead
     x.copy_(out)
     return (x if gain is None else _unit(x, n, eps) * gain).to(dtype, copy=True)
 

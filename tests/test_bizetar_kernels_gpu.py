@@ -59,13 +59,27 @@ def test_gated_residual(rows, cols, n, yt, dtype, form, depth):
         t[..., n:] = 0
     last = depth == 6  # (its result is not kept, a norm follows)
     x, xg, og = torch.zeros_like(src), src.to(DEV), over.to(DEV)
-    tail = lambda f: dict(depth=(f[0], f[1], depth) if depth else None, gain=f[2] if last else None)  # noqa: E731
-    want = ops.gated_residual(src, x, y, (g, 16, bias), post, n, 1e-4, dtype, own, **tail((over, w, gain)))
+    ahead = rnd(rows, cols, seed=10, dtype=F32) if last else None
+    if last:
+        ahead[:, n:] = 0
+    tail = lambda f: dict(depth=(f[0], f[1], depth, f[3], 4 if last else 0) if depth else None,  # noqa: E731
+                          gain=f[2] if last else None)
+    want = ops.gated_residual(src, x, y, (g, 16, bias), post, n, 1e-4, dtype, own, **tail((over, w, gain, ahead)))
     gown = None if own is None else ops.RoutedRows(dev(own.rows), dev(own.idx), dev(own.wt), 6)
-    got = ops.gated_residual(xg, xg, dev(y), (dev(g), 16, dev(bias)), dev(post), n, 1e-4, dtype, gown, **tail((og, dev(w), dev(gain))))
+    got = ops.gated_residual(xg, xg, dev(y), (dev(g), 16, dev(bias)), dev(post), n, 1e-4, dtype, gown, **tail((og, dev(w), dev(gain), dev(ahead))))
     close(xg, x, 3e-6)
     close(og, over, 3e-6)
     close(got, want, 6e-3 if dtype == BF else 4e-6)
+
+
+@pytest.mark.parametrize("T,C,n,m", [(1, 128, 9, 8), (7, 4096, 25, 8), (300, 640, 17, 3), (5, 256, 1, 1), (64, 2048, 9, 5), (2, 128, 10, 7),
+                                     (3, 384, 8, 2), (3, 384, 12, 4), (3, 384, 15, 6)])
+def test_depth_ahead(T, C, n, m):
+    over, w = rnd(n + 2, T, C, dtype=F32), rnd(m, n, seed=1, dtype=F32)
+    out = torch.zeros(8, T, C, device=DEV)
+    ops.depth_ahead(dev(over), dev(w), out)
+    close(out[:m], torch.einsum("mn,ntc->mtc", w.double(), over[:n].double()), 2e-6)
+    assert float(out[m:].abs().sum()) == 0
 
 
 @pytest.mark.parametrize("rows,cols,n", [(1, 128, 65), (700, 4096, 4000), (9, 8192, 8192)])
@@ -134,7 +148,7 @@ def test_attn_inputs(shape, whole, yt, dtype, mix):
     H, G, D = shape[:3]
     lens, starts, dec = [1, 2, 21, 9], [0, 5, 0, 100], [3, 0, 77, 1, 130]
     T0, T = sum(lens), sum(lens) + len(dec)
-    a, col, y, ring = input_case(*shape, whole, T, yt, dtype, slabs=3 if yt == F32 else 1, slots=12)
+    a, col, y, ring = input_case(*shape, whole, T, yt, dtype, slabs=3 if yt != dtype else 1, slots=12)
     pos = torch.cat([torch.arange(s, s + n) for s, n in zip(starts, lens)] + [torch.tensor(dec)]).int()
     cu = torch.tensor([0, *torch.tensor(lens).cumsum(0).tolist()], dtype=torch.int32)
     bs = 16
@@ -230,6 +244,38 @@ def test_sloped_attention(H, G, D, dtype, sloped):
             close(dg, d, tol)
     ops.chunk_decode(a[0][:4], *a[1:4], a[5], scale, 0, dev(sink), dg, slopes=dev(slopes))
     close(dg, d, tol)
+    for per in (1, D):  # with an output gate, from finished rows and from slabs
+        y = rnd(*((3,) if per == 1 else ()), 4, 16 + -(-H * D // per // 8) * 8, seed=5, dtype=dtype)
+        d.zero_()
+        ops.chunk_decode(q[:4], kc, vc, bt, cx, scale, 0, sink, d, slopes=slopes, gate=(y, 16, per))
+        ops.chunk_decode(a[0][:4], *a[1:4], a[5], scale, 0, dev(sink), dg, 1.0, 512, ws, None, dev(slopes), (dev(y), 16, per))
+        close(dg, d, tol)
+
+
+@pytest.mark.parametrize("sloped,sunk", [(True, True), (True, False), (False, True)])
+@pytest.mark.parametrize("lens,done", [([700, 1, 384, 129, 513], [0, 64, 100, 0, 300]), ([2100], [130]), ([90] * 40, [7] * 40)])
+def test_prompts_of_many_blocks(lens, done, sloped, sunk):
+    """Heads of 128 with enough query blocks for the paired walk, portions that go on from cached keys among them."""
+    H, G, D, bs = 32, 4, 128, 64
+    ctx = [a + b for a, b in zip(lens, done)]
+    blocks = [-(-c // bs) for c in ctx]
+    bt = torch.zeros(len(lens), max(blocks), dtype=torch.int32)
+    perm = torch.randperm(sum(blocks), generator=torch.Generator().manual_seed(0)).int()
+    for i, n in enumerate(blocks):
+        bt[i, :n] = perm[sum(blocks[:i]):sum(blocks[:i + 1])]
+    kc, vc = (rnd(sum(blocks), G, bs, D, seed=s) for s in (1, 2))
+    q, sink = rnd(sum(lens), H, D, seed=3), rnd(H, seed=4, dtype=F32) + 2
+    slopes = oracle.slopes(H).float() if sloped else None
+    cu = torch.tensor([0, *torch.tensor(lens).cumsum(0).tolist()], dtype=torch.int32)
+    got = torch.zeros(sum(lens), H * D, dtype=BF, device=DEV)
+    ops.chunk_prefill(*(dev(t) for t in (q, kc, vc, bt, cu, i32(*ctx))), max(lens), 0.11, 0, dev(sink) if sunk else None, got,
+                      slopes=dev(slopes))
+    some = sorted({0, len(lens) // 2, len(lens) - 1})
+    for i in some:  # (the reference of a few sequences)
+        want = torch.zeros(lens[i], H * D, dtype=BF)
+        ops.chunk_prefill(q[cu[i]:cu[i + 1]], kc, vc, bt[i:i + 1], i32(0, lens[i]), i32(ctx[i]), lens[i], 0.11, 0, sink if sunk else None,
+                          want, slopes=slopes)
+        close(got[cu[i]:cu[i + 1]], want, 1e-2)
 
 
 @pytest.mark.parametrize("T,E,top,S", [(1, 3, 1, 1), (70, 72, 8, 4), (5, 9, 9, 2), (300, 260, 6, 1), (33, 1024, 64, 1)])

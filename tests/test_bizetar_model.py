@@ -82,6 +82,9 @@ CONFIGS = {
         sloped(4, 2, 128, 96, 0.09, None)]),
     # no convolution anywhere: everything is paged, so prefixes are shared
     "paged": config(96, [sloped(4, 2, 64, 48, 0.14, dense(64)), sloped(2, 1, 32, 32, 0.2, moe(5, 1, 2, 24))]),
+    # enough layers for several blocks of sums over depth
+    "deep": config(64, [(sloped(2, 1, 32, 32, 0.2, None, v_mix=True), convolved(2, 1, 32, 32, 0.15, 3, 16, dense(48), v_mix=i % 4 == 1),
+                         sloped(2, 2, 16, 24, 0.25, dense(40)))[i % 3] for i in range(19)]),
     # projection sizes that take the streaming decode GEMM (K % 128) and a split-K of several slabs
     "stream": config(512, [
         convolved(8, 2, 128, 128, 0.09, 4, 128, dense(1024), v_mix=True, base=10000.0, yarn=(4.0, 200, 32.0, 1.0)),
@@ -275,12 +278,16 @@ def test_sublayer_and_feed_forward_mechanisms():
         res = want if k == 3 else want * 1.0
         total = sum(w[j] * over[j] for j in range(k)) + w[k] * res
         o = pad(over)
-        h = ops.gated_residual(pad(x), xs, yy, (gg, 8, pad(b)), pad(post), n, eps, torch.float32, depth=(o, w.float(), k),
+        h = ops.gated_residual(pad(x), xs, yy, (gg, 8, pad(b)), pad(post), n, eps, torch.float32, depth=(o, w.float(), k, None, 0),
                                gain=None if gain is None else pad(gain))
         near(xs, pad(total))
         near(h, pad(total if gain is None else oracle.norm(total, gain, eps)))
         if k < 3:
             near(o[k], pad(want))
+        sums = ops.depth_ahead(o, torch.stack([w[:1], 2 * w[:1]]).float(), torch.zeros(8, T, C))
+        near(sums[1], 2 * w[0] * o[0])
+        h = ops.gated_residual(pad(x), xs, yy, (gg, 8, pad(b)), pad(post), n, eps, torch.float32, depth=(o, w.float(), k, sums[0], 1))
+        near(xs, pad(total))
     # the embedding
     table, ids = R(7, n), torch.tensor([3, 0, 6, 6, 1], dtype=torch.int32)
     h = ops.norm_embed(ids, pad(table), pad(post), n, eps, xs)
@@ -740,7 +747,9 @@ def test_memory_of_the_layers(models):
     assert [r is not None for r in kv.ring] == [True, False, True, False, True] and not any(s is not None for s in kv.state)
     assert eng.model.state_bytes(5) == sum(t.numel() * t.element_size() for t in kv.ring if t is not None)
     assert eng.model.cache_bytes_per_block(64) * eng.blocks.num_blocks() == sum(t.numel() * t.element_size() for t in kv.k + kv.v)
-    assert eng.model.step_bytes(10) == 10 * 5 * 256 * 4
+    assert eng.model.step_bytes(10) == 10 * 5 * 256 * 4 and not eng.model.ahead
+    deep = engine(models("deep")[0], ("cpu", torch.float32)).model
+    assert {b: tuple(t.shape) for b, t in deep.ahead.items()} == {8: (8, 9), 16: (3, 17)}
 
 
 def test_feed_guards(models):
