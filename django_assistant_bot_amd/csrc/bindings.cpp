@@ -165,11 +165,14 @@ PYBIND11_MODULE(_native, m) {
   // chunked / sink attention over the paged cache
   m.def("flash_attention_chunk",
         [](u q, long qst, long qsh, u kc, u vc, u bt, int max_blocks, int bs, u out, long ost, long osh, u cu_q, u ctx_k,
-           int batch, int max_sq, int Hq, int Hkv, int D, float scale, int chunk, u sink, u slopes, float out_scale, u s) {
+           int batch, int max_sq, int Hq, int Hkv, int D, float scale, int chunk, u sink, u slopes, float out_scale,
+           const std::tuple<u, int, int, long, long, int, int>& gate, u s) {
+          const dab::OutputGate og{{CVP(std::get<0>(gate)), std::get<1>(gate), std::get<2>(gate), std::get<3>(gate), std::get<4>(gate)},
+                                   std::get<5>(gate), std::get<6>(gate)};
           check(dab::flash_attention(CVP(q), qst, qsh, nullptr, nullptr, 0, 0, CVP(kc), CVP(vc), (const int*)bt,
                                      max_blocks, bs, VP(out), ost, osh, (const int*)cu_q, nullptr, (const int*)ctx_k,
                                      batch, max_sq, Hq, Hkv, D, 1, 1, scale, ST(s), nullptr, nullptr, 0,
-                                     (const float*)sink, chunk, out_scale, (const float*)slopes),
+                                     (const float*)sink, chunk, out_scale, (const float*)slopes, &og),
                 "flash_attention_chunk");
         });
   m.def("any_attention", [](u q, u kc, u vc, int f32, u bt, int max_blocks, int bs, u cu, u ctx, int B, int T, int H,

@@ -72,6 +72,7 @@ struct FlashParams {
   const float* sink;
   float out_scale;
   const float* slopes;  // slopes[h] times the distance i - j is taken off the score of key j (null: none)
+  OutputGate gate;      // flash_d128 BIAS only (gate.y.p): the output times its sigmoid; bf16 rows
 };
 
 // first key position that the query at position i sees
@@ -799,6 +800,34 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void flash_d128_kernel(Fl
     if (q_valid) {
       const float inv = l_tot > 0.f ? 1.f / l_tot : 0.f;
       bf16* orow = p.out + (size_t)(q_start + my_q) * p.o_stride_tok + (size_t)h * p.o_stride_head;
+      if constexpr (BIAS) {
+        if (p.gate.y.p) {
+          const bf16* g = (const bf16*)p.gate.y.p + (size_t)(q_start + my_q) * p.gate.y.ld + p.gate.col;
+          if (p.gate.per > 1) {  // one number a head
+            const float f = inv / (1.f + __expf(-bf2f(g[h])));
+#pragma unroll
+            for (int db = 0; db < 4; ++db) o[db] *= f;
+          } else {
+            u32x2 gv[16];
+#pragma unroll
+            for (int e = 0; e < 16; ++e) gv[e] = *reinterpret_cast<const u32x2*>(g + h * D + 32 * (e >> 2) + 8 * (e & 3) + 4 * hi);
+#pragma unroll
+            for (int e = 0; e < 16; ++e)
+#pragma unroll
+              for (int j = 0; j < 4; ++j) {
+                const float z = __uint_as_float(j & 1 ? gv[e][j >> 1] & 0xffff0000u : gv[e][j >> 1] << 16);
+                o[e >> 2][4 * (e & 3) + j] *= inv / (1.f + __expf(-z));
+              }
+          }
+#pragma unroll
+          for (int db = 0; db < 4; ++db)
+#pragma unroll
+            for (int rg = 0; rg < 4; ++rg)
+              *reinterpret_cast<u32x2*>(orow + 32 * db + 8 * rg + 4 * hi) =
+                  u32x2{pack2bf(o[db][4 * rg], o[db][4 * rg + 1]), pack2bf(o[db][4 * rg + 2], o[db][4 * rg + 3])};
+          return;
+        }
+      }
 #pragma unroll
       for (int db = 0; db < 4; ++db)
 #pragma unroll
@@ -1916,7 +1945,7 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
                     long o_stride_head, const int* cu_q, const int* cu_k, const int* ctx_k, int batch,
                     int max_seqlen_q, int Hq, int Hkv, int D, int causal, int paged, float scale, hipStream_t s,
                     const int* rope_pos, const void* rope_cs, int window, const float* sink, int chunk,
-                    float out_scale, const float* slopes) {
+                    float out_scale, const float* slopes, const OutputGate* gate) {
   if (batch <= 0 || max_seqlen_q <= 0) return 0;
   if (Hq % Hkv || (paged && block_size % 64)) return hipErrorInvalidValue;
   FlashParams prm{};
@@ -1947,6 +1976,11 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
   if (D == 128 && paged && causal && !rope_cs && (sink || slopes) && window == 0 && chunk == 0 && out_scale == 1.f && scale > 0.f) {
     prm.sink = sink;
     prm.slopes = slopes;
+    if (gate) {
+      prm.gate = *gate;
+      if (gate->y.p && (gate->y.S != 1 || gate->y.f32 || (gate->per != 1 && gate->per != D) || gate->col % 4 || gate->y.ld % 4))
+        return hipErrorInvalidValue;
+    }
     // query blocks in pairs and walked heaviest-first as below, unless that leaves CUs idle
     const int npairs = ((max_seqlen_q + 127) / 128 + 1) / 2;
     const long wgs = (long)npairs * Hq * batch;
@@ -1962,6 +1996,7 @@ int flash_attention(const void* q, long q_stride_tok, long q_stride_head, const 
     }
     return hipGetLastError();
   }
+  if (gate && gate->y.p) return hipErrorInvalidValue;
   if (window > 0 || chunk > 0 || sink || slopes || D == 256 || out_scale != 1.f) {  // windowed / chunked / sink form: 16-query sub-tiles
     if (!causal || rope_cs || (window > 0 && chunk > 0) || (slopes && !paged)) return hipErrorInvalidValue;
     prm.slopes = slopes;

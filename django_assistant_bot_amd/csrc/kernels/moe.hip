@@ -10,60 +10,91 @@
 //
 // Which rows an expert gets does not change a row's result, so the order within an expert is left to the
 // LDS atomics.
+#include <type_traits>
+
 #include "launchers.h"
 #include "proj.h"
 
 namespace dab {
 
-template <typename GT, int EI>
+// the largest value of the wave, in every lane (DPP: rows of 16, then the rows)
+__device__ __forceinline__ float wave_top(float v) {
+  const auto step = [](float x, auto ctrl) {
+    const int i = __float_as_int(x);  // (lanes without a source keep their own)
+    return fmaxf(x, __int_as_float(__builtin_amdgcn_update_dpp(i, i, decltype(ctrl)::value, 0xf, 0xf, false)));
+  };
+  v = step(v, std::integral_constant<int, 0xb1>{});   // neighbours
+  v = step(v, std::integral_constant<int, 0x4e>{});   // pairs
+  v = step(v, std::integral_constant<int, 0x141>{});  // quads, mirrored within 8
+  v = step(v, std::integral_constant<int, 0x140>{});  // eights, mirrored within 16
+  v = step(v, std::integral_constant<int, 0x142>{});  // a row's last lane to the next row
+  v = step(v, std::integral_constant<int, 0x143>{});  // the lower half's last lane to the upper half
+  return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), 63));
+}
+
+template <int EI>
 __global__ __launch_bounds__(256) void moe_route_kernel(Proj z, int col0, int E, int top, float scale, int scores,
                                                         const float* correction, int* idx, float* wt, int T) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= T) return;
   const bool sigmoid = scores == 1;
   float s[EI], w[EI];  // scores as experts are chosen by them, as weights
-  float mx = -__builtin_huge_valf();
+  const float* q = (const float*)z.p + (long)t * z.ld + col0;
+  int col[EI];
 #pragma unroll
   for (int i = 0; i < EI; ++i) {
-    const int e = lane + 64 * i;
-    s[i] = e < E ? proj_f32<GT>(z, t, col0 + e) : -__builtin_huge_valf();
-    mx = fmaxf(mx, s[i]);
+    col[i] = min(lane + 64 * i, E - 1);
+    s[i] = q[col[i]];
+    w[i] = correction ? correction[col[i]] : 0.f;
   }
-  mx = wave_max(mx);
+  int k = 1;
+  for (; k + 4 <= z.S; k += 4) {  // four slabs requested at a time
+    float x[4][EI];
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+#pragma unroll
+      for (int i = 0; i < EI; ++i) x[u][i] = q[(k + u) * z.slab + col[i]];
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+#pragma unroll
+      for (int i = 0; i < EI; ++i) s[i] += x[u][i];
+  }
+  for (; k < z.S; ++k)
+#pragma unroll
+    for (int i = 0; i < EI; ++i) s[i] += q[k * z.slab + col[i]];
+  float mx = s[0];
+#pragma unroll
+  for (int i = 1; i < EI; ++i) mx = fmaxf(mx, s[i]);  // (clamped columns repeat a score)
+  mx = wave_top(mx);
   float sum = 0.f;
 #pragma unroll
   for (int i = 0; i < EI; ++i) {
     s[i] = sigmoid ? 1.f / (1.f + __expf(-s[i])) : __expf(s[i] - mx);
-    sum += s[i];
+    sum += lane + 64 * i < E ? s[i] : 0.f;
   }
   sum = wave_sum(sum);
 #pragma unroll
   for (int i = 0; i < EI; ++i) {
-    const int e = lane + 64 * i;
+    const float c = w[i];
     w[i] = sigmoid ? s[i] : s[i] / sum;
-    s[i] = e < E ? w[i] + (correction ? correction[e] : 0.f) : -__builtin_huge_valf();
+    s[i] = lane + 64 * i < E ? w[i] + c : -__builtin_huge_valf();
   }
   float total = 0.f, mine = 0.f;  // lane k keeps the k-th choice
   int mine_e = 0;
-  for (int k = 0; k < top; ++k) {
-    float best = -__builtin_huge_valf(), bw = 0.f;
-    int be = E;  // (behind every expert: a lane without one left)
+  for (k = 0; k < top; ++k) {
+    float best = s[0];
 #pragma unroll
-    for (int i = 0; i < EI; ++i)
-      if (s[i] > best) {
-        best = s[i];
-        bw = w[i];
-        be = lane + 64 * i;
-      }
+    for (int i = 1; i < EI; ++i) best = fmaxf(best, s[i]);
+    best = wave_top(best);
+    int be = E, at = 0;  // (E: no score is a number)
+    float bw = 0.f;
 #pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ob = __shfl_xor(best, o, 64);
-      const int oe = __shfl_xor(be, o, 64);
-      const float ow = __shfl_xor(bw, o, 64);
-      if (ob > best || (ob == best && oe < be)) {
-        best = ob;
-        be = oe;
-        bw = ow;
+    for (int i = EI - 1; i >= 0; --i) {  // the lowest of equal ones
+      const unsigned long long m = __ballot(s[i] == best);
+      if (m) {
+        at = __ffsll(m) - 1;
+        be = at + 64 * i;
+        bw = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(w[i]), at));
       }
     }
     total += bw;
@@ -86,12 +117,13 @@ int moe_route(Proj z, int col0, int E, int top, float scale, int scores, const f
   if (T <= 0) return 0;
   if (E < 1 || E > 1024 || top < 1 || top > 64 || top > E || !z.f32 || z.S < 1 || scores < 0 || scores > 2) return hipErrorInvalidValue;
   const dim3 grid((T + 3) / 4);
-  if (E <= 64) hipLaunchKernelGGL((moe_route_kernel<float, 1>), grid, dim3(256), 0, s, z, col0, E, top, scale, scores,
-                                  correction, idx, wt, T);
-  else if (E <= 256) hipLaunchKernelGGL((moe_route_kernel<float, 4>), grid, dim3(256), 0, s, z, col0, E, top, scale, scores,
-                                  correction, idx, wt, T);
-  else hipLaunchKernelGGL((moe_route_kernel<float, 16>), grid, dim3(256), 0, s, z, col0, E, top, scale, scores,
-                                  correction, idx, wt, T);
+#define ROUTE_L(EI) \
+  hipLaunchKernelGGL(moe_route_kernel<EI>, grid, dim3(256), 0, s, z, col0, E, top, scale, scores, correction, idx, wt, T)
+  if (E <= 64) ROUTE_L(1);
+  else if (E <= 128) ROUTE_L(2);
+  else if (E <= 256) ROUTE_L(4);
+  else ROUTE_L(16);
+#undef ROUTE_L
   return hipGetLastError();
 }
 

@@ -191,8 +191,7 @@ class BizetarModel(HybridProjections):
         o = torch.empty((T, a.H * a.D), dtype=self.dtype, device=h.device)
         if Tp:
             ops.chunk_prefill(q[:Tp], kc, vc, meta.block_tables, meta.cu_q, meta.ctx_lens, meta.max_q, L.mixer.scale, 0, L.sink,
-                              o[:Tp], slopes=L.slopes)
-            ops.sigmoid_gate(y, at["g"], o[:Tp], per)
+                              o[:Tp], slopes=L.slopes, gate=(y, at["g"], per))
         if Tp < T:  # (mixed steps have finished projections)
             bt, ctx = (meta.block_tables, meta.ctx_lens) if meta.decode else (meta.dec_block_tables, meta.dec_ctx_lens)
             ops.chunk_decode(q[Tp:], kc, vc, bt, ctx, L.mixer.scale, 0, L.sink, o[Tp:], 1.0, meta.part_size, meta.workspace,

@@ -158,27 +158,48 @@ def _check_attn(q, kc, vc, bt, ctx, B, sink, out, slopes=None):
     same_device(q, kc, bt, ctx, sink, slopes, out)
 
 
+_NO_GATE = (0, 0, 1, 0, 0, 0, 1)
+
+
+def _output_gate(gate, T: int, n: int):
+    """(projection, column, per) of a gate of [T, n] outputs as the kernels take it."""
+    if gate is None:
+        return _NO_GATE
+    y, col, per = gate
+    expect(per >= 1 and n % per == 0, "whole groups of gated columns")
+    return (*_proj(y, T, col + n // per, "gate"), int(col), int(per))
+
+
 def chunk_prefill(q, kc, vc, bt, cu, ctx, max_q: int, scale: float, chunk: int, sink, out, out_scale: float = 1.0,
-                  slopes=None):
+                  slopes=None, gate=None):
     """Causal attention of prompt portions over the paged cache in which query i sees the keys of its own chunk,
     i // chunk * chunk .. i (0: all before it).  ``sink`` fp32 [H]: one more score in the denominator.  ``slopes`` fp32
-    [H]: slope * (i - j) is taken off the score of key j.  Writes out_scale * result to ``out``, rows [T, >= H D]."""
-    if not q.is_cuda:
-        T = q.shape[0]
-        out[:T, :q.shape[1] * q.shape[2]] = ref.chunk_attention(
-            q, kc, vc, bt, cu, ctx, scale, chunk, sink, out_scale, slopes).view(T, -1).to(out.dtype)
-        return out
+    [H]: slope * (i - j) is taken off the score of key j.  Writes out_scale * result to ``out``, rows [T, >= H D]; with ``gate``
+    = (projection, column, per) times the sigmoid of its columns, as ``sigmoid_gate``."""
     T, H, D = q.shape
+
+    def gated():
+        if gate is not None:
+            sigmoid_gate(gate[0], gate[1], out[:T, :H * D], gate[2])
+        return out
+
+    if not q.is_cuda:
+        out[:T, :H * D] = ref.chunk_attention(q, kc, vc, bt, cu, ctx, scale, chunk, sink, out_scale, slopes).view(T, -1).to(out.dtype)
+        return gated()
     _i32(cu)
     B = cu.numel() - 1
     _check_attn(q, kc, vc, bt, ctx, B, sink, out, slopes)
     if q.dtype == torch.float32 or D not in CHUNK_FLASH_DIMS or kc.shape[2] % 64:
-        return _any(q, kc, vc, bt, cu, ctx, B, scale, chunk, sink, out, out_scale, slopes)
+        _any(q, kc, vc, bt, cu, ctx, B, scale, chunk, sink, out, out_scale, slopes)
+        return gated()
+    og = _output_gate(gate, T, H * D)
+    fused = (gate is not None and D == 128 and chunk == 0 and out_scale == 1.0 and scale > 0 and (sink is not None or slopes is not None)
+             and gate[0].dtype == torch.bfloat16 and gate[0].dim() == 2 and gate[1] % 4 == 0 and og[4] % 4 == 0 and gate[2] in (1, D))
     qst, qsh = _head_strides(q)
     native().flash_attention_chunk(ptr(q), qst, qsh, ptr(kc), ptr(vc), ptr(bt), bt.shape[1], kc.shape[2], ptr(out),
                                    out.stride(0), D, ptr(cu), ptr(ctx), B, int(max_q), H, kc.shape[1], D, float(scale),
-                                   int(chunk), ptr(sink), ptr(slopes), float(out_scale), stream(q))
-    return out
+                                   int(chunk), ptr(sink), ptr(slopes), float(out_scale), og if fused else _NO_GATE, stream(q))
+    return out if fused else gated()
 
 
 def chunk_decode(q, kc, vc, bt, ctx, scale: float, chunk: int, sink, out, out_scale: float = 1.0, part_size: int = 512,
@@ -213,16 +234,10 @@ def chunk_decode(q, kc, vc, bt, ctx, scale: float, chunk: int, sink, out, out_sc
     if order is not None:
         _i32(order)
         expect(order.numel() >= B, "decode order must hold the batch")
-    og = (0, 0, 1, 0, 0, 0, 1)
-    if gate is not None:
-        y, col, per = gate
-        expect(per >= 1 and H * D % per == 0, "whole groups of gated columns")
-        og = (*_proj(y, B, col + H * D // per, "gate"), int(col), int(per))
-        same_device(q, y)
     native().paged_decode_attention(ptr(q), ptr(kc), ptr(vc), ptr(bt), bt.shape[1], bs, ptr(ctx), ptr(out), *ws, B, H, G,
                                     D, int(part_size), int(parts), float(scale), stream(q), ptr(order), chunk=int(chunk),
                                     sink=ptr(sink), out_scale=float(out_scale), o_stride=out.stride(0), slopes=ptr(slopes),
-                                    gate=og)
+                                    gate=_output_gate(gate, B, H * D))
     return out
 
 

@@ -267,15 +267,18 @@ def test_prompts_of_many_blocks(lens, done, sloped, sunk):
     q, sink = rnd(sum(lens), H, D, seed=3), rnd(H, seed=4, dtype=F32) + 2
     slopes = oracle.slopes(H).float() if sloped else None
     cu = torch.tensor([0, *torch.tensor(lens).cumsum(0).tolist()], dtype=torch.int32)
-    got = torch.zeros(sum(lens), H * D, dtype=BF, device=DEV)
-    ops.chunk_prefill(*(dev(t) for t in (q, kc, vc, bt, cu, i32(*ctx))), max(lens), 0.11, 0, dev(sink) if sunk else None, got,
-                      slopes=dev(slopes))
+    got = [torch.zeros(sum(lens), H * D, dtype=BF, device=DEV) for _ in range(3)]
+    gates = [None] + [(rnd(sum(lens), 16 + H * D // per, seed=per), 16, per) for per in (1, D)]
+    for g, o in zip(gates, got):
+        ops.chunk_prefill(*(dev(t) for t in (q, kc, vc, bt, cu, i32(*ctx))), max(lens), 0.11, 0, dev(sink) if sunk else None, o,
+                          slopes=dev(slopes), gate=None if g is None else (dev(g[0]), *g[1:]))
     some = sorted({0, len(lens) // 2, len(lens) - 1})
     for i in some:  # (the reference of a few sequences)
         want = torch.zeros(lens[i], H * D, dtype=BF)
         ops.chunk_prefill(q[cu[i]:cu[i + 1]], kc, vc, bt[i:i + 1], i32(0, lens[i]), i32(ctx[i]), lens[i], 0.11, 0, sink if sunk else None,
                           want, slopes=slopes)
-        close(got[cu[i]:cu[i + 1]], want, 1e-2)
+        for g, o in zip(gates, got):
+            close(o[cu[i]:cu[i + 1]], want if g is None else ops.sigmoid_gate(g[0][cu[i]:cu[i + 1]], g[1], want.clone(), g[2]), 1e-2)
 
 
 @pytest.mark.parametrize("T,E,top,S", [(1, 3, 1, 1), (70, 72, 8, 4), (5, 9, 9, 2), (300, 260, 6, 1), (33, 1024, 64, 1)])
