@@ -328,8 +328,9 @@ PYBIND11_MODULE(_native, m) {
                             u s) {
     check(dab::moe_route(proj(z), col0, E, top, scale, scores, (const float*)correction, (int*)idx, (float*)wt, T, ST(s)), "moe_route");
   });
-  m.def("moe_plan", [](u idx, int pairs, int E, int bm, u perm, u tiles, int max_tiles, u s) {
-    check(dab::moe_plan((const int*)idx, pairs, E, bm, (int*)perm, VP(tiles), max_tiles, ST(s)), "moe_plan");
+  m.def("moe_plan_words", &dab::moe_plan_words);
+  m.def("moe_plan", [](u idx, int pairs, int E, int bm, u perm, u tiles, int max_tiles, u ws, u s) {
+    check(dab::moe_plan((const int*)idx, pairs, E, bm, (int*)perm, VP(tiles), max_tiles, (int*)ws, ST(s)), "moe_plan");
   });
   m.def("shared_glu", [proj](const P& y, int col0, int F, const P& z, int sg_col, u out, long ldo, int act_f32, int T, u s) {
     check(dab::shared_glu(proj(y), col0, F, proj(z), sg_col, VP(out), ldo, act_f32, T, ST(s)), "shared_glu");

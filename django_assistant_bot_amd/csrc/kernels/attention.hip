@@ -1861,21 +1861,24 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
     const int np = min(p.max_parts, div_up(ctx - k_org, p.part_size));
     const bool direct = np == 1;
     // the finished output of head hq: the sink's term joins the denominator here, once
-    auto finish = [&](int qh, int d, float M, float L, float O) {
+    auto gate_of = [&](int qh, int d) {  // (requested ahead of what it multiplies)
+      if (!p.gate.y.p) return 0.f;
+      const int c = p.gate.col + ((hk * G + qh) * D + d) / p.gate.per;
+      return p.gate.y.f32 ? proj_f32<float>(p.gate.y, b, c) : proj_f32<bf16>(p.gate.y, b, c);
+    };
+    auto finish = [&](int qh, int d, float M, float L, float O, float gate) {
       const int hh = hk * G + qh;
       if (p.sink) {
         const float sk = p.sink[hh] * 1.4426950408889634f, M2 = fmaxf(M, sk), f = exp2f(M - M2);
         L = L * f + exp2f(sk - M2);
         O *= f;
       }
-      if (p.gate.y.p) {
-        const int c = p.gate.col + (hh * D + d) / p.gate.per;
-        O /= 1.f + __expf(-(p.gate.y.f32 ? proj_f32<float>(p.gate.y, b, c) : proj_f32<bf16>(p.gate.y, b, c)));
-      }
+      if (p.gate.y.p) O /= 1.f + __expf(-gate);
       p.out[(size_t)b * p.o_stride_tok + (size_t)hh * D + d] = f2bf(L > 0.f ? O / L * p.out_scale : 0.f);
     };
     for (int e = tid; e < G * D; e += 256) {
       const int qh = e / D, d = e % D;
+      const float gate = direct ? gate_of(qh, d) : 0.f;
       float M = -1e30f;
 #pragma unroll
       for (int ww = 0; ww < 4; ++ww) M = fmaxf(M, mred[ww * 16 + qh]);
@@ -1888,7 +1891,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
       }
       const size_t hq = (size_t)b * p.Hq + hk * G + qh;
       if (direct) {
-        finish(qh, d, M, L, O);
+        finish(qh, d, M, L, O, gate);
       } else {
         const size_t pi = hq * p.max_parts + part;
         // write-through (sc1) stores: visible to the combining workgroup on any XCD without a
@@ -1919,6 +1922,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
         auto ld = [](const float* a) { return __hip_atomic_load(a, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); };
         for (int e = tid; e < G * D; e += 256) {
           const int qh = e / D, d = e % D;
+          const float gate = gate_of(qh, d);
           const size_t hq = (size_t)b * p.Hq + hk * G + qh;
           const size_t base = hq * p.max_parts;
           float M = -1e30f;
@@ -1929,7 +1933,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
             L += f * ld(p.part_l + base + i);
             O += f * ld(p.part_o + (base + i) * D + d);
           }
-          finish(qh, d, M, L, O);
+          finish(qh, d, M, L, O, gate);
         }
       }
     }

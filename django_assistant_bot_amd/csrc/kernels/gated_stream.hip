@@ -44,17 +44,20 @@ __global__ __launch_bounds__(1024) void gated_residual_kernel(GatedResidual p) {
     if (p.src) ElemIO<float>::load8(p.src + at, s[i]);
     if (p.y.p) proj8<PT>(p.y, yrow, c, f[i]);
     if (p.pairs) {
-      for (int k = 0; k < p.top; ++k) {
-        const size_t e = (size_t)row * p.top + k;
-        if (p.idx[e] < p.experts) {
-          float v[8];
-          ElemIO<AT>::load8((const AT*)p.pairs + e * p.cols + c, v);
+      const int* idx = p.idx + (size_t)row * p.top;
+      const float* wt = p.wt + (size_t)row * p.top;
+      const AT* q = (const AT*)p.pairs + (size_t)row * p.top * p.cols + c;
+      for (int k0 = 0; k0 < p.top; k0 += 4) {  // four choices requested at a time
+        float v[4][8];
 #pragma unroll
-          for (int j = 0; j < 8; ++j) f[i][j] += v[j];
-        } else {
-          const float w = p.wt[e];
+        for (int u = 0; u < 4; ++u) ElemIO<AT>::load8(q + (size_t)min(k0 + u, p.top - 1) * p.cols, v[u]);
 #pragma unroll
-          for (int j = 0; j < 8; ++j) f[i][j] = fmaf(w, s[i][j], f[i][j]);
+        for (int u = 0; u < 4; ++u) {
+          if (k0 + u >= p.top) break;
+          const bool real = idx[k0 + u] < p.experts;  // (an identity expert's row was not written)
+          const float w = wt[k0 + u];
+#pragma unroll
+          for (int j = 0; j < 8; ++j) f[i][j] += real ? v[u][j] : w * s[i][j];
         }
       }
     }

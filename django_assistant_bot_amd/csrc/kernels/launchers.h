@@ -199,7 +199,8 @@ int selective_step(const void* u, int act_f32, SelectiveShape d, const void* dt_
 int moe_route(Proj z, int col0, int E, int top, float scale, int scores, const float* correction, int* idx, float* wt, int T,
               hipStream_t s);
 // pairs whose index is E or more (identity experts) come last in perm and are in no tile
-int moe_plan(const int* idx, int P, int E, int bm, int* perm, void* tiles, int max_tiles, hipStream_t s);
+int moe_plan(const int* idx, int P, int E, int bm, int* perm, void* tiles, int max_tiles, int* ws, hipStream_t s);
+int moe_plan_words(int P, int E);  // ints of ws (0: none)
 int shared_glu(Proj y, int col0, int F, Proj z, int sg_col, void* out, long ldo, int act_f32, int T, hipStream_t s);
 
 // dyt.hip (Dynamic Tanh norms around an fp32 residual stream)

@@ -4,8 +4,8 @@
 //                times ``scale``; or (sigmoid, raw softmax) the ``top`` largest as they are times ``scale``.  A correction
 //                per expert joins the score where the experts are chosen, not in the weight; one wave per token
 //   plan         (token, expert) pairs grouped by expert: perm[sorted position] = pair, and the row tiles of
-//                the grouped GEMM, each {expert, first sorted position, rows}; one workgroup.  Pairs of identity experts
-//                (index >= E) come last and are in no tile
+//                the grouped GEMM, each {expert, first sorted position, rows}; one workgroup, or
+//                for many pairs three launches.  Pairs of identity experts (index >= E) come last and are in no tile
 //   shared_glu   silu(gate) up sigmoid(w_sg h) of the expert that every token runs
 //
 // Which rows an expert gets does not change a row's result, so the order within an expert is left to the
@@ -127,56 +127,122 @@ int moe_route(Proj z, int col0, int E, int top, float scale, int scores, const f
   return hipGetLastError();
 }
 
+// Offsets of the experts' rows and tiles from their counts cnt[0 .. E] (entry E: identity experts), by the first wave
+__device__ __forceinline__ void plan_offsets(const int* cnt, int* off, int* tof, int E, int bm) {
+  const int lane = threadIdx.x;
+  int base = 0, tbase = 0;
+  for (int e0 = 0; e0 < E; e0 += 64) {
+    const int e = e0 + lane;
+    const int c = e < E ? cnt[e] : 0, tc = (c + bm - 1) / bm;
+    int a = c, b = tc;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const int x = __shfl_up(a, o, 64), y = __shfl_up(b, o, 64);
+      if (lane >= o) {
+        a += x;
+        b += y;
+      }
+    }
+    if (e < E) {
+      off[e] = base + a - c;
+      tof[e] = tbase + b - tc;
+    }
+    base += __shfl(a, 63, 64);
+    tbase += __shfl(b, 63, 64);
+  }
+  if (lane == 0) {
+    off[E] = base;
+    tof[E] = tbase;
+  }
+}
+
 // tiles[i] = {expert, first sorted position, rows, 0}; rows 0 past the last tile
+__device__ __forceinline__ void plan_tiles(const int* cnt, const int* off, const int* tof, int E, int bm, int4* tiles, int max_tiles) {
+  for (int e = threadIdx.x; e < E; e += 1024) {
+    const int n = cnt[e];
+    for (int k = 0, t = tof[e]; k < n; k += bm, ++t)
+      if (t < max_tiles) tiles[t] = make_int4(e, off[e] + k, min(bm, n - k), 0);
+  }
+  for (int t = tof[E] + threadIdx.x; t < max_tiles; t += 1024) tiles[t] = make_int4(0, 0, 0, 0);
+}
+
 __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ idx, int P, int E, int bm, int* perm,
                                                         int4* tiles, int max_tiles) {
-  __shared__ int cnt[1025], off[1025], tof[1025];  // entry E: identity experts
+  __shared__ int cnt[1025], off[1025], tof[1025];
   const int tid = threadIdx.x;
   for (int e = tid; e <= E; e += 1024) cnt[e] = 0;
   __syncthreads();
   for (int i = tid; i < P; i += 1024) atomicAdd(&cnt[min(idx[i], E)], 1);
   __syncthreads();
-  if (tid < 64) {  // prefix sums of rows and tiles, 64 experts a step
-    int base = 0, tbase = 0;
-    for (int e0 = 0; e0 < E; e0 += 64) {
-      const int e = e0 + tid;
-      const int c = e < E ? cnt[e] : 0, tc = (c + bm - 1) / bm;
-      int a = c, b = tc;
-#pragma unroll
-      for (int o = 1; o < 64; o <<= 1) {
-        const int x = __shfl_up(a, o, 64), y = __shfl_up(b, o, 64);
-        if (tid >= o) {
-          a += x;
-          b += y;
-        }
-      }
-      if (e < E) {
-        off[e] = base + a - c;
-        tof[e] = tbase + b - tc;
-      }
-      base += __shfl(a, 63, 64);
-      tbase += __shfl(b, 63, 64);
-    }
-    if (tid == 0) {
-      off[E] = base;
-      tof[E] = tbase;
-    }
-  }
+  if (tid < 64) plan_offsets(cnt, off, tof, E, bm);
   __syncthreads();
-  for (int e = tid; e < E; e += 1024) {
-    const int n = cnt[e];
-    for (int k = 0, t = tof[e]; k < n; k += bm, ++t)
-      if (t < max_tiles) tiles[t] = make_int4(e, off[e] + k, min(bm, n - k), 0);
-  }
-  for (int t = tof[E] + tid; t < max_tiles; t += 1024) tiles[t] = make_int4(0, 0, 0, 0);
+  plan_tiles(cnt, off, tof, E, bm, tiles, max_tiles);
   __syncthreads();
   for (int i = tid; i < P; i += 1024) perm[atomicAdd(&off[min(idx[i], E)], 1)] = i;
 }
 
-int moe_plan(const int* idx, int P, int E, int bm, int* perm, void* tiles, int max_tiles, hipStream_t s) {
+// The same for many pairs in three launches: kPlanParts workgroups count their parts, one turns the counts ws[part][E + 1] into
+// each part's first positions and writes the tiles, and the parts place their pairs.
+constexpr int kPlanParts = 32;
+
+__global__ __launch_bounds__(1024) void moe_count_kernel(const int* __restrict__ idx, int P, int E, int part, int* __restrict__ ws) {
+  __shared__ int cnt[1025];
+  for (int e = threadIdx.x; e <= E; e += 1024) cnt[e] = 0;
+  __syncthreads();
+  const int i1 = min(P, (int)(blockIdx.x + 1) * part);
+  for (int i = blockIdx.x * part + threadIdx.x; i < i1; i += 1024) atomicAdd(&cnt[min(idx[i], E)], 1);
+  __syncthreads();
+  for (int e = threadIdx.x; e <= E; e += 1024) ws[blockIdx.x * (E + 1) + e] = cnt[e];
+}
+
+__global__ __launch_bounds__(1024) void moe_offsets_kernel(int* __restrict__ ws, int E, int bm, int4* tiles, int max_tiles) {
+  __shared__ int cnt[1025], off[1025], tof[1025];
+  const int tid = threadIdx.x;
+  for (int e = tid; e <= E; e += 1024) {
+    int n = 0;
+#pragma unroll
+    for (int b = 0; b < kPlanParts; ++b) n += ws[b * (E + 1) + e];
+    cnt[e] = n;
+  }
+  __syncthreads();
+  if (tid < 64) plan_offsets(cnt, off, tof, E, bm);
+  __syncthreads();
+  plan_tiles(cnt, off, tof, E, bm, tiles, max_tiles);
+  for (int e = tid; e <= E; e += 1024) {
+    int n[kPlanParts], at = off[e];
+#pragma unroll
+    for (int b = 0; b < kPlanParts; ++b) n[b] = ws[b * (E + 1) + e];
+#pragma unroll
+    for (int b = 0; b < kPlanParts; ++b) {
+      ws[b * (E + 1) + e] = at;
+      at += n[b];
+    }
+  }
+}
+
+__global__ __launch_bounds__(1024) void moe_place_kernel(const int* __restrict__ idx, int P, int E, int part, const int* __restrict__ ws,
+                                                         int* __restrict__ perm) {
+  __shared__ int off[1025];
+  for (int e = threadIdx.x; e <= E; e += 1024) off[e] = ws[blockIdx.x * (E + 1) + e];
+  __syncthreads();
+  const int i1 = min(P, (int)(blockIdx.x + 1) * part);
+  for (int i = blockIdx.x * part + threadIdx.x; i < i1; i += 1024) perm[atomicAdd(&off[min(idx[i], E)], 1)] = i;
+}
+
+int moe_plan_words(int P, int E) { return P < 16384 ? 0 : kPlanParts * (E + 1); }
+
+int moe_plan(const int* idx, int P, int E, int bm, int* perm, void* tiles, int max_tiles, int* ws, hipStream_t s) {
   if (P <= 0) return 0;
   if (E < 1 || E > 1024 || bm < 1 || max_tiles < 1) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), 0, s, idx, P, E, bm, perm, (int4*)tiles, max_tiles);
+  if (!moe_plan_words(P, E)) {
+    hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), 0, s, idx, P, E, bm, perm, (int4*)tiles, max_tiles);
+    return hipGetLastError();
+  }
+  if (!ws) return hipErrorInvalidValue;
+  const int part = (P + kPlanParts - 1) / kPlanParts;
+  hipLaunchKernelGGL(moe_count_kernel, dim3(kPlanParts), dim3(1024), 0, s, idx, P, E, part, ws);
+  hipLaunchKernelGGL(moe_offsets_kernel, dim3(1), dim3(1024), 0, s, ws, E, bm, (int4*)tiles, max_tiles);
+  hipLaunchKernelGGL(moe_place_kernel, dim3(kPlanParts), dim3(1024), 0, s, idx, P, E, part, ws, perm);
   return hipGetLastError();
 }
 

@@ -508,7 +508,9 @@ def moe_experts(h, idx, wt, gate_up, down, E: int, group: int, weigh: str = "out
     dev, s, nat = h.device, stream(h), native()
     perm = torch.empty((P,), dtype=torch.int32, device=dev)
     tiles = torch.empty((n_tiles, 4), dtype=torch.int32, device=dev)
-    nat.moe_plan(ptr(idx), P, E, bm, ptr(perm), ptr(tiles), n_tiles, s)
+    words = nat.moe_plan_words(P, E)
+    ws = torch.empty((words,), dtype=torch.int32, device=dev) if words else None
+    nat.moe_plan(ptr(idx), P, E, bm, ptr(perm), ptr(tiles), n_tiles, ptr(ws), s)
     act = torch.empty((P, F2 // 2), dtype=h.dtype, device=dev)
     out = torch.empty((P, W), dtype=h.dtype, device=dev)
     if f32:

@@ -293,7 +293,7 @@ def test_corrected_routing(T, E, top, S, scores):
     close(wt.cpu().gather(-1, a.indices), rw.gather(-1, b.indices), 1e-5)
 
 
-@pytest.mark.parametrize("T,E,extra,top", [(1, 4, 2, 3), (40, 6, 6, 6), (300, 8, 1, 2), (9, 3, 9, 2), (2000, 16, 4, 5)])
+@pytest.mark.parametrize("T,E,extra,top", [(1, 4, 2, 3), (40, 6, 6, 6), (300, 8, 1, 2), (9, 3, 9, 2), (2000, 16, 4, 5), (4100, 8, 3, 4), (5000, 70, 2, 4)])
 @pytest.mark.parametrize("dtype", [BF, F32])
 def test_identity_experts(T, E, extra, top, dtype):
     """Choices behind the experts take no row of the grouped products and give the stream itself."""
