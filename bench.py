@@ -285,7 +285,7 @@ def main():
                          "5 = bge-large + Llama-3-70B, TP = --gpus, serve mode at a fixed QPS (--qps, default 4)")
     ap.add_argument("--decoder-bench", default=None, metavar="MODEL[,MODEL]",
                     help="instead of the RAG workload: prefill / decode throughput of these decoder presets side by side "
-                         "(benchmarks/decoder_bench.py), e.g. vunelix-8b,llama-3-8b")
+                         "(benchmarks/decoder_bench.py), e.g. bizetar-8b,llama-3-8b")
     ap.add_argument("--decoder-shapes", default=None, metavar="KIND:BATCHxLEN[,...]",
                     help="shapes of --decoder-bench, e.g. prefill:16x1024,decode:128x2048")
     args = ap.parse_args()
