@@ -1588,10 +1588,10 @@ struct DecodeParams {
   // holds the chunk's first key.  sink (or null): one more score in head h's denominator
   int chunk;
   const float* sink;
-  const float* slopes;  // SLOPE: slopes[h] times the distance is taken off a key's score
+  const float* slopes;  // EXT: slopes[h] times the distance is taken off a key's score (null: none)
   float out_scale;
   long o_stride_tok;
-  OutputGate gate;  // optional (gate.y.p): the finished output times its sigmoid
+  OutputGate gate;  // EXT, optional (gate.y.p): the finished output times its sigmoid
   L3Warm warm;  // optional: the next projections' weights, warmed into L3 by appended workgroups
 };
 
@@ -1606,7 +1606,9 @@ struct DecodeParams {
 // the first copy.  At batch 1 - 8 a workgroup's waves walk their sub-tiles back to back with the
 // whole GPU otherwise idle: one copy round trip per sub-tile was the critical path.  128 KB of LDS:
 // one workgroup per CU, which small batches never fill anyway.
-template <int D, bool KV_NT, bool DMA = false, int NSLOT = 1, bool SLOPE = false>
+//
+// EXT: slopes (may be null) and the output gate; the plain form is free of both.
+template <int D, bool KV_NT, bool DMA = false, int NSLOT = 1, bool EXT = false>
 __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(DecodeParams p, int total_items) {
   static_assert(NSLOT == 1 || (NSLOT == 2 && DMA), "two slots: DMA staging only");
   // appended workgroups (small batches leave most CUs idle during this latency-bound launch): warm
@@ -1709,7 +1711,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
 #pragma unroll
     for (int t = 0; t < NTD; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m_run = -1e30f, l_run = 0.f;
-    const float slope = SLOPE ? p.slopes[hk * G + min(li, G - 1)] * 1.4426950408889634f : 0.f;
+    const float slope = EXT && p.slopes ? p.slopes[hk * G + min(li, G - 1)] * 1.4426950408889634f : 0.f;
 
     auto compute = [&](const int k0) {
       __builtin_amdgcn_s_waitcnt(0xc07f);  // lgkmcnt(0): this wave's LDS writes landed
@@ -1731,7 +1733,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
         for (int r = 0; r < 4; ++r) {
           const int key = k0 + 16 * m + 4 * g + r;
           float v = s[m][r] * p.scale_log2;
-          if (SLOPE) v = fmaf(slope, (float)(key - (ctx - 1)), v);
+          if (EXT) v = fmaf(slope, (float)(key - (ctx - 1)), v);
           if (key >= k_end || key < k_lo) v = kNegInf;
           s[m][r] = v;
           mx = fmaxf(mx, v);
@@ -1862,7 +1864,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
     const bool direct = np == 1;
     // the finished output of head hq: the sink's term joins the denominator here, once
     auto gate_of = [&](int qh, int d) {  // (requested ahead of what it multiplies)
-      if (!p.gate.y.p) return 0.f;
+      if (!EXT || !p.gate.y.p) return 0.f;
       const int c = p.gate.col + ((hk * G + qh) * D + d) / p.gate.per;
       return p.gate.y.f32 ? proj_f32<float>(p.gate.y, b, c) : proj_f32<bf16>(p.gate.y, b, c);
     };
@@ -1873,7 +1875,7 @@ __global__ __launch_bounds__(256, NSLOT == 1 ? 2 : 1) void paged_decode_kernel(D
         L = L * f + exp2f(sk - M2);
         O *= f;
       }
-      if (p.gate.y.p) O /= 1.f + __expf(-gate);
+      if (EXT && p.gate.y.p) O /= 1.f + __expf(-gate);
       p.out[(size_t)b * p.o_stride_tok + (size_t)hh * D + d] = f2bf(L > 0.f ? O / L * p.out_scale : 0.f);
     };
     for (int e = tid; e < G * D; e += 256) {
@@ -2194,6 +2196,7 @@ int paged_decode_attention(const void* q, const void* k_cache, const void* v_cac
   if (prm.warm.blocks < 0 || prm.warm.blocks > 1024 || ((prm.warm.bytes[0] | prm.warm.bytes[1]) & 15) ||
       (prm.warm.blocks && prm.warm.bytes[0] + prm.warm.bytes[1] <= 0))
     return hipErrorInvalidValue;
+  const bool ext = slopes || prm.gate.y.p;
   const int total_items = max_parts * Hkv * batch;
   dim3 grid((total_items < 2048 ? total_items : 2048) + prm.warm.blocks);
   // K/V are read exactly once per step: non-temporal loads (aux = 2) -- in the Llama-3-8B decode step
@@ -2204,14 +2207,14 @@ int paged_decode_attention(const void* q, const void* k_cache, const void* v_cac
     // small batches: two LDS slots per wave (at batch 128 the one-slot kernel's two workgroups per CU
     // are 2.8 % faster per step: 7.44 vs 7.65 ms, profiles/low_load_latency.md)
     const bool two = batch * Hkv <= 64 && part_size <= 64 * 4 * 32;
-    if (two && slopes)
+    if (two && ext)
       hipLaunchKernelGGL((paged_decode_kernel<128, true, true, 2, true>), grid, dim3(256), 0, s, prm, total_items);
     else if (two) hipLaunchKernelGGL((paged_decode_kernel<128, true, true, 2>), grid, dim3(256), 0, s, prm, total_items);
-    else if (slopes)
+    else if (ext)
       hipLaunchKernelGGL((paged_decode_kernel<128, true, true, 1, true>), grid, dim3(256), 0, s, prm, total_items);
     else hipLaunchKernelGGL((paged_decode_kernel<128, true, true>), grid, dim3(256), 0, s, prm, total_items);
   } else if (D == 64) {
-    if (slopes)
+    if (ext)
       hipLaunchKernelGGL((paged_decode_kernel<64, true, false, 1, true>), grid, dim3(256), 0, s, prm, total_items);
     else hipLaunchKernelGGL((paged_decode_kernel<64, true>), grid, dim3(256), 0, s, prm, total_items);
   } else {
